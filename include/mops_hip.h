@@ -327,6 +327,128 @@ int mops_hip_linear_tune(int64_t m, int64_t n, int64_t k, int64_t distinct_weigh
                          void* workspace, int64_t workspace_bytes,
                          int* best_solution_index, float* best_us, float* heuristic_us);
 
+/* ---------------------------------------------------------------------------------------------------------------------
+ * Operators of models with recurrent layers, latent attention and a float32 residual stream.  No counterpart in the
+ * reference.  They exist for two element types of activations, weights and caches, named by `dtype`; everything they
+ * reduce, scale or carry from token to token is float32 either way.
+ * Positions, state slots and sequence metadata are int32 on the device.
+ * ------------------------------------------------------------------------------------------------------------------- */
+#define MOPS_HIP_BF16 0
+#define MOPS_HIP_F32 1
+
+/* residual[i, :] = float(table[ids[i], :]) and act[i, :] = table[ids[i], :]; an id outside [0, vocab) gives zeros. */
+int mops_hip_embed_residual(const int64_t* ids, const void* table, int64_t table_row_stride, int dtype,
+                            float* residual, void* act, int64_t n_ids, int64_t vocab, int64_t width, void* stream);
+
+/* residual += y / sqrt(mean(y^2) + eps) * (weight_offset + weight), rowwise and in place; act = the new residual in `dtype`. */
+int mops_hip_norm_residual_add(float* residual, const void* y, int64_t y_row_stride, const void* weight, float weight_offset,
+                               float eps, void* act, int dtype, int64_t rows, int64_t n, void* stream);
+
+/* out = x / sqrt(mean(x^2) + eps) * (weight_offset + weight) of float32 rows. */
+int mops_hip_rms_norm_f32(const float* x, const void* weight, float weight_offset, float eps, void* out, int dtype,
+                          int64_t rows, int64_t n, void* stream);
+
+/*
+ * Rows of groups * group_size elements, every group divided by its own root mean square:
+ *   gate_first == 0:  out = rms(y) * silu(gate) [* weight];  else  out = rms(y * silu(gate)) [* weight].   weight may be NULL.
+ * out is contiguous and may be y itself when y is contiguous.
+ */
+int mops_hip_gated_group_norm(const void* y, int64_t y_row_stride, const void* gate, int64_t gate_row_stride,
+                              const void* weight, float eps, int gate_first, void* out, int dtype,
+                              int64_t rows, int64_t groups, int64_t group_size, void* stream);
+
+/* out = g * sigmoid(alpha * g) * (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit). */
+int mops_hip_clamped_glu(const void* gate, int64_t gate_row_stride, const void* up, int64_t up_row_stride, void* out,
+                         int dtype, int64_t rows, int64_t n, float alpha, float limit, void* stream);
+
+/*
+ * A linear recurrence with one decay per head and token (see csrc/decayed_recurrence.hip):
+ *   S_t = a_t S_(t-1) + k_t (s_t v_t)^T,   o_t = S_t^T q_t + skip v_t
+ * q, k: [tokens, groups * d], v, out: [tokens, heads * vd] with token strides in elements; value head h uses q/k head
+ * h / (heads / groups).  Exactly one of `decay` (float [heads]: constant) and `dt` ([tokens, heads] in `dtype`, with
+ * dt_bias and neg_a float [heads]: s = softplus(dt + dt_bias), a = exp(neg_a * s)) is given; skip may be NULL.
+ * rot > 0 rotates dimensions i and i + rot/2 of q and k (i < rot/2) by row `position` of cos_sin [max_positions, rot]
+ * (cosines, then sines); k is multiplied by k_scale afterwards.
+ * cu_seqlens: int32 [batch + 1], or NULL when every sequence brings one token.  starts[b]: position of the first token of
+ * the portion; 0 starts from a zero state whatever the slot holds.
+ * state: float [num_slots, heads, vd, pitch], pitch = mops_hip_recurrence_state_pitch(d); state_slots[b] < 0: a padding
+ * row, out is zeros and nothing is stored.
+ * conv_weight != NULL (one token per sequence only): the short convolution of mops_hip_short_conv is applied to q, k and v
+ * on the way in, channels q_channel.. k_channel.. v_channel.. of `channels`, and the ring receives the token.
+ * d <= 256.
+ */
+typedef struct {
+  const void *q, *k, *v;
+  int64_t q_stride, k_stride, v_stride;
+  void* out;
+  int64_t out_stride;
+  float* state;
+  int64_t num_slots;
+  const int32_t *state_slots, *cu_seqlens, *starts;
+  const float *decay, *neg_a, *dt_bias, *skip, *cos_sin;
+  const void* dt;
+  int64_t dt_stride;
+  int64_t batch, heads, groups, d, vd, rot, max_positions;
+  const float *conv_weight, *conv_bias;
+  void* conv_ring;
+  int64_t taps, channels, q_channel, k_channel, v_channel;
+  float k_scale;
+  int dtype;
+} mops_hip_recurrence;
+int64_t mops_hip_recurrence_state_pitch(int64_t d);
+int mops_hip_decayed_recurrence(const mops_hip_recurrence* r, void* stream);
+
+/*
+ * out[t, c] = silu(bias[c] + sum over lags l < taps of weight[taps-1-l, c] * x(position - l)[c]) for packed portions.
+ * weight: float [taps, channels]; x of earlier portions comes from ring [num_slots, taps, channels] (`dtype`), row
+ * position % taps; positions before 0 count as zeros.  token_seq: int32 [tokens], the sequence of each token.
+ */
+int mops_hip_short_conv(const void* x, int64_t x_row_stride, const float* weight, const float* bias, const void* ring,
+                        int64_t num_slots, const int32_t* token_seq, const int32_t* cu_seqlens, const int32_t* starts,
+                        const int32_t* state_slots, void* out, int dtype, int64_t tokens, int64_t channels, int64_t taps,
+                        void* stream);
+/* Files the last taps-1 inputs of every portion in the ring; launch it behind everything that still reads the ring. */
+int mops_hip_short_conv_update(const void* x, int64_t x_row_stride, void* ring, int64_t num_slots, const int32_t* cu_seqlens,
+                               const int32_t* starts, const int32_t* state_slots, int dtype, int64_t batch, int64_t channels,
+                               int64_t taps, void* stream);
+
+/*
+ * Latent attention (see csrc/latent_attention.hip).  latent_prepare: down [tokens, q_rank + kv_rank + rot_dim] ->
+ * q_latent [tokens, q_rank] = RMS norm * q_weight; cache row slot_mapping[t] of [num_slots, pitch] =
+ * [RMS norm of the kv latent * kv_weight | key part rotated in pairs (2i, 2i+1) | zeros]; slot < 0: no cache row.
+ */
+int mops_hip_latent_prepare(const void* down, int64_t down_stride, const void* q_weight, const void* kv_weight, float eps,
+                            const float* cos_sin, int64_t max_positions, const int32_t* positions, const int32_t* slot_mapping,
+                            void* q_latent, void* cache, int64_t num_slots, int64_t pitch, int dtype, int64_t tokens,
+                            int64_t q_rank, int64_t kv_rank, int64_t rot_dim, void* stream);
+
+/* y[t, h, :] = w[h] x[t, h, :] with w [heads, n, k] contiguous; token and head strides in elements. */
+int mops_hip_head_linear(const void* x, int64_t x_token_stride, int64_t x_head_stride, const void* w, void* y,
+                         int64_t y_token_stride, int64_t y_head_stride, int dtype, int64_t tokens, int64_t heads, int64_t n,
+                         int64_t k, void* stream);
+
+/*
+ * Query rows against the latent cache: row r sees the first context_lens[r] tokens of sequence row_seq[r] (row r itself when
+ * row_seq is NULL), its own position being context_lens[r] - 1; 0 gives zeros.  q_latent [rows, heads, kv_rank] contiguous,
+ * q_rot the rot_dim query values (not yet rotated) at token / head strides, out [rows, heads, kv_rank] contiguous.
+ * cache: [num_blocks, block_size, pitch]; a block table entry outside [0, num_blocks) counts as an empty block.
+ */
+typedef struct {
+  const void *q_latent, *q_rot;
+  int64_t q_rot_token_stride, q_rot_head_stride;
+  const void* cache;
+  int64_t pitch;
+  const float* cos_sin;
+  int64_t max_positions;
+  const int32_t *row_seq, *context_lens, *block_table;
+  int64_t block_table_stride, block_size, num_blocks, max_blocks;
+  void* out;
+  int64_t rows, heads, kv_rank, rot_dim;
+  float scale;
+  int dtype;
+} mops_hip_latent_rows;
+int mops_hip_latent_attention_rows(const mops_hip_latent_rows* a, void* stream);
+
 #ifdef __cplusplus
 }
 #endif

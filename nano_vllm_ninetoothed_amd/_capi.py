@@ -7,11 +7,32 @@ from __future__ import annotations
 
 import ctypes
 import os
-from ctypes import c_char_p, c_float, c_int, c_int64, c_void_p
+from ctypes import POINTER, Structure, c_char_p, c_float, c_int, c_int64, c_void_p
 from pathlib import Path
 
 # MOPS_HIP_LIB points at another build of the same ABI (kernel tuning experiments)
 LIB_PATH = Path(os.environ.get("MOPS_HIP_LIB") or Path(__file__).resolve().parent / "lib" / "libmops_hip.so")
+
+class Recurrence(Structure):
+    """mops_hip_recurrence of the header, field by field."""
+    _fields_ = ([(n, c_void_p) for n in ("q", "k", "v")] + [(n, c_int64) for n in ("q_stride", "k_stride", "v_stride")]
+                + [("out", c_void_p), ("out_stride", c_int64), ("state", c_void_p), ("num_slots", c_int64)]
+                + [(n, c_void_p) for n in ("state_slots", "cu_seqlens", "starts", "decay", "neg_a", "dt_bias", "skip", "cos_sin", "dt")]
+                + [(n, c_int64) for n in ("dt_stride", "batch", "heads", "groups", "d", "vd", "rot", "max_positions")]
+                + [(n, c_void_p) for n in ("conv_weight", "conv_bias", "conv_ring")]
+                + [(n, c_int64) for n in ("taps", "channels", "q_channel", "k_channel", "v_channel")]
+                + [("k_scale", c_float), ("dtype", c_int)])
+
+
+class LatentRows(Structure):
+    """mops_hip_latent_rows of the header, field by field."""
+    _fields_ = ([(n, c_void_p) for n in ("q_latent", "q_rot")] + [(n, c_int64) for n in ("q_rot_token_stride", "q_rot_head_stride")]
+                + [("cache", c_void_p), ("pitch", c_int64), ("cos_sin", c_void_p), ("max_positions", c_int64)]
+                + [(n, c_void_p) for n in ("row_seq", "context_lens", "block_table")]
+                + [(n, c_int64) for n in ("block_table_stride", "block_size", "num_blocks", "max_blocks")]
+                + [("out", c_void_p)] + [(n, c_int64) for n in ("rows", "heads", "kv_rank", "rot_dim")]
+                + [("scale", c_float), ("dtype", c_int)])
+
 
 # name -> (restype, argtypes); the exported surface declared in include/mops_hip.h
 SIGNATURES = {
@@ -52,11 +73,29 @@ SIGNATURES = {
                                             c_int64, c_int64, c_float, c_void_p]),
     "mops_hip_linear_bf16": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int64, c_int64,
                                      c_int64, c_void_p, c_int64, c_void_p]),
+    "mops_hip_embed_residual": (c_int, [c_void_p, c_void_p, c_int64, c_int, c_void_p, c_void_p, c_int64, c_int64, c_int64, c_void_p]),
+    "mops_hip_norm_residual_add": (c_int, [c_void_p, c_void_p, c_int64, c_void_p, c_float, c_float, c_void_p, c_int, c_int64, c_int64,
+                                           c_void_p]),
+    "mops_hip_rms_norm_f32": (c_int, [c_void_p, c_void_p, c_float, c_float, c_void_p, c_int, c_int64, c_int64, c_void_p]),
+    "mops_hip_gated_group_norm": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_float, c_int, c_void_p, c_int, c_int64,
+                                          c_int64, c_int64, c_void_p]),
+    "mops_hip_clamped_glu": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int, c_int64, c_int64, c_float, c_float, c_void_p]),
+    "mops_hip_recurrence_state_pitch": (c_int64, [c_int64]),
+    "mops_hip_decayed_recurrence": (c_int, [POINTER(Recurrence), c_void_p]),
+    "mops_hip_short_conv": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p,
+                                    c_void_p, c_int, c_int64, c_int64, c_int64, c_void_p]),
+    "mops_hip_short_conv_update": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int, c_int64, c_int64,
+                                           c_int64, c_void_p]),
+    "mops_hip_latent_prepare": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_float, c_void_p, c_int64, c_void_p, c_void_p, c_void_p,
+                                        c_void_p, c_int64, c_int64, c_int, c_int64, c_int64, c_int64, c_int64, c_void_p]),
+    "mops_hip_head_linear": (c_int, [c_void_p, c_int64, c_int64, c_void_p, c_void_p, c_int64, c_int64, c_int, c_int64, c_int64, c_int64,
+                                     c_int64, c_void_p]),
+    "mops_hip_latent_attention_rows": (c_int, [POINTER(LatentRows), c_void_p]),
     "mops_hip_linear_pin_solution": (c_int, [c_int64, c_int64, c_int64, c_int]),
     "mops_hip_linear_tune": (c_int, [c_int64, c_int64, c_int64, c_int64, c_int, c_void_p, c_int64, c_void_p, c_void_p, c_void_p]),
 }
 
-ABI_VERSION = 9
+ABI_VERSION = 10
 
 _lib = None
 

@@ -1,0 +1,231 @@
+// A float32 residual stream and the norms around it, for models whose residual sum and norms are kept in 32 bits.
+//
+//   embed_residual     x = table[id], as float32 (the residual) and in the activation type (the first projection's input)
+//   norm_residual_add  x += rms(y) * (offset + w): the norm sits on the sublayer's output, the sum runs on in float32 and
+//                      leaves a copy in the activation type for the next projection
+//   rms_norm_f32       out = rms(x) * (offset + w) of the float32 stream
+//   gated_group_norm   rms over equal parts of a row, with silu(gate) multiplied in before or after the division
+//
+// A row belongs to one workgroup of 64 or 256 threads; the elements a thread owns stay in its registers between the
+// statistics and the scaling (up to kKeep pieces; longer rows read the rest again).
+#include "mixed_types.h"
+
+namespace mops {
+
+constexpr int kKeep = 4;
+
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void embed_residual_kernel(const int64_t* __restrict__ ids, const T* __restrict__ table,
+                                                             int64_t table_stride, float* __restrict__ x, T* __restrict__ act,
+                                                             int64_t vocab, int width) {
+  const int64_t row = blockIdx.x;
+  const int64_t id = ids[row];
+  const bool ok = id >= 0 && id < vocab;
+  for (int c = threadIdx.x * VEC; c < width; c += 256 * VEC) {
+    float v[VEC];
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) v[e] = 0.f;
+    if (ok) load_vec<VEC>(table + id * table_stride + c, v);
+    store_vec<VEC>(x + row * width + c, v);
+    store_vec<VEC>(act + row * width + c, v);
+  }
+}
+
+// MODE 0: out = norm(x) with x float32; MODE 1: residual += norm(y), out = the new residual in the activation type.
+template <typename T, int VEC, int THREADS, int MODE>
+__global__ __launch_bounds__(THREADS) void norm_kernel(float* __restrict__ residual, const T* __restrict__ y, int64_t y_stride,
+                                                       const T* __restrict__ w, float offset, float eps, T* __restrict__ out,
+                                                       int n) {
+  __shared__ float scratch[THREADS / kWave];
+  const int64_t row = blockIdx.x;
+  float* xr = residual + row * n;
+  const T* yr = y + row * y_stride;
+  float keep[kKeep][VEC];
+  float ss = 0.f;
+#pragma unroll
+  for (int it = 0; it < kKeep; ++it) {
+    const int c = (it * THREADS + threadIdx.x) * VEC;
+    if (c < n) {
+      if (MODE == 0) load_vec<VEC>(xr + c, keep[it]);
+      else load_vec<VEC>(yr + c, keep[it]);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) ss += keep[it][e] * keep[it][e];
+    }
+  }
+  for (int c = (kKeep * THREADS + threadIdx.x) * VEC; c < n; c += THREADS * VEC) {
+    float v[VEC];
+    if (MODE == 0) load_vec<VEC>(xr + c, v);
+    else load_vec<VEC>(yr + c, v);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) ss += v[e] * v[e];
+  }
+  const float rstd = 1.0f / sqrtf(block_sum<THREADS>(ss, scratch) / (float)n + eps);
+  auto finish = [&](int c, const float (&v)[VEC]) {
+    float wv[VEC], o[VEC];
+    load_vec<VEC>(w + c, wv);
+    if (MODE == 1) {
+      load_vec<VEC>(xr + c, o);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) o[e] += v[e] * rstd * (offset + wv[e]);
+      store_vec<VEC>(xr + c, o);
+    } else {
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) o[e] = v[e] * rstd * (offset + wv[e]);
+    }
+    store_vec<VEC>(out + row * n + c, o);
+  };
+#pragma unroll
+  for (int it = 0; it < kKeep; ++it) {
+    const int c = (it * THREADS + threadIdx.x) * VEC;
+    if (c < n) finish(c, keep[it]);
+  }
+  for (int c = (kKeep * THREADS + threadIdx.x) * VEC; c < n; c += THREADS * VEC) {
+    float v[VEC];
+    if (MODE == 0) load_vec<VEC>(xr + c, v);
+    else load_vec<VEC>(yr + c, v);
+    finish(c, v);
+  }
+}
+
+// One wave per (row, part): parts of `size` consecutive elements.
+template <typename T, int VEC, bool GATE_FIRST>
+__global__ __launch_bounds__(256) void gated_group_norm_kernel(const T* __restrict__ y, int64_t y_stride, const T* __restrict__ gate,
+                                                               int64_t gate_stride, const T* __restrict__ w, float eps,
+                                                               T* __restrict__ out, int64_t rows, int groups, int size) {
+  const int64_t item = (int64_t)blockIdx.x * 4 + threadIdx.x / kWave;
+  if (item >= rows * groups) return;
+  const int lane = threadIdx.x & (kWave - 1);
+  const int64_t row = item / groups;
+  const int col0 = (int)(item % groups) * size;
+  const T* yr = y + row * y_stride + col0;
+  const T* gr = gate + row * gate_stride + col0;
+  T* orow = out + row * (int64_t)groups * size + col0;
+  float keep[kKeep][VEC], gk[kKeep][VEC];
+  float ss = 0.f;
+  auto read = [&](int c, float (&v)[VEC], float (&g)[VEC]) {
+    load_vec<VEC>(yr + c, v);
+    load_vec<VEC>(gr + c, g);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) {
+      g[e] = silu_f32(g[e]);
+      if (GATE_FIRST) v[e] *= g[e];
+    }
+  };
+#pragma unroll
+  for (int it = 0; it < kKeep; ++it) {
+    const int c = (it * kWave + lane) * VEC;
+    if (c < size) {
+      read(c, keep[it], gk[it]);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) ss += keep[it][e] * keep[it][e];
+    }
+  }
+  for (int c = (kKeep * kWave + lane) * VEC; c < size; c += kWave * VEC) {
+    float v[VEC], g[VEC];
+    read(c, v, g);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) ss += v[e] * v[e];
+  }
+  const float rstd = 1.0f / sqrtf(group_sum<kWave>(ss) / (float)size + eps);
+  auto finish = [&](int c, const float (&v)[VEC], const float (&g)[VEC]) {
+    float o[VEC];
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) o[e] = GATE_FIRST ? v[e] * rstd : v[e] * rstd * g[e];
+    if (w) {
+      float wv[VEC];
+      load_vec<VEC>(w + col0 + c, wv);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) o[e] *= wv[e];
+    }
+    store_vec<VEC>(orow + c, o);
+  };
+#pragma unroll
+  for (int it = 0; it < kKeep; ++it) {
+    const int c = (it * kWave + lane) * VEC;
+    if (c < size) finish(c, keep[it], gk[it]);
+  }
+  for (int c = (kKeep * kWave + lane) * VEC; c < size; c += kWave * VEC) {
+    float v[VEC], g[VEC];
+    read(c, v, g);
+    finish(c, v, g);
+  }
+}
+
+template <typename T, int MODE>
+static void launch_norm(float* residual, const void* y, int64_t y_stride, const void* w, float offset, float eps, void* out,
+                        int64_t rows, int64_t n, hipStream_t s) {
+  const bool vec = n % 8 == 0 && y_stride % 8 == 0 && aligned16(residual) && (MODE == 0 || aligned16(y)) && aligned16(w) && aligned16(out);
+  const dim3 grid((unsigned)rows);
+#define MOPS_NORM(V, TH) hipLaunchKernelGGL((norm_kernel<T, V, TH, MODE>), grid, dim3(TH), 0, s, residual, (const T*)y, y_stride, \
+                                            (const T*)w, offset, eps, (T*)out, (int)n)
+  if (vec && n <= 1024) MOPS_NORM(8, 64);
+  else if (vec) MOPS_NORM(8, 256);
+  else if (n <= 512) MOPS_NORM(1, 64);
+  else MOPS_NORM(1, 256);
+#undef MOPS_NORM
+}
+
+}  // namespace mops
+
+extern "C" int mops_hip_embed_residual(const int64_t* ids, const void* table, int64_t table_row_stride, int dtype, float* residual,
+                                       void* act, int64_t n_ids, int64_t vocab, int64_t width, void* stream) {
+  using namespace mops;
+  if (!known_dtype(dtype) || n_ids < 0 || vocab <= 0 || width <= 0 || width > (1 << 20) || n_ids > 0x7fffffffLL) return MOPS_HIP_EINVAL;
+  if (n_ids == 0) return MOPS_HIP_OK;
+  if (!ids || !table || !residual || !act || table_row_stride < width) return MOPS_HIP_EINVAL;
+  const bool vec = width % 8 == 0 && table_row_stride % 8 == 0 && aligned16(table) && aligned16(residual) && aligned16(act);
+  const dim3 grid((unsigned)n_ids), block(256);
+  hipStream_t s = (hipStream_t)stream;
+#define MOPS_EMBED(T, V) hipLaunchKernelGGL((embed_residual_kernel<T, V>), grid, block, 0, s, ids, (const T*)table, table_row_stride, \
+                                            residual, (T*)act, vocab, (int)width)
+  if (dtype == MOPS_HIP_BF16) { if (vec) MOPS_EMBED(bf16_t, 8); else MOPS_EMBED(bf16_t, 1); }
+  else { if (vec) MOPS_EMBED(float, 8); else MOPS_EMBED(float, 1); }
+#undef MOPS_EMBED
+  return finish_launch();
+}
+
+extern "C" int mops_hip_norm_residual_add(float* residual, const void* y, int64_t y_row_stride, const void* weight, float weight_offset,
+                                          float eps, void* act, int dtype, int64_t rows, int64_t n, void* stream) {
+  using namespace mops;
+  if (!known_dtype(dtype) || rows < 0 || n <= 0 || n > (1 << 20) || rows > 0x7fffffffLL) return MOPS_HIP_EINVAL;
+  if (rows == 0) return MOPS_HIP_OK;
+  if (!residual || !y || !weight || !act || y_row_stride < n || y == act) return MOPS_HIP_EINVAL;
+  if (dtype == MOPS_HIP_BF16) launch_norm<bf16_t, 1>(residual, y, y_row_stride, weight, weight_offset, eps, act, rows, n, (hipStream_t)stream);
+  else launch_norm<float, 1>(residual, y, y_row_stride, weight, weight_offset, eps, act, rows, n, (hipStream_t)stream);
+  return finish_launch();
+}
+
+extern "C" int mops_hip_rms_norm_f32(const float* x, const void* weight, float weight_offset, float eps, void* out, int dtype,
+                                     int64_t rows, int64_t n, void* stream) {
+  using namespace mops;
+  if (!known_dtype(dtype) || rows < 0 || n <= 0 || n > (1 << 20) || rows > 0x7fffffffLL) return MOPS_HIP_EINVAL;
+  if (rows == 0) return MOPS_HIP_OK;
+  if (!x || !weight || !out || (const void*)x == out) return MOPS_HIP_EINVAL;
+  float* xr = const_cast<float*>(x);   // mode 0 only reads it
+  if (dtype == MOPS_HIP_BF16) launch_norm<bf16_t, 0>(xr, nullptr, 0, weight, weight_offset, eps, out, rows, n, (hipStream_t)stream);
+  else launch_norm<float, 0>(xr, nullptr, 0, weight, weight_offset, eps, out, rows, n, (hipStream_t)stream);
+  return finish_launch();
+}
+
+extern "C" int mops_hip_gated_group_norm(const void* y, int64_t y_row_stride, const void* gate, int64_t gate_row_stride,
+                                         const void* weight, float eps, int gate_first, void* out, int dtype,
+                                         int64_t rows, int64_t groups, int64_t group_size, void* stream) {
+  using namespace mops;
+  if (!known_dtype(dtype) || rows < 0 || groups <= 0 || group_size <= 0 || groups * group_size > (1 << 24)) return MOPS_HIP_EINVAL;
+  if (rows == 0) return MOPS_HIP_OK;
+  const int64_t n = groups * group_size;
+  if (!y || !gate || !out || y_row_stride < n || gate_row_stride < n || out == gate) return MOPS_HIP_EINVAL;
+  const int64_t wgs = (rows * groups + 3) / 4;
+  if (wgs > 0x7fffffffLL) return MOPS_HIP_EUNSUPPORTED;
+  const bool vec = group_size % 8 == 0 && y_row_stride % 8 == 0 && gate_row_stride % 8 == 0 && aligned16(y) && aligned16(gate) &&
+                   aligned16(out) && (!weight || aligned16(weight));
+  hipStream_t s = (hipStream_t)stream;
+#define MOPS_GGN(T, V, F) hipLaunchKernelGGL((gated_group_norm_kernel<T, V, F>), dim3((unsigned)wgs), dim3(256), 0, s, (const T*)y, \
+                          y_row_stride, (const T*)gate, gate_row_stride, (const T*)weight, eps, (T*)out, rows, (int)groups, (int)group_size)
+#define MOPS_GGN2(T, V) do { if (gate_first) MOPS_GGN(T, V, true); else MOPS_GGN(T, V, false); } while (0)
+  if (dtype == MOPS_HIP_BF16) { if (vec) MOPS_GGN2(bf16_t, 8); else MOPS_GGN2(bf16_t, 1); }
+  else { if (vec) MOPS_GGN2(float, 8); else MOPS_GGN2(float, 1); }
+#undef MOPS_GGN2
+#undef MOPS_GGN
+  return finish_launch();
+}

@@ -1,0 +1,29 @@
+"""Feed-forward sublayers."""
+from __future__ import annotations
+
+from . import hip_op, pack, register_feed_forward, require_size
+
+
+@register_feed_forward("dense")
+class ClampedGLU:
+    """W_down(g * sigmoid(1.702 g) * (u + 1)) with g = min(W_gate x, limit) and u = clamp(W_up x, -limit, limit)."""
+    ALPHA = 1.702
+
+    @staticmethod
+    def validate(sizes):
+        require_size(sizes, "ff")
+        float(sizes["limit"])
+
+    def __init__(self, sizes, weights, prefix, m):
+        self.ff, self.limit = sizes["ff"], float(sizes["limit"])
+        # the halves start at multiples of eight columns
+        self.half = (self.ff + 7) // 8 * 8
+        gate, up = (weights.take(prefix + n, (self.ff, m.width)) for n in ("gate", "up"))
+        self.gate_up = pack([pack([gate]), pack([up])])
+        self.down = weights.take(prefix + "down", (m.width, self.ff))
+        self.linear, self.glu = hip_op("linear"), hip_op("clamped_glu")
+
+    def __call__(self, x):
+        p = self.linear(x, self.gate_up)
+        y = self.glu(p[:, :self.ff], p[:, self.half:self.half + self.ff], self.limit, self.ALPHA)
+        return self.linear(y, self.down)

@@ -31,7 +31,21 @@ OP_NAMES = (
 )
 
 # Operators this backend adds to the reference's eleven; a backend need not provide them.
-EXTENSION_OP_NAMES = ("qk_norm_rope_store",)
+EXTENSION_OP_NAMES = (
+    "qk_norm_rope_store",
+    # recurrent layers, latent attention, float32 residual stream
+    "embed_residual",
+    "norm_residual_add",
+    "rms_norm_f32",
+    "gated_group_norm",
+    "clamped_glu",
+    "decayed_recurrence",
+    "short_conv",
+    "short_conv_update",
+    "latent_prepare",
+    "head_linear",
+    "latent_attention_rows",
+)
 
 
 def rebind(backend: str = None) -> None:

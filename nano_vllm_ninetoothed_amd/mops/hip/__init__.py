@@ -1,1 +1,1 @@
-from . import ops  # noqa: F401
+from . import ops, recurrent_ops  # noqa: F401

@@ -1,0 +1,277 @@
+"""Extension ops of the `hip` backend for models with recurrent layers, latent attention and a float32 residual stream.
+They run in bfloat16 and in float32 (the tensors' dtype decides); the rules of ops.py hold: layouts are checked here with
+exceptions, outputs come from the torch allocator, everything runs on the current stream and nothing synchronises.
+"""
+from __future__ import annotations
+
+from ctypes import byref
+
+import torch
+
+from ... import _capi
+from .ops import _require, _stream
+from .registry import register_hip_op
+
+_DTYPES = {torch.bfloat16: 0, torch.float32: 1}
+
+
+def _dtype(name: str, t: torch.Tensor) -> int:
+    if not t.is_cuda:
+        raise ValueError(f"{name} must live on the GPU")
+    code = _DTYPES.get(t.dtype)
+    if code is None:
+        raise ValueError(f"{name} must be bfloat16 or float32, got {t.dtype}")
+    return code
+
+
+def _rows(name: str, t: torch.Tensor, cols: int, dtype: torch.dtype) -> int:
+    """Checks a 2-D tensor with contiguous rows of `cols` elements; returns its row stride."""
+    if not (t.is_cuda and t.dim() == 2 and t.shape[1] == cols and t.dtype == dtype and (t.stride(1) == 1 or cols == 1)):
+        raise ValueError(f"{name} must be a GPU tensor [rows, {cols}] of {dtype} with contiguous rows, got {tuple(t.shape)} {t.dtype}")
+    return t.stride(0) if t.shape[0] > 1 else max(t.stride(0), cols)
+
+
+def _flat(name: str, t: torch.Tensor, n: int, dtype: torch.dtype) -> int:
+    """Checks a contiguous tensor of n elements; returns its address."""
+    if not (t.is_cuda and t.numel() == n and t.dtype == dtype and t.is_contiguous()):
+        raise ValueError(f"{name} must be a contiguous GPU tensor of {n} x {dtype}, got {tuple(t.shape)} {t.dtype}")
+    return t.data_ptr()
+
+
+@register_hip_op
+def embed_residual(ids: torch.Tensor, table: torch.Tensor):
+    """Embedding rows as (float32 residual, activation copy in the table's dtype)."""
+    code = _dtype("table", table)
+    _require(table.dim() == 2 and table.stride(1) == 1, "table must be [vocab, width] with contiguous rows")
+    _require(ids.is_cuda and ids.dtype == torch.int64 and ids.dim() == 1 and ids.is_contiguous(), "ids must be a contiguous int64 GPU vector")
+    n, (vocab, width) = ids.numel(), table.shape
+    residual = torch.empty((n, width), dtype=torch.float32, device=table.device)
+    act = torch.empty((n, width), dtype=table.dtype, device=table.device)
+    st = _capi.load().mops_hip_embed_residual(ids.data_ptr(), table.data_ptr(), table.stride(0), code, residual.data_ptr(), act.data_ptr(),
+                                              n, vocab, width, _stream(table))
+    _capi.check("mops_hip_embed_residual", st)
+    return residual, act
+
+
+@register_hip_op
+def norm_residual_add(residual: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: float, weight_offset: float = 0.0):
+    """residual += rms(y) * (weight_offset + weight), in place; returns the new residual in y's dtype."""
+    code = _dtype("y", y)
+    rows, n = residual.shape
+    _flat("residual", residual, rows * n, torch.float32)
+    stride = _rows("y", y, n, y.dtype)
+    _require(y.shape[0] == rows, "y must have as many rows as the residual")
+    act = torch.empty((rows, n), dtype=y.dtype, device=y.device)
+    st = _capi.load().mops_hip_norm_residual_add(residual.data_ptr(), y.data_ptr(), stride, _flat("weight", weight, n, y.dtype),
+                                                 float(weight_offset), float(eps), act.data_ptr(), code, rows, n, _stream(y))
+    _capi.check("mops_hip_norm_residual_add", st)
+    return act
+
+
+@register_hip_op
+def rms_norm_f32(x: torch.Tensor, weight: torch.Tensor, eps: float, weight_offset: float = 0.0):
+    """rms(x) * (weight_offset + weight) of float32 rows, in the weight's dtype."""
+    code = _dtype("weight", weight)
+    rows, n = x.shape
+    out = torch.empty((rows, n), dtype=weight.dtype, device=x.device)
+    st = _capi.load().mops_hip_rms_norm_f32(_flat("x", x, rows * n, torch.float32), _flat("weight", weight, n, weight.dtype),
+                                            float(weight_offset), float(eps), out.data_ptr(), code, rows, n, _stream(x))
+    _capi.check("mops_hip_rms_norm_f32", st)
+    return out
+
+
+@register_hip_op
+def gated_group_norm(y: torch.Tensor, gate: torch.Tensor, groups: int, eps: float, weight=None, gate_first: bool = False):
+    """rms over `groups` equal parts of every row, multiplied by silu(gate) before (gate_first) or after the division."""
+    code = _dtype("y", y)
+    rows, n = y.shape
+    _require(groups > 0 and n % groups == 0, "the row must divide into the groups")
+    ys, gs = _rows("y", y, n, y.dtype), _rows("gate", gate, n, y.dtype)
+    _require(gate.shape[0] == rows, "gate must have as many rows as y")
+    out = torch.empty((rows, n), dtype=y.dtype, device=y.device)
+    st = _capi.load().mops_hip_gated_group_norm(y.data_ptr(), ys, gate.data_ptr(), gs, None if weight is None else _flat("weight", weight, n, y.dtype),
+                                                float(eps), 1 if gate_first else 0, out.data_ptr(), code, rows, groups, n // groups, _stream(y))
+    _capi.check("mops_hip_gated_group_norm", st)
+    return out
+
+
+@register_hip_op
+def clamped_glu(gate: torch.Tensor, up: torch.Tensor, limit: float, alpha: float = 1.702):
+    """g * sigmoid(alpha g) * (u + 1) with g = min(gate, limit) and u = clamp(up, -limit, limit)."""
+    code = _dtype("gate", gate)
+    rows, n = gate.shape
+    gs, us = _rows("gate", gate, n, gate.dtype), _rows("up", up, n, gate.dtype)
+    _require(up.shape[0] == rows, "gate and up must have the same shape")
+    out = torch.empty((rows, n), dtype=gate.dtype, device=gate.device)
+    st = _capi.load().mops_hip_clamped_glu(gate.data_ptr(), gs, up.data_ptr(), us, out.data_ptr(), code, rows, n, float(alpha), float(limit),
+                                           _stream(gate))
+    _capi.check("mops_hip_clamped_glu", st)
+    return out
+
+
+def recurrence_state_pitch(d: int) -> int:
+    """Row pitch (elements) of the recurrent state [slots, heads, vd, pitch]."""
+    return _capi.load().mops_hip_recurrence_state_pitch(d)
+
+
+def _recurrence_args(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, *, cu_seqlens=None, decay=None, dt=None,
+                     dt_bias=None, neg_a=None, skip=None, cos_sin=None, k_scale=1.0, conv=None):
+    code = _dtype("v", v)
+    tokens = v.shape[0]
+    batch = state_slots.numel()
+    r = _capi.Recurrence()
+    _require(heads > 0 and groups > 0 and heads % groups == 0, "heads must be a multiple of groups")
+    _require(state.is_cuda and state.dtype == torch.float32 and state.is_contiguous() and state.dim() == 4
+             and tuple(state.shape[1:]) == (heads, vd, recurrence_state_pitch(d)), "state must be float32 [slots, heads, vd, pitch]")
+    r.q_stride, r.k_stride = _rows("q", q, groups * d, v.dtype), _rows("k", k, groups * d, v.dtype)
+    r.v_stride, r.out_stride = _rows("v", v, heads * vd, v.dtype), _rows("out", out, heads * vd, v.dtype)
+    r.q, r.k, r.v, r.out = q.data_ptr(), k.data_ptr(), v.data_ptr(), out.data_ptr()
+    _require(q.shape[0] == k.shape[0] == out.shape[0] == tokens, "q, k, v and out must have the same number of tokens")
+    r.state, r.num_slots = state.data_ptr(), state.shape[0]
+    r.state_slots, r.starts = _flat("state_slots", state_slots, batch, torch.int32), _flat("starts", starts, batch, torch.int32)
+    if cu_seqlens is None:
+        _require(tokens == batch, "without cu_seqlens every sequence brings one token")
+    else:
+        r.cu_seqlens = _flat("cu_seqlens", cu_seqlens, batch + 1, torch.int32)
+    _require((decay is None) != (dt is None), "give either a constant decay or time steps")
+    if decay is not None:
+        r.decay = _flat("decay", decay, heads, torch.float32)
+    else:
+        r.dt, r.dt_stride = dt.data_ptr(), _rows("dt", dt, heads, v.dtype)
+        _require(dt.shape[0] == tokens, "dt must have one row per token")
+        r.dt_bias, r.neg_a = _flat("dt_bias", dt_bias, heads, torch.float32), _flat("neg_a", neg_a, heads, torch.float32)
+    if skip is not None:
+        r.skip = _flat("skip", skip, heads, torch.float32)
+    if cos_sin is not None:
+        r.rot, r.max_positions = cos_sin.shape[1], cos_sin.shape[0]
+        r.cos_sin = _flat("cos_sin", cos_sin, cos_sin.numel(), torch.float32)
+    if conv is not None:
+        weight, bias, ring, (r.q_channel, r.k_channel, r.v_channel) = conv
+        r.taps, r.channels = weight.shape
+        r.conv_weight = _flat("conv weight", weight, weight.numel(), torch.float32)
+        r.conv_bias = _flat("conv bias", bias, weight.shape[1], torch.float32)
+        r.conv_ring = _flat("conv ring", ring, state.shape[0] * weight.numel(), v.dtype)
+    r.batch, r.heads, r.groups, r.d, r.vd = batch, heads, groups, d, vd
+    r.k_scale, r.dtype = float(k_scale), code
+    return r
+
+
+@register_hip_op
+def decayed_recurrence(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, **options):
+    """S <- a S + k (s v)^T, o = S^T q + skip v, token by token with the state of state_slots[b] in float32 (layout and options:
+    mops_hip_recurrence in include/mops_hip.h).  Options: cu_seqlens (None: one token per sequence), decay | dt + dt_bias +
+    neg_a, skip, cos_sin (rotates q and k), k_scale, conv = (weight [taps, channels] float32, bias, ring, (q, k, v channel
+    offsets)).  Writes `out` and the state in place."""
+    r = _recurrence_args(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, **options)
+    st = _capi.load().mops_hip_decayed_recurrence(byref(r), _stream(v))
+    _capi.check("mops_hip_decayed_recurrence", st)
+    return out
+
+
+@register_hip_op
+def short_conv(x, weight, bias, ring, token_seq, cu_seqlens, starts, state_slots):
+    """silu(causal convolution per channel + bias) of packed portions; inputs before a portion come from the ring."""
+    code = _dtype("x", x)
+    tokens, channels = x.shape
+    taps = weight.shape[0]
+    batch = state_slots.numel()
+    stride = _rows("x", x, channels, x.dtype)
+    _require(ring.dim() == 3 and ring.shape[1:] == (taps, channels), "ring must be [slots, taps, channels]")
+    out = torch.empty((tokens, channels), dtype=x.dtype, device=x.device)
+    st = _capi.load().mops_hip_short_conv(x.data_ptr(), stride, _flat("weight", weight, taps * channels, torch.float32),
+                                          _flat("bias", bias, channels, torch.float32), _flat("ring", ring, ring.numel(), x.dtype), ring.shape[0],
+                                          _flat("token_seq", token_seq, tokens, torch.int32), _flat("cu_seqlens", cu_seqlens, batch + 1, torch.int32),
+                                          _flat("starts", starts, batch, torch.int32), _flat("state_slots", state_slots, batch, torch.int32),
+                                          out.data_ptr(), code, tokens, channels, taps, _stream(x))
+    _capi.check("mops_hip_short_conv", st)
+    return out
+
+
+@register_hip_op
+def short_conv_update(x, ring, cu_seqlens, starts, state_slots):
+    """Files the last taps-1 rows of every portion in the ring."""
+    code = _dtype("x", x)
+    channels = x.shape[1]
+    batch = state_slots.numel()
+    stride = _rows("x", x, channels, x.dtype)
+    _require(ring.dim() == 3 and ring.shape[2] == channels, "ring must be [slots, taps, channels]")
+    st = _capi.load().mops_hip_short_conv_update(x.data_ptr(), stride, _flat("ring", ring, ring.numel(), x.dtype), ring.shape[0],
+                                                 _flat("cu_seqlens", cu_seqlens, batch + 1, torch.int32),
+                                                 _flat("starts", starts, batch, torch.int32), _flat("state_slots", state_slots, batch, torch.int32),
+                                                 code, batch, channels, ring.shape[1], _stream(x))
+    _capi.check("mops_hip_short_conv_update", st)
+
+
+def _latent_cache(cache, width, dtype):
+    _require(cache.dim() == 3 and cache.dtype == dtype and cache.is_cuda and cache.is_contiguous() and cache.shape[2] >= width,
+             "the latent cache must be a contiguous [blocks, block_size, pitch] tensor of the activation dtype")
+    return cache.shape
+
+
+@register_hip_op
+def latent_prepare(down, q_weight, kv_weight, eps, cos_sin, positions, slot_mapping, cache, q_rank, kv_rank, rot_dim):
+    """Norms of the query and kv latents, rotation of the shared key part, scatter of the cache rows; returns the query latent."""
+    code = _dtype("down", down)
+    tokens = down.shape[0]
+    _require(down.dim() == 2 and down.shape[1] >= q_rank + kv_rank + rot_dim and down.stride(1) == 1, "down must be [tokens, q_rank + kv_rank + rot_dim]")
+    nblk, bs, pitch = _latent_cache(cache, kv_rank + rot_dim, down.dtype)
+    _require(cos_sin.dim() == 2 and cos_sin.shape[1] == rot_dim, "cos_sin must be [positions, rot_dim]")
+    cq = torch.empty((tokens, q_rank), dtype=down.dtype, device=down.device)
+    st = _capi.load().mops_hip_latent_prepare(down.data_ptr(), down.stride(0) if tokens > 1 else down.shape[1],
+                                              _flat("q_weight", q_weight, q_rank, down.dtype), _flat("kv_weight", kv_weight, kv_rank, down.dtype),
+                                              float(eps), _flat("cos_sin", cos_sin, cos_sin.numel(), torch.float32), cos_sin.shape[0],
+                                              _flat("positions", positions, tokens, torch.int32), _flat("slot_mapping", slot_mapping, tokens, torch.int32),
+                                              cq.data_ptr(), cache.data_ptr(), nblk * bs, pitch, code, tokens, q_rank, kv_rank, rot_dim, _stream(down))
+    _capi.check("mops_hip_latent_prepare", st)
+    return cq
+
+
+@register_hip_op
+def head_linear(x, weight):
+    """y[t, h, :] = weight[h] @ x[t, h, :]; x [tokens, heads, k] (last dimension contiguous), weight [heads, n, k]."""
+    code = _dtype("x", x)
+    tokens, heads, k = x.shape
+    _require(x.stride(2) == 1 or k == 1, "x must have a contiguous last dimension")
+    _require(weight.dim() == 3 and weight.shape[0] == heads and weight.shape[2] == k and weight.is_contiguous() and weight.dtype == x.dtype,
+             "weight must be a contiguous [heads, n, k] tensor of x's dtype")
+    n = weight.shape[1]
+    y = torch.empty((tokens, heads, n), dtype=x.dtype, device=x.device)
+    st = _capi.load().mops_hip_head_linear(x.data_ptr(), x.stride(0), x.stride(1), weight.data_ptr(), y.data_ptr(), heads * n, n, code, tokens,
+                                           heads, n, k, _stream(x))
+    _capi.check("mops_hip_head_linear", st)
+    return y
+
+
+def _latent_rows(q_latent, q_rot, cache, cos_sin, context_lens, block_table, scale, row_seq, out):
+    code = _dtype("q_latent", q_latent)
+    rows, heads, kv_rank = q_latent.shape
+    rot_dim = q_rot.shape[2]
+    _require(q_latent.is_contiguous() and q_rot.shape[:2] == (rows, heads) and q_rot.dtype == q_latent.dtype and q_rot.stride(2) == 1,
+             "q_latent must be contiguous [rows, heads, kv_rank], q_rot [rows, heads, rot_dim]")
+    nblk, bs, pitch = _latent_cache(cache, kv_rank + rot_dim, q_latent.dtype)
+    _require(cos_sin.dim() == 2 and cos_sin.shape[1] == rot_dim, "cos_sin must be [positions, rot_dim]")
+    _require(block_table.dtype == torch.int32 and block_table.is_cuda and block_table.dim() == 2 and block_table.stride(1) == 1
+             and (row_seq is not None or block_table.shape[0] >= rows), "block_table must be an int32 GPU tensor [sequences, blocks]")
+    a = _capi.LatentRows()
+    a.q_latent, a.q_rot, a.q_rot_token_stride, a.q_rot_head_stride = q_latent.data_ptr(), q_rot.data_ptr(), q_rot.stride(0), q_rot.stride(1)
+    a.cache, a.pitch = cache.data_ptr(), pitch
+    a.cos_sin, a.max_positions = _flat("cos_sin", cos_sin, cos_sin.numel(), torch.float32), cos_sin.shape[0]
+    a.row_seq = None if row_seq is None else _flat("row_seq", row_seq, rows, torch.int32)
+    a.context_lens = _flat("context_lens", context_lens, rows, torch.int32)
+    a.block_table, a.max_blocks = block_table.data_ptr(), block_table.shape[1]
+    a.block_table_stride = block_table.stride(0) if block_table.shape[0] > 1 else block_table.shape[1]
+    a.block_size, a.num_blocks = bs, nblk
+    a.out, a.rows, a.heads, a.kv_rank, a.rot_dim = out.data_ptr(), rows, heads, kv_rank, rot_dim
+    a.scale, a.dtype = float(scale), code
+    return a
+
+
+@register_hip_op
+def latent_attention_rows(q_latent, q_rot, cache, cos_sin, context_lens, block_table, scale, row_seq=None):
+    """Attention of single query rows against the paged latent cache, in the latent space; returns [rows, heads, kv_rank].
+    Row r sees the first context_lens[r] tokens of block table row row_seq[r] (r itself without row_seq)."""
+    out = torch.empty_like(q_latent)
+    a = _latent_rows(q_latent, q_rot, cache, cos_sin, context_lens, block_table, scale, row_seq, out)
+    st = _capi.load().mops_hip_latent_attention_rows(byref(a), _stream(q_latent))
+    _capi.check("mops_hip_latent_attention_rows", st)
+    return out
