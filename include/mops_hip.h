@@ -385,7 +385,7 @@ typedef struct {
   float* state;
   int64_t num_slots;
   const int32_t *state_slots, *cu_seqlens, *starts;
-  const float *decay, *neg_a, *dt_bias, *skip, *cos_sin;
+  const float *decay, *log_decay, *neg_a, *dt_bias, *skip, *cos_sin;
   const void* dt;
   int64_t dt_stride;
   int64_t batch, heads, groups, d, vd, rot, max_positions;
@@ -397,6 +397,17 @@ typedef struct {
 } mops_hip_recurrence;
 int64_t mops_hip_recurrence_state_pitch(int64_t d);
 int mops_hip_decayed_recurrence(const mops_hip_recurrence* r, void* stream);
+
+/*
+ * The same for portions of many tokens, 64 tokens at a time on the matrix cores (csrc/decayed_chunks.hip).  bf16 only, no
+ * convolution, cu_seqlens required; a constant decay is read from log_decay (natural logarithms, finite) instead of decay.
+ * segments: int32 [num_segments][3] = (sequence, first token, one past the last); the segments of a sequence are consecutive,
+ * in order, and cover it.  seg_state == NULL: one segment per sequence.  Otherwise seg_state: float [num_segments, heads,
+ * vd, pitch], seg_decay: float [num_segments, heads] are scratch, and seq_segments: int32 [batch + 1] bounds each
+ * sequence's segments.
+ */
+int mops_hip_decayed_chunks(const mops_hip_recurrence* r, const int32_t* segments, int64_t num_segments,
+                            const int32_t* seq_segments, float* seg_state, float* seg_decay, void* stream);
 
 /*
  * out[t, c] = silu(bias[c] + sum over lags l < taps of weight[taps-1-l, c] * x(position - l)[c]) for packed portions.
@@ -448,6 +459,33 @@ typedef struct {
   int dtype;
 } mops_hip_latent_rows;
 int mops_hip_latent_attention_rows(const mops_hip_latent_rows* a, void* stream);
+
+/*
+ * The same on the matrix cores (csrc/latent_decode.hip): bf16, kv_rank <= 512, kv_rank + rot_dim <= 576, block_size a
+ * multiple of 32, pitch a multiple of 8; MOPS_HIP_EUNSUPPORTED otherwise.  workspace: device scratch of at least
+ * mops_hip_latent_decode_workspace_bytes(...), private to the call until it completes.
+ */
+int64_t mops_hip_latent_decode_workspace_bytes(int64_t rows, int64_t heads, int64_t kv_rank, int64_t max_blocks,
+                                               int64_t block_size);
+int mops_hip_latent_decode(const mops_hip_latent_rows* a, void* workspace, int64_t workspace_bytes, void* stream);
+
+/*
+ * Long portions (csrc/latent_prefill.hip), bf16.  latent_gather: row i of c [rows, c_pitch] and kr [rows, kr_pitch] = latent and
+ * key part of token row_pos[i] of sequence row_seq[i] (zeros for row_pos < 0 and in the padding columns).
+ * latent_prefill: q [tokens, heads, dim + rot_dim] (rot_dim part not yet rotated), k [rows, heads * dim], kr [rows, rot_dim],
+ * vt [heads * vdim, rows] (row stride a multiple of 8), out [tokens, heads, vdim] contiguous.
+ * tiles: int32 [num_tiles][5] = (first query token, queries <= 128, position of the first query, first key row, keys of the
+ * context); the key rows of a context start at a multiple of 64 and the rows up to the next multiple of 64 exist.
+ * dim + rot_dim <= 256, vdim <= 256.
+ */
+int mops_hip_latent_gather(const void* cache, int64_t pitch, const int32_t* block_table, int64_t table_stride, int64_t block_size,
+                           int64_t num_blocks, int64_t max_blocks, const int32_t* row_seq, const int32_t* row_pos, void* c,
+                           int64_t c_pitch, void* kr, int64_t kr_pitch, int64_t rows, int64_t kv_rank, int64_t rot_dim,
+                           void* stream);
+int mops_hip_latent_prefill(const void* q, int64_t q_token_stride, int64_t q_head_stride, const void* k, int64_t k_stride,
+                            const void* kr, int64_t kr_stride, const void* vt, int64_t vt_stride, const int32_t* tiles,
+                            int64_t num_tiles, void* out, const float* cos_sin, int64_t max_positions, int64_t heads, int64_t dim,
+                            int64_t rot_dim, int64_t vdim, float scale, void* stream);
 
 #ifdef __cplusplus
 }

@@ -17,7 +17,7 @@ class Recurrence(Structure):
     """mops_hip_recurrence of the header, field by field."""
     _fields_ = ([(n, c_void_p) for n in ("q", "k", "v")] + [(n, c_int64) for n in ("q_stride", "k_stride", "v_stride")]
                 + [("out", c_void_p), ("out_stride", c_int64), ("state", c_void_p), ("num_slots", c_int64)]
-                + [(n, c_void_p) for n in ("state_slots", "cu_seqlens", "starts", "decay", "neg_a", "dt_bias", "skip", "cos_sin", "dt")]
+                + [(n, c_void_p) for n in ("state_slots", "cu_seqlens", "starts", "decay", "log_decay", "neg_a", "dt_bias", "skip", "cos_sin", "dt")]
                 + [(n, c_int64) for n in ("dt_stride", "batch", "heads", "groups", "d", "vd", "rot", "max_positions")]
                 + [(n, c_void_p) for n in ("conv_weight", "conv_bias", "conv_ring")]
                 + [(n, c_int64) for n in ("taps", "channels", "q_channel", "k_channel", "v_channel")]
@@ -82,6 +82,7 @@ SIGNATURES = {
     "mops_hip_clamped_glu": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int, c_int64, c_int64, c_float, c_float, c_void_p]),
     "mops_hip_recurrence_state_pitch": (c_int64, [c_int64]),
     "mops_hip_decayed_recurrence": (c_int, [POINTER(Recurrence), c_void_p]),
+    "mops_hip_decayed_chunks": (c_int, [POINTER(Recurrence), c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p]),
     "mops_hip_short_conv": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p,
                                     c_void_p, c_int, c_int64, c_int64, c_int64, c_void_p]),
     "mops_hip_short_conv_update": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int, c_int64, c_int64,
@@ -91,6 +92,12 @@ SIGNATURES = {
     "mops_hip_head_linear": (c_int, [c_void_p, c_int64, c_int64, c_void_p, c_void_p, c_int64, c_int64, c_int, c_int64, c_int64, c_int64,
                                      c_int64, c_void_p]),
     "mops_hip_latent_attention_rows": (c_int, [POINTER(LatentRows), c_void_p]),
+    "mops_hip_latent_decode_workspace_bytes": (c_int64, [c_int64] * 5),
+    "mops_hip_latent_decode": (c_int, [POINTER(LatentRows), c_void_p, c_int64, c_void_p]),
+    "mops_hip_latent_gather": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int64, c_int64, c_int64, c_void_p, c_void_p, c_void_p,
+                                       c_int64, c_void_p, c_int64, c_int64, c_int64, c_int64, c_void_p]),
+    "mops_hip_latent_prefill": (c_int, [c_void_p, c_int64, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_void_p,
+                                        c_int64, c_void_p, c_void_p, c_int64, c_int64, c_int64, c_int64, c_int64, c_float, c_void_p]),
     "mops_hip_linear_pin_solution": (c_int, [c_int64, c_int64, c_int64, c_int]),
     "mops_hip_linear_tune": (c_int, [c_int64, c_int64, c_int64, c_int64, c_int, c_void_p, c_int64, c_void_p, c_void_p, c_void_p]),
 }

@@ -244,8 +244,8 @@ class Engine:
         return [table[t // bs] * bs + t % bs for t in range(begin, end)]
 
     def _prepare_portions(self, seqs, counts):
-        """Batch of the next counts[i] tokens of seqs[i] behind the num_cached tokens of earlier steps.  Sequences that bring
-        one token come first (the layers' decode kernels take that part of the batch); the order is the caller's duty."""
+        """Batch of the next counts[i] tokens of seqs[i] behind the num_cached tokens of earlier steps.  Layers run single
+        tokens, short and long portions on different kernels, each on a run of the batch: callers sort by count."""
         n_decode = 0
         while n_decode < len(seqs) and counts[n_decode] == 1:
             n_decode += 1
@@ -301,7 +301,7 @@ class Engine:
             q.token_ids.extend(tokens[max(0, len(q) - q.num_cached):])
             self._check_length(q, q.num_cached + len(tokens))
             self.cache.hold(q, q.num_cached + len(tokens))
-        order = sorted(range(len(portions)), key=lambda i: len(portions[i][1]) != 1)      # stable: single tokens first
+        order = sorted(range(len(portions)), key=lambda i: len(portions[i][1]))      # stable
         seqs, counts = [portions[i][0] for i in order], [len(portions[i][1]) for i in order]
         first = {}
         at = 0
@@ -347,8 +347,7 @@ class Engine:
             self.running.append(q)
             batch.append(q)
         if batch:
-            # sequences of one token lead a batch of portions
-            return sorted(batch, key=lambda q: len(q) != 1), True
+            return sorted(batch, key=len), True
         batch = list(self.running)[: self.max_num_seqs]
         for q in batch:   # the token about to be written may open a new block
             self.cache.hold(q, len(q))

@@ -12,6 +12,7 @@ from dataclasses import dataclass
 import torch
 
 from .. import mops
+from ..mops.hip.recurrent_ops import CHUNK_MAX_DIM, recurrence_segments
 
 MIXERS: dict = {}
 FEED_FORWARDS: dict = {}
@@ -73,6 +74,31 @@ class Rotary:
             a = torch.outer(torch.arange(self.max_positions, dtype=torch.float64), float(base) ** (-2.0 * i / dims))
             self._tables[key] = torch.cat((a.cos(), a.sin()), dim=-1).float().to(self.device).contiguous()
         return self._tables[key]
+
+
+class ChunkedRecurrence:
+    """Runs a decayed recurrence over the portions of a batch: in chunks on the matrix cores in bf16, token by token for what
+    those kernels do not cover (float32, head sizes beyond theirs)."""
+
+    def __init__(self, heads, groups, d, vd, dtype):
+        self.sizes = (heads, groups, d, vd)
+        self.chunked = dtype == torch.bfloat16 and d <= CHUNK_MAX_DIM
+        self.recurrence, self.chunks = hip_op("decayed_recurrence"), hip_op("decayed_chunks")
+
+    def __call__(self, q, k, v, out, state, ctx, **options):
+        """q, k, v, out: the rows of the portions.  The cut into segments is shared by the layers of a step."""
+        heads, _, _, vd = self.sizes
+        nd = ctx["n_decode"]
+        slots, starts, cu = ctx["state_slots"][nd:], ctx["starts"][nd:], ctx["portion_cu"]
+        if not self.chunked:
+            return self.recurrence(q, k, v, out, state, slots, starts, *self.sizes, cu_seqlens=cu, **options)
+        cuts = ctx.setdefault("segment_cuts", {})
+        key = (heads, vd)
+        if key not in cuts:
+            segments, bounds = recurrence_segments(ctx["seq_counts"][nd:], heads, vd)
+            flat = torch.tensor([x for s in segments for x in s] + bounds, dtype=torch.int32).to(v.device, non_blocking=True)
+            cuts[key] = (flat[:3 * len(segments)].view(-1, 3), flat[3 * len(segments):])
+        return self.chunks(q, k, v, out, state, slots, starts, *self.sizes, *cuts[key], cu_seqlens=cu, **options)
 
 
 def hip_op(name):

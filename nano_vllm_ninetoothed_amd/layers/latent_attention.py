@@ -5,6 +5,9 @@ from __future__ import annotations
 import torch
 
 from . import hip_op, pack, register_mixer, require_size
+from ..mops.hip.recurrent_ops import latent_decode_covers, latent_prefill_covers, latent_prefill_plan
+
+EXPAND_FROM = 64     # portions of at least this many tokens expand keys and values instead of absorbing the projections
 
 
 @register_mixer("latent_attention")
@@ -33,7 +36,14 @@ class LatentAttention:
         self.pages = m.cache.paged((kr + r + 7) // 8 * 8, dtype=m.dtype)
         self.cos_sin = m.rotary.table(sizes["rot"]["base"], r)
         self.linear, self.prepare, self.head_linear = hip_op("linear"), hip_op("latent_prepare"), hip_op("head_linear")
-        self.rows = hip_op("latent_attention_rows")
+        self.rows = hip_op("latent_decode" if latent_decode_covers(m.dtype, kr, r, m.cache.block_size) else "latent_attention_rows")
+        self.expands = latent_prefill_covers(m.dtype, d, r, v)
+        if self.expands:
+            # the expansion reads gathered latents whose row length is a multiple of eight
+            pad = -kr % 8
+            self.w_k = pack([torch.nn.functional.pad(uk, (0, pad))])
+            self.w_v = torch.nn.functional.pad(uv, (0, pad)).contiguous()
+            self.gather, self.prefill = hip_op("latent_gather"), hip_op("latent_prefill")
 
     def __call__(self, x, ctx):
         h, d, r, v = self.heads, self.dim, self.rot_dim, self.vdim
@@ -42,7 +52,15 @@ class LatentAttention:
         cq = self.prepare(down, self.q_norm, self.kv_norm, self.eps, self.cos_sin, ctx["positions32"], ctx["slot_mapping"], self.pages,
                           self.q_rank, self.kv_rank, r)
         q = self.linear(cq, self.uq)[:, :h * (d + r)].unflatten(1, (h, d + r))
-        o = self._absorbed(q, ctx["token_context"], ctx["token_seq"], ctx)
+        plan = self._plan(ctx, x.device) if self.expands else None
+        if plan is None:
+            o = self._absorbed(q, ctx["token_context"], ctx["token_seq"], ctx)
+        else:
+            first = plan[0]
+            o = torch.empty((t, h, v), dtype=x.dtype, device=x.device)
+            if first:
+                o[:first] = self._absorbed(q[:first], ctx["token_context"][:first], ctx["token_seq"][:first], ctx)
+            self._expanded(q, plan, ctx, o)
         return self.linear(o.reshape(t, h * v), self.o)
 
     def _absorbed(self, q, context_lens, row_seq, ctx):
@@ -50,3 +68,29 @@ class LatentAttention:
         q_latent = self.head_linear(q[..., :self.dim], self.q_to_latent)
         o = self.rows(q_latent, q[..., self.dim:], self.pages, self.cos_sin, context_lens, ctx["block_tables"], self.scale, row_seq)
         return self.head_linear(o, self.latent_to_v)
+
+    def _plan(self, ctx, device):
+        """(first token row, row_seq, row_pos, tiles) of the batch's long portions, which come last; None without any.
+        Shared by the layers of a step."""
+        if not ctx["is_prefill"]:
+            return None
+        if "latent_plan" not in ctx:
+            counts, starts = ctx["seq_counts"], ctx["seq_starts"]
+            i = next((i for i, n in enumerate(counts) if n >= EXPAND_FROM), len(counts))
+            plan = None
+            if i < len(counts):
+                first = sum(counts[:i])
+                row_seq, row_pos, tiles = latent_prefill_plan(counts[i:], starts[i:], first, i)
+                n = len(row_pos)
+                flat = torch.tensor(row_seq + row_pos + [x for t in tiles for x in t], dtype=torch.int32).to(device, non_blocking=True)
+                plan = (first, flat[:n], flat[n:2 * n], flat[2 * n:].view(-1, 5))
+            ctx["latent_plan"] = plan
+        return ctx["latent_plan"]
+
+    def _expanded(self, q, plan, ctx, out):
+        """Long portions: keys and values of the whole context are expanded once, then ordinary attention."""
+        _, row_seq, row_pos, tiles = plan
+        c, kr = self.gather(self.pages, ctx["block_tables"], row_seq, row_pos, self.kv_rank, self.rot_dim)
+        k = self.linear(c, self.w_k)
+        vt = self.linear(self.w_v, c)
+        self.prefill(q, k, kr, vt, tiles, self.cos_sin, self.scale, self.dim, self.rot_dim, self.vdim, out)

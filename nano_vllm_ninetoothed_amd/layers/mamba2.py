@@ -3,7 +3,7 @@ from __future__ import annotations
 
 import torch
 
-from . import hip_op, pack, register_mixer, require_size
+from . import ChunkedRecurrence, hip_op, pack, register_mixer, require_size
 from ..mops.hip.recurrent_ops import recurrence_state_pitch
 
 
@@ -36,6 +36,7 @@ class Mamba2:
         self.o = take(prefix + "o", (m.width, inner))
         self.state = m.cache.per_slot(h, v, recurrence_state_pitch(n))
         self.ring = m.cache.per_slot(self.taps, ch, dtype=m.dtype)
+        self.portions = ChunkedRecurrence(h, g, n, v, m.dtype)
         self.linear, self.recurrence, self.group_norm = hip_op("linear"), hip_op("decayed_recurrence"), hip_op("gated_group_norm")
         self.conv, self.conv_update = hip_op("short_conv"), hip_op("short_conv_update")
 
@@ -45,7 +46,7 @@ class Mamba2:
         z, xbc, dt = p[:, :inner], p[:, inner:inner + ch], p[:, inner + ch:inner + ch + h]
         y = torch.empty((x.shape[0], inner), dtype=x.dtype, device=x.device)
         nd = ctx["n_decode"]
-        slots, starts, cu = ctx["state_slots"], ctx["starts"], ctx["cu_seqlens"]
+        slots, starts = ctx["state_slots"], ctx["starts"]
         opts = dict(dt_bias=self.dt_bias, neg_a=self.neg_a, skip=self.skip)
 
         def parts(t):
@@ -58,7 +59,7 @@ class Mamba2:
         if nd < slots.numel():
             c = self.conv(xbc[nd:], self.conv_w, self.conv_b, self.ring, ctx["portion_token_seq"], ctx["portion_cu"], starts[nd:], slots[nd:])
             q, k, vv = parts(c)
-            self.recurrence(q, k, vv, y[nd:], self.state, slots[nd:], starts[nd:], h, g, n, v, dt=dt[nd:], cu_seqlens=ctx["portion_cu"], **opts)
+            self.portions(q, k, vv, y[nd:], self.state, ctx, dt=dt[nd:], **opts)
             self.conv_update(xbc[nd:], self.ring, ctx["portion_cu"], starts[nd:], slots[nd:])
         y = self.group_norm(y, z, self.norm_groups, self.eps, weight=self.norm, gate_first=True)
         return self.linear(y, self.o)

@@ -5,7 +5,7 @@ import math
 
 import torch
 
-from . import hip_op, pack, register_mixer, require_size
+from . import ChunkedRecurrence, hip_op, pack, register_mixer, require_size
 from ..mops.hip.recurrent_ops import recurrence_state_pitch
 
 
@@ -38,6 +38,7 @@ class Retention:
         self.cos_sin = m.rotary.table(sizes["rot"]["base"], sizes["rot"]["dims"]) if sizes["rot"]["dims"] else None
         self.k_scale = d ** -0.5
         self.state = m.cache.per_slot(h, v, recurrence_state_pitch(d))
+        self.portions = ChunkedRecurrence(h, h, d, v, m.dtype)
         self.linear, self.recurrence, self.group_norm = hip_op("linear"), hip_op("decayed_recurrence"), hip_op("gated_group_norm")
 
     def __call__(self, x, ctx):
@@ -47,9 +48,9 @@ class Retention:
         o = torch.empty((x.shape[0], h * v), dtype=x.dtype, device=x.device)
         nd = ctx["n_decode"]
         slots, starts = ctx["state_slots"], ctx["starts"]
-        opts = dict(decay=self.decay, cos_sin=self.cos_sin, k_scale=self.k_scale)
+        opts = dict(decay=self.decay, log_decay=self.log_decay, cos_sin=self.cos_sin, k_scale=self.k_scale)
         if nd:
             self.recurrence(q[:nd], k[:nd], vv[:nd], o[:nd], self.state, slots[:nd], starts[:nd], h, h, d, v, **opts)
         if nd < slots.numel():
-            self.recurrence(q, k, vv, o, self.state, slots[nd:], starts[nd:], h, h, d, v, cu_seqlens=ctx["cu_seqlens"][nd:], **opts)
+            self.portions(q[nd:], k[nd:], vv[nd:], o[nd:], self.state, ctx, **opts)
         return self.linear(self.group_norm(o, gate, h, self.eps), self.o)

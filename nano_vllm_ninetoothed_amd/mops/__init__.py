@@ -40,11 +40,15 @@ EXTENSION_OP_NAMES = (
     "gated_group_norm",
     "clamped_glu",
     "decayed_recurrence",
+    "decayed_chunks",
     "short_conv",
     "short_conv_update",
     "latent_prepare",
     "head_linear",
     "latent_attention_rows",
+    "latent_decode",
+    "latent_gather",
+    "latent_prefill",
 )
 
 

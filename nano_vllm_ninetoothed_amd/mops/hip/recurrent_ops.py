@@ -114,7 +114,7 @@ def recurrence_state_pitch(d: int) -> int:
     return _capi.load().mops_hip_recurrence_state_pitch(d)
 
 
-def _recurrence_args(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, *, cu_seqlens=None, decay=None, dt=None,
+def _recurrence_args(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, *, cu_seqlens=None, decay=None, log_decay=None, dt=None,
                      dt_bias=None, neg_a=None, skip=None, cos_sin=None, k_scale=1.0, conv=None):
     code = _dtype("v", v)
     tokens = v.shape[0]
@@ -136,6 +136,8 @@ def _recurrence_args(q, k, v, out, state, state_slots, starts, heads, groups, d,
     _require((decay is None) != (dt is None), "give either a constant decay or time steps")
     if decay is not None:
         r.decay = _flat("decay", decay, heads, torch.float32)
+        if log_decay is not None:
+            r.log_decay = _flat("log_decay", log_decay, heads, torch.float32)
     else:
         r.dt, r.dt_stride = dt.data_ptr(), _rows("dt", dt, heads, v.dtype)
         _require(dt.shape[0] == tokens, "dt must have one row per token")
@@ -165,6 +167,44 @@ def decayed_recurrence(q, k, v, out, state, state_slots, starts, heads, groups, 
     r = _recurrence_args(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, **options)
     st = _capi.load().mops_hip_decayed_recurrence(byref(r), _stream(v))
     _capi.check("mops_hip_decayed_recurrence", st)
+    return out
+
+
+CHUNK_MAX_DIM = 256       # head sizes (d) the chunked kernels cover
+
+
+def recurrence_segments(counts, heads: int, vd: int, wanted: int = 768):
+    """Cuts portions of counts[i] tokens (packed one behind the other) into segments for decayed_chunks: one per portion if
+    those give enough workgroups, else about `wanted` workgroups in all.  Returns host lists (segments, bounds per portion)."""
+    lanes = heads * ((vd + 63) // 64)
+    length = max(counts)
+    if len(counts) * lanes < wanted // 2 and length > 256:
+        length = max(128, -(-sum(counts) * lanes // wanted // 64) * 64)
+    segments, bounds, at = [], [0], 0
+    for i, n in enumerate(counts):
+        for begin in range(0, n, length):
+            segments.append((i, at + begin, at + min(n, begin + length)))
+        bounds.append(len(segments))
+        at += n
+    return segments, bounds
+
+
+@register_hip_op
+def decayed_chunks(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, segments, seq_segments, **options):
+    """decayed_recurrence for packed portions of many tokens, on the matrix cores (bf16).  segments [n, 3] and seq_segments
+    [sequences + 1] are the int32 device copies of what recurrence_segments returns; cu_seqlens is required."""
+    r = _recurrence_args(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, **options)
+    n = segments.shape[0]
+    _require(r.batch == seq_segments.numel() - 1, "seq_segments must bound the segments of every sequence")
+    seg_state = seg_decay = None
+    if n > r.batch:
+        seg_state = torch.empty((n, heads, vd, state.shape[3]), dtype=torch.float32, device=v.device)
+        seg_decay = torch.empty((n, heads), dtype=torch.float32, device=v.device)
+    st = _capi.load().mops_hip_decayed_chunks(byref(r), _flat("segments", segments, 3 * n, torch.int32), n,
+                                              _flat("seq_segments", seq_segments, r.batch + 1, torch.int32),
+                                              None if seg_state is None else seg_state.data_ptr(),
+                                              None if seg_decay is None else seg_decay.data_ptr(), _stream(v))
+    _capi.check("mops_hip_decayed_chunks", st)
     return out
 
 
@@ -269,9 +309,92 @@ def _latent_rows(q_latent, q_rot, cache, cos_sin, context_lens, block_table, sca
 @register_hip_op
 def latent_attention_rows(q_latent, q_rot, cache, cos_sin, context_lens, block_table, scale, row_seq=None):
     """Attention of single query rows against the paged latent cache, in the latent space; returns [rows, heads, kv_rank].
-    Row r sees the first context_lens[r] tokens of block table row row_seq[r] (r itself without row_seq)."""
+    Row r sees the first context_lens[r] tokens of block table row row_seq[r] (r itself without row_seq).  The plain form:
+    any size, bf16 or float32; latent_decode is the one on the matrix cores."""
     out = torch.empty_like(q_latent)
     a = _latent_rows(q_latent, q_rot, cache, cos_sin, context_lens, block_table, scale, row_seq, out)
     st = _capi.load().mops_hip_latent_attention_rows(byref(a), _stream(q_latent))
     _capi.check("mops_hip_latent_attention_rows", st)
+    return out
+
+
+def latent_decode_covers(dtype, kv_rank: int, rot_dim: int, block_size: int) -> bool:
+    return dtype == torch.bfloat16 and kv_rank <= 512 and kv_rank + rot_dim <= 576 and block_size % 32 == 0
+
+
+@register_hip_op
+def latent_decode(q_latent, q_rot, cache, cos_sin, context_lens, block_table, scale, row_seq=None):
+    """latent_attention_rows on the matrix cores (sizes: latent_decode_covers)."""
+    out = torch.empty_like(q_latent)
+    a = _latent_rows(q_latent, q_rot, cache, cos_sin, context_lens, block_table, scale, row_seq, out)
+    lib = _capi.load()
+    nbytes = lib.mops_hip_latent_decode_workspace_bytes(a.rows, a.heads, a.kv_rank, a.max_blocks, a.block_size)
+    ws = torch.empty(max(nbytes, 16), dtype=torch.uint8, device=out.device)
+    st = lib.mops_hip_latent_decode(byref(a), ws.data_ptr(), ws.numel(), _stream(q_latent))
+    _capi.check("mops_hip_latent_decode", st)
+    return out
+
+
+def latent_prefill_covers(dtype, dim: int, rot_dim: int, vdim: int) -> bool:
+    return dtype == torch.bfloat16 and dim + rot_dim <= 256 and vdim <= 256
+
+
+PREFILL_QUERIES, PREFILL_KEYS = 128, 64
+
+
+def latent_prefill_plan(counts, starts, first_token: int, first_seq: int):
+    """Host lists for latent_gather and latent_prefill: portions of counts[i] tokens at positions starts[i].., packed from token
+    row first_token on; sequence i of the list is block table row first_seq + i.  Returns (row_seq, row_pos, tiles)."""
+    row_seq, row_pos, tiles = [], [], []
+    at = first_token
+    for i, (n, start) in enumerate(zip(counts, starts)):
+        keys, base = start + n, len(row_pos)
+        pad = -keys % PREFILL_KEYS
+        row_seq += [first_seq + i] * (keys + pad)
+        row_pos += list(range(keys)) + [-1] * pad
+        for q in range(0, n, PREFILL_QUERIES):
+            tiles.append((at + q, min(PREFILL_QUERIES, n - q), start + q, base, keys))
+        at += n
+    tiles.sort(key=lambda t: -(t[1] + t[2]))      # the longest first: they bound the launch
+    return row_seq, row_pos, tiles
+
+
+@register_hip_op
+def latent_gather(cache, block_table, row_seq, row_pos, kv_rank, rot_dim):
+    """Latent rows and key parts of whole contexts out of the pages: (c [rows, kv_rank], kr [rows, rot_dim]), row strides
+    multiples of eight."""
+    nblk, bs, pitch = _latent_cache(cache, kv_rank + rot_dim, torch.bfloat16)
+    rows = row_pos.numel()
+    _require(block_table.dtype == torch.int32 and block_table.is_cuda and block_table.dim() == 2 and block_table.stride(1) == 1,
+             "block_table must be an int32 GPU tensor [sequences, blocks]")
+    c = torch.empty((rows, (kv_rank + 7) // 8 * 8), dtype=cache.dtype, device=cache.device)
+    kr = torch.empty((rows, (rot_dim + 7) // 8 * 8), dtype=cache.dtype, device=cache.device)
+    st = _capi.load().mops_hip_latent_gather(cache.data_ptr(), pitch, block_table.data_ptr(),
+                                             block_table.stride(0) if block_table.shape[0] > 1 else block_table.shape[1], bs, nblk,
+                                             block_table.shape[1], _flat("row_seq", row_seq, rows, torch.int32),
+                                             _flat("row_pos", row_pos, rows, torch.int32), c.data_ptr(), c.shape[1], kr.data_ptr(), kr.shape[1],
+                                             rows, kv_rank, rot_dim, _stream(cache))
+    _capi.check("mops_hip_latent_gather", st)
+    return c, kr
+
+
+@register_hip_op
+def latent_prefill(q, k, kr, vt, tiles, cos_sin, scale, dim, rot_dim, vdim, out):
+    """Causal attention of long portions over expanded keys and values (layout: mops_hip_latent_prefill); writes the portions'
+    rows of out [tokens, heads, vdim]."""
+    _require(q.dim() == 3 and q.dtype == torch.bfloat16 and q.is_cuda and q.stride(2) == 1 and q.shape[2] == dim + rot_dim,
+             "q must be [tokens, heads, dim + rot_dim] in bfloat16")
+    heads = q.shape[1]
+    _require(out.shape == (q.shape[0], heads, vdim) and out.is_contiguous() and out.dtype == q.dtype, "out must be contiguous [tokens, heads, vdim]")
+    rows = k.shape[0]
+    _require(k.shape[1] >= heads * dim and k.stride(1) == 1 and kr.shape[0] == rows and kr.stride(1) == 1 and kr.shape[1] >= rot_dim
+             and vt.shape == (heads * vdim, rows) and vt.stride(1) == 1 and k.dtype == kr.dtype == vt.dtype == q.dtype
+             and rows % PREFILL_KEYS == 0, "k [rows, heads * dim], kr [rows, rot_dim], vt [heads * vdim, rows], rows a multiple of 64")
+    _require(cos_sin.dim() == 2 and cos_sin.shape[1] == rot_dim, "cos_sin must be [positions, rot_dim]")
+    n = tiles.shape[0]
+    st = _capi.load().mops_hip_latent_prefill(q.data_ptr(), q.stride(0), q.stride(1), k.data_ptr(), k.stride(0), kr.data_ptr(), kr.stride(0),
+                                              vt.data_ptr(), vt.stride(0), _flat("tiles", tiles, 5 * n, torch.int32), n, out.data_ptr(),
+                                              _flat("cos_sin", cos_sin, cos_sin.numel(), torch.float32), cos_sin.shape[0], heads, dim, rot_dim,
+                                              vdim, float(scale), _stream(q))
+    _capi.check("mops_hip_latent_prefill", st)
     return out
