@@ -6,9 +6,40 @@ Weights come as a dict of tensors under the checkpoint's names, the configuratio
 """
 from __future__ import annotations
 
+import contextlib
 import math
 
 import torch
+
+_round = None      # see sixteen_bit_products
+
+
+@contextlib.contextmanager
+def sixteen_bit_products(seed=0):
+    """Inside, every matrix product takes and gives values rounded to bfloat16 (to nearest for seed 0, else stochastically):
+    what rounding alone does to the result of a 16-bit run."""
+    global _round
+    g = torch.Generator().manual_seed(seed)
+
+    def nearest(x):
+        return x.to(torch.bfloat16).to(x.dtype)
+
+    def stochastic(x):
+        step = torch.exp2(torch.floor(torch.log2(x.abs().clamp(min=1e-30))) - 7)
+        return nearest(x + (torch.rand(x.shape, generator=g, dtype=x.dtype) - 0.5) * step)
+
+    _round = stochastic if seed else nearest
+    try:
+        yield
+    finally:
+        _round = None
+
+
+def product(x, w):
+    """x W^T"""
+    if _round is None:
+        return x @ w.T
+    return _round(_round(x) @ w.T)
 
 
 def rms(x, eps):
@@ -69,15 +100,15 @@ def retention(h, w, m, eps, positions, state=None):
     """Returns (output [T, width], final state).  w: the mixer's tensors by their short names."""
     H, D, V = m["heads"], m["dim"], m["vdim"]
     T = h.shape[0]
-    q = (h @ w["q"].T).view(T, H, D)
-    k = (h @ w["k"].T).view(T, H, D)
-    v = (h @ w["v"].T).view(T, H, V)
+    q = product(h, w["q"]).view(T, H, D)
+    k = product(h, w["k"]).view(T, H, D)
+    v = product(h, w["v"]).view(T, H, V)
     q = rotate_half(q, positions, m["rot"]["base"], m["rot"]["dims"])
     k = rotate_half(k, positions, m["rot"]["base"], m["rot"]["dims"]) * D ** -0.5
     decay = torch.tensor(m["decay"], dtype=h.dtype)[None, :].expand(T, H)
     o, S = decayed_recurrence(q, k, v, decay, state)
     o = rms(o, eps).reshape(T, H * V)
-    return (o * silu(h @ w["g"].T)) @ w["o"].T, S
+    return product(o * silu(product(h, w["g"])), w["o"]), S
 
 
 def causal_conv(x, kernel, bias, before=None):
@@ -99,7 +130,7 @@ def mamba2(h, w, m, eps, positions, state=None):
     H, V, N, G = m["heads"], m["vdim"], m["state"], m["groups"]
     inner = H * V
     T = h.shape[0]
-    p = h @ w["in"].T
+    p = product(h, w["in"])
     z, xbc, dt = p[:, :inner], p[:, inner: 2 * inner + 2 * G * N], p[:, 2 * inner + 2 * G * N:]
     xbc = silu(causal_conv(xbc, w["conv"], w["conv.b"]))
     x = xbc[:, :inner].reshape(T, H, V)
@@ -110,31 +141,31 @@ def mamba2(h, w, m, eps, positions, state=None):
     y, S = decayed_recurrence(C, B, x * dt[:, :, None], decay, state)
     y = (y + w["D"][None, :, None] * x).reshape(T, inner)
     y = group_rms(y * silu(z), m["norm_groups"], eps) * w["norm"]
-    return y @ w["o"].T, S
+    return product(y, w["o"]), S
 
 
 def latent_attention(h, w, m, eps, positions, state=None):
     H, D, R, V, K = m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"]
     T = h.shape[0]
-    cq = rms(h @ w["dq"].T, eps) * w["dq.norm"]
-    q = (cq @ w["uq"].T).view(T, H, D + R)
-    down = h @ w["dkv"].T
+    cq = rms(product(h, w["dq"]), eps) * w["dq.norm"]
+    q = product(cq, w["uq"]).view(T, H, D + R)
+    down = product(h, w["dkv"])
     c = rms(down[:, :K], eps) * w["dkv.norm"]
     kr = rotate_interleaved(down[:, None, K:], positions, m["rot"]["base"], m["rot"]["dims"])[:, 0]
     qr = rotate_interleaved(q[..., D:], positions, m["rot"]["base"], m["rot"]["dims"])
-    ku = (c @ w["uk"].T).view(T, H, D)
-    v = (c @ w["uv"].T).view(T, H, V)
+    ku = product(c, w["uk"]).view(T, H, D)
+    v = product(c, w["uv"]).view(T, H, V)
     s = (torch.einsum("ihd,jhd->hij", q[..., :D], ku) + torch.einsum("ihd,jd->hij", qr, kr)) * m["scale"]
     s = s.masked_fill(~torch.ones((T, T), dtype=torch.bool).tril(), -math.inf)
     p = torch.exp(s - s.max(dim=-1, keepdim=True).values)
     p = p / p.sum(dim=-1, keepdim=True)
-    return torch.einsum("hij,jhd->ihd", p, v).reshape(T, H * V) @ w["o"].T, None
+    return product(torch.einsum("hij,jhd->ihd", p, v).reshape(T, H * V), w["o"]), None
 
 
 def dense_ff(h, w, m):
-    g = torch.clamp(h @ w["gate"].T, max=m["limit"])
-    u = torch.clamp(h @ w["up"].T, min=-m["limit"], max=m["limit"])
-    return (g / (1 + torch.exp(-1.702 * g)) * (u + 1)) @ w["down"].T
+    g = torch.clamp(product(h, w["gate"]), max=m["limit"])
+    u = torch.clamp(product(h, w["up"]), min=-m["limit"], max=m["limit"])
+    return product(g / (1 + torch.exp(-1.702 * g)) * (u + 1), w["down"])
 
 
 MIXERS = {"retention": retention, "mamba2": mamba2, "latent_attention": latent_attention}
@@ -160,7 +191,7 @@ def forward(config, weights, tokens, dtype=torch.float64, layers_out=None):
         if layers_out is not None:
             layers_out.append(x.clone())
     x = norm_unit_offset(x, weights["final.norm"].to(dtype), eps)
-    return x @ weights["embed"].to(dtype).T
+    return product(x, weights["embed"].to(dtype))
 
 
 def greedy(config, weights, prompt, n, dtype=torch.float64):
