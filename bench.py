@@ -9,6 +9,9 @@ A step is one flash_attn_with_kvcache call over the whole batch, KV cache reside
   e2e  = end-to-end generation on a randomly initialised Qwen3-0.6B-shaped model through the engine
          counterpart (256 random-token prompts of 100..1024 tokens, 100..1024 output tokens each,
          temperature 0.6, no EOS): output tokens per second; --steps/--warmup are ignored.
+  nepulix = prefill and decode throughput of Nepulix models with layers of real sizes beside Qwen3 models of equal size, and
+         every kernel of that design beside the like kernel of the Qwen3 path (--nepulix-part, --nepulix-sizes choose);
+         the line's value is the decode throughput of the last size at the largest batch.
   copy = a plain 1 GiB device-to-device tensor copy (not a mops op): the known-size kernel against which
          the FETCH_SIZE / WRITE_SIZE counters of a profile are calibrated.
   launch_floor = an empty kernel: the floor under the durations of the small operators (value 0, read the time).
@@ -57,10 +60,12 @@ def parse_args():
     ap.add_argument("--steps", type=int, default=None, help="timed steps (default 50; 500 for the prefill ops)")
     ap.add_argument("--warmup", type=int, default=None, help="untimed warm-up steps (default 10; 300 for the prefill ops)")
     ap.add_argument("--op", default="decode",
-                    choices=["decode", "decode8b", "prefill", "prefill_long", "prefix_prefill", "prefix_prefill_short", "store", "silu", "sampler", "qk_rope_store", "add_rms", "rms", "embedding", "copy", "launch_floor", "e2e"])
+                    choices=["decode", "decode8b", "prefill", "prefill_long", "prefix_prefill", "prefix_prefill_short", "store", "silu", "sampler", "qk_rope_store", "add_rms", "rms", "embedding", "copy", "launch_floor", "e2e", "nepulix"])
     ap.add_argument("--e2e-seqs", type=int, default=256, help="number of prompts of the e2e workload")
     ap.add_argument("--e2e-eager", action="store_true", help="e2e: no HIP-graph replay of the decode step")
     ap.add_argument("--e2e-stepwise", action="store_true", help="e2e: read every step's tokens back before the next step, as the reference does")
+    ap.add_argument("--nepulix-part", default="all", choices=["all", "models", "kernels"], help="nepulix: throughput of whole models, kernels, or both")
+    ap.add_argument("--nepulix-sizes", default="", help="nepulix: sizes to run, with commas between them (default: all)")
     ap.add_argument("--no-cpu-baseline", action="store_true")
     ap.add_argument("--no-e2e", action="store_true", help="default op only: skip the end-to-end block of the line (profiling runs)")
     ap.add_argument("--seed", type=int, default=0)
@@ -163,6 +168,28 @@ def run_e2e(args, torch, dev, mops):
     print(json.dumps(out))
 
 
+def run_nepulix(args, torch, dev):
+    """`--op nepulix`: throughput of the models and the table of kernels, in one line."""
+    from nano_vllm_ninetoothed_amd import bench_layers as B
+    from nano_vllm_ninetoothed_amd.models.nepulix import NepulixConfig
+    out = {"metric": "nepulix_decode_tok_per_s", "value": None, "unit": "tok/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
+           "ms_per_step": None, "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+           "config": {"model": "Nepulix, random weights, beside Qwen3 of equal width, depth, feed-forward and vocabulary"}}
+    if args.nepulix_part != "kernels":
+        out["models"] = {}
+        for name, (cfg, qwen) in B.sizes().items():
+            if args.nepulix_sizes and name not in args.nepulix_sizes.split(","):
+                continue
+            out["models"][name] = {"nepulix": B.model_throughput(NepulixConfig.from_dict(cfg), args.seed, steps=args.steps, warmup=args.warmup),
+                                   "qwen3": B.model_throughput(qwen, args.seed, steps=args.steps, warmup=args.warmup)}
+            last = out["models"][name]["nepulix"]["decode"][-1]
+            out.update(value=last["tok_per_s"], ms_per_step=last["ms"])
+            out["config"].update(size=name, global_batch=last["batch"], seq_len=last["context"])
+    if args.nepulix_part != "models":
+        out["kernels"] = B.kernel_table(dev, args.seed)
+    print(json.dumps(out))
+
+
 def main():
     args = parse_args()
     if args.gpus != 1:
@@ -201,6 +228,9 @@ def main():
 
     if args.op == "e2e":
         run_e2e(args, torch, dev, mops)
+        return
+    if args.op == "nepulix":
+        run_nepulix(args, torch, dev)
         return
     bound = "hbm"
     dtype = "bf16"
