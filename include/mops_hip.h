@@ -472,8 +472,9 @@ int mops_hip_latent_decode(const mops_hip_latent_rows* a, void* workspace, int64
 /*
  * Long portions (csrc/latent_prefill.hip), bf16.  latent_gather: row i of c [rows, c_pitch] and kr [rows, kr_pitch] = latent and
  * key part of token row_pos[i] of sequence row_seq[i] (zeros for row_pos < 0 and in the padding columns).
- * latent_prefill: q [tokens, heads, dim + rot_dim] (rot_dim part not yet rotated), k [rows, heads * dim], kr [rows, rot_dim],
- * vt [heads * vdim, rows] (row stride a multiple of 8), out [tokens, heads, vdim] contiguous.
+ * rotate_pairs: x [tokens, heads, rot], pairs (2i, 2i+1) rotated in place by row positions[t] of cos_sin.
+ * latent_prefill: q [tokens, heads, dim + rot_dim] (rotated), k [rows, heads * dim], kr [rows, rot_dim], vt [heads * vdim, rows],
+ * out [tokens, heads, vdim] contiguous; dim, rot_dim and all strides of the inputs are multiples of 8 (pad with zeros).
  * tiles: int32 [num_tiles][5] = (first query token, queries <= 128, position of the first query, first key row, keys of the
  * context); the key rows of a context start at a multiple of 64 and the rows up to the next multiple of 64 exist.
  * dim + rot_dim <= 256, vdim <= 256.
@@ -482,10 +483,12 @@ int mops_hip_latent_gather(const void* cache, int64_t pitch, const int32_t* bloc
                            int64_t num_blocks, int64_t max_blocks, const int32_t* row_seq, const int32_t* row_pos, void* c,
                            int64_t c_pitch, void* kr, int64_t kr_pitch, int64_t rows, int64_t kv_rank, int64_t rot_dim,
                            void* stream);
+int mops_hip_rotate_pairs(void* x, int64_t token_stride, int64_t head_stride, const int32_t* positions, const float* cos_sin,
+                          int64_t max_positions, int64_t tokens, int64_t heads, int64_t rot, void* stream);
 int mops_hip_latent_prefill(const void* q, int64_t q_token_stride, int64_t q_head_stride, const void* k, int64_t k_stride,
                             const void* kr, int64_t kr_stride, const void* vt, int64_t vt_stride, const int32_t* tiles,
-                            int64_t num_tiles, void* out, const float* cos_sin, int64_t max_positions, int64_t heads, int64_t dim,
-                            int64_t rot_dim, int64_t vdim, float scale, void* stream);
+                            int64_t num_tiles, void* out, int64_t heads, int64_t dim, int64_t rot_dim, int64_t vdim, float scale,
+                            void* stream);
 
 #ifdef __cplusplus
 }

@@ -97,7 +97,8 @@ SIGNATURES = {
     "mops_hip_latent_gather": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int64, c_int64, c_int64, c_void_p, c_void_p, c_void_p,
                                        c_int64, c_void_p, c_int64, c_int64, c_int64, c_int64, c_void_p]),
     "mops_hip_latent_prefill": (c_int, [c_void_p, c_int64, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_void_p,
-                                        c_int64, c_void_p, c_void_p, c_int64, c_int64, c_int64, c_int64, c_int64, c_float, c_void_p]),
+                                        c_int64, c_void_p, c_int64, c_int64, c_int64, c_int64, c_float, c_void_p]),
+    "mops_hip_rotate_pairs": (c_int, [c_void_p, c_int64, c_int64, c_void_p, c_void_p, c_int64, c_int64, c_int64, c_int64, c_void_p]),
     "mops_hip_linear_pin_solution": (c_int, [c_int64, c_int64, c_int64, c_int]),
     "mops_hip_linear_tune": (c_int, [c_int64, c_int64, c_int64, c_int64, c_int, c_void_p, c_int64, c_void_p, c_void_p, c_void_p]),
 }

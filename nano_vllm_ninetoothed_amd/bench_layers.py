@@ -176,16 +176,18 @@ def kernel_table(dev, seed=0):
     add("head_linear", "256 rows, 16 x 512 -> 128", graph_time(lambda i: op("head_linear")(ql, wv), 16),
         nbytes=H * kr * vdim * 2 + 256 * H * (vdim + kr) * 2, flops=2.0 * 256 * H * vdim * kr, like="linear decode")
     del cache
+    p32 = (torch.arange(T, device=dev) % 1024).to(torch.int32)
     row_seq, row_pos, tiles = R.latent_prefill_plan(plens, [0] * 16, 0, 0)
     row_seq, row_pos, tiles = i32(row_seq), i32(row_pos), i32(tiles)
     qp, kp, krp, vt = rnd(T, H, dim + rot), rnd(T, H * dim), rnd(T, rot), rnd(H * vdim, T)
     op_out = torch.empty((T, H, vdim), dtype=torch.bfloat16, device=dev)
-    add("latent_prefill", "16 x 1024, 16 heads, 192/128", _events(lambda: op("latent_prefill")(qp, kp, krp, vt, tiles, trig, 0.07, dim, rot, vdim, op_out), 300, 200),
+    add("latent_prefill", "16 x 1024, 16 heads, 192/128", _events(lambda: op("latent_prefill")(qp, kp, krp, vt, tiles, 0.07, op_out), 300, 200),
         flops=sum(2.0 * H * (dim + rot + vdim) * n * (n + 1) / 2 for n in plens), like="varlen_prefill")
+    add("rotate_pairs", f"{T} x 16 heads x 64", graph_time(lambda i: op("rotate_pairs")(qp[..., dim:], p32, trig), 8), nbytes=T * H * rot * 4.0, like="qk_norm_rope_store")
     pages = rnd(T // 256, 256, kr + rot)
     ptab = torch.arange(T // 256, dtype=torch.int32, device=dev).view(16, -1)
     add("latent_gather", f"{T} rows", graph_time(lambda i: op("latent_gather")(pages, ptab, row_seq, row_pos, kr, rot), 8), nbytes=T * (kr + rot) * 4, like="siluAndMul")
-    down, wq, wk, p32 = [rnd(T, 768 + kr + rot) for _ in range(4)], rnd(768), rnd(kr), (torch.arange(T, device=dev) % 1024).to(torch.int32)
+    down, wq, wk = [rnd(T, 768 + kr + rot) for _ in range(4)], rnd(768), rnd(kr)
     add("latent_prepare", f"{T} tokens, 768 / 512+64", graph_time(lambda i: op("latent_prepare")(down[i % 4], wq, wk, 1e-6, trig, p32, slots, pages, 768, kr, rot), 8),
         nbytes=T * (768 + kr + rot) * 4, like="qk_norm_rope_store")
 

@@ -60,6 +60,7 @@ __device__ __forceinline__ void load_qk_tile(uint16_t* tile, const uint16_t* src
   constexpr int kPitch = DP + 8;
   const int half = a.rot >> 1;
   if (vec) {
+#pragma unroll 2
     for (int i = threadIdx.x; i < kChunk * (DP / 8); i += THREADS) {
       const int r = i / (DP / 8), c = (i % (DP / 8)) * 8;
       u32x4 w = {0u, 0u, 0u, 0u};
@@ -91,6 +92,7 @@ __device__ __forceinline__ void load_qk_tile(uint16_t* tile, const uint16_t* src
     }
     return;
   }
+#pragma unroll 1
   for (int i = threadIdx.x; i < kChunk * DP; i += THREADS) {
     const int r = i / DP, c = i % DP;
     float x = 0.f;
@@ -110,7 +112,7 @@ __device__ __forceinline__ void load_qk_tile(uint16_t* tile, const uint16_t* src
 }
 
 template <int DP, int VT, bool STATE_ONLY>
-__global__ __launch_bounds__(VT * 4) void decayed_chunk_kernel(const ChunkArgs a) {
+__global__ __launch_bounds__(VT * 4, 2) void decayed_chunk_kernel(const ChunkArgs a) {
   using S = ChunkShape<DP, VT>;
   constexpr int kVTiles = VT / 32;
   constexpr int kDTiles = DP >= 64 ? DP / 64 : 1;         // 32-wide tiles of d per wave in the state
@@ -168,8 +170,10 @@ __global__ __launch_bounds__(VT * 4) void decayed_chunk_kernel(const ChunkArgs a
     const int c = 32 * (half_id * kDTiles + i) + col;
 #pragma unroll
     for (int r = 0; r < 16; ++r) {
-      st[i][r] = 0.f;
-      if (load_state && has_state_tile && c < a.pitch && state_row(r) < vlen) st[i][r] = gstate[(int64_t)state_row(r) * a.pitch + c];
+      // no branch per element (the accumulators would be copied at each): every lane reads some valid element, then selects
+      const bool ok = load_state && c < a.pitch && state_row(r) < vlen;
+      const float x = STATE_ONLY ? 0.f : gstate[ok ? state_row(r) * a.pitch + c : 0];
+      st[i][r] = ok ? x : 0.f;
     }
   }
 
@@ -188,6 +192,7 @@ __global__ __launch_bounds__(VT * 4) void decayed_chunk_kernel(const ChunkArgs a
         store16(tv + r * S::kVPitch + c, w);
       }
     } else {
+#pragma unroll 1
       for (int i = threadIdx.x; i < kChunk * VT; i += S::kThreads) {
         const int r = i / VT, c = i % VT;
         tv[r * S::kVPitch + c] = r < n && c < vlen ? vp[(int64_t)(t0 + r) * a.v_stride + c] : (uint16_t)0;
@@ -317,13 +322,20 @@ __global__ __launch_bounds__(VT * 4) void decayed_chunk_kernel(const ChunkArgs a
   if (STATE_ONLY) dst = a.seg_state + (((int64_t)seg * a.heads + h) * a.vd + v0) * a.pitch;
   else if (!a.seg_state) dst = gstate;
   if (dst && has_state_tile) {
+    // the addresses and bounds are those of the load in front of the loop; the compiler must not keep them in registers
+    // all the way, so it is not told that this is the same lane number
+    int again = lane;
+    asm volatile("" : "+v"(again));
+    const int c0 = again & 31, r0 = 32 * vt + 4 * (again >> 5);
 #pragma unroll
     for (int i = 0; i < kDTiles; ++i) {
-      const int c = 32 * (half_id * kDTiles + i) + col;
+      const int c = 32 * (half_id * kDTiles + i) + c0;
       if (c < a.pitch)
 #pragma unroll
-        for (int r = 0; r < 16; ++r)
-          if (state_row(r) < vlen) dst[(int64_t)state_row(r) * a.pitch + c] = st[i][r];
+        for (int r = 0; r < 16; ++r) {
+          const int row = r0 + 8 * (r >> 2) + (r & 3);
+          if (row < vlen) dst[(int64_t)row * a.pitch + c] = st[i][r];
+        }
     }
   }
   if (STATE_ONLY && v0 == 0 && threadIdx.x == 0) a.seg_decay[(int64_t)seg * a.heads + h] = total_log;

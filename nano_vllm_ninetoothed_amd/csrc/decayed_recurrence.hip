@@ -226,6 +226,59 @@ __global__ __launch_bounds__(256) void short_conv_kernel(const T* __restrict__ x
   store_vec<VEC>(out + t * channels + c, acc);
 }
 
+// The same for the usual tap counts: a thread keeps the weights and the last TAPS inputs of eight channels in registers and
+// walks kConvRun tokens, reading each input once.
+constexpr int kConvRun = 16;
+
+template <typename T, int TAPS>
+__global__ __launch_bounds__(256) void short_conv_run_kernel(const T* __restrict__ x, int64_t x_stride, const float* __restrict__ w,
+                                                             const float* __restrict__ bias, const T* __restrict__ ring,
+                                                             const int32_t* __restrict__ token_seq, const int32_t* __restrict__ cu_seqlens,
+                                                             const int32_t* __restrict__ starts, const int32_t* __restrict__ state_slots,
+                                                             int64_t num_slots, T* __restrict__ out, int64_t tokens, int64_t channels) {
+  const int64_t pieces = channels / 8;
+  const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  const int64_t t0 = i / pieces * kConvRun;
+  if (t0 >= tokens) return;
+  const int64_t c = (i % pieces) * 8;
+  const int64_t t1 = t0 + kConvRun < tokens ? t0 + kConvRun : tokens;
+  float wv[TAPS][8], b[8], win[TAPS][8];       // win[l]: the input l tokens back
+#pragma unroll
+  for (int l = 0; l < TAPS; ++l) load_vec<8>(w + (int64_t)(TAPS - 1 - l) * channels + c, wv[l]);
+  load_vec<8>(bias + c, b);
+  int seq = -1;
+  for (int64_t t = t0; t < t1; ++t) {
+    const int s = token_seq[t];
+    if (s != seq) {      // the window in front of this token: rows of the portion, the ring behind them, zeros before the start
+      seq = s;
+      const int slot = state_slots[s], in_portion = (int)t - cu_seqlens[s], pos = starts[s] + in_portion;
+#pragma unroll
+      for (int l = 1; l < TAPS; ++l) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) win[l - 1][e] = 0.f;
+        if (pos - l >= 0) {
+          if (l <= in_portion) load_vec<8>(x + (t - l) * x_stride + c, win[l - 1]);
+          else if (slot >= 0 && slot < num_slots) load_vec<8>(ring + ((int64_t)slot * TAPS + (pos - l) % TAPS) * channels + c, win[l - 1]);
+        }
+      }
+    }
+#pragma unroll
+    for (int l = TAPS - 1; l > 0; --l)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) win[l][e] = win[l - 1][e];
+    load_vec<8>(x + t * x_stride + c, win[0]);
+    float acc[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      acc[e] = b[e];
+#pragma unroll
+      for (int l = 0; l < TAPS; ++l) acc[e] += wv[l][e] * win[l][e];
+      acc[e] = silu_f32(acc[e]);
+    }
+    store_vec<8>(out + t * channels + c, acc);
+  }
+}
+
 template <typename T>
 __global__ __launch_bounds__(256) void short_conv_update_kernel(const T* __restrict__ x, int64_t x_stride, T* __restrict__ ring,
                                                                 const int32_t* __restrict__ cu_seqlens, const int32_t* __restrict__ starts,
@@ -314,6 +367,17 @@ extern "C" int mops_hip_short_conv(const void* x, int64_t x_row_stride, const fl
   const int64_t wgs = (tokens * (channels / (vec ? 8 : 1)) + 255) / 256;
   if (wgs > 0x7fffffffLL) return MOPS_HIP_EUNSUPPORTED;
   hipStream_t s = (hipStream_t)stream;
+  if (vec && tokens >= 256 && taps >= 2 && taps <= 4) {
+    const dim3 grid((unsigned)(((tokens + kConvRun - 1) / kConvRun * (channels / 8) + 255) / 256));
+#define MOPS_CONV_RUN(T, N) hipLaunchKernelGGL((short_conv_run_kernel<T, N>), grid, dim3(256), 0, s, (const T*)x, x_row_stride, weight, bias, \
+                            (const T*)ring, token_seq, cu_seqlens, starts, state_slots, num_slots, (T*)out, tokens, channels)
+#define MOPS_CONV_TAPS(T) do { if (taps == 2) MOPS_CONV_RUN(T, 2); else if (taps == 3) MOPS_CONV_RUN(T, 3); else MOPS_CONV_RUN(T, 4); } while (0)
+    if (dtype == MOPS_HIP_BF16) MOPS_CONV_TAPS(bf16_t);
+    else MOPS_CONV_TAPS(float);
+#undef MOPS_CONV_TAPS
+#undef MOPS_CONV_RUN
+    return finish_launch();
+  }
 #define MOPS_CONV(T, V) hipLaunchKernelGGL((short_conv_kernel<T, V>), dim3((unsigned)wgs), dim3(256), 0, s, (const T*)x, x_row_stride, weight, \
                         bias, (const T*)ring, token_seq, cu_seqlens, starts, state_slots, num_slots, (T*)out, tokens, channels, (int)taps)
   if (dtype == MOPS_HIP_BF16) { if (vec) MOPS_CONV(bf16_t, 8); else MOPS_CONV(bf16_t, 1); }

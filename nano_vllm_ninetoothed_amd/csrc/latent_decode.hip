@@ -25,7 +25,7 @@ struct LatentDecodeArgs {
 
 // NQ: 32-wide k steps per wave (kv_rank + rot_dim <= 64 NQ); NT: 16-wide latent pieces per wave (kv_rank <= 64 NT)
 template <int NQ, int NT>
-__global__ __launch_bounds__(256) void latent_decode_kernel(const LatentDecodeArgs p) {
+__global__ __launch_bounds__(256, 2) void latent_decode_kernel(const LatentDecodeArgs p) {
   constexpr int kMaxPitch = 64 * NQ + 8;
   __shared__ __align__(16) uint16_t tile[kTileTokens * kMaxPitch];
   __shared__ __align__(16) float part_s[2][kTileTokens][kHeadTile + 1];
@@ -81,6 +81,7 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(const LatentDecodeAr
   {
     const int pos = len - 1;
     const float* trig = a.cos_sin + (int64_t)(pos < a.max_positions ? pos : a.max_positions - 1) * rot;
+#pragma unroll 1
     for (int i = tid; i < kHeadTile * (lp >> 3); i += 256) {
       const int hr = i / (lp >> 3), c = (i % (lp >> 3)) * 8;
       const int head = ht * kHeadTile + hr;
@@ -91,7 +92,7 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(const LatentDecodeAr
           w = load16(ql + c);
         } else {
           const uint16_t* qr = (const uint16_t*)a.q_rot + row * a.q_rot_token_stride + head * a.q_rot_head_stride;
-#pragma unroll
+#pragma unroll 1
           for (int e = 0; e < 8; ++e) {
             const int k = c + e;
             uint32_t bits = 0;
@@ -102,8 +103,9 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(const LatentDecodeAr
               const float u = bf16lo_to_f32(qr[2 * i2]), v = bf16lo_to_f32(qr[2 * i2 + 1]), cs = trig[i2], sn = trig[rot / 2 + i2];
               bits = f32_to_bf16_bits((d & 1) ? v * cs + u * sn : u * cs - v * sn);
             }
-            w[e >> 1] |= bits << (16 * (e & 1));
+            tile[hr * lp + k] = (uint16_t)bits;
           }
+          continue;
         }
       }
       store16(tile + hr * lp + c, w);

@@ -87,14 +87,14 @@ __global__ __launch_bounds__(THREADS) void norm_kernel(float* __restrict__ resid
   }
 }
 
-// One wave per (row, part): parts of `size` consecutive elements.
-template <typename T, int VEC, bool GATE_FIRST>
+// LANES lanes per (row, part): parts of `size` consecutive elements.
+template <typename T, int VEC, int LANES, bool GATE_FIRST>
 __global__ __launch_bounds__(256) void gated_group_norm_kernel(const T* __restrict__ y, int64_t y_stride, const T* __restrict__ gate,
                                                                int64_t gate_stride, const T* __restrict__ w, float eps,
                                                                T* __restrict__ out, int64_t rows, int groups, int size) {
-  const int64_t item = (int64_t)blockIdx.x * 4 + threadIdx.x / kWave;
-  if (item >= rows * groups) return;
-  const int lane = threadIdx.x & (kWave - 1);
+  const int64_t item = (int64_t)blockIdx.x * (256 / LANES) + threadIdx.x / LANES;
+  if (item >= rows * groups) return;      // whole groups of lanes leave; the sums below stay inside a group
+  const int lane = threadIdx.x & (LANES - 1);
   const int64_t row = item / groups;
   const int col0 = (int)(item % groups) * size;
   const T* yr = y + row * y_stride + col0;
@@ -113,20 +113,20 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(const T* __restri
   };
 #pragma unroll
   for (int it = 0; it < kKeep; ++it) {
-    const int c = (it * kWave + lane) * VEC;
+    const int c = (it * LANES + lane) * VEC;
     if (c < size) {
       read(c, keep[it], gk[it]);
 #pragma unroll
       for (int e = 0; e < VEC; ++e) ss += keep[it][e] * keep[it][e];
     }
   }
-  for (int c = (kKeep * kWave + lane) * VEC; c < size; c += kWave * VEC) {
+  for (int c = (kKeep * LANES + lane) * VEC; c < size; c += LANES * VEC) {
     float v[VEC], g[VEC];
     read(c, v, g);
 #pragma unroll
     for (int e = 0; e < VEC; ++e) ss += v[e] * v[e];
   }
-  const float rstd = 1.0f / sqrtf(group_sum<kWave>(ss) / (float)size + eps);
+  const float rstd = 1.0f / sqrtf(group_sum<LANES>(ss) / (float)size + eps);
   auto finish = [&](int c, const float (&v)[VEC], const float (&g)[VEC]) {
     float o[VEC];
 #pragma unroll
@@ -141,10 +141,10 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(const T* __restri
   };
 #pragma unroll
   for (int it = 0; it < kKeep; ++it) {
-    const int c = (it * kWave + lane) * VEC;
+    const int c = (it * LANES + lane) * VEC;
     if (c < size) finish(c, keep[it], gk[it]);
   }
-  for (int c = (kKeep * kWave + lane) * VEC; c < size; c += kWave * VEC) {
+  for (int c = (kKeep * LANES + lane) * VEC; c < size; c += LANES * VEC) {
     float v[VEC], g[VEC];
     read(c, v, g);
     finish(c, v, g);
@@ -215,14 +215,18 @@ extern "C" int mops_hip_gated_group_norm(const void* y, int64_t y_row_stride, co
   if (rows == 0) return MOPS_HIP_OK;
   const int64_t n = groups * group_size;
   if (!y || !gate || !out || y_row_stride < n || gate_row_stride < n || out == gate) return MOPS_HIP_EINVAL;
-  const int64_t wgs = (rows * groups + 3) / 4;
+  const bool narrow = group_size <= 512;
+  const int64_t per_wg = narrow ? 16 : 4, wgs = (rows * groups + per_wg - 1) / per_wg;
   if (wgs > 0x7fffffffLL) return MOPS_HIP_EUNSUPPORTED;
   const bool vec = group_size % 8 == 0 && y_row_stride % 8 == 0 && gate_row_stride % 8 == 0 && aligned16(y) && aligned16(gate) &&
                    aligned16(out) && (!weight || aligned16(weight));
   hipStream_t s = (hipStream_t)stream;
-#define MOPS_GGN(T, V, F) hipLaunchKernelGGL((gated_group_norm_kernel<T, V, F>), dim3((unsigned)wgs), dim3(256), 0, s, (const T*)y, \
+#define MOPS_GGN(T, V, L, F) hipLaunchKernelGGL((gated_group_norm_kernel<T, V, L, F>), dim3((unsigned)wgs), dim3(256), 0, s, (const T*)y, \
                           y_row_stride, (const T*)gate, gate_row_stride, (const T*)weight, eps, (T*)out, rows, (int)groups, (int)group_size)
-#define MOPS_GGN2(T, V) do { if (gate_first) MOPS_GGN(T, V, true); else MOPS_GGN(T, V, false); } while (0)
+#define MOPS_GGN2(T, V) do {                                    \
+    if (narrow) { if (gate_first) MOPS_GGN(T, V, 16, true); else MOPS_GGN(T, V, 16, false); }  \
+    else { if (gate_first) MOPS_GGN(T, V, 64, true); else MOPS_GGN(T, V, 64, false); }         \
+  } while (0)
   if (dtype == MOPS_HIP_BF16) { if (vec) MOPS_GGN2(bf16_t, 8); else MOPS_GGN2(bf16_t, 1); }
   else { if (vec) MOPS_GGN2(float, 8); else MOPS_GGN2(float, 1); }
 #undef MOPS_GGN2

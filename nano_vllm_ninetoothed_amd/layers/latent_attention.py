@@ -10,6 +10,11 @@ from ..mops.hip.recurrent_ops import latent_decode_covers, latent_prefill_covers
 EXPAND_FROM = 64     # portions of at least this many tokens expand keys and values instead of absorbing the projections
 
 
+def pad_rows(w, rows):
+    """w [heads, n, k] with zero rows up to `rows` per head."""
+    return torch.nn.functional.pad(w, (0, 0, 0, rows - w.shape[1]))
+
+
 @register_mixer("latent_attention")
 class LatentAttention:
     uses_pages, uses_slots = True, False
@@ -28,7 +33,10 @@ class LatentAttention:
         self.down = pack([take(prefix + "dq", (qr, m.width)), take(prefix + "dkv", (kr + r, m.width))])
         self.q_norm = take(prefix + "dq.norm", (qr,), "norm")
         self.kv_norm = take(prefix + "dkv.norm", (kr,), "norm")
-        self.uq = pack([take(prefix + "uq", (h * (d + r), qr))])
+        # queries leave the projection with both parts of a head padded to multiples of eight: [dim | 0 | rot_dim | 0]
+        self.dim_pad, self.rot_pad = dp, rp = (d + 7) // 8 * 8, (r + 7) // 8 * 8
+        uq = take(prefix + "uq", (h * (d + r), qr)).view(h, d + r, qr)
+        self.uq = torch.cat((pad_rows(uq[:, :d], dp), pad_rows(uq[:, d:], rp)), dim=1).reshape(h * (dp + rp), qr).contiguous()
         uk, uv = take(prefix + "uk", (h * d, kr)), take(prefix + "uv", (h * v, kr))
         self.q_to_latent = uk.view(h, d, kr).transpose(1, 2).contiguous()     # [H, kv_rank, dim]
         self.latent_to_v = uv.view(h, v, kr)                                  # [H, vdim, kv_rank]
@@ -39,11 +47,11 @@ class LatentAttention:
         self.rows = hip_op("latent_decode" if latent_decode_covers(m.dtype, kr, r, m.cache.block_size) else "latent_attention_rows")
         self.expands = latent_prefill_covers(m.dtype, d, r, v)
         if self.expands:
-            # the expansion reads gathered latents whose row length is a multiple of eight
+            # the expansion reads gathered latents whose row length is a multiple of eight, and gives keys in the queries' layout
             pad = -kr % 8
-            self.w_k = pack([torch.nn.functional.pad(uk, (0, pad))])
+            self.w_k = torch.nn.functional.pad(pad_rows(uk.view(h, d, kr), dp), (0, pad)).reshape(h * dp, kr + pad).contiguous()
             self.w_v = torch.nn.functional.pad(uv, (0, pad)).contiguous()
-            self.gather, self.prefill = hip_op("latent_gather"), hip_op("latent_prefill")
+            self.gather, self.rotate, self.prefill = hip_op("latent_gather"), hip_op("rotate_pairs"), hip_op("latent_prefill")
 
     def __call__(self, x, ctx):
         h, d, r, v = self.heads, self.dim, self.rot_dim, self.vdim
@@ -51,7 +59,7 @@ class LatentAttention:
         down = self.linear(x, self.down)
         cq = self.prepare(down, self.q_norm, self.kv_norm, self.eps, self.cos_sin, ctx["positions32"], ctx["slot_mapping"], self.pages,
                           self.q_rank, self.kv_rank, r)
-        q = self.linear(cq, self.uq)[:, :h * (d + r)].unflatten(1, (h, d + r))
+        q = self.linear(cq, self.uq).view(t, h, self.dim_pad + self.rot_pad)
         plan = self._plan(ctx, x.device) if self.expands else None
         if plan is None:
             o = self._absorbed(q, ctx["token_context"], ctx["token_seq"], ctx)
@@ -66,7 +74,7 @@ class LatentAttention:
     def _absorbed(self, q, context_lens, row_seq, ctx):
         """Query rows against the cache in the latent space: cheap per row, no key or value is ever expanded."""
         q_latent = self.head_linear(q[..., :self.dim], self.q_to_latent)
-        o = self.rows(q_latent, q[..., self.dim:], self.pages, self.cos_sin, context_lens, ctx["block_tables"], self.scale, row_seq)
+        o = self.rows(q_latent, q[..., self.dim_pad:self.dim_pad + self.rot_dim], self.pages, self.cos_sin, context_lens, ctx["block_tables"], self.scale, row_seq)
         return self.head_linear(o, self.latent_to_v)
 
     def _plan(self, ctx, device):
@@ -89,8 +97,9 @@ class LatentAttention:
 
     def _expanded(self, q, plan, ctx, out):
         """Long portions: keys and values of the whole context are expanded once, then ordinary attention."""
-        _, row_seq, row_pos, tiles = plan
+        first, row_seq, row_pos, tiles = plan
         c, kr = self.gather(self.pages, ctx["block_tables"], row_seq, row_pos, self.kv_rank, self.rot_dim)
         k = self.linear(c, self.w_k)
         vt = self.linear(self.w_v, c)
-        self.prefill(q, k, kr, vt, tiles, self.cos_sin, self.scale, self.dim, self.rot_dim, self.vdim, out)
+        self.rotate(q[first:, :, self.dim_pad:self.dim_pad + self.rot_dim], ctx["positions32"][first:], self.cos_sin)
+        self.prefill(q, k, kr, vt, tiles, self.scale, out)

@@ -48,6 +48,7 @@ EXTENSION_OP_NAMES = (
     "latent_attention_rows",
     "latent_decode",
     "latent_gather",
+    "rotate_pairs",
     "latent_prefill",
 )
 

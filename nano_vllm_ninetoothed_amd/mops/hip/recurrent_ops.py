@@ -336,7 +336,7 @@ def latent_decode(q_latent, q_rot, cache, cos_sin, context_lens, block_table, sc
 
 
 def latent_prefill_covers(dtype, dim: int, rot_dim: int, vdim: int) -> bool:
-    return dtype == torch.bfloat16 and dim + rot_dim <= 256 and vdim <= 256
+    return dtype == torch.bfloat16 and (dim + 7) // 8 * 8 + (rot_dim + 7) // 8 * 8 <= 256 and vdim <= 256
 
 
 PREFILL_QUERIES, PREFILL_KEYS = 128, 64
@@ -379,22 +379,33 @@ def latent_gather(cache, block_table, row_seq, row_pos, kv_rank, rot_dim):
 
 
 @register_hip_op
-def latent_prefill(q, k, kr, vt, tiles, cos_sin, scale, dim, rot_dim, vdim, out):
-    """Causal attention of long portions over expanded keys and values (layout: mops_hip_latent_prefill); writes the portions'
-    rows of out [tokens, heads, vdim]."""
-    _require(q.dim() == 3 and q.dtype == torch.bfloat16 and q.is_cuda and q.stride(2) == 1 and q.shape[2] == dim + rot_dim,
-             "q must be [tokens, heads, dim + rot_dim] in bfloat16")
-    heads = q.shape[1]
+def rotate_pairs(x, positions, cos_sin):
+    """Rotates the pairs (2i, 2i+1) of x [tokens, heads, rot] (bf16, any token and head strides) in place."""
+    _require(x.dim() == 3 and x.is_cuda and x.dtype == torch.bfloat16 and x.stride(2) == 1 and cos_sin.dim() == 2 and cos_sin.shape[1] == x.shape[2],
+             "x must be [tokens, heads, rot] in bfloat16 and cos_sin [positions, rot]")
+    tokens, heads, rot = x.shape
+    st = _capi.load().mops_hip_rotate_pairs(x.data_ptr(), x.stride(0), x.stride(1) if heads > 1 else max(rot, x.stride(1)),
+                                            _flat("positions", positions, tokens, torch.int32), _flat("cos_sin", cos_sin, cos_sin.numel(), torch.float32),
+                                            cos_sin.shape[0], tokens, heads, rot, _stream(x))
+    _capi.check("mops_hip_rotate_pairs", st)
+    return x
+
+
+@register_hip_op
+def latent_prefill(q, k, kr, vt, tiles, scale, out):
+    """Causal attention of long portions over expanded keys and values: q [tokens, heads, dim + rot] (rotated), k [rows,
+    heads * dim], kr [rows, rot], vt [heads * vdim, rows]; writes the portions' rows of out [tokens, heads, vdim].  dim, rot and
+    the strides are multiples of eight."""
+    _require(q.dim() == 3 and q.dtype == torch.bfloat16 and q.is_cuda and q.stride(2) == 1, "q must be [tokens, heads, dim + rot] in bfloat16")
+    heads, rot, rows = q.shape[1], kr.shape[1], k.shape[0]
+    dim, vdim = q.shape[2] - rot, out.shape[2]
     _require(out.shape == (q.shape[0], heads, vdim) and out.is_contiguous() and out.dtype == q.dtype, "out must be contiguous [tokens, heads, vdim]")
-    rows = k.shape[0]
-    _require(k.shape[1] >= heads * dim and k.stride(1) == 1 and kr.shape[0] == rows and kr.stride(1) == 1 and kr.shape[1] >= rot_dim
+    _require(dim > 0 and k.shape[1] == heads * dim and k.stride(1) == 1 and kr.shape[0] == rows and kr.stride(1) == 1
              and vt.shape == (heads * vdim, rows) and vt.stride(1) == 1 and k.dtype == kr.dtype == vt.dtype == q.dtype
-             and rows % PREFILL_KEYS == 0, "k [rows, heads * dim], kr [rows, rot_dim], vt [heads * vdim, rows], rows a multiple of 64")
-    _require(cos_sin.dim() == 2 and cos_sin.shape[1] == rot_dim, "cos_sin must be [positions, rot_dim]")
+             and rows % PREFILL_KEYS == 0, "k [rows, heads * dim], kr [rows, rot], vt [heads * vdim, rows], rows a multiple of 64")
     n = tiles.shape[0]
     st = _capi.load().mops_hip_latent_prefill(q.data_ptr(), q.stride(0), q.stride(1), k.data_ptr(), k.stride(0), kr.data_ptr(), kr.stride(0),
-                                              vt.data_ptr(), vt.stride(0), _flat("tiles", tiles, 5 * n, torch.int32), n, out.data_ptr(),
-                                              _flat("cos_sin", cos_sin, cos_sin.numel(), torch.float32), cos_sin.shape[0], heads, dim, rot_dim,
+                                              vt.data_ptr(), vt.stride(0), _flat("tiles", tiles, 5 * n, torch.int32), n, out.data_ptr(), heads, dim, rot,
                                               vdim, float(scale), _stream(q))
     _capi.check("mops_hip_latent_prefill", st)
     return out

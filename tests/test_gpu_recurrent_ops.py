@@ -261,6 +261,27 @@ def test_short_conv_in_portions(gpu, dtype, channels, taps):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("taps", [2, 3, 4, 5])
+def test_short_conv_of_many_tokens(gpu, dtype, taps):
+    """Unequal portions packed into one long launch, some behind earlier tokens."""
+    g = torch.Generator().manual_seed(taps + 40)
+    channels, lens, before = 48, [100, 1, 2, 3, 17, 260], [0, 7, 1, 2, 0, 31]
+    w, b = torch.randn((channels, taps), generator=g), torch.randn(channels, generator=g)
+    i32 = lambda t: torch.tensor(t, dtype=torch.int32, device=gpu)   # noqa: E731
+    ring = torch.full((7, taps, channels), 99.0, dtype=dtype, device=gpu)
+    slots, cu, xs, wants = [3, 6, 0, 5, 1, 2], [0], [], []
+    for n, p, s in zip(lens, before, slots):
+        full = rnd(g, p + n, channels, dtype=dtype)
+        wants.append(O.silu(O.causal_conv(full.double(), w.double(), b.double()))[p:])
+        op("short_conv_update")(full[:p].to(gpu), ring, i32([0, p]), i32([0]), i32([s])) if p else None
+        xs.append(full[p:])
+        cu.append(cu[-1] + n)
+    seqs = [i for i, n in enumerate(lens) for _ in range(n)]
+    got = op("short_conv")(torch.cat(xs).to(gpu), w.t().contiguous().to(gpu), b.to(gpu), ring, i32(seqs), i32(cu), i32(before), i32(slots))
+    close(got, torch.cat(wants), dtype, f"{taps} taps", 2)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("sizes", [(4, 2, 16, 24, 4), (6, 3, 20, 70, 3), (2, 1, 128, 64, 1)])
 def test_decode_step_with_the_convolution_inside(gpu, dtype, sizes):
     """One launch per token against convolution, then recurrence, in float64; two sequences at different positions."""
@@ -395,14 +416,19 @@ def test_latent_prefill(gpu, sizes):
     row_seq, row_pos, tiles = R.latent_prefill_plan(counts, starts, 3, 0)
     i32 = lambda t: torch.tensor(t, dtype=torch.int32, device=gpu)   # noqa: E731
     c, kpart = op("latent_gather")(cache, table, i32(row_seq), i32(row_pos), kr, rot)
-    pad = -kr % 8
+    pad, dp, rp = -kr % 8, (dim + 7) // 8 * 8, (rot + 7) // 8 * 8
+    assert c.shape[1] == kr + pad and kpart.shape[1] == rp and float(kpart[:, rot:].abs().sum()) == 0.0
     lin = op("linear")
-    from nano_vllm_ninetoothed_amd.layers import pack
-    k = lin(c, pack([torch.nn.functional.pad(uk.bfloat16().to(gpu), (0, pad))]))
-    vt = lin(torch.nn.functional.pad(uv.bfloat16().to(gpu), (0, pad)).contiguous(), c)
+    F = torch.nn.functional
+    k = lin(c, F.pad(uk.view(heads, dim, kr), (0, pad, 0, dp - dim)).reshape(heads * dp, -1).bfloat16().to(gpu))
+    vt = lin(F.pad(uv.bfloat16().to(gpu), (0, pad)).contiguous(), c)
     out = torch.full((T, heads, vdim), 3.0, dtype=torch.bfloat16, device=gpu)
     scale = (dim + rot) ** -0.5
-    op("latent_prefill")(q.bfloat16().to(gpu), k, kpart, vt, i32(tiles), cos_sin, scale, dim, rot, vdim, out)
+    qp = torch.cat((F.pad(q[..., :dim], (0, dp - dim)), F.pad(q[..., dim:], (0, rp - rot))), -1).bfloat16().to(gpu)
+    positions = i32([0, 0, 0] + [p for n, st in zip(counts, starts) for p in range(st, st + n)])
+    op("rotate_pairs")(qp[3:, :, dp:dp + rot], positions[3:], cos_sin)
+    assert torch.equal(qp[:3, :, dp:dp + rot].cpu(), q[:3, :, dim:].bfloat16())
+    op("latent_prefill")(qp, k, kpart, vt, i32(tiles), scale, out)
     assert float(out[:3].float().min()) == 3.0
     at = 3
     for s, (n, start) in enumerate(zip(counts, starts)):
