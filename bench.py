@@ -65,6 +65,7 @@ def parse_args():
     ap.add_argument("--e2e-eager", action="store_true", help="e2e: no HIP-graph replay of the decode step")
     ap.add_argument("--e2e-stepwise", action="store_true", help="e2e: read every step's tokens back before the next step, as the reference does")
     ap.add_argument("--nepulix-part", default="all", choices=["all", "models", "kernels"], help="nepulix: throughput of whole models, kernels, or both")
+    ap.add_argument("--nepulix-kernels", default="", help="nepulix: kernels to time, by the beginning of their names, with commas between them (default: all)")
     ap.add_argument("--nepulix-sizes", default="", help="nepulix: sizes to run, with commas between them (default: all)")
     ap.add_argument("--no-cpu-baseline", action="store_true")
     ap.add_argument("--no-e2e", action="store_true", help="default op only: skip the end-to-end block of the line (profiling runs)")
@@ -186,7 +187,7 @@ def run_nepulix(args, torch, dev):
             out.update(value=last["tok_per_s"], ms_per_step=last["ms"])
             out["config"].update(size=name, global_batch=last["batch"], seq_len=last["context"])
     if args.nepulix_part != "models":
-        out["kernels"] = B.kernel_table(dev, args.seed)
+        out["kernels"] = B.kernel_table(dev, args.seed, args.nepulix_kernels)
     print(json.dumps(out))
 
 

@@ -465,8 +465,7 @@ int mops_hip_latent_attention_rows(const mops_hip_latent_rows* a, void* stream);
  * multiple of 32, pitch a multiple of 8; MOPS_HIP_EUNSUPPORTED otherwise.  workspace: device scratch of at least
  * mops_hip_latent_decode_workspace_bytes(...), private to the call until it completes.
  */
-int64_t mops_hip_latent_decode_workspace_bytes(int64_t rows, int64_t heads, int64_t kv_rank, int64_t max_blocks,
-                                               int64_t block_size);
+int64_t mops_hip_latent_decode_workspace_bytes(int64_t rows, int64_t heads, int64_t kv_rank, int64_t rot_dim);
 int mops_hip_latent_decode(const mops_hip_latent_rows* a, void* workspace, int64_t workspace_bytes, void* stream);
 
 /*

@@ -92,7 +92,7 @@ SIGNATURES = {
     "mops_hip_head_linear": (c_int, [c_void_p, c_int64, c_int64, c_void_p, c_void_p, c_int64, c_int64, c_int, c_int64, c_int64, c_int64,
                                      c_int64, c_void_p]),
     "mops_hip_latent_attention_rows": (c_int, [POINTER(LatentRows), c_void_p]),
-    "mops_hip_latent_decode_workspace_bytes": (c_int64, [c_int64] * 5),
+    "mops_hip_latent_decode_workspace_bytes": (c_int64, [c_int64] * 4),
     "mops_hip_latent_decode": (c_int, [POINTER(LatentRows), c_void_p, c_int64, c_void_p]),
     "mops_hip_latent_gather": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int64, c_int64, c_int64, c_void_p, c_void_p, c_void_p,
                                        c_int64, c_void_p, c_int64, c_int64, c_int64, c_int64, c_void_p]),

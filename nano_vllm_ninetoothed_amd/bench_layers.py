@@ -100,7 +100,7 @@ def graph_time(fn, calls=10, replays=10):
     return _events(graph.replay, 3, replays) / calls
 
 
-def kernel_table(dev, seed=0):
+def kernel_table(dev, seed=0, only=""):
     """[{kernel, us, bound, achieved, unit, frac, like, like_frac}]: algorithmic work over time, as a fraction of the roof."""
     from . import mops
     from . import workloads as W
@@ -112,7 +112,10 @@ def kernel_table(dev, seed=0):
     i32 = lambda x: torch.tensor(x, dtype=torch.int32, device=dev)      # noqa: E731
     rows, likes = [], {}
 
-    def add(name, shape, seconds, nbytes=0.0, flops=0.0, like=None):
+    def add(name, shape, timed, nbytes=0.0, flops=0.0, like=None):
+        if only and not name.startswith(tuple(only.split(","))):
+            return
+        seconds = timed()
         t_mem, t_math = nbytes / (HBM * 1e9), flops / (MFMA * 1e12)
         bound = "hbm" if t_mem >= t_math else "mfma"
         value, unit = (nbytes / seconds / 1e9, "GB/s") if bound == "hbm" else (flops / seconds / 1e12, "TFLOP/s")
@@ -121,7 +124,7 @@ def kernel_table(dev, seed=0):
         if like is None:
             likes[name] = r["frac"]
         else:
-            r.update(like=like, like_frac=likes[like], times_further=round(likes[like] / r["frac"], 2))
+            r.update(like=like, like_frac=likes.get(like), times_further=round(likes[like] / r["frac"], 2) if like in likes else None)
         rows.append(r)
 
     # ---- the Qwen3 path's kernels, the yardstick
@@ -134,46 +137,46 @@ def kernel_table(dev, seed=0):
         at += n
     table, lens_g = table.to(dev), i32(ctx)
     kc, vc, q = rnd(sum(nb), 256, 8, 128), rnd(sum(nb), 256, 8, 128), rnd(256, 1, 16, 128)
-    add("paged_decode", "256 x uniform[512,4096], 16/8 heads", graph_time(lambda i: op("flash_attn_with_kvcache")(
+    add("paged_decode", "256 x uniform[512,4096], 16/8 heads", lambda: graph_time(lambda i: op("flash_attn_with_kvcache")(
         q, kc, vc, cache_seqlens=lens_g, block_table=table, softmax_scale=0.088, causal=True), 4), nbytes=W.decode_bytes(ctx, 16, 8, max(nb)))
     del kc, vc
     plens = [1024] * 16
     T = sum(plens)
     d = W.to_device(W.prefill_inputs(plens, seed=seed), dev)
-    add("varlen_prefill", "16 x 1024, 16/8 heads of 128", _events(lambda: op("flash_attn_varlen_func")(
+    add("varlen_prefill", "16 x 1024, 16/8 heads of 128", lambda: _events(lambda: op("flash_attn_varlen_func")(
         d["q"], d["k"], d["v"], max_seqlen_q=1024, cu_seqlens_q=d["cu_seqlens"], max_seqlen_k=1024, cu_seqlens_k=d["cu_seqlens"], softmax_scale=d["scale"],
         causal=True, block_table=None), 300, 200), flops=W.prefill_flops(plens, 16))
     bufs = [rnd(T, 6144) for _ in range(4)]
     halves = [b.chunk(2, dim=-1) for b in bufs]
-    add("siluAndMul", f"{T} x 3072", graph_time(lambda i: op("siluAndMul")(*halves[i % 4]), 8), nbytes=T * 3072 * 6)
+    add("siluAndMul", f"{T} x 3072", lambda: graph_time(lambda i: op("siluAndMul")(*halves[i % 4]), 8), nbytes=T * 3072 * 6)
     x4, r4, w4 = [rnd(512, 4096) for _ in range(24)], [rnd(512, 4096) for _ in range(24)], rnd(4096)
-    add("add_rms", "512 x 4096", graph_time(lambda i: op("add_rms_forward")(x4[i % 24], r4[i % 24], w4, 1e-6), 24), nbytes=512 * 4096 * 8)
+    add("add_rms", "512 x 4096", lambda: graph_time(lambda i: op("add_rms_forward")(x4[i % 24], r4[i % 24], w4, 1e-6), 24), nbytes=512 * 4096 * 8)
     xt, rt, w1 = [rnd(T, 1024) for _ in range(4)], [rnd(T, 1024) for _ in range(4)], rnd(1024)
-    add("add_rms prefill", f"{T} x 1024", graph_time(lambda i: op("add_rms_forward")(xt[i % 4], rt[i % 4], w1, 1e-6), 8), nbytes=T * 1024 * 8)
+    add("add_rms prefill", f"{T} x 1024", lambda: graph_time(lambda i: op("add_rms_forward")(xt[i % 4], rt[i % 4], w1, 1e-6), 8), nbytes=T * 1024 * 8)
     qkv, kc2 = [rnd(T, 4096) for _ in range(2)], torch.zeros((T // 256, 256, 8, 128), dtype=torch.bfloat16, device=dev)
     vc2, ang, slots = torch.zeros_like(kc2), torch.rand((T, 1, 64), device=dev), torch.randperm(T, device=dev).to(torch.int32)
     nw = rnd(128)
     cs, sn = ang.cos(), ang.sin()
-    add("qk_norm_rope_store", f"{T} tokens, 16/8 heads", graph_time(lambda i: op("qk_norm_rope_store")(
+    add("qk_norm_rope_store", f"{T} tokens, 16/8 heads", lambda: graph_time(lambda i: op("qk_norm_rope_store")(
         qkv[i % 2], nw, nw, 1e-6, cs, sn, kc2, vc2, slots, 16, 8, need_k=False), 8), nbytes=T * (4096 * 2 + 512 + 4 + 2048 * 2 + 2 * 1024 * 2))
     wl = rnd(1024, 1024)
     xl = [rnd(T, 1024) for _ in range(4)]
-    add("linear", f"{T} x 1024 x 1024 (library)", graph_time(lambda i: op("linear")(xl[i % 4], wl), 8), flops=2.0 * T * 1024 * 1024, nbytes=T * 1024 * 4)
+    add("linear", f"{T} x 1024 x 1024 (library)", lambda: graph_time(lambda i: op("linear")(xl[i % 4], wl), 8), flops=2.0 * T * 1024 * 1024, nbytes=T * 1024 * 4)
     wls = [rnd(1024, 1024) for _ in range(64)]
     xs = rnd(256, 1024)
-    add("linear decode", "256 x 1024 x 1024 (library)", graph_time(lambda i: op("linear")(xs, wls[i % 64]), 64), nbytes=1024 * 1024 * 2 + 256 * 1024 * 4)
+    add("linear decode", "256 x 1024 x 1024 (library)", lambda: graph_time(lambda i: op("linear")(xs, wls[i % 64]), 64), nbytes=1024 * 1024 * 2 + 256 * 1024 * 4)
 
     # ---- the design's kernels
     H, kr, rot, dim, vdim = 16, 512, 64, 128, 128
     cache, ql, qn = rnd(sum(nb), 256, kr + rot), rnd(256, H, kr), rnd(256, H, dim + rot)
     trig = Rotary(8192, dev).table(1e4, rot)
-    add("latent_decode", "256 x uniform[512,4096], 16 heads, 512+64", graph_time(lambda i: op("latent_decode")(
+    add("latent_decode", "256 x uniform[512,4096], 16 heads, 512+64", lambda: graph_time(lambda i: op("latent_decode")(
         ql, qn[..., dim:], cache, trig, lens_g, table, 0.07), 4), nbytes=sum(ctx) * (kr + rot) * 2 + 256 * H * (2 * kr + rot) * 2,
         flops=2.0 * sum(ctx) * H * (2 * kr + rot), like="paged_decode")
     wabs, wv = rnd(H, kr, dim), rnd(H, vdim, kr)
-    add("head_linear", "256 rows, 16 x 128 -> 512", graph_time(lambda i: op("head_linear")(qn[..., :dim], wabs), 16),
+    add("head_linear", "256 rows, 16 x 128 -> 512", lambda: graph_time(lambda i: op("head_linear")(qn[..., :dim], wabs), 16),
         nbytes=H * kr * dim * 2 + 256 * H * (dim + kr) * 2, flops=2.0 * 256 * H * dim * kr, like="linear decode")
-    add("head_linear", "256 rows, 16 x 512 -> 128", graph_time(lambda i: op("head_linear")(ql, wv), 16),
+    add("head_linear", "256 rows, 16 x 512 -> 128", lambda: graph_time(lambda i: op("head_linear")(ql, wv), 16),
         nbytes=H * kr * vdim * 2 + 256 * H * (vdim + kr) * 2, flops=2.0 * 256 * H * vdim * kr, like="linear decode")
     del cache
     p32 = (torch.arange(T, device=dev) % 1024).to(torch.int32)
@@ -181,14 +184,14 @@ def kernel_table(dev, seed=0):
     row_seq, row_pos, tiles = i32(row_seq), i32(row_pos), i32(tiles)
     qp, kp, krp, vt = rnd(T, H, dim + rot), rnd(T, H * dim), rnd(T, rot), rnd(H * vdim, T)
     op_out = torch.empty((T, H, vdim), dtype=torch.bfloat16, device=dev)
-    add("latent_prefill", "16 x 1024, 16 heads, 192/128", _events(lambda: op("latent_prefill")(qp, kp, krp, vt, tiles, 0.07, op_out), 300, 200),
+    add("latent_prefill", "16 x 1024, 16 heads, 192/128", lambda: _events(lambda: op("latent_prefill")(qp, kp, krp, vt, tiles, 0.07, op_out), 300, 200),
         flops=sum(2.0 * H * (dim + rot + vdim) * n * (n + 1) / 2 for n in plens), like="varlen_prefill")
-    add("rotate_pairs", f"{T} x 16 heads x 64", graph_time(lambda i: op("rotate_pairs")(qp[..., dim:], p32, trig), 8), nbytes=T * H * rot * 4.0, like="qk_norm_rope_store")
+    add("rotate_pairs", f"{T} x 16 heads x 64", lambda: graph_time(lambda i: op("rotate_pairs")(qp[..., dim:], p32, trig), 8), nbytes=T * H * rot * 4.0, like="qk_norm_rope_store")
     pages = rnd(T // 256, 256, kr + rot)
     ptab = torch.arange(T // 256, dtype=torch.int32, device=dev).view(16, -1)
-    add("latent_gather", f"{T} rows", graph_time(lambda i: op("latent_gather")(pages, ptab, row_seq, row_pos, kr, rot), 8), nbytes=T * (kr + rot) * 4, like="siluAndMul")
+    add("latent_gather", f"{T} rows", lambda: graph_time(lambda i: op("latent_gather")(pages, ptab, row_seq, row_pos, kr, rot), 8), nbytes=T * (kr + rot) * 4, like="siluAndMul")
     down, wq, wk = [rnd(T, 768 + kr + rot) for _ in range(4)], rnd(768), rnd(kr)
-    add("latent_prepare", f"{T} tokens, 768 / 512+64", graph_time(lambda i: op("latent_prepare")(down[i % 4], wq, wk, 1e-6, trig, p32, slots, pages, 768, kr, rot), 8),
+    add("latent_prepare", f"{T} tokens, 768 / 512+64", lambda: graph_time(lambda i: op("latent_prepare")(down[i % 4], wq, wk, 1e-6, trig, p32, slots, pages, 768, kr, rot), 8),
         nbytes=T * (768 + kr + rot) * 4, like="qk_norm_rope_store")
 
     def recurrent(tag, heads, groups, dd, vd, const):
@@ -209,7 +212,7 @@ def kernel_table(dev, seed=0):
         x, dt, o = rnd(bs, width), rnd(bs, heads), torch.empty((bs, inner), dtype=torch.bfloat16, device=dev)
         sl, st = torch.arange(bs, dtype=torch.int32, device=dev), torch.full((bs,), 1000, dtype=torch.int32, device=dev)
         more = {} if const else {"dt": dt, "conv": conv}
-        add("decayed_recurrence " + tag, f"{bs} sequences, {heads} x {dd} x {vd}", graph_time(lambda i: op("decayed_recurrence")(
+        add("decayed_recurrence " + tag, f"{bs} sequences, {heads} x {dd} x {vd}", lambda: graph_time(lambda i: op("decayed_recurrence")(
             x[:, inner + gn:], x[:, inner:inner + gn], x[:, :inner], o, state, sl, st, heads, groups, dd, vd, **opts, **more), 6),
             nbytes=2.0 * bs * heads * dd * vd * 4 + bs * (width + inner) * 2, like="paged_decode")
         xs = [rnd(T, width) for _ in range(2)]
@@ -220,7 +223,7 @@ def kernel_table(dev, seed=0):
             segs, bounds, cu = i32(segs), i32(bounds), i32(cu)
             more = {} if const else {"dt": dts}
             # least arithmetic at 64 tokens a chunk: scores and their product below the diagonal, state in and out
-            add("decayed_chunks " + tag, f"{nseq} x {T // nseq}, {heads} x {dd} x {vd}", _events(lambda: op("decayed_chunks")(
+            add("decayed_chunks " + tag, f"{nseq} x {T // nseq}, {heads} x {dd} x {vd}", lambda: _events(lambda: op("decayed_chunks")(
                 xs[0][:, inner + gn:], xs[0][:, inner:inner + gn], xs[0][:, :inner], oT, state, sl[:nseq], torch.zeros_like(st[:nseq]), heads, groups, dd, vd, segs,
                 bounds, cu_seqlens=cu, **opts, **more), 20, 50), flops=T * heads * (65.0 * (dd + vd) + 4.0 * dd * vd), nbytes=T * (width + inner) * 2.0,
                 like="varlen_prefill")
@@ -228,21 +231,21 @@ def kernel_table(dev, seed=0):
             tok_seq, sl16 = torch.arange(T, device=dev).div(1024, rounding_mode="floor").to(torch.int32), sl[:16]
             cu16, z16 = i32(list(range(0, T + 1, 1024))), torch.zeros(16, dtype=torch.int32, device=dev)
             big = [rnd(T, width + inner + heads) for _ in range(2)]
-            add("short_conv", f"{T} x {width}, 4 taps", graph_time(lambda i: op("short_conv")(
+            add("short_conv", f"{T} x {width}, 4 taps", lambda: graph_time(lambda i: op("short_conv")(
                 big[i % 2][:, inner:inner + width], conv[0], conv[1], conv[2], tok_seq, cu16, z16, sl16), 4), nbytes=T * width * 4.0, like="siluAndMul")
 
     recurrent("retention", 16, 16, 128, 128, True)
     recurrent("mamba2", 64, 8, 128, 64, False)
     lim = lambda i: op("clamped_glu")(*halves[i % 4], 7.0)      # noqa: E731
-    add("clamped_glu", f"{T} x 3072", graph_time(lim, 8), nbytes=T * 3072 * 6, like="siluAndMul")
-    add("gated_group_norm", f"{T} x 3072, 24 groups", graph_time(lambda i: op("gated_group_norm")(*halves[i % 4], 24, 1e-6), 8), nbytes=T * 3072 * 6, like="siluAndMul")
-    add("gated_group_norm", f"{T} x 3072, 1 group", graph_time(lambda i: op("gated_group_norm")(*halves[i % 4], 1, 1e-6, gate_first=True), 8), nbytes=T * 3072 * 6,
+    add("clamped_glu", f"{T} x 3072", lambda: graph_time(lim, 8), nbytes=T * 3072 * 6, like="siluAndMul")
+    add("gated_group_norm", f"{T} x 3072, 24 groups", lambda: graph_time(lambda i: op("gated_group_norm")(*halves[i % 4], 24, 1e-6), 8), nbytes=T * 3072 * 6, like="siluAndMul")
+    add("gated_group_norm", f"{T} x 3072, 1 group", lambda: graph_time(lambda i: op("gated_group_norm")(*halves[i % 4], 1, 1e-6, gate_first=True), 8), nbytes=T * 3072 * 6,
         like="siluAndMul")
     f4 = [x.float() for x in r4]
-    add("norm_residual_add", "512 x 4096", graph_time(lambda i: op("norm_residual_add")(f4[i % 24], x4[i % 24], w4, 1e-6, 1.0), 24), nbytes=512 * 4096 * 12, like="add_rms")
+    add("norm_residual_add", "512 x 4096", lambda: graph_time(lambda i: op("norm_residual_add")(f4[i % 24], x4[i % 24], w4, 1e-6, 1.0), 24), nbytes=512 * 4096 * 12, like="add_rms")
     ft = [x.float() for x in rt]
-    add("norm_residual_add", f"{T} x 1024", graph_time(lambda i: op("norm_residual_add")(ft[i % 4], xt[i % 4], w1, 1e-6, 1.0), 8), nbytes=T * 1024 * 12, like="add_rms prefill")
-    add("rms_norm_f32", "512 x 4096", graph_time(lambda i: op("rms_norm_f32")(f4[i % 24], w4, 1e-6, 1.0), 24), nbytes=512 * 4096 * 6, like="add_rms")
+    add("norm_residual_add", f"{T} x 1024", lambda: graph_time(lambda i: op("norm_residual_add")(ft[i % 4], xt[i % 4], w1, 1e-6, 1.0), 8), nbytes=T * 1024 * 12, like="add_rms prefill")
+    add("rms_norm_f32", "512 x 4096", lambda: graph_time(lambda i: op("rms_norm_f32")(f4[i % 24], w4, 1e-6, 1.0), 24), nbytes=512 * 4096 * 6, like="add_rms")
     emb, ids = rnd(32768, 1024), [torch.randint(0, 32768, (T,), device=dev) for _ in range(4)]
-    add("embed_residual", f"{T} x 1024", graph_time(lambda i: op("embed_residual")(ids[i % 4], emb), 8), nbytes=T * 1024 * 8.0, like="add_rms prefill")
+    add("embed_residual", f"{T} x 1024", lambda: graph_time(lambda i: op("embed_residual")(ids[i % 4], emb), 8), nbytes=T * 1024 * 8.0, like="add_rms prefill")
     return rows

@@ -5,12 +5,12 @@
 //   O_i = e^{L_i} S^T q_i + sum_{j <= i} e^{L_i - L_j} s_j (q_i . k_j) v_j + skip v_i
 //   S  <- e^{L_end} S + sum_j e^{L_end - L_j} s_j k_j v_j^T
 //
-// Workgroup = (segment, head, tile of VT value columns), walking the chunks of its segment with S^T [VT x d] in the
+// Workgroup = (segment, head, tile of VT value columns), walking the chunks of its segment with S [d x VT] in the
 // accumulators.  All products are v_mfma_f32_32x32x16_bf16:
 //   P^T [j, i] = K Q^T                 rows of the two LDS tiles as they are
 //   O^T [v, i] = S^T Q^T + V^T P^T     the accumulator layout of P^T is the B-operand layout of the second product, up to
 //                                      the order of the tokens inside a step, which V^T takes over
-//   S^T [v, d] += (w V)^T K            both operands through transposing LDS reads (ds_read_b64_tr_b16)
+//   S [d, v] += K^T (w V)              both operands through transposing LDS reads (ds_read_b64_tr_b16)
 // What the recurrence keeps in 32 bits - the state, the decayed scores, the decayed values - enters a product as the sum of two
 // bf16 numbers (value = hi + lo, 16 significant bits), at the price of a second MFMA.
 //
@@ -41,7 +41,6 @@ struct ChunkArgs {
   float k_scale;
   float* seg_state;             // [n][heads][vd][pitch], or nullptr: one segment per sequence
   float* seg_decay;             // [n][heads]: natural logarithm of the segment's total decay
-  bool vec_qk, vec_v;
 };
 
 template <int DP, int VT>
@@ -50,48 +49,105 @@ struct ChunkShape {
   static constexpr int kPitch = DP + 8;                   // elements; keeps 16-byte rows off each other's banks
   static constexpr int kVPitch = VT + 8;
   static constexpr int kQ = kChunk * kPitch, kV = kChunk * kVPitch, kS = VT * kPitch;
-  static constexpr int bytes(bool state_only) { return ((state_only ? 0 : kQ + 2 * kS) + kQ + kV) * 2 + 3 * kChunk * 4; }
+  static constexpr int bytes(bool state_only) { return ((state_only ? 0 : kQ + 2 * kS) + kQ + kV) * 2 + (3 * kChunk + 32) * 4; }
 };
 
-// Tile rows [0, 64) x columns [0, DP) of q or k: rotated, scaled, rounded to bf16, zeros outside [0, n) x [0, d).
-template <int DP, int THREADS>
-__device__ __forceinline__ void load_qk_tile(uint16_t* tile, const uint16_t* src, int64_t stride, int n, int pos0, const ChunkArgs& a,
-                                             float scale, bool vec) {
-  constexpr int kPitch = DP + 8;
-  const int half = a.rot >> 1;
-  if (vec) {
-#pragma unroll 2
-    for (int i = threadIdx.x; i < kChunk * (DP / 8); i += THREADS) {
-      const int r = i / (DP / 8), c = (i % (DP / 8)) * 8;
-      u32x4 w = {0u, 0u, 0u, 0u};
-      if (r < n && c < a.d) {
-        w = load16(src + r * stride + c);
-        if (c < a.rot || scale != 1.f) {
-          float x[8];
+// q, k and v rows of a chunk on their way from memory into the LDS tiles: q and k rotated, scaled and rounded to bf16, zeros
+// outside the chunk and the head.  fetch() issues every load of a chunk at once, so that it can be called while the chunk
+// before is still being worked on; store() finishes the values and writes the tiles.
+// A thread owns pairs of 16-byte pieces of a row, for q and k alike: pair p < rot / 16 is columns (8p, 8p + rot/2), which
+// rotate with each other; the pairs behind take two pieces that pass unchanged.
+template <int DP, int VT, bool STATE_ONLY, int PAIRS>
+struct ChunkLoader {
+  static constexpr int kThreads = ChunkShape<DP, VT>::kThreads, kPitch = DP + 8, kVPitch = VT + 8;
+  static constexpr int kVPieces = kChunk * (VT / 8) / kThreads;
+  u32x4 k[PAIRS][2], q[STATE_ONLY ? 1 : PAIRS][2], v[kVPieces];
+  float cs[PAIRS][8], sn[PAIRS][8];
+
+  static __device__ __forceinline__ bool place(int i, const ChunkArgs& a, int& r, int& c0, int& c1, bool& rotates) {
+    r = i / (DP / 16);
+    const int p = i % (DP / 16), half = a.rot >> 1;
+    rotates = 8 * p < half;
+    c0 = rotates ? 8 * p : 16 * p;       // behind the rotated pairs: rot + 16 (p - rot / 16) = 16 p
+    c1 = rotates ? c0 + half : c0 + 8;
+    return i < kChunk * (DP / 16);
+  }
+  __device__ __forceinline__ void fetch_qk(int first, const uint16_t* kp, const uint16_t* qp, int n, const ChunkArgs& a) {
 #pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            x[2 * e] = bf16lo_to_f32(w[e]);
-            x[2 * e + 1] = bf16hi_to_f32(w[e]);
-          }
-          if (c < a.rot) {
-            const bool lower = c < half;
-            float mate[8], cs[8], sn[8];
-            load_vec<8>(reinterpret_cast<const bf16_t*>(src + r * stride + (lower ? c + half : c - half)), mate);
-            const int64_t pos = pos0 + r < a.max_positions ? pos0 + r : a.max_positions - 1;
-            const float* trig = a.cos_sin + pos * a.rot + (lower ? c : c - half);
-            load_vec<8>(trig, cs);
-            load_vec<8>(trig + half, sn);
+    for (int j = 0; j < PAIRS; ++j) {
+      int r, c0, c1;
+      bool rotates;
+      const bool in = place((first + j) * kThreads + (int)threadIdx.x, a, r, c0, c1, rotates) && r < n;
+      const u32x4 zero = {0u, 0u, 0u, 0u};
+      k[j][0] = in && c0 < a.d ? load16(kp + r * a.k_stride + c0) : zero;
+      k[j][1] = in && c1 < a.d ? load16(kp + r * a.k_stride + c1) : zero;
+      if (!STATE_ONLY) {
+        q[j][0] = in && c0 < a.d ? load16(qp + r * a.q_stride + c0) : zero;
+        q[j][1] = in && c1 < a.d ? load16(qp + r * a.q_stride + c1) : zero;
+      }
+    }
+  }
+  __device__ __forceinline__ void fetch_trig(int first, int n, int pos0, const ChunkArgs& a) {
 #pragma unroll
-            for (int e = 0; e < 8; ++e) x[e] = x[e] * cs[e] + (lower ? -mate[e] : mate[e]) * sn[e];
-          }
+    for (int j = 0; j < PAIRS; ++j) {
+      int r, c0, c1;
+      bool rotates;
+      const bool in = place((first + j) * kThreads + (int)threadIdx.x, a, r, c0, c1, rotates) && r < n;
+      if (in && rotates) {
+        const int64_t pos = pos0 + r < a.max_positions ? pos0 + r : a.max_positions - 1;
+        load_vec<8>(a.cos_sin + pos * a.rot + c0, cs[j]);
+        load_vec<8>(a.cos_sin + pos * a.rot + (a.rot >> 1) + c0, sn[j]);
+      } else {
 #pragma unroll
-          for (int e = 0; e < 4; ++e) w[e] = pack_bf16x2(x[2 * e] * scale, x[2 * e + 1] * scale);
+        for (int e = 0; e < 8; ++e) {
+          cs[j][e] = 1.f;
+          sn[j][e] = 0.f;
         }
       }
-      store16(tile + r * kPitch + c, w);
     }
-    return;
   }
+  __device__ __forceinline__ void fetch_v(const uint16_t* vp, int n, int vlen, const ChunkArgs& a) {
+#pragma unroll
+    for (int j = 0; j < kVPieces; ++j) {
+      const int i = j * kThreads + (int)threadIdx.x, r = i / (VT / 8), c = (i % (VT / 8)) * 8;
+      v[j] = r < n && c < vlen ? load16(vp + r * a.v_stride + c) : u32x4{0u, 0u, 0u, 0u};
+    }
+  }
+  static __device__ __forceinline__ void finish(uint16_t* tile, int at0, int at1, const u32x4 (&w)[2], const float (&cs)[8], const float (&sn)[8],
+                                                float scale) {
+    u32x4 o0, o1;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const float x0 = bf16lo_to_f32(w[0][e]), x1 = bf16hi_to_f32(w[0][e]), y0 = bf16lo_to_f32(w[1][e]), y1 = bf16hi_to_f32(w[1][e]);
+      o0[e] = pack_bf16x2((x0 * cs[2 * e] - y0 * sn[2 * e]) * scale, (x1 * cs[2 * e + 1] - y1 * sn[2 * e + 1]) * scale);
+      o1[e] = pack_bf16x2((y0 * cs[2 * e] + x0 * sn[2 * e]) * scale, (y1 * cs[2 * e + 1] + x1 * sn[2 * e + 1]) * scale);
+    }
+    store16(tile + at0, o0);
+    store16(tile + at1, o1);
+  }
+  __device__ __forceinline__ void store_qk(int first, uint16_t* tk, uint16_t* tq, const ChunkArgs& a) const {
+#pragma unroll
+    for (int j = 0; j < PAIRS; ++j) {
+      int r, c0, c1;
+      bool rotates;
+      if (!place((first + j) * kThreads + (int)threadIdx.x, a, r, c0, c1, rotates)) continue;
+      finish(tk, r * kPitch + c0, r * kPitch + c1, k[j], cs[j], sn[j], a.k_scale);
+      if (!STATE_ONLY) finish(tq, r * kPitch + c0, r * kPitch + c1, q[j], cs[j], sn[j], 1.f);
+    }
+  }
+  __device__ __forceinline__ void store_v(uint16_t* tv) const {
+#pragma unroll
+    for (int j = 0; j < kVPieces; ++j) {
+      const int i = j * kThreads + (int)threadIdx.x;
+      store16(tv + i / (VT / 8) * kVPitch + (i % (VT / 8)) * 8, v[j]);
+    }
+  }
+};
+
+// The same for any alignment, element by element.
+template <int DP, int THREADS>
+__device__ __forceinline__ void load_tile_scalar(uint16_t* tile, const uint16_t* src, int64_t stride, int n, int pos0, const ChunkArgs& a, float scale) {
+  const int half = a.rot >> 1;
 #pragma unroll 1
   for (int i = threadIdx.x; i < kChunk * DP; i += THREADS) {
     const int r = i / DP, c = i % DP;
@@ -107,11 +163,11 @@ __device__ __forceinline__ void load_qk_tile(uint16_t* tile, const uint16_t* src
       }
       x *= scale;
     }
-    tile[r * kPitch + c] = (uint16_t)f32_to_bf16_bits(x);
+    tile[r * (DP + 8) + c] = (uint16_t)f32_to_bf16_bits(x);
   }
 }
 
-template <int DP, int VT, bool STATE_ONLY>
+template <int DP, int VT, bool STATE_ONLY, bool VEC>
 __global__ __launch_bounds__(VT * 4, 2) void decayed_chunk_kernel(const ChunkArgs a) {
   using S = ChunkShape<DP, VT>;
   constexpr int kVTiles = VT / 32;
@@ -124,6 +180,7 @@ __global__ __launch_bounds__(VT * 4, 2) void decayed_chunk_kernel(const ChunkArg
   uint16_t* const ts_lo = ts_hi + S::kS;
   float* const cum = reinterpret_cast<float*>(STATE_ONLY ? tq : ts_lo + S::kS);   // [64] L, base 2
   float* const scl = cum + kChunk;                                                  // [64] input scale
+  float* const wgt0 = scl + 2 * kChunk;                                             // [32] scale * 2^(L_31 - L)
   float* const wgt = scl + kChunk;                                                  // [64] scale * 2^(L_end - L)
 
   // consecutive workgroups go to different XCDs: give each XCD a contiguous run of items, so that the tiles and heads that
@@ -150,10 +207,11 @@ __global__ __launch_bounds__(VT * 4, 2) void decayed_chunk_kernel(const ChunkArg
   const float la_const = a.log_decay ? a.log_decay[h] * kLog2e : 0.f;
   const float dt_bias = a.dt ? a.dt_bias[h] : 0.f, neg_a = a.dt ? a.neg_a[h] * kLog2e : 0.f;
 
-  // S^T: rows v0 + 32 vt + .., columns 32 * (half_id * kDTiles + i) + (lane & 31)
+  // S: rows d = 32 (half_id kDTiles + i) + 8 q + 4 hh + e (four consecutive ones per q), column v0 + 32 vt + (lane & 31)
   f32x16 st[kDTiles];
   const bool has_state_tile = half_id * kDTiles * 32 < DP;
-  auto state_row = [&](int r) { return 32 * vt + 8 * (r >> 2) + 4 * hh + (r & 3); };
+  const int v_col = 32 * vt + col;
+  auto state_d = [&](int i, int q4) { return 32 * (half_id * kDTiles + i) + 8 * q4 + 4 * hh; };
   float* gstate = nullptr;
   bool load_state = false;
   if (!STATE_ONLY) {
@@ -166,32 +224,51 @@ __global__ __launch_bounds__(VT * 4, 2) void decayed_chunk_kernel(const ChunkArg
     }
   }
 #pragma unroll
-  for (int i = 0; i < kDTiles; ++i) {
-    const int c = 32 * (half_id * kDTiles + i) + col;
+  for (int i = 0; i < kDTiles; ++i)
 #pragma unroll
-    for (int r = 0; r < 16; ++r) {
+    for (int q4 = 0; q4 < 4; ++q4) {
       // no branch per element (the accumulators would be copied at each): every lane reads some valid element, then selects
-      const bool ok = load_state && c < a.pitch && state_row(r) < vlen;
-      const float x = STATE_ONLY ? 0.f : gstate[ok ? state_row(r) * a.pitch + c : 0];
-      st[i][r] = ok ? x : 0.f;
+      const bool ok = load_state && state_d(i, q4) < a.pitch && v_col < vlen;
+      f32x4 x = {0.f, 0.f, 0.f, 0.f};
+      if (!STATE_ONLY) x = *reinterpret_cast<const f32x4*>(gstate + (ok ? v_col * a.pitch + state_d(i, q4) : 0));
+#pragma unroll
+      for (int e = 0; e < 4; ++e) st[i][4 * q4 + e] = ok ? x[e] : 0.f;
     }
-  }
 
+  constexpr int kPairsAll = (kChunk * (DP / 16) + S::kThreads - 1) / S::kThreads;
+  constexpr bool kAhead = VEC && kPairsAll <= 2;          // a whole chunk fits the registers next to the accumulators
+  constexpr int kPairs = kPairsAll <= 2 ? kPairsAll : 2;
+  ChunkLoader<DP, VT, STATE_ONLY, kPairs> ld;
+  float dt_next = 0.f;
+  auto fetch = [&](int t) {
+    const int m = t_end - t < kChunk ? t_end - t : kChunk;
+    ld.fetch_qk(0, kp + (int64_t)t * a.k_stride, qp + (int64_t)t * a.q_stride, m, a);
+    ld.fetch_trig(0, m, start + (t - seq_begin), a);
+    ld.fetch_v(vp + (int64_t)t * a.v_stride, m, vlen, a);
+  };
+  auto fetch_dt = [&](int t) { dt_next = a.dt && wave == 0 && t + lane < t_end ? bf16lo_to_f32(a.dt[(int64_t)(t + lane) * a.dt_stride + h]) : 0.f; };
+  if (kAhead) fetch(t_begin);
+  fetch_dt(t_begin);
   float total_log = 0.f;
   for (int t0 = t_begin; t0 < t_end; t0 += kChunk) {
     const int n = t_end - t0 < kChunk ? t_end - t0 : kChunk;
     const int pos0 = start + (t0 - seq_begin);
     __syncthreads();     // the last chunk's tiles have been read
-    load_qk_tile<DP, S::kThreads>(tk, kp + (int64_t)t0 * a.k_stride, a.k_stride, n, pos0, a, a.k_scale, a.vec_qk);
-    if (!STATE_ONLY) load_qk_tile<DP, S::kThreads>(tq, qp + (int64_t)t0 * a.q_stride, a.q_stride, n, pos0, a, 1.f, a.vec_qk);
-    if (a.vec_v) {
-      for (int i = threadIdx.x; i < kChunk * (VT / 8); i += S::kThreads) {
-        const int r = i / (VT / 8), c = (i % (VT / 8)) * 8;
-        u32x4 w = {0u, 0u, 0u, 0u};
-        if (r < n && c < vlen) w = load16(vp + (int64_t)(t0 + r) * a.v_stride + c);
-        store16(tv + r * S::kVPitch + c, w);
+    if (kAhead) {
+      ld.store_qk(0, tk, tq, a);
+      ld.store_v(tv);
+    } else if (VEC) {
+      ld.fetch_v(vp + (int64_t)t0 * a.v_stride, n, vlen, a);
+#pragma unroll 1
+      for (int first = 0; first < kPairsAll; first += kPairs) {
+        ld.fetch_qk(first, kp + (int64_t)t0 * a.k_stride, qp + (int64_t)t0 * a.q_stride, n, a);
+        ld.fetch_trig(first, n, pos0, a);
+        ld.store_qk(first, tk, tq, a);
       }
+      ld.store_v(tv);
     } else {
+      load_tile_scalar<DP, S::kThreads>(tk, kp + (int64_t)t0 * a.k_stride, a.k_stride, n, pos0, a, a.k_scale);
+      if (!STATE_ONLY) load_tile_scalar<DP, S::kThreads>(tq, qp + (int64_t)t0 * a.q_stride, a.q_stride, n, pos0, a, 1.f);
 #pragma unroll 1
       for (int i = threadIdx.x; i < kChunk * VT; i += S::kThreads) {
         const int r = i / VT, c = i % VT;
@@ -202,7 +279,7 @@ __global__ __launch_bounds__(VT * 4, 2) void decayed_chunk_kernel(const ChunkArg
       float la = 0.f, s = 0.f, l;
       if (a.dt) {
         if (lane < n) {
-          s = softplus_f32(bf16lo_to_f32(a.dt[(int64_t)(t0 + lane) * a.dt_stride + h]) + dt_bias);
+          s = softplus_f32(dt_next + dt_bias);
           la = neg_a * s;
         }
         l = la;
@@ -219,22 +296,26 @@ __global__ __launch_bounds__(VT * 4, 2) void decayed_chunk_kernel(const ChunkArg
       cum[lane] = l;
       scl[lane] = s;
       wgt[lane] = s * __builtin_amdgcn_exp2f(l_end - l);
+      const float l_mid = __shfl(l, 31, 64);
+      if (lane < 32) wgt0[lane] = s * __builtin_amdgcn_exp2f(l_mid - l);
     }
     if (!STATE_ONLY && has_state_tile) {
 #pragma unroll
-      for (int i = 0; i < kDTiles; ++i) {
-        const int c = 32 * (half_id * kDTiles + i) + col;
+      for (int i = 0; i < kDTiles; ++i)
 #pragma unroll
-        for (int r = 0; r < 16; ++r) {
-          const float hi = round_to_bf16(st[i][r]);
-          ts_hi[state_row(r) * S::kPitch + c] = (uint16_t)(__float_as_uint(hi) >> 16);
-          ts_lo[state_row(r) * S::kPitch + c] = (uint16_t)f32_to_bf16_bits(st[i][r] - hi);
+        for (int q4 = 0; q4 < 4; ++q4) {
+          const uint32_t h0 = pack_bf16x2(st[i][4 * q4], st[i][4 * q4 + 1]), h1 = pack_bf16x2(st[i][4 * q4 + 2], st[i][4 * q4 + 3]);
+          const uint32_t l0 = pack_bf16x2(st[i][4 * q4] - bf16lo_to_f32(h0), st[i][4 * q4 + 1] - bf16hi_to_f32(h0));
+          const uint32_t l1 = pack_bf16x2(st[i][4 * q4 + 2] - bf16lo_to_f32(h1), st[i][4 * q4 + 3] - bf16hi_to_f32(h1));
+          *reinterpret_cast<u32x2*>(ts_hi + v_col * S::kPitch + state_d(i, q4)) = u32x2{h0, h1};
+          *reinterpret_cast<u32x2*>(ts_lo + v_col * S::kPitch + state_d(i, q4)) = u32x2{l0, l1};
         }
-      }
     }
     __syncthreads();
     const float l_end = cum[kChunk - 1];
     total_log += l_end;
+    const bool more = t0 + kChunk < t_end;
+    if (more) fetch_dt(t0 + kChunk);
 
     if (!STATE_ONLY) {
       const int i_tok = 32 * half_id + col;      // this lane's output token
@@ -248,7 +329,7 @@ __global__ __launch_bounds__(VT * 4, 2) void decayed_chunk_kernel(const ChunkArg
         o = mfma32(tile_row(ts_hi, S::kPitch, 32 * vt + col, 16 * kk + 8 * hh), qb, o);
         o = mfma32(tile_row(ts_lo, S::kPitch, 32 * vt + col, 16 * kk + 8 * hh), qb, o);
       }
-      const float e_i = __builtin_amdgcn_exp2f(l_i);
+      const float e_i = __builtin_amdgcn_exp2f(l_i), e_mid = __builtin_amdgcn_exp2f(half_id ? l_i - cum[31] : 0.f);
 #pragma unroll
       for (int r = 0; r < 16; ++r) o[r] *= e_i;
       for (int jt = 0; jt <= half_id; ++jt) {
@@ -265,7 +346,9 @@ __global__ __launch_bounds__(VT * 4, 2) void decayed_chunk_kernel(const ChunkArg
 #pragma unroll
           for (int e = 0; e < 8; ++e) {
             const int j = j0 + (e & 3) + 8 * (e >> 2);
-            pv[e] = j <= i_tok ? p[8 * ks + e] * (scl[j] * __builtin_amdgcn_exp2f(l_i - cum[j])) : 0.f;
+            // below the diagonal tile the weight is a product of one factor per token on either side of the tile border
+            if (jt < half_id) pv[e] = p[8 * ks + e] * (wgt0[j] * e_mid);
+            else pv[e] = j <= i_tok ? p[8 * ks + e] * (scl[j] * __builtin_amdgcn_exp2f(l_i - cum[j])) : 0.f;
           }
           bf16x8 hi, lo;
           split8(pv, hi, lo);
@@ -274,25 +357,37 @@ __global__ __launch_bounds__(VT * 4, 2) void decayed_chunk_kernel(const ChunkArg
           o = mfma32(va, lo, o);
         }
       }
-      if (i_tok < n) {
-        uint16_t* orow = a.out + (int64_t)(t0 + i_tok) * a.out_stride + (int64_t)h * a.vd + v0;
+      if (skip != 0.f) {
 #pragma unroll
-        for (int q4 = 0; q4 < 4; ++q4) {
-          const int v = 32 * vt + 8 * q4 + 4 * hh;
-          float x[4];
+        for (int q4 = 0; q4 < 4; ++q4)
 #pragma unroll
-          for (int e = 0; e < 4; ++e) x[e] = o[4 * q4 + e] + skip * bf16lo_to_f32(tv[i_tok * S::kVPitch + v + e]);
-          if (a.vec_v && v + 4 <= vlen) {
-            *reinterpret_cast<u32x2*>(orow + v) = u32x2{pack_bf16x2(x[0], x[1]), pack_bf16x2(x[2], x[3])};
+          for (int e = 0; e < 4; ++e)
+            o[4 * q4 + e] += skip * bf16lo_to_f32(tv[i_tok * S::kVPitch + 32 * vt + 8 * q4 + 4 * hh + e]);
+      }
+      uint16_t* orow = a.out + (int64_t)(t0 + i_tok) * a.out_stride + (int64_t)h * a.vd + v0;
+#pragma unroll
+      for (int half = 0; half < 2; ++half) {
+        // eight consecutive columns per lane: the lower half of the wave completes piece 2 half, the upper half 2 half + 1
+        const u32x2 even = {pack_bf16x2(o[8 * half], o[8 * half + 1]), pack_bf16x2(o[8 * half + 2], o[8 * half + 3])};
+        const u32x2 odd = {pack_bf16x2(o[8 * half + 4], o[8 * half + 5]), pack_bf16x2(o[8 * half + 6], o[8 * half + 7])};
+        const u32x2 mine = hh ? odd : even, give = hh ? even : odd;
+        const u32x2 got = {(uint32_t)__shfl_xor((int)give[0], 32, 64), (uint32_t)__shfl_xor((int)give[1], 32, 64)};
+        const u32x4 w = hh ? u32x4{got[0], got[1], mine[0], mine[1]} : u32x4{mine[0], mine[1], got[0], got[1]};
+        const int v = 32 * vt + 16 * half + 8 * hh;
+        if (i_tok < n) {
+          if (VEC) {
+            if (v < vlen) store16(orow + v, w);
           } else {
 #pragma unroll
-            for (int e = 0; e < 4; ++e)
-              if (v + e < vlen) orow[v + e] = (uint16_t)f32_to_bf16_bits(x[e]);
+            for (int e = 0; e < 8; ++e)
+              if (v + e < vlen) orow[v + e] = (uint16_t)(w[e >> 1] >> (16 * (e & 1)));
           }
         }
       }
     }
-    // ---- S^T <- e^{L_end} S^T + (w V)^T K
+    // the next chunk is on its way while the state takes this one in
+    if (kAhead && more) fetch(t0 + kChunk);
+    // ---- S <- e^{L_end} S + K^T (w V)
     if (has_state_tile) {
       const float e_end = __builtin_amdgcn_exp2f(l_end);
 #pragma unroll
@@ -310,9 +405,9 @@ __global__ __launch_bounds__(VT * 4, 2) void decayed_chunk_kernel(const ChunkArg
         split8(x, hi, lo);
 #pragma unroll
         for (int i = 0; i < kDTiles; ++i) {
-          const bf16x8 kb = __builtin_bit_cast(bf16x8, tile_columns(tk, S::kPitch, j0, j0 + 8, 32 * (half_id * kDTiles + i), lane));
-          st[i] = mfma32(hi, kb, st[i]);
-          st[i] = mfma32(lo, kb, st[i]);
+          const bf16x8 ka = __builtin_bit_cast(bf16x8, tile_columns(tk, S::kPitch, j0, j0 + 8, 32 * (half_id * kDTiles + i), lane));
+          st[i] = mfma32(ka, hi, st[i]);
+          st[i] = mfma32(ka, lo, st[i]);
         }
       }
     }
@@ -322,21 +417,12 @@ __global__ __launch_bounds__(VT * 4, 2) void decayed_chunk_kernel(const ChunkArg
   if (STATE_ONLY) dst = a.seg_state + (((int64_t)seg * a.heads + h) * a.vd + v0) * a.pitch;
   else if (!a.seg_state) dst = gstate;
   if (dst && has_state_tile) {
-    // the addresses and bounds are those of the load in front of the loop; the compiler must not keep them in registers
-    // all the way, so it is not told that this is the same lane number
-    int again = lane;
-    asm volatile("" : "+v"(again));
-    const int c0 = again & 31, r0 = 32 * vt + 4 * (again >> 5);
 #pragma unroll
-    for (int i = 0; i < kDTiles; ++i) {
-      const int c = 32 * (half_id * kDTiles + i) + c0;
-      if (c < a.pitch)
+    for (int i = 0; i < kDTiles; ++i)
 #pragma unroll
-        for (int r = 0; r < 16; ++r) {
-          const int row = r0 + 8 * (r >> 2) + (r & 3);
-          if (row < vlen) dst[(int64_t)row * a.pitch + c] = st[i][r];
-        }
-    }
+      for (int q4 = 0; q4 < 4; ++q4)
+        if (v_col < vlen && state_d(i, q4) < a.pitch)
+          *reinterpret_cast<f32x4*>(dst + v_col * a.pitch + state_d(i, q4)) = f32x4{st[i][4 * q4], st[i][4 * q4 + 1], st[i][4 * q4 + 2], st[i][4 * q4 + 3]};
   }
   if (STATE_ONLY && v0 == 0 && threadIdx.x == 0) a.seg_decay[(int64_t)seg * a.heads + h] = total_log;
 }
@@ -363,23 +449,23 @@ __global__ __launch_bounds__(256) void decayed_segment_scan_kernel(const ChunkAr
   *reinterpret_cast<f32x4*>(gs) = s;
 }
 
-template <int DP, int VT>
+template <int DP, int VT, bool VEC>
 static int launch_chunks(const ChunkArgs& a, const int32_t* seq_segments, int64_t batch, hipStream_t s) {
   using S = ChunkShape<DP, VT>;
   const int64_t items = (int64_t)a.num_segments * a.heads * ((a.vd + VT - 1) / VT);
   const dim3 grid((unsigned)((items + 7) / 8 * 8)), block(S::kThreads);
-  static const hipError_t lds = hipFuncSetAttribute(reinterpret_cast<const void*>(&decayed_chunk_kernel<DP, VT, false>),
+  static const hipError_t lds = hipFuncSetAttribute(reinterpret_cast<const void*>(&decayed_chunk_kernel<DP, VT, false, VEC>),
                                                     hipFuncAttributeMaxDynamicSharedMemorySize, S::bytes(false));
-  static const hipError_t lds_state = hipFuncSetAttribute(reinterpret_cast<const void*>(&decayed_chunk_kernel<DP, VT, true>),
+  static const hipError_t lds_state = hipFuncSetAttribute(reinterpret_cast<const void*>(&decayed_chunk_kernel<DP, VT, true, VEC>),
                                                           hipFuncAttributeMaxDynamicSharedMemorySize, S::bytes(true));
   if (lds != hipSuccess) return record_hip_error(lds);
   if (lds_state != hipSuccess) return record_hip_error(lds_state);
   if (a.seg_state) {
-    hipLaunchKernelGGL((decayed_chunk_kernel<DP, VT, true>), grid, block, S::bytes(true), s, a);
+    hipLaunchKernelGGL((decayed_chunk_kernel<DP, VT, true, VEC>), grid, block, S::bytes(true), s, a);
     const int64_t quads = ((int64_t)a.vd * a.pitch / 4 + 255) / 256;
     hipLaunchKernelGGL(decayed_segment_scan_kernel, dim3((unsigned)quads, (unsigned)a.heads, (unsigned)batch), dim3(256), 0, s, a, seq_segments);
   }
-  hipLaunchKernelGGL((decayed_chunk_kernel<DP, VT, false>), grid, block, S::bytes(false), s, a);
+  hipLaunchKernelGGL((decayed_chunk_kernel<DP, VT, false, VEC>), grid, block, S::bytes(false), s, a);
   return finish_launch();
 }
 
@@ -414,11 +500,12 @@ extern "C" int mops_hip_decayed_chunks(const mops_hip_recurrence* r, const int32
   a.log_decay = r->log_decay; a.dt_bias = r->dt_bias; a.neg_a = r->neg_a; a.skip = r->skip; a.cos_sin = r->cos_sin;
   a.rot = (int)r->rot; a.max_positions = r->max_positions; a.k_scale = r->k_scale;
   a.seg_state = seg_state; a.seg_decay = seg_decay;
-  a.vec_qk = r->d % 8 == 0 && r->q_stride % 8 == 0 && r->k_stride % 8 == 0 && aligned16(r->q) && aligned16(r->k) &&
-             (r->rot == 0 || ((r->rot / 2) % 8 == 0 && aligned16(r->cos_sin)));
-  a.vec_v = r->vd % 8 == 0 && r->v_stride % 8 == 0 && r->out_stride % 8 == 0 && aligned16(r->v) && aligned16(r->out);
+  const bool vec = r->d % 8 == 0 && r->q_stride % 8 == 0 && r->k_stride % 8 == 0 && aligned16(r->q) && aligned16(r->k) &&
+                   (r->rot == 0 || (r->rot % 16 == 0 && aligned16(r->cos_sin))) && r->vd % 8 == 0 && r->v_stride % 8 == 0 &&
+                   r->out_stride % 8 == 0 && aligned16(r->v) && aligned16(r->out);
   hipStream_t s = (hipStream_t)stream;
-#define MOPS_CHUNKS(D) (a.vd <= 32 ? launch_chunks<D, 32>(a, seq_segments, r->batch, s) : launch_chunks<D, 64>(a, seq_segments, r->batch, s))
+  if (!vec) return a.d <= 64 ? launch_chunks<64, 64, false>(a, seq_segments, r->batch, s) : launch_chunks<256, 64, false>(a, seq_segments, r->batch, s);
+#define MOPS_CHUNKS(D) (a.vd <= 32 ? launch_chunks<D, 32, true>(a, seq_segments, r->batch, s) : launch_chunks<D, 64, true>(a, seq_segments, r->batch, s))
   if (a.d <= 32) return MOPS_CHUNKS(32);
   if (a.d <= 64) return MOPS_CHUNKS(64);
   if (a.d <= 128) return MOPS_CHUNKS(128);

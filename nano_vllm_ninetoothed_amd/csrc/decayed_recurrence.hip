@@ -246,36 +246,57 @@ __global__ __launch_bounds__(256) void short_conv_run_kernel(const T* __restrict
 #pragma unroll
   for (int l = 0; l < TAPS; ++l) load_vec<8>(w + (int64_t)(TAPS - 1 - l) * channels + c, wv[l]);
   load_vec<8>(bias + c, b);
-  int seq = -1;
-  for (int64_t t = t0; t < t1; ++t) {
-    const int s = token_seq[t];
-    if (s != seq) {      // the window in front of this token: rows of the portion, the ring behind them, zeros before the start
-      seq = s;
-      const int slot = state_slots[s], in_portion = (int)t - cu_seqlens[s], pos = starts[s] + in_portion;
+  // the window in front of token t: rows of the portion, the ring behind them, zeros before the start
+  auto fill = [&](int64_t t, int sq) {
+    const int slot = state_slots[sq], in_portion = (int)t - cu_seqlens[sq], pos = starts[sq] + in_portion;
 #pragma unroll
-      for (int l = 1; l < TAPS; ++l) {
+    for (int l = 1; l < TAPS; ++l) {
 #pragma unroll
-        for (int e = 0; e < 8; ++e) win[l - 1][e] = 0.f;
-        if (pos - l >= 0) {
-          if (l <= in_portion) load_vec<8>(x + (t - l) * x_stride + c, win[l - 1]);
-          else if (slot >= 0 && slot < num_slots) load_vec<8>(ring + ((int64_t)slot * TAPS + (pos - l) % TAPS) * channels + c, win[l - 1]);
-        }
+      for (int e = 0; e < 8; ++e) win[l - 1][e] = 0.f;
+      if (pos - l >= 0) {
+        if (l <= in_portion) load_vec<8>(x + (t - l) * x_stride + c, win[l - 1]);
+        else if (slot >= 0 && slot < num_slots) load_vec<8>(ring + ((int64_t)slot * TAPS + (pos - l) % TAPS) * channels + c, win[l - 1]);
       }
     }
+  };
+  auto next = [&](int64_t t, const float (&in)[8]) {
 #pragma unroll
     for (int l = TAPS - 1; l > 0; --l)
 #pragma unroll
       for (int e = 0; e < 8; ++e) win[l][e] = win[l - 1][e];
-    load_vec<8>(x + t * x_stride + c, win[0]);
     float acc[8];
 #pragma unroll
     for (int e = 0; e < 8; ++e) {
+      win[0][e] = in[e];
       acc[e] = b[e];
 #pragma unroll
       for (int l = 0; l < TAPS; ++l) acc[e] += wv[l][e] * win[l][e];
       acc[e] = silu_f32(acc[e]);
     }
     store_vec<8>(out + t * channels + c, acc);
+  };
+  int seq = token_seq[t0];
+  fill(t0, seq);
+  if (t1 - t0 == kConvRun && token_seq[t1 - 1] == seq) {      // one sequence throughout: inputs four tokens ahead
+#pragma unroll
+    for (int j = 0; j < kConvRun; j += 4) {
+      float in[4][8];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) load_vec<8>(x + (t0 + j + i) * x_stride + c, in[i]);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) next(t0 + j + i, in[i]);
+    }
+    return;
+  }
+  for (int64_t t = t0; t < t1; ++t) {
+    const int sq = token_seq[t];
+    if (sq != seq) {
+      seq = sq;
+      fill(t, sq);
+    }
+    float in[8];
+    load_vec<8>(x + t * x_stride + c, in);
+    next(t, in);
   }
 }
 

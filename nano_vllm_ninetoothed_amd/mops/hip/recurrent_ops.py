@@ -328,7 +328,7 @@ def latent_decode(q_latent, q_rot, cache, cos_sin, context_lens, block_table, sc
     out = torch.empty_like(q_latent)
     a = _latent_rows(q_latent, q_rot, cache, cos_sin, context_lens, block_table, scale, row_seq, out)
     lib = _capi.load()
-    nbytes = lib.mops_hip_latent_decode_workspace_bytes(a.rows, a.heads, a.kv_rank, a.max_blocks, a.block_size)
+    nbytes = lib.mops_hip_latent_decode_workspace_bytes(a.rows, a.heads, a.kv_rank, a.rot_dim)
     ws = torch.empty(max(nbytes, 16), dtype=torch.uint8, device=out.device)
     st = lib.mops_hip_latent_decode(byref(a), ws.data_ptr(), ws.numel(), _stream(q_latent))
     _capi.check("mops_hip_latent_decode", st)
