@@ -375,7 +375,7 @@ int mops_hip_clamped_glu(const void* gate, int64_t gate_row_stride, const void* 
  * row, out is zeros and nothing is stored.
  * conv_weight != NULL (one token per sequence only): the short convolution of mops_hip_short_conv is applied to q, k and v
  * on the way in, channels q_channel.. k_channel.. v_channel.. of `channels`, and the ring receives the token.
- * d <= 256.
+ * d <= 512.
  */
 typedef struct {
   const void *q, *k, *v;
@@ -399,13 +399,14 @@ int64_t mops_hip_recurrence_state_pitch(int64_t d);
 int mops_hip_decayed_recurrence(const mops_hip_recurrence* r, void* stream);
 
 /*
- * The same for portions of many tokens, 64 tokens at a time on the matrix cores (csrc/decayed_chunks.hip).  bf16 only, no
+ * The same for portions of many tokens, 64 tokens at a time on the matrix cores (csrc/decayed_chunks.hip).  bf16 only, d <= 256, no
  * convolution, cu_seqlens required; a constant decay is read from log_decay (natural logarithms, finite) instead of decay.
  * segments: int32 [num_segments][3] = (sequence, first token, one past the last); the segments of a sequence are consecutive,
  * in order, and cover it.  seg_state == NULL: one segment per sequence.  Otherwise seg_state: float [num_segments, heads,
  * vd, pitch], seg_decay: float [num_segments, heads] are scratch, and seq_segments: int32 [batch + 1] bounds each
- * sequence's segments.
+ * sequence's segments.  mops_hip_decayed_chunks_workgroups: workgroups one segment gives, for the choice of their number.
  */
+int64_t mops_hip_decayed_chunks_workgroups(int64_t heads, int64_t groups, int64_t vd);
 int mops_hip_decayed_chunks(const mops_hip_recurrence* r, const int32_t* segments, int64_t num_segments,
                             const int32_t* seq_segments, float* seg_state, float* seg_decay, void* stream);
 

@@ -219,7 +219,7 @@ def kernel_table(dev, seed=0, only=""):
         dts, oT = rnd(T, heads), torch.empty((T, inner), dtype=torch.bfloat16, device=dev)
         for nseq in (16, 1):
             cu = list(range(0, T + 1, T // nseq))
-            segs, bounds = R.recurrence_segments([T // nseq] * nseq, heads, vd)
+            segs, bounds = R.recurrence_segments([T // nseq] * nseq, heads, groups, vd)
             segs, bounds, cu = i32(segs), i32(bounds), i32(cu)
             more = {} if const else {"dt": dts}
             # least arithmetic at 64 tokens a chunk: scores and their product below the diagonal, state in and out

@@ -5,12 +5,14 @@
 //   O_i = e^{L_i} S^T q_i + sum_{j <= i} e^{L_i - L_j} s_j (q_i . k_j) v_j + skip v_i
 //   S  <- e^{L_end} S + sum_j e^{L_end - L_j} s_j k_j v_j^T
 //
-// Workgroup = (segment, head, tile of VT value columns), walking the chunks of its segment with S [d x VT] in the
-// accumulators.  All products are v_mfma_f32_32x32x16_bf16:
-//   P^T [j, i] = K Q^T                 rows of the two LDS tiles as they are
-//   O^T [v, i] = S^T Q^T + V^T P^T     the accumulator layout of P^T is the B-operand layout of the second product, up to
-//                                      the order of the tokens inside a step, which V^T takes over
-//   S [d, v] += K^T (w V)              both operands through transposing LDS reads (ds_read_b64_tr_b16)
+// Workgroup (four waves) = (segment, NH heads of one q/k group, 128 / NH value columns of each), walking the chunks of its
+// segment.  A wave owns 32 value columns of one head, with S [d x 32] in its accumulators from the first chunk to the last.
+// All products are v_mfma_f32_32x32x16_bf16:
+//   P^T [j, i] = K Q^T             one 32 x 32 tile per (head, tile below or on the diagonal), dealt out to the waves, weighted
+//                                  and left in LDS for all of them
+//   O^T [v, i] = S^T Q^T + V^T P^T S^T straight from the accumulators: their layout is an operand layout up to the order of the
+//                                  d's inside a step, which Q's reads follow; V^T through transposing LDS reads
+//   S [d, v]  += K^T (w V)         both operands through transposing LDS reads (ds_read_b64_tr_b16)
 // What the recurrence keeps in 32 bits - the state, the decayed scores, the decayed values - enters a product as the sum of two
 // bf16 numbers (value = hi + lo, 16 significant bits), at the price of a second MFMA.
 //
@@ -40,16 +42,19 @@ struct ChunkArgs {
   int64_t max_positions;
   float k_scale;
   float* seg_state;             // [n][heads][vd][pitch], or nullptr: one segment per sequence
-  float* seg_decay;             // [n][heads]: natural logarithm of the segment's total decay
+  float* seg_decay;             // [n][heads]: base-2 logarithm of the segment's total decay
 };
 
-template <int DP, int VT>
+constexpr int kColumns = 128, kVPitch = kColumns + 8;     // value columns of a workgroup
+constexpr int kPPitch = 32 + 8, kPTile = 32 * kPPitch;     // a weighted score tile [i][j]
+
+template <int DP, int NH>
 struct ChunkShape {
-  static constexpr int kThreads = VT * 4;                 // a wave per 32 x 32 tile of [VT, 64 tokens]
-  static constexpr int kPitch = DP + 8;                   // elements; keeps 16-byte rows off each other's banks
-  static constexpr int kVPitch = VT + 8;
-  static constexpr int kQ = kChunk * kPitch, kV = kChunk * kVPitch, kS = VT * kPitch;
-  static constexpr int bytes(bool state_only) { return ((state_only ? 0 : kQ + 2 * kS) + kQ + kV) * 2 + (3 * kChunk + 32) * 4; }
+  static constexpr int kPitch = DP + 8;                    // elements; keeps 16-byte rows off each other's banks
+  static constexpr int kK = kChunk * kPitch, kV = kChunk * kVPitch;
+  static constexpr int kP = NH * 3 * 2 * kPTile;           // hi and lo of three tiles per head; takes the place of Q
+  static constexpr int kQP = kK > kP ? kK : kP;
+  static constexpr int bytes(bool state_only) { return (kK + kV + (state_only ? 0 : kQP)) * 2 + NH * (3 * kChunk + 32) * 4; }
 };
 
 // q, k and v rows of a chunk on their way from memory into the LDS tiles: q and k rotated, scaled and rounded to bf16, zeros
@@ -57,17 +62,18 @@ struct ChunkShape {
 // before is still being worked on; store() finishes the values and writes the tiles.
 // A thread owns pairs of 16-byte pieces of a row, for q and k alike: pair p < rot / 16 is columns (8p, 8p + rot/2), which
 // rotate with each other; the pairs behind take two pieces that pass unchanged.
-template <int DP, int VT, bool STATE_ONLY, int PAIRS>
+// ROT: rotation is compiled in (the tables take 16 registers a pair).
+template <int DP, bool STATE_ONLY, int PAIRS, bool ROT>
 struct ChunkLoader {
-  static constexpr int kThreads = ChunkShape<DP, VT>::kThreads, kPitch = DP + 8, kVPitch = VT + 8;
-  static constexpr int kVPieces = kChunk * (VT / 8) / kThreads;
+  static constexpr int kThreads = 256, kPitch = DP + 8;
+  static constexpr int kVPieces = kChunk * (kColumns / 8) / kThreads;
   u32x4 k[PAIRS][2], q[STATE_ONLY ? 1 : PAIRS][2], v[kVPieces];
-  float cs[PAIRS][8], sn[PAIRS][8];
+  float cs[ROT ? PAIRS : 1][8], sn[ROT ? PAIRS : 1][8];
 
   static __device__ __forceinline__ bool place(int i, const ChunkArgs& a, int& r, int& c0, int& c1, bool& rotates) {
     r = i / (DP / 16);
     const int p = i % (DP / 16), half = a.rot >> 1;
-    rotates = 8 * p < half;
+    rotates = ROT && 8 * p < half;
     c0 = rotates ? 8 * p : 16 * p;       // behind the rotated pairs: rot + 16 (p - rot / 16) = 16 p
     c1 = rotates ? c0 + half : c0 + 8;
     return i < kChunk * (DP / 16);
@@ -88,6 +94,7 @@ struct ChunkLoader {
     }
   }
   __device__ __forceinline__ void fetch_trig(int first, int n, int pos0, const ChunkArgs& a) {
+    if (!ROT) return;
 #pragma unroll
     for (int j = 0; j < PAIRS; ++j) {
       int r, c0, c1;
@@ -106,21 +113,31 @@ struct ChunkLoader {
       }
     }
   }
-  __device__ __forceinline__ void fetch_v(const uint16_t* vp, int n, int vlen, const ChunkArgs& a) {
+  // vp: the first head's columns; column c of the tile is value column (c % span) of head c / span
+  __device__ __forceinline__ void fetch_v(const uint16_t* vp, int n, int span, int vlen, const ChunkArgs& a) {
 #pragma unroll
     for (int j = 0; j < kVPieces; ++j) {
-      const int i = j * kThreads + (int)threadIdx.x, r = i / (VT / 8), c = (i % (VT / 8)) * 8;
-      v[j] = r < n && c < vlen ? load16(vp + r * a.v_stride + c) : u32x4{0u, 0u, 0u, 0u};
+      const int i = j * kThreads + (int)threadIdx.x, r = i / (kColumns / 8), c = (i % (kColumns / 8)) * 8;
+      const int x = c % span, head = c / span;
+      v[j] = r < n && x < vlen ? load16(vp + r * a.v_stride + (int64_t)head * a.vd + x) : u32x4{0u, 0u, 0u, 0u};
     }
   }
-  static __device__ __forceinline__ void finish(uint16_t* tile, int at0, int at1, const u32x4 (&w)[2], const float (&cs)[8], const float (&sn)[8],
-                                                float scale) {
-    u32x4 o0, o1;
+  __device__ __forceinline__ void finish(uint16_t* tile, int at0, int at1, const u32x4 (&w)[2], int j, float scale) const {
+    u32x4 o0 = w[0], o1 = w[1];
+    if (ROT || scale != 1.f) {
 #pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const float x0 = bf16lo_to_f32(w[0][e]), x1 = bf16hi_to_f32(w[0][e]), y0 = bf16lo_to_f32(w[1][e]), y1 = bf16hi_to_f32(w[1][e]);
-      o0[e] = pack_bf16x2((x0 * cs[2 * e] - y0 * sn[2 * e]) * scale, (x1 * cs[2 * e + 1] - y1 * sn[2 * e + 1]) * scale);
-      o1[e] = pack_bf16x2((y0 * cs[2 * e] + x0 * sn[2 * e]) * scale, (y1 * cs[2 * e + 1] + x1 * sn[2 * e + 1]) * scale);
+      for (int e = 0; e < 4; ++e) {
+        const float x0 = bf16lo_to_f32(w[0][e]) * scale, x1 = bf16hi_to_f32(w[0][e]) * scale;
+        const float y0 = bf16lo_to_f32(w[1][e]) * scale, y1 = bf16hi_to_f32(w[1][e]) * scale;
+        if (ROT) {
+          const float *c = cs[ROT ? j : 0], *s = sn[ROT ? j : 0];
+          o0[e] = pack_bf16x2(x0 * c[2 * e] - y0 * s[2 * e], x1 * c[2 * e + 1] - y1 * s[2 * e + 1]);
+          o1[e] = pack_bf16x2(y0 * c[2 * e] + x0 * s[2 * e], y1 * c[2 * e + 1] + x1 * s[2 * e + 1]);
+        } else {
+          o0[e] = pack_bf16x2(x0, x1);
+          o1[e] = pack_bf16x2(y0, y1);
+        }
+      }
     }
     store16(tile + at0, o0);
     store16(tile + at1, o1);
@@ -131,15 +148,15 @@ struct ChunkLoader {
       int r, c0, c1;
       bool rotates;
       if (!place((first + j) * kThreads + (int)threadIdx.x, a, r, c0, c1, rotates)) continue;
-      finish(tk, r * kPitch + c0, r * kPitch + c1, k[j], cs[j], sn[j], a.k_scale);
-      if (!STATE_ONLY) finish(tq, r * kPitch + c0, r * kPitch + c1, q[j], cs[j], sn[j], 1.f);
+      finish(tk, r * kPitch + c0, r * kPitch + c1, k[j], j, a.k_scale);
+      if (!STATE_ONLY) finish(tq, r * kPitch + c0, r * kPitch + c1, q[j], j, 1.f);
     }
   }
   __device__ __forceinline__ void store_v(uint16_t* tv) const {
 #pragma unroll
     for (int j = 0; j < kVPieces; ++j) {
       const int i = j * kThreads + (int)threadIdx.x;
-      store16(tv + i / (VT / 8) * kVPitch + (i % (VT / 8)) * 8, v[j]);
+      store16(tv + i / (kColumns / 8) * kVPitch + (i % (kColumns / 8)) * 8, v[j]);
     }
   }
 };
@@ -167,51 +184,50 @@ __device__ __forceinline__ void load_tile_scalar(uint16_t* tile, const uint16_t*
   }
 }
 
-template <int DP, int VT, bool STATE_ONLY, bool VEC>
-__global__ __launch_bounds__(VT * 4, 2) void decayed_chunk_kernel(const ChunkArgs a) {
-  using S = ChunkShape<DP, VT>;
-  constexpr int kVTiles = VT / 32;
-  constexpr int kDTiles = DP >= 64 ? DP / 64 : 1;         // 32-wide tiles of d per wave in the state
+template <int DP, int NH, bool STATE_ONLY, bool VEC>
+__global__ __launch_bounds__(256, DP <= 128 ? 2 : 1) void decayed_chunk_kernel(const ChunkArgs a) {
+  using S = ChunkShape<DP, NH>;
+  constexpr int kDTiles = DP / 32, kSpan = kColumns / NH, kTilesPerHead = kSpan / 32;
+  constexpr int kItems = NH * 3, kMine = (kItems + 3) / 4;        // weighted score tiles of the workgroup, of a wave
   extern __shared__ __align__(16) unsigned char smem[];
   uint16_t* const tk = reinterpret_cast<uint16_t*>(smem);
-  uint16_t* const tv = tk + S::kQ;
-  uint16_t* const tq = tv + S::kV;
-  uint16_t* const ts_hi = tq + S::kQ;
-  uint16_t* const ts_lo = ts_hi + S::kS;
-  float* const cum = reinterpret_cast<float*>(STATE_ONLY ? tq : ts_lo + S::kS);   // [64] L, base 2
-  float* const scl = cum + kChunk;                                                  // [64] input scale
-  float* const wgt0 = scl + 2 * kChunk;                                             // [32] scale * 2^(L_31 - L)
-  float* const wgt = scl + kChunk;                                                  // [64] scale * 2^(L_end - L)
+  uint16_t* const tv = tk + S::kK;
+  uint16_t* const tq = tv + S::kV;                                // Q, then the weighted scores
+  float* const tables = reinterpret_cast<float*>(tq + (STATE_ONLY ? 0 : S::kQP));
+  // per head: [64] L, [64] input scale, [64] scale * 2^(L_end - L), [32] scale * 2^(L_31 - L), logarithms to base 2
+  auto table = [&](int head) { return tables + head * (3 * kChunk + 32); };
 
-  // consecutive workgroups go to different XCDs: give each XCD a contiguous run of items, so that the tiles and heads that
-  // read the same q and k rows share an L2
-  const int vtiles = (a.vd + VT - 1) / VT;
-  const int total = a.num_segments * a.heads * vtiles;
+  // consecutive workgroups go to different XCDs: give each XCD a contiguous run of items, so that the heads that read the
+  // same q and k rows share an L2
+  const int blocks = NH == 1 ? (a.vd + kColumns - 1) / kColumns : 1, head_sets = a.heads / NH;
+  const int total = a.num_segments * head_sets * blocks;
   const int per_xcd = (total + 7) / 8;
   const int item = (blockIdx.x % 8) * per_xcd + blockIdx.x / 8;
   if (blockIdx.x / 8 >= per_xcd || item >= total) return;
-  const int v0 = (item % vtiles) * VT;
-  const int h = (item / vtiles) % a.heads;
-  const int seg = item / (vtiles * a.heads);
+  const int v0 = (item % blocks) * kColumns;
+  const int h0 = (item / blocks) % head_sets * NH;
+  const int seg = item / (blocks * head_sets);
   const int b = a.segments[3 * seg], t_begin = a.segments[3 * seg + 1], t_end = a.segments[3 * seg + 2];
   const int slot = a.state_slots[b], start = a.starts[b], seq_begin = a.cu_seqlens[b];
   if (slot < 0 || slot >= a.num_slots) return;
-  const int lane = threadIdx.x & 63, wave = threadIdx.x / 64;
-  const int col = lane & 31, hh = lane >> 5;
-  const int vt = wave % kVTiles, half_id = wave / kVTiles;   // half_id: which 32 tokens, and which half of d
-  const int g = h / (a.heads / a.groups);
-  const uint16_t *qp = a.q + (int64_t)g * a.d, *kp = a.k + (int64_t)g * a.d, *vp = a.v + (int64_t)h * a.vd + v0;
-  const int vlen = a.vd - v0 < VT ? a.vd - v0 : VT;
-  const float skip = a.skip ? a.skip[h] : 0.f;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x / 64, col = lane & 31, hh = lane >> 5;
+  const int my_head = wave / kTilesPerHead, h = h0 + my_head;     // this wave's columns: head h, v0 + vx .. vx + 31
+  const int vx = (wave % kTilesPerHead) * 32;
+  const int vlen = a.vd - v0 < kSpan ? a.vd - v0 : kSpan;
+  const bool active = vx < vlen;
+  const int g = h0 / (a.heads / a.groups);
+  const uint16_t *qp = a.q + (int64_t)g * a.d, *kp = a.k + (int64_t)g * a.d, *vp = a.v + (int64_t)h0 * a.vd + v0;
   constexpr float kLog2e = 1.4426950408889634f;
-  const float la_const = a.log_decay ? a.log_decay[h] * kLog2e : 0.f;
-  const float dt_bias = a.dt ? a.dt_bias[h] : 0.f, neg_a = a.dt ? a.neg_a[h] * kLog2e : 0.f;
+  // wave w also looks after the decays of head h0 + w
+  const int decay_head = h0 + (wave < NH ? wave : 0);
+  const float la_const = a.log_decay ? a.log_decay[decay_head] * kLog2e : 0.f;
+  const float dt_bias = a.dt ? a.dt_bias[decay_head] : 0.f, neg_a = a.dt ? a.neg_a[decay_head] * kLog2e : 0.f;
+  const float skip = a.skip ? a.skip[h] : 0.f;
 
-  // S: rows d = 32 (half_id kDTiles + i) + 8 q + 4 hh + e (four consecutive ones per q), column v0 + 32 vt + (lane & 31)
+  // S: tile i, register 4 q + e = row d = 32 i + 8 q + 4 hh + e, column vx + (lane & 31)
   f32x16 st[kDTiles];
-  const bool has_state_tile = half_id * kDTiles * 32 < DP;
-  const int v_col = 32 * vt + col;
-  auto state_d = [&](int i, int q4) { return 32 * (half_id * kDTiles + i) + 8 * q4 + 4 * hh; };
+  const int v_col = vx + col;
+  auto state_d = [&](int i, int q4) { return 32 * i + 8 * q4 + 4 * hh; };
   float* gstate = nullptr;
   bool load_state = false;
   if (!STATE_ONLY) {
@@ -235,20 +251,23 @@ __global__ __launch_bounds__(VT * 4, 2) void decayed_chunk_kernel(const ChunkArg
       for (int e = 0; e < 4; ++e) st[i][4 * q4 + e] = ok ? x[e] : 0.f;
     }
 
-  constexpr int kPairsAll = (kChunk * (DP / 16) + S::kThreads - 1) / S::kThreads;
+  constexpr int kPairsAll = (kChunk * (DP / 16) + 255) / 256;
   constexpr bool kAhead = VEC && kPairsAll <= 2;          // a whole chunk fits the registers next to the accumulators
   constexpr int kPairs = kPairsAll <= 2 ? kPairsAll : 2;
-  ChunkLoader<DP, VT, STATE_ONLY, kPairs> ld;
+  ChunkLoader<DP, STATE_ONLY, kPairs, NH == 1> ld;      // heads that rotate do not share keys
   float dt_next = 0.f;
   auto fetch = [&](int t) {
     const int m = t_end - t < kChunk ? t_end - t : kChunk;
     ld.fetch_qk(0, kp + (int64_t)t * a.k_stride, qp + (int64_t)t * a.q_stride, m, a);
     ld.fetch_trig(0, m, start + (t - seq_begin), a);
-    ld.fetch_v(vp + (int64_t)t * a.v_stride, m, vlen, a);
+    ld.fetch_v(vp + (int64_t)t * a.v_stride, m, kSpan, vlen, a);
   };
-  auto fetch_dt = [&](int t) { dt_next = a.dt && wave == 0 && t + lane < t_end ? bf16lo_to_f32(a.dt[(int64_t)(t + lane) * a.dt_stride + h]) : 0.f; };
+  auto fetch_dt = [&](int t) {
+    dt_next = a.dt && wave < NH && t + lane < t_end ? bf16lo_to_f32(a.dt[(int64_t)(t + lane) * a.dt_stride + decay_head]) : 0.f;
+  };
   if (kAhead) fetch(t_begin);
   fetch_dt(t_begin);
+
   float total_log = 0.f;
   for (int t0 = t_begin; t0 < t_end; t0 += kChunk) {
     const int n = t_end - t0 < kChunk ? t_end - t0 : kChunk;
@@ -258,24 +277,24 @@ __global__ __launch_bounds__(VT * 4, 2) void decayed_chunk_kernel(const ChunkArg
       ld.store_qk(0, tk, tq, a);
       ld.store_v(tv);
     } else if (VEC) {
-      ld.fetch_v(vp + (int64_t)t0 * a.v_stride, n, vlen, a);
+      ld.fetch_v(vp + (int64_t)t0 * a.v_stride, n, kSpan, vlen, a);
+      ld.store_v(tv);
 #pragma unroll 1
       for (int first = 0; first < kPairsAll; first += kPairs) {
         ld.fetch_qk(first, kp + (int64_t)t0 * a.k_stride, qp + (int64_t)t0 * a.q_stride, n, a);
         ld.fetch_trig(first, n, pos0, a);
         ld.store_qk(first, tk, tq, a);
       }
-      ld.store_v(tv);
     } else {
-      load_tile_scalar<DP, S::kThreads>(tk, kp + (int64_t)t0 * a.k_stride, a.k_stride, n, pos0, a, a.k_scale);
-      if (!STATE_ONLY) load_tile_scalar<DP, S::kThreads>(tq, qp + (int64_t)t0 * a.q_stride, a.q_stride, n, pos0, a, 1.f);
+      load_tile_scalar<DP, 256>(tk, kp + (int64_t)t0 * a.k_stride, a.k_stride, n, pos0, a, a.k_scale);
+      if (!STATE_ONLY) load_tile_scalar<DP, 256>(tq, qp + (int64_t)t0 * a.q_stride, a.q_stride, n, pos0, a, 1.f);
 #pragma unroll 1
-      for (int i = threadIdx.x; i < kChunk * VT; i += S::kThreads) {
-        const int r = i / VT, c = i % VT;
-        tv[r * S::kVPitch + c] = r < n && c < vlen ? vp[(int64_t)(t0 + r) * a.v_stride + c] : (uint16_t)0;
+      for (int i = threadIdx.x; i < kChunk * kColumns; i += 256) {
+        const int r = i / kColumns, c = i % kColumns;
+        tv[r * kVPitch + c] = r < n && c % kSpan < vlen ? vp[(int64_t)(t0 + r) * a.v_stride + (int64_t)(c / kSpan) * a.vd + c % kSpan] : (uint16_t)0;
       }
     }
-    if (wave == 0) {     // decays of the chunk: lane = token
+    if (wave < NH) {     // decays of the chunk: lane = token
       float la = 0.f, s = 0.f, l;
       if (a.dt) {
         if (lane < n) {
@@ -292,120 +311,174 @@ __global__ __launch_bounds__(VT * 4, 2) void decayed_chunk_kernel(const ChunkArg
         s = lane < n ? 1.f : 0.f;
         l = la_const * (float)(lane + 1 < n ? lane + 1 : n);
       }
-      const float l_end = __shfl(l, 63, 64);
-      cum[lane] = l;
-      scl[lane] = s;
-      wgt[lane] = s * __builtin_amdgcn_exp2f(l_end - l);
-      const float l_mid = __shfl(l, 31, 64);
-      if (lane < 32) wgt0[lane] = s * __builtin_amdgcn_exp2f(l_mid - l);
-    }
-    if (!STATE_ONLY && has_state_tile) {
-#pragma unroll
-      for (int i = 0; i < kDTiles; ++i)
-#pragma unroll
-        for (int q4 = 0; q4 < 4; ++q4) {
-          const uint32_t h0 = pack_bf16x2(st[i][4 * q4], st[i][4 * q4 + 1]), h1 = pack_bf16x2(st[i][4 * q4 + 2], st[i][4 * q4 + 3]);
-          const uint32_t l0 = pack_bf16x2(st[i][4 * q4] - bf16lo_to_f32(h0), st[i][4 * q4 + 1] - bf16hi_to_f32(h0));
-          const uint32_t l1 = pack_bf16x2(st[i][4 * q4 + 2] - bf16lo_to_f32(h1), st[i][4 * q4 + 3] - bf16hi_to_f32(h1));
-          *reinterpret_cast<u32x2*>(ts_hi + v_col * S::kPitch + state_d(i, q4)) = u32x2{h0, h1};
-          *reinterpret_cast<u32x2*>(ts_lo + v_col * S::kPitch + state_d(i, q4)) = u32x2{l0, l1};
-        }
+      const float l_end = __shfl(l, 63, 64), l_mid = __shfl(l, 31, 64);
+      float* t = table(wave);
+      t[lane] = l;
+      t[kChunk + lane] = s;
+      t[2 * kChunk + lane] = s * __builtin_amdgcn_exp2f(l_end - l);
+      if (lane < 32) t[3 * kChunk + lane] = s * __builtin_amdgcn_exp2f(l_mid - l);
     }
     __syncthreads();
-    const float l_end = cum[kChunk - 1];
+    const float* const mine = table(my_head);
+    const float l_end = mine[kChunk - 1];
     total_log += l_end;
     const bool more = t0 + kChunk < t_end;
     if (more) fetch_dt(t0 + kChunk);
 
     if (!STATE_ONLY) {
-      const int i_tok = 32 * half_id + col;      // this lane's output token
-      const float l_i = cum[i_tok];
-      f32x16 o;
+      // ---- weighted scores: item = 3 * head + tile, tile 0: tokens 0..31 on themselves, 1: 32..63 on 0..31, 2: 32..63 on themselves
+      bf16x8 p_hi[kMine][2], p_lo[kMine][2];
 #pragma unroll
-      for (int r = 0; r < 16; ++r) o[r] = 0.f;
+      for (int m = 0; m < kMine; ++m) {
+        const int it = wave + 4 * m;
+        if (it < kItems) {
+          const int tile = it % 3, i_tok = (tile ? 32 : 0) + col, j_base = tile == 2 ? 32 : 0;
+          const float* t = table(it / 3);
+          f32x16 p;
 #pragma unroll
-      for (int kk = 0; kk < DP / 16; ++kk) {
-        const bf16x8 qb = tile_row(tq, S::kPitch, i_tok, 16 * kk + 8 * hh);
-        o = mfma32(tile_row(ts_hi, S::kPitch, 32 * vt + col, 16 * kk + 8 * hh), qb, o);
-        o = mfma32(tile_row(ts_lo, S::kPitch, 32 * vt + col, 16 * kk + 8 * hh), qb, o);
-      }
-      const float e_i = __builtin_amdgcn_exp2f(l_i), e_mid = __builtin_amdgcn_exp2f(half_id ? l_i - cum[31] : 0.f);
+          for (int r = 0; r < 16; ++r) p[r] = 0.f;
 #pragma unroll
-      for (int r = 0; r < 16; ++r) o[r] *= e_i;
-      for (int jt = 0; jt <= half_id; ++jt) {
-        f32x16 p;
+          for (int kk = 0; kk < DP / 16; ++kk)
+            p = mfma32(tile_row(tk, S::kPitch, j_base + col, 16 * kk + 8 * hh), tile_row(tq, S::kPitch, i_tok, 16 * kk + 8 * hh), p);
+          const float l_i = t[i_tok];
+          const float e_mid = tile == 1 ? __builtin_amdgcn_exp2f(l_i - t[31]) : 0.f;
 #pragma unroll
-        for (int r = 0; r < 16; ++r) p[r] = 0.f;
+          for (int half = 0; half < 2; ++half) {
+            float w[8];
 #pragma unroll
-        for (int kk = 0; kk < DP / 16; ++kk)
-          p = mfma32(tile_row(tk, S::kPitch, 32 * jt + col, 16 * kk + 8 * hh), tile_row(tq, S::kPitch, i_tok, 16 * kk + 8 * hh), p);
+            for (int q4 = 0; q4 < 2; ++q4) {
+              const int j0 = j_base + 16 * half + 8 * q4 + 4 * hh;
+              const f32x4 l_j = *reinterpret_cast<const f32x4*>(t + j0), s_j = *reinterpret_cast<const f32x4*>(t + kChunk + j0);
+              const f32x4 m_j = *reinterpret_cast<const f32x4*>(t + 3 * kChunk + (tile == 1 ? j0 : 0));
 #pragma unroll
-        for (int ks = 0; ks < 2; ++ks) {
-          const int j0 = 32 * jt + 16 * ks + 4 * hh;       // tokens j0 .. j0+3 and j0+8 .. j0+11
-          float pv[8];
-#pragma unroll
-          for (int e = 0; e < 8; ++e) {
-            const int j = j0 + (e & 3) + 8 * (e >> 2);
-            // below the diagonal tile the weight is a product of one factor per token on either side of the tile border
-            if (jt < half_id) pv[e] = p[8 * ks + e] * (wgt0[j] * e_mid);
-            else pv[e] = j <= i_tok ? p[8 * ks + e] * (scl[j] * __builtin_amdgcn_exp2f(l_i - cum[j])) : 0.f;
+              for (int e = 0; e < 4; ++e) {
+                // below the diagonal tiles the weight is a product of one factor per token on either side of the tile border
+                const float on = j0 + e <= i_tok ? s_j[e] * __builtin_amdgcn_exp2f(l_i - l_j[e]) : 0.f;
+                w[4 * q4 + e] = p[8 * half + 4 * q4 + e] * (tile == 1 ? m_j[e] * e_mid : on);
+              }
+            }
+            split8(w, p_hi[m][half], p_lo[m][half]);
           }
-          bf16x8 hi, lo;
-          split8(pv, hi, lo);
-          const bf16x8 va = __builtin_bit_cast(bf16x8, tile_columns(tv, S::kVPitch, j0, j0 + 8, 32 * vt, lane));
-          o = mfma32(va, hi, o);
-          o = mfma32(va, lo, o);
         }
       }
-      if (skip != 0.f) {
+      __builtin_amdgcn_sched_barrier(0);
+      // ---- O^T = S^T Q^T, decayed
+      f32x16 o[2];
 #pragma unroll
-        for (int q4 = 0; q4 < 4; ++q4)
+      for (int it = 0; it < 2; ++it)
 #pragma unroll
-          for (int e = 0; e < 4; ++e)
-            o[4 * q4 + e] += skip * bf16lo_to_f32(tv[i_tok * S::kVPitch + 32 * vt + 8 * q4 + 4 * hh + e]);
+        for (int r = 0; r < 16; ++r) o[it][r] = 0.f;
+      if (active) {
+#pragma unroll
+        for (int i = 0; i < kDTiles; ++i)
+#pragma unroll
+          for (int half = 0; half < 2; ++half) {
+            float x[8];
+#pragma unroll
+            for (int e = 0; e < 8; ++e) x[e] = st[i][8 * half + e];
+            bf16x8 hi, lo;
+            split8(x, hi, lo);
+            const int d0 = 32 * i + 16 * half + 4 * hh;      // the d's of x: d0 .. d0+3, d0+8 .. d0+11
+#pragma unroll
+            for (int it = 0; it < 2; ++it) {
+              const uint16_t* qr = tq + (32 * it + col) * S::kPitch + d0;
+              const u32x2 w0 = *reinterpret_cast<const u32x2*>(qr), w1 = *reinterpret_cast<const u32x2*>(qr + 8);
+              const bf16x8 qb = __builtin_bit_cast(bf16x8, u32x4{w0[0], w0[1], w1[0], w1[1]});
+              o[it] = mfma32(hi, qb, o[it]);
+              o[it] = mfma32(lo, qb, o[it]);
+            }
+          }
+#pragma unroll
+        for (int it = 0; it < 2; ++it) o[it] *= __builtin_amdgcn_exp2f(mine[32 * it + col]);
       }
-      uint16_t* orow = a.out + (int64_t)(t0 + i_tok) * a.out_stride + (int64_t)h * a.vd + v0;
+      __syncthreads();     // Q has been read: the scores take its place
 #pragma unroll
-      for (int half = 0; half < 2; ++half) {
-        // eight consecutive columns per lane: the lower half of the wave completes piece 2 half, the upper half 2 half + 1
-        const u32x2 even = {pack_bf16x2(o[8 * half], o[8 * half + 1]), pack_bf16x2(o[8 * half + 2], o[8 * half + 3])};
-        const u32x2 odd = {pack_bf16x2(o[8 * half + 4], o[8 * half + 5]), pack_bf16x2(o[8 * half + 6], o[8 * half + 7])};
-        const u32x2 mine = hh ? odd : even, give = hh ? even : odd;
-        const u32x2 got = {(uint32_t)__shfl_xor((int)give[0], 32, 64), (uint32_t)__shfl_xor((int)give[1], 32, 64)};
-        const u32x4 w = hh ? u32x4{got[0], got[1], mine[0], mine[1]} : u32x4{mine[0], mine[1], got[0], got[1]};
-        const int v = 32 * vt + 16 * half + 8 * hh;
-        if (i_tok < n) {
-          if (VEC) {
-            if (v < vlen) store16(orow + v, w);
-          } else {
+      for (int m = 0; m < kMine; ++m) {
+        const int it = wave + 4 * m;
+        if (it < kItems) {
+          uint16_t* dst = tq + it * 2 * kPTile + col * kPPitch + 4 * hh;
 #pragma unroll
-            for (int e = 0; e < 8; ++e)
-              if (v + e < vlen) orow[v + e] = (uint16_t)(w[e >> 1] >> (16 * (e & 1)));
+          for (int half = 0; half < 2; ++half) {
+            const u32x4 hw = __builtin_bit_cast(u32x4, p_hi[m][half]), lw = __builtin_bit_cast(u32x4, p_lo[m][half]);
+            *reinterpret_cast<u32x2*>(dst + 16 * half) = u32x2{hw[0], hw[1]};
+            *reinterpret_cast<u32x2*>(dst + 16 * half + 8) = u32x2{hw[2], hw[3]};
+            *reinterpret_cast<u32x2*>(dst + kPTile + 16 * half) = u32x2{lw[0], lw[1]};
+            *reinterpret_cast<u32x2*>(dst + kPTile + 16 * half + 8) = u32x2{lw[2], lw[3]};
+          }
+        }
+      }
+      __syncthreads();
+      if (active) {
+        const uint16_t* ph = tq + my_head * 6 * kPTile;
+#pragma unroll
+        for (int jt = 0; jt < 2; ++jt)
+#pragma unroll
+          for (int ks = 0; ks < 2; ++ks) {
+            const int j0 = 32 * jt + 16 * ks + 8 * hh;
+            const bf16x8 va = __builtin_bit_cast(bf16x8, tile_columns(tv, kVPitch, j0, j0 + 4, 32 * wave, lane));
+#pragma unroll
+            for (int it = jt; it < 2; ++it) {
+              const uint16_t* tile = ph + (it + jt) * 2 * kPTile;      // (0,0) -> 0, (1,0) -> 1, (1,1) -> 2
+              o[it] = mfma32(va, tile_row(tile, kPPitch, col, 16 * ks + 8 * hh), o[it]);
+              o[it] = mfma32(va, tile_row(tile + kPTile, kPPitch, col, 16 * ks + 8 * hh), o[it]);
+            }
+          }
+#pragma unroll
+        for (int it = 0; it < 2; ++it) {
+          const int i_tok = 32 * it + col;
+          if (skip != 0.f) {
+#pragma unroll
+            for (int q4 = 0; q4 < 4; ++q4)
+#pragma unroll
+              for (int e = 0; e < 4; ++e) o[it][4 * q4 + e] += skip * bf16lo_to_f32(tv[i_tok * kVPitch + 32 * wave + 8 * q4 + 4 * hh + e]);
+          }
+          uint16_t* orow = a.out + (int64_t)(t0 + i_tok) * a.out_stride + (int64_t)h * a.vd + v0 + vx;
+#pragma unroll
+          for (int half = 0; half < 2; ++half) {
+            // eight consecutive columns per lane: the lower half of the wave completes piece 2 half, the upper half 2 half + 1
+            const u32x2 even = {pack_bf16x2(o[it][8 * half], o[it][8 * half + 1]), pack_bf16x2(o[it][8 * half + 2], o[it][8 * half + 3])};
+            const u32x2 odd = {pack_bf16x2(o[it][8 * half + 4], o[it][8 * half + 5]), pack_bf16x2(o[it][8 * half + 6], o[it][8 * half + 7])};
+            const u32x2 keep = hh ? odd : even, give = hh ? even : odd;
+            const u32x2 got = {(uint32_t)__shfl_xor((int)give[0], 32, 64), (uint32_t)__shfl_xor((int)give[1], 32, 64)};
+            const u32x4 w = hh ? u32x4{got[0], got[1], keep[0], keep[1]} : u32x4{keep[0], keep[1], got[0], got[1]};
+            const int v = 16 * half + 8 * hh;
+            if (i_tok < n) {
+              if (VEC) {
+                if (vx + v < vlen) store16(orow + v, w);
+              } else {
+#pragma unroll
+                for (int e = 0; e < 8; ++e)
+                  if (vx + v + e < vlen) orow[v + e] = (uint16_t)(w[e >> 1] >> (16 * (e & 1)));
+              }
+            }
           }
         }
       }
     }
-    // the next chunk is on its way while the state takes this one in
+    // the next chunk is on its way while the state takes this one in; not before: its registers are in use above
+    __builtin_amdgcn_sched_barrier(0);
     if (kAhead && more) fetch(t0 + kChunk);
     // ---- S <- e^{L_end} S + K^T (w V)
-    if (has_state_tile) {
+    if (active) {
       const float e_end = __builtin_amdgcn_exp2f(l_end);
 #pragma unroll
-      for (int i = 0; i < kDTiles; ++i)
-#pragma unroll
-        for (int r = 0; r < 16; ++r) st[i][r] *= e_end;
+      for (int i = 0; i < kDTiles; ++i) st[i] *= e_end;
 #pragma unroll
       for (int ks = 0; ks < kChunk / 16; ++ks) {
-        const int j0 = 16 * ks + 4 * hh;
-        const s16x8 raw = tile_columns(tv, S::kVPitch, j0, j0 + 8, 32 * vt, lane);
+        const int j0 = 16 * ks + 8 * hh;
+        const s16x8 raw = tile_columns(tv, kVPitch, j0, j0 + 4, 32 * wave, lane);
+        const f32x4 w0 = *reinterpret_cast<const f32x4*>(mine + 2 * kChunk + j0), w1 = *reinterpret_cast<const f32x4*>(mine + 2 * kChunk + j0 + 4);
         float x[8];
 #pragma unroll
-        for (int e = 0; e < 8; ++e) x[e] = bf16lo_to_f32((uint16_t)raw[e]) * wgt[j0 + (e & 3) + 8 * (e >> 2)];
+        for (int e = 0; e < 4; ++e) {
+          x[e] = bf16lo_to_f32((uint16_t)raw[e]) * w0[e];
+          x[4 + e] = bf16lo_to_f32((uint16_t)raw[4 + e]) * w1[e];
+        }
         bf16x8 hi, lo;
         split8(x, hi, lo);
 #pragma unroll
         for (int i = 0; i < kDTiles; ++i) {
-          const bf16x8 ka = __builtin_bit_cast(bf16x8, tile_columns(tk, S::kPitch, j0, j0 + 8, 32 * (half_id * kDTiles + i), lane));
+          const bf16x8 ka = __builtin_bit_cast(bf16x8, tile_columns(tk, S::kPitch, j0, j0 + 4, 32 * i, lane));
           st[i] = mfma32(ka, hi, st[i]);
           st[i] = mfma32(ka, lo, st[i]);
         }
@@ -416,7 +489,7 @@ __global__ __launch_bounds__(VT * 4, 2) void decayed_chunk_kernel(const ChunkArg
   float* dst = nullptr;
   if (STATE_ONLY) dst = a.seg_state + (((int64_t)seg * a.heads + h) * a.vd + v0) * a.pitch;
   else if (!a.seg_state) dst = gstate;
-  if (dst && has_state_tile) {
+  if (dst && active) {
 #pragma unroll
     for (int i = 0; i < kDTiles; ++i)
 #pragma unroll
@@ -424,7 +497,7 @@ __global__ __launch_bounds__(VT * 4, 2) void decayed_chunk_kernel(const ChunkArg
         if (v_col < vlen && state_d(i, q4) < a.pitch)
           *reinterpret_cast<f32x4*>(dst + v_col * a.pitch + state_d(i, q4)) = f32x4{st[i][4 * q4], st[i][4 * q4 + 1], st[i][4 * q4 + 2], st[i][4 * q4 + 3]};
   }
-  if (STATE_ONLY && v0 == 0 && threadIdx.x == 0) a.seg_decay[(int64_t)seg * a.heads + h] = total_log;
+  if (STATE_ONLY && v0 == 0 && vx == 0 && lane == 0) a.seg_decay[(int64_t)seg * a.heads + h] = total_log;
 }
 
 // Start state of every segment (in place of its contribution) and the final state of every sequence.  Segments of a sequence
@@ -449,27 +522,49 @@ __global__ __launch_bounds__(256) void decayed_segment_scan_kernel(const ChunkAr
   *reinterpret_cast<f32x4*>(gs) = s;
 }
 
-template <int DP, int VT, bool VEC>
+template <int DP, int NH, bool VEC>
 static int launch_chunks(const ChunkArgs& a, const int32_t* seq_segments, int64_t batch, hipStream_t s) {
-  using S = ChunkShape<DP, VT>;
-  const int64_t items = (int64_t)a.num_segments * a.heads * ((a.vd + VT - 1) / VT);
-  const dim3 grid((unsigned)((items + 7) / 8 * 8)), block(S::kThreads);
-  static const hipError_t lds = hipFuncSetAttribute(reinterpret_cast<const void*>(&decayed_chunk_kernel<DP, VT, false, VEC>),
+  using S = ChunkShape<DP, NH>;
+  const int64_t items = (int64_t)a.num_segments * (a.heads / NH) * (NH == 1 ? (a.vd + kColumns - 1) / kColumns : 1);
+  const dim3 grid((unsigned)((items + 7) / 8 * 8)), block(256);
+  static const hipError_t lds = hipFuncSetAttribute(reinterpret_cast<const void*>(&decayed_chunk_kernel<DP, NH, false, VEC>),
                                                     hipFuncAttributeMaxDynamicSharedMemorySize, S::bytes(false));
-  static const hipError_t lds_state = hipFuncSetAttribute(reinterpret_cast<const void*>(&decayed_chunk_kernel<DP, VT, true, VEC>),
+  static const hipError_t lds_state = hipFuncSetAttribute(reinterpret_cast<const void*>(&decayed_chunk_kernel<DP, NH, true, VEC>),
                                                           hipFuncAttributeMaxDynamicSharedMemorySize, S::bytes(true));
   if (lds != hipSuccess) return record_hip_error(lds);
   if (lds_state != hipSuccess) return record_hip_error(lds_state);
   if (a.seg_state) {
-    hipLaunchKernelGGL((decayed_chunk_kernel<DP, VT, true, VEC>), grid, block, S::bytes(true), s, a);
+    hipLaunchKernelGGL((decayed_chunk_kernel<DP, NH, true, VEC>), grid, block, S::bytes(true), s, a);
     const int64_t quads = ((int64_t)a.vd * a.pitch / 4 + 255) / 256;
     hipLaunchKernelGGL(decayed_segment_scan_kernel, dim3((unsigned)quads, (unsigned)a.heads, (unsigned)batch), dim3(256), 0, s, a, seq_segments);
   }
-  hipLaunchKernelGGL((decayed_chunk_kernel<DP, VT, false, VEC>), grid, block, S::bytes(false), s, a);
+  hipLaunchKernelGGL((decayed_chunk_kernel<DP, NH, false, VEC>), grid, block, S::bytes(false), s, a);
   return finish_launch();
 }
 
+template <int NH>
+static int launch_chunks_for(const ChunkArgs& a, const int32_t* seq_segments, int64_t batch, bool vec, hipStream_t s) {
+  if (!vec) return a.d <= 64 ? launch_chunks<64, NH, false>(a, seq_segments, batch, s) : launch_chunks<256, NH, false>(a, seq_segments, batch, s);
+  if (a.d <= 32) return launch_chunks<32, NH, true>(a, seq_segments, batch, s);
+  if (a.d <= 64) return launch_chunks<64, NH, true>(a, seq_segments, batch, s);
+  if (a.d <= 128) return launch_chunks<128, NH, true>(a, seq_segments, batch, s);
+  return launch_chunks<256, NH, true>(a, seq_segments, batch, s);
+}
+
+// Heads of one workgroup: as many of a q/k group as fill its 128 value columns.
+static int heads_together(int64_t heads, int64_t groups, int64_t vd, bool rotates) {
+  const int64_t per = heads / groups;
+  if (rotates) return 1;
+  return vd <= 32 && per % 4 == 0 ? 4 : (vd <= 64 && per % 2 == 0 ? 2 : 1);
+}
+
 }  // namespace mops
+
+extern "C" int64_t mops_hip_decayed_chunks_workgroups(int64_t heads, int64_t groups, int64_t vd) {
+  if (heads <= 0 || groups <= 0 || heads % groups || vd <= 0) return MOPS_HIP_EINVAL;
+  const int64_t nh = mops::heads_together(heads, groups, vd, false);
+  return heads / nh * (nh == 1 ? (vd + mops::kColumns - 1) / mops::kColumns : 1);
+}
 
 extern "C" int mops_hip_decayed_chunks(const mops_hip_recurrence* r, const int32_t* segments, int64_t num_segments,
                                        const int32_t* seq_segments, float* seg_state, float* seg_decay, void* stream) {
@@ -503,12 +598,9 @@ extern "C" int mops_hip_decayed_chunks(const mops_hip_recurrence* r, const int32
   const bool vec = r->d % 8 == 0 && r->q_stride % 8 == 0 && r->k_stride % 8 == 0 && aligned16(r->q) && aligned16(r->k) &&
                    (r->rot == 0 || (r->rot % 16 == 0 && aligned16(r->cos_sin))) && r->vd % 8 == 0 && r->v_stride % 8 == 0 &&
                    r->out_stride % 8 == 0 && aligned16(r->v) && aligned16(r->out);
-  hipStream_t s = (hipStream_t)stream;
-  if (!vec) return a.d <= 64 ? launch_chunks<64, 64, false>(a, seq_segments, r->batch, s) : launch_chunks<256, 64, false>(a, seq_segments, r->batch, s);
-#define MOPS_CHUNKS(D) (a.vd <= 32 ? launch_chunks<D, 32, true>(a, seq_segments, r->batch, s) : launch_chunks<D, 64, true>(a, seq_segments, r->batch, s))
-  if (a.d <= 32) return MOPS_CHUNKS(32);
-  if (a.d <= 64) return MOPS_CHUNKS(64);
-  if (a.d <= 128) return MOPS_CHUNKS(128);
-  return MOPS_CHUNKS(256);
-#undef MOPS_CHUNKS
+  switch (heads_together(r->heads, r->groups, r->vd, r->rot > 0)) {
+    case 4: return launch_chunks_for<4>(a, seq_segments, r->batch, vec, (hipStream_t)stream);
+    case 2: return launch_chunks_for<2>(a, seq_segments, r->batch, vec, (hipStream_t)stream);
+    default: return launch_chunks_for<1>(a, seq_segments, r->batch, vec, (hipStream_t)stream);
+  }
 }

@@ -331,6 +331,7 @@ static int launch_recurrence(const RecurrenceArgs& a, int64_t batch, bool conv, 
   else if (a.d <= 64) launch_recurrence_rows<T, 4>(a, batch, conv, s);
   else if (a.d <= 128) launch_recurrence_rows<T, 8>(a, batch, conv, s);
   else if (a.d <= 256) launch_recurrence_rows<T, 16>(a, batch, conv, s);
+  else if (a.d <= 512) launch_recurrence_rows<T, 32>(a, batch, conv, s);
   else return MOPS_HIP_EUNSUPPORTED;
   return finish_launch();
 }
@@ -345,7 +346,7 @@ extern "C" int mops_hip_decayed_recurrence(const mops_hip_recurrence* r, void* s
   if (r->batch == 0) return MOPS_HIP_OK;
   if (!r->q || !r->k || !r->v || !r->out || !r->state || !r->state_slots || !r->starts) return MOPS_HIP_EINVAL;
   if (r->heads <= 0 || r->groups <= 0 || r->heads % r->groups || r->d <= 0 || r->vd <= 0 || r->num_slots <= 0) return MOPS_HIP_EINVAL;
-  if (r->d > 256 || r->heads > 65536 || r->vd > 65536) return MOPS_HIP_EUNSUPPORTED;
+  if (r->d > 512 || r->heads > 65536 || r->vd > 65536) return MOPS_HIP_EUNSUPPORTED;
   if (r->q_stride < r->groups * r->d || r->k_stride < r->groups * r->d || r->v_stride < r->heads * r->vd ||
       r->out_stride < r->heads * r->vd)
     return MOPS_HIP_EINVAL;

@@ -87,15 +87,15 @@ class ChunkedRecurrence:
 
     def __call__(self, q, k, v, out, state, ctx, **options):
         """q, k, v, out: the rows of the portions.  The cut into segments is shared by the layers of a step."""
-        heads, _, _, vd = self.sizes
+        heads, groups, _, vd = self.sizes
         nd = ctx["n_decode"]
         slots, starts, cu = ctx["state_slots"][nd:], ctx["starts"][nd:], ctx["portion_cu"]
         if not self.chunked:
             return self.recurrence(q, k, v, out, state, slots, starts, *self.sizes, cu_seqlens=cu, **options)
         cuts = ctx.setdefault("segment_cuts", {})
-        key = (heads, vd)
+        key = (heads, groups, vd)
         if key not in cuts:
-            segments, bounds = recurrence_segments(ctx["seq_counts"][nd:], heads, vd)
+            segments, bounds = recurrence_segments(ctx["seq_counts"][nd:], heads, groups, vd)
             flat = torch.tensor([x for s in segments for x in s] + bounds, dtype=torch.int32).to(v.device, non_blocking=True)
             cuts[key] = (flat[:3 * len(segments)].view(-1, 3), flat[3 * len(segments):])
         return self.chunks(q, k, v, out, state, slots, starts, *self.sizes, *cuts[key], cu_seqlens=cu, **options)

@@ -173,13 +173,13 @@ def decayed_recurrence(q, k, v, out, state, state_slots, starts, heads, groups, 
 CHUNK_MAX_DIM = 256       # head sizes (d) the chunked kernels cover
 
 
-def recurrence_segments(counts, heads: int, vd: int, wanted: int = 768):
+def recurrence_segments(counts, heads: int, groups: int, vd: int, wanted: int = 512):
     """Cuts portions of counts[i] tokens (packed one behind the other) into segments for decayed_chunks: one per portion if
     those give enough workgroups, else about `wanted` workgroups in all.  Returns host lists (segments, bounds per portion)."""
-    lanes = heads * ((vd + 63) // 64)
+    per_segment = _capi.load().mops_hip_decayed_chunks_workgroups(heads, groups, vd)
     length = max(counts)
-    if len(counts) * lanes < wanted // 2 and length > 256:
-        length = max(128, -(-sum(counts) * lanes // wanted // 64) * 64)
+    if len(counts) * per_segment < wanted // 2 and length > 256:
+        length = max(128, -(-sum(counts) * per_segment // wanted // 64) * 64)
     segments, bounds, at = [], [0], 0
     for i, n in enumerate(counts):
         for begin in range(0, n, length):

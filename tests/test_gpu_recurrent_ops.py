@@ -143,7 +143,7 @@ def run_recurrence(gpu, case, heads, groups, d, vd, cuts, chunked, segment=None,
     return out, state[slot, :, :, :d].transpose(1, 2)
 
 
-SIZES = [(1, 1, 16, 16), (4, 2, 24, 40), (3, 3, 42, 25), (2, 1, 64, 64), (2, 2, 128, 130), (2, 1, 200, 32)]
+SIZES = [(1, 1, 16, 16), (4, 2, 24, 40), (3, 3, 42, 25), (2, 1, 64, 64), (2, 2, 128, 130), (2, 1, 200, 32), (8, 2, 32, 24), (4, 1, 48, 27), (2, 2, 256, 300)]
 
 
 @pytest.mark.parametrize("kind", ["const", "steps"])
@@ -205,7 +205,7 @@ def test_chunks_of_several_sequences_and_padding_slots(gpu):
     i32 = lambda x: torch.tensor(x, dtype=torch.int32, device=gpu)   # noqa: E731
     init = torch.randn((6, heads, vd, R.recurrence_state_pitch(d)), generator=g).to(gpu)
     slots = [4, 0, -1, 2]
-    segs, bounds = R.recurrence_segments(lens, heads, vd)
+    segs, bounds = R.recurrence_segments(lens, heads, heads, vd)
     for cut in (1, 64):
         state, out = init.clone(), torch.zeros((cu[-1], heads * vd), dtype=torch.bfloat16, device=gpu)
         if cut == 64:
@@ -228,7 +228,7 @@ def test_chunks_of_several_sequences_and_padding_slots(gpu):
 
 def test_segments_cover_every_portion():
     for counts in ([5000], [64], [2, 3, 700], [100] * 40, [16384, 1000]):
-        segs, bounds = R.recurrence_segments(counts, 4, 64)
+        segs, bounds = R.recurrence_segments(counts, 4, 2, 64)
         at = 0
         for i, n in enumerate(counts):
             mine = segs[bounds[i]:bounds[i + 1]]
