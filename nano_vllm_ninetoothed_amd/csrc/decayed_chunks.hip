@@ -58,7 +58,7 @@ struct ChunkShape {
 };
 
 // q, k and v rows of a chunk on their way from memory into the LDS tiles: q and k rotated, scaled and rounded to bf16, zeros
-// outside the chunk and the head.  fetch() issues every load of a chunk at once, so that it can be called while the chunk
+// behind the head.  fetch() issues every load of a chunk at once, so that it can be called while the chunk
 // before is still being worked on; store() finishes the values and writes the tiles.
 // A thread owns pairs of 16-byte pieces of a row, for q and k alike: pair p < rot / 16 is columns (8p, 8p + rot/2), which
 // rotate with each other; the pairs behind take two pieces that pass unchanged.
@@ -68,7 +68,7 @@ struct ChunkLoader {
   static constexpr int kThreads = 256, kPitch = DP + 8;
   static constexpr int kVPieces = kChunk * (kColumns / 8) / kThreads;
   u32x4 k[PAIRS][2], q[STATE_ONLY ? 1 : PAIRS][2], v[kVPieces];
-  float cs[ROT ? PAIRS : 1][8], sn[ROT ? PAIRS : 1][8];
+  f32x4 cs[ROT ? PAIRS : 1][2], sn[ROT ? PAIRS : 1][2];
 
   static __device__ __forceinline__ bool place(int i, const ChunkArgs& a, int& r, int& c0, int& c1, bool& rotates) {
     r = i / (DP / 16);
@@ -78,38 +78,42 @@ struct ChunkLoader {
     c1 = rotates ? c0 + half : c0 + 8;
     return i < kChunk * (DP / 16);
   }
+  // Loads carry no condition: a row behind the chunk's end is the last row again (its input scale is zero, so it has no
+  // weight anywhere), a column behind the head is column 0 and is dropped when the tile is written or by whoever reads the
+  // tile.  Addresses are a uniform base and a 32-bit offset.
+  static __device__ __forceinline__ u32x4 at(const void* base, uint32_t bytes) { return load16(static_cast<const char*>(base) + bytes); }
   __device__ __forceinline__ void fetch_qk(int first, const uint16_t* kp, const uint16_t* qp, int n, const ChunkArgs& a) {
 #pragma unroll
     for (int j = 0; j < PAIRS; ++j) {
       int r, c0, c1;
       bool rotates;
-      const bool in = place((first + j) * kThreads + (int)threadIdx.x, a, r, c0, c1, rotates) && r < n;
-      const u32x4 zero = {0u, 0u, 0u, 0u};
-      k[j][0] = in && c0 < a.d ? load16(kp + r * a.k_stride + c0) : zero;
-      k[j][1] = in && c1 < a.d ? load16(kp + r * a.k_stride + c1) : zero;
+      place((first + j) * kThreads + (int)threadIdx.x, a, r, c0, c1, rotates);
+      r = r < n ? r : n - 1;
+      c0 = c0 < a.d ? c0 : 0;
+      c1 = c1 < a.d ? c1 : 0;
+      const uint32_t kr = (uint32_t)r * (uint32_t)a.k_stride, qr = (uint32_t)r * (uint32_t)a.q_stride;
+      k[j][0] = at(kp, 2 * (kr + c0));
+      k[j][1] = at(kp, 2 * (kr + c1));
       if (!STATE_ONLY) {
-        q[j][0] = in && c0 < a.d ? load16(qp + r * a.q_stride + c0) : zero;
-        q[j][1] = in && c1 < a.d ? load16(qp + r * a.q_stride + c1) : zero;
+        q[j][0] = at(qp, 2 * (qr + c0));
+        q[j][1] = at(qp, 2 * (qr + c1));
       }
     }
   }
   __device__ __forceinline__ void fetch_trig(int first, int n, int pos0, const ChunkArgs& a) {
-    if (!ROT) return;
+    if (!ROT || a.rot == 0) return;
 #pragma unroll
     for (int j = 0; j < PAIRS; ++j) {
       int r, c0, c1;
       bool rotates;
-      const bool in = place((first + j) * kThreads + (int)threadIdx.x, a, r, c0, c1, rotates) && r < n;
-      if (in && rotates) {
-        const int64_t pos = pos0 + r < a.max_positions ? pos0 + r : a.max_positions - 1;
-        load_vec<8>(a.cos_sin + pos * a.rot + c0, cs[j]);
-        load_vec<8>(a.cos_sin + pos * a.rot + (a.rot >> 1) + c0, sn[j]);
-      } else {
+      place((first + j) * kThreads + (int)threadIdx.x, a, r, c0, c1, rotates);
+      r = pos0 + (r < n ? r : n - 1);
+      r = r < (int)a.max_positions ? r : (int)a.max_positions - 1;
+      const uint32_t from = 4 * ((uint32_t)r * (uint32_t)a.rot + (rotates ? c0 : 0));
 #pragma unroll
-        for (int e = 0; e < 8; ++e) {
-          cs[j][e] = 1.f;
-          sn[j][e] = 0.f;
-        }
+      for (int i = 0; i < 2; ++i) {
+        cs[j][i] = __builtin_bit_cast(f32x4, at(a.cos_sin, from + 16 * i));
+        sn[j][i] = __builtin_bit_cast(f32x4, at(a.cos_sin, from + 2 * a.rot + 16 * i));
       }
     }
   }
@@ -119,10 +123,11 @@ struct ChunkLoader {
     for (int j = 0; j < kVPieces; ++j) {
       const int i = j * kThreads + (int)threadIdx.x, r = i / (kColumns / 8), c = (i % (kColumns / 8)) * 8;
       const int x = c % span, head = c / span;
-      v[j] = r < n && x < vlen ? load16(vp + r * a.v_stride + (int64_t)head * a.vd + x) : u32x4{0u, 0u, 0u, 0u};
+      v[j] = at(vp, 2 * ((uint32_t)(r < n ? r : n - 1) * (uint32_t)a.v_stride + head * a.vd + (x < vlen ? x : 0)));
     }
   }
-  __device__ __forceinline__ void finish(uint16_t* tile, int at0, int at1, const u32x4 (&w)[2], int j, float scale) const {
+  __device__ __forceinline__ void finish(uint16_t* tile, int r, int c0, int c1, const u32x4 (&w)[2], int j, bool rotates, float scale,
+                                         const ChunkArgs& a) const {
     u32x4 o0 = w[0], o1 = w[1];
     if (ROT || scale != 1.f) {
 #pragma unroll
@@ -130,17 +135,20 @@ struct ChunkLoader {
         const float x0 = bf16lo_to_f32(w[0][e]) * scale, x1 = bf16hi_to_f32(w[0][e]) * scale;
         const float y0 = bf16lo_to_f32(w[1][e]) * scale, y1 = bf16hi_to_f32(w[1][e]) * scale;
         if (ROT) {
-          const float *c = cs[ROT ? j : 0], *s = sn[ROT ? j : 0];
-          o0[e] = pack_bf16x2(x0 * c[2 * e] - y0 * s[2 * e], x1 * c[2 * e + 1] - y1 * s[2 * e + 1]);
-          o1[e] = pack_bf16x2(y0 * c[2 * e] + x0 * s[2 * e], y1 * c[2 * e + 1] + x1 * s[2 * e + 1]);
+          const int jj = ROT ? j : 0;
+          const float ca = rotates ? cs[jj][e >> 1][2 * (e & 1)] : 1.f, cb = rotates ? cs[jj][e >> 1][2 * (e & 1) + 1] : 1.f;
+          const float sa = rotates ? sn[jj][e >> 1][2 * (e & 1)] : 0.f, sb = rotates ? sn[jj][e >> 1][2 * (e & 1) + 1] : 0.f;
+          o0[e] = pack_bf16x2(x0 * ca - y0 * sa, x1 * cb - y1 * sb);
+          o1[e] = pack_bf16x2(y0 * ca + x0 * sa, y1 * cb + x1 * sb);
         } else {
           o0[e] = pack_bf16x2(x0, x1);
           o1[e] = pack_bf16x2(y0, y1);
         }
       }
     }
-    store16(tile + at0, o0);
-    store16(tile + at1, o1);
+    const u32x4 zero = {0u, 0u, 0u, 0u};
+    store16(tile + r * kPitch + c0, c0 < a.d ? o0 : zero);
+    store16(tile + r * kPitch + c1, c1 < a.d ? o1 : zero);
   }
   __device__ __forceinline__ void store_qk(int first, uint16_t* tk, uint16_t* tq, const ChunkArgs& a) const {
 #pragma unroll
@@ -148,8 +156,8 @@ struct ChunkLoader {
       int r, c0, c1;
       bool rotates;
       if (!place((first + j) * kThreads + (int)threadIdx.x, a, r, c0, c1, rotates)) continue;
-      finish(tk, r * kPitch + c0, r * kPitch + c1, k[j], j, a.k_scale);
-      if (!STATE_ONLY) finish(tq, r * kPitch + c0, r * kPitch + c1, q[j], j, 1.f);
+      finish(tk, r, c0, c1, k[j], j, rotates, a.k_scale, a);
+      if (!STATE_ONLY) finish(tq, r, c0, c1, q[j], j, rotates, 1.f, a);
     }
   }
   __device__ __forceinline__ void store_v(uint16_t* tv) const {
@@ -255,7 +263,7 @@ __global__ __launch_bounds__(256, DP <= 128 ? 2 : 1) void decayed_chunk_kernel(c
   constexpr bool kAhead = VEC && kPairsAll <= 2;          // a whole chunk fits the registers next to the accumulators
   constexpr int kPairs = kPairsAll <= 2 ? kPairsAll : 2;
   ChunkLoader<DP, STATE_ONLY, kPairs, NH == 1> ld;      // heads that rotate do not share keys
-  float dt_next = 0.f;
+  uint32_t dt_next = 0;      // this lane's time step of the next chunk, raw
   auto fetch = [&](int t) {
     const int m = t_end - t < kChunk ? t_end - t : kChunk;
     ld.fetch_qk(0, kp + (int64_t)t * a.k_stride, qp + (int64_t)t * a.q_stride, m, a);
@@ -263,7 +271,7 @@ __global__ __launch_bounds__(256, DP <= 128 ? 2 : 1) void decayed_chunk_kernel(c
     ld.fetch_v(vp + (int64_t)t * a.v_stride, m, kSpan, vlen, a);
   };
   auto fetch_dt = [&](int t) {
-    dt_next = a.dt && wave < NH && t + lane < t_end ? bf16lo_to_f32(a.dt[(int64_t)(t + lane) * a.dt_stride + decay_head]) : 0.f;
+    if (a.dt) dt_next = a.dt[(int64_t)(t + lane < t_end ? t + lane : t_end - 1) * a.dt_stride + decay_head];
   };
   if (kAhead) fetch(t_begin);
   fetch_dt(t_begin);
@@ -298,7 +306,7 @@ __global__ __launch_bounds__(256, DP <= 128 ? 2 : 1) void decayed_chunk_kernel(c
       float la = 0.f, s = 0.f, l;
       if (a.dt) {
         if (lane < n) {
-          s = softplus_f32(dt_next + dt_bias);
+          s = softplus_f32(bf16lo_to_f32(dt_next) + dt_bias);
           la = neg_a * s;
         }
         l = la;
@@ -582,6 +590,8 @@ extern "C" int mops_hip_decayed_chunks(const mops_hip_recurrence* r, const int32
   if (r->dt && (!r->dt_bias || !r->neg_a || r->dt_stride < r->heads)) return MOPS_HIP_EINVAL;
   if (r->rot < 0 || (r->rot & 1) || r->rot > r->d || (r->rot && (!r->cos_sin || r->max_positions <= 0))) return MOPS_HIP_EINVAL;
   if (!aligned16(r->state) || (seg_state && !aligned16(seg_state))) return MOPS_HIP_EALIGN;
+  // offsets inside a chunk and into the table are 32 bits
+  if (r->q_stride > (1 << 24) || r->k_stride > (1 << 24) || r->v_stride > (1 << 24) || r->max_positions * r->rot > (1 << 29)) return MOPS_HIP_EUNSUPPORTED;
   if (num_segments * r->heads * ((r->vd + 31) / 32) > 0x3fffffffLL) return MOPS_HIP_EUNSUPPORTED;
   ChunkArgs a;
   a.q = (const uint16_t*)r->q; a.k = (const uint16_t*)r->k; a.v = (const uint16_t*)r->v; a.dt = (const uint16_t*)r->dt;
