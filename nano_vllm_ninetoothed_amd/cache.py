@@ -44,6 +44,8 @@ class CacheManager:
 
     def hold(self, seq, n_tokens: int) -> None:
         """Gives seq the pages for n_tokens tokens and, if the model keeps state, a slot."""
+        if len(seq.block_table) * self.block_size >= n_tokens and (not self.uses_slots or seq.state_slot >= 0):
+            return      # the usual decode step
         if not self.can_hold(seq, n_tokens):
             raise RuntimeError("KV cache exhausted: this engine does not preempt; raise num_blocks or the number of state slots")
         if self.uses_slots and seq.state_slot < 0:

@@ -218,7 +218,8 @@ class Engine:
         self.g_pos[:bs] = pos
         self.g_pos32[:bs] = ctx["positions32"]
         self.g_states.fill_(-1)
-        self.g_states[:bs] = ctx["state_slots"]
+        if ctx["state_slots"] is not None:
+            self.g_states[:bs] = ctx["state_slots"]
         self.g_slots.fill_(-1)
         self.g_slots[:bs] = ctx["slot_mapping"]
         self.g_lens.zero_()
@@ -242,6 +243,13 @@ class Engine:
             return [-1] * (end - begin)
         bs, table = self.block_size, q.block_table
         return [table[t // bs] * bs + t % bs for t in range(begin, end)]
+
+    def _last_slots(self, seqs):
+        """Cache row of the last token of each sequence (the whole list at once: a decode step pays for every call)."""
+        if not self.cache.uses_pages:
+            return [-1] * len(seqs)
+        bs = self.block_size
+        return [q.block_table[-1] * bs + (len(q.token_ids) - 1) % bs for q in seqs]
 
     def _prepare_portions(self, seqs, counts):
         """Batch of the next counts[i] tokens of seqs[i] behind the num_cached tokens of earlier steps.  Layers run single
@@ -284,12 +292,13 @@ class Engine:
     def _prepare_decode(self, seqs):
         ids = [q.token_ids[-1] for q in seqs]
         pos = [len(q) - 1 for q in seqs]
-        slots = [self._slots(q, len(q) - 1, len(q))[0] for q in seqs]
+        slots = self._last_slots(seqs)
         p32 = self._to_dev(pos, torch.int32)
         lens = self._to_dev([len(q) for q in seqs], torch.int32)
         ctx = dict(is_prefill=False, slot_mapping=self._to_dev(slots, torch.int32), context_lens=lens,
                    block_tables=self._block_tables(seqs), n_decode=len(seqs), starts=p32, positions32=p32, token_context=lens,
-                   token_seq=None, cu_seqlens=None, state_slots=self._to_dev([q.state_slot for q in seqs], torch.int32))
+                   token_seq=None, cu_seqlens=None,
+                   state_slots=self._to_dev([q.state_slot for q in seqs], torch.int32) if self.cache.uses_slots else None)
         return self._to_dev(ids, torch.int64), self._to_dev(pos, torch.int64), ctx
 
     @torch.inference_mode()
@@ -478,9 +487,10 @@ class Engine:
                 a[4 * n:] = -1                       # state slots and block tables
                 a[:bs] = [q.row for q in seqs]
                 a[n:n + bs] = [len(q) - 1 for q in seqs]
-                a[2 * n:2 * n + bs] = [self._slots(q, len(q) - 1, len(q))[0] for q in seqs]
+                a[2 * n:2 * n + bs] = self._last_slots(seqs)
                 a[3 * n:3 * n + bs] = [len(q) for q in seqs]
-                a[4 * n:4 * n + bs] = [q.state_slot for q in seqs]
+                if self.cache.uses_slots:
+                    a[4 * n:4 * n + bs] = [q.state_slot for q in seqs]
                 tab = a[5 * n:].reshape(n, max_blocks)
                 for j, q in enumerate(seqs):
                     tab[j, :len(q.block_table)] = q.block_table
