@@ -20,7 +20,7 @@ __global__ __launch_bounds__(256) void clamped_glu_kernel(const T* __restrict__ 
   for (int e = 0; e < VEC; ++e) {
     const float gg = fminf(g[e], limit);
     const float uu = fminf(fmaxf(u[e], -limit), limit);
-    o[e] = gg * sigmoid_f32(alpha * gg) * (uu + 1.0f);
+    o[e] = gg * sigmoid_for<T>(alpha * gg) * (uu + 1.0f);
   }
   store_vec<VEC>(out + row * n + c, o);
 }

@@ -109,7 +109,7 @@ __global__ __launch_bounds__(256) void decayed_recurrence_kernel(const Recurrenc
       if (pos - lag >= 0)
         acc += a.conv_w[(int64_t)(a.taps - 1 - lag) * a.channels + c] * to_f32(ring[(int64_t)((pos - lag) % a.taps) * a.channels + c]);
     if (keep) ring[(int64_t)(pos % a.taps) * a.channels + c] = from_f32<T>(x);
-    return silu_f32(acc);
+    return silu_for<T>(acc);
   };
   for (int t = t_begin; t < t_end; ++t) {
     const int pos = start + (t - t_begin);
@@ -222,7 +222,7 @@ __global__ __launch_bounds__(256) void short_conv_kernel(const T* __restrict__ x
     for (int e = 0; e < VEC; ++e) acc[e] += wv[e] * v[e];
   }
 #pragma unroll
-  for (int e = 0; e < VEC; ++e) acc[e] = silu_f32(acc[e]);
+  for (int e = 0; e < VEC; ++e) acc[e] = silu_for<T>(acc[e]);
   store_vec<VEC>(out + t * channels + c, acc);
 }
 
@@ -271,7 +271,7 @@ __global__ __launch_bounds__(256) void short_conv_run_kernel(const T* __restrict
       acc[e] = b[e];
 #pragma unroll
       for (int l = 0; l < TAPS; ++l) acc[e] += wv[l][e] * win[l][e];
-      acc[e] = silu_f32(acc[e]);
+      acc[e] = silu_for<T>(acc[e]);
     }
     store_vec<8>(out + t * channels + c, acc);
   };

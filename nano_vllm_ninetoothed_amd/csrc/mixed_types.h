@@ -72,11 +72,13 @@ template <int VEC> __device__ __forceinline__ void store_vec(bf16_t* p, const fl
   }
 }
 
-// 1 / (1 + e^-v) from the hardware's base-2 exponential and reciprocal (about one ulp each).
-__device__ __forceinline__ float sigmoid_f32(float v) {
+// 1 / (1 + e^-v) for results of type T: bf16 from the hardware's base-2 exponential and reciprocal (about one ulp of float32
+// each), float from the library's exponential and a true division.
+template <typename T> __device__ __forceinline__ float sigmoid_for(float v) {
   return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * v));
 }
-__device__ __forceinline__ float silu_f32(float v) { return v * sigmoid_f32(v); }
+template <> __device__ __forceinline__ float sigmoid_for<float>(float v) { return 1.0f / (1.0f + expf(-v)); }
+template <typename T> __device__ __forceinline__ float silu_for(float v) { return v * sigmoid_for<T>(v); }
 // log(1 + e^v); beyond 20 the difference to v is below one ulp of v.
 __device__ __forceinline__ float softplus_f32(float v) { return v > 20.0f ? v : log1pf(expf(v)); }
 

@@ -107,7 +107,7 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(const T* __restri
     load_vec<VEC>(gr + c, g);
 #pragma unroll
     for (int e = 0; e < VEC; ++e) {
-      g[e] = silu_f32(g[e]);
+      g[e] = silu_for<T>(g[e]);
       if (GATE_FIRST) v[e] *= g[e];
     }
   };
