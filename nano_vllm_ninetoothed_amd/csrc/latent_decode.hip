@@ -122,154 +122,154 @@ __global__ __launch_bounds__(256, 2) void latent_decode_kernel(const LatentDecod
   const float scale_log2 = a.scale * 1.4426950408889634f;
 
   for (; remaining > 0; ++row, tile0 = 0) {
-  const int len = length_of(row), row_tiles = (len + kTileTokens - 1) / kTileTokens;
-  const int run = row_tiles - tile0 < remaining ? row_tiles - tile0 : remaining;
-  if (run <= 0) continue;
-  remaining -= run;
-  const int tok_begin = tile0 * kTileTokens;
-  tok_end = tok_begin + run * kTileTokens < len ? tok_begin + run * kTileTokens : len;
-  table = a.block_table + (int64_t)(a.row_seq ? a.row_seq[row] : row) * a.block_table_stride;
-  bool ok_next = issue(tok_begin);
-  __syncthreads();      // the last piece's tile has been read
+    const int len = length_of(row), row_tiles = (len + kTileTokens - 1) / kTileTokens;
+    const int run = row_tiles - tile0 < remaining ? row_tiles - tile0 : remaining;
+    if (run <= 0) continue;
+    remaining -= run;
+    const int tok_begin = tile0 * kTileTokens;
+    tok_end = tok_begin + run * kTileTokens < len ? tok_begin + run * kTileTokens : len;
+    table = a.block_table + (int64_t)(a.row_seq ? a.row_seq[row] : row) * a.block_table_stride;
+    bool ok_next = issue(tok_begin);
+    __syncthreads();      // the last piece's tile has been read
 
-  // ---- query rows [16 heads][k] through LDS into B operands: [latent | rotated part | zeros]
-  {
-    const int pos = len - 1;
-    const float* trig = a.cos_sin + (int64_t)(pos < a.max_positions ? pos : a.max_positions - 1) * rot;
+    // ---- query rows [16 heads][k] through LDS into B operands: [latent | rotated part | zeros]
+    {
+      const int pos = len - 1;
+      const float* trig = a.cos_sin + (int64_t)(pos < a.max_positions ? pos : a.max_positions - 1) * rot;
 #pragma unroll 1
-    for (int i = tid; i < kHeadTile * (lp >> 3); i += 256) {
-      const int hr = i / (lp >> 3), c = (i % (lp >> 3)) * 8;
-      const int head = ht * kHeadTile + hr;
-      u32x4 w = {0u, 0u, 0u, 0u};
-      if (head < heads && c < width) {
-        const uint16_t* ql = (const uint16_t*)a.q_latent + (row * heads + head) * kv_rank;
-        const uint16_t* qr = (const uint16_t*)a.q_rot + (int64_t)row * a.q_rot_token_stride + head * a.q_rot_head_stride;
-        if (p.vec_q && c + 8 <= kv_rank) {
-          w = load16(ql + c);
-        } else if (p.vec_q) {       // four pairs of the rotated part
-          const int d = c - kv_rank;
-          const u32x4 raw = load16(qr + d);
-          const f32x4 cs = *reinterpret_cast<const f32x4*>(trig + d / 2), sn = *reinterpret_cast<const f32x4*>(trig + rot / 2 + d / 2);
+      for (int i = tid; i < kHeadTile * (lp >> 3); i += 256) {
+        const int hr = i / (lp >> 3), c = (i % (lp >> 3)) * 8;
+        const int head = ht * kHeadTile + hr;
+        u32x4 w = {0u, 0u, 0u, 0u};
+        if (head < heads && c < width) {
+          const uint16_t* ql = (const uint16_t*)a.q_latent + (row * heads + head) * kv_rank;
+          const uint16_t* qr = (const uint16_t*)a.q_rot + (int64_t)row * a.q_rot_token_stride + head * a.q_rot_head_stride;
+          if (p.vec_q && c + 8 <= kv_rank) {
+            w = load16(ql + c);
+          } else if (p.vec_q) {       // four pairs of the rotated part
+            const int d = c - kv_rank;
+            const u32x4 raw = load16(qr + d);
+            const f32x4 cs = *reinterpret_cast<const f32x4*>(trig + d / 2), sn = *reinterpret_cast<const f32x4*>(trig + rot / 2 + d / 2);
 #pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            const float u = bf16lo_to_f32(raw[e]), v = bf16hi_to_f32(raw[e]);
-            w[e] = pack_bf16x2(u * cs[e] - v * sn[e], v * cs[e] + u * sn[e]);
-          }
-        } else {
-#pragma unroll 1
-          for (int e = 0; e < 8; ++e) {
-            const int k = c + e;
-            uint32_t bits = 0;
-            if (k < kv_rank) {
-              bits = ql[k];
-            } else if (k < width) {
-              const int d = k - kv_rank, i2 = d >> 1;
-              const float u = bf16lo_to_f32(qr[2 * i2]), v = bf16lo_to_f32(qr[2 * i2 + 1]), cs = trig[i2], sn = trig[rot / 2 + i2];
-              bits = f32_to_bf16_bits((d & 1) ? v * cs + u * sn : u * cs - v * sn);
+            for (int e = 0; e < 4; ++e) {
+              const float u = bf16lo_to_f32(raw[e]), v = bf16hi_to_f32(raw[e]);
+              w[e] = pack_bf16x2(u * cs[e] - v * sn[e], v * cs[e] + u * sn[e]);
             }
-            tile[hr * lp + k] = (uint16_t)bits;
+          } else {
+#pragma unroll 1
+            for (int e = 0; e < 8; ++e) {
+              const int k = c + e;
+              uint32_t bits = 0;
+              if (k < kv_rank) {
+                bits = ql[k];
+              } else if (k < width) {
+                const int d = k - kv_rank, i2 = d >> 1;
+                const float u = bf16lo_to_f32(qr[2 * i2]), v = bf16lo_to_f32(qr[2 * i2 + 1]), cs = trig[i2], sn = trig[rot / 2 + i2];
+                bits = f32_to_bf16_bits((d & 1) ? v * cs + u * sn : u * cs - v * sn);
+              }
+              tile[hr * lp + k] = (uint16_t)bits;
+            }
+            continue;
           }
-          continue;
         }
+        store16(tile + hr * lp + c, w);
       }
-      store16(tile + hr * lp + c, w);
     }
-  }
-  __syncthreads();
-  bf16x8 qb[NQ];
-#pragma unroll
-  for (int i = 0; i < NQ; ++i) {
-    const int ks = 2 * i + kh;
-    qb[i] = ks < ksteps ? tile_row(tile, lp, n, 32 * ks + 8 * jj) : __builtin_bit_cast(bf16x8, u32x4{0u, 0u, 0u, 0u});
-  }
-
-  f32x4 acc[NT];
-#pragma unroll
-  for (int i = 0; i < NT; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-  float m_run = -INFINITY, l_run = 0.f;
-
-  for (int tok0 = tok_begin; tok0 < tok_end; tok0 += kTileTokens) {
-    const bool ok = ok_next;
-    __syncthreads();      // the last tile (or the query rows) have been read
-#pragma unroll
-    for (int j = 0; j < NQ; ++j)
-      if (pr[j] < kTileTokens) store16(tile + pr[j] * lp + pc[j], reg[j]);
     __syncthreads();
-    if (tok0 + kTileTokens < tok_end) ok_next = issue(tok0 + kTileTokens);
-    f32x4 s = {0.f, 0.f, 0.f, 0.f};
+    bf16x8 qb[NQ];
 #pragma unroll
     for (int i = 0; i < NQ; ++i) {
       const int ks = 2 * i + kh;
-      if (ks < ksteps) s = mfma16(tile_row(tile, lp, 16 * tt + n, 32 * ks + 8 * jj), qb[i], s);
+      qb[i] = ks < ksteps ? tile_row(tile, lp, n, 32 * ks + 8 * jj) : __builtin_bit_cast(bf16x8, u32x4{0u, 0u, 0u, 0u});
     }
+
+    f32x4 acc[NT];
 #pragma unroll
-    for (int e = 0; e < 4; ++e) part_s[kh][16 * tt + 4 * jj + e][n] = s[e];
-    __syncthreads();
-    const int valid = ok ? tok_end - tok0 : 0;
-    float sv[8], m_loc = -INFINITY;
+    for (int i = 0; i < NT; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    float m_run = -INFINITY, l_run = 0.f;
+
+    for (int tok0 = tok_begin; tok0 < tok_end; tok0 += kTileTokens) {
+      const bool ok = ok_next;
+      __syncthreads();      // the last tile (or the query rows) have been read
 #pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      const int t = 4 * jj + (e & 3) + 16 * (e >> 2);
-      sv[e] = t < valid ? (part_s[0][t][n] + part_s[1][t][n]) * scale_log2 : -INFINITY;
-      m_loc = fmaxf(m_loc, sv[e]);
-    }
-    m_loc = fmaxf(m_loc, __shfl_xor(m_loc, 16, kWave));
-    m_loc = fmaxf(m_loc, __shfl_xor(m_loc, 32, kWave));
-    const float m_new = fmaxf(m_run, m_loc);
-    const float m_safe = m_new == -INFINITY ? 0.f : m_new;
-    const float alpha = __builtin_amdgcn_exp2f(m_run - m_safe);
-    float pv[8], psum = 0.f;
+      for (int j = 0; j < NQ; ++j)
+        if (pr[j] < kTileTokens) store16(tile + pr[j] * lp + pc[j], reg[j]);
+      __syncthreads();
+      if (tok0 + kTileTokens < tok_end) ok_next = issue(tok0 + kTileTokens);
+      f32x4 s = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      pv[e] = __builtin_amdgcn_exp2f(sv[e] - m_safe);
-      psum += pv[e];
-    }
-    l_run = l_run * alpha + psum;
-    m_run = m_new;
-    if (__any(alpha != 1.0f)) {
+      for (int i = 0; i < NQ; ++i) {
+        const int ks = 2 * i + kh;
+        if (ks < ksteps) s = mfma16(tile_row(tile, lp, 16 * tt + n, 32 * ks + 8 * jj), qb[i], s);
+      }
 #pragma unroll
-      for (int i = 0; i < NT; ++i) acc[i] *= alpha;
-    }
-    bf16x8 hi, lo;
-    split8(pv, hi, lo);
+      for (int e = 0; e < 4; ++e) part_s[kh][16 * tt + 4 * jj + e][n] = s[e];
+      __syncthreads();
+      const int valid = ok ? tok_end - tok0 : 0;
+      float sv[8], m_loc = -INFINITY;
 #pragma unroll
-    for (int i = 0; i < NT; ++i) {
-      const int c0 = 16 * (wave + 4 * i);
-      if (c0 < kv_rank) {
-        const bf16x8 ca = __builtin_bit_cast(bf16x8, join(tile_block_columns(tile, lp, 4 * jj, c0, lane), tile_block_columns(tile, lp, 16 + 4 * jj, c0, lane)));
-        acc[i] = mfma16(ca, hi, acc[i]);
-        acc[i] = mfma16(ca, lo, acc[i]);
+      for (int e = 0; e < 8; ++e) {
+        const int t = 4 * jj + (e & 3) + 16 * (e >> 2);
+        sv[e] = t < valid ? (part_s[0][t][n] + part_s[1][t][n]) * scale_log2 : -INFINITY;
+        m_loc = fmaxf(m_loc, sv[e]);
+      }
+      m_loc = fmaxf(m_loc, __shfl_xor(m_loc, 16, kWave));
+      m_loc = fmaxf(m_loc, __shfl_xor(m_loc, 32, kWave));
+      const float m_new = fmaxf(m_run, m_loc);
+      const float m_safe = m_new == -INFINITY ? 0.f : m_new;
+      const float alpha = __builtin_amdgcn_exp2f(m_run - m_safe);
+      float pv[8], psum = 0.f;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        pv[e] = __builtin_amdgcn_exp2f(sv[e] - m_safe);
+        psum += pv[e];
+      }
+      l_run = l_run * alpha + psum;
+      m_run = m_new;
+      if (__any(alpha != 1.0f)) {
+#pragma unroll
+        for (int i = 0; i < NT; ++i) acc[i] *= alpha;
+      }
+      bf16x8 hi, lo;
+      split8(pv, hi, lo);
+#pragma unroll
+      for (int i = 0; i < NT; ++i) {
+        const int c0 = 16 * (wave + 4 * i);
+        if (c0 < kv_rank) {
+          const bf16x8 ca = __builtin_bit_cast(bf16x8, join(tile_block_columns(tile, lp, 4 * jj, c0, lane), tile_block_columns(tile, lp, 16 + 4 * jj, c0, lane)));
+          acc[i] = mfma16(ca, hi, acc[i]);
+          acc[i] = mfma16(ca, lo, acc[i]);
+        }
       }
     }
-  }
-  float l_tot = l_run + __shfl_xor(l_run, 16, kWave);
-  l_tot += __shfl_xor(l_tot, 32, kWave);
-  if (h >= heads) continue;
-  if (run == row_tiles) {
-    const float inv = l_tot > 0.f ? 1.0f / l_tot : 0.f;
-    uint16_t* orow = (uint16_t*)a.out + ((int64_t)row * heads + h) * kv_rank;
+    float l_tot = l_run + __shfl_xor(l_run, 16, kWave);
+    l_tot += __shfl_xor(l_tot, 32, kWave);
+    if (h >= heads) continue;
+    if (run == row_tiles) {
+      const float inv = l_tot > 0.f ? 1.0f / l_tot : 0.f;
+      uint16_t* orow = (uint16_t*)a.out + ((int64_t)row * heads + h) * kv_rank;
+#pragma unroll
+      for (int i = 0; i < NT; ++i) {
+        const int r = 16 * (wave + 4 * i) + 4 * jj;
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          if (r + e < kv_rank) orow[r + e] = (uint16_t)f32_to_bf16_bits(acc[i][e] * inv);
+      }
+      continue;
+    }
+    const int64_t slot = (((int64_t)ht * p.columns + column) * 2 + (tile0 > 0 ? 0 : 1)) * kHeadTile + n;
+    float* prow = p.part + slot * kv_rank;
 #pragma unroll
     for (int i = 0; i < NT; ++i) {
       const int r = 16 * (wave + 4 * i) + 4 * jj;
 #pragma unroll
       for (int e = 0; e < 4; ++e)
-        if (r + e < kv_rank) orow[r + e] = (uint16_t)f32_to_bf16_bits(acc[i][e] * inv);
+        if (r + e < kv_rank) prow[r + e] = acc[i][e];
     }
-    continue;
-  }
-  const int64_t slot = (((int64_t)ht * p.columns + column) * 2 + (tile0 > 0 ? 0 : 1)) * kHeadTile + n;
-  float* prow = p.part + slot * kv_rank;
-#pragma unroll
-  for (int i = 0; i < NT; ++i) {
-    const int r = 16 * (wave + 4 * i) + 4 * jj;
-#pragma unroll
-    for (int e = 0; e < 4; ++e)
-      if (r + e < kv_rank) prow[r + e] = acc[i][e];
-  }
-  if (wave == 0 && jj == 0) {
-    p.ml[2 * slot] = m_run;
-    p.ml[2 * slot + 1] = l_tot;
-  }
+    if (wave == 0 && jj == 0) {
+      p.ml[2 * slot] = m_run;
+      p.ml[2 * slot + 1] = l_tot;
+    }
   }
 }
 
