@@ -142,7 +142,7 @@ __global__ __launch_bounds__(256, 2) void latent_decode_kernel(const LatentDecod
         const int head = ht * kHeadTile + hr;
         u32x4 w = {0u, 0u, 0u, 0u};
         if (head < heads && c < width) {
-          const uint16_t* ql = (const uint16_t*)a.q_latent + (row * heads + head) * kv_rank;
+          const uint16_t* ql = (const uint16_t*)a.q_latent + ((int64_t)row * heads + head) * kv_rank;
           const uint16_t* qr = (const uint16_t*)a.q_rot + (int64_t)row * a.q_rot_token_stride + head * a.q_rot_head_stride;
           if (p.vec_q && c + 8 <= kv_rank) {
             w = load16(ql + c);
