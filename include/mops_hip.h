@@ -336,13 +336,21 @@ int mops_hip_linear_tune(int64_t m, int64_t n, int64_t k, int64_t distinct_weigh
 #define MOPS_HIP_BF16 0
 #define MOPS_HIP_F32 1
 
-/* residual[i, :] = float(table[ids[i], :]) and act[i, :] = table[ids[i], :]; an id outside [0, vocab) gives zeros. */
-int mops_hip_embed_residual(const int64_t* ids, const void* table, int64_t table_row_stride, int dtype,
+/* residual[i, :] = scale * table[ids[i], :] and act[i, :] = the same in `dtype` (act may be NULL); an id outside [0, vocab)
+ * gives zeros. */
+int mops_hip_embed_residual(const int64_t* ids, const void* table, int64_t table_row_stride, int dtype, float scale,
                             float* residual, void* act, int64_t n_ids, int64_t vocab, int64_t width, void* stream);
 
 /* residual += y / sqrt(mean(y^2) + eps) * (weight_offset + weight), rowwise and in place; act = the new residual in `dtype`. */
 int mops_hip_norm_residual_add(float* residual, const void* y, int64_t y_row_stride, const void* weight, float weight_offset,
                                float eps, void* act, int dtype, int64_t rows, int64_t n, void* stream);
+
+/*
+ * Norms behind one sublayer and in front of the next: with y_r the sum of the rows r * parts .. r * parts + parts - 1 of y,
+ * residual_r += y_r / sqrt(mean(y_r^2) + eps) * w_out in place, out_r = residual_r / sqrt(mean(residual_r^2) + eps) * w_in.
+ */
+int mops_hip_add_norm_norm(float* residual, const void* y, int64_t y_row_stride, int64_t parts, const void* w_out,
+                           const void* w_in, float eps, void* out, int dtype, int64_t rows, int64_t n, void* stream);
 
 /* out = x / sqrt(mean(x^2) + eps) * (weight_offset + weight) of float32 rows. */
 int mops_hip_rms_norm_f32(const float* x, const void* weight, float weight_offset, float eps, void* out, int dtype,
@@ -365,8 +373,11 @@ int mops_hip_clamped_glu(const void* gate, int64_t gate_row_stride, const void* 
  * A linear recurrence with one decay per head and token (see csrc/decayed_recurrence.hip):
  *   S_t = a_t S_(t-1) + k_t (s_t v_t)^T,   o_t = S_t^T q_t + skip v_t
  * q, k: [tokens, groups * d], v, out: [tokens, heads * vd] with token strides in elements; value head h uses q/k head
- * h / (heads / groups).  Exactly one of `decay` (float [heads]: constant) and `dt` ([tokens, heads] in `dtype`, with
- * dt_bias and neg_a float [heads]: s = softplus(dt + dt_bias), a = exp(neg_a * s)) is given; skip may be NULL.
+ * h / (heads / groups).  Exactly one of `decay` (float [heads]: constant), `dt` ([tokens, heads] in `dtype`, with
+ * dt_bias and neg_a float [heads]: s = softplus(dt + dt_bias), a = exp(neg_a * s)) and `channel_decay` is given; skip may be NULL.
+ * channel_decay: float [tokens, heads * d], natural logarithms of a decay per token, head and key channel, with a token stride
+ * in elements; then groups == heads, no skip and no convolution, and with bonus u (float [heads * d])
+ *   o_t = (S_(t-1) + diag(u) k_t v_t^T)^T q_t,   S_t = diag(a_t) S_(t-1) + k_t v_t^T
  * rot > 0 rotates dimensions i and i + rot/2 of q and k (i < rot/2) by row `position` of cos_sin [max_positions, rot]
  * (cosines, then sines); k is multiplied by k_scale afterwards.
  * cu_seqlens: int32 [batch + 1], or NULL when every sequence brings one token.  starts[b]: position of the first token of
@@ -392,6 +403,8 @@ typedef struct {
   const float *conv_weight, *conv_bias;
   void* conv_ring;
   int64_t taps, channels, q_channel, k_channel, v_channel;
+  const float *channel_decay, *bonus;
+  int64_t channel_decay_stride;
   float k_scale;
   int dtype;
 } mops_hip_recurrence;
@@ -489,6 +502,84 @@ int mops_hip_latent_prefill(const void* q, int64_t q_token_stride, int64_t q_hea
                             const void* kr, int64_t kr_stride, const void* vt, int64_t vt_stride, const int32_t* tiles,
                             int64_t num_tiles, void* out, int64_t heads, int64_t dim, int64_t rot_dim, int64_t vdim, float scale,
                             void* stream);
+
+/*
+ * Time mixing (csrc/token_mix.hip).  token_mix: out[p][t] = x[t] + (x[t-1] - x[t]) * mu[p], mu float [parts, width], out
+ * [parts, tokens, width].  The row in front of a sequence's first token of the step is row state_slots[b] of before
+ * [num_slots, width] (zeros where starts[b] == 0 or the slot is negative), which receives the sequence's last row.
+ * token_seq and cu_seqlens (both or neither): packed portions; NULL: one token per sequence.
+ * low_rank_decay: out[t, c] = -exp(sum over r of w2[c, r] tanh(z[t, r]) + w0[c]), float; rank <= 4096.
+ */
+int mops_hip_token_mix(const void* x, int64_t x_row_stride, const float* mu, int64_t parts, void* before, int64_t num_slots,
+                       const int32_t* token_seq, const int32_t* cu_seqlens, const int32_t* starts, const int32_t* state_slots,
+                       void* out, int dtype, int64_t tokens, int64_t width, void* stream);
+int mops_hip_low_rank_decay(const void* z, int64_t z_row_stride, const void* w2, const float* w0, float* out, int dtype,
+                            int64_t tokens, int64_t channels, int64_t rank, void* stream);
+
+/* out = max(x, 0)^2. */
+int mops_hip_squared_relu(const void* x, int64_t x_row_stride, void* out, int dtype, int64_t rows, int64_t n, void* stream);
+
+/*
+ * Attention with a linear distance bias (csrc/biased_attention.hip).  With dp and vp the sizes dim and vdim rounded up to
+ * multiples of 8: q [rows, heads, dp], k_pages [num_slots or num_blocks * block_size, kv_heads, dp], v_pages [.., kv_heads, vp].
+ * attention_prepare: qkv rows [heads * dim | kv_heads * dim | kv_heads * vdim]; q = RMS norm over all of its elements * q_weight *
+ * q_factor[position] (q_factor: float [max_positions], or NULL), k = RMS norm over all of its elements * k_weight; k and v go to
+ * row slot_mapping[t] of the pages (slot < 0: nowhere).  Padding is written as zeros.
+ */
+typedef struct {
+  const void* qkv;
+  int64_t qkv_stride;
+  const void *q_weight, *k_weight;
+  const float* q_factor;
+  int64_t max_positions;
+  const int32_t *positions, *slot_mapping;
+  void *q, *k_pages, *v_pages;
+  int64_t num_slots, tokens, heads, kv_heads, dim, vdim;
+  float eps;
+  int dtype;
+} mops_hip_attention_prepare_args;
+int mops_hip_attention_prepare(const mops_hip_attention_prepare_args* a, void* stream);
+
+/*
+ * Query row r (at position context_lens[r] - 1) sees the first context_lens[r] tokens of sequence row_seq[r] (row r itself when
+ * row_seq is NULL); 0 gives zeros.  score = q . k * scale - slopes[h] * distance (slopes float [heads], or NULL), softmax,
+ * out [rows, heads, vdim].  A block table entry outside [0, num_blocks) counts as an empty block.
+ * biased_attention_rows: the plain form; dim <= 2048, vdim <= 1024.
+ */
+typedef struct {
+  const void *q, *k_pages, *v_pages;
+  const float* slopes;
+  const int32_t *row_seq, *context_lens, *block_table;
+  int64_t block_table_stride, block_size, num_blocks, max_blocks;
+  void* out;
+  int64_t rows, heads, kv_heads, dim, vdim;
+  float scale;
+  int dtype;
+} mops_hip_biased_attention;
+int mops_hip_biased_attention_rows(const mops_hip_biased_attention* a, void* stream);
+
+/*
+ * Mixture of experts (csrc/moe.hip).  moe_route: logits = router [experts, width] h in float32; chosen, score [tokens * top] =
+ * the experts with the largest logits and the sigmoids of these; rank [tokens * top] is scratch, counts [experts] must be zeros
+ * and receives the choices per expert; rows [tokens * top] lists the choices (token * top + place) ordered by expert, tiles
+ * [1 + 3 * moe_max_tiles] = number of blocks, then (expert, first row, rows) of each.  block_rows: 32, or 128 (bf16).
+ * moe_gate_up: w [experts][2 * up_at][width], gate rows from 0, up rows from up_at on; y [tokens * top rows in the order of
+ * `rows`], y = silu(score W_gate h) * (score W_up h).  moe_down: w [experts][width][depth], depth >= ff, the columns behind ff
+ * zeros in w and finite in y; z [tokens * top] in the order of the choices.  experts <= 1024.
+ */
+typedef struct {
+  int32_t *rows, *tiles;
+  float* score;
+  int64_t tokens, experts, top, width, ff, block_rows;
+  int dtype;
+} mops_hip_moe;
+int64_t mops_hip_moe_max_tiles(int64_t tokens, int64_t experts, int64_t top, int64_t block_rows);
+int mops_hip_moe_route(const void* h, int64_t h_row_stride, const void* router, int32_t* chosen, int32_t* rank, int32_t* counts,
+                       const mops_hip_moe* m, void* stream);
+int mops_hip_moe_gate_up(const void* h, int64_t h_row_stride, const void* w, int64_t up_at, void* y, int64_t y_row_stride,
+                         const mops_hip_moe* m, void* stream);
+int mops_hip_moe_down(const void* y, int64_t y_row_stride, const void* w, int64_t depth, void* z, int64_t z_row_stride,
+                      const mops_hip_moe* m, void* stream);
 
 #ifdef __cplusplus
 }

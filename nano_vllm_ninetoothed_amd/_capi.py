@@ -21,6 +21,7 @@ class Recurrence(Structure):
                 + [(n, c_int64) for n in ("dt_stride", "batch", "heads", "groups", "d", "vd", "rot", "max_positions")]
                 + [(n, c_void_p) for n in ("conv_weight", "conv_bias", "conv_ring")]
                 + [(n, c_int64) for n in ("taps", "channels", "q_channel", "k_channel", "v_channel")]
+                + [("channel_decay", c_void_p), ("bonus", c_void_p), ("channel_decay_stride", c_int64)]
                 + [("k_scale", c_float), ("dtype", c_int)])
 
 
@@ -32,6 +33,27 @@ class LatentRows(Structure):
                 + [(n, c_int64) for n in ("block_table_stride", "block_size", "num_blocks", "max_blocks")]
                 + [("out", c_void_p)] + [(n, c_int64) for n in ("rows", "heads", "kv_rank", "rot_dim")]
                 + [("scale", c_float), ("dtype", c_int)])
+
+
+class AttentionPrepare(Structure):
+    """mops_hip_attention_prepare_args of the header, field by field."""
+    _fields_ = ([("qkv", c_void_p), ("qkv_stride", c_int64)] + [(n, c_void_p) for n in ("q_weight", "k_weight", "q_factor")]
+                + [("max_positions", c_int64)] + [(n, c_void_p) for n in ("positions", "slot_mapping", "q", "k_pages", "v_pages")]
+                + [(n, c_int64) for n in ("num_slots", "tokens", "heads", "kv_heads", "dim", "vdim")] + [("eps", c_float), ("dtype", c_int)])
+
+
+class BiasedAttention(Structure):
+    """mops_hip_biased_attention of the header, field by field."""
+    _fields_ = ([(n, c_void_p) for n in ("q", "k_pages", "v_pages", "slopes", "row_seq", "context_lens", "block_table")]
+                + [(n, c_int64) for n in ("block_table_stride", "block_size", "num_blocks", "max_blocks")]
+                + [("out", c_void_p)] + [(n, c_int64) for n in ("rows", "heads", "kv_heads", "dim", "vdim")]
+                + [("scale", c_float), ("dtype", c_int)])
+
+
+class Moe(Structure):
+    """mops_hip_moe of the header, field by field."""
+    _fields_ = ([(n, c_void_p) for n in ("rows", "tiles", "score")]
+                + [(n, c_int64) for n in ("tokens", "experts", "top", "width", "ff", "block_rows")] + [("dtype", c_int)])
 
 
 # name -> (restype, argtypes); the exported surface declared in include/mops_hip.h
@@ -73,9 +95,11 @@ SIGNATURES = {
                                             c_int64, c_int64, c_float, c_void_p]),
     "mops_hip_linear_bf16": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int64, c_int64,
                                      c_int64, c_void_p, c_int64, c_void_p]),
-    "mops_hip_embed_residual": (c_int, [c_void_p, c_void_p, c_int64, c_int, c_void_p, c_void_p, c_int64, c_int64, c_int64, c_void_p]),
+    "mops_hip_embed_residual": (c_int, [c_void_p, c_void_p, c_int64, c_int, c_float, c_void_p, c_void_p, c_int64, c_int64, c_int64, c_void_p]),
     "mops_hip_norm_residual_add": (c_int, [c_void_p, c_void_p, c_int64, c_void_p, c_float, c_float, c_void_p, c_int, c_int64, c_int64,
                                            c_void_p]),
+    "mops_hip_add_norm_norm": (c_int, [c_void_p, c_void_p, c_int64, c_int64, c_void_p, c_void_p, c_float, c_void_p, c_int, c_int64, c_int64,
+                                       c_void_p]),
     "mops_hip_rms_norm_f32": (c_int, [c_void_p, c_void_p, c_float, c_float, c_void_p, c_int, c_int64, c_int64, c_void_p]),
     "mops_hip_gated_group_norm": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_float, c_int, c_void_p, c_int, c_int64,
                                           c_int64, c_int64, c_void_p]),
@@ -100,11 +124,21 @@ SIGNATURES = {
     "mops_hip_latent_prefill": (c_int, [c_void_p, c_int64, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_void_p,
                                         c_int64, c_void_p, c_int64, c_int64, c_int64, c_int64, c_float, c_void_p]),
     "mops_hip_rotate_pairs": (c_int, [c_void_p, c_int64, c_int64, c_void_p, c_void_p, c_int64, c_int64, c_int64, c_int64, c_void_p]),
+    "mops_hip_token_mix": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
+                                   c_int, c_int64, c_int64, c_void_p]),
+    "mops_hip_low_rank_decay": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int, c_int64, c_int64, c_int64, c_void_p]),
+    "mops_hip_squared_relu": (c_int, [c_void_p, c_int64, c_void_p, c_int, c_int64, c_int64, c_void_p]),
+    "mops_hip_attention_prepare": (c_int, [POINTER(AttentionPrepare), c_void_p]),
+    "mops_hip_biased_attention_rows": (c_int, [POINTER(BiasedAttention), c_void_p]),
+    "mops_hip_moe_max_tiles": (c_int64, [c_int64] * 4),
+    "mops_hip_moe_route": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p, POINTER(Moe), c_void_p]),
+    "mops_hip_moe_gate_up": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, POINTER(Moe), c_void_p]),
+    "mops_hip_moe_down": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, POINTER(Moe), c_void_p]),
     "mops_hip_linear_pin_solution": (c_int, [c_int64, c_int64, c_int64, c_int]),
     "mops_hip_linear_tune": (c_int, [c_int64, c_int64, c_int64, c_int64, c_int, c_void_p, c_int64, c_void_p, c_void_p, c_void_p]),
 }
 
-ABI_VERSION = 10
+ABI_VERSION = 11
 
 _lib = None
 

@@ -579,7 +579,7 @@ extern "C" int mops_hip_decayed_chunks(const mops_hip_recurrence* r, const int32
   using namespace mops;
   if (!r || r->batch < 0 || num_segments < 0) return MOPS_HIP_EINVAL;
   if (r->batch == 0 || num_segments == 0) return MOPS_HIP_OK;
-  if (r->dtype != MOPS_HIP_BF16 || r->conv_weight) return MOPS_HIP_EUNSUPPORTED;
+  if (r->dtype != MOPS_HIP_BF16 || r->conv_weight || r->channel_decay) return MOPS_HIP_EUNSUPPORTED;
   if (!r->q || !r->k || !r->v || !r->out || !r->state || !r->state_slots || !r->starts || !r->cu_seqlens || !segments) return MOPS_HIP_EINVAL;
   if (!seg_state != !seg_decay || (seg_state && !seq_segments) || (!seg_state && num_segments > r->batch)) return MOPS_HIP_EINVAL;
   if (r->heads <= 0 || r->groups <= 0 || r->heads % r->groups || r->d <= 0 || r->vd <= 0 || r->num_slots <= 0) return MOPS_HIP_EINVAL;

@@ -1,11 +1,14 @@
-// Linear recurrences with one decay per head and token, carried from token to token in float32:
+// Linear recurrences with one decay per head (or key channel) and token, carried from token to token in float32:
 //
 //   S_t = a_t S_(t-1) + k_t (s_t v_t)^T        S is [d x vd] per head, kept transposed in memory: state[slot][head][vd][pitch]
 //   o_t = S_t^T q_t + skip v_t
 //
-// Two ways to the decay a and the input scale s:
+// Ways to the decay a and the input scale s:
 //   constant      a = decay[head], s = 1                                     (linear attention with a fixed decay)
 //   time steps    s = softplus(dt + dt_bias[head]), a = exp(neg_a[head] s)   (state-space layers; skip = D[head])
+//   per channel   S_t = diag(exp(channel_decay_t)) S_(t-1) + k_t v_t^T, channel_decay a float logarithm per token, head and key
+//                 channel; the output looks at the state in front of the token and weighs the token itself by a bonus u per
+//                 channel: o_t = (S_(t-1) + diag(u) k_t v_t^T)^T q_t
 // q and k may be rotated on their first rot dimensions (dimension i with i + rot/2) by the row of a cos/sin table, and k is
 // multiplied by k_scale after that.  Query/key heads may be shared by heads / groups consecutive value heads.
 //
@@ -38,6 +41,8 @@ struct RecurrenceArgs {
   const void* dt;
   int64_t dt_stride;
   const float *dt_bias, *neg_a, *skip;
+  const float *channel_decay, *bonus;
+  int64_t channel_decay_stride;
   const float* cos_sin;
   int rot;
   int64_t max_positions;
@@ -50,11 +55,11 @@ struct RecurrenceArgs {
 };
 
 // cu_seqlens == nullptr: sequence b is the single token b.
-template <typename T, int DPT, int RPT, bool CONV>
+template <typename T, int DPT, int RPT, bool CONV, bool CHANNEL>
 __global__ __launch_bounds__(256) void decayed_recurrence_kernel(const RecurrenceArgs a) {
   constexpr int kRows = 16 * RPT;
   constexpr int kDim = 16 * DPT;
-  __shared__ __align__(16) float sq[kDim], sk[kDim], sv[kRows];
+  __shared__ __align__(16) float sq[kDim], sk[kDim], sv[kRows], sa[CHANNEL ? kDim : 1], su[CHANNEL ? kDim : 1];
   const int tiles = (a.vd + kRows - 1) / kRows;
   const int tile = blockIdx.x % tiles;
   const int h = (blockIdx.x / tiles) % a.heads;
@@ -136,6 +141,10 @@ __global__ __launch_bounds__(256) void decayed_recurrence_kernel(const Recurrenc
       }
       sq[i] = qv;
       sk[i] = kv;
+      if (CHANNEL) {
+        sa[i] = i < a.d ? expf(a.channel_decay[t * a.channel_decay_stride + (int64_t)g * a.d + i]) : 0.f;
+        su[i] = i < a.d ? a.bonus[(int64_t)g * a.d + i] * kv : 0.f;
+      }
     }
     for (int i = tid; i < kRows; i += 256) {
       float x = 0.f;
@@ -151,13 +160,18 @@ __global__ __launch_bounds__(256) void decayed_recurrence_kernel(const Recurrenc
       decay = expf(neg_a * scale);
     }
     __syncthreads();
-    float kk[DPT], qq[DPT];
+    float kk[DPT], qq[DPT], aa[CHANNEL ? DPT : 1];
+    float direct = 0.f;      // CHANNEL: this lane's part of sum u k q
 #pragma unroll
     for (int p = 0; p < DPT / kPiece; ++p)
 #pragma unroll
       for (int e = 0; e < kPiece; ++e) {
         kk[p * kPiece + e] = sk[piece_at(p) + e];
         qq[p * kPiece + e] = sq[piece_at(p) + e];
+        if (CHANNEL) {
+          aa[p * kPiece + e] = sa[piece_at(p) + e];
+          direct += su[piece_at(p) + e] * qq[p * kPiece + e];
+        }
       }
 #pragma unroll
     for (int r = 0; r < RPT; ++r) {
@@ -166,9 +180,15 @@ __global__ __launch_bounds__(256) void decayed_recurrence_kernel(const Recurrenc
       float dot = 0.f;
 #pragma unroll
       for (int e = 0; e < DPT; ++e) {
-        s[r][e] = decay * s[r][e] + kk[e] * xs;
-        dot += s[r][e] * qq[e];
+        if (CHANNEL) {
+          dot += s[r][e] * qq[e];
+          s[r][e] = aa[CHANNEL ? e : 0] * s[r][e] + kk[e] * x;
+        } else {
+          s[r][e] = decay * s[r][e] + kk[e] * xs;
+          dot += s[r][e] * qq[e];
+        }
       }
+      if (CHANNEL) dot += direct * x;
       dot = group_sum<16>(dot);
       if (ln == 0 && row0 + row < a.vd) out[t * a.out_stride + row] = from_f32<T>(dot + skip * x);
     }
@@ -316,13 +336,19 @@ __global__ __launch_bounds__(256) void short_conv_update_kernel(const T* __restr
 
 template <typename T, int DPT>
 static void launch_recurrence_rows(const RecurrenceArgs& a, int64_t batch, bool conv, hipStream_t s) {
-#define MOPS_REC(R, C)                                                                                                   \
-  hipLaunchKernelGGL((decayed_recurrence_kernel<T, DPT, R, C>), dim3((unsigned)(batch * a.heads * ((a.vd + 16 * (R) - 1) / (16 * (R))))), \
+#define MOPS_REC(R, C) MOPS_REC2(R, C, false)
+#define MOPS_REC2(R, C, CH)                                                                                              \
+  hipLaunchKernelGGL((decayed_recurrence_kernel<T, DPT, R, C, CH>), dim3((unsigned)(batch * a.heads * ((a.vd + 16 * (R) - 1) / (16 * (R))))), \
                      dim3(256), 0, s, a)
-  if (a.vd <= 16) { if (conv) MOPS_REC(1, true); else MOPS_REC(1, false); }
+  if (a.channel_decay) {
+    if (a.vd <= 16) MOPS_REC2(1, false, true);
+    else if (a.vd <= 32) MOPS_REC2(2, false, true);
+    else MOPS_REC2(4, false, true);
+  } else if (a.vd <= 16) { if (conv) MOPS_REC(1, true); else MOPS_REC(1, false); }
   else if (a.vd <= 32) { if (conv) MOPS_REC(2, true); else MOPS_REC(2, false); }
   else { if (conv) MOPS_REC(4, true); else MOPS_REC(4, false); }
 #undef MOPS_REC
+#undef MOPS_REC2
 }
 
 template <typename T>
@@ -350,7 +376,8 @@ extern "C" int mops_hip_decayed_recurrence(const mops_hip_recurrence* r, void* s
   if (r->q_stride < r->groups * r->d || r->k_stride < r->groups * r->d || r->v_stride < r->heads * r->vd ||
       r->out_stride < r->heads * r->vd)
     return MOPS_HIP_EINVAL;
-  if (!r->decay == !r->dt) return MOPS_HIP_EINVAL;                    // one source of the decay
+  if ((r->decay != nullptr) + (r->dt != nullptr) + (r->channel_decay != nullptr) != 1) return MOPS_HIP_EINVAL;      // one source of the decay
+  if (r->channel_decay && (!r->bonus || r->groups != r->heads || r->skip || r->conv_weight || r->channel_decay_stride < r->heads * r->d)) return MOPS_HIP_EINVAL;
   if (r->dt && (!r->dt_bias || !r->neg_a || r->dt_stride < r->heads)) return MOPS_HIP_EINVAL;
   if (r->rot < 0 || (r->rot & 1) || r->rot > r->d || (r->rot && (!r->cos_sin || r->max_positions <= 0))) return MOPS_HIP_EINVAL;
   const bool conv = r->conv_weight != nullptr;
@@ -369,6 +396,7 @@ extern "C" int mops_hip_decayed_recurrence(const mops_hip_recurrence* r, void* s
   a.heads = (int)r->heads; a.groups = (int)r->groups; a.d = (int)r->d; a.vd = (int)r->vd;
   a.pitch = (int)mops_hip_recurrence_state_pitch(r->d);
   a.decay = r->decay; a.dt = r->dt; a.dt_stride = r->dt_stride; a.dt_bias = r->dt_bias; a.neg_a = r->neg_a; a.skip = r->skip;
+  a.channel_decay = r->channel_decay; a.channel_decay_stride = r->channel_decay_stride; a.bonus = r->bonus;
   a.cos_sin = r->cos_sin; a.rot = (int)r->rot; a.max_positions = r->max_positions; a.k_scale = r->k_scale;
   a.conv_w = r->conv_weight; a.conv_b = r->conv_bias; a.ring = r->conv_ring; a.taps = (int)r->taps; a.channels = r->channels;
   a.q_channel = (int)r->q_channel; a.k_channel = (int)r->k_channel; a.v_channel = (int)r->v_channel;

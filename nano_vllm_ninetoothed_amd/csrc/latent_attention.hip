@@ -7,7 +7,7 @@
 //                          latent result out of it
 //   latent_attention_rows  one query row at a time against the cache, in the latent space: the key of a head is
 //                          [W_uk[h]^T q | q_rot] . [c | key part], the value is c.  Plain form: any size, bf16 or float.
-#include "mixed_types.h"
+#include "mfma_tiles.h"
 
 namespace mops {
 
@@ -53,16 +53,6 @@ __global__ __launch_bounds__(128) void latent_prepare_kernel(const T* __restrict
     dst[kv_rank + 2 * i + 1] = from_f32<T>(v * c + u * s);
   }
   for (int i = kv_rank + rot + lane; i < pitch; i += kWave) dst[i] = from_f32<T>(0.f);
-}
-
-// Eight consecutive bf16 of a row of `n` elements from offset i on, zeros behind the end.
-__device__ __forceinline__ u32x4 load8_guarded(const uint16_t* row, int i, int n, bool aligned) {
-  if (aligned && i + 8 <= n) return load16(row + i);
-  u32x4 w = {0u, 0u, 0u, 0u};
-#pragma unroll
-  for (int e = 0; e < 8; ++e)
-    if (i + e < n) w[e >> 1] |= (uint32_t)row[i + e] << (16 * (e & 1));
-  return w;
 }
 
 // Wave = 16 tokens x 64 outputs; the four waves of a workgroup take four token tiles against the same weights.

@@ -29,6 +29,16 @@ __device__ __forceinline__ s16x8 tile_columns(const uint16_t* tile, int pitch, i
   return join(tile_block_columns(tile, pitch, r0, c, lane), tile_block_columns(tile, pitch, r1, c, lane));
 }
 
+// Eight consecutive bf16 of a row of `n` elements from offset i on, zeros behind the end.
+__device__ __forceinline__ u32x4 load8_guarded(const uint16_t* row, int i, int n, bool aligned) {
+  if (aligned && i + 8 <= n) return load16(row + i);
+  u32x4 w = {0u, 0u, 0u, 0u};
+#pragma unroll
+  for (int e = 0; e < 8; ++e)
+    if (i + e < n) w[e >> 1] |= (uint32_t)row[i + e] << (16 * (e & 1));
+  return w;
+}
+
 // value = hi + lo in bf16: what is kept in 32 bits enters a bf16 product as two operands with 16 significant bits together.
 __device__ __forceinline__ void split8(const float (&v)[8], bf16x8& hi, bf16x8& lo) {
   u32x4 h, l;

@@ -1,0 +1,569 @@
+// Mixture of experts: every token is sent to the `top` experts with the largest router logits.
+//
+//   moe_route    logits = router h in float32, the top choices per token, their sigmoid scores, and where each choice lands when
+//                all choices are ordered by expert: row = (choices of earlier experts) + rank.  rows[] lists the choices (token *
+//                top + place) by row; tiles[] cuts each expert's rows into blocks of `block_rows`.
+//   moe_gate_up  y[row] = silu(s W_gate h) * (s W_up h) with h the token's row and s its score: the score scales the expert's input
+//   moe_down     z[choice] = W_down y[row]
+//
+// The products are grouped: a workgroup takes a block of rows of one expert and some of its outputs.  Nothing comes back to the
+// host: the grids are sized for the largest possible number of blocks, and workgroups without one leave.  The order of an
+// expert's rows depends on the order in which workgroups count them; no row's result depends on it.
+//   large blocks   128 rows x 128 weight rows x 64 deep tiles through LDS, the next tile in flight into registers
+//   small blocks   32 rows: weights are read once, straight into registers; the four waves split the depth
+//   float          plain tiles on vector units
+#include "mfma_tiles.h"
+
+namespace mops {
+
+constexpr int kMaxExperts = 1024;
+
+struct RouteArgs {
+  const void *h, *router;
+  int64_t h_stride;
+  int tokens, width, experts, top;
+  int32_t *chosen, *rank, *counts;     // [tokens * top], [tokens * top], [experts] (zeroed)
+  float* score;                        // [tokens * top]
+};
+
+// Counts this workgroup's choices per expert and ranks them among all: one addition to the global counter per expert.
+template <int THREADS>
+__device__ __forceinline__ void rank_choices(const RouteArgs& a, int* hist, int* base, int t0, int n_tokens) {
+  __syncthreads();
+  for (int e = threadIdx.x; e < a.experts; e += THREADS) hist[e] = 0;
+  __syncthreads();
+  const int64_t i0 = (int64_t)t0 * a.top;
+  const int n = n_tokens * a.top;
+  for (int i = threadIdx.x; i < n; i += THREADS) a.rank[i0 + i] = atomicAdd(&hist[a.chosen[i0 + i]], 1);
+  __syncthreads();
+  for (int e = threadIdx.x; e < a.experts; e += THREADS) base[e] = hist[e] ? atomicAdd(&a.counts[e], hist[e]) : 0;
+  __syncthreads();
+  for (int i = threadIdx.x; i < n; i += THREADS) a.rank[i0 + i] += base[a.chosen[i0 + i]];
+}
+
+// Logits of 16 tokens per wave on the matrix cores: bf16 operands, exact products, float32 sums.  ET: tiles of 16 experts.
+template <int ET>
+__global__ __launch_bounds__(256) void moe_route_mfma_kernel(const RouteArgs a, bool aligned) {
+  constexpr int kPitch = ET * 16 + 1;
+  __shared__ float logits[4][16][kPitch];
+  __shared__ int hist[ET * 16], base[ET * 16];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, n = lane & 15, jj = lane >> 4;
+  const int t0 = blockIdx.x * 64, t = t0 + wave * 16 + n;
+  const uint16_t* h = (const uint16_t*)a.h + (int64_t)(t < a.tokens ? t : a.tokens - 1) * a.h_stride;
+  f32x4 acc[ET];
+#pragma unroll
+  for (int i = 0; i < ET; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int k0 = 0; k0 < a.width; k0 += 32) {
+    const bf16x8 b = __builtin_bit_cast(bf16x8, load8_guarded(h, k0 + 8 * jj, a.width, aligned));
+#pragma unroll
+    for (int i = 0; i < ET; ++i) {
+      const int e = 16 * i + n;
+      const u32x4 w = e < a.experts ? load8_guarded((const uint16_t*)a.router + (int64_t)e * a.width, k0 + 8 * jj, a.width, aligned) : u32x4{0u, 0u, 0u, 0u};
+      acc[i] = mfma16(__builtin_bit_cast(bf16x8, w), b, acc[i]);
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < ET; ++i)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) logits[wave][n][16 * i + 4 * jj + e] = acc[i][e];
+  __syncthreads();
+  // four lanes per token: lane jj looks at the experts jj, jj + 4, ...
+  float* mine = logits[wave][n];
+  for (int s = 0; s < a.top; ++s) {
+    float best = -INFINITY;
+    int who = 0x7fffffff;
+    for (int e = jj; e < a.experts; e += 4)
+      if (mine[e] > best) {
+        best = mine[e];
+        who = e;
+      }
+#pragma unroll
+    for (int off = 16; off < 64; off <<= 1) {
+      const float ob = __shfl_xor(best, off, kWave);
+      const int ow = __shfl_xor(who, off, kWave);
+      if (ob > best || (ob == best && ow < who)) {
+        best = ob;
+        who = ow;
+      }
+    }
+    if (who >= a.experts) {      // logits that compare with nothing: any expert that is left over, and a score that shows it
+      who = s;
+      best = NAN;
+    }
+    if ((who & 3) == jj) mine[who] = -INFINITY;
+    if (jj == 0 && t < a.tokens) {
+      a.chosen[(int64_t)t * a.top + s] = who;
+      a.score[(int64_t)t * a.top + s] = 1.0f / (1.0f + expf(-best));
+    }
+  }
+  rank_choices<256>(a, hist, base, t0, a.tokens - t0 < 64 ? a.tokens - t0 : 64);
+}
+
+// One token per workgroup, any size.
+template <typename T>
+__global__ __launch_bounds__(64) void moe_route_kernel(const RouteArgs a) {
+  __shared__ float logits[kMaxExperts];
+  __shared__ int hist[kMaxExperts], base[kMaxExperts];
+  const int t = blockIdx.x, lane = threadIdx.x;
+  const T* h = (const T*)a.h + (int64_t)t * a.h_stride;
+  for (int e = 0; e < a.experts; ++e) {
+    const T* w = (const T*)a.router + (int64_t)e * a.width;
+    float dot = 0.f;
+    for (int k = lane; k < a.width; k += kWave) dot += to_f32(h[k]) * to_f32(w[k]);
+    dot = group_sum<kWave>(dot);
+    if (lane == 0) logits[e] = dot;
+  }
+  __syncthreads();
+  for (int s = 0; s < a.top; ++s) {
+    float best = -INFINITY;
+    int who = 0x7fffffff;
+    for (int e = lane; e < a.experts; e += kWave)
+      if (logits[e] > best) {
+        best = logits[e];
+        who = e;
+      }
+#pragma unroll
+    for (int off = 1; off < 64; off <<= 1) {
+      const float ob = __shfl_xor(best, off, kWave);
+      const int ow = __shfl_xor(who, off, kWave);
+      if (ob > best || (ob == best && ow < who)) {
+        best = ob;
+        who = ow;
+      }
+    }
+    if (who >= a.experts) {
+      who = s;
+      best = NAN;
+    }
+    __syncthreads();
+    if (lane == 0) {
+      logits[who] = -INFINITY;
+      a.chosen[(int64_t)t * a.top + s] = who;
+      a.score[(int64_t)t * a.top + s] = 1.0f / (1.0f + expf(-best));
+    }
+    __syncthreads();
+  }
+  rank_choices<64>(a, hist, base, t, 1);
+}
+
+// rows[] and tiles[].  tiles: [0] their number, then {expert, first row, rows} each.
+__global__ __launch_bounds__(256) void moe_place_kernel(const int32_t* __restrict__ chosen, const int32_t* __restrict__ rank,
+                                                        const int32_t* __restrict__ counts, int32_t* __restrict__ rows,
+                                                        int32_t* __restrict__ tiles, int choices, int experts, int block_rows) {
+  __shared__ int begin[kMaxExperts + 1], first_tile[kMaxExperts + 1];
+  __shared__ int wave_rows[4], wave_tiles[4];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  {
+    // a thread owns four consecutive experts
+    int c[4], r = 0, n = 0;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int e = 4 * tid + i;
+      c[i] = e < experts ? counts[e] : 0;
+      r += c[i];
+      n += (c[i] + block_rows - 1) / block_rows;
+    }
+    int ri = r, ni = n;
+#pragma unroll
+    for (int off = 1; off < 64; off <<= 1) {
+      const int ru = __shfl_up(ri, off, 64), nu = __shfl_up(ni, off, 64);
+      if (lane >= off) {
+        ri += ru;
+        ni += nu;
+      }
+    }
+    if (lane == 63) {
+      wave_rows[wave] = ri;
+      wave_tiles[wave] = ni;
+    }
+    __syncthreads();
+    r = ri - r;
+    n = ni - n;
+    for (int w = 0; w < wave; ++w) {
+      r += wave_rows[w];
+      n += wave_tiles[w];
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int e = 4 * tid + i;
+      begin[e] = r;
+      first_tile[e] = n;
+      r += c[i];
+      n += (c[i] + block_rows - 1) / block_rows;
+    }
+    if (tid == 255) {
+      begin[kMaxExperts] = r;
+      first_tile[kMaxExperts] = n;
+    }
+  }
+  __syncthreads();
+  const int i = blockIdx.x * 256 + tid;
+  if (i < choices) rows[begin[chosen[i]] + rank[i]] = i;
+  if (blockIdx.x == 0) {
+    if (tid == 0) tiles[0] = first_tile[kMaxExperts];
+    for (int e = tid; e < experts; e += 256)
+      for (int r = begin[e], k = first_tile[e]; r < begin[e + 1]; r += block_rows, ++k) {
+        tiles[1 + 3 * k] = e;
+        tiles[2 + 3 * k] = r;
+        tiles[3 + 3 * k] = begin[e + 1] - r < block_rows ? begin[e + 1] - r : block_rows;
+      }
+  }
+}
+
+struct GroupedArgs {
+  const void* x;            // gate_up: h [tokens, x_stride]; down: y [rows, x_stride]
+  int64_t x_stride;
+  const void* w;            // [experts][w_rows][depth]
+  int64_t w_expert;         // elements per expert
+  int n, up_at, depth;      // outputs, first up row behind the gate rows, depth of the product
+  void* out;
+  int64_t out_stride;
+  const int32_t *rows, *tiles;
+  const float* score;
+  int top, blocks;          // blocks of outputs in the grid
+};
+
+// ---------------------------------------------------------------------------------------------------- large blocks
+constexpr int kGM = 128, kGK = 64, kGPitch = kGK + 8, kGTile = 128 * kGPitch;
+
+template <bool GATED, bool ALIGNED>
+__global__ __launch_bounds__(256, 2) void moe_grouped_large_kernel(const GroupedArgs a) {
+  extern __shared__ __align__(16) unsigned char smem[];
+  uint16_t* const lds = reinterpret_cast<uint16_t*>(smem);      // two buffers of [x tile | w tile]
+  const int tile = blockIdx.x / a.blocks, block = blockIdx.x % a.blocks;
+  if (tile >= a.tiles[0]) return;
+  const int e = a.tiles[1 + 3 * tile], row0 = a.tiles[2 + 3 * tile], count = a.tiles[3 + 3 * tile];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 31, hh = lane >> 5;
+  const int wm = wave & 1, wn = wave >> 1;
+  constexpr int kOut = GATED ? 64 : 128;                         // outputs of the workgroup
+  const int n0 = block * kOut;
+  const uint16_t* w = (const uint16_t*)a.w + (int64_t)e * a.w_expert;
+  // pieces of 16 bytes: thread -> row tid / 8 + 32 j, depth 8 (tid % 8)
+  const int prow = tid >> 3, pk = (tid & 7) * 8;
+  const uint16_t *xp[4], *wp[4];
+  bool w_ok[4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const int r = prow + 32 * j;
+    const int src = row0 + (r < count ? r : count - 1);
+    xp[j] = (const uint16_t*)a.x + (int64_t)(GATED ? a.rows[src] / a.top : src) * a.x_stride;
+    const int n = GATED ? (r < 64 ? n0 + r : n0 + r - 64) : n0 + r;
+    w_ok[j] = n < a.n;
+    wp[j] = w + (int64_t)((w_ok[j] ? n : 0) + (GATED && r >= 64 ? a.up_at : 0)) * a.depth;
+  }
+  u32x4 xr[4], wr[4];
+  auto issue = [&](int k0) {
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int k = k0 + pk;
+      if (ALIGNED) {      // columns behind the depth are zeros on the weights' side; the other side reads something finite
+        const bool ok = k < a.depth;
+        xr[j] = load16(xp[j] + (ok ? k : 0));
+        wr[j] = load16(wp[j] + (ok ? k : 0));
+        if (!ok || !w_ok[j]) wr[j] = u32x4{0u, 0u, 0u, 0u};
+        if (!ok) xr[j] = u32x4{0u, 0u, 0u, 0u};
+      } else {
+        xr[j] = load8_guarded(xp[j], k, a.depth, false);
+        wr[j] = w_ok[j] ? load8_guarded(wp[j], k, a.depth, false) : u32x4{0u, 0u, 0u, 0u};
+      }
+    }
+  };
+  auto stash = [&](int buf) {
+    uint16_t* d = lds + buf * 2 * kGTile + prow * kGPitch + pk;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      store16(d + 32 * j * kGPitch, xr[j]);
+      store16(d + kGTile + 32 * j * kGPitch, wr[j]);
+    }
+  };
+  f32x16 acc[2][2];      // [weight rows][tokens]
+#pragma unroll
+  for (int i = 0; i < 2; ++i)
+#pragma unroll
+    for (int j = 0; j < 2; ++j)
+#pragma unroll
+      for (int r = 0; r < 16; ++r) acc[i][j][r] = 0.f;
+  issue(0);
+  stash(0);
+  __syncthreads();
+  int buf = 0;
+  for (int k0 = 0; k0 < a.depth; k0 += kGK, buf ^= 1) {
+    const bool more = k0 + kGK < a.depth;
+    if (more) issue(k0 + kGK);
+    const uint16_t *tx = lds + buf * 2 * kGTile, *tw = tx + kGTile;
+#pragma unroll
+    for (int kk = 0; kk < kGK / 16; ++kk) {
+      bf16x8 wf[2], xf[2];
+#pragma unroll
+      for (int i = 0; i < 2; ++i) wf[i] = tile_row(tw, kGPitch, (GATED ? 64 * i + 32 * wn : 64 * wn + 32 * i) + col, 16 * kk + 8 * hh);
+#pragma unroll
+      for (int j = 0; j < 2; ++j) xf[j] = tile_row(tx, kGPitch, 64 * wm + 32 * j + col, 16 * kk + 8 * hh);
+#pragma unroll
+      for (int i = 0; i < 2; ++i)
+#pragma unroll
+        for (int j = 0; j < 2; ++j) acc[i][j] = mfma32(wf[i], xf[j], acc[i][j]);
+    }
+    if (more) stash(buf ^ 1);
+    __syncthreads();
+  }
+#pragma unroll
+  for (int j = 0; j < 2; ++j) {
+    const int r = 64 * wm + 32 * j + col;
+    if (r >= count) continue;
+    const int choice = a.rows[row0 + r];
+    const float s = GATED ? a.score[choice] : 1.f;
+    uint16_t* o = (uint16_t*)a.out + (int64_t)(GATED ? row0 + r : choice) * a.out_stride;
+#pragma unroll
+    for (int i = 0; i < (GATED ? 1 : 2); ++i)
+#pragma unroll
+      for (int q4 = 0; q4 < 4; ++q4) {
+        const int n = n0 + (GATED ? 32 * wn : 64 * wn + 32 * i) + 8 * q4 + 4 * hh;
+        float v[4];
+#pragma unroll
+        for (int x = 0; x < 4; ++x) v[x] = GATED ? silu_for<bf16_t>(s * acc[0][j][4 * q4 + x]) * (s * acc[1][j][4 * q4 + x]) : acc[i][j][4 * q4 + x];
+        if (ALIGNED && n + 4 <= a.n) {
+          *reinterpret_cast<u32x2*>(o + n) = u32x2{pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3])};
+        } else {
+#pragma unroll
+          for (int x = 0; x < 4; ++x)
+            if (n + x < a.n) o[n + x] = (uint16_t)f32_to_bf16_bits(v[x]);
+        }
+      }
+  }
+}
+
+// ---------------------------------------------------------------------------------------------------- small blocks
+constexpr int kSM = 32;
+
+// GATED: 32 outputs, tile 0 gate rows and tile 1 up rows; else 64 outputs.
+template <bool GATED, bool ALIGNED>
+__global__ __launch_bounds__(256, 2) void moe_grouped_small_kernel(const GroupedArgs a) {
+  __shared__ __align__(16) float part[4][2][16][64];      // [wave][tile][accumulator][lane]
+  const int tile = blockIdx.x / a.blocks, block = blockIdx.x % a.blocks;
+  if (tile >= a.tiles[0]) return;
+  const int e = a.tiles[1 + 3 * tile], row0 = a.tiles[2 + 3 * tile], count = a.tiles[3 + 3 * tile];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 31, hh = lane >> 5;
+  const int n0 = block * (GATED ? 32 : 64);
+  const int src = row0 + (col < count ? col : count - 1);
+  const uint16_t* x = (const uint16_t*)a.x + (int64_t)(GATED ? a.rows[src] / a.top : src) * a.x_stride;
+  const uint16_t* w[2];
+  bool w_ok[2];
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const int n = GATED ? n0 + col : n0 + 32 * i + col;
+    w_ok[i] = n < a.n;
+    w[i] = (const uint16_t*)a.w + (int64_t)e * a.w_expert + (int64_t)((w_ok[i] ? n : 0) + (GATED && i ? a.up_at : 0)) * a.depth;
+  }
+  f32x16 acc[2];
+#pragma unroll
+  for (int i = 0; i < 2; ++i)
+#pragma unroll
+    for (int r = 0; r < 16; ++r) acc[i][r] = 0.f;
+  for (int k0 = 64 * wave; k0 < a.depth; k0 += 256) {
+    u32x4 xr[4], wr[2][4];
+#pragma unroll
+    for (int kk = 0; kk < 4; ++kk) {
+      const int k = k0 + 16 * kk + 8 * hh;
+      if (ALIGNED) {
+        const bool ok = k < a.depth;
+        xr[kk] = load16(x + (ok ? k : 0));
+        if (!ok) xr[kk] = u32x4{0u, 0u, 0u, 0u};
+#pragma unroll
+        for (int i = 0; i < 2; ++i) {
+          wr[i][kk] = load16_stream(w[i] + (ok ? k : 0));
+          if (!ok) wr[i][kk] = u32x4{0u, 0u, 0u, 0u};
+        }
+      } else {
+        xr[kk] = load8_guarded(x, k, a.depth, false);
+#pragma unroll
+        for (int i = 0; i < 2; ++i) wr[i][kk] = load8_guarded(w[i], k, a.depth, false);
+      }
+    }
+#pragma unroll
+    for (int kk = 0; kk < 4; ++kk)
+#pragma unroll
+      for (int i = 0; i < 2; ++i) acc[i] = mfma32(__builtin_bit_cast(bf16x8, wr[i][kk]), __builtin_bit_cast(bf16x8, xr[kk]), acc[i]);
+  }
+#pragma unroll
+  for (int i = 0; i < 2; ++i)
+#pragma unroll
+    for (int r = 0; r < 16; ++r) part[wave][i][r][lane] = acc[i][r];
+  __syncthreads();
+  // wave q4 finishes accumulators 4 q4 .. 4 q4 + 3 of both tiles
+  float v[2][4];
+#pragma unroll
+  for (int i = 0; i < 2; ++i)
+#pragma unroll
+    for (int x4 = 0; x4 < 4; ++x4) {
+      const int r = 4 * wave + x4;
+      v[i][x4] = (part[0][i][r][lane] + part[1][i][r][lane]) + (part[2][i][r][lane] + part[3][i][r][lane]);
+    }
+  if (col >= count) return;
+  const int choice = a.rows[row0 + col];
+  uint16_t* o = (uint16_t*)a.out + (int64_t)(GATED ? row0 + col : choice) * a.out_stride;
+  const float s = GATED ? a.score[choice] : 1.f;
+#pragma unroll
+  for (int i = 0; i < (GATED ? 1 : 2); ++i) {
+    const int n = n0 + 32 * i + 8 * wave + 4 * hh;
+    float y[4];
+#pragma unroll
+    for (int x4 = 0; x4 < 4; ++x4) y[x4] = GATED ? silu_for<bf16_t>(s * v[0][x4]) * (s * v[1][x4]) : v[i][x4];
+    if (ALIGNED && n + 4 <= a.n) {
+      *reinterpret_cast<u32x2*>(o + n) = u32x2{pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3])};
+    } else {
+#pragma unroll
+      for (int x4 = 0; x4 < 4; ++x4)
+        if (n + x4 < a.n) o[n + x4] = (uint16_t)f32_to_bf16_bits(y[x4]);
+    }
+  }
+}
+
+// ---------------------------------------------------------------------------------------------------- float
+// 32 rows x 64 outputs per workgroup; a thread takes one output of eight rows.
+template <bool GATED>
+__global__ __launch_bounds__(256) void moe_grouped_f32_kernel(const GroupedArgs a) {
+  __shared__ float tx[kSM][33], tw[GATED ? 2 : 1][64][33];
+  const int tile = blockIdx.x / a.blocks, block = blockIdx.x % a.blocks;
+  if (tile >= a.tiles[0]) return;
+  const int e = a.tiles[1 + 3 * tile], row0 = a.tiles[2 + 3 * tile], count = a.tiles[3 + 3 * tile];
+  const int tid = threadIdx.x, n_loc = tid & 63, r0 = tid >> 6;
+  const int n0 = block * 64;
+  const float* w = (const float*)a.w + (int64_t)e * a.w_expert;
+  float acc[GATED ? 2 : 1][8];
+#pragma unroll
+  for (int i = 0; i < (GATED ? 2 : 1); ++i)
+#pragma unroll
+    for (int r = 0; r < 8; ++r) acc[i][r] = 0.f;
+  for (int k0 = 0; k0 < a.depth; k0 += 32) {
+    for (int i = tid; i < kSM * 32; i += 256) {
+      const int r = i / 32, k = k0 + i % 32;
+      const int src = row0 + (r < count ? r : count - 1);
+      tx[r][i % 32] = k < a.depth ? ((const float*)a.x)[(int64_t)(GATED ? a.rows[src] / a.top : src) * a.x_stride + k] : 0.f;
+    }
+    for (int i = tid; i < (GATED ? 2 : 1) * 64 * 32; i += 256) {
+      const int half = i / (64 * 32), r = i / 32 % 64, k = k0 + i % 32;
+      tw[half][r][i % 32] = k < a.depth && n0 + r < a.n ? w[(int64_t)(n0 + r + (half ? a.up_at : 0)) * a.depth + k] : 0.f;
+    }
+    __syncthreads();
+    for (int k = 0; k < 32; ++k)
+#pragma unroll
+      for (int i = 0; i < (GATED ? 2 : 1); ++i)
+#pragma unroll
+        for (int r = 0; r < 8; ++r) acc[i][r] += tw[i][n_loc][k] * tx[r0 + 4 * r][k];
+    __syncthreads();
+  }
+  const int n = n0 + n_loc;
+  if (n >= a.n) return;
+#pragma unroll
+  for (int r = 0; r < 8; ++r) {
+    const int row = r0 + 4 * r;
+    if (row >= count) continue;
+    const int choice = a.rows[row0 + row];
+    const float s = GATED ? a.score[choice] : 1.f;
+    ((float*)a.out)[(int64_t)(GATED ? row0 + row : choice) * a.out_stride + n] =
+        GATED ? silu_for<float>(s * acc[0][r]) * (s * acc[GATED ? 1 : 0][r]) : acc[0][r];
+  }
+}
+
+template <bool GATED>
+static int launch_grouped(GroupedArgs a, int dtype, int64_t block_rows, int64_t choices, int64_t experts, hipStream_t s) {
+  const int64_t tiles = choices / block_rows + (experts < choices ? experts : choices);
+  const int per = dtype == MOPS_HIP_F32 ? 64 : (block_rows == kSM ? (GATED ? 32 : 64) : (GATED ? 64 : 128));
+  a.blocks = (a.n + per - 1) / per;
+  if (tiles * a.blocks > 0x7fffffffLL) return MOPS_HIP_EUNSUPPORTED;
+  const dim3 grid((unsigned)(tiles * a.blocks)), block(256);
+  const bool aligned = a.depth % 8 == 0 && a.x_stride % 8 == 0 && a.out_stride % 4 == 0 && a.w_expert % 8 == 0 && aligned16(a.x) && aligned16(a.w) &&
+                       aligned16(a.out);
+  if (dtype == MOPS_HIP_F32) {
+    hipLaunchKernelGGL((moe_grouped_f32_kernel<GATED>), grid, block, 0, s, a);
+  } else if (block_rows == kSM) {
+    if (aligned) hipLaunchKernelGGL((moe_grouped_small_kernel<GATED, true>), grid, block, 0, s, a);
+    else hipLaunchKernelGGL((moe_grouped_small_kernel<GATED, false>), grid, block, 0, s, a);
+  } else {
+    constexpr int kLds = 4 * kGTile * 2;
+    static const hipError_t lds0 = hipFuncSetAttribute(reinterpret_cast<const void*>(&moe_grouped_large_kernel<GATED, true>),
+                                                       hipFuncAttributeMaxDynamicSharedMemorySize, kLds);
+    static const hipError_t lds1 = hipFuncSetAttribute(reinterpret_cast<const void*>(&moe_grouped_large_kernel<GATED, false>),
+                                                       hipFuncAttributeMaxDynamicSharedMemorySize, kLds);
+    if (lds0 != hipSuccess) return record_hip_error(lds0);
+    if (lds1 != hipSuccess) return record_hip_error(lds1);
+    if (aligned) hipLaunchKernelGGL((moe_grouped_large_kernel<GATED, true>), grid, block, kLds, s, a);
+    else hipLaunchKernelGGL((moe_grouped_large_kernel<GATED, false>), grid, block, kLds, s, a);
+  }
+  return finish_launch();
+}
+
+static int check_grouped(const mops_hip_moe* m) {
+  if (!m || !known_dtype(m->dtype) || m->tokens < 0) return MOPS_HIP_EINVAL;
+  if (m->tokens == 0) return MOPS_HIP_OK;
+  if (m->experts <= 0 || m->top <= 0 || m->top > m->experts || m->width <= 0 || m->ff <= 0) return MOPS_HIP_EINVAL;
+  if (m->block_rows != kSM && (m->block_rows != kGM || m->dtype != MOPS_HIP_BF16)) return MOPS_HIP_EINVAL;
+  if (m->experts > kMaxExperts || m->tokens * m->top > (1 << 28) || m->width > (1 << 20) || m->ff > (1 << 20)) return MOPS_HIP_EUNSUPPORTED;
+  if (!m->rows || !m->tiles || !m->score) return MOPS_HIP_EINVAL;
+  return 1;
+}
+
+}  // namespace mops
+
+extern "C" int64_t mops_hip_moe_max_tiles(int64_t tokens, int64_t experts, int64_t top, int64_t block_rows) {
+  if (tokens < 0 || experts <= 0 || top <= 0 || block_rows <= 0) return MOPS_HIP_EINVAL;
+  const int64_t choices = tokens * top;
+  return choices / block_rows + (experts < choices ? experts : choices);
+}
+
+extern "C" int mops_hip_moe_route(const void* h, int64_t h_row_stride, const void* router, int32_t* chosen, int32_t* rank, int32_t* counts,
+                                  const mops_hip_moe* m, void* stream) {
+  using namespace mops;
+  const int pre = check_grouped(m);
+  if (pre != 1) return pre;
+  if (!h || !router || !chosen || !rank || !counts || h_row_stride < m->width) return MOPS_HIP_EINVAL;
+  RouteArgs a;
+  a.h = h; a.router = router; a.h_stride = h_row_stride;
+  a.tokens = (int)m->tokens; a.width = (int)m->width; a.experts = (int)m->experts; a.top = (int)m->top;
+  a.chosen = chosen; a.rank = rank; a.counts = counts; a.score = m->score;
+  hipStream_t s = (hipStream_t)stream;
+  if (m->dtype == MOPS_HIP_BF16 && m->experts <= 128) {
+    const dim3 grid((unsigned)((m->tokens + 63) / 64)), block(256);
+    const bool aligned = m->width % 8 == 0 && h_row_stride % 8 == 0 && aligned16(h) && aligned16(router);
+    if (m->experts <= 16) hipLaunchKernelGGL((moe_route_mfma_kernel<1>), grid, block, 0, s, a, aligned);
+    else if (m->experts <= 32) hipLaunchKernelGGL((moe_route_mfma_kernel<2>), grid, block, 0, s, a, aligned);
+    else if (m->experts <= 64) hipLaunchKernelGGL((moe_route_mfma_kernel<4>), grid, block, 0, s, a, aligned);
+    else hipLaunchKernelGGL((moe_route_mfma_kernel<8>), grid, block, 0, s, a, aligned);
+  } else if (m->dtype == MOPS_HIP_BF16) {
+    hipLaunchKernelGGL((moe_route_kernel<bf16_t>), dim3((unsigned)m->tokens), dim3(64), 0, s, a);
+  } else {
+    hipLaunchKernelGGL((moe_route_kernel<float>), dim3((unsigned)m->tokens), dim3(64), 0, s, a);
+  }
+  int st = finish_launch();
+  if (st != MOPS_HIP_OK) return st;
+  const int choices = (int)(m->tokens * m->top);
+  hipLaunchKernelGGL(moe_place_kernel, dim3((unsigned)((choices + 255) / 256)), dim3(256), 0, s, chosen, rank, counts, m->rows, m->tiles, choices,
+                     (int)m->experts, (int)m->block_rows);
+  return finish_launch();
+}
+
+extern "C" int mops_hip_moe_gate_up(const void* h, int64_t h_row_stride, const void* w, int64_t up_at, void* y, int64_t y_row_stride,
+                                    const mops_hip_moe* m, void* stream) {
+  using namespace mops;
+  const int pre = check_grouped(m);
+  if (pre != 1) return pre;
+  if (!h || !w || !y || h_row_stride < m->width || y_row_stride < m->ff || up_at < m->ff || up_at > (1 << 20)) return MOPS_HIP_EINVAL;
+  GroupedArgs a;
+  a.x = h; a.x_stride = h_row_stride; a.w = w; a.w_expert = 2 * up_at * m->width;
+  a.n = (int)m->ff; a.up_at = (int)up_at; a.depth = (int)m->width; a.out = y; a.out_stride = y_row_stride;
+  a.rows = m->rows; a.tiles = m->tiles; a.score = m->score; a.top = (int)m->top; a.blocks = 0;
+  return launch_grouped<true>(a, m->dtype, m->block_rows, m->tokens * m->top, m->experts, (hipStream_t)stream);
+}
+
+extern "C" int mops_hip_moe_down(const void* y, int64_t y_row_stride, const void* w, int64_t depth, void* z, int64_t z_row_stride,
+                                 const mops_hip_moe* m, void* stream) {
+  using namespace mops;
+  const int pre = check_grouped(m);
+  if (pre != 1) return pre;
+  if (!y || !w || !z || depth < m->ff || depth > (1 << 20) || y_row_stride < depth || z_row_stride < m->width) return MOPS_HIP_EINVAL;
+  GroupedArgs a;
+  a.x = y; a.x_stride = y_row_stride; a.w = w; a.w_expert = depth * m->width;
+  a.n = (int)m->width; a.up_at = 0; a.depth = (int)depth; a.out = z; a.out_stride = z_row_stride;
+  a.rows = m->rows; a.tiles = m->tiles; a.score = m->score; a.top = (int)m->top; a.blocks = 0;
+  return launch_grouped<false>(a, m->dtype, m->block_rows, m->tokens * m->top, m->experts, (hipStream_t)stream);
+}

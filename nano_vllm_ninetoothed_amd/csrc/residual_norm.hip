@@ -1,9 +1,10 @@
 // A float32 residual stream and the norms around it, for models whose residual sum and norms are kept in 32 bits.
 //
-//   embed_residual     x = table[id], as float32 (the residual) and in the activation type (the first projection's input)
+//   embed_residual     x = scale * table[id], as float32 (the residual) and in the activation type (the first projection's input)
 //   norm_residual_add  x += rms(y) * (offset + w): the norm sits on the sublayer's output, the sum runs on in float32 and
 //                      leaves a copy in the activation type for the next projection
 //   rms_norm_f32       out = rms(x) * (offset + w) of the float32 stream
+//   add_norm_norm      x += rms(y) * w_out, out = rms(x) * w_in: norms behind one sublayer and in front of the next, in one pass
 //   gated_group_norm   rms over equal parts of a row, with silu(gate) multiplied in before or after the division
 //
 // A row belongs to one workgroup of 64 or 256 threads; the elements a thread owns stay in its registers between the
@@ -16,7 +17,7 @@ constexpr int kKeep = 4;
 
 template <typename T, int VEC>
 __global__ __launch_bounds__(256) void embed_residual_kernel(const int64_t* __restrict__ ids, const T* __restrict__ table,
-                                                             int64_t table_stride, float* __restrict__ x, T* __restrict__ act,
+                                                             int64_t table_stride, float scale, float* __restrict__ x, T* __restrict__ act,
                                                              int64_t vocab, int width) {
   const int64_t row = blockIdx.x;
   const int64_t id = ids[row];
@@ -26,8 +27,10 @@ __global__ __launch_bounds__(256) void embed_residual_kernel(const int64_t* __re
 #pragma unroll
     for (int e = 0; e < VEC; ++e) v[e] = 0.f;
     if (ok) load_vec<VEC>(table + id * table_stride + c, v);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) v[e] *= scale;
     store_vec<VEC>(x + row * width + c, v);
-    store_vec<VEC>(act + row * width + c, v);
+    if (act) store_vec<VEC>(act + row * width + c, v);
   }
 }
 
@@ -83,6 +86,84 @@ __global__ __launch_bounds__(THREADS) void norm_kernel(float* __restrict__ resid
     float v[VEC];
     if (MODE == 0) load_vec<VEC>(xr + c, v);
     else load_vec<VEC>(yr + c, v);
+    finish(c, v);
+  }
+}
+
+// residual += norm(sum of the row's `parts` rows of y) * w_out; out = norm(residual) * w_in.
+template <typename T, int VEC, int THREADS>
+__global__ __launch_bounds__(THREADS) void add_norm_norm_kernel(float* __restrict__ residual, const T* __restrict__ y, int64_t y_stride,
+                                                                int parts, const T* __restrict__ w_out, const T* __restrict__ w_in,
+                                                                float eps, T* __restrict__ out, int n) {
+  __shared__ float scratch[THREADS / kWave];
+  const int64_t row = blockIdx.x;
+  float* xr = residual + row * n;
+  const T* yr = y + row * parts * y_stride;
+  auto read = [&](int c, float (&v)[VEC]) {
+    load_vec<VEC>(yr + c, v);
+    for (int p = 1; p < parts; ++p) {
+      float u[VEC];
+      load_vec<VEC>(yr + p * y_stride + c, u);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) v[e] += u[e];
+    }
+  };
+  float keep[kKeep][VEC];
+  float ss = 0.f;
+#pragma unroll
+  for (int it = 0; it < kKeep; ++it) {
+    const int c = (it * THREADS + threadIdx.x) * VEC;
+    if (c < n) {
+      read(c, keep[it]);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) ss += keep[it][e] * keep[it][e];
+    }
+  }
+  for (int c = (kKeep * THREADS + threadIdx.x) * VEC; c < n; c += THREADS * VEC) {
+    float v[VEC];
+    read(c, v);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) ss += v[e] * v[e];
+  }
+  const float rstd_out = 1.0f / sqrtf(block_sum<THREADS>(ss, scratch) / (float)n + eps);
+  ss = 0.f;
+  auto add = [&](int c, float (&v)[VEC]) {      // v: the sublayer's output, then the new residual
+    float wv[VEC], x[VEC];
+    load_vec<VEC>(w_out + c, wv);
+    load_vec<VEC>(xr + c, x);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) {
+      v[e] = x[e] + v[e] * rstd_out * wv[e];
+      ss += v[e] * v[e];
+    }
+    store_vec<VEC>(xr + c, v);
+  };
+#pragma unroll
+  for (int it = 0; it < kKeep; ++it) {
+    const int c = (it * THREADS + threadIdx.x) * VEC;
+    if (c < n) add(c, keep[it]);
+  }
+  for (int c = (kKeep * THREADS + threadIdx.x) * VEC; c < n; c += THREADS * VEC) {
+    float v[VEC];
+    read(c, v);
+    add(c, v);
+  }
+  const float rstd_in = 1.0f / sqrtf(block_sum<THREADS>(ss, scratch) / (float)n + eps);
+  auto finish = [&](int c, const float (&v)[VEC]) {
+    float wv[VEC], o[VEC];
+    load_vec<VEC>(w_in + c, wv);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) o[e] = v[e] * rstd_in * wv[e];
+    store_vec<VEC>(out + row * n + c, o);
+  };
+#pragma unroll
+  for (int it = 0; it < kKeep; ++it) {
+    const int c = (it * THREADS + threadIdx.x) * VEC;
+    if (c < n) finish(c, keep[it]);
+  }
+  for (int c = (kKeep * THREADS + threadIdx.x) * VEC; c < n; c += THREADS * VEC) {
+    float v[VEC];
+    load_vec<VEC>(xr + c, v);      // this thread's own stores
     finish(c, v);
   }
 }
@@ -167,17 +248,17 @@ static void launch_norm(float* residual, const void* y, int64_t y_stride, const 
 
 }  // namespace mops
 
-extern "C" int mops_hip_embed_residual(const int64_t* ids, const void* table, int64_t table_row_stride, int dtype, float* residual,
-                                       void* act, int64_t n_ids, int64_t vocab, int64_t width, void* stream) {
+extern "C" int mops_hip_embed_residual(const int64_t* ids, const void* table, int64_t table_row_stride, int dtype, float scale,
+                                       float* residual, void* act, int64_t n_ids, int64_t vocab, int64_t width, void* stream) {
   using namespace mops;
   if (!known_dtype(dtype) || n_ids < 0 || vocab <= 0 || width <= 0 || width > (1 << 20) || n_ids > 0x7fffffffLL) return MOPS_HIP_EINVAL;
   if (n_ids == 0) return MOPS_HIP_OK;
-  if (!ids || !table || !residual || !act || table_row_stride < width) return MOPS_HIP_EINVAL;
-  const bool vec = width % 8 == 0 && table_row_stride % 8 == 0 && aligned16(table) && aligned16(residual) && aligned16(act);
+  if (!ids || !table || !residual || table_row_stride < width) return MOPS_HIP_EINVAL;
+  const bool vec = width % 8 == 0 && table_row_stride % 8 == 0 && aligned16(table) && aligned16(residual) && (!act || aligned16(act));
   const dim3 grid((unsigned)n_ids), block(256);
   hipStream_t s = (hipStream_t)stream;
 #define MOPS_EMBED(T, V) hipLaunchKernelGGL((embed_residual_kernel<T, V>), grid, block, 0, s, ids, (const T*)table, table_row_stride, \
-                                            residual, (T*)act, vocab, (int)width)
+                                            scale, residual, (T*)act, vocab, (int)width)
   if (dtype == MOPS_HIP_BF16) { if (vec) MOPS_EMBED(bf16_t, 8); else MOPS_EMBED(bf16_t, 1); }
   else { if (vec) MOPS_EMBED(float, 8); else MOPS_EMBED(float, 1); }
 #undef MOPS_EMBED
@@ -204,6 +285,30 @@ extern "C" int mops_hip_rms_norm_f32(const float* x, const void* weight, float w
   float* xr = const_cast<float*>(x);   // mode 0 only reads it
   if (dtype == MOPS_HIP_BF16) launch_norm<bf16_t, 0>(xr, nullptr, 0, weight, weight_offset, eps, out, rows, n, (hipStream_t)stream);
   else launch_norm<float, 0>(xr, nullptr, 0, weight, weight_offset, eps, out, rows, n, (hipStream_t)stream);
+  return finish_launch();
+}
+
+extern "C" int mops_hip_add_norm_norm(float* residual, const void* y, int64_t y_row_stride, int64_t parts, const void* w_out, const void* w_in,
+                                      float eps, void* out, int dtype, int64_t rows, int64_t n, void* stream) {
+  using namespace mops;
+  if (!known_dtype(dtype) || rows < 0 || n <= 0 || n > (1 << 20) || rows > 0x7fffffffLL || parts <= 0 || parts > (1 << 20)) return MOPS_HIP_EINVAL;
+  if (rows == 0) return MOPS_HIP_OK;
+  if (!residual || !y || !w_out || !w_in || !out || y_row_stride < n || y == out) return MOPS_HIP_EINVAL;
+  const bool vec = n % 8 == 0 && y_row_stride % 8 == 0 && aligned16(residual) && aligned16(y) && aligned16(w_out) && aligned16(w_in) && aligned16(out);
+  const dim3 grid((unsigned)rows);
+  hipStream_t s = (hipStream_t)stream;
+#define MOPS_ANN(T, V, TH) hipLaunchKernelGGL((add_norm_norm_kernel<T, V, TH>), grid, dim3(TH), 0, s, residual, (const T*)y, y_row_stride, \
+                                              (int)parts, (const T*)w_out, (const T*)w_in, eps, (T*)out, (int)n)
+#define MOPS_ANN_TYPE(T) do {                          \
+    if (vec && n <= 1024) MOPS_ANN(T, 8, 64);          \
+    else if (vec) MOPS_ANN(T, 8, 256);                 \
+    else if (n <= 512) MOPS_ANN(T, 1, 64);             \
+    else MOPS_ANN(T, 1, 256);                          \
+  } while (0)
+  if (dtype == MOPS_HIP_BF16) MOPS_ANN_TYPE(bf16_t);
+  else MOPS_ANN_TYPE(float);
+#undef MOPS_ANN_TYPE
+#undef MOPS_ANN
   return finish_launch();
 }
 

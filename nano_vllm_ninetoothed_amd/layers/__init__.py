@@ -3,10 +3,14 @@
 A mixer is built as cls(sizes, weights, prefix, ModelContext) and called as mixer(x, ctx) with x [tokens, width] in the
 activation dtype and the batch description ctx of the engine; it returns [tokens, width] and updates its cache or state.
 The first ctx["n_decode"] sequences of a batch bring one token each, the others portions of any length.
-A feed-forward is built the same way and called as ff(x).
+A mixer takes its cache or state in allocate(cache); again(cache) gives another mixer on the same weights with a cache or state of
+its own, for layers that run several times in a forward pass.
+A feed-forward is built the same way and called as ff(x).  Its result may have several rows per token, one behind the other,
+that count as their sum.
 """
 from __future__ import annotations
 
+import copy
 from dataclasses import dataclass
 
 import torch
@@ -43,6 +47,16 @@ class ModelContext:
     rotary: object
 
 
+class Mixer:
+    def allocate(self, cache) -> None:
+        raise NotImplementedError
+
+    def again(self, cache) -> "Mixer":
+        other = copy.copy(self)
+        other.allocate(cache)
+        return other
+
+
 def require_size(sizes: dict, *names):
     for n in names:
         v = sizes.get(n)
@@ -61,7 +75,7 @@ def pack(tensors, multiple: int = 8) -> torch.Tensor:
 
 
 class Rotary:
-    """cos/sin tables [max_positions, dims] (cosines, then sines; float32, angles taken in float64), one per (base, dims)."""
+    """Tables over positions: cos/sin tables [max_positions, dims] (cosines, then sines; float32, angles taken in float64), one per (base, dims)."""
 
     def __init__(self, max_positions: int, device):
         self.max_positions, self.device = max_positions, device
@@ -73,6 +87,14 @@ class Rotary:
             i = torch.arange(dims // 2, dtype=torch.float64)
             a = torch.outer(torch.arange(self.max_positions, dtype=torch.float64), float(base) ** (-2.0 * i / dims))
             self._tables[key] = torch.cat((a.cos(), a.sin()), dim=-1).float().to(self.device).contiguous()
+        return self._tables[key]
+
+    def steps(self, coef: float, every: float) -> torch.Tensor:
+        """1 + coef ln(floor((p + 1) / every) + 1) for every position p (float32, taken in float64)."""
+        key = ("steps", float(coef), float(every))
+        if key not in self._tables:
+            p = torch.arange(1, self.max_positions + 1, dtype=torch.float64)
+            self._tables[key] = (1 + float(coef) * torch.log(torch.floor(p / float(every)) + 1)).float().to(self.device).contiguous()
         return self._tables[key]
 
 
@@ -101,8 +123,20 @@ class ChunkedRecurrence:
         return self.chunks(q, k, v, out, state, slots, starts, *self.sizes, *cuts[key], cu_seqlens=cu, **options)
 
 
+class ChannelRecurrence:
+    """The same for a recurrence with a decay per key channel and a bonus for the current token."""
+
+    def __init__(self, heads, d, dtype):
+        self.sizes = (heads, heads, d, d)
+        self.recurrence = hip_op("decayed_recurrence")
+
+    def __call__(self, r, k, v, out, state, ctx, **options):
+        nd = ctx["n_decode"]
+        return self.recurrence(r, k, v, out, state, ctx["state_slots"][nd:], ctx["starts"][nd:], *self.sizes, cu_seqlens=ctx["portion_cu"], **options)
+
+
 def hip_op(name):
     return mops.get_op(name, "hip")
 
 
-from . import feed_forward, latent_attention, mamba2, retention  # noqa: E402,F401  (register themselves)
+from . import biased_attention, feed_forward, latent_attention, mamba2, mixture, retention, time_mixing  # noqa: E402,F401  (register themselves)

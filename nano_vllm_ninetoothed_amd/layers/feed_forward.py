@@ -4,7 +4,7 @@ from __future__ import annotations
 from . import hip_op, pack, register_feed_forward, require_size
 
 
-@register_feed_forward("dense")
+@register_feed_forward("clamped_glu")
 class ClampedGLU:
     """W_down(g * sigmoid(1.702 g) * (u + 1)) with g = min(W_gate x, limit) and u = clamp(W_up x, -limit, limit)."""
     ALPHA = 1.702
@@ -27,3 +27,21 @@ class ClampedGLU:
         p = self.linear(x, self.gate_up)
         y = self.glu(p[:, :self.ff], p[:, self.half:self.half + self.ff], self.limit, self.ALPHA)
         return self.linear(y, self.down)
+
+
+@register_feed_forward("squared_relu")
+class SquaredReLU:
+    """W_down max(W_up x, 0)^2."""
+
+    @staticmethod
+    def validate(sizes):
+        require_size(sizes, "ff")
+
+    def __init__(self, sizes, weights, prefix, m):
+        self.ff = sizes["ff"]
+        self.up = pack([weights.take(prefix + "up", (self.ff, m.width))])
+        self.down = weights.take(prefix + "down", (m.width, self.ff))
+        self.linear, self.act = hip_op("linear"), hip_op("squared_relu")
+
+    def __call__(self, x):
+        return self.linear(self.act(self.linear(x, self.up)[:, :self.ff]), self.down)

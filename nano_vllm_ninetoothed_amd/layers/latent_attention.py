@@ -4,7 +4,7 @@ from __future__ import annotations
 
 import torch
 
-from . import hip_op, pack, register_mixer, require_size
+from . import Mixer, hip_op, pack, register_mixer, require_size
 from ..mops.hip.recurrent_ops import latent_decode_covers, latent_prefill_covers, latent_prefill_plan
 
 EXPAND_FROM = 64     # portions of at least this many tokens expand keys and values instead of absorbing the projections
@@ -16,7 +16,7 @@ def pad_rows(w, rows):
 
 
 @register_mixer("latent_attention")
-class LatentAttention:
+class LatentAttention(Mixer):
     uses_pages, uses_slots = True, False
 
     @staticmethod
@@ -41,7 +41,8 @@ class LatentAttention:
         self.q_to_latent = uk.view(h, d, kr).transpose(1, 2).contiguous()     # [H, kv_rank, dim]
         self.latent_to_v = uv.view(h, v, kr)                                  # [H, vdim, kv_rank]
         self.o = take(prefix + "o", (m.width, h * v))
-        self.pages = m.cache.paged((kr + r + 7) // 8 * 8, dtype=m.dtype)
+        self.dtype = m.dtype
+        self.allocate(m.cache)
         self.cos_sin = m.rotary.table(sizes["rot"]["base"], r)
         self.linear, self.prepare, self.head_linear = hip_op("linear"), hip_op("latent_prepare"), hip_op("head_linear")
         self.rows = hip_op("latent_decode" if latent_decode_covers(m.dtype, kr, r, m.cache.block_size) else "latent_attention_rows")
@@ -52,6 +53,9 @@ class LatentAttention:
             self.w_k = torch.nn.functional.pad(pad_rows(uk.view(h, d, kr), dp), (0, pad)).reshape(h * dp, kr + pad).contiguous()
             self.w_v = torch.nn.functional.pad(uv, (0, pad)).contiguous()
             self.gather, self.rotate, self.prefill = hip_op("latent_gather"), hip_op("rotate_pairs"), hip_op("latent_prefill")
+
+    def allocate(self, cache):
+        self.pages = cache.paged((self.kv_rank + self.rot_dim + 7) // 8 * 8, dtype=self.dtype)
 
     def __call__(self, x, ctx):
         h, d, r, v = self.heads, self.dim, self.rot_dim, self.vdim

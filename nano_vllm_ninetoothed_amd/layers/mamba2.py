@@ -3,12 +3,12 @@ from __future__ import annotations
 
 import torch
 
-from . import ChunkedRecurrence, hip_op, pack, register_mixer, require_size
+from . import ChunkedRecurrence, Mixer, hip_op, pack, register_mixer, require_size
 from ..mops.hip.recurrent_ops import recurrence_state_pitch
 
 
 @register_mixer("mamba2")
-class Mamba2:
+class Mamba2(Mixer):
     uses_pages, uses_slots = False, True
 
     @staticmethod
@@ -34,11 +34,15 @@ class Mamba2:
         self.skip = take(prefix + "D", (h,), "norm").float().contiguous()
         self.norm = take(prefix + "norm", (inner,), "norm")
         self.o = take(prefix + "o", (m.width, inner))
-        self.state = m.cache.per_slot(h, v, recurrence_state_pitch(n))
-        self.ring = m.cache.per_slot(self.taps, ch, dtype=m.dtype)
+        self.dtype = m.dtype
+        self.allocate(m.cache)
         self.portions = ChunkedRecurrence(h, g, n, v, m.dtype)
         self.linear, self.recurrence, self.group_norm = hip_op("linear"), hip_op("decayed_recurrence"), hip_op("gated_group_norm")
         self.conv, self.conv_update = hip_op("short_conv"), hip_op("short_conv_update")
+
+    def allocate(self, cache):
+        self.state = cache.per_slot(self.heads, self.vdim, recurrence_state_pitch(self.n))
+        self.ring = cache.per_slot(self.taps, self.channels, dtype=self.dtype)
 
     def __call__(self, x, ctx):
         h, v, n, g, inner, ch = self.heads, self.vdim, self.n, self.groups, self.inner, self.channels

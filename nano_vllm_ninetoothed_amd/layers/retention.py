@@ -5,12 +5,12 @@ import math
 
 import torch
 
-from . import ChunkedRecurrence, hip_op, pack, register_mixer, require_size
+from . import ChunkedRecurrence, Mixer, hip_op, pack, register_mixer, require_size
 from ..mops.hip.recurrent_ops import recurrence_state_pitch
 
 
 @register_mixer("retention")
-class Retention:
+class Retention(Mixer):
     uses_pages, uses_slots = False, True
 
     @staticmethod
@@ -37,9 +37,12 @@ class Retention:
         self.log_decay = decay.clamp(min=math.exp(-80.0)).log().float().to(m.device)
         self.cos_sin = m.rotary.table(sizes["rot"]["base"], sizes["rot"]["dims"]) if sizes["rot"]["dims"] else None
         self.k_scale = d ** -0.5
-        self.state = m.cache.per_slot(h, v, recurrence_state_pitch(d))
+        self.allocate(m.cache)
         self.portions = ChunkedRecurrence(h, h, d, v, m.dtype)
         self.linear, self.recurrence, self.group_norm = hip_op("linear"), hip_op("decayed_recurrence"), hip_op("gated_group_norm")
+
+    def allocate(self, cache):
+        self.state = cache.per_slot(self.heads, self.vdim, recurrence_state_pitch(self.dim))
 
     def __call__(self, x, ctx):
         h, d, v = self.heads, self.dim, self.vdim

@@ -15,6 +15,10 @@ from . import register_model
 from ..layers import FEED_FORWARDS, MIXERS, ModelContext, Rotary, hip_op
 
 
+TYPES = ("retention", "mamba2", "latent_attention")
+KINDS = {"dense": "clamped_glu"}      # the configuration's feed-forwards
+
+
 @dataclass
 class NepulixConfig:
     vocab: int
@@ -25,14 +29,14 @@ class NepulixConfig:
     @classmethod
     def from_dict(cls, raw: dict) -> "NepulixConfig":
         for layer in raw["layers"]:
-            if layer["type"] not in MIXERS:
+            if layer["type"] not in TYPES:
                 raise ValueError(f"unknown mixer {layer['type']!r}")
             MIXERS[layer["type"]].validate(layer["mixer"])
             mlp = layer.get("mlp")
             if mlp is not None:
-                if mlp["kind"] not in FEED_FORWARDS:
+                if mlp["kind"] not in KINDS:
                     raise ValueError(f"unknown feed-forward {mlp['kind']!r}")
-                FEED_FORWARDS[mlp["kind"]].validate(mlp)
+                FEED_FORWARDS[KINDS[mlp["kind"]]].validate(mlp)
         return cls(vocab=int(raw["vocab"]), width=int(raw["width"]), eps=float(raw["norm"]["eps"]), layers=list(raw["layers"]))
 
 
@@ -64,7 +68,7 @@ class NepulixModel:
             norm2 = ff = None
             if spec.get("mlp") is not None:
                 norm2 = take(p + "norm2", (config.width,), "norm_offset")
-                ff = FEED_FORWARDS[spec["mlp"]["kind"]](spec["mlp"], weights, p + "mlp.", m)
+                ff = FEED_FORWARDS[KINDS[spec["mlp"]["kind"]]](spec["mlp"], weights, p + "mlp.", m)
             self.layers.append((mixer, norm1, ff, norm2))
         self.final_norm = take("final.norm", (config.width,), "norm_offset")
         weights.finish()

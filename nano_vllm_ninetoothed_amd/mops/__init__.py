@@ -50,6 +50,16 @@ EXTENSION_OP_NAMES = (
     "latent_gather",
     "rotate_pairs",
     "latent_prefill",
+    # time mixing, attention with a distance bias, mixtures of experts
+    "add_norm_norm",
+    "token_mix",
+    "low_rank_decay",
+    "squared_relu",
+    "attention_prepare",
+    "biased_attention_rows",
+    "moe_route",
+    "moe_gate_up",
+    "moe_down",
 )
 
 

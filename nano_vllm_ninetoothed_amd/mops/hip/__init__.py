@@ -1,1 +1,1 @@
-from . import ops, recurrent_ops  # noqa: F401
+from . import attention_ops, mixture_ops, ops, recurrent_ops  # noqa: F401

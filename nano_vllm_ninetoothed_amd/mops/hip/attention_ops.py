@@ -1,0 +1,84 @@
+"""Extension ops of the `hip` backend for grouped-query attention with a linear distance bias over paged keys and values of any
+two sizes (the rules of recurrent_ops.py hold)."""
+from __future__ import annotations
+
+from ctypes import byref
+
+import torch
+
+from ... import _capi
+from .ops import _require, _stream
+from .recurrent_ops import _dtype, _flat
+from .registry import register_hip_op
+
+
+def padded(n: int) -> int:
+    """Head sizes in queries and pages: rounded up to 16-byte pieces of bf16."""
+    return (n + 7) // 8 * 8
+
+
+def _pages(name, pages, heads, size, dtype):
+    _require(pages.is_cuda and pages.dtype == dtype and pages.is_contiguous() and pages.dim() == 4 and pages.shape[2:] == (heads, padded(size)),
+             f"{name} must be contiguous [blocks, block_size, {heads}, {padded(size)}] of {dtype}")
+    return pages.data_ptr()
+
+
+@register_hip_op
+def attention_prepare(qkv, q_weight, k_weight, eps, positions, slot_mapping, k_pages, v_pages, heads, kv_heads, dim, vdim, q_factor=None):
+    """qkv rows [q | k | v]: RMS norms over the whole of q and of k, a factor per position on q, k and v into their pages.
+    Returns q [tokens, heads, padded dim]."""
+    code = _dtype("qkv", qkv)
+    tokens = qkv.shape[0]
+    a = _capi.AttentionPrepare()
+    _require(qkv.dim() == 2 and qkv.stride(1) == 1 and qkv.shape[1] >= (heads + kv_heads) * dim + kv_heads * vdim, "qkv must be [tokens, q | k | v]")
+    a.qkv, a.qkv_stride = qkv.data_ptr(), qkv.stride(0) if tokens > 1 else qkv.shape[1]
+    a.q_weight, a.k_weight = _flat("q_weight", q_weight, heads * dim, qkv.dtype), _flat("k_weight", k_weight, kv_heads * dim, qkv.dtype)
+    a.max_positions = 1
+    if q_factor is not None:
+        a.q_factor, a.max_positions = _flat("q_factor", q_factor, q_factor.numel(), torch.float32), q_factor.numel()
+    a.positions, a.slot_mapping = _flat("positions", positions, tokens, torch.int32), _flat("slot_mapping", slot_mapping, tokens, torch.int32)
+    q = torch.empty((tokens, heads, padded(dim)), dtype=qkv.dtype, device=qkv.device)
+    a.q, a.k_pages, a.v_pages = q.data_ptr(), _pages("k_pages", k_pages, kv_heads, dim, qkv.dtype), _pages("v_pages", v_pages, kv_heads, vdim, qkv.dtype)
+    _require(k_pages.shape[:2] == v_pages.shape[:2], "k_pages and v_pages must have the same blocks")
+    a.num_slots, a.tokens, a.heads, a.kv_heads, a.dim, a.vdim = k_pages.shape[0] * k_pages.shape[1], tokens, heads, kv_heads, dim, vdim
+    a.eps, a.dtype = float(eps), code
+    st = _capi.load().mops_hip_attention_prepare(byref(a), _stream(qkv))
+    _capi.check("mops_hip_attention_prepare", st)
+    return q
+
+
+def _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes, row_seq, out):
+    code = _dtype("q", q)
+    rows, heads, dp = q.shape
+    kv_heads = k_pages.shape[2]
+    _require(q.is_contiguous() and dp == padded(dim), "q must be contiguous [rows, heads, padded dim]")
+    _require(heads % kv_heads == 0, "query heads must be a multiple of kv heads")
+    _require(out.is_cuda and out.is_contiguous() and out.dtype == q.dtype and out.numel() == rows * heads * vdim, "out must be contiguous [rows, heads, vdim]")
+    a = _capi.BiasedAttention()
+    a.q, a.k_pages, a.v_pages = q.data_ptr(), _pages("k_pages", k_pages, kv_heads, dim, q.dtype), _pages("v_pages", v_pages, kv_heads, vdim, q.dtype)
+    _require(k_pages.shape[:2] == v_pages.shape[:2], "k_pages and v_pages must have the same blocks")
+    if slopes is not None:
+        a.slopes = _flat("slopes", slopes, heads, torch.float32)
+    if row_seq is not None:
+        a.row_seq = _flat("row_seq", row_seq, rows, torch.int32)
+    a.context_lens = _flat("context_lens", context_lens, rows, torch.int32)
+    _require(block_table.dtype == torch.int32 and block_table.is_cuda and block_table.dim() == 2 and block_table.stride(1) == 1
+             and (row_seq is not None or block_table.shape[0] >= rows), "block_table must be an int32 GPU tensor [sequences, blocks]")
+    a.block_table, a.max_blocks = block_table.data_ptr(), block_table.shape[1]
+    a.block_table_stride = block_table.stride(0) if block_table.shape[0] > 1 else block_table.shape[1]
+    a.num_blocks, a.block_size = k_pages.shape[:2]
+    a.out, a.rows, a.heads, a.kv_heads, a.dim, a.vdim = out.data_ptr(), rows, heads, kv_heads, dim, vdim
+    a.scale, a.dtype = float(scale), code
+    return a
+
+
+@register_hip_op
+def biased_attention_rows(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes=None, row_seq=None):
+    """Attention of single query rows against the pages: row r sees the first context_lens[r] tokens of block table row row_seq[r]
+    (r itself without row_seq); score = q.k scale - slope (distance).  Returns [rows, heads, vdim].  The plain form: any size, bf16
+    or float32."""
+    out = torch.empty((q.shape[0], q.shape[1], vdim), dtype=q.dtype, device=q.device)
+    a = _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes, row_seq, out)
+    st = _capi.load().mops_hip_biased_attention_rows(byref(a), _stream(q))
+    _capi.check("mops_hip_biased_attention_rows", st)
+    return out

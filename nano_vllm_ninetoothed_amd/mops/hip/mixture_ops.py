@@ -1,0 +1,79 @@
+"""Extension ops of the `hip` backend for mixtures of experts: routing and grouped products (the rules of recurrent_ops.py hold).
+Nothing comes back to the host, so that a captured step routes anew at every replay."""
+from __future__ import annotations
+
+from ctypes import byref
+from dataclasses import dataclass
+
+import torch
+
+from ... import _capi
+from .ops import _require, _stream
+from .recurrent_ops import _dtype, _flat, _rows
+from .registry import register_hip_op
+
+SMALL_BLOCK, LARGE_BLOCK = 32, 128
+
+
+@dataclass
+class Routing:
+    """Where every token goes: chosen experts and their scores [tokens, top], the choices ordered by expert, blocks of them."""
+    args: object
+    chosen: torch.Tensor
+    score: torch.Tensor
+    rows: torch.Tensor
+    tiles: torch.Tensor
+
+
+@register_hip_op
+def moe_route(h: torch.Tensor, router: torch.Tensor, top: int, block_rows: int = None) -> Routing:
+    """The `top` experts with the largest logits router @ h (float32) per token, their sigmoids, and the plan of the grouped products."""
+    code = _dtype("h", h)
+    tokens, (experts, width) = h.shape[0], router.shape
+    stride = _rows("h", h, width, h.dtype)
+    _require(0 < top <= experts, "top must lie between 1 and the number of experts")
+    if block_rows is None:
+        block_rows = LARGE_BLOCK if h.dtype == torch.bfloat16 and tokens * top >= 48 * experts else SMALL_BLOCK
+    lib = _capi.load()
+    n = tokens * top
+    tiles = lib.mops_hip_moe_max_tiles(tokens, experts, top, block_rows)
+    ints = torch.empty(3 * n + experts + 1 + 3 * tiles, dtype=torch.int32, device=h.device)
+    chosen, rank, rows, counts, tile_list = ints.split([n, n, n, experts, 1 + 3 * tiles])
+    score = torch.empty((tokens, top), dtype=torch.float32, device=h.device)
+    counts.zero_()
+    m = _capi.Moe()
+    m.rows, m.tiles, m.score = rows.data_ptr(), tile_list.data_ptr(), score.data_ptr()
+    m.tokens, m.experts, m.top, m.width, m.ff, m.block_rows, m.dtype = tokens, experts, top, width, 1, block_rows, code
+    st = lib.mops_hip_moe_route(h.data_ptr(), stride, _flat("router", router, experts * width, h.dtype), chosen.data_ptr(), rank.data_ptr(), counts.data_ptr(),
+                                byref(m), _stream(h))
+    _capi.check("mops_hip_moe_route", st)
+    return Routing(m, chosen.view(tokens, top), score, rows, tile_list)
+
+
+@register_hip_op
+def moe_gate_up(h: torch.Tensor, w: torch.Tensor, routing: Routing):
+    """silu(s W_gate h) * (s W_up h) of every choice, s its score, in the order of routing.rows.  w [experts, 2, ff, width]."""
+    code = _dtype("h", h)
+    m = routing.args
+    experts, two, ff, width = w.shape
+    _require(m.tokens == h.shape[0] and m.experts == experts and m.width == width and m.dtype == code and two == 2, "the routing was made for another problem")
+    m.ff = ff
+    y = torch.empty((m.tokens * m.top, ff), dtype=h.dtype, device=h.device)
+    st = _capi.load().mops_hip_moe_gate_up(h.data_ptr(), _rows("h", h, width, h.dtype), _flat("w", w, w.numel(), h.dtype), ff, y.data_ptr(), ff, byref(m), _stream(h))
+    _capi.check("mops_hip_moe_gate_up", st)
+    return y
+
+
+@register_hip_op
+def moe_down(y: torch.Tensor, w: torch.Tensor, routing: Routing):
+    """W_down y of every choice: [tokens * top, width], a token's choices one behind the other.  w [experts, width, ff]."""
+    code = _dtype("y", y)
+    m = routing.args
+    experts, width, ff = w.shape
+    _require(y.shape == (m.tokens * m.top, ff) and y.is_contiguous() and m.experts == experts and m.width == width and m.dtype == code,
+             "the routing was made for another problem")
+    m.ff = ff
+    z = torch.empty((m.tokens * m.top, width), dtype=y.dtype, device=y.device)
+    st = _capi.load().mops_hip_moe_down(y.data_ptr(), ff, _flat("w", w, w.numel(), y.dtype), ff, z.data_ptr(), width, byref(m), _stream(y))
+    _capi.check("mops_hip_moe_down", st)
+    return z

@@ -39,16 +39,16 @@ def _flat(name: str, t: torch.Tensor, n: int, dtype: torch.dtype) -> int:
 
 
 @register_hip_op
-def embed_residual(ids: torch.Tensor, table: torch.Tensor):
-    """Embedding rows as (float32 residual, activation copy in the table's dtype)."""
+def embed_residual(ids: torch.Tensor, table: torch.Tensor, scale: float = 1.0, need_act: bool = True):
+    """Scaled embedding rows as (float32 residual, activation copy in the table's dtype or None)."""
     code = _dtype("table", table)
     _require(table.dim() == 2 and table.stride(1) == 1, "table must be [vocab, width] with contiguous rows")
     _require(ids.is_cuda and ids.dtype == torch.int64 and ids.dim() == 1 and ids.is_contiguous(), "ids must be a contiguous int64 GPU vector")
     n, (vocab, width) = ids.numel(), table.shape
     residual = torch.empty((n, width), dtype=torch.float32, device=table.device)
-    act = torch.empty((n, width), dtype=table.dtype, device=table.device)
-    st = _capi.load().mops_hip_embed_residual(ids.data_ptr(), table.data_ptr(), table.stride(0), code, residual.data_ptr(), act.data_ptr(),
-                                              n, vocab, width, _stream(table))
+    act = torch.empty((n, width), dtype=table.dtype, device=table.device) if need_act else None
+    st = _capi.load().mops_hip_embed_residual(ids.data_ptr(), table.data_ptr(), table.stride(0), code, float(scale), residual.data_ptr(),
+                                              None if act is None else act.data_ptr(), n, vocab, width, _stream(table))
     _capi.check("mops_hip_embed_residual", st)
     return residual, act
 
@@ -66,6 +66,23 @@ def norm_residual_add(residual: torch.Tensor, y: torch.Tensor, weight: torch.Ten
                                                  float(weight_offset), float(eps), act.data_ptr(), code, rows, n, _stream(y))
     _capi.check("mops_hip_norm_residual_add", st)
     return act
+
+
+@register_hip_op
+def add_norm_norm(residual: torch.Tensor, y: torch.Tensor, w_out: torch.Tensor, w_in: torch.Tensor, eps: float):
+    """residual += rms(y) * w_out in place; returns rms(residual) * w_in in y's dtype.  y [rows * parts, n]: `parts` consecutive
+    rows are summed first (the outputs of several experts)."""
+    code = _dtype("y", y)
+    rows, n = residual.shape
+    parts = y.shape[0] // rows if rows else 1
+    _flat("residual", residual, rows * n, torch.float32)
+    stride = _rows("y", y, n, y.dtype)
+    _require(parts > 0 and y.shape[0] == rows * parts, "y must have a whole number of rows per residual row")
+    out = torch.empty((rows, n), dtype=y.dtype, device=y.device)
+    st = _capi.load().mops_hip_add_norm_norm(residual.data_ptr(), y.data_ptr(), stride, parts, _flat("w_out", w_out, n, y.dtype),
+                                             _flat("w_in", w_in, n, y.dtype), float(eps), out.data_ptr(), code, rows, n, _stream(y))
+    _capi.check("mops_hip_add_norm_norm", st)
+    return out
 
 
 @register_hip_op
@@ -109,13 +126,24 @@ def clamped_glu(gate: torch.Tensor, up: torch.Tensor, limit: float, alpha: float
     return out
 
 
+@register_hip_op
+def squared_relu(x: torch.Tensor):
+    """max(x, 0)^2"""
+    code = _dtype("x", x)
+    rows, n = x.shape
+    out = torch.empty((rows, n), dtype=x.dtype, device=x.device)
+    st = _capi.load().mops_hip_squared_relu(x.data_ptr(), _rows("x", x, n, x.dtype), out.data_ptr(), code, rows, n, _stream(x))
+    _capi.check("mops_hip_squared_relu", st)
+    return out
+
+
 def recurrence_state_pitch(d: int) -> int:
     """Row pitch (elements) of the recurrent state [slots, heads, vd, pitch]."""
     return _capi.load().mops_hip_recurrence_state_pitch(d)
 
 
 def _recurrence_args(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, *, cu_seqlens=None, decay=None, log_decay=None, dt=None,
-                     dt_bias=None, neg_a=None, skip=None, cos_sin=None, k_scale=1.0, conv=None):
+                     dt_bias=None, neg_a=None, skip=None, cos_sin=None, k_scale=1.0, conv=None, channel_decay=None, bonus=None):
     code = _dtype("v", v)
     tokens = v.shape[0]
     batch = state_slots.numel()
@@ -133,8 +161,12 @@ def _recurrence_args(q, k, v, out, state, state_slots, starts, heads, groups, d,
         _require(tokens == batch, "without cu_seqlens every sequence brings one token")
     else:
         r.cu_seqlens = _flat("cu_seqlens", cu_seqlens, batch + 1, torch.int32)
-    _require((decay is None) != (dt is None), "give either a constant decay or time steps")
-    if decay is not None:
+    _require(sum(x is not None for x in (decay, dt, channel_decay)) == 1, "give a constant decay, time steps or a decay per channel")
+    if channel_decay is not None:
+        r.channel_decay, r.channel_decay_stride = channel_decay.data_ptr(), _rows("channel_decay", channel_decay, heads * d, torch.float32)
+        _require(channel_decay.shape[0] == tokens, "channel_decay must have one row per token")
+        r.bonus = _flat("bonus", bonus, heads * d, torch.float32)
+    elif decay is not None:
         r.decay = _flat("decay", decay, heads, torch.float32)
         if log_decay is not None:
             r.log_decay = _flat("log_decay", log_decay, heads, torch.float32)
@@ -162,7 +194,7 @@ def _recurrence_args(q, k, v, out, state, state_slots, starts, heads, groups, d,
 def decayed_recurrence(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, **options):
     """S <- a S + k (s v)^T, o = S^T q + skip v, token by token with the state of state_slots[b] in float32 (layout and options:
     mops_hip_recurrence in include/mops_hip.h).  Options: cu_seqlens (None: one token per sequence), decay | dt + dt_bias +
-    neg_a, skip, cos_sin (rotates q and k), k_scale, conv = (weight [taps, channels] float32, bias, ring, (q, k, v channel
+    neg_a | channel_decay + bonus, skip, cos_sin (rotates q and k), k_scale, conv = (weight [taps, channels] float32, bias, ring, (q, k, v channel
     offsets)).  Writes `out` and the state in place."""
     r = _recurrence_args(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, **options)
     st = _capi.load().mops_hip_decayed_recurrence(byref(r), _stream(v))
@@ -240,6 +272,39 @@ def short_conv_update(x, ring, cu_seqlens, starts, state_slots):
                                                  _flat("starts", starts, batch, torch.int32), _flat("state_slots", state_slots, batch, torch.int32),
                                                  code, batch, channels, ring.shape[1], _stream(x))
     _capi.check("mops_hip_short_conv_update", st)
+
+
+@register_hip_op
+def token_mix(x, mu, before, starts, state_slots, token_seq=None, cu_seqlens=None):
+    """[parts, tokens, width]: every row of x moved by mu[p] (float32) towards the row in front of it; `before` [slots, width] holds the
+    last row of each sequence's earlier tokens and receives the new last row.  Without cu_seqlens every sequence brings one token."""
+    code = _dtype("x", x)
+    tokens, width = x.shape
+    parts, batch = mu.shape[0], state_slots.numel()
+    stride = _rows("x", x, width, x.dtype)
+    _require(before.dim() == 2 and before.shape[1] == width, "before must be [slots, width]")
+    _require((token_seq is None) == (cu_seqlens is None) and (cu_seqlens is not None or tokens == batch), "packed portions need token_seq and cu_seqlens")
+    out = torch.empty((parts, tokens, width), dtype=x.dtype, device=x.device)
+    st = _capi.load().mops_hip_token_mix(x.data_ptr(), stride, _flat("mu", mu, parts * width, torch.float32), parts,
+                                         _flat("before", before, before.numel(), x.dtype), before.shape[0],
+                                         None if token_seq is None else _flat("token_seq", token_seq, tokens, torch.int32),
+                                         None if cu_seqlens is None else _flat("cu_seqlens", cu_seqlens, batch + 1, torch.int32),
+                                         _flat("starts", starts, batch, torch.int32), _flat("state_slots", state_slots, batch, torch.int32),
+                                         out.data_ptr(), code, tokens, width, _stream(x))
+    _capi.check("mops_hip_token_mix", st)
+    return out
+
+
+@register_hip_op
+def low_rank_decay(z, w2, w0):
+    """-exp(w2 tanh(z) + w0), float32: the logarithm of a decay per channel.  w2 in z's dtype, w0 float32."""
+    code = _dtype("z", z)
+    tokens, (channels, rank) = z.shape[0], w2.shape
+    out = torch.empty((tokens, channels), dtype=torch.float32, device=z.device)
+    st = _capi.load().mops_hip_low_rank_decay(z.data_ptr(), _rows("z", z, rank, z.dtype), _flat("w2", w2, channels * rank, z.dtype),
+                                              _flat("w0", w0, channels, torch.float32), out.data_ptr(), code, tokens, channels, rank, _stream(z))
+    _capi.check("mops_hip_low_rank_decay", st)
+    return out
 
 
 def _latent_cache(cache, width, dtype):

@@ -1,7 +1,8 @@
 """Where a model's tensors come from: a folder with safetensors files, or a seeded random initialisation.
 
 Both sources answer take(name, shape, kind) with a device tensor in the model's dtype; a model asks for each of its tensors
-once, under the checkpoint's name.  `kind` only matters to the random source:
+once, under the checkpoint's name.  shape_of(name) is the shape that the source holds, or None where it makes tensors of any
+shape: for sizes that the configuration leaves to the tensors.  `kind` only matters to the random source:
   linear (std fan_in^-0.5) | embed (std 0.02, or `std`) | norm (around one) | norm_offset (around zero) | vector (std 0.1)
 """
 from __future__ import annotations
@@ -66,6 +67,12 @@ class CheckpointWeights:
             return t.to(device=self.device, dtype=self.dtype)
         return t.to(self.device)
 
+    def shape_of(self, name: str):
+        t = self._tensors.get(name)
+        if t is None:
+            raise KeyError(f"the checkpoint has no tensor {name}")
+        return tuple(t.shape)
+
     def finish(self) -> None:
         if self._tensors:
             print(f"tensors of the checkpoint that the model does not use: {', '.join(sorted(self._tensors))}", file=sys.stderr)
@@ -83,6 +90,9 @@ class RandomWeights:
             std = {"linear": shape[-1] ** -0.5, "embed": 0.02, "norm": 0.05, "norm_offset": 0.05, "vector": 0.1}[kind]
         t = torch.randn(tuple(shape), generator=self._g, device=self.device, dtype=torch.float32) * std
         return ((1.0 + t) if kind == "norm" else t).to(torch.bfloat16).to(self.dtype)
+
+    def shape_of(self, name: str):
+        return None
 
     def finish(self) -> None:
         pass
