@@ -424,6 +424,14 @@ int mops_hip_decayed_chunks(const mops_hip_recurrence* r, const int32_t* segment
                             const int32_t* seq_segments, float* seg_state, float* seg_decay, void* stream);
 
 /*
+ * The same for a decay per key channel (csrc/channel_chunks.hip): 16 tokens at a time, bf16, d <= 256, channel_decay and bonus
+ * given, no rotation, k_scale 1; a decay below 2^-28 counts as 2^-28.  seg_decay: float [num_segments, heads, pitch].
+ */
+int64_t mops_hip_channel_chunks_workgroups(int64_t heads, int64_t vd);
+int mops_hip_channel_chunks(const mops_hip_recurrence* r, const int32_t* segments, int64_t num_segments,
+                            const int32_t* seq_segments, float* seg_state, float* seg_decay, void* stream);
+
+/*
  * out[t, c] = silu(bias[c] + sum over lags l < taps of weight[taps-1-l, c] * x(position - l)[c]) for packed portions.
  * weight: float [taps, channels]; x of earlier portions comes from ring [num_slots, taps, channels] (`dtype`), row
  * position % taps; positions before 0 count as zeros.  token_seq: int32 [tokens], the sequence of each token.

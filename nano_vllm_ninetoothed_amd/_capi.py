@@ -108,6 +108,8 @@ SIGNATURES = {
     "mops_hip_decayed_recurrence": (c_int, [POINTER(Recurrence), c_void_p]),
     "mops_hip_decayed_chunks_workgroups": (c_int64, [c_int64] * 3),
     "mops_hip_decayed_chunks": (c_int, [POINTER(Recurrence), c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p]),
+    "mops_hip_channel_chunks_workgroups": (c_int64, [c_int64] * 2),
+    "mops_hip_channel_chunks": (c_int, [POINTER(Recurrence), c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p]),
     "mops_hip_short_conv": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p,
                                     c_void_p, c_int, c_int64, c_int64, c_int64, c_void_p]),
     "mops_hip_short_conv_update": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int, c_int64, c_int64,

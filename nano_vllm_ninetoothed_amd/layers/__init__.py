@@ -16,7 +16,7 @@ from dataclasses import dataclass
 import torch
 
 from .. import mops
-from ..mops.hip.recurrent_ops import CHUNK_MAX_DIM, recurrence_segments
+from ..mops.hip.recurrent_ops import CHUNK_MAX_DIM, channel_segments, recurrence_segments
 
 MIXERS: dict = {}
 FEED_FORWARDS: dict = {}
@@ -101,11 +101,16 @@ class Rotary:
 class ChunkedRecurrence:
     """Runs a decayed recurrence over the portions of a batch: in chunks on the matrix cores in bf16, token by token for what
     those kernels do not cover (float32, head sizes beyond theirs)."""
+    CHUNKS = "decayed_chunks"
 
     def __init__(self, heads, groups, d, vd, dtype):
         self.sizes = (heads, groups, d, vd)
         self.chunked = dtype == torch.bfloat16 and d <= CHUNK_MAX_DIM
-        self.recurrence, self.chunks = hip_op("decayed_recurrence"), hip_op("decayed_chunks")
+        self.recurrence, self.chunks = hip_op("decayed_recurrence"), hip_op(self.CHUNKS)
+
+    def segments(self, counts):
+        heads, groups, _, vd = self.sizes
+        return recurrence_segments(counts, heads, groups, vd)
 
     def __call__(self, q, k, v, out, state, ctx, **options):
         """q, k, v, out: the rows of the portions.  The cut into segments is shared by the layers of a step."""
@@ -115,24 +120,20 @@ class ChunkedRecurrence:
         if not self.chunked:
             return self.recurrence(q, k, v, out, state, slots, starts, *self.sizes, cu_seqlens=cu, **options)
         cuts = ctx.setdefault("segment_cuts", {})
-        key = (heads, groups, vd)
+        key = (self.CHUNKS, heads, groups, vd)
         if key not in cuts:
-            segments, bounds = recurrence_segments(ctx["seq_counts"][nd:], heads, groups, vd)
+            segments, bounds = self.segments(ctx["seq_counts"][nd:])
             flat = torch.tensor([x for s in segments for x in s] + bounds, dtype=torch.int32).to(v.device, non_blocking=True)
             cuts[key] = (flat[:3 * len(segments)].view(-1, 3), flat[3 * len(segments):])
         return self.chunks(q, k, v, out, state, slots, starts, *self.sizes, *cuts[key], cu_seqlens=cu, **options)
 
 
-class ChannelRecurrence:
+class ChannelRecurrence(ChunkedRecurrence):
     """The same for a recurrence with a decay per key channel and a bonus for the current token."""
+    CHUNKS = "channel_chunks"
 
-    def __init__(self, heads, d, dtype):
-        self.sizes = (heads, heads, d, d)
-        self.recurrence = hip_op("decayed_recurrence")
-
-    def __call__(self, r, k, v, out, state, ctx, **options):
-        nd = ctx["n_decode"]
-        return self.recurrence(r, k, v, out, state, ctx["state_slots"][nd:], ctx["starts"][nd:], *self.sizes, cu_seqlens=ctx["portion_cu"], **options)
+    def segments(self, counts):
+        return channel_segments(counts, self.sizes[0], self.sizes[3])
 
 
 def hip_op(name):

@@ -33,7 +33,7 @@ class TimeMixing(Mixer):
         self.bonus = take(prefix + "u", (h, d), "vector").float().reshape(-1).contiguous()
         self.norm = take(prefix + "norm", (h * d,), "norm")
         self.o = take(prefix + "o", (m.width, h * d))
-        self.portions = ChannelRecurrence(h, d, m.dtype)
+        self.portions = ChannelRecurrence(h, h, d, d, m.dtype)
         self.linear, self.head_linear, self.mix = hip_op("linear"), hip_op("head_linear"), hip_op("token_mix")
         self.decay, self.recurrence, self.group_norm = hip_op("low_rank_decay"), hip_op("decayed_recurrence"), hip_op("gated_group_norm")
         self.allocate(m.cache)

@@ -53,6 +53,7 @@ EXTENSION_OP_NAMES = (
     # time mixing, attention with a distance bias, mixtures of experts
     "add_norm_norm",
     "token_mix",
+    "channel_chunks",
     "low_rank_decay",
     "squared_relu",
     "attention_prepare",

@@ -208,7 +208,15 @@ CHUNK_MAX_DIM = 256       # head sizes (d) the chunked kernels cover
 def recurrence_segments(counts, heads: int, groups: int, vd: int, wanted: int = 512):
     """Cuts portions of counts[i] tokens (packed one behind the other) into segments for decayed_chunks: one per portion if
     those give enough workgroups, else about `wanted` workgroups in all.  Returns host lists (segments, bounds per portion)."""
-    per_segment = _capi.load().mops_hip_decayed_chunks_workgroups(heads, groups, vd)
+    return _segments(counts, _capi.load().mops_hip_decayed_chunks_workgroups(heads, groups, vd), wanted)
+
+
+def channel_segments(counts, heads: int, vd: int, wanted: int = 768):
+    """The same for channel_chunks."""
+    return _segments(counts, _capi.load().mops_hip_channel_chunks_workgroups(heads, vd), wanted)
+
+
+def _segments(counts, per_segment: int, wanted: int):
     length = max(counts)
     if len(counts) * per_segment < wanted // 2 and length > 256:
         length = max(128, -(-sum(counts) * per_segment // wanted // 64) * 64)
@@ -221,23 +229,34 @@ def recurrence_segments(counts, heads: int, groups: int, vd: int, wanted: int = 
     return segments, bounds
 
 
-@register_hip_op
-def decayed_chunks(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, segments, seq_segments, **options):
-    """decayed_recurrence for packed portions of many tokens, on the matrix cores (bf16).  segments [n, 3] and seq_segments
-    [sequences + 1] are the int32 device copies of what recurrence_segments returns; cu_seqlens is required."""
+def _chunks(name, seg_decay_shape, q, k, v, out, state, state_slots, starts, heads, groups, d, vd, segments, seq_segments, **options):
     r = _recurrence_args(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, **options)
     n = segments.shape[0]
     _require(r.batch == seq_segments.numel() - 1, "seq_segments must bound the segments of every sequence")
     seg_state = seg_decay = None
     if n > r.batch:
         seg_state = torch.empty((n, heads, vd, state.shape[3]), dtype=torch.float32, device=v.device)
-        seg_decay = torch.empty((n, heads), dtype=torch.float32, device=v.device)
-    st = _capi.load().mops_hip_decayed_chunks(byref(r), _flat("segments", segments, 3 * n, torch.int32), n,
-                                              _flat("seq_segments", seq_segments, r.batch + 1, torch.int32),
-                                              None if seg_state is None else seg_state.data_ptr(),
-                                              None if seg_decay is None else seg_decay.data_ptr(), _stream(v))
-    _capi.check("mops_hip_decayed_chunks", st)
+        seg_decay = torch.empty((n, *seg_decay_shape), dtype=torch.float32, device=v.device)
+    st = getattr(_capi.load(), name)(byref(r), _flat("segments", segments, 3 * n, torch.int32), n,
+                                     _flat("seq_segments", seq_segments, r.batch + 1, torch.int32),
+                                     None if seg_state is None else seg_state.data_ptr(),
+                                     None if seg_decay is None else seg_decay.data_ptr(), _stream(v))
+    _capi.check(name, st)
     return out
+
+
+@register_hip_op
+def decayed_chunks(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, segments, seq_segments, **options):
+    """decayed_recurrence for packed portions of many tokens, on the matrix cores (bf16).  segments [n, 3] and seq_segments
+    [sequences + 1] are the int32 device copies of what recurrence_segments returns; cu_seqlens is required."""
+    return _chunks("mops_hip_decayed_chunks", (heads,), q, k, v, out, state, state_slots, starts, heads, groups, d, vd, segments, seq_segments, **options)
+
+
+@register_hip_op
+def channel_chunks(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, segments, seq_segments, **options):
+    """The same for channel_decay and bonus; segments from channel_segments."""
+    return _chunks("mops_hip_channel_chunks", (heads, state.shape[3]), q, k, v, out, state, state_slots, starts, heads, groups, d, vd, segments,
+                   seq_segments, **options)
 
 
 @register_hip_op
