@@ -567,6 +567,18 @@ typedef struct {
 int mops_hip_biased_attention_rows(const mops_hip_biased_attention* a, void* stream);
 
 /*
+ * The same on the matrix cores: bf16, dim <= 256, vdim <= 256.
+ * biased_decode (csrc/biased_decode.hip): single rows; block_size a multiple of 32.  workspace: device scratch of at least
+ * mops_hip_biased_decode_workspace_bytes(...), private to the call until it completes.
+ * biased_prefill (csrc/biased_prefill.hip): long portions.  q and out cover `rows` rows; tiles: int32 [num_tiles][5] = (first query
+ * row, queries <= 128, position of the first query, block table row, tokens of the context); row_seq is not read and context_lens
+ * only has to be there.  Writes the tiles' rows of out.
+ */
+int64_t mops_hip_biased_decode_workspace_bytes(int64_t rows, int64_t heads, int64_t kv_heads, int64_t dim, int64_t vdim);
+int mops_hip_biased_decode(const mops_hip_biased_attention* a, void* workspace, int64_t workspace_bytes, void* stream);
+int mops_hip_biased_prefill(const mops_hip_biased_attention* a, const int32_t* tiles, int64_t num_tiles, void* stream);
+
+/*
  * Mixture of experts (csrc/moe.hip).  moe_route: logits = router [experts, width] h in float32; chosen, score [tokens * top] =
  * the experts with the largest logits and the sigmoids of these; rank [tokens * top] is scratch, counts [experts] must be zeros
  * and receives the choices per expert; rows [tokens * top] lists the choices (token * top + place) ordered by expert, tiles

@@ -132,6 +132,9 @@ SIGNATURES = {
     "mops_hip_squared_relu": (c_int, [c_void_p, c_int64, c_void_p, c_int, c_int64, c_int64, c_void_p]),
     "mops_hip_attention_prepare": (c_int, [POINTER(AttentionPrepare), c_void_p]),
     "mops_hip_biased_attention_rows": (c_int, [POINTER(BiasedAttention), c_void_p]),
+    "mops_hip_biased_decode_workspace_bytes": (c_int64, [c_int64] * 5),
+    "mops_hip_biased_decode": (c_int, [POINTER(BiasedAttention), c_void_p, c_int64, c_void_p]),
+    "mops_hip_biased_prefill": (c_int, [POINTER(BiasedAttention), c_void_p, c_int64, c_void_p]),
     "mops_hip_moe_max_tiles": (c_int64, [c_int64] * 4),
     "mops_hip_moe_route": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p, POINTER(Moe), c_void_p]),
     "mops_hip_moe_gate_up": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, POINTER(Moe), c_void_p]),

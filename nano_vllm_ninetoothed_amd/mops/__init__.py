@@ -58,6 +58,8 @@ EXTENSION_OP_NAMES = (
     "squared_relu",
     "attention_prepare",
     "biased_attention_rows",
+    "biased_decode",
+    "biased_prefill",
     "moe_route",
     "moe_gate_up",
     "moe_down",

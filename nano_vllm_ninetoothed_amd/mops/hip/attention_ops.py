@@ -47,7 +47,7 @@ def attention_prepare(qkv, q_weight, k_weight, eps, positions, slot_mapping, k_p
     return q
 
 
-def _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes, row_seq, out):
+def _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes, row_seq, out, own_rows=True):
     code = _dtype("q", q)
     rows, heads, dp = q.shape
     kv_heads = k_pages.shape[2]
@@ -63,7 +63,7 @@ def _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scal
         a.row_seq = _flat("row_seq", row_seq, rows, torch.int32)
     a.context_lens = _flat("context_lens", context_lens, rows, torch.int32)
     _require(block_table.dtype == torch.int32 and block_table.is_cuda and block_table.dim() == 2 and block_table.stride(1) == 1
-             and (row_seq is not None or block_table.shape[0] >= rows), "block_table must be an int32 GPU tensor [sequences, blocks]")
+             and (row_seq is not None or not own_rows or block_table.shape[0] >= rows), "block_table must be an int32 GPU tensor [sequences, blocks]")
     a.block_table, a.max_blocks = block_table.data_ptr(), block_table.shape[1]
     a.block_table_stride = block_table.stride(0) if block_table.shape[0] > 1 else block_table.shape[1]
     a.num_blocks, a.block_size = k_pages.shape[:2]
@@ -81,4 +81,48 @@ def biased_attention_rows(q, k_pages, v_pages, dim, vdim, context_lens, block_ta
     a = _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes, row_seq, out)
     st = _capi.load().mops_hip_biased_attention_rows(byref(a), _stream(q))
     _capi.check("mops_hip_biased_attention_rows", st)
+    return out
+
+
+def biased_matrix_covers(dtype, dim: int, vdim: int, block_size: int) -> bool:
+    """Whether biased_decode and biased_prefill cover these sizes."""
+    return dtype == torch.bfloat16 and dim <= 256 and vdim <= 256 and block_size % 32 == 0
+
+
+@register_hip_op
+def biased_decode(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes=None, row_seq=None, out=None):
+    """biased_attention_rows on the matrix cores (sizes: biased_matrix_covers)."""
+    if out is None:
+        out = torch.empty((q.shape[0], q.shape[1], vdim), dtype=q.dtype, device=q.device)
+    a = _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes, row_seq, out)
+    lib = _capi.load()
+    ws = torch.empty(max(16, lib.mops_hip_biased_decode_workspace_bytes(a.rows, a.heads, a.kv_heads, dim, vdim)), dtype=torch.uint8, device=q.device)
+    st = lib.mops_hip_biased_decode(byref(a), ws.data_ptr(), ws.numel(), _stream(q))
+    _capi.check("mops_hip_biased_decode", st)
+    return out
+
+
+BIASED_QUERIES = 128
+
+
+def biased_prefill_tiles(counts, starts, first_token: int, first_seq: int):
+    """Host list for biased_prefill: portions of counts[i] tokens at positions starts[i].., packed from row first_token on; sequence i
+    of the list is block table row first_seq + i.  The tiles that see most come first: they bound the launch."""
+    tiles, at = [], first_token
+    for i, (n, start) in enumerate(zip(counts, starts)):
+        tiles += [(at + q, min(BIASED_QUERIES, n - q), start + q, first_seq + i, start + n) for q in range(0, n, BIASED_QUERIES)]
+        at += n
+    return sorted(tiles, key=lambda t: -(t[1] + t[2]))
+
+
+@register_hip_op
+def biased_prefill(q, k_pages, v_pages, dim, vdim, tiles, block_table, scale, context_lens, slopes=None, out=None):
+    """Causal attention of long portions, whose keys and values are in the pages already: tiles [n, 5] is the int32 device copy of
+    biased_prefill_tiles.  context_lens: of every row.  Writes the portions' rows of out [rows, heads, vdim]."""
+    if out is None:
+        out = torch.empty((q.shape[0], q.shape[1], vdim), dtype=q.dtype, device=q.device)
+    a = _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes, None, out, own_rows=False)
+    n = tiles.shape[0]
+    st = _capi.load().mops_hip_biased_prefill(byref(a), _flat("tiles", tiles, 5 * n, torch.int32), n, _stream(q))
+    _capi.check("mops_hip_biased_prefill", st)
     return out
