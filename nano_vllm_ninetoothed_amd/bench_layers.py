@@ -1,6 +1,6 @@
-"""Measurements behind `bench.py --op nepulix`: prefill and decode throughput of Nepulix models with layers of real sizes beside
-Qwen3 models of equal width, depth, feed-forward and vocabulary, and every kernel of the design beside the like kernel of the
-Qwen3 path.  Random weights and inputs."""
+"""Measurements behind `bench.py --op nepulix` and `--op sozarax`: prefill and decode throughput of models with layers of real sizes
+beside models of equal width, depth, feed-forward and vocabulary (Qwen3; for Sozarax also Nepulix), and every kernel of the
+design beside the like kernel of those.  Random weights and inputs."""
 from __future__ import annotations
 
 import torch
@@ -35,6 +35,23 @@ def sizes():
                                {"heads": 64, "vdim": 64, "state": 128, "groups": 8, "conv": 4, "norm_groups": 8}, _latent(16, 1536)),
                   Qwen3Shape(num_layers=6, hidden=2048, intermediate=6144, vocab=32768)),
     }
+
+
+def sozarax_dict(width, layers, ff, vocab, wkv, att, experts, top):
+    """Two time-mixing layers, one attention layer and so on; dense and routed feed-forwards in turn, a token's experts together as
+    wide as the dense one."""
+    mlps = [{"kind": "dense", "ff": ff}, {"kind": "moe", "expert": {"ff": ff // top}, "router": {"experts": experts, "top": top}}]
+    out = [{"type": "attention" if i % 3 == 2 else "wkv", "mixer": att if i % 3 == 2 else wkv, "mlp": mlps[i % 2]} for i in range(layers)]
+    return {"architecture": "Sozarax", "width": width, "vocab": vocab, "norm": {"eps": 1e-6}, "embedding": {"scale": width ** 0.5}, "layers": out,
+            "loop": {"start": 0, "stop": layers, "times": 1}}
+
+
+def sozarax_sizes():
+    """name -> (Sozarax config.json dict, Nepulix dict and Qwen3Shape of equal size)"""
+    att = {"heads": 16, "kv_heads": 8, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "q_temp": {"coef": 0.1, "every": 1024}}
+    near = sizes()
+    return {"w1024": (sozarax_dict(1024, 12, 3072, 32768, {"heads": 16, "dim": 64}, att, 16, 2), *near["w1024"]),
+            "w2048": (sozarax_dict(2048, 6, 6144, 32768, {"heads": 16, "dim": 128}, att, 32, 4), *near["w2048"])}
 
 
 def _events(fn, warmup, steps):
@@ -100,20 +117,26 @@ def graph_time(fn, calls=10, replays=10):
     return _events(graph.replay, 3, replays) / calls
 
 
-def kernel_table(dev, seed=0, only=""):
-    """[{kernel, us, bound, achieved, unit, frac, like, like_frac}]: algorithmic work over time, as a fraction of the roof."""
-    from . import mops
-    from . import workloads as W
-    from .layers import Rotary
-    from .mops.hip import recurrent_ops as R
-    op = lambda n: mops.get_op(n, "hip")      # noqa: E731
-    g = torch.Generator(device=dev).manual_seed(seed)
-    rnd = lambda *s: torch.randn(s, generator=g, device=dev, dtype=torch.float32).bfloat16()      # noqa: E731
-    i32 = lambda x: torch.tensor(x, dtype=torch.int32, device=dev)      # noqa: E731
-    rows, likes = [], {}
+class KernelTable:
+    """Rows {kernel, shape, us, bound, achieved, unit, frac, like, like_frac, times_further}: algorithmic work over time, as a fraction of
+    the roof, beside the fraction of a like kernel timed before."""
 
-    def add(name, shape, timed, nbytes=0.0, flops=0.0, like=None):
-        if only and not name.startswith(tuple(only.split(","))):
+    def __init__(self, dev, seed=0, only=""):
+        self.dev, self.seed, self.only = dev, seed, tuple(x for x in only.split(",") if x)
+        self.g = torch.Generator(device=dev).manual_seed(seed)
+        self.rows, self.likes = [], {}
+
+    def rnd(self, *shape):
+        return torch.randn(shape, generator=self.g, device=self.dev, dtype=torch.float32).bfloat16()
+
+    def f32(self, *shape):
+        return torch.randn(shape, generator=self.g, device=self.dev)
+
+    def i32(self, x):
+        return torch.tensor(x, dtype=torch.int32, device=self.dev)
+
+    def add(self, name, shape, timed, nbytes=0.0, flops=0.0, like=None):
+        if self.only and not name.startswith(self.only):
             return
         seconds = timed()
         t_mem, t_math = nbytes / (HBM * 1e9), flops / (MFMA * 1e12)
@@ -122,30 +145,53 @@ def kernel_table(dev, seed=0, only=""):
         r = {"kernel": name, "shape": shape, "us": round(seconds * 1e6, 2), "bound": bound, "achieved": round(value, 1), "unit": unit,
              "frac": round(max(t_mem, t_math) / seconds, 4)}
         if like is None:
-            likes[name] = r["frac"]
+            self.likes[name] = r["frac"]
         else:
-            r.update(like=like, like_frac=likes.get(like), times_further=round(likes[like] / r["frac"], 2) if like in likes else None)
-        rows.append(r)
+            known = self.likes.get(like)
+            r.update(like=like, like_frac=known, times_further=None if known is None else round(known / r["frac"], 2))
+            self.likes.setdefault(f"{name} {shape}", r["frac"])
+        self.rows.append(r)
 
-    # ---- the Qwen3 path's kernels, the yardstick
-    ctx = W.random_seq_lens(256, 512, 4096, seed=seed)
+
+PROMPTS = [1024] * 16
+T = sum(PROMPTS)      # tokens of a prefill step
+
+
+def op(name):
+    from . import mops
+    return mops.get_op(name, "hip")
+
+
+def decode_contexts(t):
+    """Context lengths of a decode step, blocks of the pool, block table of shuffled blocks, lengths on the device."""
+    from . import workloads as W
+    ctx = W.random_seq_lens(256, 512, 4096, seed=t.seed)
     nb = [(c + 255) // 256 for c in ctx]
-    perm = torch.randperm(sum(nb), generator=torch.Generator().manual_seed(seed)).to(torch.int32)
+    perm = torch.randperm(sum(nb), generator=torch.Generator().manual_seed(t.seed)).to(torch.int32)
     table, at = torch.full((256, max(nb)), -1, dtype=torch.int32), 0
     for b, n in enumerate(nb):
         table[b, :n] = perm[at:at + n]
         at += n
-    table, lens_g = table.to(dev), i32(ctx)
-    kc, vc, q = rnd(sum(nb), 256, 8, 128), rnd(sum(nb), 256, 8, 128), rnd(256, 1, 16, 128)
+    return ctx, sum(nb), table.to(t.dev), t.i32(ctx)
+
+
+def _handles(t):
+    return t.add, t.rnd, t.i32, t.dev
+
+
+def qwen3_kernels(t):
+    """The Qwen3 path's kernels, the yardstick."""
+    from . import workloads as W
+    add, rnd, i32, dev = _handles(t)
+    ctx, blocks, table, lens_g = decode_contexts(t)
+    kc, vc, q = rnd(blocks, 256, 8, 128), rnd(blocks, 256, 8, 128), rnd(256, 1, 16, 128)
     add("paged_decode", "256 x uniform[512,4096], 16/8 heads", lambda: graph_time(lambda i: op("flash_attn_with_kvcache")(
-        q, kc, vc, cache_seqlens=lens_g, block_table=table, softmax_scale=0.088, causal=True), 4), nbytes=W.decode_bytes(ctx, 16, 8, max(nb)))
+        q, kc, vc, cache_seqlens=lens_g, block_table=table, softmax_scale=0.088, causal=True), 4), nbytes=W.decode_bytes(ctx, 16, 8, table.shape[1]))
     del kc, vc
-    plens = [1024] * 16
-    T = sum(plens)
-    d = W.to_device(W.prefill_inputs(plens, seed=seed), dev)
+    d = W.to_device(W.prefill_inputs(PROMPTS, seed=t.seed), dev)
     add("varlen_prefill", "16 x 1024, 16/8 heads of 128", lambda: _events(lambda: op("flash_attn_varlen_func")(
         d["q"], d["k"], d["v"], max_seqlen_q=1024, cu_seqlens_q=d["cu_seqlens"], max_seqlen_k=1024, cu_seqlens_k=d["cu_seqlens"], softmax_scale=d["scale"],
-        causal=True, block_table=None), 300, 200), flops=W.prefill_flops(plens, 16))
+        causal=True, block_table=None), 300, 200), flops=W.prefill_flops(PROMPTS, 16))
     bufs = [rnd(T, 6144) for _ in range(4)]
     halves = [b.chunk(2, dim=-1) for b in bufs]
     add("siluAndMul", f"{T} x 3072", lambda: graph_time(lambda i: op("siluAndMul")(*halves[i % 4]), 8), nbytes=T * 3072 * 6)
@@ -166,9 +212,15 @@ def kernel_table(dev, seed=0, only=""):
     xs = rnd(256, 1024)
     add("linear decode", "256 x 1024 x 1024 (library)", lambda: graph_time(lambda i: op("linear")(xs, wls[i % 64]), 64), nbytes=1024 * 1024 * 2 + 256 * 1024 * 4)
 
-    # ---- the design's kernels
+
+def latent_kernels(t):
+    from .layers import Rotary
+    from .mops.hip import recurrent_ops as R
+    add, rnd, i32, dev = _handles(t)
+    ctx, blocks, table, lens_g = decode_contexts(t)
+    slots = torch.randperm(T, device=dev).to(torch.int32)
     H, kr, rot, dim, vdim = 16, 512, 64, 128, 128
-    cache, ql, qn = rnd(sum(nb), 256, kr + rot), rnd(256, H, kr), rnd(256, H, dim + rot)
+    cache, ql, qn = rnd(blocks, 256, kr + rot), rnd(256, H, kr), rnd(256, H, dim + rot)
     trig = Rotary(8192, dev).table(1e4, rot)
     add("latent_decode", "256 x uniform[512,4096], 16 heads, 512+64", lambda: graph_time(lambda i: op("latent_decode")(
         ql, qn[..., dim:], cache, trig, lens_g, table, 0.07), 4), nbytes=sum(ctx) * (kr + rot) * 2 + 256 * H * (2 * kr + rot) * 2,
@@ -180,12 +232,12 @@ def kernel_table(dev, seed=0, only=""):
         nbytes=H * kr * vdim * 2 + 256 * H * (vdim + kr) * 2, flops=2.0 * 256 * H * vdim * kr, like="linear decode")
     del cache
     p32 = (torch.arange(T, device=dev) % 1024).to(torch.int32)
-    row_seq, row_pos, tiles = R.latent_prefill_plan(plens, [0] * 16, 0, 0)
+    row_seq, row_pos, tiles = R.latent_prefill_plan(PROMPTS, [0] * 16, 0, 0)
     row_seq, row_pos, tiles = i32(row_seq), i32(row_pos), i32(tiles)
     qp, kp, krp, vt = rnd(T, H, dim + rot), rnd(T, H * dim), rnd(T, rot), rnd(H * vdim, T)
     op_out = torch.empty((T, H, vdim), dtype=torch.bfloat16, device=dev)
     add("latent_prefill", "16 x 1024, 16 heads, 192/128", lambda: _events(lambda: op("latent_prefill")(qp, kp, krp, vt, tiles, 0.07, op_out), 300, 200),
-        flops=sum(2.0 * H * (dim + rot + vdim) * n * (n + 1) / 2 for n in plens), like="varlen_prefill")
+        flops=sum(2.0 * H * (dim + rot + vdim) * n * (n + 1) / 2 for n in PROMPTS), like="varlen_prefill")
     add("rotate_pairs", f"{T} x 16 heads x 64", lambda: graph_time(lambda i: op("rotate_pairs")(qp[..., dim:], p32, trig), 8), nbytes=T * H * rot * 4.0, like="qk_norm_rope_store")
     pages = rnd(T // 256, 256, kr + rot)
     ptab = torch.arange(T // 256, dtype=torch.int32, device=dev).view(16, -1)
@@ -194,48 +246,60 @@ def kernel_table(dev, seed=0, only=""):
     add("latent_prepare", f"{T} tokens, 768 / 512+64", lambda: graph_time(lambda i: op("latent_prepare")(down[i % 4], wq, wk, 1e-6, trig, p32, slots, pages, 768, kr, rot), 8),
         nbytes=T * (768 + kr + rot) * 4, like="qk_norm_rope_store")
 
-    def recurrent(tag, heads, groups, dd, vd, const):
-        bs = 256
-        pitch = R.recurrence_state_pitch(dd)
-        state = torch.randn((bs, heads, vd, pitch), generator=g, device=dev)
-        gn, inner = groups * dd, heads * vd
-        opts, conv = {"k_scale": dd ** -0.5}, None
-        if const:
-            dec = torch.tensor([1 - 2.0 ** (-5 - i % 8) for i in range(heads)], dtype=torch.float64)
-            opts.update(decay=dec.float().to(dev), log_decay=dec.log().float().to(dev), cos_sin=Rotary(8192, dev).table(1e4, dd))
-        else:
-            f = lambda *s: torch.randn(s, generator=g, device=dev)      # noqa: E731
-            ch = inner + 2 * gn
-            opts.update(dt_bias=f(heads) - 2, neg_a=-torch.exp(f(heads)), skip=f(heads))
-            conv = (f(4, ch), f(ch), torch.zeros((bs, 4, ch), dtype=torch.bfloat16, device=dev), (inner + gn, inner, 0))
-        width = 2 * gn + inner
-        x, dt, o = rnd(bs, width), rnd(bs, heads), torch.empty((bs, inner), dtype=torch.bfloat16, device=dev)
-        sl, st = torch.arange(bs, dtype=torch.int32, device=dev), torch.full((bs,), 1000, dtype=torch.int32, device=dev)
-        more = {} if const else {"dt": dt, "conv": conv}
-        add("decayed_recurrence " + tag, f"{bs} sequences, {heads} x {dd} x {vd}", lambda: graph_time(lambda i: op("decayed_recurrence")(
-            x[:, inner + gn:], x[:, inner:inner + gn], x[:, :inner], o, state, sl, st, heads, groups, dd, vd, **opts, **more), 6),
-            nbytes=2.0 * bs * heads * dd * vd * 4 + bs * (width + inner) * 2, like="paged_decode")
-        xs = [rnd(T, width) for _ in range(2)]
-        dts, oT = rnd(T, heads), torch.empty((T, inner), dtype=torch.bfloat16, device=dev)
-        for nseq in (16, 1):
-            cu = list(range(0, T + 1, T // nseq))
-            segs, bounds = R.recurrence_segments([T // nseq] * nseq, heads, groups, vd)
-            segs, bounds, cu = i32(segs), i32(bounds), i32(cu)
-            more = {} if const else {"dt": dts}
-            # least arithmetic at 64 tokens a chunk: scores and their product below the diagonal, state in and out
-            add("decayed_chunks " + tag, f"{nseq} x {T // nseq}, {heads} x {dd} x {vd}", lambda: _events(lambda: op("decayed_chunks")(
-                xs[0][:, inner + gn:], xs[0][:, inner:inner + gn], xs[0][:, :inner], oT, state, sl[:nseq], torch.zeros_like(st[:nseq]), heads, groups, dd, vd, segs,
-                bounds, cu_seqlens=cu, **opts, **more), 20, 50), flops=T * heads * (65.0 * (dd + vd) + 4.0 * dd * vd), nbytes=T * (width + inner) * 2.0,
-                like="varlen_prefill")
-        if not const:
-            tok_seq, sl16 = torch.arange(T, device=dev).div(1024, rounding_mode="floor").to(torch.int32), sl[:16]
-            cu16, z16 = i32(list(range(0, T + 1, 1024))), torch.zeros(16, dtype=torch.int32, device=dev)
-            big = [rnd(T, width + inner + heads) for _ in range(2)]
-            add("short_conv", f"{T} x {width}, 4 taps", lambda: graph_time(lambda i: op("short_conv")(
-                big[i % 2][:, inner:inner + width], conv[0], conv[1], conv[2], tok_seq, cu16, z16, sl16), 4), nbytes=T * width * 4.0, like="siluAndMul")
 
-    recurrent("retention", 16, 16, 128, 128, True)
-    recurrent("mamba2", 64, 8, 128, 64, False)
+def decayed_kernels(t, tag, heads, groups, dd, vd, const):
+    from .layers import Rotary
+    from .mops.hip import recurrent_ops as R
+    add, rnd, i32, dev = _handles(t)
+    bs = 256
+    pitch = R.recurrence_state_pitch(dd)
+    state = torch.randn((bs, heads, vd, pitch), generator=t.g, device=dev)
+    gn, inner = groups * dd, heads * vd
+    opts, conv = {"k_scale": dd ** -0.5}, None
+    if const:
+        dec = torch.tensor([1 - 2.0 ** (-5 - i % 8) for i in range(heads)], dtype=torch.float64)
+        opts.update(decay=dec.float().to(dev), log_decay=dec.log().float().to(dev), cos_sin=Rotary(8192, dev).table(1e4, dd))
+    else:
+        f = t.f32
+        ch = inner + 2 * gn
+        opts.update(dt_bias=f(heads) - 2, neg_a=-torch.exp(f(heads)), skip=f(heads))
+        conv = (f(4, ch), f(ch), torch.zeros((bs, 4, ch), dtype=torch.bfloat16, device=dev), (inner + gn, inner, 0))
+    width = 2 * gn + inner
+    x, dt, o = rnd(bs, width), rnd(bs, heads), torch.empty((bs, inner), dtype=torch.bfloat16, device=dev)
+    sl, st = torch.arange(bs, dtype=torch.int32, device=dev), torch.full((bs,), 1000, dtype=torch.int32, device=dev)
+    more = {} if const else {"dt": dt, "conv": conv}
+    add("decayed_recurrence " + tag, f"{bs} sequences, {heads} x {dd} x {vd}", lambda: graph_time(lambda i: op("decayed_recurrence")(
+        x[:, inner + gn:], x[:, inner:inner + gn], x[:, :inner], o, state, sl, st, heads, groups, dd, vd, **opts, **more), 6),
+        nbytes=2.0 * bs * heads * dd * vd * 4 + bs * (width + inner) * 2, like="paged_decode")
+    xs = [rnd(T, width) for _ in range(2)]
+    dts, oT = rnd(T, heads), torch.empty((T, inner), dtype=torch.bfloat16, device=dev)
+    for nseq in (16, 1):
+        cu = list(range(0, T + 1, T // nseq))
+        segs, bounds = R.recurrence_segments([T // nseq] * nseq, heads, groups, vd)
+        segs, bounds, cu = i32(segs), i32(bounds), i32(cu)
+        more = {} if const else {"dt": dts}
+        # least arithmetic at 64 tokens a chunk: scores and their product below the diagonal, state in and out
+        add("decayed_chunks " + tag, f"{nseq} x {T // nseq}, {heads} x {dd} x {vd}", lambda: _events(lambda: op("decayed_chunks")(
+            xs[0][:, inner + gn:], xs[0][:, inner:inner + gn], xs[0][:, :inner], oT, state, sl[:nseq], torch.zeros_like(st[:nseq]), heads, groups, dd, vd, segs,
+            bounds, cu_seqlens=cu, **opts, **more), 20, 50), flops=T * heads * (65.0 * (dd + vd) + 4.0 * dd * vd), nbytes=T * (width + inner) * 2.0,
+            like="varlen_prefill")
+    if not const:
+        tok_seq, sl16 = torch.arange(T, device=dev).div(1024, rounding_mode="floor").to(torch.int32), sl[:16]
+        cu16, z16 = i32(list(range(0, T + 1, 1024))), torch.zeros(16, dtype=torch.int32, device=dev)
+        big = [rnd(T, width + inner + heads) for _ in range(2)]
+        add("short_conv", f"{T} x {width}, 4 taps", lambda: graph_time(lambda i: op("short_conv")(
+            big[i % 2][:, inner:inner + width], conv[0], conv[1], conv[2], tok_seq, cu16, z16, sl16), 4), nbytes=T * width * 4.0, like="siluAndMul")
+
+
+def nepulix_kernels(t):
+    add, rnd, i32, dev = _handles(t)
+    latent_kernels(t)
+    decayed_kernels(t, "retention", 16, 16, 128, 128, True)
+    decayed_kernels(t, "mamba2", 64, 8, 128, 64, False)
+    bufs = [rnd(T, 6144) for _ in range(4)]
+    halves = [b.chunk(2, dim=-1) for b in bufs]
+    x4, r4, w4 = [rnd(512, 4096) for _ in range(24)], [rnd(512, 4096) for _ in range(24)], rnd(4096)
+    xt, rt, w1 = [rnd(T, 1024) for _ in range(4)], [rnd(T, 1024) for _ in range(4)], rnd(1024)
     lim = lambda i: op("clamped_glu")(*halves[i % 4], 7.0)      # noqa: E731
     add("clamped_glu", f"{T} x 3072", lambda: graph_time(lim, 8), nbytes=T * 3072 * 6, like="siluAndMul")
     add("gated_group_norm", f"{T} x 3072, 24 groups", lambda: graph_time(lambda i: op("gated_group_norm")(*halves[i % 4], 24, 1e-6), 8), nbytes=T * 3072 * 6, like="siluAndMul")
@@ -248,4 +312,89 @@ def kernel_table(dev, seed=0, only=""):
     add("rms_norm_f32", "512 x 4096", lambda: graph_time(lambda i: op("rms_norm_f32")(f4[i % 24], w4, 1e-6, 1.0), 24), nbytes=512 * 4096 * 6, like="add_rms")
     emb, ids = rnd(32768, 1024), [torch.randint(0, 32768, (T,), device=dev) for _ in range(4)]
     add("embed_residual", f"{T} x 1024", lambda: graph_time(lambda i: op("embed_residual")(ids[i % 4], emb), 8), nbytes=T * 1024 * 8.0, like="add_rms prefill")
-    return rows
+
+
+def sozarax_kernels(t):
+    from .mops.hip import recurrent_ops as R
+    from .mops.hip.attention_ops import biased_prefill_tiles
+    from .layers.biased_attention import distance_slopes
+    add, rnd, i32, dev = _handles(t)
+    # ---- attention
+    ctx, blocks, table, lens_g = decode_contexts(t)
+    H, G, d = 16, 8, 128
+    slopes = distance_slopes(H).to(dev)
+    kp, vp, q = rnd(blocks, 256, G, d), rnd(blocks, 256, G, d), rnd(256, H, d)
+    add("biased_decode", "256 x uniform[512,4096], 16/8 heads of 128", lambda: graph_time(lambda i: op("biased_decode")(q, kp, vp, d, d, lens_g, table, 0.088, slopes=slopes), 4),
+        nbytes=sum(ctx) * G * 2 * d * 2.0 + 256 * H * 2 * d * 2, like="paged_decode")
+    del kp, vp
+    kp, vp, q = rnd(T // 256, 256, G, d), rnd(T // 256, 256, G, d), rnd(T, H, d)
+    tiles, ptab = i32(biased_prefill_tiles(PROMPTS, [0] * 16, 0, 0)), torch.arange(T // 256, dtype=torch.int32, device=dev).view(16, -1)
+    out, lens = torch.empty((T, H, d), dtype=torch.bfloat16, device=dev), i32([0] * T)
+    add("biased_prefill", "16 x 1024, 16/8 heads of 128", lambda: _events(lambda: op("biased_prefill")(q, kp, vp, d, d, tiles, ptab, 0.088, lens, slopes=slopes, out=out), 300, 200),
+        flops=sum(2.0 * H * 2 * d * n * (n + 1) / 2 for n in PROMPTS), like="varlen_prefill")
+    qkv, wq, wk = [rnd(T, (H + 2 * G) * d) for _ in range(2)], rnd(H * d), rnd(G * d)
+    pos, slots = (torch.arange(T, device=dev) % 1024).to(torch.int32), torch.randperm(T, device=dev).to(torch.int32)
+    add("attention_prepare", f"{T} tokens, 16/8 heads of 128", lambda: graph_time(lambda i: op("attention_prepare")(qkv[i % 2], wq, wk, 1e-6, pos, slots, kp, vp, H, G, d, d), 8),
+        nbytes=T * (H + 2 * G) * d * 4.0, like="qk_norm_rope_store")
+    # ---- time mixing
+    for heads, dd in ((16, 64), (16, 128)):
+        n = heads * dd
+        bs, pitch = 256, R.recurrence_state_pitch(dd)
+        state, sl = torch.randn((bs, heads, dd, pitch), generator=t.g, device=dev), torch.arange(bs, dtype=torch.int32, device=dev)
+        st, u = torch.full((bs,), 1000, dtype=torch.int32, device=dev), t.f32(n)
+        x, ld, o = rnd(3, bs, n), -torch.exp(t.f32(bs, n) - 3), torch.empty((bs, n), dtype=torch.bfloat16, device=dev)
+        add("decayed_recurrence channels", f"{bs} sequences, {heads} x {dd} x {dd}", lambda: graph_time(lambda i: op("decayed_recurrence")(
+            x[0], x[1], x[2], o, state, sl, st, heads, heads, dd, dd, channel_decay=ld, bonus=u), 6), nbytes=2.0 * bs * n * dd * 4 + bs * n * 12, like="decayed_recurrence retention 256 sequences, 16 x 128 x 128")
+        xs, ldT, oT = rnd(3, T, n), -torch.exp(t.f32(T, n) - 3), torch.empty((T, n), dtype=torch.bfloat16, device=dev)
+        for nseq in (16, 1):
+            segs, ends = (i32(v) for v in R.channel_segments([T // nseq] * nseq, heads, dd))
+            cu, zero = i32(list(range(0, T + 1, T // nseq))), torch.zeros(nseq, dtype=torch.int32, device=dev)
+            add("channel_chunks", f"{nseq} x {T // nseq}, {heads} x {dd} x {dd}", lambda: _events(lambda: op("channel_chunks")(
+                xs[0], xs[1], xs[2], oT, state, sl[:nseq], zero, heads, heads, dd, dd, segs, ends, cu_seqlens=cu, channel_decay=ldT, bonus=u), 20, 50),
+                flops=T * heads * (17.0 * 2 * dd + 4.0 * dd * dd), nbytes=T * n * 12.0, like=f"decayed_chunks retention {nseq} x {T // nseq}, 16 x 128 x 128")
+    width, rank = 1024, 32
+    xw, mu, before = [rnd(T, width) for _ in range(4)], t.f32(5, width), torch.zeros((16, width), dtype=torch.bfloat16, device=dev)
+    cu16, z16, sl16 = i32(list(range(0, T + 1, 1024))), torch.zeros(16, dtype=torch.int32, device=dev), torch.arange(16, dtype=torch.int32, device=dev)
+    seq = torch.arange(T, device=dev).div(1024, rounding_mode="floor").to(torch.int32)
+    add("token_mix", f"{T} x {width}, 5 blends", lambda: graph_time(lambda i: op("token_mix")(xw[i % 4], mu, before, z16, sl16, seq, cu16), 4), nbytes=T * width * 12.0, like="siluAndMul")
+    z, w2, w0 = [rnd(T, rank) for _ in range(4)], rnd(1024, rank), t.f32(1024)
+    add("low_rank_decay", f"{T} x {rank} -> 1024", lambda: graph_time(lambda i: op("low_rank_decay")(z[i % 4], w2, w0), 4), nbytes=T * (rank * 2 + 1024 * 4.0), like="siluAndMul")
+    y, gate, wn = [rnd(T, 1024) for _ in range(4)], [rnd(T, 1024) for _ in range(4)], rnd(1024)
+    add("gated_group_norm", f"{T} x 1024, 16 groups", lambda: graph_time(lambda i: op("gated_group_norm")(y[i % 4], gate[i % 4], 16, 1e-6, weight=wn), 8), nbytes=T * 1024 * 6.0, like="siluAndMul")
+    mixes, wr = rnd(4, 256, width), [rnd(4, 1024, width) for _ in range(16)]
+    add("head_linear", "256 rows, 4 x 1024 -> 1024", lambda: graph_time(lambda i: op("head_linear")(mixes.transpose(0, 1), wr[i % 16]), 16),
+        nbytes=4 * 1024 * 1024 * 2 + 256 * 4 * 2048 * 2, flops=2.0 * 256 * 4 * 1024 * 1024, like="linear decode")
+    # ---- experts
+    for tokens, w, ff, experts, top in ((T, 1024, 1536, 16, 2), (256, 1024, 1536, 16, 2), (T, 2048, 1536, 32, 4), (256, 2048, 1536, 32, 4)):
+        tag, n = f"{tokens} x {w}, top {top} of {experts} x {ff}", tokens * top
+        sets = 2 if tokens == T else 4
+        h, router = [rnd(tokens, w) for _ in range(sets)], rnd(experts, w)
+        gu, down = [rnd(experts, 2, ff, w) for _ in range(sets)], [rnd(experts, w, ff) for _ in range(sets)]
+        routing = [op("moe_route")(x, router, top) for x in h]
+        ys = [op("moe_gate_up")(h[i], gu[i], routing[i]) for i in range(sets)]
+        like = "linear" if tokens == T else "linear decode"
+        add("moe_route", tag, lambda: graph_time(lambda i: op("moe_route")(h[i % sets], router, top), 8), nbytes=tokens * w * 2.0 + n * 24, like="add_rms prefill" if tokens == T else "linear decode")
+        add("moe_gate_up", tag, lambda: graph_time(lambda i: op("moe_gate_up")(h[i % sets], gu[i % sets], routing[i % sets]), 8),
+            nbytes=experts * 2.0 * ff * w * 2 + tokens * w * 2.0 + n * ff * 2.0, flops=4.0 * n * ff * w, like=like)
+        add("moe_down", tag, lambda: graph_time(lambda i: op("moe_down")(ys[i % sets], down[i % sets], routing[i % sets]), 8),
+            nbytes=experts * float(ff) * w * 2 + n * ff * 2.0 + n * w * 2.0, flops=2.0 * n * ff * w, like=like)
+    # ---- around the sublayers
+    sq = [rnd(T, 3072) for _ in range(4)]
+    add("squared_relu", f"{T} x 3072", lambda: graph_time(lambda i: op("squared_relu")(sq[i % 4]), 8), nbytes=T * 3072 * 4.0, like="siluAndMul")
+    for rows, n, parts, like in ((512, 4096, 1, "add_rms"), (T, 1024, 1, "add_rms prefill"), (T, 1024, 2, "add_rms prefill")):
+        sets = 24 if rows == 512 else 4
+        res, yy, wa, wb = [t.f32(rows, n) for _ in range(sets)], [rnd(rows * parts, n) for _ in range(sets)], rnd(n), rnd(n)
+        add("add_norm_norm", f"{rows} x {n}, {parts} part{'s' if parts > 1 else ''}", lambda: graph_time(lambda i: op("add_norm_norm")(res[i % sets], yy[i % sets], wa, wb, 1e-6), 24 if rows == 512 else 8),
+            nbytes=rows * n * (10.0 + 2 * parts), like=like)
+
+
+def kernel_table(dev, seed=0, only="", design="nepulix"):
+    """The rows of a design's kernels behind those of the models it is measured against."""
+    t = KernelTable(dev, seed, only)
+    qwen3_kernels(t)
+    if design == "sozarax":
+        decayed_kernels(t, "retention", 16, 16, 128, 128, True)
+        sozarax_kernels(t)
+    else:
+        nepulix_kernels(t)
+    return t.rows
