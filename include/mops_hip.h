@@ -580,8 +580,8 @@ int mops_hip_biased_prefill(const mops_hip_biased_attention* a, const int32_t* t
 
 /*
  * Mixture of experts (csrc/moe.hip).  moe_route: logits = router [experts, width] h in float32; chosen, score [tokens * top] =
- * the experts with the largest logits and the sigmoids of these; rank [tokens * top] is scratch, counts [experts] must be zeros
- * and receives the choices per expert; rows [tokens * top] lists the choices (token * top + place) ordered by expert, tiles
+ * the experts with the largest logits and the sigmoids of these; rank [tokens * top] and counts [moe_route_workgroups(tokens),
+ * experts] are scratch; rows [tokens * top] lists the choices (token * top + place) ordered by expert, tiles
  * [1 + 3 * moe_max_tiles] = number of blocks, then (expert, first row, rows) of each.  block_rows: 32, or 128 (bf16).
  * moe_gate_up: w [experts][2 * up_at][width], gate rows from 0, up rows from up_at on; y [tokens * top rows in the order of
  * `rows`], y = silu(score W_gate h) * (score W_up h).  moe_down: w [experts][width][depth], depth >= ff, the columns behind ff
@@ -594,6 +594,7 @@ typedef struct {
   int dtype;
 } mops_hip_moe;
 int64_t mops_hip_moe_max_tiles(int64_t tokens, int64_t experts, int64_t top, int64_t block_rows);
+int64_t mops_hip_moe_route_workgroups(int64_t tokens);
 int mops_hip_moe_route(const void* h, int64_t h_row_stride, const void* router, int32_t* chosen, int32_t* rank, int32_t* counts,
                        const mops_hip_moe* m, void* stream);
 int mops_hip_moe_gate_up(const void* h, int64_t h_row_stride, const void* w, int64_t up_at, void* y, int64_t y_row_stride,

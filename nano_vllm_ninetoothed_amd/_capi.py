@@ -136,6 +136,7 @@ SIGNATURES = {
     "mops_hip_biased_decode": (c_int, [POINTER(BiasedAttention), c_void_p, c_int64, c_void_p]),
     "mops_hip_biased_prefill": (c_int, [POINTER(BiasedAttention), c_void_p, c_int64, c_void_p]),
     "mops_hip_moe_max_tiles": (c_int64, [c_int64] * 4),
+    "mops_hip_moe_route_workgroups": (c_int64, [c_int64]),
     "mops_hip_moe_route": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p, POINTER(Moe), c_void_p]),
     "mops_hip_moe_gate_up": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, POINTER(Moe), c_void_p]),
     "mops_hip_moe_down": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, POINTER(Moe), c_void_p]),

@@ -8,7 +8,7 @@
 //
 // The products are grouped: a workgroup takes a block of rows of one expert and some of its outputs.  Nothing comes back to the
 // host: the grids are sized for the largest possible number of blocks, and workgroups without one leave.  The order of an
-// expert's rows depends on the order in which workgroups count them; no row's result depends on it.
+// expert's rows depends on the order in which the waves of a workgroup count them; no row's result depends on it.
 //   large blocks   128 rows x 128 weight rows x 64 deep tiles through LDS, the next tile in flight into registers
 //   small blocks   32 rows: weights are read once, straight into registers; the four waves split the depth
 //   float          plain tiles on vector units
@@ -21,145 +21,202 @@ constexpr int kMaxExperts = 1024;
 struct RouteArgs {
   const void *h, *router;
   int64_t h_stride;
-  int tokens, width, experts, top;
-  int32_t *chosen, *rank, *counts;     // [tokens * top], [tokens * top], [experts] (zeroed)
+  int tokens, width, experts, top, per_wg;      // per_wg: tokens of a workgroup, a multiple of 16
+  int32_t *chosen, *rank, *counts;     // [tokens * top], [tokens * top], [workgroups][experts]
   float* score;                        // [tokens * top]
 };
 
-// Counts this workgroup's choices per expert and ranks them among all: one addition to the global counter per expert.
-template <int THREADS>
-__device__ __forceinline__ void rank_choices(const RouteArgs& a, int* hist, int* base, int t0, int n_tokens) {
+static int tokens_per_workgroup(int64_t tokens) { return tokens <= 2048 ? 16 : 64; }
+
+// Counts this workgroup's choices per expert and ranks them among each other.
+__device__ __forceinline__ void rank_choices(const RouteArgs& a, int* hist) {
+  const int t0 = blockIdx.x * a.per_wg, n_tokens = a.tokens - t0 < a.per_wg ? a.tokens - t0 : a.per_wg;
   __syncthreads();
-  for (int e = threadIdx.x; e < a.experts; e += THREADS) hist[e] = 0;
+  for (int e = threadIdx.x; e < a.experts; e += 256) hist[e] = 0;
   __syncthreads();
   const int64_t i0 = (int64_t)t0 * a.top;
-  const int n = n_tokens * a.top;
-  for (int i = threadIdx.x; i < n; i += THREADS) a.rank[i0 + i] = atomicAdd(&hist[a.chosen[i0 + i]], 1);
+  for (int i = threadIdx.x; i < n_tokens * a.top; i += 256) a.rank[i0 + i] = atomicAdd(&hist[a.chosen[i0 + i]], 1);
   __syncthreads();
-  for (int e = threadIdx.x; e < a.experts; e += THREADS) base[e] = hist[e] ? atomicAdd(&a.counts[e], hist[e]) : 0;
-  __syncthreads();
-  for (int i = threadIdx.x; i < n; i += THREADS) a.rank[i0 + i] += base[a.chosen[i0 + i]];
+  for (int e = threadIdx.x; e < a.experts; e += 256) a.counts[(int64_t)blockIdx.x * a.experts + e] = hist[e];
 }
 
-// Logits of 16 tokens per wave on the matrix cores: bf16 operands, exact products, float32 sums.  ET: tiles of 16 experts.
+// 16 tokens at a time on the matrix cores: bf16 operands, exact products, float32 sums; the four waves split the depth.
+// ET: tiles of 16 experts.
+constexpr int kRouteTokens = 16;
+
 template <int ET>
 __global__ __launch_bounds__(256) void moe_route_mfma_kernel(const RouteArgs a, bool aligned) {
   constexpr int kPitch = ET * 16 + 1;
-  __shared__ float logits[4][16][kPitch];
-  __shared__ int hist[ET * 16], base[ET * 16];
+  constexpr int kAhead = ET <= 2 ? 4 : 2;      // steps whose loads are issued together
+  __shared__ float logits[4][kRouteTokens][kPitch];
+  __shared__ int hist[ET * 16];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, n = lane & 15, jj = lane >> 4;
-  const int t0 = blockIdx.x * 64, t = t0 + wave * 16 + n;
-  const uint16_t* h = (const uint16_t*)a.h + (int64_t)(t < a.tokens ? t : a.tokens - 1) * a.h_stride;
-  f32x4 acc[ET];
+  const uint16_t* w[ET];
+  bool w_ok[ET];
 #pragma unroll
-  for (int i = 0; i < ET; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-  for (int k0 = 0; k0 < a.width; k0 += 32) {
-    const bf16x8 b = __builtin_bit_cast(bf16x8, load8_guarded(h, k0 + 8 * jj, a.width, aligned));
-#pragma unroll
-    for (int i = 0; i < ET; ++i) {
-      const int e = 16 * i + n;
-      const u32x4 w = e < a.experts ? load8_guarded((const uint16_t*)a.router + (int64_t)e * a.width, k0 + 8 * jj, a.width, aligned) : u32x4{0u, 0u, 0u, 0u};
-      acc[i] = mfma16(__builtin_bit_cast(bf16x8, w), b, acc[i]);
-    }
+  for (int i = 0; i < ET; ++i) {
+    w_ok[i] = 16 * i + n < a.experts;
+    w[i] = (const uint16_t*)a.router + (int64_t)(w_ok[i] ? 16 * i + n : 0) * a.width;
   }
+  for (int t0 = blockIdx.x * a.per_wg; t0 < a.tokens && t0 < (int)(blockIdx.x + 1) * a.per_wg; t0 += kRouteTokens) {
+    const int t = t0 + n;
+    const uint16_t* h = (const uint16_t*)a.h + (int64_t)(t < a.tokens ? t : a.tokens - 1) * a.h_stride;
+    f32x4 acc[ET];
 #pragma unroll
-  for (int i = 0; i < ET; ++i)
+    for (int i = 0; i < ET; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int k0 = 32 * kAhead * wave; k0 < a.width; k0 += 128 * kAhead) {
+      u32x4 x[kAhead], y[kAhead][ET];
 #pragma unroll
-    for (int e = 0; e < 4; ++e) logits[wave][n][16 * i + 4 * jj + e] = acc[i][e];
-  __syncthreads();
-  // four lanes per token: lane jj looks at the experts jj, jj + 4, ...
-  float* mine = logits[wave][n];
-  for (int s = 0; s < a.top; ++s) {
-    float best = -INFINITY;
-    int who = 0x7fffffff;
-    for (int e = jj; e < a.experts; e += 4)
-      if (mine[e] > best) {
-        best = mine[e];
-        who = e;
+      for (int s = 0; s < kAhead; ++s) {
+        const int k = k0 + 32 * s + 8 * jj;
+        if (aligned) {
+          const bool ok = k < a.width;
+          x[s] = load16(h + (ok ? k : 0));
+          if (!ok) x[s] = u32x4{0u, 0u, 0u, 0u};
+#pragma unroll
+          for (int i = 0; i < ET; ++i) {
+            y[s][i] = load16(w[i] + (ok ? k : 0));
+            if (!ok) y[s][i] = u32x4{0u, 0u, 0u, 0u};
+          }
+        } else {
+          x[s] = load8_guarded(h, k, a.width, false);
+#pragma unroll
+          for (int i = 0; i < ET; ++i) y[s][i] = load8_guarded(w[i], k, a.width, false);
+        }
       }
 #pragma unroll
-    for (int off = 16; off < 64; off <<= 1) {
-      const float ob = __shfl_xor(best, off, kWave);
-      const int ow = __shfl_xor(who, off, kWave);
-      if (ob > best || (ob == best && ow < who)) {
-        best = ob;
-        who = ow;
+      for (int s = 0; s < kAhead; ++s)
+#pragma unroll
+        for (int i = 0; i < ET; ++i) acc[i] = mfma16(__builtin_bit_cast(bf16x8, y[s][i]), __builtin_bit_cast(bf16x8, x[s]), acc[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < ET; ++i)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) logits[wave][n][16 * i + 4 * jj + e] = acc[i][e];
+    __syncthreads();
+    for (int i = threadIdx.x; i < kRouteTokens * ET * 16; i += 256) {
+      const int r = i / (ET * 16), e = i % (ET * 16);
+      logits[0][r][e] = (logits[0][r][e] + logits[1][r][e]) + (logits[2][r][e] + logits[3][r][e]);
+    }
+    __syncthreads();
+    // sixteen lanes per token: lane x looks at the experts x, x + 16, ...
+    const int mt = threadIdx.x >> 4, x = threadIdx.x & 15, token = t0 + mt;
+    float* mine = logits[0][mt];
+    for (int s = 0; s < a.top; ++s) {
+      float best = -INFINITY;
+      int who = 0x7fffffff;
+#pragma unroll
+      for (int i = 0; i < ET; ++i) {
+        const int e = x + 16 * i;
+        if (e < a.experts && mine[e] > best) {
+          best = mine[e];
+          who = e;
+        }
+      }
+#pragma unroll
+      for (int off = 1; off < 16; off <<= 1) {
+        const float ob = __shfl_xor(best, off, kWave);
+        const int ow = __shfl_xor(who, off, kWave);
+        if (ob > best || (ob == best && ow < who)) {
+          best = ob;
+          who = ow;
+        }
+      }
+      if (who >= a.experts) {      // logits that compare with nothing: any expert that is left over, and a score that shows it
+        who = s;
+        best = NAN;
+      }
+      if ((who & 15) == x) mine[who] = -INFINITY;
+      if (x == 0 && token < a.tokens) {
+        a.chosen[(int64_t)token * a.top + s] = who;
+        a.score[(int64_t)token * a.top + s] = 1.0f / (1.0f + expf(-best));
       }
     }
-    if (who >= a.experts) {      // logits that compare with nothing: any expert that is left over, and a score that shows it
-      who = s;
-      best = NAN;
-    }
-    if ((who & 3) == jj) mine[who] = -INFINITY;
-    if (jj == 0 && t < a.tokens) {
-      a.chosen[(int64_t)t * a.top + s] = who;
-      a.score[(int64_t)t * a.top + s] = 1.0f / (1.0f + expf(-best));
-    }
+    __syncthreads();
   }
-  rank_choices<256>(a, hist, base, t0, a.tokens - t0 < 64 ? a.tokens - t0 : 64);
+  rank_choices(a, hist);
 }
 
-// One token per workgroup, any size.
+// A wave per token, any size.
 template <typename T>
-__global__ __launch_bounds__(64) void moe_route_kernel(const RouteArgs a) {
-  __shared__ float logits[kMaxExperts];
-  __shared__ int hist[kMaxExperts], base[kMaxExperts];
-  const int t = blockIdx.x, lane = threadIdx.x;
-  const T* h = (const T*)a.h + (int64_t)t * a.h_stride;
-  for (int e = 0; e < a.experts; ++e) {
-    const T* w = (const T*)a.router + (int64_t)e * a.width;
-    float dot = 0.f;
-    for (int k = lane; k < a.width; k += kWave) dot += to_f32(h[k]) * to_f32(w[k]);
-    dot = group_sum<kWave>(dot);
-    if (lane == 0) logits[e] = dot;
-  }
-  __syncthreads();
-  for (int s = 0; s < a.top; ++s) {
-    float best = -INFINITY;
-    int who = 0x7fffffff;
-    for (int e = lane; e < a.experts; e += kWave)
-      if (logits[e] > best) {
-        best = logits[e];
-        who = e;
-      }
+__global__ __launch_bounds__(256) void moe_route_kernel(const RouteArgs a) {
+  __shared__ float logits[4][kMaxExperts];
+  __shared__ int hist[kMaxExperts];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  float* mine = logits[wave];
+  for (int i = wave; i < a.per_wg; i += 4) {      // as often for every wave
+    const int t = blockIdx.x * a.per_wg + i;
+    const T* h = (const T*)a.h + (int64_t)(t < a.tokens ? t : a.tokens - 1) * a.h_stride;
+    for (int e = 0; e < a.experts; ++e) {
+      const T* w = (const T*)a.router + (int64_t)e * a.width;
+      float dot = 0.f;
+      for (int k = lane; k < a.width; k += kWave) dot += to_f32(h[k]) * to_f32(w[k]);
+      dot = group_sum<kWave>(dot);
+      if (lane == 0) mine[e] = dot;
+    }
+    __syncthreads();
+    for (int s = 0; s < a.top; ++s) {
+      float best = -INFINITY;
+      int who = 0x7fffffff;
+      for (int e = lane; e < a.experts; e += kWave)
+        if (mine[e] > best) {
+          best = mine[e];
+          who = e;
+        }
 #pragma unroll
-    for (int off = 1; off < 64; off <<= 1) {
-      const float ob = __shfl_xor(best, off, kWave);
-      const int ow = __shfl_xor(who, off, kWave);
-      if (ob > best || (ob == best && ow < who)) {
-        best = ob;
-        who = ow;
+      for (int off = 1; off < 64; off <<= 1) {
+        const float ob = __shfl_xor(best, off, kWave);
+        const int ow = __shfl_xor(who, off, kWave);
+        if (ob > best || (ob == best && ow < who)) {
+          best = ob;
+          who = ow;
+        }
       }
-    }
-    if (who >= a.experts) {
-      who = s;
-      best = NAN;
-    }
-    __syncthreads();
-    if (lane == 0) {
-      logits[who] = -INFINITY;
-      a.chosen[(int64_t)t * a.top + s] = who;
-      a.score[(int64_t)t * a.top + s] = 1.0f / (1.0f + expf(-best));
+      if (who >= a.experts) {
+        who = s;
+        best = NAN;
+      }
+      if ((who & 63) == lane) mine[who] = -INFINITY;      // the lane that looks at this expert
+      if (lane == 0 && t < a.tokens) {
+        a.chosen[(int64_t)t * a.top + s] = who;
+        a.score[(int64_t)t * a.top + s] = 1.0f / (1.0f + expf(-best));
+      }
     }
     __syncthreads();
   }
-  rank_choices<64>(a, hist, base, t, 1);
+  rank_choices(a, hist);
 }
 
-// rows[] and tiles[].  tiles: [0] their number, then {expert, first row, rows} each.
-__global__ __launch_bounds__(256) void moe_place_kernel(const int32_t* __restrict__ chosen, const int32_t* __restrict__ rank,
-                                                        const int32_t* __restrict__ counts, int32_t* __restrict__ rows,
-                                                        int32_t* __restrict__ tiles, int choices, int experts, int block_rows) {
+// rows[] and tiles[]; a workgroup for each one of the route.  tiles: [0] their number, then {expert, first row, rows} each.
+__global__ __launch_bounds__(256) void moe_place_kernel(const RouteArgs a, int32_t* __restrict__ rows, int32_t* __restrict__ tiles, int block_rows) {
+  __shared__ int total[kMaxExperts], earlier[kMaxExperts];
   __shared__ int begin[kMaxExperts + 1], first_tile[kMaxExperts + 1];
   __shared__ int wave_rows[4], wave_tiles[4];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  for (int e = tid; e < kMaxExperts; e += 256) total[e] = earlier[e] = 0;
+  __syncthreads();
+  {
+    // threads over (expert, part of the workgroups)
+    const int across = a.experts < 256 ? a.experts : 256, parts = 256 / across;
+    if (tid < across * parts)
+      for (int e = tid % across; e < a.experts; e += across) {
+        int all = 0, front = 0;
+        for (int w = tid / across; w < (int)gridDim.x; w += parts) {
+          const int c = a.counts[(int64_t)w * a.experts + e];
+          all += c;
+          front += w < (int)blockIdx.x ? c : 0;
+        }
+        atomicAdd(&total[e], all);
+        atomicAdd(&earlier[e], front);
+      }
+  }
+  __syncthreads();
   {
     // a thread owns four consecutive experts
     int c[4], r = 0, n = 0;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const int e = 4 * tid + i;
-      c[i] = e < experts ? counts[e] : 0;
+      c[i] = total[4 * tid + i];
       r += c[i];
       n += (c[i] + block_rows - 1) / block_rows;
     }
@@ -185,9 +242,8 @@ __global__ __launch_bounds__(256) void moe_place_kernel(const int32_t* __restric
     }
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const int e = 4 * tid + i;
-      begin[e] = r;
-      first_tile[e] = n;
+      begin[4 * tid + i] = r;
+      first_tile[4 * tid + i] = n;
       r += c[i];
       n += (c[i] + block_rows - 1) / block_rows;
     }
@@ -197,11 +253,14 @@ __global__ __launch_bounds__(256) void moe_place_kernel(const int32_t* __restric
     }
   }
   __syncthreads();
-  const int i = blockIdx.x * 256 + tid;
-  if (i < choices) rows[begin[chosen[i]] + rank[i]] = i;
+  const int t0 = blockIdx.x * a.per_wg, n_tokens = a.tokens - t0 < a.per_wg ? a.tokens - t0 : a.per_wg;
+  for (int i = tid; i < n_tokens * a.top; i += 256) {
+    const int choice = t0 * a.top + i, e = a.chosen[choice];
+    rows[begin[e] + earlier[e] + a.rank[choice]] = choice;
+  }
   if (blockIdx.x == 0) {
     if (tid == 0) tiles[0] = first_tile[kMaxExperts];
-    for (int e = tid; e < experts; e += 256)
+    for (int e = tid; e < a.experts; e += 256)
       for (int r = begin[e], k = first_tile[e]; r < begin[e + 1]; r += block_rows, ++k) {
         tiles[1 + 3 * k] = e;
         tiles[2 + 3 * k] = r;
@@ -223,6 +282,15 @@ struct GroupedArgs {
   int top, blocks;          // blocks of outputs in the grid
 };
 
+// This workgroup's tile and block of outputs.  Consecutive workgroups go to different XCDs: each XCD gets a contiguous run of
+// tiles with all their outputs, so that the rows of a tile and the weights of an expert meet in one L2.
+__device__ __forceinline__ bool grouped_item(const GroupedArgs& a, int& tile, int& block) {
+  const int n = a.tiles[0], per = (n + 7) / 8, i = blockIdx.x / 8;
+  tile = (blockIdx.x % 8) * per + i / a.blocks;
+  block = i % a.blocks;
+  return i / a.blocks < per && tile < n;
+}
+
 // ---------------------------------------------------------------------------------------------------- large blocks
 constexpr int kGM = 128, kGK = 64, kGPitch = kGK + 8, kGTile = 128 * kGPitch;
 
@@ -230,8 +298,8 @@ template <bool GATED, bool ALIGNED>
 __global__ __launch_bounds__(256, 2) void moe_grouped_large_kernel(const GroupedArgs a) {
   extern __shared__ __align__(16) unsigned char smem[];
   uint16_t* const lds = reinterpret_cast<uint16_t*>(smem);      // two buffers of [x tile | w tile]
-  const int tile = blockIdx.x / a.blocks, block = blockIdx.x % a.blocks;
-  if (tile >= a.tiles[0]) return;
+  int tile, block;
+  if (!grouped_item(a, tile, block)) return;
   const int e = a.tiles[1 + 3 * tile], row0 = a.tiles[2 + 3 * tile], count = a.tiles[3 + 3 * tile];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 31, hh = lane >> 5;
   const int wm = wave & 1, wn = wave >> 1;
@@ -241,39 +309,32 @@ __global__ __launch_bounds__(256, 2) void moe_grouped_large_kernel(const Grouped
   // pieces of 16 bytes: thread -> row tid / 8 + 32 j, depth 8 (tid % 8)
   const int prow = tid >> 3, pk = (tid & 7) * 8;
   const uint16_t *xp[4], *wp[4];
-  bool w_ok[4];
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
     const int r = prow + 32 * j;
     const int src = row0 + (r < count ? r : count - 1);
     xp[j] = (const uint16_t*)a.x + (int64_t)(GATED ? a.rows[src] / a.top : src) * a.x_stride;
     const int n = GATED ? (r < 64 ? n0 + r : n0 + r - 64) : n0 + r;
-    w_ok[j] = n < a.n;
-    wp[j] = w + (int64_t)((w_ok[j] ? n : 0) + (GATED && r >= 64 ? a.up_at : 0)) * a.depth;
+    wp[j] = w + (int64_t)((n < a.n ? n : 0) + (GATED && r >= 64 ? a.up_at : 0)) * a.depth;
   }
-  u32x4 xr[4], wr[4];
-  auto issue = [&](int k0) {
+  // Loads carry no condition: behind the depth they read the row's start, and the pieces become zeros on their way into LDS.
+  u32x4 xr[2][4], wr[2][4];
+  auto issue = [&](u32x4 (&x)[4], u32x4 (&y)[4], int k0) {
+    const int k = k0 + pk, at = k < a.depth ? k : 0;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
-      const int k = k0 + pk;
-      if (ALIGNED) {      // columns behind the depth are zeros on the weights' side; the other side reads something finite
-        const bool ok = k < a.depth;
-        xr[j] = load16(xp[j] + (ok ? k : 0));
-        wr[j] = load16(wp[j] + (ok ? k : 0));
-        if (!ok || !w_ok[j]) wr[j] = u32x4{0u, 0u, 0u, 0u};
-        if (!ok) xr[j] = u32x4{0u, 0u, 0u, 0u};
-      } else {
-        xr[j] = load8_guarded(xp[j], k, a.depth, false);
-        wr[j] = w_ok[j] ? load8_guarded(wp[j], k, a.depth, false) : u32x4{0u, 0u, 0u, 0u};
-      }
+      x[j] = ALIGNED ? load16(xp[j] + at) : load8_guarded(xp[j], k, a.depth, false);
+      y[j] = ALIGNED ? load16(wp[j] + at) : load8_guarded(wp[j], k, a.depth, false);
     }
   };
-  auto stash = [&](int buf) {
+  auto stash = [&](const u32x4 (&x)[4], const u32x4 (&y)[4], int buf, int k0) {
     uint16_t* d = lds + buf * 2 * kGTile + prow * kGPitch + pk;
+    const bool ok = k0 + pk < a.depth;
+    const u32x4 zero = {0u, 0u, 0u, 0u};
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
-      store16(d + 32 * j * kGPitch, xr[j]);
-      store16(d + kGTile + 32 * j * kGPitch, wr[j]);
+      store16(d + 32 * j * kGPitch, ok ? x[j] : zero);
+      store16(d + kGTile + 32 * j * kGPitch, ok ? y[j] : zero);
     }
   };
   f32x16 acc[2][2];      // [weight rows][tokens]
@@ -283,13 +344,7 @@ __global__ __launch_bounds__(256, 2) void moe_grouped_large_kernel(const Grouped
     for (int j = 0; j < 2; ++j)
 #pragma unroll
       for (int r = 0; r < 16; ++r) acc[i][j][r] = 0.f;
-  issue(0);
-  stash(0);
-  __syncthreads();
-  int buf = 0;
-  for (int k0 = 0; k0 < a.depth; k0 += kGK, buf ^= 1) {
-    const bool more = k0 + kGK < a.depth;
-    if (more) issue(k0 + kGK);
+  auto multiply = [&](int buf) {
     const uint16_t *tx = lds + buf * 2 * kGTile, *tw = tx + kGTile;
 #pragma unroll
     for (int kk = 0; kk < kGK / 16; ++kk) {
@@ -303,7 +358,22 @@ __global__ __launch_bounds__(256, 2) void moe_grouped_large_kernel(const Grouped
 #pragma unroll
         for (int j = 0; j < 2; ++j) acc[i][j] = mfma32(wf[i], xf[j], acc[i][j]);
     }
-    if (more) stash(buf ^ 1);
+  };
+  // a turn: two tiles, each with the loads of the tile two further on issued in front of its products
+  issue(xr[0], wr[0], 0);
+  issue(xr[1], wr[1], kGK);
+  stash(xr[0], wr[0], 0, 0);
+  __syncthreads();
+  for (int k0 = 0; k0 < a.depth; k0 += 2 * kGK) {
+    issue(xr[0], wr[0], k0 + 2 * kGK);
+    multiply(0);
+    if (k0 + kGK >= a.depth) break;
+    stash(xr[1], wr[1], 1, k0 + kGK);
+    __syncthreads();
+    issue(xr[1], wr[1], k0 + 3 * kGK);
+    multiply(1);
+    if (k0 + 2 * kGK >= a.depth) break;
+    stash(xr[0], wr[0], 0, k0 + 2 * kGK);
     __syncthreads();
   }
 #pragma unroll
@@ -335,85 +405,102 @@ __global__ __launch_bounds__(256, 2) void moe_grouped_large_kernel(const Grouped
 // ---------------------------------------------------------------------------------------------------- small blocks
 constexpr int kSM = 32;
 
-// GATED: 32 outputs, tile 0 gate rows and tile 1 up rows; else 64 outputs.
+// Four 16-row pieces of the weights: GATED two of gate rows and two of up rows (32 outputs), else 64 outputs; two pieces of 16 rows.
 template <bool GATED, bool ALIGNED>
 __global__ __launch_bounds__(256, 2) void moe_grouped_small_kernel(const GroupedArgs a) {
-  __shared__ __align__(16) float part[4][2][16][64];      // [wave][tile][accumulator][lane]
-  const int tile = blockIdx.x / a.blocks, block = blockIdx.x % a.blocks;
-  if (tile >= a.tiles[0]) return;
+  __shared__ __align__(16) f32x4 part[4][8][64];      // [wave][piece of the weights, piece of the rows][lane]
+  int tile, block;
+  if (!grouped_item(a, tile, block)) return;
   const int e = a.tiles[1 + 3 * tile], row0 = a.tiles[2 + 3 * tile], count = a.tiles[3 + 3 * tile];
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 31, hh = lane >> 5;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 15, jj = lane >> 4;
   const int n0 = block * (GATED ? 32 : 64);
-  const int src = row0 + (col < count ? col : count - 1);
-  const uint16_t* x = (const uint16_t*)a.x + (int64_t)(GATED ? a.rows[src] / a.top : src) * a.x_stride;
-  const uint16_t* w[2];
-  bool w_ok[2];
+  const uint16_t *x[2], *w[4];
 #pragma unroll
-  for (int i = 0; i < 2; ++i) {
-    const int n = GATED ? n0 + col : n0 + 32 * i + col;
-    w_ok[i] = n < a.n;
-    w[i] = (const uint16_t*)a.w + (int64_t)e * a.w_expert + (int64_t)((w_ok[i] ? n : 0) + (GATED && i ? a.up_at : 0)) * a.depth;
+  for (int j = 0; j < 2; ++j) {
+    const int r = 16 * j + col, src = row0 + (r < count ? r : count - 1);
+    x[j] = (const uint16_t*)a.x + (int64_t)(GATED ? a.rows[src] / a.top : src) * a.x_stride;
   }
-  f32x16 acc[2];
 #pragma unroll
-  for (int i = 0; i < 2; ++i)
+  for (int i = 0; i < 4; ++i) {
+    const int n = n0 + 16 * (GATED ? i & 1 : i) + col;      // outputs behind the last are row 0 again and never stored
+    w[i] = (const uint16_t*)a.w + (int64_t)e * a.w_expert + (int64_t)((n < a.n ? n : 0) + (GATED && i >= 2 ? a.up_at : 0)) * a.depth;
+  }
+  f32x4 acc[4][2];
 #pragma unroll
-    for (int r = 0; r < 16; ++r) acc[i][r] = 0.f;
-  for (int k0 = 64 * wave; k0 < a.depth; k0 += 256) {
-    u32x4 xr[4], wr[2][4];
+  for (int i = 0; i < 4; ++i)
 #pragma unroll
-    for (int kk = 0; kk < 4; ++kk) {
-      const int k = k0 + 16 * kk + 8 * hh;
+    for (int j = 0; j < 2; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+  // a wave takes every fourth piece of 64 of the depth; the next piece is in flight while this one is used
+  u32x4 xr[2][2][2], wr[2][2][4];
+  auto fetch = [&](int buf, int k0) {
+#pragma unroll
+    for (int s = 0; s < 2; ++s) {
+      const int k = k0 + 32 * s + 8 * jj;
       if (ALIGNED) {
         const bool ok = k < a.depth;
-        xr[kk] = load16(x + (ok ? k : 0));
-        if (!ok) xr[kk] = u32x4{0u, 0u, 0u, 0u};
 #pragma unroll
-        for (int i = 0; i < 2; ++i) {
-          wr[i][kk] = load16_stream(w[i] + (ok ? k : 0));
-          if (!ok) wr[i][kk] = u32x4{0u, 0u, 0u, 0u};
+        for (int i = 0; i < 4; ++i) wr[buf][s][i] = load16_stream(w[i] + (ok ? k : 0));
+#pragma unroll
+        for (int j = 0; j < 2; ++j) {
+          xr[buf][s][j] = load16(x[j] + (ok ? k : 0));
+          if (!ok) xr[buf][s][j] = u32x4{0u, 0u, 0u, 0u};
+        }
+        if (!ok) {
+#pragma unroll
+          for (int i = 0; i < 4; ++i) wr[buf][s][i] = u32x4{0u, 0u, 0u, 0u};
         }
       } else {
-        xr[kk] = load8_guarded(x, k, a.depth, false);
 #pragma unroll
-        for (int i = 0; i < 2; ++i) wr[i][kk] = load8_guarded(w[i], k, a.depth, false);
+        for (int i = 0; i < 4; ++i) wr[buf][s][i] = load8_guarded(w[i], k, a.depth, false);
+#pragma unroll
+        for (int j = 0; j < 2; ++j) xr[buf][s][j] = load8_guarded(x[j], k, a.depth, false);
       }
     }
+  };
+  auto use = [&](int buf) {
 #pragma unroll
-    for (int kk = 0; kk < 4; ++kk)
+    for (int s = 0; s < 2; ++s)
 #pragma unroll
-      for (int i = 0; i < 2; ++i) acc[i] = mfma32(__builtin_bit_cast(bf16x8, wr[i][kk]), __builtin_bit_cast(bf16x8, xr[kk]), acc[i]);
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 2; ++j) acc[i][j] = mfma16(__builtin_bit_cast(bf16x8, wr[buf][s][i]), __builtin_bit_cast(bf16x8, xr[buf][s][j]), acc[i][j]);
+  };
+  int k0 = 64 * wave;
+  if (k0 < a.depth) fetch(0, k0);
+  while (k0 < a.depth) {      // two pieces a turn: the buffers are registers
+    if (k0 + 256 < a.depth) fetch(1, k0 + 256);
+    use(0);
+    k0 += 256;
+    if (k0 >= a.depth) break;
+    if (k0 + 256 < a.depth) fetch(0, k0 + 256);
+    use(1);
+    k0 += 256;
   }
 #pragma unroll
-  for (int i = 0; i < 2; ++i)
+  for (int i = 0; i < 4; ++i)
 #pragma unroll
-    for (int r = 0; r < 16; ++r) part[wave][i][r][lane] = acc[i][r];
+    for (int j = 0; j < 2; ++j) part[wave][2 * i + j][lane] = acc[i][j];
   __syncthreads();
-  // wave q4 finishes accumulators 4 q4 .. 4 q4 + 3 of both tiles
-  float v[2][4];
-#pragma unroll
-  for (int i = 0; i < 2; ++i)
-#pragma unroll
-    for (int x4 = 0; x4 < 4; ++x4) {
-      const int r = 4 * wave + x4;
-      v[i][x4] = (part[0][i][r][lane] + part[1][i][r][lane]) + (part[2][i][r][lane] + part[3][i][r][lane]);
-    }
-  if (col >= count) return;
-  const int choice = a.rows[row0 + col];
-  uint16_t* o = (uint16_t*)a.out + (int64_t)(GATED ? row0 + col : choice) * a.out_stride;
+  // wave (i, j): rows 16 j .., outputs of the pieces i (and i + 2)
+  const int i = wave >> 1, j = wave & 1, r = 16 * j + col;
+  auto total = [&](int piece) { return (part[0][piece][lane] + part[1][piece][lane]) + (part[2][piece][lane] + part[3][piece][lane]); };
+  const f32x4 v0 = total(2 * i + j), v1 = total(2 * (i + 2) + j);
+  if (r >= count) return;
+  const int choice = a.rows[row0 + r];
+  uint16_t* o = (uint16_t*)a.out + (int64_t)(GATED ? row0 + r : choice) * a.out_stride;
   const float s = GATED ? a.score[choice] : 1.f;
 #pragma unroll
-  for (int i = 0; i < (GATED ? 1 : 2); ++i) {
-    const int n = n0 + 32 * i + 8 * wave + 4 * hh;
+  for (int half = 0; half < (GATED ? 1 : 2); ++half) {
+    const int n = n0 + 16 * (i + 2 * half) + 4 * jj;
     float y[4];
 #pragma unroll
-    for (int x4 = 0; x4 < 4; ++x4) y[x4] = GATED ? silu_for<bf16_t>(s * v[0][x4]) * (s * v[1][x4]) : v[i][x4];
+    for (int q = 0; q < 4; ++q) y[q] = GATED ? silu_for<bf16_t>(s * v0[q]) * (s * v1[q]) : (half ? v1[q] : v0[q]);
     if (ALIGNED && n + 4 <= a.n) {
       *reinterpret_cast<u32x2*>(o + n) = u32x2{pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3])};
     } else {
 #pragma unroll
-      for (int x4 = 0; x4 < 4; ++x4)
-        if (n + x4 < a.n) o[n + x4] = (uint16_t)f32_to_bf16_bits(y[x4]);
+      for (int q = 0; q < 4; ++q)
+        if (n + q < a.n) o[n + q] = (uint16_t)f32_to_bf16_bits(y[q]);
     }
   }
 }
@@ -423,8 +510,8 @@ __global__ __launch_bounds__(256, 2) void moe_grouped_small_kernel(const Grouped
 template <bool GATED>
 __global__ __launch_bounds__(256) void moe_grouped_f32_kernel(const GroupedArgs a) {
   __shared__ float tx[kSM][33], tw[GATED ? 2 : 1][64][33];
-  const int tile = blockIdx.x / a.blocks, block = blockIdx.x % a.blocks;
-  if (tile >= a.tiles[0]) return;
+  int tile, block;
+  if (!grouped_item(a, tile, block)) return;
   const int e = a.tiles[1 + 3 * tile], row0 = a.tiles[2 + 3 * tile], count = a.tiles[3 + 3 * tile];
   const int tid = threadIdx.x, n_loc = tid & 63, r0 = tid >> 6;
   const int n0 = block * 64;
@@ -470,8 +557,9 @@ static int launch_grouped(GroupedArgs a, int dtype, int64_t block_rows, int64_t 
   const int64_t tiles = choices / block_rows + (experts < choices ? experts : choices);
   const int per = dtype == MOPS_HIP_F32 ? 64 : (block_rows == kSM ? (GATED ? 32 : 64) : (GATED ? 64 : 128));
   a.blocks = (a.n + per - 1) / per;
-  if (tiles * a.blocks > 0x7fffffffLL) return MOPS_HIP_EUNSUPPORTED;
-  const dim3 grid((unsigned)(tiles * a.blocks)), block(256);
+  const int64_t grid_size = (tiles + 7) / 8 * 8 * a.blocks;
+  if (grid_size > 0x7fffffffLL) return MOPS_HIP_EUNSUPPORTED;
+  const dim3 grid((unsigned)grid_size), block(256);
   const bool aligned = a.depth % 8 == 0 && a.x_stride % 8 == 0 && a.out_stride % 4 == 0 && a.w_expert % 8 == 0 && aligned16(a.x) && aligned16(a.w) &&
                        aligned16(a.out);
   if (dtype == MOPS_HIP_F32) {
@@ -511,6 +599,12 @@ extern "C" int64_t mops_hip_moe_max_tiles(int64_t tokens, int64_t experts, int64
   return choices / block_rows + (experts < choices ? experts : choices);
 }
 
+extern "C" int64_t mops_hip_moe_route_workgroups(int64_t tokens) {
+  if (tokens < 0) return MOPS_HIP_EINVAL;
+  const int64_t per = mops::tokens_per_workgroup(tokens);
+  return (tokens + per - 1) / per;
+}
+
 extern "C" int mops_hip_moe_route(const void* h, int64_t h_row_stride, const void* router, int32_t* chosen, int32_t* rank, int32_t* counts,
                                   const mops_hip_moe* m, void* stream) {
   using namespace mops;
@@ -520,25 +614,23 @@ extern "C" int mops_hip_moe_route(const void* h, int64_t h_row_stride, const voi
   RouteArgs a;
   a.h = h; a.router = router; a.h_stride = h_row_stride;
   a.tokens = (int)m->tokens; a.width = (int)m->width; a.experts = (int)m->experts; a.top = (int)m->top;
-  a.chosen = chosen; a.rank = rank; a.counts = counts; a.score = m->score;
+  a.chosen = chosen; a.rank = rank; a.counts = counts; a.score = m->score; a.per_wg = tokens_per_workgroup(m->tokens);
+  const dim3 grid((unsigned)((m->tokens + a.per_wg - 1) / a.per_wg)), block(256);
   hipStream_t s = (hipStream_t)stream;
   if (m->dtype == MOPS_HIP_BF16 && m->experts <= 128) {
-    const dim3 grid((unsigned)((m->tokens + 63) / 64)), block(256);
     const bool aligned = m->width % 8 == 0 && h_row_stride % 8 == 0 && aligned16(h) && aligned16(router);
     if (m->experts <= 16) hipLaunchKernelGGL((moe_route_mfma_kernel<1>), grid, block, 0, s, a, aligned);
     else if (m->experts <= 32) hipLaunchKernelGGL((moe_route_mfma_kernel<2>), grid, block, 0, s, a, aligned);
     else if (m->experts <= 64) hipLaunchKernelGGL((moe_route_mfma_kernel<4>), grid, block, 0, s, a, aligned);
     else hipLaunchKernelGGL((moe_route_mfma_kernel<8>), grid, block, 0, s, a, aligned);
   } else if (m->dtype == MOPS_HIP_BF16) {
-    hipLaunchKernelGGL((moe_route_kernel<bf16_t>), dim3((unsigned)m->tokens), dim3(64), 0, s, a);
+    hipLaunchKernelGGL((moe_route_kernel<bf16_t>), grid, block, 0, s, a);
   } else {
-    hipLaunchKernelGGL((moe_route_kernel<float>), dim3((unsigned)m->tokens), dim3(64), 0, s, a);
+    hipLaunchKernelGGL((moe_route_kernel<float>), grid, block, 0, s, a);
   }
   int st = finish_launch();
   if (st != MOPS_HIP_OK) return st;
-  const int choices = (int)(m->tokens * m->top);
-  hipLaunchKernelGGL(moe_place_kernel, dim3((unsigned)((choices + 255) / 256)), dim3(256), 0, s, chosen, rank, counts, m->rows, m->tiles, choices,
-                     (int)m->experts, (int)m->block_rows);
+  hipLaunchKernelGGL(moe_place_kernel, grid, block, 0, s, a, m->rows, m->tiles, (int)m->block_rows);
   return finish_launch();
 }
 

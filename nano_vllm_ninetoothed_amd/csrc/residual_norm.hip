@@ -320,16 +320,17 @@ extern "C" int mops_hip_gated_group_norm(const void* y, int64_t y_row_stride, co
   if (rows == 0) return MOPS_HIP_OK;
   const int64_t n = groups * group_size;
   if (!y || !gate || !out || y_row_stride < n || gate_row_stride < n || out == gate) return MOPS_HIP_EINVAL;
-  const bool narrow = group_size <= 512;
-  const int64_t per_wg = narrow ? 16 : 4, wgs = (rows * groups + per_wg - 1) / per_wg;
-  if (wgs > 0x7fffffffLL) return MOPS_HIP_EUNSUPPORTED;
   const bool vec = group_size % 8 == 0 && y_row_stride % 8 == 0 && gate_row_stride % 8 == 0 && aligned16(y) && aligned16(gate) &&
                    aligned16(out) && (!weight || aligned16(weight));
+  const bool small = vec && group_size <= 64, narrow = group_size <= 512;      // eight lanes, a row of lanes, a wave per group
+  const int64_t per_wg = small ? 32 : (narrow ? 16 : 4), wgs = (rows * groups + per_wg - 1) / per_wg;
+  if (wgs > 0x7fffffffLL) return MOPS_HIP_EUNSUPPORTED;
   hipStream_t s = (hipStream_t)stream;
 #define MOPS_GGN(T, V, L, F) hipLaunchKernelGGL((gated_group_norm_kernel<T, V, L, F>), dim3((unsigned)wgs), dim3(256), 0, s, (const T*)y, \
                           y_row_stride, (const T*)gate, gate_row_stride, (const T*)weight, eps, (T*)out, rows, (int)groups, (int)group_size)
 #define MOPS_GGN2(T, V) do {                                    \
-    if (narrow) { if (gate_first) MOPS_GGN(T, V, 16, true); else MOPS_GGN(T, V, 16, false); }  \
+    if (V == 8 && small) { if (gate_first) MOPS_GGN(T, V, 8, true); else MOPS_GGN(T, V, 8, false); }  \
+    else if (narrow) { if (gate_first) MOPS_GGN(T, V, 16, true); else MOPS_GGN(T, V, 16, false); }  \
     else { if (gate_first) MOPS_GGN(T, V, 64, true); else MOPS_GGN(T, V, 64, false); }         \
   } while (0)
   if (dtype == MOPS_HIP_BF16) { if (vec) MOPS_GGN2(bf16_t, 8); else MOPS_GGN2(bf16_t, 1); }

@@ -61,17 +61,27 @@ __device__ __forceinline__ float tanh_fast(float v) {
 // Workgroup = 64 tokens x 256 channels, a wave takes 64 of the channels; tanh(z) in LDS, the rows of w2 straight from memory.
 __global__ __launch_bounds__(256) void low_rank_decay_mfma_kernel(const uint16_t* __restrict__ z, int64_t z_stride, const uint16_t* __restrict__ w2,
                                                                   const float* __restrict__ w0, float* __restrict__ out, int64_t tokens,
-                                                                  int channels, int rank, bool aligned, bool wide) {
+                                                                  int channels, int rank, bool aligned, bool z_aligned, bool wide) {
   extern __shared__ __align__(16) unsigned char smem[];
   uint16_t* const tile = reinterpret_cast<uint16_t*>(smem);
   const int ksteps = (rank + 31) / 32, pitch = ksteps * 32 + 8;
   const int64_t t0 = (int64_t)blockIdx.x * kDecayTokens;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, n = lane & 15, jj = lane >> 4;
   const int c0 = blockIdx.y * kDecayChannels + wave * 64;
-  for (int i = threadIdx.x; i < kDecayTokens * ksteps * 32; i += 256) {
-    const int r = i / (ksteps * 32), k = i % (ksteps * 32);
-    const float v = t0 + r < tokens && k < rank ? tanh_fast(bf16lo_to_f32(z[(t0 + r) * z_stride + k])) : 0.f;
-    tile[r * pitch + k] = (uint16_t)f32_to_bf16_bits(v);
+  auto weights = [&](int i, int ks) {
+    const int c = c0 + 16 * i + n;
+    return c < channels ? load8_guarded(w2 + (int64_t)c * rank, 32 * ks + 8 * jj, rank, aligned) : u32x4{0u, 0u, 0u, 0u};
+  };
+  u32x4 first[4];      // on their way while the tile is filled
+#pragma unroll
+  for (int i = 0; i < 4; ++i) first[i] = weights(i, 0);
+  for (int i = threadIdx.x; i < kDecayTokens * ksteps * 4; i += 256) {
+    const int r = i / (ksteps * 4), k = i % (ksteps * 4) * 8;
+    u32x4 w = {0u, 0u, 0u, 0u};
+    if (t0 + r < tokens) w = load8_guarded(z + (t0 + r) * z_stride, k, rank, z_aligned);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) w[e] = pack_bf16x2(tanh_fast(bf16lo_to_f32(w[e])), tanh_fast(bf16hi_to_f32(w[e])));
+    store16(tile + r * pitch + k, w);
   }
   __syncthreads();
   f32x4 acc[4][4];      // [channels][tokens]
@@ -85,8 +95,7 @@ __global__ __launch_bounds__(256) void low_rank_decay_mfma_kernel(const uint16_t
     for (int j = 0; j < 4; ++j) b[j] = tile_row(tile, pitch, 16 * j + n, 32 * ks + 8 * jj);
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const int c = c0 + 16 * i + n;
-      const u32x4 a = c < channels ? load8_guarded(w2 + (int64_t)c * rank, 32 * ks + 8 * jj, rank, aligned) : u32x4{0u, 0u, 0u, 0u};
+      const u32x4 a = ks == 0 ? first[i] : weights(i, ks);
 #pragma unroll
       for (int j = 0; j < 4; ++j) acc[i][j] = mfma16(__builtin_bit_cast(bf16x8, a), b[j], acc[i][j]);
     }
@@ -165,7 +174,7 @@ extern "C" int mops_hip_low_rank_decay(const void* z, int64_t z_row_stride, cons
     const dim3 grid((unsigned)((tokens + kDecayTokens - 1) / kDecayTokens), (unsigned)((channels + kDecayChannels - 1) / kDecayChannels));
     const size_t lds = kDecayTokens * ((rank + 31) / 32 * 32 + 8) * 2;
     hipLaunchKernelGGL(low_rank_decay_mfma_kernel, grid, dim3(256), lds, s, (const uint16_t*)z, z_row_stride, (const uint16_t*)w2, w0, out, tokens,
-                       (int)channels, (int)rank, rank % 8 == 0 && aligned16(w2), channels % 4 == 0 && aligned16(out));
+                       (int)channels, (int)rank, rank % 8 == 0 && aligned16(w2), z_row_stride % 8 == 0 && aligned16(z), channels % 4 == 0 && aligned16(out));
     return finish_launch();
   }
   const dim3 grid((unsigned)tokens, (unsigned)((channels + 255) / 256));

@@ -37,10 +37,9 @@ def moe_route(h: torch.Tensor, router: torch.Tensor, top: int, block_rows: int =
     lib = _capi.load()
     n = tokens * top
     tiles = lib.mops_hip_moe_max_tiles(tokens, experts, top, block_rows)
-    ints = torch.empty(3 * n + experts + 1 + 3 * tiles, dtype=torch.int32, device=h.device)
-    chosen, rank, rows, counts, tile_list = ints.split([n, n, n, experts, 1 + 3 * tiles])
+    sizes = [n, n, n, lib.mops_hip_moe_route_workgroups(tokens) * experts, 1 + 3 * tiles]
+    chosen, rank, rows, counts, tile_list = torch.empty(sum(sizes), dtype=torch.int32, device=h.device).split(sizes)
     score = torch.empty((tokens, top), dtype=torch.float32, device=h.device)
-    counts.zero_()
     m = _capi.Moe()
     m.rows, m.tiles, m.score = rows.data_ptr(), tile_list.data_ptr(), score.data_ptr()
     m.tokens, m.experts, m.top, m.width, m.ff, m.block_rows, m.dtype = tokens, experts, top, width, 1, block_rows, code

@@ -16,8 +16,8 @@ _round = None      # see sixteen_bit_products
 
 @contextlib.contextmanager
 def sixteen_bit_products(seed=0):
-    """Inside, every matrix product takes and gives values rounded to bfloat16 (to nearest for seed 0, else stochastically):
-    what rounding alone does to the result of a 16-bit run.  The router's product is exempt."""
+    """Inside, every matrix product takes and gives values rounded to bfloat16 (to nearest for seed 0, else stochastically), and so
+    are the values marked stored(): what rounding alone does to the result of a 16-bit run.  The router's product is exempt."""
     global _round
     g = torch.Generator().manual_seed(seed)
 
@@ -40,6 +40,11 @@ def product(x, w):
     if _round is None:
         return x @ w.T
     return _round(_round(x) @ w.T)
+
+
+def stored(x):
+    """An intermediate that a 16-bit run keeps in 16 bits."""
+    return x if _round is None else _round(x)
 
 
 def sigmoid(x):
@@ -96,7 +101,7 @@ def time_mixing(h, w, m, eps):
     r, k, v = (product(mix[n], w[n]).view(T, H, D) for n in "rkv")
     decay = channel_decay(mix["w"], w["w1"], w["w2"], w["w0"]).view(T, H, D)
     o, _ = channel_recurrence(r, k, v, decay, w["u"])
-    o = unit_rms(o, eps).reshape(T, H * D) * w["norm"]
+    o = unit_rms(stored(o), eps).reshape(T, H * D) * w["norm"]
     return product(o * silu(product(mix["g"], w["g"])), w["o"])
 
 
@@ -131,7 +136,7 @@ def attention(h, w, m, eps):
     k = norm(product(h, w["k"]), w["k.norm"], eps)
     t = m["q_temp"]
     q = q * query_temperature(torch.arange(T), t["coef"], t["every"])[:, None].to(q.dtype)
-    o = biased_attention(q.view(T, H, D), k.view(T, G, D), product(h, w["v"]).view(T, G, V), m["scale"], distance_slopes(H))
+    o = biased_attention(stored(q).view(T, H, D), stored(k).view(T, G, D), product(h, w["v"]).view(T, G, V), m["scale"], distance_slopes(H))
     return product(o.reshape(T, H * V), w["o"])
 
 

@@ -36,8 +36,8 @@ MADE = {
     # head sizes of large models; the last layers loop
     "large": config(256, 264, [wkv(2, 128, 64), attention(24, 1, 128, 128, 0.1, 64), wkv(4, 64, 32)],
                     [moe(136, 16, 4), dense(512), moe(64, 40, 1)], (1, 3, 2), 16.0),
-    # everything that can be one is one
-    "ones": config(64, 96, [wkv(1, 16, 1), attention(1, 1, 16, 8, 0.5, 1), wkv(1, 32, 8)], [moe(8, 1, 1), dense(1), moe(1, 2, 1)], (1, 2, 1), 1.0, eps=1e-3),
+    # nearly everything that can be one is one (a dense hidden size of one would make its normed result a matter of one sign)
+    "ones": config(64, 96, [wkv(1, 16, 1), attention(1, 1, 16, 8, 0.5, 1), wkv(1, 32, 8)], [moe(8, 1, 1), dense(24), moe(1, 2, 1)], (1, 2, 1), 1.0, eps=1e-3),
     # only recurrent layers, all looped, heads wider than the matrix-core kernels' smaller forms, every expert chosen
     "states": config(96, 120, [wkv(1, 200, 40), wkv(5, 20, 7)], [moe(24, 3, 3), dense(100)], (0, 2, 3), 0.5),
     # only attention, values wider than keys and keys wider than values, no loop at all
@@ -76,10 +76,15 @@ def tensor_shapes(name):
     return shapes
 
 
+CODE = 12      # channels that only the embedding writes and only the routers read, see random_weights
+
+
 def random_weights(name, seed=0):
-    """bfloat16 weights under the checkpoint's names.  Query norms are scaled up, so that attention is far from uniform; routers
-    too, so that rounding seldom changes a choice; decays reach from almost nothing lost to almost everything."""
-    g = torch.Generator().manual_seed(seed)
+    """bfloat16 weights under the checkpoint's names.  Query norms are scaled up, so that attention is far from uniform; decays reach
+    from almost nothing lost to almost everything; r and k lean towards each other, since a state's first outputs are divided by their
+    own size and r.k near zero would make that a matter of rounding.  For the same reason no choice of experts is a close call: the
+    routers read channels that no sublayer writes, where each token carries a code with a clear order of the experts."""
+    cfg, g = CONFIGS[name], torch.Generator().manual_seed(seed)
     out = {}
     for n, shape in tensor_shapes(name).items():
         t = torch.randn(shape, generator=g)
@@ -89,16 +94,41 @@ def random_weights(name, seed=0):
         elif leaf.startswith("mix.mu."):
             t = 0.5 + 0.4 * t
         elif leaf == "mix.u":
-            t = 0.7 * t
+            t = 1 + 0.5 * t
         elif leaf == "mix.q.norm":
             t = 2.5 * (1 + 0.3 * t)
         elif len(shape) == 1:
             t = 1 + 0.3 * t
+            if leaf in ("norm1b", "norm2b"):
+                t[:CODE] = 0
         elif n == "embed":
-            t = t / CONFIGS[name]["embedding"]["scale"]
+            t = t / cfg["embedding"]["scale"]
+        elif leaf == "mlp.router":
+            t = t * CODE ** -0.5
+            t[:, CODE:] = 0
         else:
-            t = t * shape[1] ** -0.5 * (6.0 if leaf == "mlp.router" else 1.0)
+            t = t * shape[1] ** -0.5
+            if leaf == "mix.k" and n.replace("mix.k", "mix.r") in tensor_shapes(name):
+                t = 0.6 * t      # and 0.8 of r, below
         out[n] = t.to(torch.bfloat16)
+    for n in [n for n in out if n.endswith("mix.r")]:
+        k = n[:-1] + "k"
+        out[k] = (out[k].float() + 0.8 * out[n].float()).to(torch.bfloat16)
+    routed = [(i, layer["mlp"]["router"]) for i, layer in enumerate(cfg["layers"]) if layer["mlp"] and layer["mlp"]["kind"] == "moe"]
+    open_, codes = torch.arange(cfg["vocab"]), out["embed"][:, :CODE].float()
+    for _ in range(400):
+        clear = torch.ones(len(open_), dtype=torch.bool)
+        for i, r in routed:
+            if r["top"] < r["experts"]:
+                z = (codes[open_] * out[f"l{i}.norm2"][:CODE].float()) @ out[f"l{i}.mlp.router"][:, :CODE].float().T
+                best = z.topk(r["top"] + 1, dim=-1).values
+                clear &= best[:, -2] - best[:, -1] > 0.1 * z.std(dim=-1)
+        open_ = open_[~clear]
+        if not len(open_):
+            break
+        codes[open_] = (torch.randn((len(open_), CODE), generator=g) / cfg["embedding"]["scale"]).to(torch.bfloat16).float()
+    assert not len(open_)
+    out["embed"][:, :CODE] = codes.to(torch.bfloat16)
     return out
 
 

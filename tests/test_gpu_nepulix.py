@@ -9,32 +9,23 @@ import numpy as np
 import pytest
 import torch
 
+import model_harness as H
 from nepulix_cases import CONFIGS, logit_error, random_tokens, random_weights, write_checkpoint
 from oracle import nepulix as O
 
 pytestmark = pytest.mark.gpu
 ROOT = Path(__file__).resolve().parent.parent
 DTYPES = [torch.float32, torch.bfloat16]
-LIMIT32 = 2e-5      # float32: per position, of the logits' root mean square
+check, feed = H.check, H.feed
 
 
-class Wanted:
-    """The oracle's logits, and per position what rounding alone does to a 16-bit run (the worst of three realisations, and
-    never less than the bulk of the positions shows)."""
+def Wanted(cfg, w, tokens):
+    return H.Wanted(O, cfg, w, tokens)
 
-    def __init__(self, cfg, w, tokens):
-        self.logits = O.forward(cfg, w, tokens)
-        errs = []
-        for seed in range(3):
-            with O.sixteen_bit_products(seed):
-                errs.append(logit_error(O.forward(cfg, w, tokens), self.logits))
-        e = torch.stack(errs).max(0).values
-        self.noise = torch.maximum(e, e.quantile(0.9))
 
-    def __getitem__(self, rows):
-        out = object.__new__(Wanted)
-        out.logits, out.noise = self.logits[rows], self.noise[rows]
-        return out
+def engine(gpu, cfg, *args, **kw):
+    from nano_vllm_ninetoothed_amd.models.nepulix import NepulixConfig
+    return H.engine(gpu, NepulixConfig.from_dict(cfg), *args, **kw)
 
 
 @pytest.fixture(scope="module")
@@ -52,31 +43,6 @@ def case():
             made[name] = (cfg, w, seqs, [Wanted(cfg, w, s) for s in seqs])
         return made[name]
     return get
-
-
-def engine(gpu, cfg, w, dtype, tokens=1024, block_size=32, slots=4, **kw):
-    from nano_vllm_ninetoothed_amd.engine import Engine
-    from nano_vllm_ninetoothed_amd.models.nepulix import NepulixConfig
-    from nano_vllm_ninetoothed_amd.weights import TensorWeights
-    return Engine(NepulixConfig.from_dict(cfg), weights=TensorWeights(w, dtype, gpu), num_blocks=-(-tokens // block_size), block_size=block_size,
-                  max_num_seqs=slots, max_model_len=tokens, device=str(gpu), **kw)
-
-
-def check(got, want, dtype, what):
-    e = logit_error(got, want.logits)
-    assert torch.isfinite(e).all(), what
-    e = e / (LIMIT32 if dtype == torch.float32 else 3 * want.noise)
-    worst, at, over = e.max().item(), int(e.argmax()), int((e > 1).sum())
-    assert worst <= 1.5 and over <= max(1, 0.02 * len(e)), f"{what}: {over} of {len(e)} positions over their limit, worst {worst:.3g} at {at}"
-
-
-def feed(eng, seq, q, cuts):
-    """Runs seq in portions that end at cuts, all logits wanted."""
-    out, at = [], 0
-    for end in cuts:
-        out.append(eng.run_portions([(q, seq[at:end], list(range(end - at)))]))
-        at = end
-    return torch.cat(out)
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -121,34 +87,10 @@ def test_mixed_batches(gpu, case, name, dtype):
     requests come and go, so that pages and slots change hands."""
     cfg, w, seqs, wants = case(name)
     eng = engine(gpu, cfg, w, dtype, tokens=32 * 24, slots=4)
-    g = torch.Generator().manual_seed(4)
-    todo = [0, 1, 2, 3, 1, 2, 1, 3, 2, 1]
-    live, got = [], []
-    while todo or live:
-        while todo and len(live) < 4 and (len(live) < 2 or torch.rand((), generator=g) < 0.4):
-            live.append([todo.pop(0), eng.open_sequence(), 0, []])
-        batch = [r for r in live if len(live) == 1 or torch.rand((), generator=g) < 0.8] or live[:1]
-        portions = []
-        for r in batch:
-            left = len(seqs[r[0]]) - r[2]
-            n = min(left, [1, 1, 1, 2, 3, 17, 64, 70][int(torch.randint(0, 8, (), generator=g))])
-            want = list(range(n)) if n != 17 else [16, 0]
-            portions.append((r[1], seqs[r[0]][r[2]:r[2] + n], want))
-        logits = eng.run_portions(portions).cpu()
-        at = 0
-        for r, (_, toks, want) in zip(batch, portions):
-            for j in want:
-                r[3].append((r[2] + j, logits[at]))
-                at += 1
-            r[2] += len(toks)
-        for r in [r for r in live if r[2] == len(seqs[r[0]])]:
-            eng.close_sequence(r[1])
-            live.remove(r)
-            got.append((r[0], r[3]))
+    got = H.mixed_batches(eng, seqs, [0, 1, 2, 3, 1, 2, 1, 3, 2, 1])
     assert len(got) == 10
-    for i, rows in got:
-        pos = torch.tensor([p for p, _ in rows])
-        check(torch.stack([x for _, x in rows]), wants[i][pos], dtype, f"request {i}")
+    for i, pos, logits in got:
+        check(logits, wants[i][pos], dtype, f"request {i}")
 
 
 def test_nothing_wanted_and_order_of_rows(gpu, case):
