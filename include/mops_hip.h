@@ -599,6 +599,10 @@ int mops_hip_moe_route(const void* h, int64_t h_row_stride, const void* router, 
                        const mops_hip_moe* m, void* stream);
 int mops_hip_moe_gate_up(const void* h, int64_t h_row_stride, const void* w, int64_t up_at, void* y, int64_t y_row_stride,
                          const mops_hip_moe* m, void* stream);
+/* bf16: y[g, t] = w[g] x[g, t] with x [groups (+ 1), tokens, k], w [groups, n, k], y [groups, tokens, n], all contiguous.  w_last
+ * [n_last <= n, k] (or NULL): weights of one more group of rows, y_last [tokens, n_last].  For batches of up to a few hundred tokens. */
+int mops_hip_grouped_linear(const void* x, const void* w, void* y, const void* w_last, void* y_last, int64_t n_last, int64_t groups,
+                            int64_t tokens, int64_t n, int64_t k, void* stream);
 int mops_hip_moe_down(const void* y, int64_t y_row_stride, const void* w, int64_t depth, void* z, int64_t z_row_stride,
                       const mops_hip_moe* m, void* stream);
 

@@ -139,6 +139,7 @@ SIGNATURES = {
     "mops_hip_moe_route_workgroups": (c_int64, [c_int64]),
     "mops_hip_moe_route": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p, POINTER(Moe), c_void_p]),
     "mops_hip_moe_gate_up": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, POINTER(Moe), c_void_p]),
+    "mops_hip_grouped_linear": (c_int, [c_void_p] * 5 + [c_int64] * 5 + [c_void_p]),
     "mops_hip_moe_down": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, POINTER(Moe), c_void_p]),
     "mops_hip_linear_pin_solution": (c_int, [c_int64, c_int64, c_int64, c_int]),
     "mops_hip_linear_tune": (c_int, [c_int64, c_int64, c_int64, c_int64, c_int, c_void_p, c_int64, c_void_p, c_void_p, c_void_p]),

@@ -361,9 +361,9 @@ def sozarax_kernels(t):
     add("low_rank_decay", f"{T} x {rank} -> 1024", lambda: graph_time(lambda i: op("low_rank_decay")(z[i % 4], w2, w0), 4), nbytes=T * (rank * 2 + 1024 * 4.0), like="siluAndMul")
     y, gate, wn = [rnd(T, 1024) for _ in range(4)], [rnd(T, 1024) for _ in range(4)], rnd(1024)
     add("gated_group_norm", f"{T} x 1024, 16 groups", lambda: graph_time(lambda i: op("gated_group_norm")(y[i % 4], gate[i % 4], 16, 1e-6, weight=wn), 8), nbytes=T * 1024 * 6.0, like="siluAndMul")
-    mixes, wr = rnd(4, 256, width), [rnd(4, 1024, width) for _ in range(16)]
-    add("head_linear", "256 rows, 4 x 1024 -> 1024", lambda: graph_time(lambda i: op("head_linear")(mixes.transpose(0, 1), wr[i % 16]), 16),
-        nbytes=4 * 1024 * 1024 * 2 + 256 * 4 * 2048 * 2, flops=2.0 * 256 * 4 * 1024 * 1024, like="linear decode")
+    mixes, wr, w1 = rnd(5, 256, width), [rnd(4, 1024, width) for _ in range(16)], rnd(rank, width)
+    add("grouped_linear", f"256 rows, 4 x 1024 -> 1024 and {rank}", lambda: graph_time(lambda i: op("grouped_linear")(mixes, wr[i % 16], w1), 16),
+        nbytes=4 * 1024 * 1024 * 2 + 256 * 9 * 1024 * 2, flops=2.0 * 256 * 4 * 1024 * 1024, like="linear decode")
     # ---- experts
     for tokens, w, ff, experts, top in ((T, 1024, 1536, 16, 2), (256, 1024, 1536, 16, 2), (T, 2048, 1536, 32, 4), (256, 2048, 1536, 32, 4)):
         tag, n = f"{tokens} x {w}, top {top} of {experts} x {ff}", tokens * top

@@ -5,6 +5,7 @@
 //                top + place) by row; tiles[] cuts each expert's rows into blocks of `block_rows`.
 //   moe_gate_up  y[row] = silu(s W_gate h) * (s W_up h) with h the token's row and s its score: the score scales the expert's input
 //   moe_down     z[choice] = W_down y[row]
+//   grouped_linear   the products of the small blocks without routing: equal runs of rows, each with weights of its own
 //
 // The products are grouped: a workgroup takes a block of rows of one expert and some of its outputs.  Nothing comes back to the
 // host: the grids are sized for the largest possible number of blocks, and workgroups without one leave.  The order of an
@@ -21,16 +22,17 @@ constexpr int kMaxExperts = 1024;
 struct RouteArgs {
   const void *h, *router;
   int64_t h_stride;
-  int tokens, width, experts, top, per_wg;      // per_wg: tokens of a workgroup, a multiple of 16
+  int tokens, width, experts, top;
   int32_t *chosen, *rank, *counts;     // [tokens * top], [tokens * top], [workgroups][experts]
   float* score;                        // [tokens * top]
 };
 
-static int tokens_per_workgroup(int64_t tokens) { return tokens <= 2048 ? 16 : 64; }
+constexpr int kRouteTokens = 16;      // tokens of a route workgroup
+constexpr int kPlaceGroups = 4;       // route workgroups of a place workgroup
 
 // Counts this workgroup's choices per expert and ranks them among each other.
 __device__ __forceinline__ void rank_choices(const RouteArgs& a, int* hist) {
-  const int t0 = blockIdx.x * a.per_wg, n_tokens = a.tokens - t0 < a.per_wg ? a.tokens - t0 : a.per_wg;
+  const int t0 = blockIdx.x * kRouteTokens, n_tokens = a.tokens - t0 < kRouteTokens ? a.tokens - t0 : kRouteTokens;
   __syncthreads();
   for (int e = threadIdx.x; e < a.experts; e += 256) hist[e] = 0;
   __syncthreads();
@@ -42,12 +44,11 @@ __device__ __forceinline__ void rank_choices(const RouteArgs& a, int* hist) {
 
 // 16 tokens at a time on the matrix cores: bf16 operands, exact products, float32 sums; the four waves split the depth.
 // ET: tiles of 16 experts.
-constexpr int kRouteTokens = 16;
 
 template <int ET>
 __global__ __launch_bounds__(256) void moe_route_mfma_kernel(const RouteArgs a, bool aligned) {
   constexpr int kPitch = ET * 16 + 1;
-  constexpr int kAhead = ET <= 2 ? 4 : 2;      // steps whose loads are issued together
+  constexpr int kAhead = ET <= 2 ? 8 : (ET <= 4 ? 4 : 2);      // steps whose loads are issued together
   __shared__ float logits[4][kRouteTokens][kPitch];
   __shared__ int hist[ET * 16];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, n = lane & 15, jj = lane >> 4;
@@ -58,81 +59,79 @@ __global__ __launch_bounds__(256) void moe_route_mfma_kernel(const RouteArgs a, 
     w_ok[i] = 16 * i + n < a.experts;
     w[i] = (const uint16_t*)a.router + (int64_t)(w_ok[i] ? 16 * i + n : 0) * a.width;
   }
-  for (int t0 = blockIdx.x * a.per_wg; t0 < a.tokens && t0 < (int)(blockIdx.x + 1) * a.per_wg; t0 += kRouteTokens) {
-    const int t = t0 + n;
-    const uint16_t* h = (const uint16_t*)a.h + (int64_t)(t < a.tokens ? t : a.tokens - 1) * a.h_stride;
-    f32x4 acc[ET];
+  const int t0 = blockIdx.x * kRouteTokens;
+  const int t = t0 + n;
+  const uint16_t* h = (const uint16_t*)a.h + (int64_t)(t < a.tokens ? t : a.tokens - 1) * a.h_stride;
+  f32x4 acc[ET];
 #pragma unroll
-    for (int i = 0; i < ET; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-    for (int k0 = 32 * kAhead * wave; k0 < a.width; k0 += 128 * kAhead) {
-      u32x4 x[kAhead], y[kAhead][ET];
+  for (int i = 0; i < ET; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int k0 = 32 * kAhead * wave; k0 < a.width; k0 += 128 * kAhead) {
+    u32x4 x[kAhead], y[kAhead][ET];
 #pragma unroll
-      for (int s = 0; s < kAhead; ++s) {
-        const int k = k0 + 32 * s + 8 * jj;
-        if (aligned) {
-          const bool ok = k < a.width;
-          x[s] = load16(h + (ok ? k : 0));
-          if (!ok) x[s] = u32x4{0u, 0u, 0u, 0u};
+    for (int s = 0; s < kAhead; ++s) {
+      const int k = k0 + 32 * s + 8 * jj;
+      if (aligned) {
+        const bool ok = k < a.width;
+        x[s] = load16(h + (ok ? k : 0));
+        if (!ok) x[s] = u32x4{0u, 0u, 0u, 0u};
 #pragma unroll
-          for (int i = 0; i < ET; ++i) {
-            y[s][i] = load16(w[i] + (ok ? k : 0));
-            if (!ok) y[s][i] = u32x4{0u, 0u, 0u, 0u};
-          }
-        } else {
-          x[s] = load8_guarded(h, k, a.width, false);
-#pragma unroll
-          for (int i = 0; i < ET; ++i) y[s][i] = load8_guarded(w[i], k, a.width, false);
+        for (int i = 0; i < ET; ++i) {
+          y[s][i] = load16(w[i] + (ok ? k : 0));
+          if (!ok) y[s][i] = u32x4{0u, 0u, 0u, 0u};
         }
+      } else {
+        x[s] = load8_guarded(h, k, a.width, false);
+#pragma unroll
+        for (int i = 0; i < ET; ++i) y[s][i] = load8_guarded(w[i], k, a.width, false);
       }
-#pragma unroll
-      for (int s = 0; s < kAhead; ++s)
-#pragma unroll
-        for (int i = 0; i < ET; ++i) acc[i] = mfma16(__builtin_bit_cast(bf16x8, y[s][i]), __builtin_bit_cast(bf16x8, x[s]), acc[i]);
     }
 #pragma unroll
-    for (int i = 0; i < ET; ++i)
+    for (int s = 0; s < kAhead; ++s)
 #pragma unroll
-      for (int e = 0; e < 4; ++e) logits[wave][n][16 * i + 4 * jj + e] = acc[i][e];
-    __syncthreads();
-    for (int i = threadIdx.x; i < kRouteTokens * ET * 16; i += 256) {
-      const int r = i / (ET * 16), e = i % (ET * 16);
-      logits[0][r][e] = (logits[0][r][e] + logits[1][r][e]) + (logits[2][r][e] + logits[3][r][e]);
-    }
-    __syncthreads();
-    // sixteen lanes per token: lane x looks at the experts x, x + 16, ...
-    const int mt = threadIdx.x >> 4, x = threadIdx.x & 15, token = t0 + mt;
-    float* mine = logits[0][mt];
-    for (int s = 0; s < a.top; ++s) {
-      float best = -INFINITY;
-      int who = 0x7fffffff;
+      for (int i = 0; i < ET; ++i) acc[i] = mfma16(__builtin_bit_cast(bf16x8, y[s][i]), __builtin_bit_cast(bf16x8, x[s]), acc[i]);
+  }
 #pragma unroll
-      for (int i = 0; i < ET; ++i) {
-        const int e = x + 16 * i;
-        if (e < a.experts && mine[e] > best) {
-          best = mine[e];
-          who = e;
-        }
-      }
+  for (int i = 0; i < ET; ++i)
 #pragma unroll
-      for (int off = 1; off < 16; off <<= 1) {
-        const float ob = __shfl_xor(best, off, kWave);
-        const int ow = __shfl_xor(who, off, kWave);
-        if (ob > best || (ob == best && ow < who)) {
-          best = ob;
-          who = ow;
-        }
-      }
-      if (who >= a.experts) {      // logits that compare with nothing: any expert that is left over, and a score that shows it
-        who = s;
-        best = NAN;
-      }
-      if ((who & 15) == x) mine[who] = -INFINITY;
-      if (x == 0 && token < a.tokens) {
-        a.chosen[(int64_t)token * a.top + s] = who;
-        a.score[(int64_t)token * a.top + s] = 1.0f / (1.0f + expf(-best));
+    for (int e = 0; e < 4; ++e) logits[wave][n][16 * i + 4 * jj + e] = acc[i][e];
+  __syncthreads();
+  for (int i = threadIdx.x; i < kRouteTokens * ET * 16; i += 256) {
+    const int r = i / (ET * 16), e = i % (ET * 16);
+    logits[0][r][e] = (logits[0][r][e] + logits[1][r][e]) + (logits[2][r][e] + logits[3][r][e]);
+  }
+  __syncthreads();
+  // sixteen lanes per token: lane x looks at the experts x, x + 16, ...
+  const int mt = threadIdx.x >> 4, x = threadIdx.x & 15, token = t0 + mt;
+  float* mine = logits[0][mt];
+  for (int s = 0; s < a.top; ++s) {
+    float best = -INFINITY;
+    int who = 0x7fffffff;
+#pragma unroll
+    for (int i = 0; i < ET; ++i) {
+      const int e = x + 16 * i;
+      if (e < a.experts && mine[e] > best) {
+        best = mine[e];
+        who = e;
       }
     }
-    __syncthreads();
+#pragma unroll
+    for (int off = 1; off < 16; off <<= 1) {
+      const float ob = __shfl_xor(best, off, kWave);
+      const int ow = __shfl_xor(who, off, kWave);
+      if (ob > best || (ob == best && ow < who)) {
+        best = ob;
+        who = ow;
+      }
+    }
+    if (who >= a.experts) {      // logits that compare with nothing: any expert that is left over, and a score that shows it
+      who = s;
+      best = NAN;
+    }
+    if ((who & 15) == x) mine[who] = -INFINITY;
+    if (x == 0 && token < a.tokens) {
+      a.chosen[(int64_t)token * a.top + s] = who;
+      a.score[(int64_t)token * a.top + s] = 1.0f / (1.0f + expf(-best));
+    }
   }
   rank_choices(a, hist);
 }
@@ -144,8 +143,8 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const RouteArgs a) {
   __shared__ int hist[kMaxExperts];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   float* mine = logits[wave];
-  for (int i = wave; i < a.per_wg; i += 4) {      // as often for every wave
-    const int t = blockIdx.x * a.per_wg + i;
+  for (int i = wave; i < kRouteTokens; i += 4) {      // as often for every wave
+    const int t = blockIdx.x * kRouteTokens + i;
     const T* h = (const T*)a.h + (int64_t)(t < a.tokens ? t : a.tokens - 1) * a.h_stride;
     for (int e = 0; e < a.experts; ++e) {
       const T* w = (const T*)a.router + (int64_t)e * a.width;
@@ -187,8 +186,8 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const RouteArgs a) {
   rank_choices(a, hist);
 }
 
-// rows[] and tiles[]; a workgroup for each one of the route.  tiles: [0] their number, then {expert, first row, rows} each.
-__global__ __launch_bounds__(256) void moe_place_kernel(const RouteArgs a, int32_t* __restrict__ rows, int32_t* __restrict__ tiles, int block_rows) {
+// rows[] and tiles[]; a workgroup for every kPlaceGroups of the route.  tiles: [0] their number, then {expert, first row, rows} each.
+__global__ __launch_bounds__(256) void moe_place_kernel(const RouteArgs a, int groups, int32_t* __restrict__ rows, int32_t* __restrict__ tiles, int block_rows) {
   __shared__ int total[kMaxExperts], earlier[kMaxExperts];
   __shared__ int begin[kMaxExperts + 1], first_tile[kMaxExperts + 1];
   __shared__ int wave_rows[4], wave_tiles[4];
@@ -197,14 +196,15 @@ __global__ __launch_bounds__(256) void moe_place_kernel(const RouteArgs a, int32
   __syncthreads();
   {
     // threads over (expert, part of the workgroups)
-    const int across = a.experts < 256 ? a.experts : 256, parts = 256 / across;
+    const int across = a.experts < 256 ? a.experts : 256, parts = 256 / across, mine = blockIdx.x * kPlaceGroups;
     if (tid < across * parts)
       for (int e = tid % across; e < a.experts; e += across) {
         int all = 0, front = 0;
-        for (int w = tid / across; w < (int)gridDim.x; w += parts) {
+#pragma unroll 8
+        for (int w = tid / across; w < groups; w += parts) {
           const int c = a.counts[(int64_t)w * a.experts + e];
           all += c;
-          front += w < (int)blockIdx.x ? c : 0;
+          front += w < mine ? c : 0;
         }
         atomicAdd(&total[e], all);
         atomicAdd(&earlier[e], front);
@@ -253,10 +253,13 @@ __global__ __launch_bounds__(256) void moe_place_kernel(const RouteArgs a, int32
     }
   }
   __syncthreads();
-  const int t0 = blockIdx.x * a.per_wg, n_tokens = a.tokens - t0 < a.per_wg ? a.tokens - t0 : a.per_wg;
+  constexpr int kTokens = kRouteTokens * kPlaceGroups;
+  const int t0 = blockIdx.x * kTokens, n_tokens = a.tokens - t0 < kTokens ? a.tokens - t0 : kTokens;
   for (int i = tid; i < n_tokens * a.top; i += 256) {
     const int choice = t0 * a.top + i, e = a.chosen[choice];
-    rows[begin[e] + earlier[e] + a.rank[choice]] = choice;
+    int at = begin[e] + earlier[e] + a.rank[choice];
+    for (int w = blockIdx.x * kPlaceGroups; w < choice / a.top / kRouteTokens; ++w) at += a.counts[(int64_t)w * a.experts + e];
+    rows[at] = choice;
   }
   if (blockIdx.x == 0) {
     if (tid == 0) tiles[0] = first_tile[kMaxExperts];
@@ -280,6 +283,13 @@ struct GroupedArgs {
   const int32_t *rows, *tiles;
   const float* score;
   int top, blocks;          // blocks of outputs in the grid
+  // small blocks without routing (rows == nullptr): group e has the rows e * per_group .., and one more group of the same rows has
+  // weights, outputs and their number of its own
+  int per_group, groups;
+  const void* w_last;
+  int n_last;
+  void* out_last;
+  int64_t out_last_stride;
 };
 
 // This workgroup's tile and block of outputs.  Consecutive workgroups go to different XCDs: each XCD gets a contiguous run of
@@ -410,8 +420,28 @@ template <bool GATED, bool ALIGNED>
 __global__ __launch_bounds__(256, 2) void moe_grouped_small_kernel(const GroupedArgs a) {
   __shared__ __align__(16) f32x4 part[4][8][64];      // [wave][piece of the weights, piece of the rows][lane]
   int tile, block;
-  if (!grouped_item(a, tile, block)) return;
-  const int e = a.tiles[1 + 3 * tile], row0 = a.tiles[2 + 3 * tile], count = a.tiles[3 + 3 * tile];
+  int e, row0, count, n_all = a.n;
+  const uint16_t* w_group;
+  bool last = false;
+  if (a.tiles) {
+    if (!grouped_item(a, tile, block)) return;
+    e = a.tiles[1 + 3 * tile];
+    row0 = a.tiles[2 + 3 * tile];
+    count = a.tiles[3 + 3 * tile];
+    w_group = (const uint16_t*)a.w + (int64_t)e * a.w_expert;
+  } else {
+    // all row tiles of a block of weights one behind the other
+    const int per = (a.per_group + kSM - 1) / kSM;
+    tile = blockIdx.x % per;
+    block = blockIdx.x / per % a.blocks;
+    e = blockIdx.x / per / a.blocks;
+    row0 = e * a.per_group + tile * kSM;
+    count = a.per_group - tile * kSM < kSM ? a.per_group - tile * kSM : kSM;
+    last = e == a.groups;
+    n_all = last ? a.n_last : a.n;
+    w_group = last ? (const uint16_t*)a.w_last : (const uint16_t*)a.w + (int64_t)e * a.w_expert;
+    if (block * 64 >= n_all) return;
+  }
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 15, jj = lane >> 4;
   const int n0 = block * (GATED ? 32 : 64);
   const uint16_t *x[2], *w[4];
@@ -423,7 +453,7 @@ __global__ __launch_bounds__(256, 2) void moe_grouped_small_kernel(const Grouped
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int n = n0 + 16 * (GATED ? i & 1 : i) + col;      // outputs behind the last are row 0 again and never stored
-    w[i] = (const uint16_t*)a.w + (int64_t)e * a.w_expert + (int64_t)((n < a.n ? n : 0) + (GATED && i >= 2 ? a.up_at : 0)) * a.depth;
+    w[i] = w_group + (int64_t)((n < n_all ? n : 0) + (GATED && i >= 2 ? a.up_at : 0)) * a.depth;
   }
   f32x4 acc[4][2];
 #pragma unroll
@@ -486,8 +516,9 @@ __global__ __launch_bounds__(256, 2) void moe_grouped_small_kernel(const Grouped
   auto total = [&](int piece) { return (part[0][piece][lane] + part[1][piece][lane]) + (part[2][piece][lane] + part[3][piece][lane]); };
   const f32x4 v0 = total(2 * i + j), v1 = total(2 * (i + 2) + j);
   if (r >= count) return;
-  const int choice = a.rows[row0 + r];
-  uint16_t* o = (uint16_t*)a.out + (int64_t)(GATED ? row0 + r : choice) * a.out_stride;
+  const int choice = a.rows ? a.rows[row0 + r] : row0 + r;
+  uint16_t* o = last ? (uint16_t*)a.out_last + (int64_t)(choice - e * a.per_group) * a.out_last_stride
+                     : (uint16_t*)a.out + (int64_t)(GATED ? row0 + r : choice) * a.out_stride;
   const float s = GATED ? a.score[choice] : 1.f;
 #pragma unroll
   for (int half = 0; half < (GATED ? 1 : 2); ++half) {
@@ -495,12 +526,12 @@ __global__ __launch_bounds__(256, 2) void moe_grouped_small_kernel(const Grouped
     float y[4];
 #pragma unroll
     for (int q = 0; q < 4; ++q) y[q] = GATED ? silu_for<bf16_t>(s * v0[q]) * (s * v1[q]) : (half ? v1[q] : v0[q]);
-    if (ALIGNED && n + 4 <= a.n) {
+    if (ALIGNED && n + 4 <= n_all) {
       *reinterpret_cast<u32x2*>(o + n) = u32x2{pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3])};
     } else {
 #pragma unroll
       for (int q = 0; q < 4; ++q)
-        if (n + q < a.n) o[n + q] = (uint16_t)f32_to_bf16_bits(y[q]);
+        if (n + q < n_all) o[n + q] = (uint16_t)f32_to_bf16_bits(y[q]);
     }
   }
 }
@@ -601,8 +632,7 @@ extern "C" int64_t mops_hip_moe_max_tiles(int64_t tokens, int64_t experts, int64
 
 extern "C" int64_t mops_hip_moe_route_workgroups(int64_t tokens) {
   if (tokens < 0) return MOPS_HIP_EINVAL;
-  const int64_t per = mops::tokens_per_workgroup(tokens);
-  return (tokens + per - 1) / per;
+  return (tokens + mops::kRouteTokens - 1) / mops::kRouteTokens;
 }
 
 extern "C" int mops_hip_moe_route(const void* h, int64_t h_row_stride, const void* router, int32_t* chosen, int32_t* rank, int32_t* counts,
@@ -614,8 +644,9 @@ extern "C" int mops_hip_moe_route(const void* h, int64_t h_row_stride, const voi
   RouteArgs a;
   a.h = h; a.router = router; a.h_stride = h_row_stride;
   a.tokens = (int)m->tokens; a.width = (int)m->width; a.experts = (int)m->experts; a.top = (int)m->top;
-  a.chosen = chosen; a.rank = rank; a.counts = counts; a.score = m->score; a.per_wg = tokens_per_workgroup(m->tokens);
-  const dim3 grid((unsigned)((m->tokens + a.per_wg - 1) / a.per_wg)), block(256);
+  a.chosen = chosen; a.rank = rank; a.counts = counts; a.score = m->score;
+  const int64_t groups = mops_hip_moe_route_workgroups(m->tokens);
+  const dim3 grid((unsigned)groups), block(256);
   hipStream_t s = (hipStream_t)stream;
   if (m->dtype == MOPS_HIP_BF16 && m->experts <= 128) {
     const bool aligned = m->width % 8 == 0 && h_row_stride % 8 == 0 && aligned16(h) && aligned16(router);
@@ -630,7 +661,7 @@ extern "C" int mops_hip_moe_route(const void* h, int64_t h_row_stride, const voi
   }
   int st = finish_launch();
   if (st != MOPS_HIP_OK) return st;
-  hipLaunchKernelGGL(moe_place_kernel, grid, block, 0, s, a, m->rows, m->tiles, (int)m->block_rows);
+  hipLaunchKernelGGL(moe_place_kernel, dim3((unsigned)((groups + kPlaceGroups - 1) / kPlaceGroups)), block, 0, s, a, (int)groups, m->rows, m->tiles, (int)m->block_rows);
   return finish_launch();
 }
 
@@ -640,7 +671,7 @@ extern "C" int mops_hip_moe_gate_up(const void* h, int64_t h_row_stride, const v
   const int pre = check_grouped(m);
   if (pre != 1) return pre;
   if (!h || !w || !y || h_row_stride < m->width || y_row_stride < m->ff || up_at < m->ff || up_at > (1 << 20)) return MOPS_HIP_EINVAL;
-  GroupedArgs a;
+  GroupedArgs a = {};
   a.x = h; a.x_stride = h_row_stride; a.w = w; a.w_expert = 2 * up_at * m->width;
   a.n = (int)m->ff; a.up_at = (int)up_at; a.depth = (int)m->width; a.out = y; a.out_stride = y_row_stride;
   a.rows = m->rows; a.tiles = m->tiles; a.score = m->score; a.top = (int)m->top; a.blocks = 0;
@@ -653,9 +684,29 @@ extern "C" int mops_hip_moe_down(const void* y, int64_t y_row_stride, const void
   const int pre = check_grouped(m);
   if (pre != 1) return pre;
   if (!y || !w || !z || depth < m->ff || depth > (1 << 20) || y_row_stride < depth || z_row_stride < m->width) return MOPS_HIP_EINVAL;
-  GroupedArgs a;
+  GroupedArgs a = {};
   a.x = y; a.x_stride = y_row_stride; a.w = w; a.w_expert = depth * m->width;
   a.n = (int)m->width; a.up_at = 0; a.depth = (int)depth; a.out = z; a.out_stride = z_row_stride;
   a.rows = m->rows; a.tiles = m->tiles; a.score = m->score; a.top = (int)m->top; a.blocks = 0;
   return launch_grouped<false>(a, m->dtype, m->block_rows, m->tokens * m->top, m->experts, (hipStream_t)stream);
+}
+
+extern "C" int mops_hip_grouped_linear(const void* x, const void* w, void* y, const void* w_last, void* y_last, int64_t n_last, int64_t groups,
+                                       int64_t tokens, int64_t n, int64_t k, void* stream) {
+  using namespace mops;
+  if (groups <= 0 || tokens < 0 || n <= 0 || k <= 0 || (w_last && (!y_last || n_last <= 0 || n_last > n))) return MOPS_HIP_EINVAL;
+  if (tokens == 0) return MOPS_HIP_OK;
+  if (!x || !w || !y) return MOPS_HIP_EINVAL;
+  if (n > (1 << 20) || k > (1 << 20) || (groups + 1) * tokens > 0x7fffffffLL) return MOPS_HIP_EUNSUPPORTED;
+  GroupedArgs a = {};
+  a.x = x; a.x_stride = k; a.w = w; a.w_expert = n * k; a.n = (int)n; a.depth = (int)k; a.out = y; a.out_stride = n; a.top = 1;
+  a.blocks = (int)((n + 63) / 64);
+  a.per_group = (int)tokens; a.groups = (int)groups; a.w_last = w_last; a.n_last = (int)n_last; a.out_last = y_last; a.out_last_stride = n_last;
+  const int64_t grid = (tokens + kSM - 1) / kSM * a.blocks * (groups + (w_last ? 1 : 0));
+  if (grid > 0x7fffffffLL) return MOPS_HIP_EUNSUPPORTED;
+  const bool aligned = k % 8 == 0 && n % 4 == 0 && aligned16(x) && aligned16(w) && aligned16(y) &&
+                       (!w_last || (n_last % 4 == 0 && aligned16(w_last) && aligned16(y_last)));
+  if (aligned) hipLaunchKernelGGL((moe_grouped_small_kernel<false, true>), dim3((unsigned)grid), dim3(256), 0, (hipStream_t)stream, a);
+  else hipLaunchKernelGGL((moe_grouped_small_kernel<false, false>), dim3((unsigned)grid), dim3(256), 0, (hipStream_t)stream, a);
+  return finish_launch();
 }

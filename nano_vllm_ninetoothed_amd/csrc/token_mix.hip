@@ -51,17 +51,19 @@ __global__ __launch_bounds__(256) void token_mix_kernel(const T* __restrict__ x,
   }
 }
 
-constexpr int kDecayTokens = 64, kDecayChannels = 256, kDecayMaxRank = 256;
+constexpr int kDecayChannels = 256, kDecayMaxRank = 256;
 
 // tanh to about one ulp of float32's neighbourhood of a bf16 result
 __device__ __forceinline__ float tanh_fast(float v) {
   return 1.0f - 2.0f * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(2.8853900817779268f * v));
 }
 
-// Workgroup = 64 tokens x 256 channels, a wave takes 64 of the channels; tanh(z) in LDS, the rows of w2 straight from memory.
+// Workgroup = 16 TT tokens x 256 channels, a wave takes 64 of the channels; tanh(z) in LDS, the rows of w2 straight from memory.
+template <int TT>
 __global__ __launch_bounds__(256) void low_rank_decay_mfma_kernel(const uint16_t* __restrict__ z, int64_t z_stride, const uint16_t* __restrict__ w2,
                                                                   const float* __restrict__ w0, float* __restrict__ out, int64_t tokens,
                                                                   int channels, int rank, bool aligned, bool z_aligned, bool wide) {
+  constexpr int kDecayTokens = 16 * TT;
   extern __shared__ __align__(16) unsigned char smem[];
   uint16_t* const tile = reinterpret_cast<uint16_t*>(smem);
   const int ksteps = (rank + 31) / 32, pitch = ksteps * 32 + 8;
@@ -84,20 +86,20 @@ __global__ __launch_bounds__(256) void low_rank_decay_mfma_kernel(const uint16_t
     store16(tile + r * pitch + k, w);
   }
   __syncthreads();
-  f32x4 acc[4][4];      // [channels][tokens]
+  f32x4 acc[4][TT];      // [channels][tokens]
 #pragma unroll
   for (int i = 0; i < 4; ++i)
 #pragma unroll
-    for (int j = 0; j < 4; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int j = 0; j < TT; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
   for (int ks = 0; ks < ksteps; ++ks) {
-    bf16x8 b[4];
+    bf16x8 b[TT];
 #pragma unroll
-    for (int j = 0; j < 4; ++j) b[j] = tile_row(tile, pitch, 16 * j + n, 32 * ks + 8 * jj);
+    for (int j = 0; j < TT; ++j) b[j] = tile_row(tile, pitch, 16 * j + n, 32 * ks + 8 * jj);
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const u32x4 a = ks == 0 ? first[i] : weights(i, ks);
 #pragma unroll
-      for (int j = 0; j < 4; ++j) acc[i][j] = mfma16(__builtin_bit_cast(bf16x8, a), b[j], acc[i][j]);
+      for (int j = 0; j < TT; ++j) acc[i][j] = mfma16(__builtin_bit_cast(bf16x8, a), b[j], acc[i][j]);
     }
   }
 #pragma unroll
@@ -107,7 +109,7 @@ __global__ __launch_bounds__(256) void low_rank_decay_mfma_kernel(const uint16_t
 #pragma unroll
     for (int e = 0; e < 4; ++e) bias[e] = c + e < channels ? w0[c + e] : 0.f;
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
+    for (int j = 0; j < TT; ++j) {
       const int64_t t = t0 + 16 * j + n;
       if (t >= tokens) continue;
       f32x4 o;
@@ -171,10 +173,15 @@ extern "C" int mops_hip_low_rank_decay(const void* z, int64_t z_row_stride, cons
   if (rank > kDecayPlainRank || tokens > 0x7fffffffLL || (channels + 255) / 256 > 65535) return MOPS_HIP_EUNSUPPORTED;
   hipStream_t s = (hipStream_t)stream;
   if (dtype == MOPS_HIP_BF16 && rank <= kDecayMaxRank) {
-    const dim3 grid((unsigned)((tokens + kDecayTokens - 1) / kDecayTokens), (unsigned)((channels + kDecayChannels - 1) / kDecayChannels));
-    const size_t lds = kDecayTokens * ((rank + 31) / 32 * 32 + 8) * 2;
-    hipLaunchKernelGGL(low_rank_decay_mfma_kernel, grid, dim3(256), lds, s, (const uint16_t*)z, z_row_stride, (const uint16_t*)w2, w0, out, tokens,
-                       (int)channels, (int)rank, rank % 8 == 0 && aligned16(w2), z_row_stride % 8 == 0 && aligned16(z), channels % 4 == 0 && aligned16(out));
+    const int per = tokens <= 2048 ? 16 : 64;
+    const dim3 grid((unsigned)((tokens + per - 1) / per), (unsigned)((channels + kDecayChannels - 1) / kDecayChannels));
+    const size_t lds = per * ((rank + 31) / 32 * 32 + 8) * 2;
+    const bool w_aligned = rank % 8 == 0 && aligned16(w2), z_aligned = z_row_stride % 8 == 0 && aligned16(z), wide = channels % 4 == 0 && aligned16(out);
+#define MOPS_LRM(TT) hipLaunchKernelGGL((low_rank_decay_mfma_kernel<TT>), grid, dim3(256), lds, s, (const uint16_t*)z, z_row_stride, (const uint16_t*)w2, w0, \
+                                        out, tokens, (int)channels, (int)rank, w_aligned, z_aligned, wide)
+    if (per == 16) MOPS_LRM(1);
+    else MOPS_LRM(4);
+#undef MOPS_LRM
     return finish_launch();
   }
   const dim3 grid((unsigned)tokens, (unsigned)((channels + 255) / 256));

@@ -7,7 +7,7 @@ import torch
 from . import ChannelRecurrence, Mixer, hip_op, pack, register_mixer, require_size
 from ..mops.hip.recurrent_ops import recurrence_state_pitch
 
-GROUPED_ROWS = 256      # batches up to this many tokens run the four projections of equal size as one launch
+GROUPED_ROWS = 256      # 16-bit batches up to this many tokens run all projections as one launch
 
 
 @register_mixer("time_mixing")
@@ -34,7 +34,8 @@ class TimeMixing(Mixer):
         self.norm = take(prefix + "norm", (h * d,), "norm")
         self.o = take(prefix + "o", (m.width, h * d))
         self.portions = ChannelRecurrence(h, h, d, d, m.dtype)
-        self.linear, self.head_linear, self.mix = hip_op("linear"), hip_op("head_linear"), hip_op("token_mix")
+        self.linear, self.grouped_linear, self.mix = hip_op("linear"), hip_op("grouped_linear"), hip_op("token_mix")
+        self.grouped_rows = GROUPED_ROWS if m.dtype == torch.bfloat16 and self.w1.shape[0] <= h * d else 0
         self.decay, self.recurrence, self.group_norm = hip_op("low_rank_decay"), hip_op("decayed_recurrence"), hip_op("gated_group_norm")
         self.allocate(m.cache)
 
@@ -47,11 +48,12 @@ class TimeMixing(Mixer):
         t, nd = x.shape[0], ctx["n_decode"]
         slots, starts = ctx["state_slots"], ctx["starts"]
         mixes = self.mix(x, self.mu, self.before, starts, slots, ctx["token_seq"], ctx["cu_seqlens"])
-        if t <= GROUPED_ROWS:
-            r, k, v, gate = self.head_linear(mixes[:4].transpose(0, 1), self.rkvg).unbind(1)
+        if t <= self.grouped_rows:
+            (r, k, v, gate), z = self.grouped_linear(mixes, self.rkvg, self.w1)
         else:
             r, k, v, gate = (self.linear(mixes[i], self.each[i]) for i in range(4))
-        log_decay = self.decay(self.linear(mixes[4], self.w1)[:, :self.rank], self.w2, self.w0)
+            z = self.linear(mixes[4], self.w1)
+        log_decay = self.decay(z[:, :self.rank], self.w2, self.w0)
         o = torch.empty((t, self.inner), dtype=x.dtype, device=x.device)
         if nd:
             self.recurrence(r[:nd], k[:nd], v[:nd], o[:nd], self.state, slots[:nd], starts[:nd], h, h, d, d, channel_decay=log_decay[:nd], bonus=self.bonus)

@@ -63,6 +63,7 @@ EXTENSION_OP_NAMES = (
     "moe_route",
     "moe_gate_up",
     "moe_down",
+    "grouped_linear",
 )
 
 

@@ -76,3 +76,19 @@ def moe_down(y: torch.Tensor, w: torch.Tensor, routing: Routing):
     st = _capi.load().mops_hip_moe_down(y.data_ptr(), ff, _flat("w", w, w.numel(), y.dtype), ff, z.data_ptr(), width, byref(m), _stream(y))
     _capi.check("mops_hip_moe_down", st)
     return z
+
+
+@register_hip_op
+def grouped_linear(x: torch.Tensor, w: torch.Tensor, w_last: torch.Tensor = None):
+    """y[g] = x[g] @ w[g].T for x [groups, tokens, k] and w [groups, n, k] (bf16, contiguous) in one launch, for small batches.  w_last
+    [at most n, k]: weights of one more group of rows behind them; then (y, y_last)."""
+    groups, n, k = w.shape
+    tokens = x.shape[1]
+    _require(x.dim() == 3 and x.shape[0] == groups + (w_last is not None) and x.shape[2] == k, "x must be [groups, tokens, k]")
+    y = torch.empty((groups, tokens, n), dtype=x.dtype, device=x.device)
+    last = None if w_last is None else torch.empty((tokens, w_last.shape[0]), dtype=x.dtype, device=x.device)
+    st = _capi.load().mops_hip_grouped_linear(_flat("x", x, x.numel(), torch.bfloat16), _flat("w", w, w.numel(), torch.bfloat16), y.data_ptr(),
+                                              None if last is None else _flat("w_last", w_last, w_last.shape[0] * k, torch.bfloat16),
+                                              None if last is None else last.data_ptr(), 0 if last is None else w_last.shape[0], groups, tokens, n, k, _stream(x))
+    _capi.check("mops_hip_grouped_linear", st)
+    return y if last is None else (y, last)

@@ -369,3 +369,15 @@ def test_all_tokens_on_one_expert_and_replay(gpu):
         a, b = torch.empty_like(y), torch.empty_like(ye)
         a[routing.rows.long()], b[eager.rows.long()] = y, ye
         assert torch.equal(a, b)
+
+
+@pytest.mark.parametrize("groups,tokens,n,k,last", [(4, 1, 64, 64, 16), (4, 70, 132, 72, 5), (3, 256, 256, 320, 256), (2, 33, 50, 44, None), (4, 16, 1024, 1024, 32)])
+def test_grouped_linear(gpu, groups, tokens, n, k, last):
+    g = torch.Generator().manual_seed(n)
+    x, w = torch.randn((groups + (last is not None), tokens, k), generator=g).bfloat16(), torch.randn((groups, n, k), generator=g).bfloat16()
+    wl = None if last is None else torch.randn((last, k), generator=g).bfloat16()
+    got = op("grouped_linear")(x.to(gpu), w.to(gpu), None if wl is None else wl.to(gpu))
+    y = got if last is None else got[0]
+    assert rel(y, torch.stack([x[i].to(D) @ w[i].to(D).T for i in range(groups)])) < 3e-3
+    if last is not None:
+        assert rel(got[1], x[-1].to(D) @ wl.to(D).T) < 3e-3
