@@ -417,7 +417,7 @@ constexpr int kSM = 32;
 
 // Four 16-row pieces of the weights: GATED two of gate rows and two of up rows (32 outputs), else 64 outputs; two pieces of 16 rows.
 template <bool GATED, bool ALIGNED>
-__global__ __launch_bounds__(256, 2) void moe_grouped_small_kernel(const GroupedArgs a) {
+__global__ __launch_bounds__(256, 3) void moe_grouped_small_kernel(const GroupedArgs a) {
   __shared__ __align__(16) f32x4 part[4][8][64];      // [wave][piece of the weights, piece of the rows][lane]
   int tile, block;
   int e, row0, count, n_all = a.n;
@@ -460,51 +460,48 @@ __global__ __launch_bounds__(256, 2) void moe_grouped_small_kernel(const Grouped
   for (int i = 0; i < 4; ++i)
 #pragma unroll
     for (int j = 0; j < 2; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
-  // a wave takes every fourth piece of 64 of the depth; the next piece is in flight while this one is used
-  u32x4 xr[2][2][2], wr[2][2][4];
-  auto fetch = [&](int buf, int k0) {
+  // a wave takes every fourth piece of 32 of the depth, with two pieces in flight while one is used
+  u32x4 xr[3][2], wr[3][4];
+  const int pieces = (a.depth - 32 * wave + 127) / 128;
+  auto fetch = [&](int buf, int piece) {
+    const int k = 32 * wave + 128 * piece + 8 * jj;
+    if (ALIGNED) {
+      const bool ok = k < a.depth;
 #pragma unroll
-    for (int s = 0; s < 2; ++s) {
-      const int k = k0 + 32 * s + 8 * jj;
-      if (ALIGNED) {
-        const bool ok = k < a.depth;
+      for (int i = 0; i < 4; ++i) wr[buf][i] = load16(w[i] + (ok ? k : 0));
 #pragma unroll
-        for (int i = 0; i < 4; ++i) wr[buf][s][i] = load16_stream(w[i] + (ok ? k : 0));
+      for (int j = 0; j < 2; ++j) xr[buf][j] = load16(x[j] + (ok ? k : 0));
+    } else {
 #pragma unroll
-        for (int j = 0; j < 2; ++j) {
-          xr[buf][s][j] = load16(x[j] + (ok ? k : 0));
-          if (!ok) xr[buf][s][j] = u32x4{0u, 0u, 0u, 0u};
-        }
-        if (!ok) {
+      for (int i = 0; i < 4; ++i) wr[buf][i] = load8_guarded(w[i], k, a.depth, false);
 #pragma unroll
-          for (int i = 0; i < 4; ++i) wr[buf][s][i] = u32x4{0u, 0u, 0u, 0u};
-        }
-      } else {
-#pragma unroll
-        for (int i = 0; i < 4; ++i) wr[buf][s][i] = load8_guarded(w[i], k, a.depth, false);
-#pragma unroll
-        for (int j = 0; j < 2; ++j) xr[buf][s][j] = load8_guarded(x[j], k, a.depth, false);
-      }
+      for (int j = 0; j < 2; ++j) xr[buf][j] = load8_guarded(x[j], k, a.depth, false);
     }
   };
-  auto use = [&](int buf) {
+  auto use = [&](int buf, int piece) {
+    const bool ok = 32 * wave + 128 * piece + 8 * jj < a.depth;      // what lies behind the depth counts as zeros on both sides
+    const u32x4 zero = {0u, 0u, 0u, 0u};
 #pragma unroll
-    for (int s = 0; s < 2; ++s)
+    for (int j = 0; j < 2; ++j) {
+      const bf16x8 b = __builtin_bit_cast(bf16x8, ok ? xr[buf][j] : zero);
 #pragma unroll
-      for (int i = 0; i < 4; ++i)
-#pragma unroll
-        for (int j = 0; j < 2; ++j) acc[i][j] = mfma16(__builtin_bit_cast(bf16x8, wr[buf][s][i]), __builtin_bit_cast(bf16x8, xr[buf][s][j]), acc[i][j]);
+      for (int i = 0; i < 4; ++i) acc[i][j] = mfma16(__builtin_bit_cast(bf16x8, ok ? wr[buf][i] : zero), b, acc[i][j]);
+    }
   };
-  int k0 = 64 * wave;
-  if (k0 < a.depth) fetch(0, k0);
-  while (k0 < a.depth) {      // two pieces a turn: the buffers are registers
-    if (k0 + 256 < a.depth) fetch(1, k0 + 256);
-    use(0);
-    k0 += 256;
-    if (k0 >= a.depth) break;
-    if (k0 + 256 < a.depth) fetch(0, k0 + 256);
-    use(1);
-    k0 += 256;
+  if (pieces > 0) {
+    fetch(0, 0);
+    fetch(1, 1);
+    for (int p = 0;; p += 3) {      // three pieces a turn: the buffers are registers
+      fetch(2, p + 2);
+      use(0, p);
+      if (p + 1 >= pieces) break;
+      fetch(0, p + 3);
+      use(1, p + 1);
+      if (p + 2 >= pieces) break;
+      fetch(1, p + 4);
+      use(2, p + 2);
+      if (p + 3 >= pieces) break;
+    }
   }
 #pragma unroll
   for (int i = 0; i < 4; ++i)

@@ -208,17 +208,17 @@ CHUNK_MAX_DIM = 256       # head sizes (d) the chunked kernels cover
 def recurrence_segments(counts, heads: int, groups: int, vd: int, wanted: int = 512):
     """Cuts portions of counts[i] tokens (packed one behind the other) into segments for decayed_chunks: one per portion if
     those give enough workgroups, else about `wanted` workgroups in all.  Returns host lists (segments, bounds per portion)."""
-    return _segments(counts, _capi.load().mops_hip_decayed_chunks_workgroups(heads, groups, vd), wanted)
+    return _segments(counts, _capi.load().mops_hip_decayed_chunks_workgroups(heads, groups, vd), wanted, wanted // 2)
 
 
-def channel_segments(counts, heads: int, vd: int, wanted: int = 768):
+def channel_segments(counts, heads: int, vd: int, wanted: int = 1024, enough: int = 192):
     """The same for channel_chunks."""
-    return _segments(counts, _capi.load().mops_hip_channel_chunks_workgroups(heads, vd), wanted)
+    return _segments(counts, _capi.load().mops_hip_channel_chunks_workgroups(heads, vd), wanted, enough)
 
 
-def _segments(counts, per_segment: int, wanted: int):
+def _segments(counts, per_segment: int, wanted: int, enough: int):
     length = max(counts)
-    if len(counts) * per_segment < wanted // 2 and length > 256:
+    if len(counts) * per_segment < enough and length > 256:
         length = max(128, -(-sum(counts) * per_segment // wanted // 64) * 64)
     segments, bounds, at = [], [0], 0
     for i, n in enumerate(counts):
