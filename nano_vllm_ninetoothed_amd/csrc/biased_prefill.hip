@@ -55,11 +55,20 @@ __global__ __launch_bounds__(256, NK <= 8 && NV <= 4 ? 2 : 1) void biased_prefil
   const int visible = pos0 + q_count < keys ? pos0 + q_count : keys;      // keys any query of the tile sees
   const int krow = tid >> 2, kcol = (tid & 3) * 8;
   u32x4 kreg[kLoadsK], vreg[kLoadsV];
-  auto page_of = [&](int k0) {      // row of this thread's token in the pages, -1 without one
-    const int j = k0 + krow, blk = j / bs;
-    if (j >= visible || blk >= a.max_blocks) return (int64_t)-1;
-    const int id = table[blk];
-    return id < 0 || id >= a.num_blocks ? (int64_t)-1 : (int64_t)id * bs + j % bs;
+  int j_next = krow, blk_next = krow / bs, in_blk = krow % bs;      // the token page_of looks up next
+  auto page_of = [&]() {      // row of this thread's next token in the pages, -1 without one
+    int64_t row = -1;
+    if (j_next < visible && blk_next < a.max_blocks) {
+      const int id = table[blk_next];
+      if (id >= 0 && id < a.num_blocks) row = (int64_t)id * bs + in_blk;
+    }
+    j_next += kPrefillKeys;
+    in_blk += kPrefillKeys;
+    while (in_blk >= bs) {
+      in_blk -= bs;
+      ++blk_next;
+    }
+    return row;
   };
   auto issue = [&](int64_t row) {
     const uint16_t *ks = (const uint16_t*)a.k_pages + ((row < 0 ? 0 : row) * groups + g) * dp;
@@ -74,8 +83,8 @@ __global__ __launch_bounds__(256, NK <= 8 && NV <= 4 ? 2 : 1) void biased_prefil
   };
   const float scale = a.scale * 1.4426950408889634f;
   const float slope = a.slopes ? a.slopes[h] * 1.4426950408889634f : 0.f;
-  issue(page_of(0));
-  int64_t next_row = page_of(kPrefillKeys);
+  issue(page_of());
+  int64_t next_row = page_of();
   for (int k0 = 0; k0 < visible; k0 += kPrefillKeys) {
     __syncthreads();
 #pragma unroll
@@ -85,7 +94,7 @@ __global__ __launch_bounds__(256, NK <= 8 && NV <= 4 ? 2 : 1) void biased_prefil
     __syncthreads();
     if (k0 + kPrefillKeys < visible) {
       issue(next_row);
-      next_row = page_of(k0 + 2 * kPrefillKeys);
+      next_row = page_of();
     }
     if (k0 > pos0 + 32 * wave + 31) continue;           // this wave's queries see none of the tile
     f32x16 s[2];
@@ -100,17 +109,25 @@ __global__ __launch_bounds__(256, NK <= 8 && NV <= 4 ? 2 : 1) void biased_prefil
     float m_loc = -INFINITY;
     const int last = pos < keys - 1 ? pos : keys - 1;
     const float dist = (float)(k0 + 4 * hh - pos);      // of the lane's first key, in front of the query by its negative
-    const bool edge = k0 + kPrefillKeys - 1 > pos0 + 32 * wave || k0 + kPrefillKeys > keys;      // the diagonal or the end of the context
+    if (k0 + kPrefillKeys - 1 > pos0 + 32 * wave || k0 + kPrefillKeys > keys) {      // the diagonal or the end of the context: mask
 #pragma unroll
-    for (int kt = 0; kt < 2; ++kt)
+      for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
-      for (int r = 0; r < 16; ++r) {
-        const int off = 32 * kt + 8 * (r >> 2) + (r & 3);
-        float x = s[kt][r] * scale + slope * (dist + (float)off);
-        if (edge && k0 + 4 * hh + off > last) x = -INFINITY;
-        s[kt][r] = x;
-        m_loc = fmaxf(m_loc, x);
-      }
+        for (int r = 0; r < 16; ++r) {
+          const int off = 32 * kt + 8 * (r >> 2) + (r & 3);
+          s[kt][r] = k0 + 4 * hh + off <= last ? s[kt][r] * scale + slope * (dist + (float)off) : -INFINITY;
+          m_loc = fmaxf(m_loc, s[kt][r]);
+        }
+    } else {
+#pragma unroll
+      for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+        for (int r = 0; r < 16; ++r) {
+          const int off = 32 * kt + 8 * (r >> 2) + (r & 3);
+          s[kt][r] = s[kt][r] * scale + slope * (dist + (float)off);
+          m_loc = fmaxf(m_loc, s[kt][r]);
+        }
+    }
     m_loc = fmaxf(m_loc, __shfl_xor(m_loc, 32, kWave));
     const float m_new = fmaxf(m_run, m_loc);
     const float m_safe = m_new == -INFINITY ? 0.f : m_new;
