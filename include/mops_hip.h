@@ -581,7 +581,7 @@ int mops_hip_biased_prefill(const mops_hip_biased_attention* a, const int32_t* t
 /*
  * Mixture of experts (csrc/moe.hip).  moe_route: logits = router [experts, width] h in float32; chosen, score [tokens * top] =
  * the experts with the largest logits and the sigmoids of these; rank [tokens * top] and counts [moe_route_workgroups(tokens),
- * experts] are scratch; rows [tokens * top] lists the choices (token * top + place) ordered by expert, tiles
+ * experts] (aligned to 16 bytes) are scratch; rows [tokens * top] lists the choices (token * top + place) ordered by expert, tiles
  * [1 + 3 * moe_max_tiles] = number of blocks, then (expert, first row, rows) of each.  block_rows: 32, or 128 (bf16).
  * moe_gate_up: w [experts][2 * up_at][width], gate rows from 0, up rows from up_at on; y [tokens * top rows in the order of
  * `rows`], y = silu(score W_gate h) * (score W_up h).  moe_down: w [experts][width][depth], depth >= ff, the columns behind ff

@@ -22,17 +22,18 @@ constexpr int kMaxExperts = 1024;
 struct RouteArgs {
   const void *h, *router;
   int64_t h_stride;
-  int tokens, width, experts, top;
+  int tokens, width, experts, top, per_wg;      // per_wg: tokens of a route workgroup, 16 or 32
   int32_t *chosen, *rank, *counts;     // [tokens * top], [tokens * top], [workgroups][experts]
   float* score;                        // [tokens * top]
 };
 
-constexpr int kRouteTokens = 16;      // tokens of a route workgroup
 constexpr int kPlaceGroups = 4;       // route workgroups of a place workgroup
+// Tokens of a route workgroup: the router's weights are read once for all of them; small batches need the workgroups more.
+static int route_tokens(int64_t tokens) { return tokens <= 2048 ? 16 : 32; }
 
 // Counts this workgroup's choices per expert and ranks them among each other.
 __device__ __forceinline__ void rank_choices(const RouteArgs& a, int* hist) {
-  const int t0 = blockIdx.x * kRouteTokens, n_tokens = a.tokens - t0 < kRouteTokens ? a.tokens - t0 : kRouteTokens;
+  const int t0 = blockIdx.x * a.per_wg, n_tokens = a.tokens - t0 < a.per_wg ? a.tokens - t0 : a.per_wg;
   __syncthreads();
   for (int e = threadIdx.x; e < a.experts; e += 256) hist[e] = 0;
   __syncthreads();
@@ -42,45 +43,49 @@ __device__ __forceinline__ void rank_choices(const RouteArgs& a, int* hist) {
   for (int e = threadIdx.x; e < a.experts; e += 256) a.counts[(int64_t)blockIdx.x * a.experts + e] = hist[e];
 }
 
-// 16 tokens at a time on the matrix cores: bf16 operands, exact products, float32 sums; the four waves split the depth.
+// 16 TT tokens per workgroup on the matrix cores: bf16 operands, exact products, float32 sums; the four waves split the depth.
 // ET: tiles of 16 experts.
-
-template <int ET>
+template <int ET, int TT>
 __global__ __launch_bounds__(256) void moe_route_mfma_kernel(const RouteArgs a, bool aligned) {
   constexpr int kPitch = ET * 16 + 1;
-  constexpr int kAhead = ET <= 2 ? 8 : (ET <= 4 ? 4 : 2);      // steps whose loads are issued together
-  __shared__ float logits[4][kRouteTokens][kPitch];
+  constexpr int kAhead = TT == 1 ? (ET <= 2 ? 8 : (ET <= 4 ? 4 : 2)) : (ET <= 2 ? 4 : (ET <= 4 ? 2 : 1));      // steps whose loads are issued together
+  __shared__ float logits[2][16 * TT][kPitch];
   __shared__ int hist[ET * 16];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, n = lane & 15, jj = lane >> 4;
-  const uint16_t* w[ET];
-  bool w_ok[ET];
+  const int t0 = blockIdx.x * 16 * TT;
+  const uint16_t *h[TT], *w[ET];
 #pragma unroll
-  for (int i = 0; i < ET; ++i) {
-    w_ok[i] = 16 * i + n < a.experts;
-    w[i] = (const uint16_t*)a.router + (int64_t)(w_ok[i] ? 16 * i + n : 0) * a.width;
+  for (int j = 0; j < TT; ++j) {
+    const int t = t0 + 16 * j + n;
+    h[j] = (const uint16_t*)a.h + (int64_t)(t < a.tokens ? t : a.tokens - 1) * a.h_stride;
   }
-  const int t0 = blockIdx.x * kRouteTokens;
-  const int t = t0 + n;
-  const uint16_t* h = (const uint16_t*)a.h + (int64_t)(t < a.tokens ? t : a.tokens - 1) * a.h_stride;
-  f32x4 acc[ET];
 #pragma unroll
-  for (int i = 0; i < ET; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int i = 0; i < ET; ++i) w[i] = (const uint16_t*)a.router + (int64_t)(16 * i + n < a.experts ? 16 * i + n : 0) * a.width;
+  f32x4 acc[ET][TT];
+#pragma unroll
+  for (int i = 0; i < ET; ++i)
+#pragma unroll
+    for (int j = 0; j < TT; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
   for (int k0 = 32 * kAhead * wave; k0 < a.width; k0 += 128 * kAhead) {
-    u32x4 x[kAhead], y[kAhead][ET];
+    u32x4 x[kAhead][TT], y[kAhead][ET];
 #pragma unroll
     for (int s = 0; s < kAhead; ++s) {
       const int k = k0 + 32 * s + 8 * jj;
       if (aligned) {
         const bool ok = k < a.width;
-        x[s] = load16(h + (ok ? k : 0));
-        if (!ok) x[s] = u32x4{0u, 0u, 0u, 0u};
+#pragma unroll
+        for (int j = 0; j < TT; ++j) {
+          x[s][j] = load16(h[j] + (ok ? k : 0));
+          if (!ok) x[s][j] = u32x4{0u, 0u, 0u, 0u};
+        }
 #pragma unroll
         for (int i = 0; i < ET; ++i) {
           y[s][i] = load16(w[i] + (ok ? k : 0));
           if (!ok) y[s][i] = u32x4{0u, 0u, 0u, 0u};
         }
       } else {
-        x[s] = load8_guarded(h, k, a.width, false);
+#pragma unroll
+        for (int j = 0; j < TT; ++j) x[s][j] = load8_guarded(h[j], k, a.width, false);
 #pragma unroll
         for (int i = 0; i < ET; ++i) y[s][i] = load8_guarded(w[i], k, a.width, false);
       }
@@ -88,49 +93,63 @@ __global__ __launch_bounds__(256) void moe_route_mfma_kernel(const RouteArgs a, 
 #pragma unroll
     for (int s = 0; s < kAhead; ++s)
 #pragma unroll
-      for (int i = 0; i < ET; ++i) acc[i] = mfma16(__builtin_bit_cast(bf16x8, y[s][i]), __builtin_bit_cast(bf16x8, x[s]), acc[i]);
-  }
+      for (int i = 0; i < ET; ++i)
 #pragma unroll
-  for (int i = 0; i < ET; ++i)
-#pragma unroll
-    for (int e = 0; e < 4; ++e) logits[wave][n][16 * i + 4 * jj + e] = acc[i][e];
-  __syncthreads();
-  for (int i = threadIdx.x; i < kRouteTokens * ET * 16; i += 256) {
-    const int r = i / (ET * 16), e = i % (ET * 16);
-    logits[0][r][e] = (logits[0][r][e] + logits[1][r][e]) + (logits[2][r][e] + logits[3][r][e]);
+        for (int j = 0; j < TT; ++j) acc[i][j] = mfma16(__builtin_bit_cast(bf16x8, y[s][i]), __builtin_bit_cast(bf16x8, x[s][j]), acc[i][j]);
   }
-  __syncthreads();
+  // the waves' parts: the first two leave theirs, the others add to them
+#pragma unroll
+  for (int round = 0; round < 2; ++round) {
+    if (wave >> 1 == round) {
+#pragma unroll
+      for (int i = 0; i < ET; ++i)
+#pragma unroll
+        for (int j = 0; j < TT; ++j)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            float& to = logits[wave & 1][16 * j + n][16 * i + 4 * jj + e];
+            to = round ? to + acc[i][j][e] : acc[i][j][e];
+          }
+    }
+    __syncthreads();
+  }
   // sixteen lanes per token: lane x looks at the experts x, x + 16, ...
-  const int mt = threadIdx.x >> 4, x = threadIdx.x & 15, token = t0 + mt;
-  float* mine = logits[0][mt];
-  for (int s = 0; s < a.top; ++s) {
-    float best = -INFINITY;
-    int who = 0x7fffffff;
+  const int x = threadIdx.x & 15;
 #pragma unroll
-    for (int i = 0; i < ET; ++i) {
-      const int e = x + 16 * i;
-      if (e < a.experts && mine[e] > best) {
-        best = mine[e];
-        who = e;
-      }
-    }
+  for (int j = 0; j < TT; ++j) {
+    const int mt = 16 * j + (threadIdx.x >> 4), token = t0 + mt;
+    float mine[ET];
 #pragma unroll
-    for (int off = 1; off < 16; off <<= 1) {
-      const float ob = __shfl_xor(best, off, kWave);
-      const int ow = __shfl_xor(who, off, kWave);
-      if (ob > best || (ob == best && ow < who)) {
-        best = ob;
-        who = ow;
+    for (int i = 0; i < ET; ++i) mine[i] = x + 16 * i < a.experts ? logits[0][mt][x + 16 * i] + logits[1][mt][x + 16 * i] : -INFINITY;
+    for (int s = 0; s < a.top; ++s) {
+      float best = -INFINITY;
+      int who = 0x7fffffff;
+#pragma unroll
+      for (int i = 0; i < ET; ++i)
+        if (mine[i] > best) {
+          best = mine[i];
+          who = x + 16 * i;
+        }
+#pragma unroll
+      for (int off = 1; off < 16; off <<= 1) {
+        const float ob = __shfl_xor(best, off, kWave);
+        const int ow = __shfl_xor(who, off, kWave);
+        if (ob > best || (ob == best && ow < who)) {
+          best = ob;
+          who = ow;
+        }
       }
-    }
-    if (who >= a.experts) {      // logits that compare with nothing: any expert that is left over, and a score that shows it
-      who = s;
-      best = NAN;
-    }
-    if ((who & 15) == x) mine[who] = -INFINITY;
-    if (x == 0 && token < a.tokens) {
-      a.chosen[(int64_t)token * a.top + s] = who;
-      a.score[(int64_t)token * a.top + s] = 1.0f / (1.0f + expf(-best));
+      if (who >= a.experts) {      // logits that compare with nothing: any expert that is left over, and a score that shows it
+        who = s;
+        best = NAN;
+      }
+#pragma unroll
+      for (int i = 0; i < ET; ++i)
+        if (who == x + 16 * i) mine[i] = -INFINITY;
+      if (x == 0 && token < a.tokens) {
+        a.chosen[(int64_t)token * a.top + s] = who;
+        a.score[(int64_t)token * a.top + s] = 1.0f / (1.0f + expf(-best));
+      }
     }
   }
   rank_choices(a, hist);
@@ -143,8 +162,8 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const RouteArgs a) {
   __shared__ int hist[kMaxExperts];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   float* mine = logits[wave];
-  for (int i = wave; i < kRouteTokens; i += 4) {      // as often for every wave
-    const int t = blockIdx.x * kRouteTokens + i;
+  for (int i = wave; i < a.per_wg; i += 4) {      // as often for every wave
+    const int t = blockIdx.x * a.per_wg + i;
     const T* h = (const T*)a.h + (int64_t)(t < a.tokens ? t : a.tokens - 1) * a.h_stride;
     for (int e = 0; e < a.experts; ++e) {
       const T* w = (const T*)a.router + (int64_t)e * a.width;
@@ -195,19 +214,34 @@ __global__ __launch_bounds__(256) void moe_place_kernel(const RouteArgs a, int g
   for (int e = tid; e < kMaxExperts; e += 256) total[e] = earlier[e] = 0;
   __syncthreads();
   {
-    // threads over (expert, part of the workgroups)
-    const int across = a.experts < 256 ? a.experts : 256, parts = 256 / across, mine = blockIdx.x * kPlaceGroups;
+    // threads over (experts, part of the workgroups); four experts at a time where rows of counts are aligned
+    const int mine = blockIdx.x * kPlaceGroups, step = a.experts % 4 == 0 ? 4 : 1, columns = a.experts / step;
+    const int across = columns < 256 ? columns : 256, parts = 256 / across;
     if (tid < across * parts)
-      for (int e = tid % across; e < a.experts; e += across) {
-        int all = 0, front = 0;
+      for (int c = tid % across; c < columns; c += across) {
+        int all[4] = {0, 0, 0, 0}, front[4] = {0, 0, 0, 0};
+        if (step == 4) {
+#pragma unroll 4
+          for (int w = tid / across; w < groups; w += parts) {
+            const u32x4 v = load16(a.counts + (int64_t)w * a.experts + 4 * c);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+              all[e] += (int)v[e];
+              front[e] += w < mine ? (int)v[e] : 0;
+            }
+          }
+        } else {
 #pragma unroll 8
-        for (int w = tid / across; w < groups; w += parts) {
-          const int c = a.counts[(int64_t)w * a.experts + e];
-          all += c;
-          front += w < mine ? c : 0;
+          for (int w = tid / across; w < groups; w += parts) {
+            const int v = a.counts[(int64_t)w * a.experts + c];
+            all[0] += v;
+            front[0] += w < mine ? v : 0;
+          }
         }
-        atomicAdd(&total[e], all);
-        atomicAdd(&earlier[e], front);
+        for (int e = 0; e < step; ++e) {
+          atomicAdd(&total[c * step + e], all[e]);
+          atomicAdd(&earlier[c * step + e], front[e]);
+        }
       }
   }
   __syncthreads();
@@ -253,12 +287,11 @@ __global__ __launch_bounds__(256) void moe_place_kernel(const RouteArgs a, int g
     }
   }
   __syncthreads();
-  constexpr int kTokens = kRouteTokens * kPlaceGroups;
-  const int t0 = blockIdx.x * kTokens, n_tokens = a.tokens - t0 < kTokens ? a.tokens - t0 : kTokens;
+  const int per = a.per_wg * kPlaceGroups, t0 = blockIdx.x * per, n_tokens = a.tokens - t0 < per ? a.tokens - t0 : per;
   for (int i = tid; i < n_tokens * a.top; i += 256) {
     const int choice = t0 * a.top + i, e = a.chosen[choice];
     int at = begin[e] + earlier[e] + a.rank[choice];
-    for (int w = blockIdx.x * kPlaceGroups; w < choice / a.top / kRouteTokens; ++w) at += a.counts[(int64_t)w * a.experts + e];
+    for (int w = blockIdx.x * kPlaceGroups; w < choice / a.top / a.per_wg; ++w) at += a.counts[(int64_t)w * a.experts + e];
     rows[at] = choice;
   }
   if (blockIdx.x == 0) {
@@ -629,7 +662,7 @@ extern "C" int64_t mops_hip_moe_max_tiles(int64_t tokens, int64_t experts, int64
 
 extern "C" int64_t mops_hip_moe_route_workgroups(int64_t tokens) {
   if (tokens < 0) return MOPS_HIP_EINVAL;
-  return (tokens + mops::kRouteTokens - 1) / mops::kRouteTokens;
+  return (tokens + mops::route_tokens(tokens) - 1) / mops::route_tokens(tokens);
 }
 
 extern "C" int mops_hip_moe_route(const void* h, int64_t h_row_stride, const void* router, int32_t* chosen, int32_t* rank, int32_t* counts,
@@ -638,19 +671,26 @@ extern "C" int mops_hip_moe_route(const void* h, int64_t h_row_stride, const voi
   const int pre = check_grouped(m);
   if (pre != 1) return pre;
   if (!h || !router || !chosen || !rank || !counts || h_row_stride < m->width) return MOPS_HIP_EINVAL;
+  if (!aligned16(counts)) return MOPS_HIP_EALIGN;
   RouteArgs a;
   a.h = h; a.router = router; a.h_stride = h_row_stride;
   a.tokens = (int)m->tokens; a.width = (int)m->width; a.experts = (int)m->experts; a.top = (int)m->top;
   a.chosen = chosen; a.rank = rank; a.counts = counts; a.score = m->score;
+  a.per_wg = route_tokens(m->tokens);
   const int64_t groups = mops_hip_moe_route_workgroups(m->tokens);
   const dim3 grid((unsigned)groups), block(256);
   hipStream_t s = (hipStream_t)stream;
   if (m->dtype == MOPS_HIP_BF16 && m->experts <= 128) {
     const bool aligned = m->width % 8 == 0 && h_row_stride % 8 == 0 && aligned16(h) && aligned16(router);
-    if (m->experts <= 16) hipLaunchKernelGGL((moe_route_mfma_kernel<1>), grid, block, 0, s, a, aligned);
-    else if (m->experts <= 32) hipLaunchKernelGGL((moe_route_mfma_kernel<2>), grid, block, 0, s, a, aligned);
-    else if (m->experts <= 64) hipLaunchKernelGGL((moe_route_mfma_kernel<4>), grid, block, 0, s, a, aligned);
-    else hipLaunchKernelGGL((moe_route_mfma_kernel<8>), grid, block, 0, s, a, aligned);
+#define MOPS_ROUTE(E) do {                                                                                                \
+    if (a.per_wg == 16) hipLaunchKernelGGL((moe_route_mfma_kernel<E, 1>), grid, block, 0, s, a, aligned);                \
+    else hipLaunchKernelGGL((moe_route_mfma_kernel<E, 2>), grid, block, 0, s, a, aligned);                               \
+  } while (0)
+    if (m->experts <= 16) MOPS_ROUTE(1);
+    else if (m->experts <= 32) MOPS_ROUTE(2);
+    else if (m->experts <= 64) MOPS_ROUTE(4);
+    else MOPS_ROUTE(8);
+#undef MOPS_ROUTE
   } else if (m->dtype == MOPS_HIP_BF16) {
     hipLaunchKernelGGL((moe_route_kernel<bf16_t>), grid, block, 0, s, a);
   } else {

@@ -37,8 +37,8 @@ def moe_route(h: torch.Tensor, router: torch.Tensor, top: int, block_rows: int =
     lib = _capi.load()
     n = tokens * top
     tiles = lib.mops_hip_moe_max_tiles(tokens, experts, top, block_rows)
-    sizes = [n, n, n, lib.mops_hip_moe_route_workgroups(tokens) * experts, 1 + 3 * tiles]
-    chosen, rank, rows, counts, tile_list = torch.empty(sum(sizes), dtype=torch.int32, device=h.device).split(sizes)
+    sizes = [lib.mops_hip_moe_route_workgroups(tokens) * experts, n, n, n, 1 + 3 * tiles]      # the counts first: their rows are aligned
+    counts, chosen, rank, rows, tile_list = torch.empty(sum(sizes), dtype=torch.int32, device=h.device).split(sizes)
     score = torch.empty((tokens, top), dtype=torch.float32, device=h.device)
     m = _capi.Moe()
     m.rows, m.tiles, m.score = rows.data_ptr(), tile_list.data_ptr(), score.data_ptr()

@@ -308,7 +308,7 @@ def test_long_portions(gpu, H, G, d, v):
 # ---------------------------------------------------------------------------------------------------- mixture of experts
 @pytest.mark.parametrize("dtype,block", [(torch.float32, 32), (torch.bfloat16, 32), (torch.bfloat16, 128)])
 @pytest.mark.parametrize("tokens,width,ff,experts,top", [(1, 64, 32, 4, 1), (70, 72, 24, 5, 2), (300, 256, 136, 16, 4), (40, 50, 17, 3, 3), (33, 128, 40, 130, 2),
-                                                         (129, 96, 64, 1, 1), (257, 64, 200, 33, 1)])
+                                                         (129, 96, 64, 1, 1), (257, 64, 200, 33, 1), (2500, 64, 32, 20, 3), (2111, 48, 16, 7, 2)])
 def test_mixture(gpu, dtype, block, tokens, width, ff, experts, top):
     g = torch.Generator().manual_seed(experts)
     h, router = torch.randn((tokens, width), generator=g).to(dtype), (torch.randn((experts, width), generator=g) * 4 * width ** -0.5).to(dtype)
