@@ -116,13 +116,14 @@ def random_weights(name, seed=0):
         out[k] = (out[k].float() + 0.8 * out[n].float()).to(torch.bfloat16)
     routed = [(i, layer["mlp"]["router"]) for i, layer in enumerate(cfg["layers"]) if layer["mlp"] and layer["mlp"]["kind"] == "moe"]
     open_, codes = torch.arange(cfg["vocab"]), out["embed"][:, :CODE].float()
+    read = {i: (out[f"l{i}.mlp.router"][:, :CODE].float() * out[f"l{i}.norm2"][:CODE].float()).T for i, _ in routed}
+    usual = {i: (codes @ r).pow(2).mean().sqrt() for i, r in read.items()}
     for _ in range(400):
         clear = torch.ones(len(open_), dtype=torch.bool)
         for i, r in routed:
             if r["top"] < r["experts"]:
-                z = (codes[open_] * out[f"l{i}.norm2"][:CODE].float()) @ out[f"l{i}.mlp.router"][:, :CODE].float().T
-                best = z.topk(r["top"] + 1, dim=-1).values
-                clear &= best[:, -2] - best[:, -1] > 0.1 * z.std(dim=-1)
+                best = (codes[open_] @ read[i]).topk(r["top"] + 1, dim=-1).values
+                clear &= best[:, -2] - best[:, -1] > 0.1 * usual[i]
         open_ = open_[~clear]
         if not len(open_):
             break
