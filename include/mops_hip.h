@@ -346,11 +346,36 @@ int mops_hip_norm_residual_add(float* residual, const void* y, int64_t y_row_str
                                float eps, void* act, int dtype, int64_t rows, int64_t n, void* stream);
 
 /*
- * Norms behind one sublayer and in front of the next: with y_r the sum of the rows r * parts .. r * parts + parts - 1 of y,
- * residual_r += y_r / sqrt(mean(y_r^2) + eps) * w_out in place, out_r = residual_r / sqrt(mean(residual_r^2) + eps) * w_in.
+ * residual = scale * table[id] + pairs[(token in front * mul_prev + id * mul_cur) mod buckets], and pairs[buckets] for a sequence's
+ * first token; table [vocab, width], pairs [buckets + 1, width].  The token in front of a sequence's first token of the step is
+ * before[state_slots[b]] (none where starts[b] == 0 or the slot is negative), which receives the sequence's last token.
+ * token_seq and cu_seqlens (both or neither): packed portions; NULL: one token per sequence.
  */
-int mops_hip_add_norm_norm(float* residual, const void* y, int64_t y_row_stride, int64_t parts, const void* w_out,
-                           const void* w_in, float eps, void* out, int dtype, int64_t rows, int64_t n, void* stream);
+typedef struct {
+  const int64_t* ids;
+  const void *table, *pairs;
+  int64_t table_stride, pairs_stride, buckets, mul_prev, mul_cur;
+  int32_t* before;
+  int64_t num_slots;
+  const int32_t *token_seq, *cu_seqlens, *starts, *state_slots;
+  float* residual;
+  int64_t tokens, vocab, width;
+  float scale;
+  int dtype;
+} mops_hip_embed_pairs_args;
+int mops_hip_embed_pairs(const mops_hip_embed_pairs_args* a, void* stream);
+
+/*
+ * Norms behind one sublayer and in front of the next: with y_r the sum of the rows r * parts .. r * parts + parts - 1 of y and of
+ * row r of extra ([rows, n], or NULL),
+ * residual_r += y_r / sqrt(mean(y_r^2) + eps) * w_out in place, out_r = residual_r / sqrt(mean(residual_r^2) + eps) * w_in.
+ * center: both norms take the mean of their row off first.
+ */
+int mops_hip_add_norm_norm(float* residual, const void* y, int64_t y_row_stride, int64_t parts, const void* extra, const void* w_out,
+                           const void* w_in, float eps, int center, void* out, int dtype, int64_t rows, int64_t n, void* stream);
+
+/* out = (x - mean(x)) / sqrt(mean((x - mean(x))^2) + eps) * weight of float32 rows. */
+int mops_hip_layer_norm_f32(const float* x, const void* weight, float eps, void* out, int dtype, int64_t rows, int64_t n, void* stream);
 
 /* out = x / sqrt(mean(x^2) + eps) * (weight_offset + weight) of float32 rows. */
 int mops_hip_rms_norm_f32(const float* x, const void* weight, float weight_offset, float eps, void* out, int dtype,
@@ -368,6 +393,9 @@ int mops_hip_gated_group_norm(const void* y, int64_t y_row_stride, const void* g
 /* out = g * sigmoid(alpha * g) * (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit). */
 int mops_hip_clamped_glu(const void* gate, int64_t gate_row_stride, const void* up, int64_t up_row_stride, void* out,
                          int dtype, int64_t rows, int64_t n, float alpha, float limit, void* stream);
+/* out = gelu(gate) * up, gelu(z) = z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))) / 2. */
+int mops_hip_gelu_glu(const void* gate, int64_t gate_row_stride, const void* up, int64_t up_row_stride, void* out, int dtype,
+                      int64_t rows, int64_t n, void* stream);
 
 /*
  * A linear recurrence with one decay per head and token (see csrc/decayed_recurrence.hip):
@@ -549,9 +577,35 @@ typedef struct {
 int mops_hip_attention_prepare(const mops_hip_attention_prepare_args* a, void* stream);
 
 /*
+ * rotary_prepare (csrc/rotary_prepare.hip): the same for rotated queries and keys.  q_weight, k_weight [dim] or NULL: an RMS norm over
+ * every head of q or k.  Then the pairs (i, i + rot / 2) of a head's first `rot` elements turn by the angles of the token's position:
+ * cos_sin float [max_positions, rot], cosines, then sines.
+ */
+typedef struct {
+  const void* qkv;
+  int64_t qkv_stride;
+  const void *q_weight, *k_weight;
+  const float* cos_sin;
+  int64_t max_positions, rot;
+  const int32_t *positions, *slot_mapping;
+  void *q, *k_pages, *v_pages;
+  int64_t num_slots, tokens, heads, kv_heads, dim, vdim;
+  float eps;
+  int dtype;
+} mops_hip_rotary_prepare_args;
+int mops_hip_rotary_prepare(const mops_hip_rotary_prepare_args* a, void* stream);
+
+/*
  * Query row r (at position context_lens[r] - 1) sees the first context_lens[r] tokens of sequence row_seq[r] (row r itself when
  * row_seq is NULL); 0 gives zeros.  score = q . k * scale - slopes[h] * distance (slopes float [heads], or NULL), softmax,
  * out [rows, heads, vdim].  A block table entry outside [0, num_blocks) counts as an empty block.
+ * Zeros in the fields behind dtype leave out what they describe:
+ *   softcap     score = softcap * tanh(q . k * scale / softcap); not together with slopes
+ *   window      position i sees the last `window` tokens up to itself
+ *   chunk       position i sees the tokens of its chunk up to itself, chunks of `chunk` tokens from position 0 on; not with window
+ *   keep_first  the first keep_first tokens stay visible
+ *   sinks       float [heads]: exp(sinks[h]) is one more term of the softmax's denominator
+ *   gate        `dtype` [rows, heads] with rows gate_stride apart: out is multiplied by its sigmoid
  * biased_attention_rows: the plain form; dim <= 2048, vdim <= 1024.
  */
 typedef struct {
@@ -563,6 +617,11 @@ typedef struct {
   int64_t rows, heads, kv_heads, dim, vdim;
   float scale;
   int dtype;
+  float softcap;
+  int64_t window, chunk, keep_first;
+  const float* sinks;
+  const void* gate;
+  int64_t gate_stride;
 } mops_hip_biased_attention;
 int mops_hip_biased_attention_rows(const mops_hip_biased_attention* a, void* stream);
 
@@ -586,12 +645,21 @@ int mops_hip_biased_prefill(const mops_hip_biased_attention* a, const int32_t* t
  * moe_gate_up: w [experts][2 * up_at][width], gate rows from 0, up rows from up_at on; y [tokens * top rows in the order of
  * `rows`], y = silu(score W_gate h) * (score W_up h).  moe_down: w [experts][width][depth], depth >= ff, the columns behind ff
  * zeros in w and finite in y; z [tokens * top] in the order of the choices.  experts <= 1024.
+ * The weighted form, groups > 0: the experts are `groups` equal runs of neighbours; a choice score is sigmoid(logit) + correction[e]
+ * (float [experts]), a group's score the sum of its two largest ones; the best `top` experts of the best `keep` groups are chosen, and
+ * score = factor * sigmoid(logit) over the sum of the chosen ones' + 1e-20.  moe_down multiplies by it, and moe_gate_up does not.
+ * unit 1: moe_gate_up gives g sigmoid(alpha g) (u + 1) with g = min(W_gate h, limit), u = W_up h between -limit and limit.
  */
 typedef struct {
   int32_t *rows, *tiles;
   float* score;
   int64_t tokens, experts, top, width, ff, block_rows;
   int dtype;
+  int unit;
+  float limit, alpha;
+  const float* correction;
+  int64_t groups, keep;
+  float factor;
 } mops_hip_moe;
 int64_t mops_hip_moe_max_tiles(int64_t tokens, int64_t experts, int64_t top, int64_t block_rows);
 int64_t mops_hip_moe_route_workgroups(int64_t tokens);

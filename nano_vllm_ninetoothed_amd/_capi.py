@@ -47,13 +47,30 @@ class BiasedAttention(Structure):
     _fields_ = ([(n, c_void_p) for n in ("q", "k_pages", "v_pages", "slopes", "row_seq", "context_lens", "block_table")]
                 + [(n, c_int64) for n in ("block_table_stride", "block_size", "num_blocks", "max_blocks")]
                 + [("out", c_void_p)] + [(n, c_int64) for n in ("rows", "heads", "kv_heads", "dim", "vdim")]
-                + [("scale", c_float), ("dtype", c_int)])
+                + [("scale", c_float), ("dtype", c_int), ("softcap", c_float)] + [(n, c_int64) for n in ("window", "chunk", "keep_first")]
+                + [("sinks", c_void_p), ("gate", c_void_p), ("gate_stride", c_int64)])
+
+
+class RotaryPrepare(Structure):
+    """mops_hip_rotary_prepare_args of the header, field by field."""
+    _fields_ = ([("qkv", c_void_p), ("qkv_stride", c_int64)] + [(n, c_void_p) for n in ("q_weight", "k_weight", "cos_sin")]
+                + [("max_positions", c_int64), ("rot", c_int64)] + [(n, c_void_p) for n in ("positions", "slot_mapping", "q", "k_pages", "v_pages")]
+                + [(n, c_int64) for n in ("num_slots", "tokens", "heads", "kv_heads", "dim", "vdim")] + [("eps", c_float), ("dtype", c_int)])
+
+
+class EmbedPairs(Structure):
+    """mops_hip_embed_pairs_args of the header, field by field."""
+    _fields_ = ([(n, c_void_p) for n in ("ids", "table", "pairs")]
+                + [(n, c_int64) for n in ("table_stride", "pairs_stride", "buckets", "mul_prev", "mul_cur")] + [("before", c_void_p), ("num_slots", c_int64)]
+                + [(n, c_void_p) for n in ("token_seq", "cu_seqlens", "starts", "state_slots", "residual")]
+                + [(n, c_int64) for n in ("tokens", "vocab", "width")] + [("scale", c_float), ("dtype", c_int)])
 
 
 class Moe(Structure):
     """mops_hip_moe of the header, field by field."""
     _fields_ = ([(n, c_void_p) for n in ("rows", "tiles", "score")]
-                + [(n, c_int64) for n in ("tokens", "experts", "top", "width", "ff", "block_rows")] + [("dtype", c_int)])
+                + [(n, c_int64) for n in ("tokens", "experts", "top", "width", "ff", "block_rows")] + [("dtype", c_int), ("unit", c_int)]
+                + [("limit", c_float), ("alpha", c_float), ("correction", c_void_p), ("groups", c_int64), ("keep", c_int64), ("factor", c_float)])
 
 
 # name -> (restype, argtypes); the exported surface declared in include/mops_hip.h
@@ -98,12 +115,15 @@ SIGNATURES = {
     "mops_hip_embed_residual": (c_int, [c_void_p, c_void_p, c_int64, c_int, c_float, c_void_p, c_void_p, c_int64, c_int64, c_int64, c_void_p]),
     "mops_hip_norm_residual_add": (c_int, [c_void_p, c_void_p, c_int64, c_void_p, c_float, c_float, c_void_p, c_int, c_int64, c_int64,
                                            c_void_p]),
-    "mops_hip_add_norm_norm": (c_int, [c_void_p, c_void_p, c_int64, c_int64, c_void_p, c_void_p, c_float, c_void_p, c_int, c_int64, c_int64,
-                                       c_void_p]),
+    "mops_hip_add_norm_norm": (c_int, [c_void_p, c_void_p, c_int64, c_int64, c_void_p, c_void_p, c_void_p, c_float, c_int, c_void_p, c_int, c_int64,
+                                       c_int64, c_void_p]),
+    "mops_hip_layer_norm_f32": (c_int, [c_void_p, c_void_p, c_float, c_void_p, c_int, c_int64, c_int64, c_void_p]),
+    "mops_hip_embed_pairs": (c_int, [POINTER(EmbedPairs), c_void_p]),
     "mops_hip_rms_norm_f32": (c_int, [c_void_p, c_void_p, c_float, c_float, c_void_p, c_int, c_int64, c_int64, c_void_p]),
     "mops_hip_gated_group_norm": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_float, c_int, c_void_p, c_int, c_int64,
                                           c_int64, c_int64, c_void_p]),
     "mops_hip_clamped_glu": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int, c_int64, c_int64, c_float, c_float, c_void_p]),
+    "mops_hip_gelu_glu": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int, c_int64, c_int64, c_void_p]),
     "mops_hip_recurrence_state_pitch": (c_int64, [c_int64]),
     "mops_hip_decayed_recurrence": (c_int, [POINTER(Recurrence), c_void_p]),
     "mops_hip_decayed_chunks_workgroups": (c_int64, [c_int64] * 3),
@@ -131,6 +151,7 @@ SIGNATURES = {
     "mops_hip_low_rank_decay": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int, c_int64, c_int64, c_int64, c_void_p]),
     "mops_hip_squared_relu": (c_int, [c_void_p, c_int64, c_void_p, c_int, c_int64, c_int64, c_void_p]),
     "mops_hip_attention_prepare": (c_int, [POINTER(AttentionPrepare), c_void_p]),
+    "mops_hip_rotary_prepare": (c_int, [POINTER(RotaryPrepare), c_void_p]),
     "mops_hip_biased_attention_rows": (c_int, [POINTER(BiasedAttention), c_void_p]),
     "mops_hip_biased_decode_workspace_bytes": (c_int64, [c_int64] * 5),
     "mops_hip_biased_decode": (c_int, [POINTER(BiasedAttention), c_void_p, c_int64, c_void_p]),
@@ -145,7 +166,7 @@ SIGNATURES = {
     "mops_hip_linear_tune": (c_int, [c_int64, c_int64, c_int64, c_int64, c_int, c_void_p, c_int64, c_void_p, c_void_p, c_void_p]),
 }
 
-ABI_VERSION = 11
+ABI_VERSION = 12
 
 _lib = None
 

@@ -1,11 +1,13 @@
 // Causal attention over paged keys and values with a linear distance bias per head:
 //   score(i, j) = (q_i . k_j) * scale - slope_h (i - j),  j <= i,  softmax over j,  query head h reads key/value head h / (H / G).
+// Instead of the bias a cap on the scores, and as options: a window or chunks with kept first tokens (visible.h), a sink in the
+// softmax's denominator, a gate on the output.
 // Key and value sizes are independent of each other; pages hold [block][offset][G][size rounded up to 8], zeros behind the size.
 //
 //   attention_prepare       from the packed projections [q | k | v] of every token: RMS norm with plain weights over the whole of
 //                           q and over the whole of k, a factor per position on q, scatter of k and v into their pages
 //   biased_attention_rows   one query row at a time, on vector units.  The plain form: any size, bf16 or float.
-#include "mixed_types.h"
+#include "visible.h"
 
 namespace mops {
 
@@ -78,6 +80,7 @@ __global__ __launch_bounds__(256) void biased_attention_rows_kernel(const mops_h
   const T* q = (const T*)a.q + (row * a.heads + h) * dp;
   for (int i = tid; i < dim; i += 256) sq[i] = to_f32(q[i]);
   const float slope = a.slopes ? a.slopes[h] : 0.f;
+  const Visible see = visible_at(a, len);
   const int seq = a.row_seq ? a.row_seq[row] : (int)row;
   const int32_t* table = a.block_table + (int64_t)seq * a.block_table_stride;
   auto token_row = [&](int j) -> int64_t {      // the row of token j in the pages, -1 without one
@@ -86,22 +89,27 @@ __global__ __launch_bounds__(256) void biased_attention_rows_kernel(const mops_h
     const int id = table[blk];
     return id < 0 || id >= a.num_blocks ? -1 : (int64_t)id * a.block_size + j % (int)a.block_size;
   };
-  float m = -INFINITY, l = 0.f;
+  float m = a.sinks ? a.sinks[h] : -INFINITY, l = a.sinks ? 1.f : 0.f;      // a sink is a key with a value of zeros
   float acc[kRowMaxValue / 256];
 #pragma unroll
   for (int i = 0; i < kRowMaxValue / 256; ++i) acc[i] = 0.f;
   for (int k0 = 0; k0 < len; k0 += kRowKeys) {
+    if (k0 >= see.kept && k0 + kRowKeys <= see.lo) k0 = see.lo / kRowKeys * kRowKeys;      // nothing to see up to there
     __syncthreads();
     for (int kk = r16; kk < kRowKeys; kk += 16) {
       const int j = k0 + kk;
-      const int64_t r = j < len ? token_row(j) : -1;
+      const int64_t r = j < len && (j >= see.lo || j < see.kept) ? token_row(j) : -1;
       float dot = 0.f;
       if (r >= 0) {
         const T* kr = (const T*)a.k_pages + (r * groups + g) * dp;
         for (int i = ln; i < dim; i += 16) dot += sq[i] * to_f32(kr[i]);
       }
       dot = group_sum<16>(dot);
-      if (ln == 0) sp[kk] = r >= 0 ? dot * a.scale - slope * (float)(len - 1 - j) : -INFINITY;
+      if (ln == 0) {
+        dot *= a.scale;
+        if (a.softcap > 0.f) dot = a.softcap * tanhf(dot / a.softcap);
+        sp[kk] = r >= 0 ? dot - slope * (float)(len - 1 - j) : -INFINITY;
+      }
     }
     __syncthreads();
     float mx = group_max<kWave>(sp[tid]);
@@ -123,16 +131,17 @@ __global__ __launch_bounds__(256) void biased_attention_rows_kernel(const mops_h
     for (int i = 0; i < kRowMaxValue / 256; ++i) acc[i] *= alpha;
     const int n = len - k0 < kRowKeys ? len - k0 : kRowKeys;
     for (int kk = 0; kk < n; ++kk) {
-      const int64_t r = token_row(k0 + kk);
-      if (r < 0) continue;
       const float w = sp[kk];
+      const int64_t r = w != 0.f ? token_row(k0 + kk) : -1;
+      if (r < 0) continue;
       const T* vr = (const T*)a.v_pages + (r * groups + g) * vp;
 #pragma unroll
       for (int i = 0; i < kRowMaxValue / 256; ++i)
         if (tid + 256 * i < vdim) acc[i] += w * to_f32(vr[tid + 256 * i]);
     }
   }
-  const float inv = l > 0.f ? 1.0f / l : 0.f;
+  float inv = l > 0.f ? 1.0f / l : 0.f;
+  if (a.gate) inv *= sigmoid_for<T>(to_f32(((const T*)a.gate)[row * a.gate_stride + h]));
 #pragma unroll
   for (int i = 0; i < kRowMaxValue / 256; ++i)
     if (tid + 256 * i < vdim) out[tid + 256 * i] = from_f32<T>(acc[i] * inv);
@@ -145,6 +154,9 @@ int check_biased_attention(const mops_hip_biased_attention* a) {
   if (!a->q || !a->k_pages || !a->v_pages || !a->context_lens || !a->block_table || !a->out) return MOPS_HIP_EINVAL;
   if (a->heads <= 0 || a->kv_heads <= 0 || a->heads % a->kv_heads || a->dim <= 0 || a->vdim <= 0) return MOPS_HIP_EINVAL;
   if (a->block_size <= 0 || a->num_blocks <= 0 || a->max_blocks <= 0 || a->block_table_stride < a->max_blocks) return MOPS_HIP_EINVAL;
+  if (a->window < 0 || a->chunk < 0 || a->keep_first < 0 || (a->window && a->chunk)) return MOPS_HIP_EINVAL;
+  if (!(a->softcap >= 0.f) || (a->softcap > 0.f && a->slopes) || (a->gate && a->gate_stride < a->heads)) return MOPS_HIP_EINVAL;
+  if (a->window > kMaxRange || a->chunk > kMaxRange || a->keep_first > kMaxRange) return MOPS_HIP_EUNSUPPORTED;
   if (a->rows * a->heads > 0x7fffffffLL || a->block_size > (1 << 20) || a->max_blocks * a->block_size > (1 << 28)) return MOPS_HIP_EUNSUPPORTED;
   return 1;
 }

@@ -10,7 +10,10 @@
 //   O^T [v, head]    += V^T P^T      V^T through transposing LDS reads, P as the sum of two bf16 numbers
 // A row that lies inside one run is written at once.  A row that is cut leaves (max, sum, unnormalised O) in one of the two slots
 // of each run it touches; biased_combine_kernel merges them and writes the rows without any context as zeros.
+// Where rows see a part of their sequence only, their stages are those with something to see.  A sink enters with a row's first
+// stage, as a token with a value of zeros.
 #include "mfma_tiles.h"
+#include "visible.h"
 
 namespace mops {
 
@@ -27,7 +30,7 @@ struct BiasedDecodeArgs {
 };
 
 // NK: 32-deep steps of the key (dim <= 32 NK); NV: 16-wide pieces of the value (vdim <= 16 NV)
-template <int NK, int NV>
+template <int NK, int NV, ScoreKind KIND>
 __global__ __launch_bounds__(64, NK * 32 + NV * 16 <= 256 ? 2 : 1) void biased_decode_kernel(const BiasedDecodeArgs p) {
   constexpr int kPitchK = 32 * NK + 8, kPitchV = 16 * NV + 8;
   constexpr int kPiecesK = 4 * NK, kPiecesV = 2 * NV;               // 16-byte pieces of a row
@@ -48,7 +51,12 @@ __global__ __launch_bounds__(64, NK * 32 + NV * 16 <= 256 ? 2 : 1) void biased_d
     const int l = a.context_lens[r];
     return l < 0 ? 0 : (l < max_tokens ? l : max_tokens);
   };
-  auto stages_of = [&](int r) { return (length_of(r) + kStage - 1) / kStage; };
+  const int keep_first = (int)a.keep_first;
+  auto blocks_of = [&](int len) { return VisibleBlocks<kStage>(visible_at(a, len).lo, keep_first); };
+  auto stages_of = [&](int r) {
+    const int len = length_of(r);
+    return blocks_of(len).count(len);
+  };
 
   // ---- this workgroup's run
   int row = 0, stage0 = 0, remaining;
@@ -120,15 +128,18 @@ __global__ __launch_bounds__(64, NK * 32 + NV * 16 <= 256 ? 2 : 1) void biased_d
     return ok;
   };
   const float scale = a.scale * 1.4426950408889634f;
-  const float slope = a.slopes ? a.slopes[h] * 1.4426950408889634f : 0.f;
+  const float slope = KIND == kSloped && a.slopes ? a.slopes[h] * 1.4426950408889634f : 0.f;
+  const CappedScore capped(a);
+  const float sink = a.sinks ? a.sinks[h] * 1.4426950408889634f : -INFINITY;
 
   for (; remaining > 0; ++row, stage0 = 0) {
-    const int len = __builtin_amdgcn_readfirstlane(length_of(row)), row_stages = (len + kStage - 1) / kStage;
+    const int len = __builtin_amdgcn_readfirstlane(length_of(row));
+    const Visible see = visible_at(a, len);
+    const VisibleBlocks<kStage> blocks(see.lo, keep_first);
+    const int row_stages = blocks.count(len);
     const int run = row_stages - stage0 < remaining ? row_stages - stage0 : remaining;
     if (run <= 0) continue;
     remaining -= run;
-    const int tok_begin = stage0 * kStage;
-    const int tok_end = tok_begin + run * kStage < len ? tok_begin + run * kStage : len;
     table = a.block_table + (int64_t)(a.row_seq ? a.row_seq[row] : row) * a.block_table_stride;
     const uint16_t* q = (const uint16_t*)a.q + ((int64_t)row * heads + h) * dp;
     bf16x8 qb[NK];
@@ -137,14 +148,16 @@ __global__ __launch_bounds__(64, NK * 32 + NV * 16 <= 256 ? 2 : 1) void biased_d
       const int c = 32 * i + 8 * jj;
       qb[i] = __builtin_bit_cast(bf16x8, head_ok && c < dp ? load16(q + c) : u32x4{0u, 0u, 0u, 0u});
     }
-    bool ok_next = issue(tok_begin);
+    bool ok_next = issue(blocks.token(stage0));
     f32x4 acc[NV];
 #pragma unroll
     for (int i = 0; i < NV; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-    float m_run = -INFINITY, l_run = 0.f;
+    float m_run = KIND == kCappedFixed ? 0.f : (stage0 == 0 ? sink : -INFINITY);
+    float l_run = stage0 == 0 && jj == 0 && a.sinks ? __builtin_amdgcn_exp2f(sink - m_run) : 0.f;
 
-    for (int tok0 = tok_begin; tok0 < tok_end; tok0 += kStage) {
-      const int valid = ok_next ? (tok_end - tok0 < kStage ? tok_end - tok0 : kStage) : 0;
+    for (int st = stage0; st < stage0 + run; ++st) {
+      const int tok0 = blocks.token(st);
+      const int valid = ok_next ? (len - tok0 < kStage ? len - tok0 : kStage) : 0;
 #pragma unroll
       for (int j = 0; j < kLoadsK; ++j) store16(tk + k_lds[j], kreg[j]);
 #pragma unroll
@@ -154,7 +167,7 @@ __global__ __launch_bounds__(64, NK * 32 + NV * 16 <= 256 ? 2 : 1) void biased_d
         for (int j = 0; j < kLoadsV; ++j)
           if ((lane + 64 * j) / kPiecesV >= valid) store16(tv + v_lds[j], u32x4{0u, 0u, 0u, 0u});
       }
-      if (tok0 + kStage < tok_end) ok_next = issue(tok0 + kStage);
+      if (st + 1 < stage0 + run) ok_next = issue(blocks.token(st + 1));
       __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
       __builtin_amdgcn_wave_barrier();
       __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
@@ -170,15 +183,27 @@ __global__ __launch_bounds__(64, NK * 32 + NV * 16 <= 256 ? 2 : 1) void biased_d
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
         const int t = 4 * jj + (e & 3) + 16 * (e >> 2);
-        const float x = s[e >> 2][e & 3] * scale + slope * (dist + (float)((e & 3) + 16 * (e >> 2)));
+        const float x = KIND == kSloped ? s[e >> 2][e & 3] * scale + slope * (dist + (float)((e & 3) + 16 * (e >> 2))) : capped(s[e >> 2][e & 3]);
         sv[e] = t < valid ? x : -INFINITY;
-        m_loc = fmaxf(m_loc, sv[e]);
       }
-      m_loc = fmaxf(m_loc, __shfl_xor(m_loc, 16, kWave));
-      m_loc = fmaxf(m_loc, __shfl_xor(m_loc, 32, kWave));
-      const float m_new = fmaxf(m_run, m_loc);
-      const float m_safe = m_new == -INFINITY ? 0.f : m_new;
-      const float alpha = __builtin_amdgcn_exp2f(m_run - m_safe);
+      if (tok0 < see.lo && tok0 + kStage > see.kept) {      // the edge of what the row sees
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          const int t = tok0 + 4 * jj + (e & 3) + 16 * (e >> 2);
+          sv[e] = t >= see.lo || t < see.kept ? sv[e] : -INFINITY;
+        }
+      }
+      float m_safe = 0.f, alpha = 1.f;
+      if (KIND != kCappedFixed) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) m_loc = fmaxf(m_loc, sv[e]);
+        m_loc = fmaxf(m_loc, __shfl_xor(m_loc, 16, kWave));
+        m_loc = fmaxf(m_loc, __shfl_xor(m_loc, 32, kWave));
+        const float m_new = fmaxf(m_run, m_loc);
+        m_safe = m_new == -INFINITY ? 0.f : m_new;
+        alpha = __builtin_amdgcn_exp2f(m_run - m_safe);
+        m_run = m_new;
+      }
       float pv[8], psum = 0.f;
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
@@ -186,8 +211,7 @@ __global__ __launch_bounds__(64, NK * 32 + NV * 16 <= 256 ? 2 : 1) void biased_d
         psum += pv[e];
       }
       l_run = l_run * alpha + psum;
-      m_run = m_new;
-      if (__any(alpha != 1.0f)) {
+      if (KIND != kCappedFixed && __any(alpha != 1.0f)) {
 #pragma unroll
         for (int i = 0; i < NV; ++i) acc[i] *= alpha;
       }
@@ -207,7 +231,8 @@ __global__ __launch_bounds__(64, NK * 32 + NV * 16 <= 256 ? 2 : 1) void biased_d
     l_tot += __shfl_xor(l_tot, 32, kWave);
     if (!head_ok) continue;
     if (run == row_stages) {
-      const float inv = l_tot > 0.f ? 1.0f / l_tot : 0.f;
+      float inv = l_tot > 0.f ? 1.0f / l_tot : 0.f;
+      if (a.gate) inv *= sigmoid_for<bf16_t>(to_f32(((const bf16_t*)a.gate)[row * a.gate_stride + h]));
       uint16_t* orow = (uint16_t*)a.out + ((int64_t)row * heads + h) * vdim;
 #pragma unroll
       for (int i = 0; i < NV; ++i) {
@@ -257,7 +282,8 @@ __global__ __launch_bounds__(64) void biased_combine_kernel(const BiasedDecodeAr
   float l = 0.f;
   for (int j = j0 + lane; j <= j1; j += kWave) l += __builtin_amdgcn_exp2f(p.ml[2 * slot_of(j)] - safe) * p.ml[2 * slot_of(j) + 1];
   l = group_sum<kWave>(l);
-  const float inv = l > 0.f ? 1.0f / l : 0.f;
+  float inv = l > 0.f ? 1.0f / l : 0.f;
+  if (a.gate) inv *= sigmoid_for<bf16_t>(to_f32(((const bf16_t*)a.gate)[row * a.gate_stride + h]));
   for (int v0 = 0; v0 < vdim; v0 += 4 * kWave) {
     float o[4] = {0.f, 0.f, 0.f, 0.f};
     for (int j = j0; j <= j1; ++j) {
@@ -288,13 +314,21 @@ static int decode_columns(int64_t dim, int64_t vdim, int64_t planes) {
 static int64_t decode_plan_bytes(int64_t rows) { return ((rows + 2) * 4 + 255) / 256 * 256; }
 static int64_t head_tiles_of(int64_t heads, int64_t kv_heads) { return (heads / kv_heads + kPlaneHeads - 1) / kPlaneHeads; }
 
-template <int NK>
+template <int NK, ScoreKind KIND>
 static void launch_decode_keys(const BiasedDecodeArgs& p, dim3 grid, hipStream_t s) {
   const int64_t v = p.a.vdim;
-  if (v <= 32) hipLaunchKernelGGL((biased_decode_kernel<NK, 2>), grid, dim3(64), 0, s, p);
-  else if (v <= 64) hipLaunchKernelGGL((biased_decode_kernel<NK, 4>), grid, dim3(64), 0, s, p);
-  else if (v <= 128) hipLaunchKernelGGL((biased_decode_kernel<NK, 8>), grid, dim3(64), 0, s, p);
-  else hipLaunchKernelGGL((biased_decode_kernel<NK, 16>), grid, dim3(64), 0, s, p);
+  if (v <= 32) hipLaunchKernelGGL((biased_decode_kernel<NK, 2, KIND>), grid, dim3(64), 0, s, p);
+  else if (v <= 64) hipLaunchKernelGGL((biased_decode_kernel<NK, 4, KIND>), grid, dim3(64), 0, s, p);
+  else if (v <= 128) hipLaunchKernelGGL((biased_decode_kernel<NK, 8, KIND>), grid, dim3(64), 0, s, p);
+  else hipLaunchKernelGGL((biased_decode_kernel<NK, 16, KIND>), grid, dim3(64), 0, s, p);
+}
+template <ScoreKind KIND>
+static void launch_decode(const BiasedDecodeArgs& p, dim3 grid, hipStream_t s) {
+  const int64_t d = p.a.dim;
+  if (d <= 32) launch_decode_keys<1, KIND>(p, grid, s);
+  else if (d <= 64) launch_decode_keys<2, KIND>(p, grid, s);
+  else if (d <= 128) launch_decode_keys<4, KIND>(p, grid, s);
+  else launch_decode_keys<8, KIND>(p, grid, s);
 }
 
 }  // namespace mops
@@ -327,10 +361,10 @@ extern "C" int mops_hip_biased_decode(const mops_hip_biased_attention* a, void* 
   p.ml = p.part + planes * p.columns * 2 * kPlaneHeads * a->vdim;
   const dim3 grid((unsigned)(planes * p.columns));
   hipStream_t s = (hipStream_t)stream;
-  if (a->dim <= 32) launch_decode_keys<1>(p, grid, s);
-  else if (a->dim <= 64) launch_decode_keys<2>(p, grid, s);
-  else if (a->dim <= 128) launch_decode_keys<4>(p, grid, s);
-  else launch_decode_keys<8>(p, grid, s);
+  const ScoreKind kind = score_kind(*a);
+  if (kind == kCappedFixed) launch_decode<kCappedFixed>(p, grid, s);
+  else if (kind == kCapped) launch_decode<kCapped>(p, grid, s);
+  else launch_decode<kSloped>(p, grid, s);
   hipLaunchKernelGGL(biased_combine_kernel, dim3((unsigned)(a->rows * a->heads)), dim3(64), 0, s, p);
   return finish_launch();
 }

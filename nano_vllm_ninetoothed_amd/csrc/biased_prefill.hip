@@ -5,7 +5,9 @@
 // flight into registers; a thread looks its token's page up one tile ahead.  v_mfma_f32_32x32x16_bf16 throughout:
 //   S^T [key, query] = K Q^T        the softmax runs over keys: in a lane and its partner in the other half
 //   O^T [v, query]  += V^T P^T      V^T through transposing LDS reads, P from the accumulators of S^T as the sum of two bf16 numbers
+// Key tiles of which no query of a workgroup sees anything are left out, and a wave leaves out those of which its queries see nothing.
 #include "mfma_tiles.h"
+#include "visible.h"
 
 namespace mops {
 
@@ -18,7 +20,7 @@ struct BiasedPrefillArgs {
 };
 
 // NK: 16-deep steps of the key (dim <= 16 NK), NV: 32-wide pieces of the value (vdim <= 32 NV)
-template <int NK, int NV>
+template <int NK, int NV, ScoreKind KIND>
 __global__ __launch_bounds__(256, NK <= 8 && NV <= 4 ? 2 : 1) void biased_prefill_kernel(const BiasedPrefillArgs p) {
   constexpr int kPitchK = NK * 16 + 8, kPitchV = NV * 32 + 8;
   constexpr int kLoadsK = NK / 2, kLoadsV = NV;      // 16-byte pieces of a thread: columns 8 (tid % 4) + 32 j of token tid / 4
@@ -50,13 +52,23 @@ __global__ __launch_bounds__(256, NK <= 8 && NV <= 4 ? 2 : 1) void biased_prefil
   for (int i = 0; i < NV; ++i)
 #pragma unroll
     for (int r = 0; r < 16; ++r) o[i][r] = 0.f;
-  float m_run = -INFINITY, l_run = 0.f;
+  const float sink = a.sinks ? a.sinks[h] * 1.4426950408889634f : -INFINITY;      // a token with a value of zeros
+  float m_run = KIND == kCappedFixed ? 0.f : sink, l_run = a.sinks && hh == 0 ? __builtin_amdgcn_exp2f(sink - m_run) : 0.f;
 
   const int visible = pos0 + q_count < keys ? pos0 + q_count : keys;      // keys any query of the tile sees
+  const int keep = (int)a.keep_first, pos_first = pos0 + 32 * wave;      // of the wave's queries
+  const VisibleBlocks<kPrefillKeys> blocks(first_visible(a, pos0), keep);
+  const int n_blocks = blocks.count(visible);
+  const int lo = first_visible(a, pos), lo_first = first_visible(a, pos_first), lo_last = first_visible(a, pos_first + 31);
   const int krow = tid >> 2, kcol = (tid & 3) * 8;
   u32x4 kreg[kLoadsK], vreg[kLoadsV];
-  int j_next = krow, blk_next = krow / bs, in_blk = krow % bs;      // the token page_of looks up next
+  int block_next = 0, j_next = krow, blk_next = krow / bs, in_blk = krow % bs;      // the token page_of looks up next
   auto page_of = [&]() {      // row of this thread's next token in the pages, -1 without one
+    if (block_next++ == blocks.kept && blocks.first > blocks.kept) {
+      j_next = kPrefillKeys * blocks.first + krow;
+      blk_next = j_next / bs;
+      in_blk = j_next % bs;
+    }
     int64_t row = -1;
     if (j_next < visible && blk_next < a.max_blocks) {
       const int id = table[blk_next];
@@ -82,21 +94,23 @@ __global__ __launch_bounds__(256, NK <= 8 && NV <= 4 ? 2 : 1) void biased_prefil
     }
   };
   const float scale = a.scale * 1.4426950408889634f;
-  const float slope = a.slopes ? a.slopes[h] * 1.4426950408889634f : 0.f;
+  const float slope = KIND == kSloped && a.slopes ? a.slopes[h] * 1.4426950408889634f : 0.f;
+  const CappedScore capped(a);
   issue(page_of());
   int64_t next_row = page_of();
-  for (int k0 = 0; k0 < visible; k0 += kPrefillKeys) {
+  for (int block = 0; block < n_blocks; ++block) {
+    const int k0 = blocks.token(block);
     __syncthreads();
 #pragma unroll
     for (int j = 0; j < kLoadsK; ++j) store16(tk + krow * kPitchK + kcol + 32 * j, kreg[j]);
 #pragma unroll
     for (int j = 0; j < kLoadsV; ++j) store16(tv + krow * kPitchV + kcol + 32 * j, vreg[j]);
     __syncthreads();
-    if (k0 + kPrefillKeys < visible) {
+    if (block + 1 < n_blocks) {
       issue(next_row);
       next_row = page_of();
     }
-    if (k0 > pos0 + 32 * wave + 31) continue;           // this wave's queries see none of the tile
+    if (k0 > pos_first + 31 || (k0 >= keep && k0 + kPrefillKeys <= lo_first)) continue;      // this wave's queries see none of the tile
     f32x16 s[2];
 #pragma unroll
     for (int kt = 0; kt < 2; ++kt)
@@ -109,13 +123,16 @@ __global__ __launch_bounds__(256, NK <= 8 && NV <= 4 ? 2 : 1) void biased_prefil
     float m_loc = -INFINITY;
     const int last = pos < keys - 1 ? pos : keys - 1;
     const float dist = (float)(k0 + 4 * hh - pos);      // of the lane's first key, in front of the query by its negative
-    if (k0 + kPrefillKeys - 1 > pos0 + 32 * wave || k0 + kPrefillKeys > keys) {      // the diagonal or the end of the context: mask
+    // the diagonal, the end of the context or of what is visible: mask
+    if (k0 + kPrefillKeys - 1 > pos_first || k0 + kPrefillKeys > keys || (k0 < lo_last && k0 + kPrefillKeys > keep)) {
 #pragma unroll
       for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
         for (int r = 0; r < 16; ++r) {
           const int off = 32 * kt + 8 * (r >> 2) + (r & 3);
-          s[kt][r] = k0 + 4 * hh + off <= last ? s[kt][r] * scale + slope * (dist + (float)off) : -INFINITY;
+          const int j = k0 + 4 * hh + off;
+          const float x = KIND == kSloped ? s[kt][r] * scale + slope * (dist + (float)off) : capped(s[kt][r]);
+          s[kt][r] = j <= last && (j >= lo || j < keep) ? x : -INFINITY;
           m_loc = fmaxf(m_loc, s[kt][r]);
         }
     } else {
@@ -124,19 +141,22 @@ __global__ __launch_bounds__(256, NK <= 8 && NV <= 4 ? 2 : 1) void biased_prefil
 #pragma unroll
         for (int r = 0; r < 16; ++r) {
           const int off = 32 * kt + 8 * (r >> 2) + (r & 3);
-          s[kt][r] = s[kt][r] * scale + slope * (dist + (float)off);
+          s[kt][r] = KIND == kSloped ? s[kt][r] * scale + slope * (dist + (float)off) : capped(s[kt][r]);
           m_loc = fmaxf(m_loc, s[kt][r]);
         }
     }
-    m_loc = fmaxf(m_loc, __shfl_xor(m_loc, 32, kWave));
-    const float m_new = fmaxf(m_run, m_loc);
-    const float m_safe = m_new == -INFINITY ? 0.f : m_new;
-    const float alpha = __builtin_amdgcn_exp2f(m_run - m_safe);
-    m_run = m_new;
-    if (__any(alpha != 1.0f)) {
-      l_run *= alpha;
+    float m_safe = 0.f;
+    if (KIND != kCappedFixed) {
+      m_loc = fmaxf(m_loc, __shfl_xor(m_loc, 32, kWave));
+      const float m_new = fmaxf(m_run, m_loc);
+      m_safe = m_new == -INFINITY ? 0.f : m_new;
+      const float alpha = __builtin_amdgcn_exp2f(m_run - m_safe);
+      m_run = m_new;
+      if (__any(alpha != 1.0f)) {
+        l_run *= alpha;
 #pragma unroll
-      for (int i = 0; i < NV; ++i) o[i] *= alpha;
+        for (int i = 0; i < NV; ++i) o[i] *= alpha;
+      }
     }
 #pragma unroll
     for (int kt = 0; kt < 2; ++kt)
@@ -162,7 +182,8 @@ __global__ __launch_bounds__(256, NK <= 8 && NV <= 4 ? 2 : 1) void biased_prefil
   }
   if (!q_ok) return;
   const float l = l_run + __shfl_xor(l_run, 32, kWave);
-  const float inv = l > 0.f ? 1.0f / l : 0.f;
+  float inv = l > 0.f ? 1.0f / l : 0.f;
+  if (a.gate) inv *= sigmoid_for<bf16_t>(to_f32(((const bf16_t*)a.gate)[(q_begin + qi) * a.gate_stride + h]));
   uint16_t* orow = (uint16_t*)a.out + ((int64_t)(q_begin + qi) * heads + h) * vdim;
 #pragma unroll
   for (int i = 0; i < NV; ++i)
@@ -182,6 +203,17 @@ __global__ __launch_bounds__(256, NK <= 8 && NV <= 4 ? 2 : 1) void biased_prefil
 
 int check_biased_attention(const mops_hip_biased_attention* a);   // biased_attention.hip
 
+template <ScoreKind KIND>
+static void launch_prefill(const BiasedPrefillArgs& p, dim3 grid, hipStream_t s) {
+#define MOPS_BP(K, V) hipLaunchKernelGGL((biased_prefill_kernel<K, V, KIND>), grid, dim3(256), 0, s, p)
+#define MOPS_BP_K(V) do { if (p.a.dim <= 64) MOPS_BP(4, V); else if (p.a.dim <= 128) MOPS_BP(8, V); else MOPS_BP(16, V); } while (0)
+  if (p.a.vdim <= 64) MOPS_BP_K(2);
+  else if (p.a.vdim <= 128) MOPS_BP_K(4);
+  else MOPS_BP_K(8);
+#undef MOPS_BP_K
+#undef MOPS_BP
+}
+
 }  // namespace mops
 
 extern "C" int mops_hip_biased_prefill(const mops_hip_biased_attention* args, const int32_t* tiles, int64_t num_tiles, void* stream) {
@@ -196,14 +228,11 @@ extern "C" int mops_hip_biased_prefill(const mops_hip_biased_attention* args, co
   p.a = *args;
   p.tiles = tiles;
   p.vec_out = args->vdim % 4 == 0 && aligned16(args->out);
-  const dim3 grid((unsigned)(num_tiles * args->heads)), block(256);
+  const dim3 grid((unsigned)(num_tiles * args->heads));
   hipStream_t s = (hipStream_t)stream;
-#define MOPS_BP(K, V) hipLaunchKernelGGL((biased_prefill_kernel<K, V>), grid, block, 0, s, p)
-#define MOPS_BP_K(V) do { if (args->dim <= 64) MOPS_BP(4, V); else if (args->dim <= 128) MOPS_BP(8, V); else MOPS_BP(16, V); } while (0)
-  if (args->vdim <= 64) MOPS_BP_K(2);
-  else if (args->vdim <= 128) MOPS_BP_K(4);
-  else MOPS_BP_K(8);
-#undef MOPS_BP_K
-#undef MOPS_BP
+  const ScoreKind kind = score_kind(*args);
+  if (kind == kCappedFixed) launch_prefill<kCappedFixed>(p, grid, s);
+  else if (kind == kCapped) launch_prefill<kCapped>(p, grid, s);
+  else launch_prefill<kSloped>(p, grid, s);
   return finish_launch();
 }

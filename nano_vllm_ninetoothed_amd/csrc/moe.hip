@@ -3,8 +3,11 @@
 //   moe_route    logits = router h in float32, the top choices per token, their sigmoid scores, and where each choice lands when
 //                all choices are ordered by expert: row = (choices of earlier experts) + rank.  rows[] lists the choices (token *
 //                top + place) by row; tiles[] cuts each expert's rows into blocks of `block_rows`.
-//   moe_gate_up  y[row] = silu(s W_gate h) * (s W_up h) with h the token's row and s its score: the score scales the expert's input
-//   moe_down     z[choice] = W_down y[row]
+//                Or the score is a choice's weight: experts are chosen by sigmoid + correction among those of the best groups of
+//                neighbours, and the weights are their sigmoids over the sum of these, times a factor.
+//   moe_gate_up  y[row] = silu(s W_gate h) * (s W_up h) with h the token's row and s its score: the score scales the expert's input;
+//                or g sigmoid(alpha g) (u + 1) with g = min(W_gate h, limit), u = W_up h between -limit and limit
+//   moe_down     z[choice] = W_down y[row], times the choice's weight in the second form
 //   grouped_linear   the products of the small blocks without routing: equal runs of rows, each with weights of its own
 //
 // The products are grouped: a workgroup takes a block of rows of one expert and some of its outputs.  Nothing comes back to the
@@ -25,7 +28,89 @@ struct RouteArgs {
   int tokens, width, experts, top, per_wg;      // per_wg: tokens of a route workgroup, 16 or 32
   int32_t *chosen, *rank, *counts;     // [tokens * top], [tokens * top], [workgroups][experts]
   float* score;                        // [tokens * top]
+  // the weighted form, with groups > 0
+  const float* correction;             // [experts]
+  int groups, keep;
+  float factor;
 };
+
+// The weighted form, for LANES lanes per token (lane x owns the experts x, x + LANES, ...; N of them at most).  On entry score[e] is
+// the sigmoid of expert e, choice[e] the same plus its correction, in LDS for all lanes of the token; group_score has room for the
+// groups.  The lanes of a token run together: `together` orders their accesses to LDS.
+template <int LANES, int N, typename Sync>
+__device__ __forceinline__ void choose_weighted(const RouteArgs& a, const float* score, const float* choice, float* group_score, int x, int token, Sync together) {
+  const int size = a.experts / a.groups;
+  for (int g = x; g < a.groups; g += LANES) {      // the two best of a group
+    float first = -INFINITY, second = -INFINITY;
+    for (int e = g * size; e < (g + 1) * size; ++e) {
+      const float c = choice[e];
+      second = fmaxf(second, fminf(first, c));
+      first = fmaxf(first, c);
+    }
+    group_score[g] = size > 1 ? first + second : first;
+  }
+  together();
+  float mine[N];
+  int place[N];
+#pragma unroll
+  for (int i = 0; i < N; ++i) {
+    const int e = x + LANES * i;
+    mine[i] = -INFINITY;
+    place[i] = -1;
+    if (e < a.experts) {
+      bool open = a.keep >= a.groups;
+      if (!open) {
+        const int g = e / size;
+        const float s = group_score[g];
+        int better = 0;
+        for (int o = 0; o < a.groups; ++o) better += group_score[o] > s || (group_score[o] == s && o < g);
+        open = better < a.keep;
+      }
+      if (open) mine[i] = choice[e];
+    }
+  }
+  float sum = 0.f;
+  for (int s = 0; s < a.top; ++s) {
+    float best = -INFINITY;
+    int who = 0x7fffffff;
+#pragma unroll
+    for (int i = 0; i < N; ++i)
+      if (mine[i] > best) {
+        best = mine[i];
+        who = x + LANES * i;
+      }
+#pragma unroll
+    for (int off = 1; off < LANES; off <<= 1) {
+      const float ob = __shfl_xor(best, off, kWave);
+      const int ow = __shfl_xor(who, off, kWave);
+      if (ob > best || (ob == best && ow < who)) {
+        best = ob;
+        who = ow;
+      }
+    }
+    if (who >= a.experts) {      // scores that compare with nothing: any expert, and a weight that shows it
+      if (x == 0 && token < a.tokens) {
+        a.chosen[(int64_t)token * a.top + s] = s;
+        a.score[(int64_t)token * a.top + s] = NAN;
+      }
+      continue;
+    }
+    sum += score[who];
+#pragma unroll
+    for (int i = 0; i < N; ++i)
+      if (who == x + LANES * i) {
+        mine[i] = -INFINITY;
+        place[i] = s;
+      }
+  }
+  const float f = a.factor / (sum + 1e-20f);
+#pragma unroll
+  for (int i = 0; i < N; ++i)
+    if (place[i] >= 0 && token < a.tokens) {
+      a.chosen[(int64_t)token * a.top + place[i]] = x + LANES * i;
+      a.score[(int64_t)token * a.top + place[i]] = score[x + LANES * i] * f;
+    }
+}
 
 constexpr int kPlaceGroups = 4;       // route workgroups of a place workgroup
 // Tokens of a route workgroup: the router's weights are read once for all of them; small batches need the workgroups more.
@@ -50,6 +135,7 @@ __global__ __launch_bounds__(256) void moe_route_mfma_kernel(const RouteArgs a, 
   constexpr int kPitch = ET * 16 + 1;
   constexpr int kAhead = TT == 1 ? (ET <= 2 ? 8 : (ET <= 4 ? 4 : 2)) : (ET <= 2 ? 4 : (ET <= 4 ? 2 : 1));      // steps whose loads are issued together
   __shared__ float logits[2][16 * TT][kPitch];
+  __shared__ float group_scores[16 * TT][kPitch];
   __shared__ int hist[ET * 16];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, n = lane & 15, jj = lane >> 4;
   const int t0 = blockIdx.x * 16 * TT;
@@ -118,6 +204,16 @@ __global__ __launch_bounds__(256) void moe_route_mfma_kernel(const RouteArgs a, 
 #pragma unroll
   for (int j = 0; j < TT; ++j) {
     const int mt = 16 * j + (threadIdx.x >> 4), token = t0 + mt;
+    if (a.groups > 0) {
+      for (int e = x; e < a.experts; e += 16) {
+        const float sg = 1.0f / (1.0f + expf(-(logits[0][mt][e] + logits[1][mt][e])));
+        logits[0][mt][e] = sg + a.correction[e];
+        logits[1][mt][e] = sg;
+      }
+      __syncthreads();
+      choose_weighted<16, ET>(a, logits[1][mt], logits[0][mt], group_scores[mt], x, token, [] { __syncthreads(); });
+      continue;
+    }
     float mine[ET];
 #pragma unroll
     for (int i = 0; i < ET; ++i) mine[i] = x + 16 * i < a.experts ? logits[0][mt][x + 16 * i] + logits[1][mt][x + 16 * i] : -INFINITY;
@@ -158,12 +254,13 @@ __global__ __launch_bounds__(256) void moe_route_mfma_kernel(const RouteArgs a, 
 // A wave per token, any size.
 template <typename T>
 __global__ __launch_bounds__(256) void moe_route_kernel(const RouteArgs a) {
-  __shared__ float logits[4][kMaxExperts];
+  __shared__ float logits[4][kMaxExperts], choices[4][kMaxExperts], group_scores[4][kMaxExperts];
   __shared__ int hist[kMaxExperts];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   float* mine = logits[wave];
+  auto t0_of = [&](int i) { return (int)blockIdx.x * a.per_wg + i; };
   for (int i = wave; i < a.per_wg; i += 4) {      // as often for every wave
-    const int t = blockIdx.x * a.per_wg + i;
+    const int t = t0_of(i);
     const T* h = (const T*)a.h + (int64_t)(t < a.tokens ? t : a.tokens - 1) * a.h_stride;
     for (int e = 0; e < a.experts; ++e) {
       const T* w = (const T*)a.router + (int64_t)e * a.width;
@@ -173,6 +270,16 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const RouteArgs a) {
       if (lane == 0) mine[e] = dot;
     }
     __syncthreads();
+    if (a.groups > 0) {
+      for (int e = lane; e < a.experts; e += kWave) {
+        mine[e] = 1.0f / (1.0f + expf(-mine[e]));
+        choices[wave][e] = mine[e] + a.correction[e];
+      }
+      __syncthreads();
+      choose_weighted<kWave, kMaxExperts / kWave>(a, mine, choices[wave], group_scores[wave], lane, t0_of(i), [] { __syncthreads(); });
+      __syncthreads();
+      continue;
+    }
     for (int s = 0; s < a.top; ++s) {
       float best = -INFINITY;
       int who = 0x7fffffff;
@@ -316,6 +423,9 @@ struct GroupedArgs {
   const int32_t *rows, *tiles;
   const float* score;
   int top, blocks;          // blocks of outputs in the grid
+  int unit;                 // of gate_up: 0 silu of scaled inputs, 1 clamped
+  float limit, alpha;
+  bool weigh;               // the choice's score multiplies the result of down instead of the input of gate_up
   // small blocks without routing (rows == nullptr): group e has the rows e * per_group .., and one more group of the same rows has
   // weights, outputs and their number of its own
   int per_group, groups;
@@ -324,6 +434,15 @@ struct GroupedArgs {
   void* out_last;
   int64_t out_last_stride;
 };
+
+// The gated unit of an expert: s the choice's score, g and u the products of its token.
+template <typename T>
+__device__ __forceinline__ float gated_unit(const GroupedArgs& a, float s, float g, float u) {
+  if (a.unit == 0) return silu_for<T>(s * g) * (s * u);
+  g = fminf(g, a.limit);
+  u = fminf(fmaxf(u, -a.limit), a.limit);
+  return g * sigmoid_for<T>(a.alpha * g) * (u + 1.0f);
+}
 
 // This workgroup's tile and block of outputs.  Consecutive workgroups go to different XCDs: each XCD gets a contiguous run of
 // tiles with all their outputs, so that the rows of a tile and the weights of an expert meet in one L2.
@@ -424,7 +543,7 @@ __global__ __launch_bounds__(256, 2) void moe_grouped_large_kernel(const Grouped
     const int r = 64 * wm + 32 * j + col;
     if (r >= count) continue;
     const int choice = a.rows[row0 + r];
-    const float s = GATED ? a.score[choice] : 1.f;
+    const float s = GATED != a.weigh ? a.score[choice] : 1.f;
     uint16_t* o = (uint16_t*)a.out + (int64_t)(GATED ? row0 + r : choice) * a.out_stride;
 #pragma unroll
     for (int i = 0; i < (GATED ? 1 : 2); ++i)
@@ -433,7 +552,7 @@ __global__ __launch_bounds__(256, 2) void moe_grouped_large_kernel(const Grouped
         const int n = n0 + (GATED ? 32 * wn : 64 * wn + 32 * i) + 8 * q4 + 4 * hh;
         float v[4];
 #pragma unroll
-        for (int x = 0; x < 4; ++x) v[x] = GATED ? silu_for<bf16_t>(s * acc[0][j][4 * q4 + x]) * (s * acc[1][j][4 * q4 + x]) : acc[i][j][4 * q4 + x];
+        for (int x = 0; x < 4; ++x) v[x] = GATED ? gated_unit<bf16_t>(a, s, acc[0][j][4 * q4 + x], acc[1][j][4 * q4 + x]) : s * acc[i][j][4 * q4 + x];
         if (ALIGNED && n + 4 <= a.n) {
           *reinterpret_cast<u32x2*>(o + n) = u32x2{pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3])};
         } else {
@@ -549,13 +668,13 @@ __global__ __launch_bounds__(256, 3) void moe_grouped_small_kernel(const Grouped
   const int choice = a.rows ? a.rows[row0 + r] : row0 + r;
   uint16_t* o = last ? (uint16_t*)a.out_last + (int64_t)(choice - e * a.per_group) * a.out_last_stride
                      : (uint16_t*)a.out + (int64_t)(GATED ? row0 + r : choice) * a.out_stride;
-  const float s = GATED ? a.score[choice] : 1.f;
+  const float s = GATED != a.weigh ? a.score[choice] : 1.f;
 #pragma unroll
   for (int half = 0; half < (GATED ? 1 : 2); ++half) {
     const int n = n0 + 16 * (i + 2 * half) + 4 * jj;
     float y[4];
 #pragma unroll
-    for (int q = 0; q < 4; ++q) y[q] = GATED ? silu_for<bf16_t>(s * v0[q]) * (s * v1[q]) : (half ? v1[q] : v0[q]);
+    for (int q = 0; q < 4; ++q) y[q] = GATED ? gated_unit<bf16_t>(a, s, v0[q], v1[q]) : s * (half ? v1[q] : v0[q]);
     if (ALIGNED && n + 4 <= n_all) {
       *reinterpret_cast<u32x2*>(o + n) = u32x2{pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3])};
     } else {
@@ -607,9 +726,9 @@ __global__ __launch_bounds__(256) void moe_grouped_f32_kernel(const GroupedArgs 
     const int row = r0 + 4 * r;
     if (row >= count) continue;
     const int choice = a.rows[row0 + row];
-    const float s = GATED ? a.score[choice] : 1.f;
+    const float s = GATED != a.weigh ? a.score[choice] : 1.f;
     ((float*)a.out)[(int64_t)(GATED ? row0 + row : choice) * a.out_stride + n] =
-        GATED ? silu_for<float>(s * acc[0][r]) * (s * acc[GATED ? 1 : 0][r]) : acc[0][r];
+        GATED ? gated_unit<float>(a, s, acc[0][r], acc[GATED ? 1 : 0][r]) : s * acc[0][r];
   }
 }
 
@@ -649,6 +768,9 @@ static int check_grouped(const mops_hip_moe* m) {
   if (m->block_rows != kSM && (m->block_rows != kGM || m->dtype != MOPS_HIP_BF16)) return MOPS_HIP_EINVAL;
   if (m->experts > kMaxExperts || m->tokens * m->top > (1 << 28) || m->width > (1 << 20) || m->ff > (1 << 20)) return MOPS_HIP_EUNSUPPORTED;
   if (!m->rows || !m->tiles || !m->score) return MOPS_HIP_EINVAL;
+  if (m->groups < 0 || (m->groups > 0 && (m->experts % m->groups || m->keep <= 0 || m->keep > m->groups || m->top > m->experts / m->groups * m->keep)))
+    return MOPS_HIP_EINVAL;
+  if (m->unit != 0 && m->unit != 1) return MOPS_HIP_EINVAL;
   return 1;
 }
 
@@ -677,6 +799,8 @@ extern "C" int mops_hip_moe_route(const void* h, int64_t h_row_stride, const voi
   a.tokens = (int)m->tokens; a.width = (int)m->width; a.experts = (int)m->experts; a.top = (int)m->top;
   a.chosen = chosen; a.rank = rank; a.counts = counts; a.score = m->score;
   a.per_wg = route_tokens(m->tokens);
+  if (m->groups > 0 && !m->correction) return MOPS_HIP_EINVAL;
+  a.correction = m->correction; a.groups = (int)m->groups; a.keep = (int)m->keep; a.factor = m->factor;
   const int64_t groups = mops_hip_moe_route_workgroups(m->tokens);
   const dim3 grid((unsigned)groups), block(256);
   hipStream_t s = (hipStream_t)stream;
@@ -712,6 +836,7 @@ extern "C" int mops_hip_moe_gate_up(const void* h, int64_t h_row_stride, const v
   a.x = h; a.x_stride = h_row_stride; a.w = w; a.w_expert = 2 * up_at * m->width;
   a.n = (int)m->ff; a.up_at = (int)up_at; a.depth = (int)m->width; a.out = y; a.out_stride = y_row_stride;
   a.rows = m->rows; a.tiles = m->tiles; a.score = m->score; a.top = (int)m->top; a.blocks = 0;
+  a.unit = m->unit; a.limit = m->limit; a.alpha = m->alpha; a.weigh = m->groups > 0;
   return launch_grouped<true>(a, m->dtype, m->block_rows, m->tokens * m->top, m->experts, (hipStream_t)stream);
 }
 
@@ -724,7 +849,7 @@ extern "C" int mops_hip_moe_down(const void* y, int64_t y_row_stride, const void
   GroupedArgs a = {};
   a.x = y; a.x_stride = y_row_stride; a.w = w; a.w_expert = depth * m->width;
   a.n = (int)m->width; a.up_at = 0; a.depth = (int)depth; a.out = z; a.out_stride = z_row_stride;
-  a.rows = m->rows; a.tiles = m->tiles; a.score = m->score; a.top = (int)m->top; a.blocks = 0;
+  a.rows = m->rows; a.tiles = m->tiles; a.score = m->score; a.top = (int)m->top; a.blocks = 0; a.weigh = m->groups > 0;
   return launch_grouped<false>(a, m->dtype, m->block_rows, m->tokens * m->top, m->experts, (hipStream_t)stream);
 }
 

@@ -4,7 +4,10 @@
 //   norm_residual_add  x += rms(y) * (offset + w): the norm sits on the sublayer's output, the sum runs on in float32 and
 //                      leaves a copy in the activation type for the next projection
 //   rms_norm_f32       out = rms(x) * (offset + w) of the float32 stream
-//   add_norm_norm      x += rms(y) * w_out, out = rms(x) * w_in: norms behind one sublayer and in front of the next, in one pass
+//   add_norm_norm      x += norm(y) * w_out, out = norm(x) * w_in: norms behind one sublayer and in front of the next, in one pass;
+//                      RMS norms or layer norms
+//   layer_norm_f32     out = (x - mean) / sqrt(variance + eps) * w of the float32 stream
+//   embed_pairs        embed_residual plus a row of a table of pairs of tokens
 //   gated_group_norm   rms over equal parts of a row, with silu(gate) multiplied in before or after the division
 //
 // A row belongs to one workgroup of 64 or 256 threads; the elements a thread owns stay in its registers between the
@@ -31,6 +34,42 @@ __global__ __launch_bounds__(256) void embed_residual_kernel(const int64_t* __re
     for (int e = 0; e < VEC; ++e) v[e] *= scale;
     store_vec<VEC>(x + row * width + c, v);
     if (act) store_vec<VEC>(act + row * width + c, v);
+  }
+}
+
+// The same plus a row of a table of pairs: (token in front * mul_prev + token * mul_cur) mod buckets, and row `buckets` for a
+// sequence's first token.  The token in front of a portion is kept per state slot: the workgroup of the portion's first token is the
+// only one that reads it, and it files the portion's last token behind its read.
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void embed_pairs_kernel(const mops_hip_embed_pairs_args a) {
+  const int64_t t = blockIdx.x;
+  const int width = (int)a.width;
+  const int64_t b = a.token_seq ? a.token_seq[t] : t;
+  const int64_t first = a.cu_seqlens ? a.cu_seqlens[b] : t;
+  const int64_t id = a.ids[t];
+  int64_t pair = a.buckets, prev = -1;
+  if (t > first) {
+    prev = a.ids[t - 1];
+  } else {
+    const int slot = a.state_slots[b];
+    const bool filed = slot >= 0 && slot < a.num_slots;
+    if (filed && a.starts[b] > 0) prev = a.before[slot];
+    __syncthreads();
+    if (filed && threadIdx.x == 0) a.before[slot] = (int32_t)a.ids[a.cu_seqlens ? a.cu_seqlens[b + 1] - 1 : t];
+  }
+  if (prev >= 0) {
+    pair = (prev * a.mul_prev + id * a.mul_cur) % a.buckets;
+    if (pair < 0) pair += a.buckets;
+  }
+  const bool ok = id >= 0 && id < a.vocab;
+  const T *row = (const T*)a.table + (ok ? id : 0) * a.table_stride, *row2 = (const T*)a.pairs + pair * a.pairs_stride;
+  for (int c = threadIdx.x * VEC; c < width; c += 256 * VEC) {
+    float v[VEC], u[VEC];
+    load_vec<VEC>(row + c, v);
+    load_vec<VEC>(row2 + c, u);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) v[e] = (ok ? a.scale * v[e] : 0.f) + u[e];
+    store_vec<VEC>(a.residual + t * width + c, v);
   }
 }
 
@@ -90,82 +129,131 @@ __global__ __launch_bounds__(THREADS) void norm_kernel(float* __restrict__ resid
   }
 }
 
-// residual += norm(sum of the row's `parts` rows of y) * w_out; out = norm(residual) * w_in.
-template <typename T, int VEC, int THREADS>
+// residual += norm(sum of the row's `parts` rows of y, and of extra) * w_out; out = norm(residual) * w_in.  CENTER: the norms take
+// the mean off first.
+template <typename T, int VEC, int THREADS, bool CENTER>
 __global__ __launch_bounds__(THREADS) void add_norm_norm_kernel(float* __restrict__ residual, const T* __restrict__ y, int64_t y_stride,
-                                                                int parts, const T* __restrict__ w_out, const T* __restrict__ w_in,
-                                                                float eps, T* __restrict__ out, int n) {
+                                                                int parts, const T* __restrict__ extra, const T* __restrict__ w_out,
+                                                                const T* __restrict__ w_in, float eps, T* __restrict__ out, int n) {
   __shared__ float scratch[THREADS / kWave];
   const int64_t row = blockIdx.x;
   float* xr = residual + row * n;
   const T* yr = y + row * parts * y_stride;
   auto read = [&](int c, float (&v)[VEC]) {
     load_vec<VEC>(yr + c, v);
-    for (int p = 1; p < parts; ++p) {
+    auto more = [&](const T* p) {
       float u[VEC];
-      load_vec<VEC>(yr + p * y_stride + c, u);
+      load_vec<VEC>(p + c, u);
 #pragma unroll
       for (int e = 0; e < VEC; ++e) v[e] += u[e];
+    };
+    for (int p = 1; p < parts; ++p) more(yr + p * y_stride);
+    if (extra) more(extra + row * n);
+  };
+  auto stream = [&](int c, float (&v)[VEC]) { load_vec<VEC>(xr + c, v); };      // this thread's own stores, once it has made them
+  float keep[kKeep][VEC];
+  // f(column, values) for all pieces of this thread; those behind the kept ones come from `again`
+  auto each = [&](auto&& again, auto&& f) {
+#pragma unroll
+    for (int it = 0; it < kKeep; ++it) {
+      const int c = (it * THREADS + threadIdx.x) * VEC;
+      if (c < n) f(c, keep[it]);
+    }
+    for (int c = (kKeep * THREADS + threadIdx.x) * VEC; c < n; c += THREADS * VEC) {
+      float v[VEC];
+      again(c, v);
+      f(c, v);
     }
   };
-  float keep[kKeep][VEC];
-  float ss = 0.f;
+  // mean (0 without CENTER) and reciprocal root of the mean squared deviation from it
+  auto statistics = [&](auto&& again, float sum, float squares, float& mean, float& rstd) {
+    mean = 0.f;
+    if (CENTER) {
+      mean = block_sum<THREADS>(sum, scratch) / (float)n;
+      squares = 0.f;
+      each(again, [&](int, float (&v)[VEC]) {
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) squares += (v[e] - mean) * (v[e] - mean);
+      });
+    }
+    rstd = 1.0f / sqrtf(block_sum<THREADS>(squares, scratch) / (float)n + eps);
+  };
+  float sum = 0.f, squares = 0.f, mean, rstd;
+  auto count = [&](const float (&v)[VEC]) {
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) {
+      if (CENTER) sum += v[e];
+      else squares += v[e] * v[e];
+    }
+  };
 #pragma unroll
   for (int it = 0; it < kKeep; ++it) {
     const int c = (it * THREADS + threadIdx.x) * VEC;
-    if (c < n) {
-      read(c, keep[it]);
-#pragma unroll
-      for (int e = 0; e < VEC; ++e) ss += keep[it][e] * keep[it][e];
-    }
+    if (c < n) read(c, keep[it]);
   }
-  for (int c = (kKeep * THREADS + threadIdx.x) * VEC; c < n; c += THREADS * VEC) {
-    float v[VEC];
-    read(c, v);
-#pragma unroll
-    for (int e = 0; e < VEC; ++e) ss += v[e] * v[e];
-  }
-  const float rstd_out = 1.0f / sqrtf(block_sum<THREADS>(ss, scratch) / (float)n + eps);
-  ss = 0.f;
-  auto add = [&](int c, float (&v)[VEC]) {      // v: the sublayer's output, then the new residual
+  each(read, [&](int, float (&v)[VEC]) { count(v); });
+  statistics(read, sum, squares, mean, rstd);
+  sum = squares = 0.f;
+  each(read, [&](int c, float (&v)[VEC]) {      // v: the sublayer's output, then the new residual
     float wv[VEC], x[VEC];
     load_vec<VEC>(w_out + c, wv);
     load_vec<VEC>(xr + c, x);
 #pragma unroll
-    for (int e = 0; e < VEC; ++e) {
-      v[e] = x[e] + v[e] * rstd_out * wv[e];
-      ss += v[e] * v[e];
-    }
+    for (int e = 0; e < VEC; ++e) v[e] = x[e] + (v[e] - mean) * rstd * wv[e];
     store_vec<VEC>(xr + c, v);
-  };
-#pragma unroll
-  for (int it = 0; it < kKeep; ++it) {
-    const int c = (it * THREADS + threadIdx.x) * VEC;
-    if (c < n) add(c, keep[it]);
-  }
-  for (int c = (kKeep * THREADS + threadIdx.x) * VEC; c < n; c += THREADS * VEC) {
-    float v[VEC];
-    read(c, v);
-    add(c, v);
-  }
-  const float rstd_in = 1.0f / sqrtf(block_sum<THREADS>(ss, scratch) / (float)n + eps);
-  auto finish = [&](int c, const float (&v)[VEC]) {
+    count(v);
+  });
+  statistics(stream, sum, squares, mean, rstd);
+  each(stream, [&](int c, float (&v)[VEC]) {
     float wv[VEC], o[VEC];
     load_vec<VEC>(w_in + c, wv);
 #pragma unroll
-    for (int e = 0; e < VEC; ++e) o[e] = v[e] * rstd_in * wv[e];
+    for (int e = 0; e < VEC; ++e) o[e] = (v[e] - mean) * rstd * wv[e];
     store_vec<VEC>(out + row * n + c, o);
+  });
+}
+
+// out = (x - mean) / sqrt(variance + eps) * w of the float32 stream.
+template <typename T, int VEC, int THREADS>
+__global__ __launch_bounds__(THREADS) void layer_norm_kernel(const float* __restrict__ x, const T* __restrict__ w, float eps, T* __restrict__ out, int n) {
+  __shared__ float scratch[THREADS / kWave];
+  const float* xr = x + (int64_t)blockIdx.x * n;
+  float keep[kKeep][VEC];
+  auto each = [&](auto&& f) {
+#pragma unroll
+    for (int it = 0; it < kKeep; ++it) {
+      const int c = (it * THREADS + threadIdx.x) * VEC;
+      if (c < n) f(c, keep[it]);
+    }
+    for (int c = (kKeep * THREADS + threadIdx.x) * VEC; c < n; c += THREADS * VEC) {
+      float v[VEC];
+      load_vec<VEC>(xr + c, v);
+      f(c, v);
+    }
   };
 #pragma unroll
   for (int it = 0; it < kKeep; ++it) {
     const int c = (it * THREADS + threadIdx.x) * VEC;
-    if (c < n) finish(c, keep[it]);
+    if (c < n) load_vec<VEC>(xr + c, keep[it]);
   }
-  for (int c = (kKeep * THREADS + threadIdx.x) * VEC; c < n; c += THREADS * VEC) {
-    float v[VEC];
-    load_vec<VEC>(xr + c, v);      // this thread's own stores
-    finish(c, v);
-  }
+  float sum = 0.f, squares = 0.f;
+  each([&](int, float (&v)[VEC]) {
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) sum += v[e];
+  });
+  const float mean = block_sum<THREADS>(sum, scratch) / (float)n;
+  each([&](int, float (&v)[VEC]) {
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) squares += (v[e] - mean) * (v[e] - mean);
+  });
+  const float rstd = 1.0f / sqrtf(block_sum<THREADS>(squares, scratch) / (float)n + eps);
+  each([&](int c, float (&v)[VEC]) {
+    float wv[VEC], o[VEC];
+    load_vec<VEC>(w + c, wv);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) o[e] = (v[e] - mean) * rstd * wv[e];
+    store_vec<VEC>(out + (int64_t)blockIdx.x * n + c, o);
+  });
 }
 
 // LANES lanes per (row, part): parts of `size` consecutive elements.
@@ -288,27 +376,69 @@ extern "C" int mops_hip_rms_norm_f32(const float* x, const void* weight, float w
   return finish_launch();
 }
 
-extern "C" int mops_hip_add_norm_norm(float* residual, const void* y, int64_t y_row_stride, int64_t parts, const void* w_out, const void* w_in,
-                                      float eps, void* out, int dtype, int64_t rows, int64_t n, void* stream) {
+extern "C" int mops_hip_add_norm_norm(float* residual, const void* y, int64_t y_row_stride, int64_t parts, const void* extra, const void* w_out,
+                                      const void* w_in, float eps, int center, void* out, int dtype, int64_t rows, int64_t n, void* stream) {
   using namespace mops;
   if (!known_dtype(dtype) || rows < 0 || n <= 0 || n > (1 << 20) || rows > 0x7fffffffLL || parts <= 0 || parts > (1 << 20)) return MOPS_HIP_EINVAL;
   if (rows == 0) return MOPS_HIP_OK;
-  if (!residual || !y || !w_out || !w_in || !out || y_row_stride < n || y == out) return MOPS_HIP_EINVAL;
-  const bool vec = n % 8 == 0 && y_row_stride % 8 == 0 && aligned16(residual) && aligned16(y) && aligned16(w_out) && aligned16(w_in) && aligned16(out);
+  if (!residual || !y || !w_out || !w_in || !out || y_row_stride < n || y == out || (extra && extra == out)) return MOPS_HIP_EINVAL;
+  const bool vec = n % 8 == 0 && y_row_stride % 8 == 0 && aligned16(residual) && aligned16(y) && aligned16(w_out) && aligned16(w_in) && aligned16(out) &&
+                   (!extra || aligned16(extra));
   const dim3 grid((unsigned)rows);
   hipStream_t s = (hipStream_t)stream;
-#define MOPS_ANN(T, V, TH) hipLaunchKernelGGL((add_norm_norm_kernel<T, V, TH>), grid, dim3(TH), 0, s, residual, (const T*)y, y_row_stride, \
-                                              (int)parts, (const T*)w_out, (const T*)w_in, eps, (T*)out, (int)n)
-#define MOPS_ANN_TYPE(T) do {                          \
-    if (vec && n <= 1024) MOPS_ANN(T, 8, 64);          \
-    else if (vec) MOPS_ANN(T, 8, 256);                 \
-    else if (n <= 512) MOPS_ANN(T, 1, 64);             \
-    else MOPS_ANN(T, 1, 256);                          \
+#define MOPS_ANN(T, V, TH, C) hipLaunchKernelGGL((add_norm_norm_kernel<T, V, TH, C>), grid, dim3(TH), 0, s, residual, (const T*)y, y_row_stride, \
+                                                 (int)parts, (const T*)extra, (const T*)w_out, (const T*)w_in, eps, (T*)out, (int)n)
+#define MOPS_ANN_TYPE(T, C) do {                          \
+    if (vec && n <= 1024) MOPS_ANN(T, 8, 64, C);          \
+    else if (vec) MOPS_ANN(T, 8, 256, C);                 \
+    else if (n <= 512) MOPS_ANN(T, 1, 64, C);             \
+    else MOPS_ANN(T, 1, 256, C);                          \
   } while (0)
-  if (dtype == MOPS_HIP_BF16) MOPS_ANN_TYPE(bf16_t);
-  else MOPS_ANN_TYPE(float);
+  if (dtype == MOPS_HIP_BF16) { if (center) MOPS_ANN_TYPE(bf16_t, true); else MOPS_ANN_TYPE(bf16_t, false); }
+  else { if (center) MOPS_ANN_TYPE(float, true); else MOPS_ANN_TYPE(float, false); }
 #undef MOPS_ANN_TYPE
 #undef MOPS_ANN
+  return finish_launch();
+}
+
+extern "C" int mops_hip_layer_norm_f32(const float* x, const void* weight, float eps, void* out, int dtype, int64_t rows, int64_t n, void* stream) {
+  using namespace mops;
+  if (!known_dtype(dtype) || rows < 0 || n <= 0 || n > (1 << 20) || rows > 0x7fffffffLL) return MOPS_HIP_EINVAL;
+  if (rows == 0) return MOPS_HIP_OK;
+  if (!x || !weight || !out || (const void*)x == out) return MOPS_HIP_EINVAL;
+  const bool vec = n % 8 == 0 && aligned16(x) && aligned16(weight) && aligned16(out);
+  const dim3 grid((unsigned)rows);
+  hipStream_t s = (hipStream_t)stream;
+#define MOPS_LN(T, V, TH) hipLaunchKernelGGL((layer_norm_kernel<T, V, TH>), grid, dim3(TH), 0, s, x, (const T*)weight, eps, (T*)out, (int)n)
+#define MOPS_LN_TYPE(T) do {                          \
+    if (vec && n <= 1024) MOPS_LN(T, 8, 64);          \
+    else if (vec) MOPS_LN(T, 8, 256);                 \
+    else if (n <= 512) MOPS_LN(T, 1, 64);             \
+    else MOPS_LN(T, 1, 256);                          \
+  } while (0)
+  if (dtype == MOPS_HIP_BF16) MOPS_LN_TYPE(bf16_t);
+  else MOPS_LN_TYPE(float);
+#undef MOPS_LN_TYPE
+#undef MOPS_LN
+  return finish_launch();
+}
+
+extern "C" int mops_hip_embed_pairs(const mops_hip_embed_pairs_args* a, void* stream) {
+  using namespace mops;
+  if (!a || !known_dtype(a->dtype) || a->tokens < 0 || a->vocab <= 0 || a->width <= 0 || a->width > (1 << 20) || a->buckets <= 0 || a->num_slots <= 0)
+    return MOPS_HIP_EINVAL;
+  if (a->tokens == 0) return MOPS_HIP_OK;
+  if (!a->ids || !a->table || !a->pairs || !a->residual || !a->before || !a->starts || !a->state_slots) return MOPS_HIP_EINVAL;
+  if (a->table_stride < a->width || a->pairs_stride < a->width || (a->token_seq == nullptr) != (a->cu_seqlens == nullptr)) return MOPS_HIP_EINVAL;
+  const int64_t most = 0x7fffffffLL;      // products of token ids and factors stay inside 64 bits
+  if (a->tokens > most || a->vocab > most || a->mul_prev > most || a->mul_cur > most || a->mul_prev < -most || a->mul_cur < -most) return MOPS_HIP_EUNSUPPORTED;
+  const bool vec = a->width % 8 == 0 && a->table_stride % 8 == 0 && a->pairs_stride % 8 == 0 && aligned16(a->table) && aligned16(a->pairs) && aligned16(a->residual);
+  const dim3 grid((unsigned)a->tokens), block(256);
+  hipStream_t s = (hipStream_t)stream;
+#define MOPS_PAIRS(T, V) hipLaunchKernelGGL((embed_pairs_kernel<T, V>), grid, block, 0, s, *a)
+  if (a->dtype == MOPS_HIP_BF16) { if (vec) MOPS_PAIRS(bf16_t, 8); else MOPS_PAIRS(bf16_t, 1); }
+  else { if (vec) MOPS_PAIRS(float, 8); else MOPS_PAIRS(float, 1); }
+#undef MOPS_PAIRS
   return finish_launch();
 }
 

@@ -6,7 +6,7 @@ The first ctx["n_decode"] sequences of a batch bring one token each, the others 
 A mixer takes its cache or state in allocate(cache); again(cache) gives another mixer on the same weights with a cache or state of
 its own, for layers that run several times in a forward pass.
 A feed-forward is built the same way and called as ff(x).  Its result may have several rows per token, one behind the other,
-that count as their sum.
+that count as their sum; or be a pair of such a result and one more [tokens, width] that is added.
 """
 from __future__ import annotations
 
@@ -140,4 +140,4 @@ def hip_op(name):
     return mops.get_op(name, "hip")
 
 
-from . import biased_attention, feed_forward, latent_attention, mamba2, mixture, retention, time_mixing  # noqa: E402,F401  (register themselves)
+from . import biased_attention, feed_forward, latent_attention, mamba2, mixture, retention, rotary_attention, time_mixing  # noqa: E402,F401  (register themselves)

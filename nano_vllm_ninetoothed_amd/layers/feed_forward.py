@@ -4,29 +4,58 @@ from __future__ import annotations
 from . import hip_op, pack, register_feed_forward, require_size
 
 
-@register_feed_forward("clamped_glu")
-class ClampedGLU:
-    """W_down(g * sigmoid(1.702 g) * (u + 1)) with g = min(W_gate x, limit) and u = clamp(W_up x, -limit, limit)."""
-    ALPHA = 1.702
+class GatedLinearUnit:
+    """W_down f(W_gate x, W_up x); a subclass says what f is."""
 
     @staticmethod
     def validate(sizes):
         require_size(sizes, "ff")
-        float(sizes["limit"])
 
     def __init__(self, sizes, weights, prefix, m):
-        self.ff, self.limit = sizes["ff"], float(sizes["limit"])
+        self.ff = sizes["ff"]
         # the halves start at multiples of eight columns
         self.half = (self.ff + 7) // 8 * 8
         gate, up = (weights.take(prefix + n, (self.ff, m.width)) for n in ("gate", "up"))
         self.gate_up = pack([pack([gate]), pack([up])])
         self.down = weights.take(prefix + "down", (m.width, self.ff))
-        self.linear, self.glu = hip_op("linear"), hip_op("clamped_glu")
+        self.linear = hip_op("linear")
+
+    def unit(self, gate, up):
+        raise NotImplementedError
 
     def __call__(self, x):
         p = self.linear(x, self.gate_up)
-        y = self.glu(p[:, :self.ff], p[:, self.half:self.half + self.ff], self.limit, self.ALPHA)
-        return self.linear(y, self.down)
+        return self.linear(self.unit(p[:, :self.ff], p[:, self.half:self.half + self.ff]), self.down)
+
+
+@register_feed_forward("clamped_glu")
+class ClampedGLU(GatedLinearUnit):
+    """f = g * sigmoid(1.702 g) * (u + 1) with g = min(W_gate x, limit) and u = clamp(W_up x, -limit, limit)."""
+    ALPHA = 1.702
+
+    @staticmethod
+    def validate(sizes):
+        GatedLinearUnit.validate(sizes)
+        float(sizes["limit"])
+
+    def __init__(self, sizes, weights, prefix, m):
+        super().__init__(sizes, weights, prefix, m)
+        self.limit, self.glu = float(sizes["limit"]), hip_op("clamped_glu")
+
+    def unit(self, gate, up):
+        return self.glu(gate, up, self.limit, self.ALPHA)
+
+
+@register_feed_forward("gelu_glu")
+class GeluGLU(GatedLinearUnit):
+    """f = gelu(W_gate x) * W_up x, gelu in its tanh form."""
+
+    def __init__(self, sizes, weights, prefix, m):
+        super().__init__(sizes, weights, prefix, m)
+        self.glu = hip_op("gelu_glu")
+
+    def unit(self, gate, up):
+        return self.glu(gate, up)
 
 
 @register_feed_forward("squared_relu")

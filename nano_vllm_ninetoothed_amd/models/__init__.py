@@ -50,4 +50,4 @@ def load_config(path):
     return cls.config_class.from_dict(raw)
 
 
-from . import nepulix, qwen3, sozarax  # noqa: E402,F401  (register themselves)
+from . import lulizen, nepulix, qwen3, sozarax  # noqa: E402,F401  (register themselves)

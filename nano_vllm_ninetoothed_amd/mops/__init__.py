@@ -64,6 +64,11 @@ EXTENSION_OP_NAMES = (
     "moe_gate_up",
     "moe_down",
     "grouped_linear",
+    # embeddings of pairs, layer norms, rotated attention over part of a sequence, GELU units
+    "embed_pairs",
+    "layer_norm_f32",
+    "gelu_glu",
+    "rotary_prepare",
 )
 
 

@@ -1,14 +1,15 @@
-"""Extension ops of the `hip` backend for grouped-query attention with a linear distance bias over paged keys and values of any
-two sizes (the rules of recurrent_ops.py hold)."""
+"""Extension ops of the `hip` backend for grouped-query attention over paged keys and values of any two sizes, with a linear distance
+bias or capped scores, over all of a sequence or a part of it (the rules of recurrent_ops.py hold)."""
 from __future__ import annotations
 
 from ctypes import byref
+from dataclasses import dataclass
 
 import torch
 
 from ... import _capi
 from .ops import _require, _stream
-from .recurrent_ops import _dtype, _flat
+from .recurrent_ops import _dtype, _flat, _rows
 from .registry import register_hip_op
 
 
@@ -47,7 +48,51 @@ def attention_prepare(qkv, q_weight, k_weight, eps, positions, slot_mapping, k_p
     return q
 
 
-def _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes, row_seq, out, own_rows=True):
+@register_hip_op
+def rotary_prepare(qkv, positions, slot_mapping, k_pages, v_pages, heads, kv_heads, dim, vdim, cos_sin=None, q_weight=None, k_weight=None, eps=0.0):
+    """qkv rows [q | k | v | anything]: an RMS norm per head on q and k where there are weights [dim], their first cos_sin.shape[1]
+    elements turned by the token's position, k and v into their pages.  Returns q [tokens, heads, padded dim]."""
+    a = _capi.RotaryPrepare()
+    a.dtype = _dtype("qkv", qkv)
+    tokens = qkv.shape[0]
+    _require(qkv.dim() == 2 and qkv.stride(1) == 1 and qkv.shape[1] >= (heads + kv_heads) * dim + kv_heads * vdim, "qkv must be [tokens, q | k | v]")
+    a.qkv, a.qkv_stride = qkv.data_ptr(), qkv.stride(0) if tokens > 1 else qkv.shape[1]
+    if q_weight is not None:
+        a.q_weight = _flat("q_weight", q_weight, dim, qkv.dtype)
+    if k_weight is not None:
+        a.k_weight = _flat("k_weight", k_weight, dim, qkv.dtype)
+    a.max_positions = 1
+    if cos_sin is not None:
+        a.max_positions, a.rot = cos_sin.shape
+        a.cos_sin = _flat("cos_sin", cos_sin, a.max_positions * a.rot, torch.float32)
+    a.positions, a.slot_mapping = _flat("positions", positions, tokens, torch.int32), _flat("slot_mapping", slot_mapping, tokens, torch.int32)
+    q = torch.empty((tokens, heads, padded(dim)), dtype=qkv.dtype, device=qkv.device)
+    a.q, a.k_pages, a.v_pages = q.data_ptr(), _pages("k_pages", k_pages, kv_heads, dim, qkv.dtype), _pages("v_pages", v_pages, kv_heads, vdim, qkv.dtype)
+    _require(k_pages.shape[:2] == v_pages.shape[:2], "k_pages and v_pages must have the same blocks")
+    a.num_slots, a.tokens, a.heads, a.kv_heads, a.dim, a.vdim = k_pages.shape[0] * k_pages.shape[1], tokens, heads, kv_heads, dim, vdim
+    a.eps = float(eps)
+    st = _capi.load().mops_hip_rotary_prepare(byref(a), _stream(qkv))
+    _capi.check("mops_hip_rotary_prepare", st)
+    return q
+
+
+@dataclass(frozen=True)
+class Scores:
+    """What a design does to the scores of attention beside scaling them, and what a token sees.  Zeros and None leave it out.
+    softcap: softcap tanh(score / softcap).  window: the last `window` tokens; chunk: the token's chunk of a sequence cut from its start;
+    both up to the token itself, and the first keep_first tokens with them.  sinks (float32 [heads]): logarithms of one more term of
+    the denominator."""
+    softcap: float = 0.0
+    window: int = 0
+    chunk: int = 0
+    keep_first: int = 0
+    sinks: torch.Tensor = None
+
+
+WIDEST = 1 << 30      # more than any sequence holds: a window or chunk without effect
+
+
+def _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes, row_seq, out, own_rows=True, scores=None, gate=None):
     code = _dtype("q", q)
     rows, heads, dp = q.shape
     kv_heads = k_pages.shape[2]
@@ -69,16 +114,25 @@ def _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scal
     a.num_blocks, a.block_size = k_pages.shape[:2]
     a.out, a.rows, a.heads, a.kv_heads, a.dim, a.vdim = out.data_ptr(), rows, heads, kv_heads, dim, vdim
     a.scale, a.dtype = float(scale), code
+    if scores is not None:
+        a.softcap = float(scores.softcap)
+        a.window, a.chunk, a.keep_first = (min(int(n), WIDEST) for n in (scores.window, scores.chunk, scores.keep_first))
+        if scores.sinks is not None:
+            a.sinks = _flat("sinks", scores.sinks, heads, torch.float32)
+    if gate is not None:
+        a.gate, a.gate_stride = gate.data_ptr(), _rows("gate", gate, heads, q.dtype)
+        _require(gate.shape[0] == rows, "gate must be [rows, heads]")
     return a
 
 
 @register_hip_op
-def biased_attention_rows(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes=None, row_seq=None):
+def biased_attention_rows(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes=None, row_seq=None, scores=None, gate=None, out=None):
     """Attention of single query rows against the pages: row r sees the first context_lens[r] tokens of block table row row_seq[r]
-    (r itself without row_seq); score = q.k scale - slope (distance).  Returns [rows, heads, vdim].  The plain form: any size, bf16
-    or float32."""
-    out = torch.empty((q.shape[0], q.shape[1], vdim), dtype=q.dtype, device=q.device)
-    a = _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes, row_seq, out)
+    (r itself without row_seq), or of these what scores lets it see; score = q.k scale - slope (distance), or capped.  gate [rows,
+    heads]: the result is multiplied by its sigmoid.  Returns [rows, heads, vdim].  The plain form: any size, bf16 or float32."""
+    if out is None:
+        out = torch.empty((q.shape[0], q.shape[1], vdim), dtype=q.dtype, device=q.device)
+    a = _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes, row_seq, out, scores=scores, gate=gate)
     st = _capi.load().mops_hip_biased_attention_rows(byref(a), _stream(q))
     _capi.check("mops_hip_biased_attention_rows", st)
     return out
@@ -90,11 +144,11 @@ def biased_matrix_covers(dtype, dim: int, vdim: int, block_size: int) -> bool:
 
 
 @register_hip_op
-def biased_decode(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes=None, row_seq=None, out=None):
+def biased_decode(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes=None, row_seq=None, out=None, scores=None, gate=None):
     """biased_attention_rows on the matrix cores (sizes: biased_matrix_covers)."""
     if out is None:
         out = torch.empty((q.shape[0], q.shape[1], vdim), dtype=q.dtype, device=q.device)
-    a = _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes, row_seq, out)
+    a = _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes, row_seq, out, scores=scores, gate=gate)
     lib = _capi.load()
     ws = torch.empty(max(16, lib.mops_hip_biased_decode_workspace_bytes(a.rows, a.heads, a.kv_heads, dim, vdim)), dtype=torch.uint8, device=q.device)
     st = lib.mops_hip_biased_decode(byref(a), ws.data_ptr(), ws.numel(), _stream(q))
@@ -116,12 +170,12 @@ def biased_prefill_tiles(counts, starts, first_token: int, first_seq: int):
 
 
 @register_hip_op
-def biased_prefill(q, k_pages, v_pages, dim, vdim, tiles, block_table, scale, context_lens, slopes=None, out=None):
+def biased_prefill(q, k_pages, v_pages, dim, vdim, tiles, block_table, scale, context_lens, slopes=None, out=None, scores=None, gate=None):
     """Causal attention of long portions, whose keys and values are in the pages already: tiles [n, 5] is the int32 device copy of
     biased_prefill_tiles.  context_lens: of every row.  Writes the portions' rows of out [rows, heads, vdim]."""
     if out is None:
         out = torch.empty((q.shape[0], q.shape[1], vdim), dtype=q.dtype, device=q.device)
-    a = _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes, None, out, own_rows=False)
+    a = _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes, None, out, own_rows=False, scores=scores, gate=gate)
     n = tiles.shape[0]
     st = _capi.load().mops_hip_biased_prefill(byref(a), _flat("tiles", tiles, 5 * n, torch.int32), n, _stream(q))
     _capi.check("mops_hip_biased_prefill", st)

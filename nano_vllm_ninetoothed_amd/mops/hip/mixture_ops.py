@@ -25,9 +25,22 @@ class Routing:
     tiles: torch.Tensor
 
 
+@dataclass(frozen=True)
+class Weighted:
+    """The weighted form of routing: experts chosen by sigmoid + correction (float32 [experts]) among those of the `keep` best of `groups`
+    equal groups of neighbours (by the sum of a group's two best); a choice's weight is its sigmoid over the sum of the chosen ones,
+    times factor."""
+    correction: torch.Tensor
+    groups: int = 1
+    keep: int = 1
+    factor: float = 1.0
+
+
 @register_hip_op
-def moe_route(h: torch.Tensor, router: torch.Tensor, top: int, block_rows: int = None) -> Routing:
-    """The `top` experts with the largest logits router @ h (float32) per token, their sigmoids, and the plan of the grouped products."""
+def moe_route(h: torch.Tensor, router: torch.Tensor, top: int, block_rows: int = None, weighted: Weighted = None) -> Routing:
+    """The `top` experts with the largest logits router @ h (float32) per token, their sigmoids, and the plan of the grouped products.
+    weighted: another choice, and weights instead of sigmoids; moe_gate_up then leaves its inputs as they are, and moe_down multiplies
+    its results."""
     code = _dtype("h", h)
     tokens, (experts, width) = h.shape[0], router.shape
     stride = _rows("h", h, width, h.dtype)
@@ -43,6 +56,9 @@ def moe_route(h: torch.Tensor, router: torch.Tensor, top: int, block_rows: int =
     m = _capi.Moe()
     m.rows, m.tiles, m.score = rows.data_ptr(), tile_list.data_ptr(), score.data_ptr()
     m.tokens, m.experts, m.top, m.width, m.ff, m.block_rows, m.dtype = tokens, experts, top, width, 1, block_rows, code
+    if weighted is not None:
+        m.correction = _flat("correction", weighted.correction, experts, torch.float32)
+        m.groups, m.keep, m.factor = weighted.groups, weighted.keep, weighted.factor
     st = lib.mops_hip_moe_route(h.data_ptr(), stride, _flat("router", router, experts * width, h.dtype), chosen.data_ptr(), rank.data_ptr(), counts.data_ptr(),
                                 byref(m), _stream(h))
     _capi.check("mops_hip_moe_route", st)
@@ -50,13 +66,15 @@ def moe_route(h: torch.Tensor, router: torch.Tensor, top: int, block_rows: int =
 
 
 @register_hip_op
-def moe_gate_up(h: torch.Tensor, w: torch.Tensor, routing: Routing):
-    """silu(s W_gate h) * (s W_up h) of every choice, s its score, in the order of routing.rows.  w [experts, 2, ff, width]."""
+def moe_gate_up(h: torch.Tensor, w: torch.Tensor, routing: Routing, limit: float = None, alpha: float = 1.702):
+    """silu(s W_gate h) * (s W_up h) of every choice, s its score, in the order of routing.rows.  w [experts, 2, ff, width].  With a
+    limit the unit of clamped_glu instead, which takes no score."""
     code = _dtype("h", h)
     m = routing.args
     experts, two, ff, width = w.shape
     _require(m.tokens == h.shape[0] and m.experts == experts and m.width == width and m.dtype == code and two == 2, "the routing was made for another problem")
-    m.ff = ff
+    m.ff, m.unit = ff, 0 if limit is None else 1
+    m.limit, m.alpha = limit or 0.0, alpha
     y = torch.empty((m.tokens * m.top, ff), dtype=h.dtype, device=h.device)
     st = _capi.load().mops_hip_moe_gate_up(h.data_ptr(), _rows("h", h, width, h.dtype), _flat("w", w, w.numel(), h.dtype), ff, y.data_ptr(), ff, byref(m), _stream(h))
     _capi.check("mops_hip_moe_gate_up", st)
@@ -65,7 +83,8 @@ def moe_gate_up(h: torch.Tensor, w: torch.Tensor, routing: Routing):
 
 @register_hip_op
 def moe_down(y: torch.Tensor, w: torch.Tensor, routing: Routing):
-    """W_down y of every choice: [tokens * top, width], a token's choices one behind the other.  w [experts, width, ff]."""
+    """W_down y of every choice, times its weight if the routing has weights: [tokens * top, width], a token's choices one behind the
+    other.  w [experts, width, ff]."""
     code = _dtype("y", y)
     m = routing.args
     experts, width, ff = w.shape

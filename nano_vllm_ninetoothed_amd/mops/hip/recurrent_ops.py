@@ -54,6 +54,30 @@ def embed_residual(ids: torch.Tensor, table: torch.Tensor, scale: float = 1.0, n
 
 
 @register_hip_op
+def embed_pairs(ids, table, pairs, mul_prev: int, mul_cur: int, before, starts, state_slots, token_seq=None, cu_seqlens=None, scale: float = 1.0):
+    """float32 residual: scaled embedding rows plus a row of `pairs` [buckets + 1, width], picked by a hash of the token and the one in
+    front of it (the last row for a sequence's first token).  `before` [slots] int32 holds each sequence's last token of earlier steps
+    and receives the new one.  Without cu_seqlens every sequence brings one token."""
+    _require(table.dim() == 2 and pairs.dim() == 2 and table.shape[1] == pairs.shape[1] and pairs.shape[0] > 1, "table and pairs must be [rows, width]")
+    n, (vocab, width), batch = ids.numel(), table.shape, state_slots.numel()
+    _require((token_seq is None) == (cu_seqlens is None) and (cu_seqlens is not None or n == batch), "packed portions need token_seq and cu_seqlens")
+    a = _capi.EmbedPairs()
+    a.dtype, a.scale = _dtype("table", table), float(scale)
+    a.ids = _flat("ids", ids, n, torch.int64)
+    a.table, a.table_stride, a.pairs, a.pairs_stride = table.data_ptr(), _rows("table", table, width, table.dtype), pairs.data_ptr(), _rows("pairs", pairs, width, table.dtype)
+    a.buckets, a.mul_prev, a.mul_cur = pairs.shape[0] - 1, mul_prev, mul_cur
+    a.before, a.num_slots = _flat("before", before, before.numel(), torch.int32), before.numel()
+    if cu_seqlens is not None:
+        a.token_seq, a.cu_seqlens = _flat("token_seq", token_seq, n, torch.int32), _flat("cu_seqlens", cu_seqlens, batch + 1, torch.int32)
+    a.starts, a.state_slots = _flat("starts", starts, batch, torch.int32), _flat("state_slots", state_slots, batch, torch.int32)
+    residual = torch.empty((n, width), dtype=torch.float32, device=table.device)
+    a.residual, a.tokens, a.vocab, a.width = residual.data_ptr(), n, vocab, width
+    st = _capi.load().mops_hip_embed_pairs(byref(a), _stream(table))
+    _capi.check("mops_hip_embed_pairs", st)
+    return residual
+
+
+@register_hip_op
 def norm_residual_add(residual: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: float, weight_offset: float = 0.0):
     """residual += rms(y) * (weight_offset + weight), in place; returns the new residual in y's dtype."""
     code = _dtype("y", y)
@@ -69,9 +93,10 @@ def norm_residual_add(residual: torch.Tensor, y: torch.Tensor, weight: torch.Ten
 
 
 @register_hip_op
-def add_norm_norm(residual: torch.Tensor, y: torch.Tensor, w_out: torch.Tensor, w_in: torch.Tensor, eps: float):
+def add_norm_norm(residual: torch.Tensor, y: torch.Tensor, w_out: torch.Tensor, w_in: torch.Tensor, eps: float, center: bool = False, extra=None):
     """residual += rms(y) * w_out in place; returns rms(residual) * w_in in y's dtype.  y [rows * parts, n]: `parts` consecutive
-    rows are summed first (the outputs of several experts)."""
+    rows are summed first (the outputs of several experts), and those of extra [rows, n] with them.  center: layer norms instead
+    of RMS norms."""
     code = _dtype("y", y)
     rows, n = residual.shape
     parts = y.shape[0] // rows if rows else 1
@@ -79,9 +104,22 @@ def add_norm_norm(residual: torch.Tensor, y: torch.Tensor, w_out: torch.Tensor, 
     stride = _rows("y", y, n, y.dtype)
     _require(parts > 0 and y.shape[0] == rows * parts, "y must have a whole number of rows per residual row")
     out = torch.empty((rows, n), dtype=y.dtype, device=y.device)
-    st = _capi.load().mops_hip_add_norm_norm(residual.data_ptr(), y.data_ptr(), stride, parts, _flat("w_out", w_out, n, y.dtype),
-                                             _flat("w_in", w_in, n, y.dtype), float(eps), out.data_ptr(), code, rows, n, _stream(y))
+    st = _capi.load().mops_hip_add_norm_norm(residual.data_ptr(), y.data_ptr(), stride, parts, None if extra is None else _flat("extra", extra, rows * n, y.dtype),
+                                             _flat("w_out", w_out, n, y.dtype), _flat("w_in", w_in, n, y.dtype), float(eps), 1 if center else 0,
+                                             out.data_ptr(), code, rows, n, _stream(y))
     _capi.check("mops_hip_add_norm_norm", st)
+    return out
+
+
+@register_hip_op
+def layer_norm_f32(x: torch.Tensor, weight: torch.Tensor, eps: float):
+    """(x - mean) / sqrt(variance + eps) * weight of float32 rows, in the weight's dtype."""
+    code = _dtype("weight", weight)
+    rows, n = x.shape
+    out = torch.empty((rows, n), dtype=weight.dtype, device=x.device)
+    st = _capi.load().mops_hip_layer_norm_f32(_flat("x", x, rows * n, torch.float32), _flat("weight", weight, n, weight.dtype), float(eps), out.data_ptr(),
+                                              code, rows, n, _stream(x))
+    _capi.check("mops_hip_layer_norm_f32", st)
     return out
 
 
@@ -123,6 +161,19 @@ def clamped_glu(gate: torch.Tensor, up: torch.Tensor, limit: float, alpha: float
     st = _capi.load().mops_hip_clamped_glu(gate.data_ptr(), gs, up.data_ptr(), us, out.data_ptr(), code, rows, n, float(alpha), float(limit),
                                            _stream(gate))
     _capi.check("mops_hip_clamped_glu", st)
+    return out
+
+
+@register_hip_op
+def gelu_glu(gate: torch.Tensor, up: torch.Tensor):
+    """gelu(gate) * up, gelu in its tanh form."""
+    code = _dtype("gate", gate)
+    rows, n = gate.shape
+    gs, us = _rows("gate", gate, n, gate.dtype), _rows("up", up, n, gate.dtype)
+    _require(up.shape[0] == rows, "gate and up must have the same shape")
+    out = torch.empty((rows, n), dtype=gate.dtype, device=gate.device)
+    st = _capi.load().mops_hip_gelu_glu(gate.data_ptr(), gs, up.data_ptr(), us, out.data_ptr(), code, rows, n, _stream(gate))
+    _capi.check("mops_hip_gelu_glu", st)
     return out
 
 
