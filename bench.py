@@ -13,6 +13,7 @@ A step is one flash_attn_with_kvcache call over the whole batch, KV cache reside
          every kernel of that design beside the like kernel of the Qwen3 path (--part, --kernels, --sizes choose);
          the line's value is the decode throughput of the last size at the largest batch.
   sozarax = the same for Sozarax, beside Nepulix and Qwen3 models of equal size and their kernels.
+  lulizen = the same for Lulizen, beside Sozarax and Qwen3 models of equal size and their kernels.
   copy = a plain 1 GiB device-to-device tensor copy (not a mops op): the known-size kernel against which
          the FETCH_SIZE / WRITE_SIZE counters of a profile are calibrated.
   launch_floor = an empty kernel: the floor under the durations of the small operators (value 0, read the time).
@@ -61,13 +62,13 @@ def parse_args():
     ap.add_argument("--steps", type=int, default=None, help="timed steps (default 50; 500 for the prefill ops)")
     ap.add_argument("--warmup", type=int, default=None, help="untimed warm-up steps (default 10; 300 for the prefill ops)")
     ap.add_argument("--op", default="decode",
-                    choices=["decode", "decode8b", "prefill", "prefill_long", "prefix_prefill", "prefix_prefill_short", "store", "silu", "sampler", "qk_rope_store", "add_rms", "rms", "embedding", "copy", "launch_floor", "e2e", "nepulix", "sozarax"])
+                    choices=["decode", "decode8b", "prefill", "prefill_long", "prefix_prefill", "prefix_prefill_short", "store", "silu", "sampler", "qk_rope_store", "add_rms", "rms", "embedding", "copy", "launch_floor", "e2e", "nepulix", "sozarax", "lulizen"])
     ap.add_argument("--e2e-seqs", type=int, default=256, help="number of prompts of the e2e workload")
     ap.add_argument("--e2e-eager", action="store_true", help="e2e: no HIP-graph replay of the decode step")
     ap.add_argument("--e2e-stepwise", action="store_true", help="e2e: read every step's tokens back before the next step, as the reference does")
-    ap.add_argument("--part", "--nepulix-part", default="all", choices=["all", "models", "kernels"], help="nepulix, sozarax: throughput of whole models, kernels, or both")
-    ap.add_argument("--kernels", "--nepulix-kernels", default="", help="nepulix, sozarax: kernels to time, by the beginning of their names, with commas between them (default: all)")
-    ap.add_argument("--sizes", "--nepulix-sizes", default="", help="nepulix, sozarax: sizes to run, with commas between them (default: all)")
+    ap.add_argument("--part", "--nepulix-part", default="all", choices=["all", "models", "kernels"], help="nepulix, sozarax, lulizen: throughput of whole models, kernels, or both")
+    ap.add_argument("--kernels", "--nepulix-kernels", default="", help="nepulix, sozarax, lulizen: kernels to time, by the beginning of their names, with commas between them (default: all)")
+    ap.add_argument("--sizes", "--nepulix-sizes", default="", help="nepulix, sozarax, lulizen: sizes to run, with commas between them (default: all)")
     ap.add_argument("--no-cpu-baseline", action="store_true")
     ap.add_argument("--no-e2e", action="store_true", help="default op only: skip the end-to-end block of the line (profiling runs)")
     ap.add_argument("--seed", type=int, default=0)
@@ -171,27 +172,24 @@ def run_e2e(args, torch, dev, mops):
 
 
 def run_design(args, torch, dev):
-    """`--op nepulix`, `--op sozarax`: throughput of the models and the table of kernels, in one line."""
+    """`--op nepulix`, `--op sozarax`, `--op lulizen`: throughput of the models and the table of kernels, in one line."""
     from nano_vllm_ninetoothed_amd import bench_layers as B
-    from nano_vllm_ninetoothed_amd.models.nepulix import NepulixConfig
-    from nano_vllm_ninetoothed_amd.models.sozarax import SozaraxConfig
+    from nano_vllm_ninetoothed_amd.models import parse_config
     design = args.op
-    others = "Qwen3" if design == "nepulix" else "Nepulix and Qwen3"
+    sizes, others = B.DESIGNS[design]
     out = {"metric": f"{design}_decode_tok_per_s", "value": None, "unit": "tok/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
            "ms_per_step": None, "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
            "config": {"model": f"{design.capitalize()}, random weights, beside {others} of equal width, depth, feed-forward and vocabulary"}}
     if args.part != "kernels":
         out["models"] = {}
-        for name, configs in (B.sizes() if design == "nepulix" else B.sozarax_sizes()).items():
+        for name, configs in sizes().items():
             if args.sizes and name not in args.sizes.split(","):
                 continue
             out["models"][name] = r = {}
             for cfg in configs:
                 label = cfg["architecture"].lower() if isinstance(cfg, dict) else "qwen3"
-                if label == "sozarax":
-                    cfg = SozaraxConfig.from_dict(cfg)
-                elif label == "nepulix":
-                    cfg = NepulixConfig.from_dict(cfg)
+                if isinstance(cfg, dict):
+                    cfg = parse_config(cfg)
                 r[label] = B.model_throughput(cfg, args.seed, steps=args.steps, warmup=args.warmup)
             last = r[design]["decode"][-1]
             out.update(value=last["tok_per_s"], ms_per_step=last["ms"])
@@ -240,7 +238,7 @@ def main():
     if args.op == "e2e":
         run_e2e(args, torch, dev, mops)
         return
-    if args.op in ("nepulix", "sozarax"):
+    if args.op in ("nepulix", "sozarax", "lulizen"):
         run_design(args, torch, dev)
         return
     bound = "hbm"

@@ -1,6 +1,6 @@
-"""Measurements behind `bench.py --op nepulix` and `--op sozarax`: prefill and decode throughput of models with layers of real sizes
-beside models of equal width, depth, feed-forward and vocabulary (Qwen3; for Sozarax also Nepulix), and every kernel of the
-design beside the like kernel of those.  Random weights and inputs."""
+"""Measurements behind `bench.py --op nepulix`, `--op sozarax` and `--op lulizen`: prefill and decode throughput of models with layers
+of real sizes beside models of equal width, depth, feed-forward and vocabulary (Qwen3 and the designs that came before), and every
+kernel of the design beside the like kernel of those.  Random weights and inputs."""
 from __future__ import annotations
 
 import torch
@@ -54,6 +54,29 @@ def sozarax_sizes():
             "w2048": (sozarax_dict(2048, 6, 6144, 32768, {"heads": 16, "dim": 128}, att, 32, 4), *near["w2048"])}
 
 
+def lulizen_dict(width, layers, ff, vocab, heads, experts, top):
+    """Layers over chunks and over windows in turn; of three layers one is dense, and a token's experts and the shared one are together
+    as wide as the dense one."""
+    att = {"heads": heads, "kv_heads": heads // 2, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 30.0, "rot": {"base": 5e5, "dims": 128}}
+    kinds = [("attention", dict(att, mask={"size": 8192})), ("attention_2", dict(att, mask={"size": 512, "keep_first": 16}, rot={"base": 1e4, "dims": 64}))]
+    unit = ff // 3 if top == 2 else ff // 6
+    moe = {"kind": "moe", "expert": {"ff": unit, "limit": 7.0}, "shared": {"ff": ff - top * unit, "limit": 7.0},
+           "router": {"experts": experts, "top": top, "scale": 2.5, "groups": {"count": 4, "keep": 2}}}
+    out = [{"type": kinds[i % 2][0], "mixer": kinds[i % 2][1], "mlp": {"kind": "dense", "ff": ff} if i % 3 == 0 else moe} for i in range(layers)]
+    return {"architecture": "Lulizen", "width": width, "vocab": vocab, "norm": {"eps": 1e-6}, "layers": out,
+            "embedding": {"bigram": {"buckets": vocab - 1, "mul_prev": 31, "mul_cur": 17}}}
+
+
+def lulizen_sizes():
+    """name -> (Lulizen config.json dict, Sozarax dict and Qwen3Shape of equal size)"""
+    near = {n: (c[0], c[-1]) for n, c in sozarax_sizes().items()}
+    return {"w1024": (lulizen_dict(1024, 12, 3072, 32768, 16, 16, 2), *near["w1024"]),
+            "w2048": (lulizen_dict(2048, 6, 6144, 32768, 16, 32, 4), *near["w2048"])}
+
+
+DESIGNS = {"nepulix": (sizes, "Qwen3"), "sozarax": (sozarax_sizes, "Nepulix and Qwen3"), "lulizen": (lulizen_sizes, "Sozarax and Qwen3")}
+
+
 def _events(fn, warmup, steps):
     for _ in range(warmup):
         fn()
@@ -92,7 +115,7 @@ def model_throughput(config, seed=0, prompts=16, prompt_len=1024, decode=((64, 1
         live = []
         for _ in range(bs):
             q = eng.open_sequence()
-            q.token_ids = [1] * context
+            q.token_ids = [1] * (context - 1) + [int(torch.randint(0, eng.model.vocab, (), generator=g))]
             eng.cache.hold(q, context)
             live.append(q)
         ids, pos, dctx = eng._prepare_decode(live)
@@ -314,12 +337,10 @@ def nepulix_kernels(t):
     add("embed_residual", f"{T} x 1024", lambda: graph_time(lambda i: op("embed_residual")(ids[i % 4], emb), 8), nbytes=T * 1024 * 8.0, like="add_rms prefill")
 
 
-def sozarax_kernels(t):
-    from .mops.hip import recurrent_ops as R
+def sozarax_attention(t):
     from .mops.hip.attention_ops import biased_prefill_tiles
     from .layers.biased_attention import distance_slopes
     add, rnd, i32, dev = _handles(t)
-    # ---- attention
     ctx, blocks, table, lens_g = decode_contexts(t)
     H, G, d = 16, 8, 128
     slopes = distance_slopes(H).to(dev)
@@ -336,7 +357,11 @@ def sozarax_kernels(t):
     pos, slots = (torch.arange(T, device=dev) % 1024).to(torch.int32), torch.randperm(T, device=dev).to(torch.int32)
     add("attention_prepare", f"{T} tokens, 16/8 heads of 128", lambda: graph_time(lambda i: op("attention_prepare")(qkv[i % 2], wq, wk, 1e-6, pos, slots, kp, vp, H, G, d, d), 8),
         nbytes=T * (H + 2 * G) * d * 4.0, like="qk_norm_rope_store")
-    # ---- time mixing
+
+
+def time_mixing_kernels(t):
+    from .mops.hip import recurrent_ops as R
+    add, rnd, i32, dev = _handles(t)
     for heads, dd in ((16, 64), (16, 128)):
         n = heads * dd
         bs, pitch = 256, R.recurrence_state_pitch(dd)
@@ -364,8 +389,14 @@ def sozarax_kernels(t):
     mixes, wr, w1 = rnd(5, 256, width), [rnd(4, 1024, width) for _ in range(16)], rnd(rank, width)
     add("grouped_linear", f"256 rows, 4 x 1024 -> 1024 and {rank}", lambda: graph_time(lambda i: op("grouped_linear")(mixes, wr[i % 16], w1), 16),
         nbytes=4 * 1024 * 1024 * 2 + 256 * 9 * 1024 * 2, flops=2.0 * 256 * 4 * 1024 * 1024, like="linear decode")
-    # ---- experts
-    for tokens, w, ff, experts, top in ((T, 1024, 1536, 16, 2), (256, 1024, 1536, 16, 2), (T, 2048, 1536, 32, 4), (256, 2048, 1536, 32, 4)):
+
+
+EXPERTS = ((T, 1024, 1536, 16, 2), (256, 1024, 1536, 16, 2), (T, 2048, 1536, 32, 4), (256, 2048, 1536, 32, 4))      # tokens, width, ff, experts, top
+
+
+def sozarax_experts(t):
+    add, rnd, i32, dev = _handles(t)
+    for tokens, w, ff, experts, top in EXPERTS:
         tag, n = f"{tokens} x {w}, top {top} of {experts} x {ff}", tokens * top
         sets = 2 if tokens == T else 4
         h, router = [rnd(tokens, w) for _ in range(sets)], rnd(experts, w)
@@ -378,7 +409,10 @@ def sozarax_kernels(t):
             nbytes=experts * 2.0 * ff * w * 2 + tokens * w * 2.0 + n * ff * 2.0, flops=4.0 * n * ff * w, like=like)
         add("moe_down", tag, lambda: graph_time(lambda i: op("moe_down")(ys[i % sets], down[i % sets], routing[i % sets]), 8),
             nbytes=experts * float(ff) * w * 2 + n * ff * 2.0 + n * w * 2.0, flops=2.0 * n * ff * w, like=like)
-    # ---- around the sublayers
+
+
+def sozarax_residual(t):
+    add, rnd, i32, dev = _handles(t)
     sq = [rnd(T, 3072) for _ in range(4)]
     add("squared_relu", f"{T} x 3072", lambda: graph_time(lambda i: op("squared_relu")(sq[i % 4]), 8), nbytes=T * 3072 * 4.0, like="siluAndMul")
     for rows, n, parts, like in ((512, 4096, 1, "add_rms"), (T, 1024, 1, "add_rms prefill"), (T, 1024, 2, "add_rms prefill")):
@@ -388,6 +422,86 @@ def sozarax_kernels(t):
             nbytes=rows * n * (10.0 + 2 * parts), like=like)
 
 
+def sozarax_kernels(t):
+    sozarax_attention(t)
+    time_mixing_kernels(t)
+    sozarax_experts(t)
+    sozarax_residual(t)
+
+
+def lulizen_kernels(t):
+    from .layers import Rotary
+    from .mops.hip.attention_ops import Scores, biased_prefill_tiles
+    from .mops.hip.mixture_ops import Weighted
+    add, rnd, i32, dev = _handles(t)
+    # ---- attention
+    ctx, blocks, table, lens_g = decode_contexts(t)
+    H, G, d, cap = 16, 8, 128, 30.0
+    sinks = t.f32(H)
+    kp, vp, q, gate = rnd(blocks, 256, G, d), rnd(blocks, 256, G, d), rnd(256, H, d), rnd(256, H)
+    like = "biased_decode 256 x uniform[512,4096], 16/8 heads of 128"
+    for label, scores, g, seen in (
+            ("chunks of 8192, sinks", Scores(softcap=cap, chunk=8192, sinks=sinks), None, lambda n: n),
+            ("chunks of 1024, sinks", Scores(softcap=cap, chunk=1024, sinks=sinks), None, lambda n: (n - 1) % 1024 + 1),
+            ("window of 1024 and 64, gate", Scores(softcap=cap, window=1024, keep_first=64), gate, lambda n: min(n, 1024 + 64)),
+            ("chunks of 8192, cap 100", Scores(softcap=100.0, chunk=8192), None, lambda n: n)):
+        add("biased_decode", f"256 x uniform[512,4096], {label}", lambda: graph_time(lambda i: op("biased_decode")(q, kp, vp, d, d, lens_g, table, 0.088, scores=scores, gate=g), 4),
+            nbytes=sum(map(seen, ctx)) * G * 2 * d * 2.0 + 256 * H * 2 * d * 2, like=like)
+    del kp, vp
+    kp, vp, q, gate = rnd(T // 256, 256, G, d), rnd(T // 256, 256, G, d), rnd(T, H, d), rnd(T, H)
+    out, lens = torch.empty((T, H, d), dtype=torch.bfloat16, device=dev), i32([0] * T)
+    for n, label, scores, g, seen in (
+            (1024, "chunks of 8192, sinks", Scores(softcap=cap, chunk=8192, sinks=sinks), None, lambda i: i + 1),
+            (1024, "cap 100", Scores(softcap=100.0, chunk=8192), None, lambda i: i + 1),
+            (4096, "chunks of 1024, sinks", Scores(softcap=cap, chunk=1024, sinks=sinks), None, lambda i: i % 1024 + 1),
+            (4096, "window of 1024 and 64, gate", Scores(softcap=cap, window=1024, keep_first=64), gate, lambda i: min(i + 1, 1024 + 64)),
+            (4096, "window of 512 and 16, gate", Scores(softcap=cap, window=512, keep_first=16), gate, lambda i: min(i + 1, 512 + 16))):
+        b = T // n
+        tiles, ptab = i32(biased_prefill_tiles([n] * b, [0] * b, 0, 0)), torch.arange(T // 256, dtype=torch.int32, device=dev).view(b, -1)
+        add("biased_prefill", f"{b} x {n}, {label}", lambda: _events(lambda: op("biased_prefill")(
+            q, kp, vp, d, d, tiles, ptab, 0.088, lens, out=out, scores=scores, gate=g), 300, 200), flops=2.0 * H * 2 * d * b * sum(map(seen, range(n))),
+            like="biased_prefill 16 x 1024, 16/8 heads of 128")
+    qkv, w = [rnd(T, (H + 2 * G) * d + 16) for _ in range(2)], rnd(d)
+    pos, slots = (torch.arange(T, device=dev) % 1024).to(torch.int32), torch.randperm(T, device=dev).to(torch.int32)
+    for label, rot, norm in (("norms, 128 rotated", 128, w), ("64 rotated", 64, None)):
+        trig = Rotary(8192, dev).table(1e4, rot)
+        add("rotary_prepare", f"{T} tokens, 16/8 heads of 128, {label}", lambda: graph_time(lambda i: op("rotary_prepare")(
+            qkv[i % 2], pos, slots, kp, vp, H, G, d, d, cos_sin=trig, q_weight=norm, k_weight=norm, eps=1e-6), 8), nbytes=T * (H + 2 * G) * d * 4.0,
+            like=f"attention_prepare {T} tokens, 16/8 heads of 128")
+    # ---- experts
+    for tokens, wd, ff, experts, top in EXPERTS:
+        tag, n = f"{tokens} x {wd}, top {top} of {experts} x {ff}", tokens * top
+        sets = 2 if tokens == T else 4
+        h, router, form = [rnd(tokens, wd) for _ in range(sets)], rnd(experts, wd), Weighted(0.1 * t.f32(experts), 4, 2, 2.5)
+        gu, down = [rnd(experts, 2, ff, wd) for _ in range(sets)], [rnd(experts, wd, ff) for _ in range(sets)]
+        routing = [op("moe_route")(x, router, top, weighted=form) for x in h]
+        ys = [op("moe_gate_up")(h[i], gu[i], routing[i], 7.0) for i in range(sets)]
+        add("moe_route", f"{tag}, 2 of 4 groups", lambda: graph_time(lambda i: op("moe_route")(h[i % sets], router, top, weighted=form), 8), nbytes=tokens * wd * 2.0 + n * 24,
+            like=f"moe_route {tag}")
+        add("moe_gate_up", f"{tag}, clamped", lambda: graph_time(lambda i: op("moe_gate_up")(h[i % sets], gu[i % sets], routing[i % sets], 7.0), 8),
+            nbytes=experts * 2.0 * ff * wd * 2 + tokens * wd * 2.0 + n * ff * 2.0, flops=4.0 * n * ff * wd, like=f"moe_gate_up {tag}")
+        add("moe_down", f"{tag}, weighted", lambda: graph_time(lambda i: op("moe_down")(ys[i % sets], down[i % sets], routing[i % sets]), 8),
+            nbytes=experts * float(ff) * wd * 2 + n * ff * 2.0 + n * wd * 2.0, flops=2.0 * n * ff * wd, like=f"moe_down {tag}")
+    # ---- around the sublayers
+    halves = [rnd(T, 6144).chunk(2, dim=-1) for _ in range(4)]
+    add("gelu_glu", f"{T} x 3072", lambda: graph_time(lambda i: op("gelu_glu")(*halves[i % 4]), 8), nbytes=T * 3072 * 6.0, like="siluAndMul")
+    add("clamped_glu", f"{T} x 3072", lambda: graph_time(lambda i: op("clamped_glu")(*halves[i % 4], 7.0), 8), nbytes=T * 3072 * 6.0, like="siluAndMul")
+    for rows, n, parts, more, like in ((512, 4096, 1, False, "512 x 4096, 1 part"), (T, 1024, 1, False, f"{T} x 1024, 1 part"), (T, 1024, 2, True, f"{T} x 1024, 2 parts")):
+        sets = 24 if rows == 512 else 4
+        res, yy, wa, wb = [t.f32(rows, n) for _ in range(sets)], [rnd(rows * parts, n) for _ in range(sets)], rnd(n), rnd(n)
+        extra = [rnd(rows, n) if more else None for _ in range(sets)]
+        add("add_norm_norm", f"{rows} x {n}, layer norms, {parts}{' + 1' if more else ''} parts", lambda: graph_time(lambda i: op("add_norm_norm")(
+            res[i % sets], yy[i % sets], wa, wb, 1e-6, center=True, extra=extra[i % sets]), 24 if rows == 512 else 8),
+            nbytes=rows * n * (10.0 + 2 * (parts + more)), like=f"add_norm_norm {like}")
+    res, w1 = [t.f32(T, 1024) for _ in range(4)], rnd(1024)
+    add("layer_norm_f32", f"{T} x 1024", lambda: graph_time(lambda i: op("layer_norm_f32")(res[i % 4], w1, 1e-6), 8), nbytes=T * 1024 * 6.0, like="add_rms prefill")
+    emb, pairs, ids = rnd(32768, 1024), rnd(32768, 1024), [torch.randint(0, 32768, (T,), device=dev) for _ in range(4)]
+    before, cu16, z16, sl16 = torch.zeros(16, dtype=torch.int32, device=dev), i32(list(range(0, T + 1, 1024))), i32([0] * 16), torch.arange(16, dtype=torch.int32, device=dev)
+    seq = torch.arange(T, device=dev).div(1024, rounding_mode="floor").to(torch.int32)
+    add("embed_pairs", f"{T} x 1024", lambda: graph_time(lambda i: op("embed_pairs")(ids[i % 4], emb, pairs, 31, 17, before, z16, sl16, seq, cu16), 8), nbytes=T * 1024 * 8.0,
+        like="add_rms prefill")
+
+
 def kernel_table(dev, seed=0, only="", design="nepulix"):
     """The rows of a design's kernels behind those of the models it is measured against."""
     t = KernelTable(dev, seed, only)
@@ -395,6 +509,11 @@ def kernel_table(dev, seed=0, only="", design="nepulix"):
     if design == "sozarax":
         decayed_kernels(t, "retention", 16, 16, 128, 128, True)
         sozarax_kernels(t)
+    elif design == "lulizen":
+        sozarax_attention(t)
+        sozarax_experts(t)
+        sozarax_residual(t)
+        lulizen_kernels(t)
     else:
         nepulix_kernels(t)
     return t.rows

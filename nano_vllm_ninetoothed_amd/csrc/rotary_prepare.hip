@@ -2,8 +2,8 @@
 // an optional RMS norm per head on q and k (one weight for all heads), a rotation of their first `rot` elements by the token's
 // position, q to its own rows, k and v to their pages.  Pair i of a rotation is (element i, element i + rot / 2).
 //
-// LANES lanes own one head of one token, eight elements each; what a lane needs of the other half of a pair it reads again.
-// Heads wider than that, or of odd sizes: a wave per head, element by element.
+// LANES lanes own one head of one token, eight elements each, and take the other half of a pair from the lane that holds it.  Heads
+// wider than that, or of odd sizes: a wave per head, element by element, with the other half read again.
 #include "mixed_types.h"
 
 namespace mops {
@@ -33,11 +33,45 @@ __global__ __launch_bounds__(256) void rotary_prepare_kernel(const mops_hip_rota
     }
     return;
   }
+  const int rot = (int)a.rot, half = rot / 2;
+  int64_t pos = a.positions[t];
+  pos = pos < 0 ? 0 : (pos < a.max_positions ? pos : a.max_positions - 1);
+  const float* trig = a.cos_sin + pos * rot;
   const bool is_q = h < heads;
   const T* src = row + h * dim;
   T* dst = is_q ? (T*)a.q + (t * heads + h) * dp : (T*)a.k_pages + (slot * groups + h - heads) * dp;
   const T* w = (const T*)(is_q ? a.q_weight : a.k_weight);
   if (!is_q && !filed) return;
+  if (VEC == 8) {
+    const int c = lane * 8;
+    const bool mine = c < dim, turns = c < rot, low = c < half;
+    float v[VEC];
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) v[e] = 0.f;
+    if (mine) load_vec<VEC>(src + c, v);
+    float cs[VEC], sn[VEC];
+    if (turns) {
+      load_vec<VEC>(trig + (low ? c : c - half), cs);
+      load_vec<VEC>(trig + half + (low ? c : c - half), sn);
+    }
+    if (w) {
+      float ss = 0.f, wv[VEC];
+      if (mine) load_vec<VEC>(w + c, wv);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) ss += v[e] * v[e];
+      const float r = 1.0f / sqrtf(group_sum<LANES>(ss) / (float)dim + a.eps);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) v[e] = mine ? v[e] * r * wv[e] : 0.f;
+    }
+    const int from = turns ? lane + (low ? half : -half) / 8 : lane;
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) {
+      const float o = __shfl(v[e], from, LANES);
+      if (turns) v[e] = low ? v[e] * cs[e] - o * sn[e] : v[e] * cs[e] + o * sn[e];
+    }
+    if (mine) store_vec<VEC>(dst + c, v);
+    return;
+  }
   float r = 1.f;
   if (w) {
     float ss = 0.f;
@@ -49,10 +83,6 @@ __global__ __launch_bounds__(256) void rotary_prepare_kernel(const mops_hip_rota
     }
     r = 1.0f / sqrtf(group_sum<LANES>(ss) / (float)dim + a.eps);
   }
-  const int rot = (int)a.rot, half = rot / 2;
-  int64_t pos = a.positions[t];
-  pos = pos < 0 ? 0 : (pos < a.max_positions ? pos : a.max_positions - 1);
-  const float* trig = a.cos_sin + pos * rot;
   auto normed = [&](int c, float (&v)[VEC]) {
     load_vec<VEC>(src + c, v);
     if (w) {
@@ -66,7 +96,7 @@ __global__ __launch_bounds__(256) void rotary_prepare_kernel(const mops_hip_rota
     float v[VEC];
 #pragma unroll
     for (int e = 0; e < VEC; ++e) v[e] = 0.f;
-    if (VEC > 1 || c < dim) {
+    if (c < dim) {
       normed(c, v);
       if (c < rot) {
         const bool low = c < half;
@@ -97,13 +127,14 @@ extern "C" int mops_hip_rotary_prepare(const mops_hip_rotary_prepare_args* a, vo
                    aligned16(a->k_pages) && aligned16(a->v_pages) && aligned16(a->cos_sin) && (!a->q_weight || aligned16(a->q_weight)) &&
                    (!a->k_weight || aligned16(a->k_weight));
   const int64_t items = a->heads + 2 * a->kv_heads, widest = a->dim > a->vdim ? a->dim : a->vdim;
-  const int lanes = !vec ? 64 : (widest <= 64 ? 8 : (widest <= 128 ? 16 : 32));
+  const bool wide = vec && widest <= 256;
+  const int lanes = !wide ? 64 : (widest <= 64 ? 8 : (widest <= 128 ? 16 : 32));
   const int64_t wgs = (a->tokens * items + 256 / lanes - 1) / (256 / lanes);
   if (wgs > 0x7fffffffLL) return MOPS_HIP_EUNSUPPORTED;
   hipStream_t s = (hipStream_t)stream;
 #define MOPS_RP(T, V, L) hipLaunchKernelGGL((rotary_prepare_kernel<T, V, L>), dim3((unsigned)wgs), dim3(256), 0, s, *a, (int)items)
 #define MOPS_RP_TYPE(T) do {              \
-    if (!vec) MOPS_RP(T, 1, 64);          \
+    if (!wide) MOPS_RP(T, 1, 64);         \
     else if (lanes == 8) MOPS_RP(T, 8, 8);   \
     else if (lanes == 16) MOPS_RP(T, 8, 16); \
     else MOPS_RP(T, 8, 32);               \

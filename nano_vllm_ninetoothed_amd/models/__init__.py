@@ -42,7 +42,11 @@ def model_class(config):
 def load_config(path):
     """The configuration object of a folder's config.json ("architecture", or the first of "architectures")."""
     p = Path(path)
-    raw = json.loads((p / "config.json" if p.is_dir() else p).read_text())
+    return parse_config(json.loads((p / "config.json" if p.is_dir() else p).read_text()))
+
+
+def parse_config(raw: dict):
+    """The same from what config.json holds."""
     name = raw.get("architecture") or (raw.get("architectures") or [None])[0]
     cls = _BY_ARCHITECTURE.get(name)
     if cls is None:

@@ -12,6 +12,7 @@ import math
 import torch
 
 _round = None      # see sixteen_bit_products
+_margins = None    # see watching_choices
 
 
 @contextlib.contextmanager
@@ -33,6 +34,18 @@ def sixteen_bit_products(seed=0):
         yield
     finally:
         _round = None
+
+
+@contextlib.contextmanager
+def watching_choices():
+    """Inside, every choice of experts appends how far it is from another one: per token the smaller of two gaps, between the last
+    expert taken and the first one left, and (halved: two scores add up) between the last group kept and the first one dropped."""
+    global _margins
+    _margins = []
+    try:
+        yield _margins
+    finally:
+        _margins = None
 
 
 def product(x, w):
@@ -154,7 +167,16 @@ def choose(scores, correction, top, groups):
     size = E // groups["count"]
     best = c.view(T, groups["count"], size).topk(min(2, size), dim=-1).values.sum(dim=-1)
     kept = torch.zeros_like(best, dtype=torch.bool).scatter(1, best.topk(groups["keep"], dim=-1).indices, True)
-    return c.masked_fill(~kept.repeat_interleave(size, dim=1), -math.inf).topk(top, dim=-1).indices
+    c = c.masked_fill(~kept.repeat_interleave(size, dim=1), -math.inf)
+    if _margins is not None:
+        _margins.append(torch.minimum(_gap(c, top), _gap(best, groups["keep"]) / 2))
+    return c.topk(top, dim=-1).indices
+
+
+def _gap(x, n):
+    """Between the n-th largest of a row and the next one."""
+    s = torch.cat((x.sort(dim=-1, descending=True).values, torch.full((x.shape[0], 1), -math.inf, dtype=x.dtype)), dim=1)
+    return s[:, n - 1] - s[:, n]
 
 
 def route(h, router, correction, m):

@@ -2,37 +2,12 @@
 import pytest
 import torch
 
+from op_harness import bounds, i32, limit, op, padded_rows, paged_case, rel
 from oracle import sozarax as O
 
 pytestmark = pytest.mark.gpu
 DTYPES = [torch.float32, torch.bfloat16]
 D = torch.float64
-
-
-def op(name):
-    from nano_vllm_ninetoothed_amd import mops
-    return mops.get_op(name, "hip")
-
-
-def rel(got, want):
-    got = got.double().cpu()
-    assert torch.isfinite(got).all()
-    return ((got - want).norm() / want.norm()).item()
-
-
-def limit(dtype, f32=1e-6, bf16=3e-3):
-    return f32 if dtype == torch.float32 else bf16
-
-
-def i32(x, gpu):
-    return torch.tensor(x, dtype=torch.int32, device=gpu)
-
-
-def bounds(counts):
-    cu = [0]
-    for n in counts:
-        cu.append(cu[-1] + n)
-    return cu
 
 
 # ---------------------------------------------------------------------------------------------------- residual, norms, activations
@@ -209,36 +184,6 @@ def test_attention_prepare(gpu, dtype, H, G, d, v):
     assert torch.equal(vf[..., :v], values[ok]) and (vf[..., v:] == 0).all()
     rest = [s for s in range(32) if s not in at]
     assert kp.view(32, -1)[rest].isnan().all() and vp.view(32, -1)[rest].isnan().all()
-
-
-def paged_case(gpu, dtype, H, G, d, v, lens, bs, seed, far=()):
-    """Random queries, keys and values of several sequences in shuffled pages that hold garbage elsewhere.  far: positions whose key
-    looks like the last query, so that it stands out of all others."""
-    from nano_vllm_ninetoothed_amd.mops.hip.attention_ops import padded
-    g = torch.Generator().manual_seed(seed)
-    blocks = [-(-n // bs) for n in lens]
-    total = sum(blocks) + 2
-    perm = torch.randperm(total, generator=g).tolist()
-    kp, vp = (torch.full((total, bs, G, padded(s)), float("nan"), dtype=dtype) for s in (d, v))
-    table = torch.full((len(lens), max(max(blocks), 1)), -1, dtype=torch.int32)
-    seqs = []
-    for i, n in enumerate(lens):
-        q, k, val = torch.randn((n, H, d), generator=g), torch.randn((n, G, d), generator=g), torch.randn((n, G, v), generator=g)
-        for p in far:
-            if p < n:
-                k[p] = 3 * q[-1].view(G, H // G, d)[:, 0]
-        q, k, val = q.to(dtype), k.to(dtype), val.to(dtype)
-        for b in range(blocks[i]):
-            table[i, b] = page = perm.pop()
-            m = min(bs, n - b * bs)
-            kp[page, :m], vp[page, :m] = 0, 0
-            kp[page, :m, :, :d], vp[page, :m, :, :v] = k[b * bs:b * bs + m], val[b * bs:b * bs + m]
-        seqs.append((q, k, val))
-    return seqs, kp.to(gpu), vp.to(gpu), table.to(gpu)
-
-
-def padded_rows(q, d):
-    return torch.nn.functional.pad(q, (0, -d % 8)).contiguous()
 
 
 SIZES = [(8, 2, 64, 64), (6, 3, 20, 13), (1, 1, 8, 40), (20, 1, 128, 128), (4, 4, 200, 24), (3, 1, 24, 256), (16, 8, 128, 128)]
