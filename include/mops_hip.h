@@ -649,6 +649,9 @@ int mops_hip_biased_prefill(const mops_hip_biased_attention* a, const int32_t* t
  * (float [experts]), a group's score the sum of its two largest ones; the best `top` experts of the best `keep` groups are chosen, and
  * score = factor * sigmoid(logit) over the sum of the chosen ones' + 1e-20.  moe_down multiplies by it, and moe_gate_up does not.
  * unit 1: moe_gate_up gives g sigmoid(alpha g) (u + 1) with g = min(W_gate h, limit), u = W_up h between -limit and limit.
+ * common_w: a unit that every token goes through, in the same launches (bf16, block_rows 32, unit 1; NULL: none).  moe_gate_up:
+ * common_x [tokens, width], common_w gate rows from 0 and up rows from common_up_at on, [.., width], common_out [tokens, common_ff];
+ * moe_down: common_x [tokens, common_ff], common_w [width, common_ff], common_out [tokens, width].
  */
 typedef struct {
   int32_t *rows, *tiles;
@@ -659,7 +662,10 @@ typedef struct {
   float limit, alpha;
   const float* correction;
   int64_t groups, keep;
-  float factor;
+  float factor, common_limit;
+  const void *common_x, *common_w;
+  void* common_out;
+  int64_t common_x_stride, common_out_stride, common_ff, common_up_at;
 } mops_hip_moe;
 int64_t mops_hip_moe_max_tiles(int64_t tokens, int64_t experts, int64_t top, int64_t block_rows);
 int64_t mops_hip_moe_route_workgroups(int64_t tokens);

@@ -70,7 +70,9 @@ class Moe(Structure):
     """mops_hip_moe of the header, field by field."""
     _fields_ = ([(n, c_void_p) for n in ("rows", "tiles", "score")]
                 + [(n, c_int64) for n in ("tokens", "experts", "top", "width", "ff", "block_rows")] + [("dtype", c_int), ("unit", c_int)]
-                + [("limit", c_float), ("alpha", c_float), ("correction", c_void_p), ("groups", c_int64), ("keep", c_int64), ("factor", c_float)])
+                + [("limit", c_float), ("alpha", c_float), ("correction", c_void_p), ("groups", c_int64), ("keep", c_int64), ("factor", c_float)]
+                + [("common_limit", c_float)] + [(n, c_void_p) for n in ("common_x", "common_w", "common_out")]
+                + [(n, c_int64) for n in ("common_x_stride", "common_out_stride", "common_ff", "common_up_at")])
 
 
 # name -> (restype, argtypes); the exported surface declared in include/mops_hip.h

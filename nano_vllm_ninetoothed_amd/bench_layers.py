@@ -432,7 +432,7 @@ def sozarax_kernels(t):
 def lulizen_kernels(t):
     from .layers import Rotary
     from .mops.hip.attention_ops import Scores, biased_prefill_tiles
-    from .mops.hip.mixture_ops import Weighted
+    from .mops.hip.mixture_ops import CommonUnit, Weighted
     add, rnd, i32, dev = _handles(t)
     # ---- attention
     ctx, blocks, table, lens_g = decode_contexts(t)
@@ -476,6 +476,14 @@ def lulizen_kernels(t):
         gu, down = [rnd(experts, 2, ff, wd) for _ in range(sets)], [rnd(experts, wd, ff) for _ in range(sets)]
         routing = [op("moe_route")(x, router, top, weighted=form) for x in h]
         ys = [op("moe_gate_up")(h[i], gu[i], routing[i], 7.0) for i in range(sets)]
+        if tokens != T:
+            fs = ff * top // 2
+            cu = [CommonUnit(rnd(2 * fs, wd), rnd(wd, fs), fs, fs, 7.0) for _ in range(sets)]
+            yc = rnd(tokens, fs)
+            add("moe_gate_up", f"{tag}, and a shared unit of {fs}", lambda: graph_time(lambda i: op("moe_gate_up")(h[i % sets], gu[i % sets], routing[i % sets], 7.0, common=cu[i % sets]), 8),
+                nbytes=(experts * ff + fs) * 2.0 * wd * 2 + tokens * wd * 2.0 + (n * ff + tokens * fs) * 2.0, flops=4.0 * (n * ff + tokens * fs) * wd, like=f"moe_gate_up {tag}")
+            add("moe_down", f"{tag}, and a shared unit of {fs}", lambda: graph_time(lambda i: op("moe_down")(ys[i % sets], down[i % sets], routing[i % sets], cu[i % sets], yc), 8),
+                nbytes=(experts * ff + fs) * wd * 2.0 + (n * ff + tokens * fs) * 2.0 + (n + tokens) * wd * 2.0, flops=2.0 * (n * ff + tokens * fs) * wd, like=f"moe_down {tag}")
         add("moe_route", f"{tag}, 2 of 4 groups", lambda: graph_time(lambda i: op("moe_route")(h[i % sets], router, top, weighted=form), 8), nbytes=tokens * wd * 2.0 + n * 24,
             like=f"moe_route {tag}")
         add("moe_gate_up", f"{tag}, clamped", lambda: graph_time(lambda i: op("moe_gate_up")(h[i % sets], gu[i % sets], routing[i % sets], 7.0), 8),

@@ -9,6 +9,7 @@
 //                or g sigmoid(alpha g) (u + 1) with g = min(W_gate h, limit), u = W_up h between -limit and limit
 //   moe_down     z[choice] = W_down y[row], times the choice's weight in the second form
 //   grouped_linear   the products of the small blocks without routing: equal runs of rows, each with weights of its own
+// A unit that all tokens share can be part of both launches of the small blocks: workgroups of its own, which come first.
 //
 // The products are grouped: a workgroup takes a block of rows of one expert and some of its outputs.  Nothing comes back to the
 // host: the grids are sized for the largest possible number of blocks, and workgroups without one leave.  The order of an
@@ -433,21 +434,27 @@ struct GroupedArgs {
   int n_last;
   void* out_last;
   int64_t out_last_stride;
+  // small blocks with a shared unit: the first `ahead` workgroups (a multiple of 8); its rows are the tokens, and more is its own
+  int ahead, tokens;
+  const void* x_last;
+  int64_t x_last_stride;
+  int up_last, depth_last;
+  float limit_last;
 };
 
 // The gated unit of an expert: s the choice's score, g and u the products of its token.
 template <typename T>
-__device__ __forceinline__ float gated_unit(const GroupedArgs& a, float s, float g, float u) {
+__device__ __forceinline__ float gated_unit(const GroupedArgs& a, float limit, float s, float g, float u) {
   if (a.unit == 0) return silu_for<T>(s * g) * (s * u);
-  g = fminf(g, a.limit);
-  u = fminf(fmaxf(u, -a.limit), a.limit);
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
   return g * sigmoid_for<T>(a.alpha * g) * (u + 1.0f);
 }
 
 // This workgroup's tile and block of outputs.  Consecutive workgroups go to different XCDs: each XCD gets a contiguous run of
 // tiles with all their outputs, so that the rows of a tile and the weights of an expert meet in one L2.
 __device__ __forceinline__ bool grouped_item(const GroupedArgs& a, int& tile, int& block) {
-  const int n = a.tiles[0], per = (n + 7) / 8, i = blockIdx.x / 8;
+  const int n = a.tiles[0], per = (n + 7) / 8, i = ((int)blockIdx.x - a.ahead) / 8;
   tile = (blockIdx.x % 8) * per + i / a.blocks;
   block = i % a.blocks;
   return i / a.blocks < per && tile < n;
@@ -552,7 +559,7 @@ __global__ __launch_bounds__(256, 2) void moe_grouped_large_kernel(const Grouped
         const int n = n0 + (GATED ? 32 * wn : 64 * wn + 32 * i) + 8 * q4 + 4 * hh;
         float v[4];
 #pragma unroll
-        for (int x = 0; x < 4; ++x) v[x] = GATED ? gated_unit<bf16_t>(a, s, acc[0][j][4 * q4 + x], acc[1][j][4 * q4 + x]) : s * acc[i][j][4 * q4 + x];
+        for (int x = 0; x < 4; ++x) v[x] = GATED ? gated_unit<bf16_t>(a, a.limit, s, acc[0][j][4 * q4 + x], acc[1][j][4 * q4 + x]) : s * acc[i][j][4 * q4 + x];
         if (ALIGNED && n + 4 <= a.n) {
           *reinterpret_cast<u32x2*>(o + n) = u32x2{pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3])};
         } else {
@@ -573,9 +580,30 @@ __global__ __launch_bounds__(256, 3) void moe_grouped_small_kernel(const Grouped
   __shared__ __align__(16) f32x4 part[4][8][64];      // [wave][piece of the weights, piece of the rows][lane]
   int tile, block;
   int e, row0, count, n_all = a.n;
-  const uint16_t* w_group;
+  int depth = a.depth, up_at = a.up_at;
+  float limit = a.limit;
+  const uint16_t *w_group, *xs = (const uint16_t*)a.x;
+  int64_t x_stride = a.x_stride;
   bool last = false;
-  if (a.tiles) {
+  const bool common = a.tiles && (int)blockIdx.x < a.ahead;
+  if (common) {
+    // each XCD takes every eighth block of weights, with all row tiles
+    const int per = (a.tokens + kSM - 1) / kSM, c = (int)blockIdx.x;
+    tile = c / 8 % per;
+    block = c % 8 + 8 * (c / 8 / per);
+    e = 0;
+    row0 = tile * kSM;
+    count = a.tokens - row0 < kSM ? a.tokens - row0 : kSM;
+    last = true;
+    n_all = a.n_last;
+    w_group = (const uint16_t*)a.w_last;
+    xs = (const uint16_t*)a.x_last;
+    x_stride = a.x_last_stride;
+    depth = a.depth_last;
+    up_at = a.up_last;
+    limit = a.limit_last;
+    if (block * (GATED ? 32 : 64) >= n_all) return;
+  } else if (a.tiles) {
     if (!grouped_item(a, tile, block)) return;
     e = a.tiles[1 + 3 * tile];
     row0 = a.tiles[2 + 3 * tile];
@@ -600,12 +628,12 @@ __global__ __launch_bounds__(256, 3) void moe_grouped_small_kernel(const Grouped
 #pragma unroll
   for (int j = 0; j < 2; ++j) {
     const int r = 16 * j + col, src = row0 + (r < count ? r : count - 1);
-    x[j] = (const uint16_t*)a.x + (int64_t)(GATED ? a.rows[src] / a.top : src) * a.x_stride;
+    x[j] = xs + (int64_t)(GATED && !common ? a.rows[src] / a.top : src) * x_stride;
   }
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int n = n0 + 16 * (GATED ? i & 1 : i) + col;      // outputs behind the last are row 0 again and never stored
-    w[i] = w_group + (int64_t)((n < n_all ? n : 0) + (GATED && i >= 2 ? a.up_at : 0)) * a.depth;
+    w[i] = w_group + (int64_t)((n < n_all ? n : 0) + (GATED && i >= 2 ? up_at : 0)) * depth;
   }
   f32x4 acc[4][2];
 #pragma unroll
@@ -614,24 +642,24 @@ __global__ __launch_bounds__(256, 3) void moe_grouped_small_kernel(const Grouped
     for (int j = 0; j < 2; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
   // a wave takes every fourth piece of 32 of the depth, with two pieces in flight while one is used
   u32x4 xr[3][2], wr[3][4];
-  const int pieces = (a.depth - 32 * wave + 127) / 128;
+  const int pieces = (depth - 32 * wave + 127) / 128;
   auto fetch = [&](int buf, int piece) {
     const int k = 32 * wave + 128 * piece + 8 * jj;
     if (ALIGNED) {
-      const bool ok = k < a.depth;
+      const bool ok = k < depth;
 #pragma unroll
       for (int i = 0; i < 4; ++i) wr[buf][i] = load16(w[i] + (ok ? k : 0));
 #pragma unroll
       for (int j = 0; j < 2; ++j) xr[buf][j] = load16(x[j] + (ok ? k : 0));
     } else {
 #pragma unroll
-      for (int i = 0; i < 4; ++i) wr[buf][i] = load8_guarded(w[i], k, a.depth, false);
+      for (int i = 0; i < 4; ++i) wr[buf][i] = load8_guarded(w[i], k, depth, false);
 #pragma unroll
-      for (int j = 0; j < 2; ++j) xr[buf][j] = load8_guarded(x[j], k, a.depth, false);
+      for (int j = 0; j < 2; ++j) xr[buf][j] = load8_guarded(x[j], k, depth, false);
     }
   };
   auto use = [&](int buf, int piece) {
-    const bool ok = 32 * wave + 128 * piece + 8 * jj < a.depth;      // what lies behind the depth counts as zeros on both sides
+    const bool ok = 32 * wave + 128 * piece + 8 * jj < depth;      // what lies behind the depth counts as zeros on both sides
     const u32x4 zero = {0u, 0u, 0u, 0u};
 #pragma unroll
     for (int j = 0; j < 2; ++j) {
@@ -665,16 +693,16 @@ __global__ __launch_bounds__(256, 3) void moe_grouped_small_kernel(const Grouped
   auto total = [&](int piece) { return (part[0][piece][lane] + part[1][piece][lane]) + (part[2][piece][lane] + part[3][piece][lane]); };
   const f32x4 v0 = total(2 * i + j), v1 = total(2 * (i + 2) + j);
   if (r >= count) return;
-  const int choice = a.rows ? a.rows[row0 + r] : row0 + r;
+  const int choice = a.rows && !common ? a.rows[row0 + r] : row0 + r;
   uint16_t* o = last ? (uint16_t*)a.out_last + (int64_t)(choice - e * a.per_group) * a.out_last_stride
                      : (uint16_t*)a.out + (int64_t)(GATED ? row0 + r : choice) * a.out_stride;
-  const float s = GATED != a.weigh ? a.score[choice] : 1.f;
+  const float s = GATED != a.weigh && !common ? a.score[choice] : 1.f;
 #pragma unroll
   for (int half = 0; half < (GATED ? 1 : 2); ++half) {
     const int n = n0 + 16 * (i + 2 * half) + 4 * jj;
     float y[4];
 #pragma unroll
-    for (int q = 0; q < 4; ++q) y[q] = GATED ? gated_unit<bf16_t>(a, s, v0[q], v1[q]) : s * (half ? v1[q] : v0[q]);
+    for (int q = 0; q < 4; ++q) y[q] = GATED ? gated_unit<bf16_t>(a, limit, s, v0[q], v1[q]) : s * (half ? v1[q] : v0[q]);
     if (ALIGNED && n + 4 <= n_all) {
       *reinterpret_cast<u32x2*>(o + n) = u32x2{pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3])};
     } else {
@@ -728,7 +756,7 @@ __global__ __launch_bounds__(256) void moe_grouped_f32_kernel(const GroupedArgs 
     const int choice = a.rows[row0 + row];
     const float s = GATED != a.weigh ? a.score[choice] : 1.f;
     ((float*)a.out)[(int64_t)(GATED ? row0 + row : choice) * a.out_stride + n] =
-        GATED ? gated_unit<float>(a, s, acc[0][r], acc[GATED ? 1 : 0][r]) : s * acc[0][r];
+        GATED ? gated_unit<float>(a, a.limit, s, acc[0][r], acc[GATED ? 1 : 0][r]) : s * acc[0][r];
   }
 }
 
@@ -737,11 +765,16 @@ static int launch_grouped(GroupedArgs a, int dtype, int64_t block_rows, int64_t 
   const int64_t tiles = choices / block_rows + (experts < choices ? experts : choices);
   const int per = dtype == MOPS_HIP_F32 ? 64 : (block_rows == kSM ? (GATED ? 32 : 64) : (GATED ? 64 : 128));
   a.blocks = (a.n + per - 1) / per;
-  const int64_t grid_size = (tiles + 7) / 8 * 8 * a.blocks;
+  int64_t grid_size = (tiles + 7) / 8 * 8 * a.blocks;
+  const int64_t ahead = a.w_last ? (int64_t)((a.n_last + per - 1) / per + 7) / 8 * 8 * ((a.tokens + kSM - 1) / kSM) : 0;
+  a.ahead = (int)(ahead < 0x7fffffffLL ? ahead : 0x7fffffffLL);
+  grid_size += ahead;
   if (grid_size > 0x7fffffffLL) return MOPS_HIP_EUNSUPPORTED;
   const dim3 grid((unsigned)grid_size), block(256);
   const bool aligned = a.depth % 8 == 0 && a.x_stride % 8 == 0 && a.out_stride % 4 == 0 && a.w_expert % 8 == 0 && aligned16(a.x) && aligned16(a.w) &&
-                       aligned16(a.out);
+                       aligned16(a.out) &&
+                       (!a.w_last || (a.depth_last % 8 == 0 && a.x_last_stride % 8 == 0 && a.out_last_stride % 4 == 0 && aligned16(a.x_last) &&
+                                      aligned16(a.w_last) && aligned16(a.out_last)));
   if (dtype == MOPS_HIP_F32) {
     hipLaunchKernelGGL((moe_grouped_f32_kernel<GATED>), grid, block, 0, s, a);
   } else if (block_rows == kSM) {
@@ -771,7 +804,22 @@ static int check_grouped(const mops_hip_moe* m) {
   if (m->groups < 0 || (m->groups > 0 && (m->experts % m->groups || m->keep <= 0 || m->keep > m->groups || m->top > m->experts / m->groups * m->keep)))
     return MOPS_HIP_EINVAL;
   if (m->unit != 0 && m->unit != 1) return MOPS_HIP_EINVAL;
+  if (m->common_w) {
+    if (m->block_rows != kSM || m->dtype != MOPS_HIP_BF16 || !m->common_x || !m->common_out || m->common_ff <= 0) return MOPS_HIP_EINVAL;
+    if (m->common_ff > (1 << 20) || m->common_up_at > (1 << 20)) return MOPS_HIP_EUNSUPPORTED;
+  }
   return 1;
+}
+
+// What both launches say about the shared unit.
+static void set_common(GroupedArgs& a, const mops_hip_moe* m) {
+  a.w_last = m->common_w;
+  a.x_last = m->common_x;
+  a.out_last = m->common_out;
+  a.x_last_stride = m->common_x_stride;
+  a.out_last_stride = m->common_out_stride;
+  a.limit_last = m->common_limit;
+  a.tokens = (int)m->tokens;
 }
 
 }  // namespace mops
@@ -837,6 +885,11 @@ extern "C" int mops_hip_moe_gate_up(const void* h, int64_t h_row_stride, const v
   a.n = (int)m->ff; a.up_at = (int)up_at; a.depth = (int)m->width; a.out = y; a.out_stride = y_row_stride;
   a.rows = m->rows; a.tiles = m->tiles; a.score = m->score; a.top = (int)m->top; a.blocks = 0;
   a.unit = m->unit; a.limit = m->limit; a.alpha = m->alpha; a.weigh = m->groups > 0;
+  if (m->common_w) {
+    if (m->unit != 1 || m->common_up_at < m->common_ff || m->common_x_stride < m->width || m->common_out_stride < m->common_ff) return MOPS_HIP_EINVAL;
+    set_common(a, m);
+    a.n_last = (int)m->common_ff; a.up_last = (int)m->common_up_at; a.depth_last = (int)m->width;
+  }
   return launch_grouped<true>(a, m->dtype, m->block_rows, m->tokens * m->top, m->experts, (hipStream_t)stream);
 }
 
@@ -850,6 +903,11 @@ extern "C" int mops_hip_moe_down(const void* y, int64_t y_row_stride, const void
   a.x = y; a.x_stride = y_row_stride; a.w = w; a.w_expert = depth * m->width;
   a.n = (int)m->width; a.up_at = 0; a.depth = (int)depth; a.out = z; a.out_stride = z_row_stride;
   a.rows = m->rows; a.tiles = m->tiles; a.score = m->score; a.top = (int)m->top; a.blocks = 0; a.weigh = m->groups > 0;
+  if (m->common_w) {
+    if (m->common_x_stride < m->common_ff || m->common_out_stride < m->width) return MOPS_HIP_EINVAL;
+    set_common(a, m);
+    a.n_last = (int)m->width; a.depth_last = (int)m->common_ff;
+  }
   return launch_grouped<false>(a, m->dtype, m->block_rows, m->tokens * m->top, m->experts, (hipStream_t)stream);
 }
 

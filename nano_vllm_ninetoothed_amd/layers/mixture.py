@@ -5,7 +5,7 @@ import torch
 
 from . import hip_op, register_feed_forward, require_size
 from .feed_forward import ClampedGLU
-from ..mops.hip.mixture_ops import Weighted
+from ..mops.hip.mixture_ops import CommonUnit, Weighted
 
 
 class Mixture:
@@ -73,8 +73,13 @@ class GroupedMixture(Mixture):
                                  float(router["scale"]))
         self.limit = float(sizes["expert"]["limit"])
         self.shared = ClampedGLU(sizes["shared"], weights, prefix + "shared.", m) if sizes.get("shared") is not None else None
+        s = self.shared
+        self.common = None if s is None else CommonUnit(s.gate_up, s.down.contiguous(), s.ff, s.half, s.limit)
 
     def __call__(self, x):
         routing = self.route(x, self.router, self.top, weighted=self.weighted)
+        if self.common is not None and routing.takes_common:      # small batches: in the experts' launches
+            y, yc = self.op_gate_up(x, self.gate_up, routing, self.limit, ClampedGLU.ALPHA, common=self.common)
+            return self.op_down(y, self.down, routing, common=self.common, common_y=yc)
         y = self.op_down(self.op_gate_up(x, self.gate_up, routing, self.limit, ClampedGLU.ALPHA), self.down, routing)
         return y if self.shared is None else (y, self.shared(x))

@@ -5,6 +5,8 @@ from __future__ import annotations
 
 from . import hip_op, pack, register_mixer, require_size
 from .paged_attention import PagedAttention
+
+PACKED_ROWS = 1024      # above, the few columns of the gates cost the packed product more than a product of their own
 from ..mops.hip.attention_ops import Scores
 
 
@@ -35,6 +37,7 @@ class RotaryAttention(PagedAttention):
             projections.append(take(prefix + "g", (h, m.width)))
         self.qkv = pack(projections)
         self.gate_at = (h + g) * d + g * v if self.GATE else None
+        self.gate_rows = pack([projections[-1]]) if self.GATE else None
         self.q_norm, self.k_norm = (take(prefix + n, (d,), "norm") if self.HEAD_NORMS else None for n in ("q.norm", "k.norm"))
         self.o = take(prefix + "o", (m.width, h * v))
         self.scores = Scores(softcap=float(sizes.get("softcap") or 0.0), **self.visible(sizes.get("mask")),
@@ -44,10 +47,13 @@ class RotaryAttention(PagedAttention):
         super().__init__(sizes, m)
 
     def __call__(self, x, ctx):
-        qkv = self.linear(x, self.qkv)
+        packed = x.shape[0] <= PACKED_ROWS or not self.GATE
+        qkv = self.linear(x, self.qkv if packed else self.qkv[:self.gate_at])
         q = self.prepare(qkv, ctx["positions32"], ctx["slot_mapping"], self.k_pages, self.v_pages, self.heads, self.kv_heads, self.dim, self.vdim,
                          cos_sin=self.trig, q_weight=self.q_norm, k_weight=self.k_norm, eps=self.eps)
-        gate = qkv[:, self.gate_at:self.gate_at + self.heads] if self.GATE else None
+        gate = None
+        if self.GATE:
+            gate = qkv[:, self.gate_at:self.gate_at + self.heads] if packed else self.linear(x, self.gate_rows)[:, :self.heads]
         return self.linear(self.attend(q, ctx, gate), self.o)
 
 

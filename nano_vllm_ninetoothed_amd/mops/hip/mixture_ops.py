@@ -24,6 +24,22 @@ class Routing:
     rows: torch.Tensor
     tiles: torch.Tensor
 
+    @property
+    def takes_common(self) -> bool:
+        """Whether the products take a unit that all tokens share along."""
+        return self.args.dtype == 0 and self.args.block_rows == SMALL_BLOCK
+
+
+@dataclass(frozen=True)
+class CommonUnit:
+    """A unit of clamped_glu's form that every token goes through: gate_up [2 * up_at or more, width] with gate rows from 0 and up rows
+    from up_at on, down [width, ff]."""
+    gate_up: torch.Tensor
+    down: torch.Tensor
+    ff: int
+    up_at: int
+    limit: float
+
 
 @dataclass(frozen=True)
 class Weighted:
@@ -66,9 +82,10 @@ def moe_route(h: torch.Tensor, router: torch.Tensor, top: int, block_rows: int =
 
 
 @register_hip_op
-def moe_gate_up(h: torch.Tensor, w: torch.Tensor, routing: Routing, limit: float = None, alpha: float = 1.702):
+def moe_gate_up(h: torch.Tensor, w: torch.Tensor, routing: Routing, limit: float = None, alpha: float = 1.702, common: CommonUnit = None):
     """silu(s W_gate h) * (s W_up h) of every choice, s its score, in the order of routing.rows.  w [experts, 2, ff, width].  With a
-    limit the unit of clamped_glu instead, which takes no score."""
+    limit the unit of clamped_glu instead, which takes no score; with a common unit (routing.takes_common) a pair, the second what
+    that unit makes of every token."""
     code = _dtype("h", h)
     m = routing.args
     experts, two, ff, width = w.shape
@@ -76,15 +93,27 @@ def moe_gate_up(h: torch.Tensor, w: torch.Tensor, routing: Routing, limit: float
     m.ff, m.unit = ff, 0 if limit is None else 1
     m.limit, m.alpha = limit or 0.0, alpha
     y = torch.empty((m.tokens * m.top, ff), dtype=h.dtype, device=h.device)
+    yc = None if common is None else torch.empty((m.tokens, common.ff), dtype=h.dtype, device=h.device)
+    if common is not None:
+        _require(limit is not None and common.gate_up.shape[0] >= common.up_at + common.ff, "a common unit comes with limits, and with all its rows")
+        _set_common(m, h, _rows("h", h, width, h.dtype), _flat("gate_up", common.gate_up, common.gate_up.shape[0] * width, h.dtype), yc, common)
     st = _capi.load().mops_hip_moe_gate_up(h.data_ptr(), _rows("h", h, width, h.dtype), _flat("w", w, w.numel(), h.dtype), ff, y.data_ptr(), ff, byref(m), _stream(h))
+    m.common_w = None
     _capi.check("mops_hip_moe_gate_up", st)
-    return y
+    return y if common is None else (y, yc)
+
+
+def _set_common(m, x, x_stride, w, out, common):
+    m.common_x, m.common_x_stride, m.common_w = x.data_ptr(), x_stride, w
+    m.common_out, m.common_out_stride = out.data_ptr(), out.shape[1]
+    m.common_ff, m.common_up_at, m.common_limit = common.ff, common.up_at, common.limit
 
 
 @register_hip_op
-def moe_down(y: torch.Tensor, w: torch.Tensor, routing: Routing):
+def moe_down(y: torch.Tensor, w: torch.Tensor, routing: Routing, common: CommonUnit = None, common_y: torch.Tensor = None):
     """W_down y of every choice, times its weight if the routing has weights: [tokens * top, width], a token's choices one behind the
-    other.  w [experts, width, ff]."""
+    other.  w [experts, width, ff].  common, common_y: the unit and its result of moe_gate_up; then a pair, the second what the unit
+    adds per token."""
     code = _dtype("y", y)
     m = routing.args
     experts, width, ff = w.shape
@@ -92,9 +121,14 @@ def moe_down(y: torch.Tensor, w: torch.Tensor, routing: Routing):
              "the routing was made for another problem")
     m.ff = ff
     z = torch.empty((m.tokens * m.top, width), dtype=y.dtype, device=y.device)
+    zc = None if common is None else torch.empty((m.tokens, width), dtype=y.dtype, device=y.device)
+    if common is not None:
+        _require(common_y.shape[0] == m.tokens, "common_y must have a row per token")
+        _set_common(m, common_y, _rows("common_y", common_y, common.ff, y.dtype), _flat("down", common.down, width * common.ff, y.dtype), zc, common)
     st = _capi.load().mops_hip_moe_down(y.data_ptr(), ff, _flat("w", w, w.numel(), y.dtype), ff, z.data_ptr(), width, byref(m), _stream(y))
+    m.common_w = None
     _capi.check("mops_hip_moe_down", st)
-    return z
+    return z if common is None else (z, zc)
 
 
 @register_hip_op

@@ -316,6 +316,28 @@ def test_weighted_mixture(gpu, dtype, block, tokens, width, ff, experts, top, co
     assert rel(z.view(tokens, top, width)[:n], want[:n]) < limit(dtype, 3e-6, 8e-3)
 
 
+@pytest.mark.parametrize("tokens,width,ff,experts,top,shared", [(1, 64, 32, 4, 1, 72), (70, 72, 24, 6, 2, 17), (33, 256, 136, 16, 4, 300), (64, 100, 16, 3, 2, 8), (150, 64, 24, 16, 2, 1030)])
+def test_a_shared_unit_in_the_launches_of_the_experts(gpu, tokens, width, ff, experts, top, shared):
+    from nano_vllm_ninetoothed_amd.mops.hip.mixture_ops import CommonUnit, Weighted
+    g = torch.Generator().manual_seed(shared)
+    rnd = lambda *s: (torch.randn(s, generator=g) * s[-1] ** -0.5).bfloat16().to(gpu)      # noqa: E731
+    h, pad, half = torch.randn((tokens, width), generator=g).bfloat16().to(gpu), (ff + 7) // 8 * 8, (shared + 7) // 8 * 8
+    gu, down, cg, cd = 2 * rnd(experts, 2, pad, width), rnd(experts, width, pad), 2 * rnd(half + (shared + 7) // 8 * 8, width), rnd(width, shared)
+    gu[:, :, ff:], down[:, :, ff:] = 0, 0
+    routing = op("moe_route")(h, rnd(experts, width), top, 32, weighted=Weighted(torch.randn(experts, generator=g).to(gpu), 1, 1, 1.0))
+    assert routing.takes_common
+    unit = CommonUnit(cg, cd, shared, half, 0.7)
+    y, yc = op("moe_gate_up")(h, gu, routing, 1.5, common=unit)
+    z, zc = op("moe_down")(y, down, routing, unit, yc)
+    assert torch.equal(y, op("moe_gate_up")(h, gu, routing, 1.5)) and torch.equal(z, op("moe_down")(y, down, routing))
+    w = {"gate": cg[:shared].double().cpu(), "up": cg[half:half + shared].double().cpu(), "down": cd.double().cpu()}
+    assert yc.shape == (tokens, shared) and rel(zc, O.clamped_unit(h.double().cpu(), w, 0.7)) < 8e-3
+    big = op("moe_route")(h, rnd(experts, width), top, 128, weighted=Weighted(torch.randn(experts, generator=g).to(gpu), 1, 1, 1.0))
+    assert not big.takes_common
+    with pytest.raises(Exception):
+        op("moe_gate_up")(h, gu, big, 1.5, common=unit)
+
+
 def test_groups_that_lose_are_out_even_with_the_best_expert(gpu):
     """The single best expert stands in a group whose two best add up to less; negative choice scores are still taken from kept groups."""
     from nano_vllm_ninetoothed_amd.mops.hip.mixture_ops import Weighted
