@@ -64,7 +64,7 @@ def lulizen_dict(width, layers, ff, vocab, heads, experts, top):
            "router": {"experts": experts, "top": top, "scale": 2.5, "groups": {"count": 4, "keep": 2}}}
     out = [{"type": kinds[i % 2][0], "mixer": kinds[i % 2][1], "mlp": {"kind": "dense", "ff": ff} if i % 3 == 0 else moe} for i in range(layers)]
     return {"architecture": "Lulizen", "width": width, "vocab": vocab, "norm": {"eps": 1e-6}, "layers": out,
-            "embedding": {"bigram": {"buckets": vocab - 1, "mul_prev": 31, "mul_cur": 17}}}
+            "embedding": {"bigram": {"buckets": vocab - 1, "mul_prev": 37, "mul_cur": 17}}}
 
 
 def lulizen_sizes():
@@ -498,7 +498,7 @@ def lulizen_kernels(t):
         sets = 24 if rows == 512 else 4
         res, yy, wa, wb = [t.f32(rows, n) for _ in range(sets)], [rnd(rows * parts, n) for _ in range(sets)], rnd(n), rnd(n)
         extra = [rnd(rows, n) if more else None for _ in range(sets)]
-        add("add_norm_norm", f"{rows} x {n}, layer norms, {parts}{' + 1' if more else ''} parts", lambda: graph_time(lambda i: op("add_norm_norm")(
+        add("add_norm_norm", f"{rows} x {n}, layer norms, {parts}{' + 1 parts' if more else ' part'}", lambda: graph_time(lambda i: op("add_norm_norm")(
             res[i % sets], yy[i % sets], wa, wb, 1e-6, center=True, extra=extra[i % sets]), 24 if rows == 512 else 8),
             nbytes=rows * n * (10.0 + 2 * (parts + more)), like=f"add_norm_norm {like}")
     res, w1 = [t.f32(T, 1024) for _ in range(4)], rnd(1024)
@@ -506,7 +506,7 @@ def lulizen_kernels(t):
     emb, pairs, ids = rnd(32768, 1024), rnd(32768, 1024), [torch.randint(0, 32768, (T,), device=dev) for _ in range(4)]
     before, cu16, z16, sl16 = torch.zeros(16, dtype=torch.int32, device=dev), i32(list(range(0, T + 1, 1024))), i32([0] * 16), torch.arange(16, dtype=torch.int32, device=dev)
     seq = torch.arange(T, device=dev).div(1024, rounding_mode="floor").to(torch.int32)
-    add("embed_pairs", f"{T} x 1024", lambda: graph_time(lambda i: op("embed_pairs")(ids[i % 4], emb, pairs, 31, 17, before, z16, sl16, seq, cu16), 8), nbytes=T * 1024 * 8.0,
+    add("embed_pairs", f"{T} x 1024", lambda: graph_time(lambda i: op("embed_pairs")(ids[i % 4], emb, pairs, 37, 17, before, z16, sl16, seq, cu16), 8), nbytes=T * 1024 * 8.0,
         like="add_rms prefill")
 
 

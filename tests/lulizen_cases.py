@@ -39,7 +39,7 @@ CONFIGS = {
     "odd": config(76, 101, [(windowed(6, 3, 22, 13, 14, 25, 5, 0.5, 9.0), moe(20, 6, 3, 3, 2, 36)), (chunked(4, 2, 19, 33, 6, 37, 0.3, 5.0), None),
                             (chunked(5, 5, 10, 9, 10, 50, 0.4, 12.0), moe(17, 5, 2, 5, 2, 9)), 0, 1, 0], (67, 13, 5)),
     # head sizes of large models, the second kind of attention first, one kv head and many, a cap beyond what needs no reference
-    "large": config(256, 264, [(chunked(24, 1, 128, 128, 128, 64, 0.09, 100.0, 5e5), moe(136, 16, 4, 4, 2, 200, 7.0, 5.0, 2.5)),
+    "large": config(256, 264, [(chunked(24, 1, 128, 128, 128, 64, 0.09, 100.0, 5e5), moe(136, 16, 4, 4, 2, 200, 7.0, 5.0, 2.2)),
                                (windowed(16, 8, 128, 128, 64, 128, 40, 0.08, 50.0), dense(512)),
                                (windowed(8, 2, 64, 64, 32, 33, 32, 0.12, 30.0), moe(64, 40, 6, 8, 3, 64, 2.0, 3.0, 1.0))], (1021, 7, 3)),
     # nearly everything that can be one is one: a token that sees itself only, or itself and the first
@@ -47,7 +47,7 @@ CONFIGS = {
                             (windowed(2, 1, 24, 16, 24, 30, 0, 0.4, 20.0), moe(8, 4, 1, 4, 1, 16))], (1, 1, 1), eps=1e-3),
     # values wider than the matrix-core kernels cover, keys wider than values, many experts in small groups, windows wider than a prompt
     "wide": config(128, 88, [(chunked(3, 3, 48, 280, 48, 1000, 0.25, 15.0), moe(24, 130, 2, 65, 60, 40)), (windowed(18, 1, 160, 24, 80, 4000, 3, 0.12, 25.0), dense(96)),
-                             (chunked(2, 1, 72, 40, 40, 90, 0.2, 8.0), moe(40, 12, 6, 2, 1, 56))], (500, 11, -3)),
+                             (chunked(2, 1, 72, 40, 40, 90, 0.2, 8.0), moe(40, 14, 6, 2, 1, 56))], (500, 11, -3)),
 }
 
 
