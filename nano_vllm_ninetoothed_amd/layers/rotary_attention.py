@@ -5,9 +5,9 @@ from __future__ import annotations
 
 from . import hip_op, pack, register_mixer, require_size
 from .paged_attention import PagedAttention
+from ..mops.hip.attention_ops import Scores
 
 PACKED_ROWS = 1024      # above, the few columns of the gates cost the packed product more than a product of their own
-from ..mops.hip.attention_ops import Scores
 
 
 class RotaryAttention(PagedAttention):
