@@ -336,10 +336,27 @@ int mops_hip_linear_tune(int64_t m, int64_t n, int64_t k, int64_t distinct_weigh
 #define MOPS_HIP_BF16 0
 #define MOPS_HIP_F32 1
 
-/* residual[i, :] = scale * table[ids[i], :] and act[i, :] = the same in `dtype` (act may be NULL); an id outside [0, vocab)
- * gives zeros. */
+/* residual[i, :] = scale * table[ids[i], :] and act[i, :] = the same in `dtype`, rows act_stride apart (act may be NULL); an id outside
+ * [0, vocab) gives zeros. */
 int mops_hip_embed_residual(const int64_t* ids, const void* table, int64_t table_row_stride, int dtype, float scale,
-                            float* residual, void* act, int64_t n_ids, int64_t vocab, int64_t width, void* stream);
+                            float* residual, void* act, int64_t act_stride, int64_t n_ids, int64_t vocab, int64_t width, void* stream);
+
+/*
+ * residual [rows, n] float += y + shift, or = y + shift with `replace`; y (`dtype`, rows y_stride apart) and shift (float [n]) may be NULL.
+ * out (`dtype`, rows out_stride apart, or NULL) = norm(residual) * w + b: RMS norms, or layer norms with `center`; w NULL: the residual.
+ */
+typedef struct {
+  float* residual;
+  const void* y;
+  int64_t y_stride;
+  const float* shift;
+  const void *w, *b;
+  void* out;
+  int64_t out_stride, rows, n;
+  float eps;
+  int replace, center, dtype;
+} mops_hip_add_norm_args;
+int mops_hip_add_norm(const mops_hip_add_norm_args* a, void* stream);
 
 /* residual += y / sqrt(mean(y^2) + eps) * (weight_offset + weight), rowwise and in place; act = the new residual in `dtype`. */
 int mops_hip_norm_residual_add(float* residual, const void* y, int64_t y_row_stride, const void* weight, float weight_offset,
@@ -384,18 +401,22 @@ int mops_hip_rms_norm_f32(const float* x, const void* weight, float weight_offse
 /*
  * Rows of groups * group_size elements, every group divided by its own root mean square:
  *   gate_first == 0:  out = rms(y) * silu(gate) [* weight];  else  out = rms(y * silu(gate)) [* weight].   weight may be NULL.
- * out is contiguous and may be y itself when y is contiguous.
+ * plain_sigmoid: sigmoid(gate) in the place of silu(gate).  shared_weight: weight [group_size] for all groups.  Everything times scale.
+ * out may be y itself when their strides agree.
  */
 int mops_hip_gated_group_norm(const void* y, int64_t y_row_stride, const void* gate, int64_t gate_row_stride,
-                              const void* weight, float eps, int gate_first, void* out, int dtype,
-                              int64_t rows, int64_t groups, int64_t group_size, void* stream);
+                              const void* weight, int shared_weight, float eps, int gate_first, int plain_sigmoid, float scale, void* out,
+                              int64_t out_row_stride, int dtype, int64_t rows, int64_t groups, int64_t group_size, void* stream);
 
 /* out = g * sigmoid(alpha * g) * (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit). */
 int mops_hip_clamped_glu(const void* gate, int64_t gate_row_stride, const void* up, int64_t up_row_stride, void* out,
-                         int dtype, int64_t rows, int64_t n, float alpha, float limit, void* stream);
+                         int64_t out_row_stride, int dtype, int64_t rows, int64_t n, float alpha, float limit, void* stream);
 /* out = gelu(gate) * up, gelu(z) = z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))) / 2. */
-int mops_hip_gelu_glu(const void* gate, int64_t gate_row_stride, const void* up, int64_t up_row_stride, void* out, int dtype,
-                      int64_t rows, int64_t n, void* stream);
+int mops_hip_gelu_glu(const void* gate, int64_t gate_row_stride, const void* up, int64_t up_row_stride, void* out,
+                      int64_t out_row_stride, int dtype, int64_t rows, int64_t n, void* stream);
+/* out = max(gate, 0) * up. */
+int mops_hip_relu_glu(const void* gate, int64_t gate_row_stride, const void* up, int64_t up_row_stride, void* out,
+                      int64_t out_row_stride, int dtype, int64_t rows, int64_t n, void* stream);
 
 /*
  * A linear recurrence with one decay per head and token (see csrc/decayed_recurrence.hip):
@@ -435,7 +456,19 @@ typedef struct {
   int64_t channel_decay_stride;
   float k_scale;
   int dtype;
+  const void *input_gate, *forget_gate;
+  int64_t gate_stride;
+  const float *input_bias, *forget_bias;
+  float* top;
+  const float *log_keep, *input_scale, *least;
+  float gate_cap;
 } mops_hip_recurrence;
+/*
+ * Matrix memory (input_gate given, in the place of a decay): gates are `dtype` [tokens, heads] with rows gate_stride apart, biases float
+ * [heads]; state [num_slots, heads, vd + copies, pitch] and top float [num_slots, heads, copies], copies = mops_hip_matrix_memory_copies.
+ * The chunked form takes the gates from mops_hip_matrix_memory_gates instead: log_keep, input_scale and least, float [tokens, heads].
+ */
+int64_t mops_hip_matrix_memory_copies(int64_t vd);
 int64_t mops_hip_recurrence_state_pitch(int64_t d);
 int mops_hip_decayed_recurrence(const mops_hip_recurrence* r, void* stream);
 
@@ -460,7 +493,34 @@ int mops_hip_channel_chunks(const mops_hip_recurrence* r, const int32_t* segment
                             const int32_t* seq_segments, float* seg_state, float* seg_decay, void* stream);
 
 /*
- * out[t, c] = silu(bias[c] + sum over lags l < taps of weight[taps-1-l, c] * x(position - l)[c]) for packed portions.
+ * The gated delta rule (csrc/delta_rule.hip): S <- exp(log_decay) S, u = sigmoid(beta) (v - S^T k), S <- S + k u^T, o = S^T q, with q and k
+ * divided by sqrt(sum of squares + unit_eps) per head and q multiplied by q_scale.  q, k: [tokens, groups * d], v, out: [tokens, heads *
+ * vd], beta: [tokens, heads] in `dtype`, log_decay: float [tokens, heads * d], all with row strides in elements; state: float [num_slots,
+ * heads, vd, pitch], pitch = mops_hip_recurrence_state_pitch(d).  Sequences, slots and the convolution (without a bias) as in
+ * mops_hip_recurrence.  d <= 512.
+ */
+typedef struct {
+  const void *q, *k, *v;
+  int64_t q_stride, k_stride, v_stride;
+  void* out;
+  int64_t out_stride;
+  float* state;
+  int64_t num_slots;
+  const int32_t *state_slots, *cu_seqlens, *starts;
+  const float* log_decay;
+  const void* beta;
+  int64_t log_decay_stride, beta_stride;
+  int64_t batch, heads, groups, d, vd;
+  const float* conv_weight;
+  void* conv_ring;
+  int64_t taps, channels, q_channel, k_channel, v_channel;
+  float q_scale, unit_eps;
+  int dtype;
+} mops_hip_delta;
+int mops_hip_delta_rule(const mops_hip_delta* a, void* stream);
+
+/*
+ * out[t, c] = silu(bias[c] (bias may be NULL) + sum over lags l < taps of weight[taps-1-l, c] * x(position - l)[c]) for packed portions.
  * weight: float [taps, channels]; x of earlier portions comes from ring [num_slots, taps, channels] (`dtype`), row
  * position % taps; positions before 0 count as zeros.  token_seq: int32 [tokens], the sequence of each token.
  */
@@ -544,13 +604,14 @@ int mops_hip_latent_prefill(const void* q, int64_t q_token_stride, int64_t q_hea
  * [parts, tokens, width].  The row in front of a sequence's first token of the step is row state_slots[b] of before
  * [num_slots, width] (zeros where starts[b] == 0 or the slot is negative), which receives the sequence's last row.
  * token_seq and cu_seqlens (both or neither): packed portions; NULL: one token per sequence.
- * low_rank_decay: out[t, c] = -exp(sum over r of w2[c, r] tanh(z[t, r]) + w0[c]), float; rank <= 4096.
+ * low_rank_decay: out[t, c] = -exp(sum over r of w2[c, r] tanh(z[t, r]) + w0[c]), float; rank <= 4096.  With rate (float
+ * [channels / head_size], else NULL) out[t, c] = rate[c / head_size] * softplus(sum over r of w2[c, r] z[t, r] + w0[c]).
  */
 int mops_hip_token_mix(const void* x, int64_t x_row_stride, const float* mu, int64_t parts, void* before, int64_t num_slots,
                        const int32_t* token_seq, const int32_t* cu_seqlens, const int32_t* starts, const int32_t* state_slots,
                        void* out, int dtype, int64_t tokens, int64_t width, void* stream);
-int mops_hip_low_rank_decay(const void* z, int64_t z_row_stride, const void* w2, const float* w0, float* out, int dtype,
-                            int64_t tokens, int64_t channels, int64_t rank, void* stream);
+int mops_hip_low_rank_decay(const void* z, int64_t z_row_stride, const void* w2, const float* w0, const float* rate, int64_t head_size,
+                            float* out, int dtype, int64_t tokens, int64_t channels, int64_t rank, void* stream);
 
 /* out = max(x, 0)^2. */
 int mops_hip_squared_relu(const void* x, int64_t x_row_stride, void* out, int dtype, int64_t rows, int64_t n, void* stream);
@@ -579,7 +640,8 @@ int mops_hip_attention_prepare(const mops_hip_attention_prepare_args* a, void* s
 /*
  * rotary_prepare (csrc/rotary_prepare.hip): the same for rotated queries and keys.  q_weight, k_weight [dim] or NULL: an RMS norm over
  * every head of q or k.  Then the pairs (i, i + rot / 2) of a head's first `rot` elements turn by the angles of the token's position:
- * cos_sin float [max_positions, rot], cosines, then sines.
+ * cos_sin float [max_positions, rot], cosines, then sines.  neighbours: the pairs are (2i, 2i + 1).  bias (`dtype`, as many elements as
+ * q, k and v have together, or NULL) is added in front of all that.
  */
 typedef struct {
   const void* qkv;
@@ -592,6 +654,8 @@ typedef struct {
   int64_t num_slots, tokens, heads, kv_heads, dim, vdim;
   float eps;
   int dtype;
+  const void* bias;
+  int64_t neighbours;
 } mops_hip_rotary_prepare_args;
 int mops_hip_rotary_prepare(const mops_hip_rotary_prepare_args* a, void* stream);
 
@@ -605,7 +669,11 @@ int mops_hip_rotary_prepare(const mops_hip_rotary_prepare_args* a, void* stream)
  *   chunk       position i sees the tokens of its chunk up to itself, chunks of `chunk` tokens from position 0 on; not with window
  *   keep_first  the first keep_first tokens stay visible
  *   sinks       float [heads]: exp(sinks[h]) is one more term of the softmax's denominator
- *   gate        `dtype` [rows, heads] with rows gate_stride apart: out is multiplied by its sigmoid
+ *   gate        `dtype` [rows, heads], or with gate_each [rows, heads * vdim], rows gate_stride apart: out is multiplied by its sigmoid
+ *   log_rate    float [heads], with log_step [heads]: score = q . k * scale - log_rate[h] * ln(1 + log_step[h] * distance)
+ *   weight_bias float [heads]: no softmax; a key counts with sigmoid(q . k * scale + weight_bias[h]).  Not with sinks
+ * At most one of softcap, slopes, log_rate and weight_bias.  Rows of out are out_stride apart (0: contiguous) and
+ * multiplied by out_scale (0: by one).
  * biased_attention_rows: the plain form; dim <= 2048, vdim <= 1024.
  */
 typedef struct {
@@ -622,6 +690,9 @@ typedef struct {
   const float* sinks;
   const void* gate;
   int64_t gate_stride;
+  const float *log_rate, *log_step, *weight_bias;
+  int64_t gate_each, out_stride;
+  float out_scale;
 } mops_hip_biased_attention;
 int mops_hip_biased_attention_rows(const mops_hip_biased_attention* a, void* stream);
 

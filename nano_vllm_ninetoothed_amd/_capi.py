@@ -22,7 +22,25 @@ class Recurrence(Structure):
                 + [(n, c_void_p) for n in ("conv_weight", "conv_bias", "conv_ring")]
                 + [(n, c_int64) for n in ("taps", "channels", "q_channel", "k_channel", "v_channel")]
                 + [("channel_decay", c_void_p), ("bonus", c_void_p), ("channel_decay_stride", c_int64)]
-                + [("k_scale", c_float), ("dtype", c_int)])
+                + [("k_scale", c_float), ("dtype", c_int)]
+                + [("input_gate", c_void_p), ("forget_gate", c_void_p), ("gate_stride", c_int64)]
+                + [(n, c_void_p) for n in ("input_bias", "forget_bias", "top", "log_keep", "input_scale", "least")] + [("gate_cap", c_float)])
+
+
+class Delta(Structure):
+    """mops_hip_delta of the header, field by field."""
+    _fields_ = ([(n, c_void_p) for n in ("q", "k", "v")] + [(n, c_int64) for n in ("q_stride", "k_stride", "v_stride")]
+                + [("out", c_void_p), ("out_stride", c_int64), ("state", c_void_p), ("num_slots", c_int64)]
+                + [(n, c_void_p) for n in ("state_slots", "cu_seqlens", "starts", "log_decay", "beta")]
+                + [(n, c_int64) for n in ("log_decay_stride", "beta_stride", "batch", "heads", "groups", "d", "vd")]
+                + [("conv_weight", c_void_p), ("conv_ring", c_void_p)] + [(n, c_int64) for n in ("taps", "channels", "q_channel", "k_channel", "v_channel")]
+                + [("q_scale", c_float), ("unit_eps", c_float), ("dtype", c_int)])
+
+
+class AddNorm(Structure):
+    """mops_hip_add_norm_args of the header, field by field."""
+    _fields_ = ([("residual", c_void_p), ("y", c_void_p), ("y_stride", c_int64)] + [(n, c_void_p) for n in ("shift", "w", "b", "out")]
+                + [(n, c_int64) for n in ("out_stride", "rows", "n")] + [("eps", c_float)] + [(n, c_int) for n in ("replace", "center", "dtype")])
 
 
 class LatentRows(Structure):
@@ -48,14 +66,16 @@ class BiasedAttention(Structure):
                 + [(n, c_int64) for n in ("block_table_stride", "block_size", "num_blocks", "max_blocks")]
                 + [("out", c_void_p)] + [(n, c_int64) for n in ("rows", "heads", "kv_heads", "dim", "vdim")]
                 + [("scale", c_float), ("dtype", c_int), ("softcap", c_float)] + [(n, c_int64) for n in ("window", "chunk", "keep_first")]
-                + [("sinks", c_void_p), ("gate", c_void_p), ("gate_stride", c_int64)])
+                + [("sinks", c_void_p), ("gate", c_void_p), ("gate_stride", c_int64)]
+                + [(n, c_void_p) for n in ("log_rate", "log_step", "weight_bias")] + [("gate_each", c_int64), ("out_stride", c_int64), ("out_scale", c_float)])
 
 
 class RotaryPrepare(Structure):
     """mops_hip_rotary_prepare_args of the header, field by field."""
     _fields_ = ([("qkv", c_void_p), ("qkv_stride", c_int64)] + [(n, c_void_p) for n in ("q_weight", "k_weight", "cos_sin")]
                 + [("max_positions", c_int64), ("rot", c_int64)] + [(n, c_void_p) for n in ("positions", "slot_mapping", "q", "k_pages", "v_pages")]
-                + [(n, c_int64) for n in ("num_slots", "tokens", "heads", "kv_heads", "dim", "vdim")] + [("eps", c_float), ("dtype", c_int)])
+                + [(n, c_int64) for n in ("num_slots", "tokens", "heads", "kv_heads", "dim", "vdim")] + [("eps", c_float), ("dtype", c_int)]
+                + [("bias", c_void_p), ("neighbours", c_int64)])
 
 
 class EmbedPairs(Structure):
@@ -114,7 +134,8 @@ SIGNATURES = {
                                             c_int64, c_int64, c_float, c_void_p]),
     "mops_hip_linear_bf16": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int64, c_int64,
                                      c_int64, c_void_p, c_int64, c_void_p]),
-    "mops_hip_embed_residual": (c_int, [c_void_p, c_void_p, c_int64, c_int, c_float, c_void_p, c_void_p, c_int64, c_int64, c_int64, c_void_p]),
+    "mops_hip_embed_residual": (c_int, [c_void_p, c_void_p, c_int64, c_int, c_float, c_void_p, c_void_p, c_int64, c_int64, c_int64, c_int64, c_void_p]),
+    "mops_hip_add_norm": (c_int, [POINTER(AddNorm), c_void_p]),
     "mops_hip_norm_residual_add": (c_int, [c_void_p, c_void_p, c_int64, c_void_p, c_float, c_float, c_void_p, c_int, c_int64, c_int64,
                                            c_void_p]),
     "mops_hip_add_norm_norm": (c_int, [c_void_p, c_void_p, c_int64, c_int64, c_void_p, c_void_p, c_void_p, c_float, c_int, c_void_p, c_int, c_int64,
@@ -122,10 +143,13 @@ SIGNATURES = {
     "mops_hip_layer_norm_f32": (c_int, [c_void_p, c_void_p, c_float, c_void_p, c_int, c_int64, c_int64, c_void_p]),
     "mops_hip_embed_pairs": (c_int, [POINTER(EmbedPairs), c_void_p]),
     "mops_hip_rms_norm_f32": (c_int, [c_void_p, c_void_p, c_float, c_float, c_void_p, c_int, c_int64, c_int64, c_void_p]),
-    "mops_hip_gated_group_norm": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_float, c_int, c_void_p, c_int, c_int64,
-                                          c_int64, c_int64, c_void_p]),
-    "mops_hip_clamped_glu": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int, c_int64, c_int64, c_float, c_float, c_void_p]),
-    "mops_hip_gelu_glu": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int, c_int64, c_int64, c_void_p]),
+    "mops_hip_gated_group_norm": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int, c_float, c_int, c_int, c_float, c_void_p, c_int64,
+                                          c_int, c_int64, c_int64, c_int64, c_void_p]),
+    "mops_hip_clamped_glu": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_int, c_int64, c_int64, c_float, c_float, c_void_p]),
+    "mops_hip_gelu_glu": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_int, c_int64, c_int64, c_void_p]),
+    "mops_hip_relu_glu": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_int, c_int64, c_int64, c_void_p]),
+    "mops_hip_matrix_memory_copies": (c_int64, [c_int64]),
+    "mops_hip_delta_rule": (c_int, [POINTER(Delta), c_void_p]),
     "mops_hip_recurrence_state_pitch": (c_int64, [c_int64]),
     "mops_hip_decayed_recurrence": (c_int, [POINTER(Recurrence), c_void_p]),
     "mops_hip_decayed_chunks_workgroups": (c_int64, [c_int64] * 3),
@@ -150,7 +174,7 @@ SIGNATURES = {
     "mops_hip_rotate_pairs": (c_int, [c_void_p, c_int64, c_int64, c_void_p, c_void_p, c_int64, c_int64, c_int64, c_int64, c_void_p]),
     "mops_hip_token_mix": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                                    c_int, c_int64, c_int64, c_void_p]),
-    "mops_hip_low_rank_decay": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int, c_int64, c_int64, c_int64, c_void_p]),
+    "mops_hip_low_rank_decay": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_void_p, c_int, c_int64, c_int64, c_int64, c_void_p]),
     "mops_hip_squared_relu": (c_int, [c_void_p, c_int64, c_void_p, c_int, c_int64, c_int64, c_void_p]),
     "mops_hip_attention_prepare": (c_int, [POINTER(AttentionPrepare), c_void_p]),
     "mops_hip_rotary_prepare": (c_int, [POINTER(RotaryPrepare), c_void_p]),
@@ -168,7 +192,7 @@ SIGNATURES = {
     "mops_hip_linear_tune": (c_int, [c_int64, c_int64, c_int64, c_int64, c_int, c_void_p, c_int64, c_void_p, c_void_p, c_void_p]),
 }
 
-ABI_VERSION = 12
+ABI_VERSION = 13
 
 _lib = None
 

@@ -1,7 +1,8 @@
 // Causal attention over paged keys and values with a linear distance bias per head:
 //   score(i, j) = (q_i . k_j) * scale - slope_h (i - j),  j <= i,  softmax over j,  query head h reads key/value head h / (H / G).
-// Instead of the bias a cap on the scores, and as options: a window or chunks with kept first tokens (visible.h), a sink in the
-// softmax's denominator, a gate on the output.
+// Instead of the bias a cap on the scores, or a bias rate_h ln(1 + step_h (i - j)), or no softmax at all: every key counts with
+// sigmoid(score + bias_h).  Options: a window or chunks with kept first tokens (visible.h), a sink in the softmax's denominator, a gate
+// per head or per element on the output, a constant factor.
 // Key and value sizes are independent of each other; pages hold [block][offset][G][size rounded up to 8], zeros behind the size.
 //
 //   attention_prepare       from the packed projections [q | k | v] of every token: RMS norm with plain weights over the whole of
@@ -71,7 +72,7 @@ __global__ __launch_bounds__(256) void biased_attention_rows_kernel(const mops_h
   const int tid = threadIdx.x, ln = tid & 15, r16 = tid >> 4;
   const int dim = (int)a.dim, vdim = (int)a.vdim, groups = (int)a.kv_heads, g = h / (int)(a.heads / a.kv_heads);
   const int dp = (dim + 7) / 8 * 8, vp = (vdim + 7) / 8 * 8;
-  T* out = (T*)a.out + (row * a.heads + h) * vdim;
+  T* out = (T*)a.out + row * a.out_stride + (int64_t)h * vdim;
   const int len = a.context_lens[row];
   if (len <= 0) {
     for (int i = tid; i < vdim; i += 256) out[i] = from_f32<T>(0.f);
@@ -79,7 +80,8 @@ __global__ __launch_bounds__(256) void biased_attention_rows_kernel(const mops_h
   }
   const T* q = (const T*)a.q + (row * a.heads + h) * dp;
   for (int i = tid; i < dim; i += 256) sq[i] = to_f32(q[i]);
-  const float slope = a.slopes ? a.slopes[h] : 0.f;
+  const float slope = a.slopes ? a.slopes[h] : 0.f, rate = a.log_rate ? a.log_rate[h] : 0.f, step = a.log_rate ? a.log_step[h] : 0.f;
+  const float bias = a.weight_bias ? a.weight_bias[h] : 0.f;
   const Visible see = visible_at(a, len);
   const int seq = a.row_seq ? a.row_seq[row] : (int)row;
   const int32_t* table = a.block_table + (int64_t)seq * a.block_table_stride;
@@ -108,7 +110,8 @@ __global__ __launch_bounds__(256) void biased_attention_rows_kernel(const mops_h
       if (ln == 0) {
         dot *= a.scale;
         if (a.softcap > 0.f) dot = a.softcap * tanhf(dot / a.softcap);
-        sp[kk] = r >= 0 ? dot - slope * (float)(len - 1 - j) : -INFINITY;
+        if (a.log_rate) dot -= rate * log1pf(step * (float)(len - 1 - j));
+        sp[kk] = r >= 0 ? dot - slope * (float)(len - 1 - j) + bias : -INFINITY;
       }
     }
     __syncthreads();
@@ -118,8 +121,8 @@ __global__ __launch_bounds__(256) void biased_attention_rows_kernel(const mops_h
     mx = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
     const float m_new = fmaxf(m, mx);
     const float safe = m_new == -INFINITY ? 0.f : m_new;
-    const float alpha = expf(m - safe);
-    const float p = expf(sp[tid] - safe);
+    const float alpha = a.weight_bias ? 1.f : expf(m - safe);
+    const float p = a.weight_bias ? 1.0f / (1.0f + expf(-sp[tid])) : expf(sp[tid] - safe);
     __syncthreads();
     sp[tid] = p;
     const float ps = group_sum<kWave>(p);
@@ -140,11 +143,11 @@ __global__ __launch_bounds__(256) void biased_attention_rows_kernel(const mops_h
         if (tid + 256 * i < vdim) acc[i] += w * to_f32(vr[tid + 256 * i]);
     }
   }
-  float inv = l > 0.f ? 1.0f / l : 0.f;
-  if (a.gate) inv *= sigmoid_for<T>(to_f32(((const T*)a.gate)[row * a.gate_stride + h]));
+  const float inv = a.weight_bias ? 1.0f : (l > 0.f ? 1.0f / l : 0.f);
+  const OutputGate<T> gate(a, row, h);
 #pragma unroll
   for (int i = 0; i < kRowMaxValue / 256; ++i)
-    if (tid + 256 * i < vdim) out[tid + 256 * i] = from_f32<T>(acc[i] * inv);
+    if (tid + 256 * i < vdim) out[tid + 256 * i] = from_f32<T>(acc[i] * inv * gate(tid + 256 * i));
 }
 
 // 1: go on; otherwise the status to return.
@@ -155,7 +158,9 @@ int check_biased_attention(const mops_hip_biased_attention* a) {
   if (a->heads <= 0 || a->kv_heads <= 0 || a->heads % a->kv_heads || a->dim <= 0 || a->vdim <= 0) return MOPS_HIP_EINVAL;
   if (a->block_size <= 0 || a->num_blocks <= 0 || a->max_blocks <= 0 || a->block_table_stride < a->max_blocks) return MOPS_HIP_EINVAL;
   if (a->window < 0 || a->chunk < 0 || a->keep_first < 0 || (a->window && a->chunk)) return MOPS_HIP_EINVAL;
-  if (!(a->softcap >= 0.f) || (a->softcap > 0.f && a->slopes) || (a->gate && a->gate_stride < a->heads)) return MOPS_HIP_EINVAL;
+  if (!(a->softcap >= 0.f) || (a->gate && a->gate_stride < (a->gate_each ? a->heads * a->vdim : a->heads))) return MOPS_HIP_EINVAL;
+  if ((a->softcap > 0.f) + (a->slopes != nullptr) + (a->log_rate != nullptr) + (a->weight_bias != nullptr) > 1) return MOPS_HIP_EINVAL;
+  if ((a->log_rate == nullptr) != (a->log_step == nullptr) || (a->weight_bias && a->sinks) || (a->out_stride && a->out_stride < a->heads * a->vdim)) return MOPS_HIP_EINVAL;
   if (a->window > kMaxRange || a->chunk > kMaxRange || a->keep_first > kMaxRange) return MOPS_HIP_EUNSUPPORTED;
   if (a->rows * a->heads > 0x7fffffffLL || a->block_size > (1 << 20) || a->max_blocks * a->block_size > (1 << 28)) return MOPS_HIP_EUNSUPPORTED;
   return 1;
@@ -192,7 +197,7 @@ extern "C" int mops_hip_biased_attention_rows(const mops_hip_biased_attention* a
   if (pre != 1) return pre;
   if (a->dim > kRowMaxDim || a->vdim > kRowMaxValue) return MOPS_HIP_EUNSUPPORTED;
   const dim3 grid((unsigned)(a->rows * a->heads));
-  if (a->dtype == MOPS_HIP_BF16) hipLaunchKernelGGL((biased_attention_rows_kernel<bf16_t>), grid, dim3(256), 0, (hipStream_t)stream, *a);
-  else hipLaunchKernelGGL((biased_attention_rows_kernel<float>), grid, dim3(256), 0, (hipStream_t)stream, *a);
+  if (a->dtype == MOPS_HIP_BF16) hipLaunchKernelGGL((biased_attention_rows_kernel<bf16_t>), grid, dim3(256), 0, (hipStream_t)stream, completed(*a));
+  else hipLaunchKernelGGL((biased_attention_rows_kernel<float>), grid, dim3(256), 0, (hipStream_t)stream, completed(*a));
   return finish_launch();
 }

@@ -10,6 +10,7 @@
 //   O^T [v, head]    += V^T P^T      V^T through transposing LDS reads, P as the sum of two bf16 numbers
 // A row that lies inside one run is written at once.  A row that is cut leaves (max, sum, unnormalised O) in one of the two slots
 // of each run it touches; biased_combine_kernel merges them and writes the rows without any context as zeros.
+// Weights that are sigmoids need no maximum and no sum; the parts of a cut row simply add up.
 // Where rows see a part of their sequence only, their stages are those with something to see.  A sink enters with a row's first
 // stage, as a token with a value of zeros.
 #include "mfma_tiles.h"
@@ -127,9 +128,7 @@ __global__ __launch_bounds__(64, NK * 32 + NV * 16 <= 256 ? 2 : 1) void biased_d
     for (int j = 0; j < kLoadsV; ++j) vreg[j] = load16_stream(vs + v_off[j]);
     return ok;
   };
-  const float scale = a.scale * 1.4426950408889634f;
-  const float slope = KIND == kSloped && a.slopes ? a.slopes[h] * 1.4426950408889634f : 0.f;
-  const CappedScore capped(a);
+  const ScoreOf<KIND> score(a, h);
   const float sink = a.sinks ? a.sinks[h] * 1.4426950408889634f : -INFINITY;
 
   for (; remaining > 0; ++row, stage0 = 0) {
@@ -152,7 +151,7 @@ __global__ __launch_bounds__(64, NK * 32 + NV * 16 <= 256 ? 2 : 1) void biased_d
     f32x4 acc[NV];
 #pragma unroll
     for (int i = 0; i < NV; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-    float m_run = KIND == kCappedFixed ? 0.f : (stage0 == 0 ? sink : -INFINITY);
+    float m_run = !needs_reference(KIND) ? 0.f : (stage0 == 0 ? sink : -INFINITY);
     float l_run = stage0 == 0 && jj == 0 && a.sinks ? __builtin_amdgcn_exp2f(sink - m_run) : 0.f;
 
     for (int st = stage0; st < stage0 + run; ++st) {
@@ -183,7 +182,7 @@ __global__ __launch_bounds__(64, NK * 32 + NV * 16 <= 256 ? 2 : 1) void biased_d
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
         const int t = 4 * jj + (e & 3) + 16 * (e >> 2);
-        const float x = KIND == kSloped ? s[e >> 2][e & 3] * scale + slope * (dist + (float)((e & 3) + 16 * (e >> 2))) : capped(s[e >> 2][e & 3]);
+        const float x = score(s[e >> 2][e & 3], dist + (float)((e & 3) + 16 * (e >> 2)));
         sv[e] = t < valid ? x : -INFINITY;
       }
       if (tok0 < see.lo && tok0 + kStage > see.kept) {      // the edge of what the row sees
@@ -194,7 +193,7 @@ __global__ __launch_bounds__(64, NK * 32 + NV * 16 <= 256 ? 2 : 1) void biased_d
         }
       }
       float m_safe = 0.f, alpha = 1.f;
-      if (KIND != kCappedFixed) {
+      if (needs_reference(KIND)) {
 #pragma unroll
         for (int e = 0; e < 8; ++e) m_loc = fmaxf(m_loc, sv[e]);
         m_loc = fmaxf(m_loc, __shfl_xor(m_loc, 16, kWave));
@@ -207,11 +206,11 @@ __global__ __launch_bounds__(64, NK * 32 + NV * 16 <= 256 ? 2 : 1) void biased_d
       float pv[8], psum = 0.f;
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
-        pv[e] = __builtin_amdgcn_exp2f(sv[e] - m_safe);
+        pv[e] = score.weight(sv[e], m_safe);
         psum += pv[e];
       }
       l_run = l_run * alpha + psum;
-      if (KIND != kCappedFixed && __any(alpha != 1.0f)) {
+      if (needs_reference(KIND) && __any(alpha != 1.0f)) {
 #pragma unroll
         for (int i = 0; i < NV; ++i) acc[i] *= alpha;
       }
@@ -231,15 +230,15 @@ __global__ __launch_bounds__(64, NK * 32 + NV * 16 <= 256 ? 2 : 1) void biased_d
     l_tot += __shfl_xor(l_tot, 32, kWave);
     if (!head_ok) continue;
     if (run == row_stages) {
-      float inv = l_tot > 0.f ? 1.0f / l_tot : 0.f;
-      if (a.gate) inv *= sigmoid_for<bf16_t>(to_f32(((const bf16_t*)a.gate)[row * a.gate_stride + h]));
-      uint16_t* orow = (uint16_t*)a.out + ((int64_t)row * heads + h) * vdim;
+      const float inv = KIND == kSigmoid ? 1.0f : (l_tot > 0.f ? 1.0f / l_tot : 0.f);
+      const OutputGate<bf16_t> gate(a, row, h);
+      uint16_t* orow = (uint16_t*)a.out + (int64_t)row * a.out_stride + (int64_t)h * vdim;
 #pragma unroll
       for (int i = 0; i < NV; ++i) {
         const int v = 16 * i + 4 * jj;
 #pragma unroll
         for (int e = 0; e < 4; ++e)
-          if (v + e < vdim) orow[v + e] = (uint16_t)f32_to_bf16_bits(acc[i][e] * inv);
+          if (v + e < vdim) orow[v + e] = (uint16_t)f32_to_bf16_bits(acc[i][e] * inv * gate(v + e));
       }
       continue;
     }
@@ -265,7 +264,7 @@ __global__ __launch_bounds__(64) void biased_combine_kernel(const BiasedDecodeAr
   const int heads = (int)a.heads, vdim = (int)a.vdim, per_group = heads / (int)a.kv_heads;
   const int h = blockIdx.x % heads, row = blockIdx.x / heads, lane = threadIdx.x;
   const int per = p.plan[0], f0 = p.plan[1 + row], f1 = p.plan[2 + row];
-  uint16_t* out = (uint16_t*)a.out + ((int64_t)row * heads + h) * vdim;
+  uint16_t* out = (uint16_t*)a.out + (int64_t)row * a.out_stride + (int64_t)h * vdim;
   if (f1 <= f0) {
     for (int v = lane; v < vdim; v += kWave) out[v] = 0;
     return;
@@ -282,8 +281,8 @@ __global__ __launch_bounds__(64) void biased_combine_kernel(const BiasedDecodeAr
   float l = 0.f;
   for (int j = j0 + lane; j <= j1; j += kWave) l += __builtin_amdgcn_exp2f(p.ml[2 * slot_of(j)] - safe) * p.ml[2 * slot_of(j) + 1];
   l = group_sum<kWave>(l);
-  float inv = l > 0.f ? 1.0f / l : 0.f;
-  if (a.gate) inv *= sigmoid_for<bf16_t>(to_f32(((const bf16_t*)a.gate)[row * a.gate_stride + h]));
+  const float inv = a.weight_bias ? 1.0f : (l > 0.f ? 1.0f / l : 0.f);
+  const OutputGate<bf16_t> gate(a, row, h);
   for (int v0 = 0; v0 < vdim; v0 += 4 * kWave) {
     float o[4] = {0.f, 0.f, 0.f, 0.f};
     for (int j = j0; j <= j1; ++j) {
@@ -298,7 +297,7 @@ __global__ __launch_bounds__(64) void biased_combine_kernel(const BiasedDecodeAr
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       const int v = v0 + e * kWave + lane;
-      if (v < vdim) out[v] = (uint16_t)f32_to_bf16_bits(o[e] * inv);
+      if (v < vdim) out[v] = (uint16_t)f32_to_bf16_bits(o[e] * inv * gate(v));
     }
   }
 }
@@ -349,7 +348,7 @@ extern "C" int mops_hip_biased_decode(const mops_hip_biased_attention* a, void* 
   const int64_t tokens = a->max_blocks * a->block_size;
   if (a->rows * ((tokens + kStage - 1) / kStage) > 0x7fffffffLL || a->kv_heads * 256 * kStage > 0x7fffffffLL) return MOPS_HIP_EUNSUPPORTED;
   BiasedDecodeArgs p;
-  p.a = *a;
+  p.a = completed(*a);
   p.head_tiles = (int)head_tiles_of(a->heads, a->kv_heads);
   const int64_t planes = a->kv_heads * p.head_tiles;
   p.columns = decode_columns(a->dim, a->vdim, planes);
@@ -364,6 +363,8 @@ extern "C" int mops_hip_biased_decode(const mops_hip_biased_attention* a, void* 
   const ScoreKind kind = score_kind(*a);
   if (kind == kCappedFixed) launch_decode<kCappedFixed>(p, grid, s);
   else if (kind == kCapped) launch_decode<kCapped>(p, grid, s);
+  else if (kind == kLogSloped) launch_decode<kLogSloped>(p, grid, s);
+  else if (kind == kSigmoid) launch_decode<kSigmoid>(p, grid, s);
   else launch_decode<kSloped>(p, grid, s);
   hipLaunchKernelGGL(biased_combine_kernel, dim3((unsigned)(a->rows * a->heads)), dim3(64), 0, s, p);
   return finish_launch();

@@ -53,7 +53,7 @@ __global__ __launch_bounds__(256, NK <= 8 && NV <= 4 ? 2 : 1) void biased_prefil
 #pragma unroll
     for (int r = 0; r < 16; ++r) o[i][r] = 0.f;
   const float sink = a.sinks ? a.sinks[h] * 1.4426950408889634f : -INFINITY;      // a token with a value of zeros
-  float m_run = KIND == kCappedFixed ? 0.f : sink, l_run = a.sinks && hh == 0 ? __builtin_amdgcn_exp2f(sink - m_run) : 0.f;
+  float m_run = !needs_reference(KIND) ? 0.f : sink, l_run = a.sinks && hh == 0 ? __builtin_amdgcn_exp2f(sink - m_run) : 0.f;
 
   const int visible = pos0 + q_count < keys ? pos0 + q_count : keys;      // keys any query of the tile sees
   const int keep = (int)a.keep_first, pos_first = pos0 + 32 * wave;      // of the wave's queries
@@ -93,9 +93,7 @@ __global__ __launch_bounds__(256, NK <= 8 && NV <= 4 ? 2 : 1) void biased_prefil
       if (row < 0) vreg[j] = u32x4{0u, 0u, 0u, 0u};      // zero weights times what a page holds must be zero
     }
   };
-  const float scale = a.scale * 1.4426950408889634f;
-  const float slope = KIND == kSloped && a.slopes ? a.slopes[h] * 1.4426950408889634f : 0.f;
-  const CappedScore capped(a);
+  const ScoreOf<KIND> score(a, h);
   issue(page_of());
   int64_t next_row = page_of();
   for (int block = 0; block < n_blocks; ++block) {
@@ -131,7 +129,7 @@ __global__ __launch_bounds__(256, NK <= 8 && NV <= 4 ? 2 : 1) void biased_prefil
         for (int r = 0; r < 16; ++r) {
           const int off = 32 * kt + 8 * (r >> 2) + (r & 3);
           const int j = k0 + 4 * hh + off;
-          const float x = KIND == kSloped ? s[kt][r] * scale + slope * (dist + (float)off) : capped(s[kt][r]);
+          const float x = score(s[kt][r], dist + (float)off);
           s[kt][r] = j <= last && (j >= lo || j < keep) ? x : -INFINITY;
           m_loc = fmaxf(m_loc, s[kt][r]);
         }
@@ -141,12 +139,12 @@ __global__ __launch_bounds__(256, NK <= 8 && NV <= 4 ? 2 : 1) void biased_prefil
 #pragma unroll
         for (int r = 0; r < 16; ++r) {
           const int off = 32 * kt + 8 * (r >> 2) + (r & 3);
-          s[kt][r] = KIND == kSloped ? s[kt][r] * scale + slope * (dist + (float)off) : capped(s[kt][r]);
+          s[kt][r] = score(s[kt][r], dist + (float)off);
           m_loc = fmaxf(m_loc, s[kt][r]);
         }
     }
     float m_safe = 0.f;
-    if (KIND != kCappedFixed) {
+    if (needs_reference(KIND)) {
       m_loc = fmaxf(m_loc, __shfl_xor(m_loc, 32, kWave));
       const float m_new = fmaxf(m_run, m_loc);
       m_safe = m_new == -INFINITY ? 0.f : m_new;
@@ -165,7 +163,7 @@ __global__ __launch_bounds__(256, NK <= 8 && NV <= 4 ? 2 : 1) void biased_prefil
         float pv[8];
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
-          pv[e] = __builtin_amdgcn_exp2f(s[kt][8 * ks + e] - m_safe);
+          pv[e] = score.weight(s[kt][8 * ks + e], m_safe);
           l_run += pv[e];
         }
         bf16x8 hi, lo;
@@ -182,21 +180,28 @@ __global__ __launch_bounds__(256, NK <= 8 && NV <= 4 ? 2 : 1) void biased_prefil
   }
   if (!q_ok) return;
   const float l = l_run + __shfl_xor(l_run, 32, kWave);
-  float inv = l > 0.f ? 1.0f / l : 0.f;
-  if (a.gate) inv *= sigmoid_for<bf16_t>(to_f32(((const bf16_t*)a.gate)[(q_begin + qi) * a.gate_stride + h]));
-  uint16_t* orow = (uint16_t*)a.out + ((int64_t)(q_begin + qi) * heads + h) * vdim;
+  const OutputGate<bf16_t> gate(a, q_begin + qi, h);
+  const float inv = (KIND == kSigmoid ? 1.0f : (l > 0.f ? 1.0f / l : 0.f)) * (gate.each ? 1.0f : gate.constant);
+  uint16_t* orow = (uint16_t*)a.out + (int64_t)(q_begin + qi) * a.out_stride + (int64_t)h * vdim;
 #pragma unroll
   for (int i = 0; i < NV; ++i)
 #pragma unroll
     for (int q4 = 0; q4 < 4; ++q4) {
       const int v = 32 * i + 8 * q4 + 4 * hh;
+      float y[4];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) y[e] = o[i][4 * q4 + e] * inv;
       if (p.vec_out && v + 4 <= vdim) {
-        *reinterpret_cast<u32x2*>(orow + v) = u32x2{pack_bf16x2(o[i][4 * q4] * inv, o[i][4 * q4 + 1] * inv),
-                                                    pack_bf16x2(o[i][4 * q4 + 2] * inv, o[i][4 * q4 + 3] * inv)};
+        if (gate.each) {
+          const u32x2 g = *reinterpret_cast<const u32x2*>(gate.g + v);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) y[e] *= gate.constant * sigmoid_for<bf16_t>(e & 1 ? bf16hi_to_f32(g[e >> 1]) : bf16lo_to_f32(g[e >> 1]));
+        }
+        *reinterpret_cast<u32x2*>(orow + v) = u32x2{pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3])};
       } else {
 #pragma unroll
         for (int e = 0; e < 4; ++e)
-          if (v + e < vdim) orow[v + e] = (uint16_t)f32_to_bf16_bits(o[i][4 * q4 + e] * inv);
+          if (v + e < vdim) orow[v + e] = (uint16_t)f32_to_bf16_bits(gate.each ? y[e] * gate(v + e) : y[e]);
       }
     }
 }
@@ -225,14 +230,17 @@ extern "C" int mops_hip_biased_prefill(const mops_hip_biased_attention* args, co
   if (args->dtype != MOPS_HIP_BF16 || args->dim > 256 || args->vdim > 256 || num_tiles * args->heads > 0x7fffffffLL) return MOPS_HIP_EUNSUPPORTED;
   if (!aligned16(args->q) || !aligned16(args->k_pages) || !aligned16(args->v_pages)) return MOPS_HIP_EALIGN;
   BiasedPrefillArgs p;
-  p.a = *args;
+  p.a = completed(*args);
   p.tiles = tiles;
-  p.vec_out = args->vdim % 4 == 0 && aligned16(args->out);
+  p.vec_out = args->vdim % 4 == 0 && p.a.out_stride % 4 == 0 && aligned16(args->out) &&
+              (!args->gate || !args->gate_each || (args->gate_stride % 4 == 0 && aligned16(args->gate)));
   const dim3 grid((unsigned)(num_tiles * args->heads));
   hipStream_t s = (hipStream_t)stream;
   const ScoreKind kind = score_kind(*args);
   if (kind == kCappedFixed) launch_prefill<kCappedFixed>(p, grid, s);
   else if (kind == kCapped) launch_prefill<kCapped>(p, grid, s);
+  else if (kind == kLogSloped) launch_prefill<kLogSloped>(p, grid, s);
+  else if (kind == kSigmoid) launch_prefill<kSigmoid>(p, grid, s);
   else launch_prefill<kSloped>(p, grid, s);
   return finish_launch();
 }

@@ -9,6 +9,10 @@
 //   per channel   S_t = diag(exp(channel_decay_t)) S_(t-1) + k_t v_t^T, channel_decay a float logarithm per token, head and key
 //                 channel; the output looks at the state in front of the token and weighs the token itself by a bonus u per
 //                 channel: o_t = (S_(t-1) + diag(u) k_t v_t^T)^T q_t
+//   matrix memory a = exp(f + m_(t-1) - m_t), s = exp(i - m_t) with gates i = cap tanh((x + bias) / cap) and f = log sigmoid(cap tanh((y +
+//                 bias) / cap)) per token and head, relative to a running maximum m_t = max(f + m_(t-1), i) that starts at 0; the same
+//                 recurrence with values of one gives n, and o_t = S_t^T q_t / (max(|n_t . q_t|, exp(-m_t)) + 1e-6).  n follows the value
+//                 rows of a head's state, once per 64 of them, and so does m in `top`: every workgroup has a copy of its own.
 // q and k may be rotated on their first rot dimensions (dimension i with i + rot/2) by the row of a cos/sin table, and k is
 // multiplied by k_scale after that.  Query/key heads may be shared by heads / groups consecutive value heads.
 //
@@ -24,7 +28,7 @@
 // reads the taps-1 rows before its own position and writes its own row, which is none of those, so the step needs no
 // second buffer and no shifting.  Positions before the start of the sequence count as zeros whatever the ring holds.
 // short_conv_update writes the last taps-1 inputs of each portion into the ring, in a launch of its own behind the readers.
-#include "mixed_types.h"
+#include "matrix_memory.h"
 
 namespace mops {
 
@@ -43,6 +47,12 @@ struct RecurrenceArgs {
   const float *dt_bias, *neg_a, *skip;
   const float *channel_decay, *bonus;
   int64_t channel_decay_stride;
+  const void *input_gate, *forget_gate;
+  int64_t gate_stride;
+  const float *input_bias, *forget_bias;
+  float gate_cap;
+  float* top;
+  int copies;                   // of n and m: 0 without a matrix memory
   const float* cos_sin;
   int rot;
   int64_t max_positions;
@@ -54,9 +64,12 @@ struct RecurrenceArgs {
   int q_channel, k_channel, v_channel;
 };
 
+enum RecurrenceKind { kPlain, kConvolved, kPerChannel, kMemory };
+
 // cu_seqlens == nullptr: sequence b is the single token b.
-template <typename T, int DPT, int RPT, bool CONV, bool CHANNEL>
+template <typename T, int DPT, int RPT, RecurrenceKind KIND>
 __global__ __launch_bounds__(256) void decayed_recurrence_kernel(const RecurrenceArgs a) {
+  constexpr bool CONV = KIND == kConvolved, CHANNEL = KIND == kPerChannel, MEMORY = KIND == kMemory;
   constexpr int kRows = 16 * RPT;
   constexpr int kDim = 16 * DPT;
   __shared__ __align__(16) float sq[kDim], sk[kDim], sv[kRows], sa[CHANNEL ? kDim : 1], su[CHANNEL ? kDim : 1];
@@ -77,7 +90,10 @@ __global__ __launch_bounds__(256) void decayed_recurrence_kernel(const Recurrenc
       if (tid < kRows && row0 + tid < a.vd) out[t * a.out_stride + tid] = from_f32<T>(0.f);
     return;
   }
-  float* state = a.state + (((int64_t)slot * a.heads + h) * a.vd + row0) * a.pitch;
+  float* const head_state = a.state + ((int64_t)slot * a.heads + h) * (a.vd + (MEMORY ? a.copies : 0)) * a.pitch;
+  float* const state = head_state + (int64_t)row0 * a.pitch;
+  float* const n_row = head_state + (int64_t)(a.vd + tile) * a.pitch;            // MEMORY
+  float* const top = MEMORY ? a.top + ((int64_t)slot * a.heads + h) * a.copies + tile : nullptr;
   float s[RPT][DPT];
   constexpr int kPiece = DPT >= 4 ? 4 : DPT;
   auto piece_at = [&](int p) { return p * 64 + ln * kPiece; };
@@ -100,6 +116,17 @@ __global__ __launch_bounds__(256) void decayed_recurrence_kernel(const Recurrenc
         for (int e = 0; e < kPiece; ++e) s[r][p * kPiece + e] = v[e];
       }
     }
+  }
+  float nn[MEMORY ? DPT : 1], m = 0.f;
+  if (MEMORY) {
+    if (start > 0) m = *top;
+#pragma unroll
+    for (int p = 0; p < DPT / kPiece; ++p)
+#pragma unroll
+      for (int e = 0; e < kPiece; ++e) {
+        const int i = piece_at(p) + e;
+        nn[MEMORY ? p * kPiece + e : 0] = start > 0 && i < a.pitch ? n_row[i] : 0.f;
+      }
   }
   const int per_group = a.heads / a.groups;
   const int g = h / per_group;
@@ -159,6 +186,16 @@ __global__ __launch_bounds__(256) void decayed_recurrence_kernel(const Recurrenc
       scale = softplus_f32(to_f32(((const T*)a.dt)[t * a.dt_stride + h]) + bias);
       decay = expf(neg_a * scale);
     }
+    float least = 0.f;
+    if (MEMORY) {
+      const float i = capped_gate(to_f32(((const T*)a.input_gate)[t * a.gate_stride + h]) + a.input_bias[h], a.gate_cap);
+      const float f = log_sigmoid(capped_gate(to_f32(((const T*)a.forget_gate)[t * a.gate_stride + h]) + a.forget_bias[h], a.gate_cap));
+      const float m_new = fmaxf(f + m, i);
+      decay = expf(f + m - m_new);
+      scale = expf(i - m_new);
+      least = expf(-m_new);
+      m = m_new;
+    }
     __syncthreads();
     float kk[DPT], qq[DPT], aa[CHANNEL ? DPT : 1];
     float direct = 0.f;      // CHANNEL: this lane's part of sum u k q
@@ -173,6 +210,16 @@ __global__ __launch_bounds__(256) void decayed_recurrence_kernel(const Recurrenc
           direct += su[piece_at(p) + e] * qq[p * kPiece + e];
         }
       }
+    float inv = 1.f;
+    if (MEMORY) {
+      float dot = 0.f;
+#pragma unroll
+      for (int e = 0; e < DPT; ++e) {
+        nn[MEMORY ? e : 0] = decay * nn[MEMORY ? e : 0] + scale * kk[e];
+        dot += nn[MEMORY ? e : 0] * qq[e];
+      }
+      inv = 1.0f / (fmaxf(fabsf(group_sum<16>(dot)), least) + kMemoryEps);
+    }
 #pragma unroll
     for (int r = 0; r < RPT; ++r) {
       const int row = r16 + 16 * r;
@@ -190,7 +237,7 @@ __global__ __launch_bounds__(256) void decayed_recurrence_kernel(const Recurrenc
       }
       if (CHANNEL) dot += direct * x;
       dot = group_sum<16>(dot);
-      if (ln == 0 && row0 + row < a.vd) out[t * a.out_stride + row] = from_f32<T>(dot + skip * x);
+      if (ln == 0 && row0 + row < a.vd) out[t * a.out_stride + row] = from_f32<T>(MEMORY ? dot * inv : dot + skip * x);
     }
     __syncthreads();
   }
@@ -212,6 +259,16 @@ __global__ __launch_bounds__(256) void decayed_recurrence_kernel(const Recurrenc
       }
     }
   }
+  if (MEMORY) {
+    if (r16 == 0) {
+#pragma unroll
+      for (int p = 0; p < DPT / kPiece; ++p)
+#pragma unroll
+        for (int e = 0; e < kPiece; ++e)
+          if (piece_at(p) + e < a.pitch) n_row[piece_at(p) + e] = nn[MEMORY ? p * kPiece + e : 0];
+    }
+    if (tid == 0) *top = m;      // behind the barriers above: everyone has read it
+  }
 }
 
 template <typename T, int VEC>
@@ -231,7 +288,9 @@ __global__ __launch_bounds__(256) void short_conv_kernel(const T* __restrict__ x
   const int in_portion = (int)t - cu_seqlens[b];
   const int pos = starts[b] + in_portion;
   float acc[VEC], v[VEC], wv[VEC];
-  load_vec<VEC>(bias + c, acc);
+#pragma unroll
+  for (int e = 0; e < VEC; ++e) acc[e] = 0.f;
+  if (bias) load_vec<VEC>(bias + c, acc);
   for (int lag = 0; lag < taps; ++lag) {
     if (pos - lag < 0) break;
     if (lag <= in_portion) load_vec<VEC>(x + (t - lag) * x_stride + c, v);
@@ -265,7 +324,9 @@ __global__ __launch_bounds__(256) void short_conv_run_kernel(const T* __restrict
   float wv[TAPS][8], b[8], win[TAPS][8];       // win[l]: the input l tokens back
 #pragma unroll
   for (int l = 0; l < TAPS; ++l) load_vec<8>(w + (int64_t)(TAPS - 1 - l) * channels + c, wv[l]);
-  load_vec<8>(bias + c, b);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) b[e] = 0.f;
+  if (bias) load_vec<8>(bias + c, b);
   // the window in front of token t: rows of the portion, the ring behind them, zeros before the start
   auto fill = [&](int64_t t, int sq) {
     const int slot = state_slots[sq], in_portion = (int)t - cu_seqlens[sq], pos = starts[sq] + in_portion;
@@ -334,21 +395,23 @@ __global__ __launch_bounds__(256) void short_conv_update_kernel(const T* __restr
     ring[((int64_t)slot * taps + (start + j) % taps) * channels + c] = x[(int64_t)(t0 + j) * x_stride + c];
 }
 
+template <typename T, int DPT, RecurrenceKind KIND>
+static void launch_recurrence_kind(const RecurrenceArgs& a, int64_t batch, hipStream_t s) {
+#define MOPS_REC(R)                                                                                                      \
+  hipLaunchKernelGGL((decayed_recurrence_kernel<T, DPT, R, KIND>), dim3((unsigned)(batch * a.heads * ((a.vd + 16 * (R) - 1) / (16 * (R))))), \
+                     dim3(256), 0, s, a)
+  if (a.vd <= 16) MOPS_REC(1);
+  else if (a.vd <= 32) MOPS_REC(2);
+  else MOPS_REC(4);
+#undef MOPS_REC
+}
+
 template <typename T, int DPT>
 static void launch_recurrence_rows(const RecurrenceArgs& a, int64_t batch, bool conv, hipStream_t s) {
-#define MOPS_REC(R, C) MOPS_REC2(R, C, false)
-#define MOPS_REC2(R, C, CH)                                                                                              \
-  hipLaunchKernelGGL((decayed_recurrence_kernel<T, DPT, R, C, CH>), dim3((unsigned)(batch * a.heads * ((a.vd + 16 * (R) - 1) / (16 * (R))))), \
-                     dim3(256), 0, s, a)
-  if (a.channel_decay) {
-    if (a.vd <= 16) MOPS_REC2(1, false, true);
-    else if (a.vd <= 32) MOPS_REC2(2, false, true);
-    else MOPS_REC2(4, false, true);
-  } else if (a.vd <= 16) { if (conv) MOPS_REC(1, true); else MOPS_REC(1, false); }
-  else if (a.vd <= 32) { if (conv) MOPS_REC(2, true); else MOPS_REC(2, false); }
-  else { if (conv) MOPS_REC(4, true); else MOPS_REC(4, false); }
-#undef MOPS_REC
-#undef MOPS_REC2
+  if (a.channel_decay) launch_recurrence_kind<T, DPT, kPerChannel>(a, batch, s);
+  else if (a.input_gate) launch_recurrence_kind<T, DPT, kMemory>(a, batch, s);
+  else if (conv) launch_recurrence_kind<T, DPT, kConvolved>(a, batch, s);
+  else launch_recurrence_kind<T, DPT, kPlain>(a, batch, s);
 }
 
 template <typename T>
@@ -364,6 +427,8 @@ static int launch_recurrence(const RecurrenceArgs& a, int64_t batch, bool conv, 
 
 }  // namespace mops
 
+extern "C" int64_t mops_hip_matrix_memory_copies(int64_t vd) { return vd <= 0 ? MOPS_HIP_EINVAL : (vd + 63) / 64; }
+
 extern "C" int64_t mops_hip_recurrence_state_pitch(int64_t d) { return d <= 0 ? MOPS_HIP_EINVAL : (d + 3) / 4 * 4; }
 
 extern "C" int mops_hip_decayed_recurrence(const mops_hip_recurrence* r, void* stream) {
@@ -376,7 +441,10 @@ extern "C" int mops_hip_decayed_recurrence(const mops_hip_recurrence* r, void* s
   if (r->q_stride < r->groups * r->d || r->k_stride < r->groups * r->d || r->v_stride < r->heads * r->vd ||
       r->out_stride < r->heads * r->vd)
     return MOPS_HIP_EINVAL;
-  if ((r->decay != nullptr) + (r->dt != nullptr) + (r->channel_decay != nullptr) != 1) return MOPS_HIP_EINVAL;      // one source of the decay
+  if ((r->decay != nullptr) + (r->dt != nullptr) + (r->channel_decay != nullptr) + (r->input_gate != nullptr) != 1) return MOPS_HIP_EINVAL;      // one source of the decay
+  if (r->input_gate && (!r->forget_gate || !r->input_bias || !r->forget_bias || !r->top || !(r->gate_cap > 0.f) || r->gate_stride < r->heads || r->skip ||
+                        r->conv_weight))
+    return MOPS_HIP_EINVAL;
   if (r->channel_decay && (!r->bonus || r->groups != r->heads || r->skip || r->conv_weight || r->channel_decay_stride < r->heads * r->d)) return MOPS_HIP_EINVAL;
   if (r->dt && (!r->dt_bias || !r->neg_a || r->dt_stride < r->heads)) return MOPS_HIP_EINVAL;
   if (r->rot < 0 || (r->rot & 1) || r->rot > r->d || (r->rot && (!r->cos_sin || r->max_positions <= 0))) return MOPS_HIP_EINVAL;
@@ -397,6 +465,9 @@ extern "C" int mops_hip_decayed_recurrence(const mops_hip_recurrence* r, void* s
   a.pitch = (int)mops_hip_recurrence_state_pitch(r->d);
   a.decay = r->decay; a.dt = r->dt; a.dt_stride = r->dt_stride; a.dt_bias = r->dt_bias; a.neg_a = r->neg_a; a.skip = r->skip;
   a.channel_decay = r->channel_decay; a.channel_decay_stride = r->channel_decay_stride; a.bonus = r->bonus;
+  a.input_gate = r->input_gate; a.forget_gate = r->forget_gate; a.gate_stride = r->gate_stride;
+  a.input_bias = r->input_bias; a.forget_bias = r->forget_bias; a.gate_cap = r->gate_cap;
+  a.top = r->top; a.copies = r->input_gate ? (int)mops_hip_matrix_memory_copies(r->vd) : 0;
   a.cos_sin = r->cos_sin; a.rot = (int)r->rot; a.max_positions = r->max_positions; a.k_scale = r->k_scale;
   a.conv_w = r->conv_weight; a.conv_b = r->conv_bias; a.ring = r->conv_ring; a.taps = (int)r->taps; a.channels = r->channels;
   a.q_channel = (int)r->q_channel; a.k_channel = (int)r->k_channel; a.v_channel = (int)r->v_channel;
@@ -411,9 +482,9 @@ extern "C" int mops_hip_short_conv(const void* x, int64_t x_row_stride, const fl
   using namespace mops;
   if (!known_dtype(dtype) || tokens < 0 || channels <= 0 || taps <= 0 || taps > 1024 || num_slots <= 0) return MOPS_HIP_EINVAL;
   if (tokens == 0) return MOPS_HIP_OK;
-  if (!x || !weight || !bias || !ring || !token_seq || !cu_seqlens || !starts || !state_slots || !out || x_row_stride < channels)
+  if (!x || !weight || !ring || !token_seq || !cu_seqlens || !starts || !state_slots || !out || x_row_stride < channels)
     return MOPS_HIP_EINVAL;
-  const bool vec = channels % 8 == 0 && x_row_stride % 8 == 0 && aligned16(x) && aligned16(weight) && aligned16(bias) && aligned16(ring) && aligned16(out);
+  const bool vec = channels % 8 == 0 && x_row_stride % 8 == 0 && aligned16(x) && aligned16(weight) && (!bias || aligned16(bias)) && aligned16(ring) && aligned16(out);
   const int64_t wgs = (tokens * (channels / (vec ? 8 : 1)) + 255) / 256;
   if (wgs > 0x7fffffffLL) return MOPS_HIP_EUNSUPPORTED;
   hipStream_t s = (hipStream_t)stream;

@@ -7,8 +7,10 @@
 //   add_norm_norm      x += norm(y) * w_out, out = norm(x) * w_in: norms behind one sublayer and in front of the next, in one pass;
 //                      RMS norms or layer norms
 //   layer_norm_f32     out = (x - mean) / sqrt(variance + eps) * w of the float32 stream
+//   add_norm           x += y + shift, or x = y + shift, then out = norm(x) * w + b (or x itself) in the activation type: a sublayer's
+//                      output as it is, the norm in front of the next one
 //   embed_pairs        embed_residual plus a row of a table of pairs of tokens
-//   gated_group_norm   rms over equal parts of a row, with silu(gate) multiplied in before or after the division
+//   gated_group_norm   rms over equal parts of a row, with silu(gate) or sigmoid(gate) multiplied in before or after the division
 //
 // A row belongs to one workgroup of 64 or 256 threads; the elements a thread owns stay in its registers between the
 // statistics and the scaling (up to kKeep pieces; longer rows read the rest again).
@@ -21,7 +23,7 @@ constexpr int kKeep = 4;
 template <typename T, int VEC>
 __global__ __launch_bounds__(256) void embed_residual_kernel(const int64_t* __restrict__ ids, const T* __restrict__ table,
                                                              int64_t table_stride, float scale, float* __restrict__ x, T* __restrict__ act,
-                                                             int64_t vocab, int width) {
+                                                             int64_t act_stride, int64_t vocab, int width) {
   const int64_t row = blockIdx.x;
   const int64_t id = ids[row];
   const bool ok = id >= 0 && id < vocab;
@@ -33,7 +35,7 @@ __global__ __launch_bounds__(256) void embed_residual_kernel(const int64_t* __re
 #pragma unroll
     for (int e = 0; e < VEC; ++e) v[e] *= scale;
     store_vec<VEC>(x + row * width + c, v);
-    if (act) store_vec<VEC>(act + row * width + c, v);
+    if (act) store_vec<VEC>(act + row * act_stride + c, v);
   }
 }
 
@@ -256,11 +258,97 @@ __global__ __launch_bounds__(THREADS) void layer_norm_kernel(const float* __rest
   });
 }
 
+// residual += y + shift (or = y + shift; y and shift may be missing), out = norm(residual) * w + b, or the residual without w.
+template <typename T, int VEC, int THREADS, bool CENTER>
+__global__ __launch_bounds__(THREADS) void add_norm_kernel(const mops_hip_add_norm_args a) {
+  __shared__ float scratch[THREADS / kWave];
+  const int64_t row = blockIdx.x;
+  const int n = (int)a.n;
+  float* xr = a.residual + row * n;
+  const T *yr = a.y ? (const T*)a.y + row * a.y_stride : nullptr, *w = (const T*)a.w, *b = (const T*)a.b;
+  T* out = a.out ? (T*)a.out + row * a.out_stride : nullptr;
+  float keep[kKeep][VEC];
+  auto each = [&](auto&& f) {      // pieces behind the kept ones: this thread's own stores, once it has made them
+#pragma unroll
+    for (int it = 0; it < kKeep; ++it) {
+      const int c = (it * THREADS + threadIdx.x) * VEC;
+      if (c < n) f(c, keep[it]);
+    }
+    for (int c = (kKeep * THREADS + threadIdx.x) * VEC; c < n; c += THREADS * VEC) {
+      float v[VEC];
+      load_vec<VEC>(xr + c, v);
+      f(c, v);
+    }
+  };
+  auto read = [&](int c, float (&v)[VEC]) {
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) v[e] = 0.f;
+    if (!a.replace) load_vec<VEC>(xr + c, v);
+    if (!yr && !a.shift) return;
+    float u[VEC];
+    if (yr) {
+      load_vec<VEC>(yr + c, u);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) v[e] += u[e];
+    }
+    if (a.shift) {
+      load_vec<VEC>(a.shift + c, u);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) v[e] += u[e];
+    }
+    store_vec<VEC>(xr + c, v);
+  };
+#pragma unroll
+  for (int it = 0; it < kKeep; ++it) {
+    const int c = (it * THREADS + threadIdx.x) * VEC;
+    if (c < n) read(c, keep[it]);
+  }
+  for (int c = (kKeep * THREADS + threadIdx.x) * VEC; c < n; c += THREADS * VEC) {
+    float v[VEC];
+    read(c, v);
+  }
+  if (!out) return;
+  float mean = 0.f, rstd = 1.f;
+  if (w) {
+    float sum = 0.f;
+    if (CENTER) {
+      each([&](int, float (&v)[VEC]) {
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) sum += v[e];
+      });
+      mean = block_sum<THREADS>(sum, scratch) / (float)n;
+    }
+    float squares = 0.f;
+    each([&](int, float (&v)[VEC]) {
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) squares += (v[e] - mean) * (v[e] - mean);
+    });
+    rstd = 1.0f / sqrtf(block_sum<THREADS>(squares, scratch) / (float)n + a.eps);
+  }
+  each([&](int c, float (&v)[VEC]) {
+    float o[VEC], u[VEC];
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) o[e] = (v[e] - mean) * rstd;
+    if (w) {
+      load_vec<VEC>(w + c, u);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) o[e] *= u[e];
+    }
+    if (b) {
+      load_vec<VEC>(b + c, u);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) o[e] += u[e];
+    }
+    store_vec<VEC>(out + c, o);
+  });
+}
+
 // LANES lanes per (row, part): parts of `size` consecutive elements.
 template <typename T, int VEC, int LANES, bool GATE_FIRST>
 __global__ __launch_bounds__(256) void gated_group_norm_kernel(const T* __restrict__ y, int64_t y_stride, const T* __restrict__ gate,
-                                                               int64_t gate_stride, const T* __restrict__ w, float eps,
-                                                               T* __restrict__ out, int64_t rows, int groups, int size) {
+                                                               int64_t gate_stride, const T* __restrict__ w, bool shared_w, bool plain_sigmoid,
+                                                               float eps, float scale, T* __restrict__ out, int64_t out_stride, int64_t rows,
+                                                               int groups, int size) {
   const int64_t item = (int64_t)blockIdx.x * (256 / LANES) + threadIdx.x / LANES;
   if (item >= rows * groups) return;      // whole groups of lanes leave; the sums below stay inside a group
   const int lane = threadIdx.x & (LANES - 1);
@@ -268,7 +356,8 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(const T* __restri
   const int col0 = (int)(item % groups) * size;
   const T* yr = y + row * y_stride + col0;
   const T* gr = gate + row * gate_stride + col0;
-  T* orow = out + row * (int64_t)groups * size + col0;
+  T* orow = out + row * out_stride + col0;
+  if (w && !shared_w) w += col0;
   float keep[kKeep][VEC], gk[kKeep][VEC];
   float ss = 0.f;
   auto read = [&](int c, float (&v)[VEC], float (&g)[VEC]) {
@@ -276,7 +365,7 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(const T* __restri
     load_vec<VEC>(gr + c, g);
 #pragma unroll
     for (int e = 0; e < VEC; ++e) {
-      g[e] = silu_for<T>(g[e]);
+      g[e] = plain_sigmoid ? sigmoid_for<T>(g[e]) : silu_for<T>(g[e]);
       if (GATE_FIRST) v[e] *= g[e];
     }
   };
@@ -295,14 +384,14 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(const T* __restri
 #pragma unroll
     for (int e = 0; e < VEC; ++e) ss += v[e] * v[e];
   }
-  const float rstd = 1.0f / sqrtf(group_sum<LANES>(ss) / (float)size + eps);
+  const float rstd = scale / sqrtf(group_sum<LANES>(ss) / (float)size + eps);
   auto finish = [&](int c, const float (&v)[VEC], const float (&g)[VEC]) {
     float o[VEC];
 #pragma unroll
     for (int e = 0; e < VEC; ++e) o[e] = GATE_FIRST ? v[e] * rstd : v[e] * rstd * g[e];
     if (w) {
       float wv[VEC];
-      load_vec<VEC>(w + col0 + c, wv);
+      load_vec<VEC>(w + c, wv);
 #pragma unroll
       for (int e = 0; e < VEC; ++e) o[e] *= wv[e];
     }
@@ -337,16 +426,17 @@ static void launch_norm(float* residual, const void* y, int64_t y_stride, const 
 }  // namespace mops
 
 extern "C" int mops_hip_embed_residual(const int64_t* ids, const void* table, int64_t table_row_stride, int dtype, float scale,
-                                       float* residual, void* act, int64_t n_ids, int64_t vocab, int64_t width, void* stream) {
+                                       float* residual, void* act, int64_t act_stride, int64_t n_ids, int64_t vocab, int64_t width,
+                                       void* stream) {
   using namespace mops;
   if (!known_dtype(dtype) || n_ids < 0 || vocab <= 0 || width <= 0 || width > (1 << 20) || n_ids > 0x7fffffffLL) return MOPS_HIP_EINVAL;
   if (n_ids == 0) return MOPS_HIP_OK;
-  if (!ids || !table || !residual || table_row_stride < width) return MOPS_HIP_EINVAL;
-  const bool vec = width % 8 == 0 && table_row_stride % 8 == 0 && aligned16(table) && aligned16(residual) && (!act || aligned16(act));
+  if (!ids || !table || !residual || table_row_stride < width || (act && act_stride < width)) return MOPS_HIP_EINVAL;
+  const bool vec = width % 8 == 0 && table_row_stride % 8 == 0 && aligned16(table) && aligned16(residual) && (!act || (aligned16(act) && act_stride % 8 == 0));
   const dim3 grid((unsigned)n_ids), block(256);
   hipStream_t s = (hipStream_t)stream;
 #define MOPS_EMBED(T, V) hipLaunchKernelGGL((embed_residual_kernel<T, V>), grid, block, 0, s, ids, (const T*)table, table_row_stride, \
-                                            scale, residual, (T*)act, vocab, (int)width)
+                                            scale, residual, (T*)act, act_stride, vocab, (int)width)
   if (dtype == MOPS_HIP_BF16) { if (vec) MOPS_EMBED(bf16_t, 8); else MOPS_EMBED(bf16_t, 1); }
   else { if (vec) MOPS_EMBED(float, 8); else MOPS_EMBED(float, 1); }
 #undef MOPS_EMBED
@@ -423,6 +513,32 @@ extern "C" int mops_hip_layer_norm_f32(const float* x, const void* weight, float
   return finish_launch();
 }
 
+extern "C" int mops_hip_add_norm(const mops_hip_add_norm_args* a, void* stream) {
+  using namespace mops;
+  if (!a || !known_dtype(a->dtype) || a->rows < 0 || a->n <= 0 || a->n > (1 << 20) || a->rows > 0x7fffffffLL) return MOPS_HIP_EINVAL;
+  if (a->rows == 0) return MOPS_HIP_OK;
+  if (!a->residual || (a->y && a->y_stride < a->n) || (a->out && a->out_stride < a->n) || (a->y && a->y == a->out) || (a->b && !a->w) ||
+      (a->replace && !a->y && !a->shift))
+    return MOPS_HIP_EINVAL;
+  auto good = [](const void* p) { return !p || aligned16(p); };
+  const bool vec = a->n % 8 == 0 && (!a->y || a->y_stride % 8 == 0) && (!a->out || a->out_stride % 8 == 0) && good(a->residual) && good(a->y) &&
+                   good(a->shift) && good(a->w) && good(a->b) && good(a->out);
+  const dim3 grid((unsigned)a->rows);
+  hipStream_t s = (hipStream_t)stream;
+#define MOPS_AN(T, V, TH, C) hipLaunchKernelGGL((add_norm_kernel<T, V, TH, C>), grid, dim3(TH), 0, s, *a)
+#define MOPS_AN_TYPE(T, C) do {                          \
+    if (vec && a->n <= 1024) MOPS_AN(T, 8, 64, C);       \
+    else if (vec) MOPS_AN(T, 8, 256, C);                 \
+    else if (a->n <= 512) MOPS_AN(T, 1, 64, C);          \
+    else MOPS_AN(T, 1, 256, C);                          \
+  } while (0)
+  if (a->dtype == MOPS_HIP_BF16) { if (a->center) MOPS_AN_TYPE(bf16_t, true); else MOPS_AN_TYPE(bf16_t, false); }
+  else { if (a->center) MOPS_AN_TYPE(float, true); else MOPS_AN_TYPE(float, false); }
+#undef MOPS_AN_TYPE
+#undef MOPS_AN
+  return finish_launch();
+}
+
 extern "C" int mops_hip_embed_pairs(const mops_hip_embed_pairs_args* a, void* stream) {
   using namespace mops;
   if (!a || !known_dtype(a->dtype) || a->tokens < 0 || a->vocab <= 0 || a->width <= 0 || a->width > (1 << 20) || a->buckets <= 0 || a->num_slots <= 0)
@@ -443,21 +559,23 @@ extern "C" int mops_hip_embed_pairs(const mops_hip_embed_pairs_args* a, void* st
 }
 
 extern "C" int mops_hip_gated_group_norm(const void* y, int64_t y_row_stride, const void* gate, int64_t gate_row_stride,
-                                         const void* weight, float eps, int gate_first, void* out, int dtype,
-                                         int64_t rows, int64_t groups, int64_t group_size, void* stream) {
+                                         const void* weight, int shared_weight, float eps, int gate_first, int plain_sigmoid, float scale,
+                                         void* out, int64_t out_row_stride, int dtype, int64_t rows, int64_t groups, int64_t group_size,
+                                         void* stream) {
   using namespace mops;
   if (!known_dtype(dtype) || rows < 0 || groups <= 0 || group_size <= 0 || groups * group_size > (1 << 24)) return MOPS_HIP_EINVAL;
   if (rows == 0) return MOPS_HIP_OK;
   const int64_t n = groups * group_size;
-  if (!y || !gate || !out || y_row_stride < n || gate_row_stride < n || out == gate) return MOPS_HIP_EINVAL;
-  const bool vec = group_size % 8 == 0 && y_row_stride % 8 == 0 && gate_row_stride % 8 == 0 && aligned16(y) && aligned16(gate) &&
+  if (!y || !gate || !out || y_row_stride < n || gate_row_stride < n || out_row_stride < n || out == gate) return MOPS_HIP_EINVAL;
+  const bool vec = group_size % 8 == 0 && out_row_stride % 8 == 0 && y_row_stride % 8 == 0 && gate_row_stride % 8 == 0 && aligned16(y) && aligned16(gate) &&
                    aligned16(out) && (!weight || aligned16(weight));
   const bool small = vec && group_size <= 64, narrow = group_size <= 512;      // eight lanes, a row of lanes, a wave per group
   const int64_t per_wg = small ? 32 : (narrow ? 16 : 4), wgs = (rows * groups + per_wg - 1) / per_wg;
   if (wgs > 0x7fffffffLL) return MOPS_HIP_EUNSUPPORTED;
   hipStream_t s = (hipStream_t)stream;
 #define MOPS_GGN(T, V, L, F) hipLaunchKernelGGL((gated_group_norm_kernel<T, V, L, F>), dim3((unsigned)wgs), dim3(256), 0, s, (const T*)y, \
-                          y_row_stride, (const T*)gate, gate_row_stride, (const T*)weight, eps, (T*)out, rows, (int)groups, (int)group_size)
+                          y_row_stride, (const T*)gate, gate_row_stride, (const T*)weight, shared_weight != 0, plain_sigmoid != 0, eps, scale, \
+                          (T*)out, out_row_stride, rows, (int)groups, (int)group_size)
 #define MOPS_GGN2(T, V) do {                                    \
     if (V == 8 && small) { if (gate_first) MOPS_GGN(T, V, 8, true); else MOPS_GGN(T, V, 8, false); }  \
     else if (narrow) { if (gate_first) MOPS_GGN(T, V, 16, true); else MOPS_GGN(T, V, 16, false); }  \

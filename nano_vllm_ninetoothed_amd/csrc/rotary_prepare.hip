@@ -1,6 +1,7 @@
 // rotary_prepare: what stands between the packed projections [q | k | v] of every token and attention over paged keys and values:
 // an optional RMS norm per head on q and k (one weight for all heads), a rotation of their first `rot` elements by the token's
-// position, q to its own rows, k and v to their pages.  Pair i of a rotation is (element i, element i + rot / 2).
+// position, q to its own rows, k and v to their pages.  Pair i of a rotation is (element i, element i + rot / 2), or with `neighbours`
+// (element 2i, element 2i + 1).  A bias over [q | k | v] is added first.
 //
 // LANES lanes own one head of one token, eight elements each, and take the other half of a pair from the lane that holds it.  Heads
 // wider than that, or of odd sizes: a wave per head, element by element, with the other half read again.
@@ -23,12 +24,21 @@ __global__ __launch_bounds__(256) void rotary_prepare_kernel(const mops_hip_rota
     h -= heads + groups;
     if (!filed) return;
     const T* src = row + (heads + groups) * dim + h * vdim;
+    const T* bias = a.bias ? (const T*)a.bias + (heads + groups) * dim + h * vdim : nullptr;
     T* dst = (T*)a.v_pages + (slot * groups + h) * vp;
     for (int c = lane * VEC; c < vp; c += LANES * VEC) {
       float v[VEC];
 #pragma unroll
       for (int e = 0; e < VEC; ++e) v[e] = 0.f;
-      if (VEC > 1 || c < vdim) load_vec<VEC>(src + c, v);
+      if (VEC > 1 || c < vdim) {
+        load_vec<VEC>(src + c, v);
+        if (bias) {
+          float bv[VEC];
+          load_vec<VEC>(bias + c, bv);
+#pragma unroll
+          for (int e = 0; e < VEC; ++e) v[e] += bv[e];
+        }
+      }
       store_vec<VEC>(dst + c, v);
     }
     return;
@@ -41,6 +51,16 @@ __global__ __launch_bounds__(256) void rotary_prepare_kernel(const mops_hip_rota
   const T* src = row + h * dim;
   T* dst = is_q ? (T*)a.q + (t * heads + h) * dp : (T*)a.k_pages + (slot * groups + h - heads) * dp;
   const T* w = (const T*)(is_q ? a.q_weight : a.k_weight);
+  const T* bias = a.bias ? (const T*)a.bias + h * dim : nullptr;
+  auto load = [&](int c, float (&v)[VEC]) {
+    load_vec<VEC>(src + c, v);
+    if (bias) {
+      float bv[VEC];
+      load_vec<VEC>(bias + c, bv);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) v[e] += bv[e];
+    }
+  };
   if (!is_q && !filed) return;
   if (VEC == 8) {
     const int c = lane * 8;
@@ -48,9 +68,9 @@ __global__ __launch_bounds__(256) void rotary_prepare_kernel(const mops_hip_rota
     float v[VEC];
 #pragma unroll
     for (int e = 0; e < VEC; ++e) v[e] = 0.f;
-    if (mine) load_vec<VEC>(src + c, v);
+    if (mine) load(c, v);
     float cs[VEC], sn[VEC];
-    if (turns) {
+    if (turns && !a.neighbours) {
       load_vec<VEC>(trig + (low ? c : c - half), cs);
       load_vec<VEC>(trig + half + (low ? c : c - half), sn);
     }
@@ -62,6 +82,21 @@ __global__ __launch_bounds__(256) void rotary_prepare_kernel(const mops_hip_rota
       const float r = 1.0f / sqrtf(group_sum<LANES>(ss) / (float)dim + a.eps);
 #pragma unroll
       for (int e = 0; e < VEC; ++e) v[e] = mine ? v[e] * r * wv[e] : 0.f;
+    }
+    if (a.neighbours) {      // whole pairs in a lane
+      if (turns) {
+        float pc[4], ps[4];
+        load_vec<4>(trig + c / 2, pc);
+        load_vec<4>(trig + half + c / 2, ps);
+#pragma unroll
+        for (int i = 0; i < VEC / 2; ++i) {
+          const float x = v[2 * i], y = v[(2 * i + 1) % VEC];
+          v[2 * i] = x * pc[i] - y * ps[i];
+          v[(2 * i + 1) % VEC] = y * pc[i] + x * ps[i];
+        }
+      }
+      if (mine) store_vec<VEC>(dst + c, v);
+      return;
     }
     const int from = turns ? lane + (low ? half : -half) / 8 : lane;
 #pragma unroll
@@ -77,14 +112,14 @@ __global__ __launch_bounds__(256) void rotary_prepare_kernel(const mops_hip_rota
     float ss = 0.f;
     for (int c = lane * VEC; c < dim; c += LANES * VEC) {
       float v[VEC];
-      load_vec<VEC>(src + c, v);
+      load(c, v);
 #pragma unroll
       for (int e = 0; e < VEC; ++e) ss += v[e] * v[e];
     }
     r = 1.0f / sqrtf(group_sum<LANES>(ss) / (float)dim + a.eps);
   }
   auto normed = [&](int c, float (&v)[VEC]) {
-    load_vec<VEC>(src + c, v);
+    load(c, v);
     if (w) {
       float wv[VEC];
       load_vec<VEC>(w + c, wv);
@@ -99,11 +134,12 @@ __global__ __launch_bounds__(256) void rotary_prepare_kernel(const mops_hip_rota
     if (c < dim) {
       normed(c, v);
       if (c < rot) {
-        const bool low = c < half;
+        const bool low = a.neighbours ? c % 2 == 0 : c < half;
+        const int pair = a.neighbours ? c / 2 : (low ? c : c - half), mate = a.neighbours ? (low ? c + 1 : c - 1) : (low ? c + half : c - half);
         float o[VEC], cs[VEC], sn[VEC];
-        normed(low ? c + half : c - half, o);
-        load_vec<VEC>(trig + (low ? c : c - half), cs);
-        load_vec<VEC>(trig + half + (low ? c : c - half), sn);
+        normed(mate, o);
+        load_vec<VEC>(trig + pair, cs);
+        load_vec<VEC>(trig + half + pair, sn);
 #pragma unroll
         for (int e = 0; e < VEC; ++e) v[e] = low ? v[e] * cs[e] - o[e] * sn[e] : v[e] * cs[e] + o[e] * sn[e];
       }
@@ -123,7 +159,7 @@ extern "C" int mops_hip_rotary_prepare(const mops_hip_rotary_prepare_args* a, vo
   if (!a->qkv || !a->positions || !a->slot_mapping || !a->q || !a->k_pages || !a->v_pages || (a->rot && !a->cos_sin)) return MOPS_HIP_EINVAL;
   if (a->qkv_stride < (a->heads + a->kv_heads) * a->dim + a->kv_heads * a->vdim) return MOPS_HIP_EINVAL;
   if (a->tokens > 0x7fffffffLL || a->heads * a->dim > (1 << 20) || a->kv_heads * (a->dim + a->vdim) > (1 << 20)) return MOPS_HIP_EUNSUPPORTED;
-  const bool vec = a->dim % 8 == 0 && a->vdim % 8 == 0 && a->rot % 16 == 0 && a->qkv_stride % 8 == 0 && aligned16(a->qkv) && aligned16(a->q) &&
+  const bool vec = a->dim % 8 == 0 && a->vdim % 8 == 0 && a->rot % (a->neighbours ? 8 : 16) == 0 && (!a->bias || aligned16(a->bias)) && a->qkv_stride % 8 == 0 && aligned16(a->qkv) && aligned16(a->q) &&
                    aligned16(a->k_pages) && aligned16(a->v_pages) && aligned16(a->cos_sin) && (!a->q_weight || aligned16(a->q_weight)) &&
                    (!a->k_weight || aligned16(a->k_weight));
   const int64_t items = a->heads + 2 * a->kv_heads, widest = a->dim > a->vdim ? a->dim : a->vdim;

@@ -3,7 +3,8 @@
 //   token_mix        out[p][t] = x[t] + (x[t-1] - x[t]) * mu[p] for several vectors mu at once: every token is moved some way
 //                    towards the token in front of it.  The row in front of a portion comes from one row per state slot (zeros
 //                    at the start of a sequence), which receives the last row of the portion.
-//   low_rank_decay   out[t, c] = -exp(sum_r w2[c, r] tanh(z[t, r]) + w0[c]): the natural logarithm of a decay per channel, float32
+//   low_rank_decay   out[t, c] = -exp(sum_r w2[c, r] tanh(z[t, r]) + w0[c]): the natural logarithm of a decay per channel, float32; or
+//                    with a rate per head out[t, c] = rate[head of c] softplus(sum_r w2[c, r] z[t, r] + w0[c])
 #include "mfma_tiles.h"
 
 namespace mops {
@@ -58,11 +59,12 @@ __device__ __forceinline__ float tanh_fast(float v) {
   return 1.0f - 2.0f * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(2.8853900817779268f * v));
 }
 
-// Workgroup = 16 TT tokens x 256 channels, a wave takes 64 of the channels; tanh(z) in LDS, the rows of w2 straight from memory.
-template <int TT>
+// Workgroup = 16 TT tokens x 256 channels, a wave takes 64 of the channels; tanh(z) (with RATED z) in LDS, the rows of w2 straight from
+// memory.
+template <int TT, bool RATED>
 __global__ __launch_bounds__(256) void low_rank_decay_mfma_kernel(const uint16_t* __restrict__ z, int64_t z_stride, const uint16_t* __restrict__ w2,
-                                                                  const float* __restrict__ w0, float* __restrict__ out, int64_t tokens,
-                                                                  int channels, int rank, bool aligned, bool z_aligned, bool wide) {
+                                                                  const float* __restrict__ w0, const float* __restrict__ rate, int head_size,
+                                                                  float* __restrict__ out, int64_t tokens, int channels, int rank, bool aligned, bool z_aligned, bool wide) {
   constexpr int kDecayTokens = 16 * TT;
   extern __shared__ __align__(16) unsigned char smem[];
   uint16_t* const tile = reinterpret_cast<uint16_t*>(smem);
@@ -81,8 +83,10 @@ __global__ __launch_bounds__(256) void low_rank_decay_mfma_kernel(const uint16_t
     const int r = i / (ksteps * 4), k = i % (ksteps * 4) * 8;
     u32x4 w = {0u, 0u, 0u, 0u};
     if (t0 + r < tokens) w = load8_guarded(z + (t0 + r) * z_stride, k, rank, z_aligned);
+    if (!RATED) {
 #pragma unroll
-    for (int e = 0; e < 4; ++e) w[e] = pack_bf16x2(tanh_fast(bf16lo_to_f32(w[e])), tanh_fast(bf16hi_to_f32(w[e])));
+      for (int e = 0; e < 4; ++e) w[e] = pack_bf16x2(tanh_fast(bf16lo_to_f32(w[e])), tanh_fast(bf16hi_to_f32(w[e])));
+    }
     store16(tile + r * pitch + k, w);
   }
   __syncthreads();
@@ -105,16 +109,22 @@ __global__ __launch_bounds__(256) void low_rank_decay_mfma_kernel(const uint16_t
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int c = c0 + 16 * i + 4 * jj;
-    float bias[4];
+    float bias[4], per[4];
 #pragma unroll
-    for (int e = 0; e < 4; ++e) bias[e] = c + e < channels ? w0[c + e] : 0.f;
+    for (int e = 0; e < 4; ++e) {
+      bias[e] = c + e < channels ? w0[c + e] : 0.f;
+      per[e] = RATED && c + e < channels ? rate[(c + e) / head_size] : 0.f;
+    }
 #pragma unroll
     for (int j = 0; j < TT; ++j) {
       const int64_t t = t0 + 16 * j + n;
       if (t >= tokens) continue;
       f32x4 o;
 #pragma unroll
-      for (int e = 0; e < 4; ++e) o[e] = -__builtin_amdgcn_exp2f(1.4426950408889634f * (acc[i][j][e] + bias[e]));
+      for (int e = 0; e < 4; ++e) {
+        const float x = acc[i][j][e] + bias[e];
+        o[e] = RATED ? per[e] * softplus_fast(x) : -__builtin_amdgcn_exp2f(1.4426950408889634f * x);
+      }
       float* dst = out + t * channels + c;
       if (wide && c + 4 <= channels) {
         *reinterpret_cast<f32x4*>(dst) = o;
@@ -131,17 +141,20 @@ constexpr int kDecayPlainRank = 4096;
 
 template <typename T>
 __global__ __launch_bounds__(256) void low_rank_decay_kernel(const T* __restrict__ z, int64_t z_stride, const T* __restrict__ w2,
-                                                             const float* __restrict__ w0, float* __restrict__ out, int64_t tokens,
-                                                             int channels, int rank) {
+                                                             const float* __restrict__ w0, const float* __restrict__ rate, int head_size,
+                                                             float* __restrict__ out, int64_t tokens, int channels, int rank) {
   __shared__ float th[kDecayPlainRank];
   const int64_t t = blockIdx.x;
-  for (int r = threadIdx.x; r < rank; r += 256) th[r] = tanhf(to_f32(z[t * z_stride + r]));
+  for (int r = threadIdx.x; r < rank; r += 256) {
+    const float x = to_f32(z[t * z_stride + r]);
+    th[r] = rate ? x : tanhf(x);
+  }
   __syncthreads();
   const int c = blockIdx.y * 256 + threadIdx.x;
   if (c >= channels) return;
   float acc = w0[c];
   for (int r = 0; r < rank; ++r) acc += to_f32(w2[(int64_t)c * rank + r]) * th[r];
-  out[t * channels + c] = -expf(acc);
+  out[t * channels + c] = rate ? rate[c / head_size] * softplus_f32(acc) : -expf(acc);
 }
 
 }  // namespace mops
@@ -164,12 +177,12 @@ extern "C" int mops_hip_token_mix(const void* x, int64_t x_row_stride, const flo
   return finish_launch();
 }
 
-extern "C" int mops_hip_low_rank_decay(const void* z, int64_t z_row_stride, const void* w2, const float* w0, float* out, int dtype,
-                                       int64_t tokens, int64_t channels, int64_t rank, void* stream) {
+extern "C" int mops_hip_low_rank_decay(const void* z, int64_t z_row_stride, const void* w2, const float* w0, const float* rate, int64_t head_size,
+                                       float* out, int dtype, int64_t tokens, int64_t channels, int64_t rank, void* stream) {
   using namespace mops;
   if (!known_dtype(dtype) || tokens < 0 || channels <= 0 || channels > (1 << 22) || rank <= 0) return MOPS_HIP_EINVAL;
   if (tokens == 0) return MOPS_HIP_OK;
-  if (!z || !w2 || !w0 || !out || z_row_stride < rank) return MOPS_HIP_EINVAL;
+  if (!z || !w2 || !w0 || !out || z_row_stride < rank || (rate && head_size <= 0)) return MOPS_HIP_EINVAL;
   if (rank > kDecayPlainRank || tokens > 0x7fffffffLL || (channels + 255) / 256 > 65535) return MOPS_HIP_EUNSUPPORTED;
   hipStream_t s = (hipStream_t)stream;
   if (dtype == MOPS_HIP_BF16 && rank <= kDecayMaxRank) {
@@ -177,16 +190,18 @@ extern "C" int mops_hip_low_rank_decay(const void* z, int64_t z_row_stride, cons
     const dim3 grid((unsigned)((tokens + per - 1) / per), (unsigned)((channels + kDecayChannels - 1) / kDecayChannels));
     const size_t lds = per * ((rank + 31) / 32 * 32 + 8) * 2;
     const bool w_aligned = rank % 8 == 0 && aligned16(w2), z_aligned = z_row_stride % 8 == 0 && aligned16(z), wide = channels % 4 == 0 && aligned16(out);
-#define MOPS_LRM(TT) hipLaunchKernelGGL((low_rank_decay_mfma_kernel<TT>), grid, dim3(256), lds, s, (const uint16_t*)z, z_row_stride, (const uint16_t*)w2, w0, \
-                                        out, tokens, (int)channels, (int)rank, w_aligned, z_aligned, wide)
+#define MOPS_LRM2(TT, R) hipLaunchKernelGGL((low_rank_decay_mfma_kernel<TT, R>), grid, dim3(256), lds, s, (const uint16_t*)z, z_row_stride, \
+                                        (const uint16_t*)w2, w0, rate, (int)head_size, out, tokens, (int)channels, (int)rank, w_aligned, z_aligned, wide)
+#define MOPS_LRM(TT) do { if (rate) MOPS_LRM2(TT, true); else MOPS_LRM2(TT, false); } while (0)
     if (per == 16) MOPS_LRM(1);
     else MOPS_LRM(4);
 #undef MOPS_LRM
+#undef MOPS_LRM2
     return finish_launch();
   }
   const dim3 grid((unsigned)tokens, (unsigned)((channels + 255) / 256));
-#define MOPS_LRD(T) hipLaunchKernelGGL((low_rank_decay_kernel<T>), grid, dim3(256), 0, s, (const T*)z, z_row_stride, (const T*)w2, w0, out, tokens, \
-                                       (int)channels, (int)rank)
+#define MOPS_LRD(T) hipLaunchKernelGGL((low_rank_decay_kernel<T>), grid, dim3(256), 0, s, (const T*)z, z_row_stride, (const T*)w2, w0, rate, (int)head_size, out, \
+                                       tokens, (int)channels, (int)rank)
   if (dtype == MOPS_HIP_BF16) MOPS_LRD(bf16_t);
   else MOPS_LRD(float);
 #undef MOPS_LRD

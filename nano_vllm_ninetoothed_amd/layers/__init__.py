@@ -7,6 +7,7 @@ A mixer takes its cache or state in allocate(cache); again(cache) gives another 
 its own, for layers that run several times in a forward pass.
 A feed-forward is built the same way and called as ff(x).  Its result may have several rows per token, one behind the other,
 that count as their sum; or be a pair of such a result and one more [tokens, width] that is added.
+Sublayers of two products (joined.py) can be run as one where they read the same input.
 """
 from __future__ import annotations
 
@@ -140,4 +141,5 @@ def hip_op(name):
     return mops.get_op(name, "hip")
 
 
-from . import biased_attention, feed_forward, latent_attention, mamba2, mixture, retention, rotary_attention, time_mixing  # noqa: E402,F401  (register themselves)
+from . import (biased_attention, feed_forward, gated_delta, latent_attention, mamba2, matrix_memory, mixture, projected_attention, retention,  # noqa: E402,F401
+               rotary_attention, side_by_side, time_mixing)  # (register themselves)

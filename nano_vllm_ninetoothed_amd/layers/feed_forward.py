@@ -2,9 +2,10 @@
 from __future__ import annotations
 
 from . import hip_op, pack, register_feed_forward, require_size
+from .joined import TwoProducts
 
 
-class GatedLinearUnit:
+class GatedLinearUnit(TwoProducts):
     """W_down f(W_gate x, W_up x); a subclass says what f is."""
 
     @staticmethod
@@ -16,16 +17,20 @@ class GatedLinearUnit:
         # the halves start at multiples of eight columns
         self.half = (self.ff + 7) // 8 * 8
         gate, up = (weights.take(prefix + n, (self.ff, m.width)) for n in ("gate", "up"))
-        self.gate_up = pack([pack([gate]), pack([up])])
         self.down = weights.take(prefix + "down", (m.width, self.ff))
-        self.linear = hip_op("linear")
+        self.products([gate, up], self.down)
+        self.gate_up, self.linear = self.w_in, hip_op("linear")
 
-    def unit(self, gate, up):
+    def unit(self, gate, up, out=None):
         raise NotImplementedError
 
-    def __call__(self, x):
-        p = self.linear(x, self.gate_up)
-        return self.linear(self.unit(p[:, :self.ff], p[:, self.half:self.half + self.ff]), self.down)
+    def mix(self, p, ctx, out, scale=1.0):
+        if scale != 1.0:
+            raise ValueError("a gated unit takes no factor")
+        self.unit(*self.parts_of(p), out=out)
+
+    def __call__(self, x, ctx=None):
+        return self.linear(self.unit(*self.parts_of(self.linear(x, self.gate_up))), self.down)
 
 
 @register_feed_forward("clamped_glu")
@@ -42,8 +47,8 @@ class ClampedGLU(GatedLinearUnit):
         super().__init__(sizes, weights, prefix, m)
         self.limit, self.glu = float(sizes["limit"]), hip_op("clamped_glu")
 
-    def unit(self, gate, up):
-        return self.glu(gate, up, self.limit, self.ALPHA)
+    def unit(self, gate, up, out=None):
+        return self.glu(gate, up, self.limit, self.ALPHA, out=out)
 
 
 @register_feed_forward("gelu_glu")
@@ -54,8 +59,20 @@ class GeluGLU(GatedLinearUnit):
         super().__init__(sizes, weights, prefix, m)
         self.glu = hip_op("gelu_glu")
 
-    def unit(self, gate, up):
-        return self.glu(gate, up)
+    def unit(self, gate, up, out=None):
+        return self.glu(gate, up, out=out)
+
+
+@register_feed_forward("relu_glu")
+class ReluGLU(GatedLinearUnit):
+    """f = max(W_gate x, 0) * W_up x."""
+
+    def __init__(self, sizes, weights, prefix, m):
+        super().__init__(sizes, weights, prefix, m)
+        self.glu = hip_op("relu_glu")
+
+    def unit(self, gate, up, out=None):
+        return self.glu(gate, up, out=out)
 
 
 @register_feed_forward("squared_relu")

@@ -34,12 +34,13 @@ class PagedAttention(Mixer):
         self.k_pages = cache.paged(self.kv_heads, padded(self.dim), dtype=self.dtype)
         self.v_pages = cache.paged(self.kv_heads, padded(self.vdim), dtype=self.dtype)
 
-    def attend(self, q, ctx, gate=None):
-        """Attention of all rows of the batch [tokens, heads * vdim]; gate [tokens, heads]: times its sigmoid."""
+    def attend(self, q, ctx, gate=None, out=None, scale=1.0):
+        """Attention of all rows of the batch [tokens, heads * vdim], into `out` if given; gate [tokens, heads] or [tokens, heads * vdim]:
+        times its sigmoid.  Everything times scale."""
         lens, seqs, table = ctx["token_context"], ctx["token_seq"], ctx["block_tables"]
-        common, options = (self.k_pages, self.v_pages, self.dim, self.vdim), {"slopes": self.slopes, "scores": self.scores}
+        common, options = (self.k_pages, self.v_pages, self.dim, self.vdim), {"slopes": self.slopes, "scores": self.scores, "out_scale": scale}
         plan = self._plan(ctx, q.device) if self.matrix else None
-        o = torch.empty((q.shape[0], self.heads, self.vdim), dtype=q.dtype, device=q.device)
+        o = torch.empty((q.shape[0], self.heads * self.vdim), dtype=q.dtype, device=q.device) if out is None else out
         if plan is None:
             self.rows(q, *common, lens, table, self.scale, row_seq=seqs, gate=gate, out=o, **options)
         else:
@@ -47,7 +48,7 @@ class PagedAttention(Mixer):
             if n:
                 self.rows(q[:n], *common, lens[:n], table, self.scale, row_seq=seqs[:n], gate=None if gate is None else gate[:n], out=o[:n], **options)
             self.prefill(q, *common, tiles, table, self.scale, lens, gate=gate, out=o, **options)
-        return o.view(q.shape[0], self.heads * self.vdim)
+        return o
 
     @staticmethod
     def _plan(ctx, device):

@@ -54,4 +54,4 @@ def parse_config(raw: dict):
     return cls.config_class.from_dict(raw)
 
 
-from . import lulizen, nepulix, qwen3, sozarax  # noqa: E402,F401  (register themselves)
+from . import fedovik, lulizen, nepulix, qwen3, sozarax  # noqa: E402,F401  (register themselves)

@@ -8,35 +8,14 @@ from __future__ import annotations
 
 import torch
 
+from .listed import ListedDecoder
 from ..layers import FEED_FORWARDS, MIXERS, ModelContext, Rotary, hip_op
 
 
-class SandwichDecoder:
-    """A subclass names its mixers and feed-forwards (the configuration's names and those they are registered under), says which norms
-    it has, takes the tensors of its embedding and computes it.  The configuration offers vocab, width, eps, layers and order(): the
-    numbers of the layers in the order in which they run."""
-    TYPES: dict = {}
-    KINDS: dict = {}
+class SandwichDecoder(ListedDecoder):
+    """A subclass also says which norms it has, takes the tensors of its embedding and computes it.  The configuration offers vocab, width,
+    eps, layers and order(): the numbers of the layers in the order in which they run."""
     CENTER = False      # layer norms instead of RMS norms
-    EMBEDDING_SLOTS = False      # whether the embedding keeps something per sequence
-    dtypes = (torch.bfloat16, torch.float32)
-
-    @classmethod
-    def validate_layer(cls, layer) -> None:
-        if layer["type"] not in cls.TYPES:
-            raise ValueError(f"unknown mixer {layer['type']!r}")
-        MIXERS[cls.TYPES[layer["type"]]].validate(layer["mixer"])
-        mlp = layer.get("mlp")
-        if mlp is not None:
-            if mlp["kind"] not in cls.KINDS:
-                raise ValueError(f"unknown feed-forward {mlp['kind']!r}")
-            FEED_FORWARDS[cls.KINDS[mlp["kind"]]].validate(mlp)
-
-    @classmethod
-    def needs(cls, config):
-        """(pages, state slots)"""
-        kinds = [MIXERS[cls.TYPES[layer["type"]]] for layer in config.layers]
-        return any(k.uses_pages for k in kinds), cls.EMBEDDING_SLOTS or any(k.uses_slots for k in kinds)
 
     def __init__(self, config, weights, cache, backend: str = "hip", max_model_len: int = 32768):
         if backend != "hip":
@@ -77,11 +56,6 @@ class SandwichDecoder:
         """The float32 residual stream [tokens, width]."""
         raise NotImplementedError
 
-    def reserve_graph_scratch(self, max_bs: int, max_blocks: int) -> None:
-        """Makes the scratch of the current stream exist before a capture."""
-        from ..mops.hip.ops import _linear_workspace
-        _linear_workspace(self.embed.device)
-
     def _add(self, residual, y, norm_behind, norm_in_front):
         y, extra = y if isinstance(y, tuple) else (y, None)
         return self.op_add_norm_norm(residual, y, norm_behind, norm_in_front, self.shape.eps, center=self.CENTER, extra=extra)
@@ -98,12 +72,4 @@ class SandwichDecoder:
                 x = self._add(residual, ff(x), norm2b, following)
             if self.layer_hook is not None:
                 self.layer_hook(i, residual)
-        if ctx.get("hidden_only"):
-            return x
-        rows = ctx.get("logit_rows")
-        if rows is None and ctx["is_prefill"]:
-            rows = ctx["cu_seqlens"][1:].long() - 1
-        return self.logits(x if rows is None else x[rows])
-
-    def logits(self, hidden):
-        return self.op_linear(hidden, self.head)
+        return self.result(x, ctx)

@@ -5,6 +5,7 @@ from __future__ import annotations
 from dataclasses import dataclass
 
 from . import register_model
+from .listed import looped, parse_loop
 from .sandwich import SandwichDecoder
 from ..layers import hip_op
 
@@ -23,17 +24,12 @@ class SozaraxConfig:
         layers = list(raw["layers"])
         for layer in layers:
             SozaraxModel.validate_layer(layer)
-        loop = raw.get("loop") or {"start": 0, "stop": 0, "times": 1}
-        start, stop, times = (int(loop[n]) for n in ("start", "stop", "times"))
-        if not 0 <= start <= stop <= len(layers) or times < 1:
-            raise ValueError(f"a loop over the layers {start} .. {stop - 1} of {len(layers)}, {times} times")
         return cls(vocab=int(raw["vocab"]), width=int(raw["width"]), eps=float(raw["norm"]["eps"]), embedding_scale=float(raw["embedding"]["scale"]),
-                   layers=layers, loop=(start, stop, times))
+                   layers=layers, loop=parse_loop(raw, len(layers)))
 
     def order(self) -> list:
         """Layer numbers in the order in which they run."""
-        start, stop, times = self.loop
-        return [*range(start), *list(range(start, stop)) * times, *range(stop, len(self.layers))]
+        return looped(self.loop, len(self.layers))
 
 
 @register_model("Sozarax")

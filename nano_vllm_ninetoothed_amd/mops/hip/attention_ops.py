@@ -49,9 +49,11 @@ def attention_prepare(qkv, q_weight, k_weight, eps, positions, slot_mapping, k_p
 
 
 @register_hip_op
-def rotary_prepare(qkv, positions, slot_mapping, k_pages, v_pages, heads, kv_heads, dim, vdim, cos_sin=None, q_weight=None, k_weight=None, eps=0.0):
-    """qkv rows [q | k | v | anything]: an RMS norm per head on q and k where there are weights [dim], their first cos_sin.shape[1]
-    elements turned by the token's position, k and v into their pages.  Returns q [tokens, heads, padded dim]."""
+def rotary_prepare(qkv, positions, slot_mapping, k_pages, v_pages, heads, kv_heads, dim, vdim, cos_sin=None, q_weight=None, k_weight=None, eps=0.0,
+                   bias=None, neighbours=False):
+    """qkv rows [q | k | v | anything], plus bias over [q | k | v]: an RMS norm per head on q and k where there are weights [dim], their
+    first cos_sin.shape[1] elements turned by the token's position (pairs half of that apart, or neighbours), k and v into their pages.
+    Returns q [tokens, heads, padded dim]."""
     a = _capi.RotaryPrepare()
     a.dtype = _dtype("qkv", qkv)
     tokens = qkv.shape[0]
@@ -70,7 +72,9 @@ def rotary_prepare(qkv, positions, slot_mapping, k_pages, v_pages, heads, kv_hea
     a.q, a.k_pages, a.v_pages = q.data_ptr(), _pages("k_pages", k_pages, kv_heads, dim, qkv.dtype), _pages("v_pages", v_pages, kv_heads, vdim, qkv.dtype)
     _require(k_pages.shape[:2] == v_pages.shape[:2], "k_pages and v_pages must have the same blocks")
     a.num_slots, a.tokens, a.heads, a.kv_heads, a.dim, a.vdim = k_pages.shape[0] * k_pages.shape[1], tokens, heads, kv_heads, dim, vdim
-    a.eps = float(eps)
+    a.eps, a.neighbours = float(eps), 1 if neighbours else 0
+    if bias is not None:
+        a.bias = _flat("bias", bias, (heads + kv_heads) * dim + kv_heads * vdim, qkv.dtype)
     st = _capi.load().mops_hip_rotary_prepare(byref(a), _stream(qkv))
     _capi.check("mops_hip_rotary_prepare", st)
     return q
@@ -81,25 +85,31 @@ class Scores:
     """What a design does to the scores of attention beside scaling them, and what a token sees.  Zeros and None leave it out.
     softcap: softcap tanh(score / softcap).  window: the last `window` tokens; chunk: the token's chunk of a sequence cut from its start;
     both up to the token itself, and the first keep_first tokens with them.  sinks (float32 [heads]): logarithms of one more term of
-    the denominator."""
+    the denominator.  log_distance (two of float32 [heads]): rate ln(1 + step distance) is taken off.  weight_bias (float32 [heads]): no
+    softmax, a key counts with sigmoid(score + weight_bias)."""
     softcap: float = 0.0
     window: int = 0
     chunk: int = 0
     keep_first: int = 0
     sinks: torch.Tensor = None
+    log_distance: tuple = None
+    weight_bias: torch.Tensor = None
 
 
 WIDEST = 1 << 30      # more than any sequence holds: a window or chunk without effect
 
 
-def _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes, row_seq, out, own_rows=True, scores=None, gate=None):
+def _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes, row_seq, out, own_rows=True, scores=None, gate=None,
+                 out_scale=1.0):
     code = _dtype("q", q)
     rows, heads, dp = q.shape
     kv_heads = k_pages.shape[2]
     _require(q.is_contiguous() and dp == padded(dim), "q must be contiguous [rows, heads, padded dim]")
     _require(heads % kv_heads == 0, "query heads must be a multiple of kv heads")
-    _require(out.is_cuda and out.is_contiguous() and out.dtype == q.dtype and out.numel() == rows * heads * vdim, "out must be contiguous [rows, heads, vdim]")
+    out = out.view(rows, heads * vdim) if out.dim() == 3 else out
     a = _capi.BiasedAttention()
+    a.out_stride, a.out_scale = _rows("out", out, heads * vdim, q.dtype), float(out_scale)
+    _require(out.shape[0] == rows, "out must have as many rows as q")
     a.q, a.k_pages, a.v_pages = q.data_ptr(), _pages("k_pages", k_pages, kv_heads, dim, q.dtype), _pages("v_pages", v_pages, kv_heads, vdim, q.dtype)
     _require(k_pages.shape[:2] == v_pages.shape[:2], "k_pages and v_pages must have the same blocks")
     if slopes is not None:
@@ -119,20 +129,27 @@ def _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scal
         a.window, a.chunk, a.keep_first = (min(int(n), WIDEST) for n in (scores.window, scores.chunk, scores.keep_first))
         if scores.sinks is not None:
             a.sinks = _flat("sinks", scores.sinks, heads, torch.float32)
+        if scores.log_distance is not None:
+            a.log_rate, a.log_step = (_flat("log_distance", x, heads, torch.float32) for x in scores.log_distance)
+        if scores.weight_bias is not None:
+            a.weight_bias = _flat("weight_bias", scores.weight_bias, heads, torch.float32)
     if gate is not None:
-        a.gate, a.gate_stride = gate.data_ptr(), _rows("gate", gate, heads, q.dtype)
-        _require(gate.shape[0] == rows, "gate must be [rows, heads]")
+        a.gate_each = 1 if gate.shape[1] != heads else 0      # values of one element: the two are the same
+        a.gate, a.gate_stride = gate.data_ptr(), _rows("gate", gate, heads * vdim if a.gate_each else heads, q.dtype)
+        _require(gate.shape[0] == rows, "gate must be [rows, heads] or [rows, heads * vdim]")
     return a
 
 
 @register_hip_op
-def biased_attention_rows(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes=None, row_seq=None, scores=None, gate=None, out=None):
+def biased_attention_rows(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes=None, row_seq=None, scores=None, gate=None, out=None,
+                          out_scale=1.0):
     """Attention of single query rows against the pages: row r sees the first context_lens[r] tokens of block table row row_seq[r]
     (r itself without row_seq), or of these what scores lets it see; score = q.k scale - slope (distance), or capped.  gate [rows,
-    heads]: the result is multiplied by its sigmoid.  Returns [rows, heads, vdim].  The plain form: any size, bf16 or float32."""
+    heads] or [rows, heads * vdim]: the result is multiplied by its sigmoid, and by out_scale.  out: [rows, heads, vdim], or rows [rows,
+    heads * vdim] with a stride.  Returns [rows, heads, vdim].  The plain form: any size, bf16 or float32."""
     if out is None:
         out = torch.empty((q.shape[0], q.shape[1], vdim), dtype=q.dtype, device=q.device)
-    a = _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes, row_seq, out, scores=scores, gate=gate)
+    a = _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes, row_seq, out, scores=scores, gate=gate, out_scale=out_scale)
     st = _capi.load().mops_hip_biased_attention_rows(byref(a), _stream(q))
     _capi.check("mops_hip_biased_attention_rows", st)
     return out
@@ -144,11 +161,12 @@ def biased_matrix_covers(dtype, dim: int, vdim: int, block_size: int) -> bool:
 
 
 @register_hip_op
-def biased_decode(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes=None, row_seq=None, out=None, scores=None, gate=None):
+def biased_decode(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes=None, row_seq=None, out=None, scores=None, gate=None,
+                  out_scale=1.0):
     """biased_attention_rows on the matrix cores (sizes: biased_matrix_covers)."""
     if out is None:
         out = torch.empty((q.shape[0], q.shape[1], vdim), dtype=q.dtype, device=q.device)
-    a = _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes, row_seq, out, scores=scores, gate=gate)
+    a = _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes, row_seq, out, scores=scores, gate=gate, out_scale=out_scale)
     lib = _capi.load()
     ws = torch.empty(max(16, lib.mops_hip_biased_decode_workspace_bytes(a.rows, a.heads, a.kv_heads, dim, vdim)), dtype=torch.uint8, device=q.device)
     st = lib.mops_hip_biased_decode(byref(a), ws.data_ptr(), ws.numel(), _stream(q))
@@ -170,12 +188,13 @@ def biased_prefill_tiles(counts, starts, first_token: int, first_seq: int):
 
 
 @register_hip_op
-def biased_prefill(q, k_pages, v_pages, dim, vdim, tiles, block_table, scale, context_lens, slopes=None, out=None, scores=None, gate=None):
+def biased_prefill(q, k_pages, v_pages, dim, vdim, tiles, block_table, scale, context_lens, slopes=None, out=None, scores=None, gate=None,
+                   out_scale=1.0):
     """Causal attention of long portions, whose keys and values are in the pages already: tiles [n, 5] is the int32 device copy of
     biased_prefill_tiles.  context_lens: of every row.  Writes the portions' rows of out [rows, heads, vdim]."""
     if out is None:
         out = torch.empty((q.shape[0], q.shape[1], vdim), dtype=q.dtype, device=q.device)
-    a = _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes, None, out, own_rows=False, scores=scores, gate=gate)
+    a = _biased_args(q, k_pages, v_pages, dim, vdim, context_lens, block_table, scale, slopes, None, out, own_rows=False, scores=scores, gate=gate, out_scale=out_scale)
     n = tiles.shape[0]
     st = _capi.load().mops_hip_biased_prefill(byref(a), _flat("tiles", tiles, 5 * n, torch.int32), n, _stream(q))
     _capi.check("mops_hip_biased_prefill", st)

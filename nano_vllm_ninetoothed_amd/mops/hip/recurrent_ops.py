@@ -5,6 +5,7 @@ exceptions, outputs come from the torch allocator, everything runs on the curren
 from __future__ import annotations
 
 from ctypes import byref
+from dataclasses import dataclass
 
 import torch
 
@@ -39,16 +40,19 @@ def _flat(name: str, t: torch.Tensor, n: int, dtype: torch.dtype) -> int:
 
 
 @register_hip_op
-def embed_residual(ids: torch.Tensor, table: torch.Tensor, scale: float = 1.0, need_act: bool = True):
-    """Scaled embedding rows as (float32 residual, activation copy in the table's dtype or None)."""
+def embed_residual(ids: torch.Tensor, table: torch.Tensor, scale: float = 1.0, need_act: bool = True, act=None):
+    """Scaled embedding rows as (float32 residual, activation copy in the table's dtype or None); act: rows for the copy."""
     code = _dtype("table", table)
     _require(table.dim() == 2 and table.stride(1) == 1, "table must be [vocab, width] with contiguous rows")
     _require(ids.is_cuda and ids.dtype == torch.int64 and ids.dim() == 1 and ids.is_contiguous(), "ids must be a contiguous int64 GPU vector")
     n, (vocab, width) = ids.numel(), table.shape
     residual = torch.empty((n, width), dtype=torch.float32, device=table.device)
-    act = torch.empty((n, width), dtype=table.dtype, device=table.device) if need_act else None
+    if act is None and need_act:
+        act = torch.empty((n, width), dtype=table.dtype, device=table.device)
+    act_stride = width if act is None else _rows("act", act, width, table.dtype)
+    _require(act is None or act.shape[0] == n, "act must have one row per id")
     st = _capi.load().mops_hip_embed_residual(ids.data_ptr(), table.data_ptr(), table.stride(0), code, float(scale), residual.data_ptr(),
-                                              None if act is None else act.data_ptr(), n, vocab, width, _stream(table))
+                                              None if act is None else act.data_ptr(), act_stride, n, vocab, width, _stream(table))
     _capi.check("mops_hip_embed_residual", st)
     return residual, act
 
@@ -112,6 +116,34 @@ def add_norm_norm(residual: torch.Tensor, y: torch.Tensor, w_out: torch.Tensor, 
 
 
 @register_hip_op
+def add_norm(residual: torch.Tensor, y=None, shift=None, replace: bool = False, weight=None, bias=None, eps: float = 0.0, center: bool = False, out=None,
+             dtype=None):
+    """residual += y + shift in place (replace: = y + shift; shift: float32 vector); returns norm(residual) * weight + bias, or the residual
+    without weight, in the dtype of `out` (rows to fill), of weight or `dtype`.  center: layer norms instead of RMS norms."""
+    rows, n = residual.shape
+    dtype = out.dtype if out is not None else (weight.dtype if weight is not None else dtype)
+    if out is None:
+        out = torch.empty((rows, n), dtype=dtype, device=residual.device)
+    a = _capi.AddNorm()
+    a.residual, a.rows, a.n = _flat("residual", residual, rows * n, torch.float32), rows, n
+    if y is not None:
+        a.y, a.y_stride = y.data_ptr(), _rows("y", y, n, dtype)
+        _require(y.shape[0] == rows, "y must have as many rows as the residual")
+    if shift is not None:
+        a.shift = _flat("shift", shift, n, torch.float32)
+    if weight is not None:
+        a.w = _flat("weight", weight, n, dtype)
+    if bias is not None:
+        a.b = _flat("bias", bias, n, dtype)
+    a.out, a.out_stride = out.data_ptr(), _rows("out", out, n, dtype)
+    _require(out.shape[0] == rows, "out must have as many rows as the residual")
+    a.eps, a.replace, a.center, a.dtype = float(eps), 1 if replace else 0, 1 if center else 0, _dtype("out", out)
+    st = _capi.load().mops_hip_add_norm(byref(a), _stream(residual))
+    _capi.check("mops_hip_add_norm", st)
+    return out
+
+
+@register_hip_op
 def layer_norm_f32(x: torch.Tensor, weight: torch.Tensor, eps: float):
     """(x - mean) / sqrt(variance + eps) * weight of float32 rows, in the weight's dtype."""
     code = _dtype("weight", weight)
@@ -136,45 +168,58 @@ def rms_norm_f32(x: torch.Tensor, weight: torch.Tensor, eps: float, weight_offse
 
 
 @register_hip_op
-def gated_group_norm(y: torch.Tensor, gate: torch.Tensor, groups: int, eps: float, weight=None, gate_first: bool = False):
-    """rms over `groups` equal parts of every row, multiplied by silu(gate) before (gate_first) or after the division."""
+def gated_group_norm(y: torch.Tensor, gate: torch.Tensor, groups: int, eps: float, weight=None, gate_first: bool = False, activation: str = "silu",
+                     scale: float = 1.0, out=None):
+    """rms over `groups` equal parts of every row, multiplied by silu(gate), or its sigmoid, before (gate_first) or after the division.
+    weight: for the whole row, or for one part and shared by all.  Everything times scale."""
     code = _dtype("y", y)
     rows, n = y.shape
     _require(groups > 0 and n % groups == 0, "the row must divide into the groups")
     ys, gs = _rows("y", y, n, y.dtype), _rows("gate", gate, n, y.dtype)
     _require(gate.shape[0] == rows, "gate must have as many rows as y")
-    out = torch.empty((rows, n), dtype=y.dtype, device=y.device)
-    st = _capi.load().mops_hip_gated_group_norm(y.data_ptr(), ys, gate.data_ptr(), gs, None if weight is None else _flat("weight", weight, n, y.dtype),
-                                                float(eps), 1 if gate_first else 0, out.data_ptr(), code, rows, groups, n // groups, _stream(y))
+    _require(activation in ("silu", "sigmoid"), "activation must be silu or sigmoid")
+    if out is None:
+        out = torch.empty((rows, n), dtype=y.dtype, device=y.device)
+    _require(out.shape[0] == rows, "out must have as many rows as y")
+    shared = weight is not None and weight.numel() != n
+    st = _capi.load().mops_hip_gated_group_norm(y.data_ptr(), ys, gate.data_ptr(), gs,
+                                                None if weight is None else _flat("weight", weight, n // groups if shared else n, y.dtype), 1 if shared else 0,
+                                                float(eps), 1 if gate_first else 0, 1 if activation == "sigmoid" else 0, float(scale), out.data_ptr(),
+                                                _rows("out", out, n, y.dtype), code, rows, groups, n // groups, _stream(y))
     _capi.check("mops_hip_gated_group_norm", st)
     return out
 
 
+def _glu(name, gate, up, out, *constants):
+    code = _dtype("gate", gate)
+    rows, n = gate.shape
+    gs, us = _rows("gate", gate, n, gate.dtype), _rows("up", up, n, gate.dtype)
+    _require(up.shape[0] == rows, "gate and up must have the same shape")
+    if out is None:
+        out = torch.empty((rows, n), dtype=gate.dtype, device=gate.device)
+    _require(out.shape[0] == rows, "out must have as many rows as gate")
+    st = getattr(_capi.load(), name)(gate.data_ptr(), gs, up.data_ptr(), us, out.data_ptr(), _rows("out", out, n, gate.dtype), code, rows, n, *constants,
+                                     _stream(gate))
+    _capi.check(name, st)
+    return out
+
+
 @register_hip_op
-def clamped_glu(gate: torch.Tensor, up: torch.Tensor, limit: float, alpha: float = 1.702):
+def clamped_glu(gate: torch.Tensor, up: torch.Tensor, limit: float, alpha: float = 1.702, out=None):
     """g * sigmoid(alpha g) * (u + 1) with g = min(gate, limit) and u = clamp(up, -limit, limit)."""
-    code = _dtype("gate", gate)
-    rows, n = gate.shape
-    gs, us = _rows("gate", gate, n, gate.dtype), _rows("up", up, n, gate.dtype)
-    _require(up.shape[0] == rows, "gate and up must have the same shape")
-    out = torch.empty((rows, n), dtype=gate.dtype, device=gate.device)
-    st = _capi.load().mops_hip_clamped_glu(gate.data_ptr(), gs, up.data_ptr(), us, out.data_ptr(), code, rows, n, float(alpha), float(limit),
-                                           _stream(gate))
-    _capi.check("mops_hip_clamped_glu", st)
-    return out
+    return _glu("mops_hip_clamped_glu", gate, up, out, float(alpha), float(limit))
 
 
 @register_hip_op
-def gelu_glu(gate: torch.Tensor, up: torch.Tensor):
+def gelu_glu(gate: torch.Tensor, up: torch.Tensor, out=None):
     """gelu(gate) * up, gelu in its tanh form."""
-    code = _dtype("gate", gate)
-    rows, n = gate.shape
-    gs, us = _rows("gate", gate, n, gate.dtype), _rows("up", up, n, gate.dtype)
-    _require(up.shape[0] == rows, "gate and up must have the same shape")
-    out = torch.empty((rows, n), dtype=gate.dtype, device=gate.device)
-    st = _capi.load().mops_hip_gelu_glu(gate.data_ptr(), gs, up.data_ptr(), us, out.data_ptr(), code, rows, n, _stream(gate))
-    _capi.check("mops_hip_gelu_glu", st)
-    return out
+    return _glu("mops_hip_gelu_glu", gate, up, out)
+
+
+@register_hip_op
+def relu_glu(gate: torch.Tensor, up: torch.Tensor, out=None):
+    """max(gate, 0) * up"""
+    return _glu("mops_hip_relu_glu", gate, up, out)
 
 
 @register_hip_op
@@ -188,20 +233,38 @@ def squared_relu(x: torch.Tensor):
     return out
 
 
+def matrix_memory_copies(vd: int) -> int:
+    """Rows behind the vd value rows of a head's state that hold a matrix memory's normalizer, and copies of its running maximum."""
+    return _capi.load().mops_hip_matrix_memory_copies(vd)
+
+
+@dataclass(frozen=True)
+class MemoryGates:
+    """A matrix memory's gates: projections [tokens, heads] in front of bias and cap, biases (float32 [heads]), the cap, and the running
+    maximum of every slot (float32 [slots, heads, copies])."""
+    input: torch.Tensor
+    forget: torch.Tensor
+    input_bias: torch.Tensor
+    forget_bias: torch.Tensor
+    cap: float
+    top: torch.Tensor
+
+
 def recurrence_state_pitch(d: int) -> int:
     """Row pitch (elements) of the recurrent state [slots, heads, vd, pitch]."""
     return _capi.load().mops_hip_recurrence_state_pitch(d)
 
 
 def _recurrence_args(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, *, cu_seqlens=None, decay=None, log_decay=None, dt=None,
-                     dt_bias=None, neg_a=None, skip=None, cos_sin=None, k_scale=1.0, conv=None, channel_decay=None, bonus=None):
+                     dt_bias=None, neg_a=None, skip=None, cos_sin=None, k_scale=1.0, conv=None, channel_decay=None, bonus=None, gates=None):
     code = _dtype("v", v)
     tokens = v.shape[0]
     batch = state_slots.numel()
     r = _capi.Recurrence()
     _require(heads > 0 and groups > 0 and heads % groups == 0, "heads must be a multiple of groups")
+    copies = 0 if gates is None else matrix_memory_copies(vd)
     _require(state.is_cuda and state.dtype == torch.float32 and state.is_contiguous() and state.dim() == 4
-             and tuple(state.shape[1:]) == (heads, vd, recurrence_state_pitch(d)), "state must be float32 [slots, heads, vd, pitch]")
+             and tuple(state.shape[1:]) == (heads, vd + copies, recurrence_state_pitch(d)), "state must be float32 [slots, heads, vd (+ copies), pitch]")
     r.q_stride, r.k_stride = _rows("q", q, groups * d, v.dtype), _rows("k", k, groups * d, v.dtype)
     r.v_stride, r.out_stride = _rows("v", v, heads * vd, v.dtype), _rows("out", out, heads * vd, v.dtype)
     r.q, r.k, r.v, r.out = q.data_ptr(), k.data_ptr(), v.data_ptr(), out.data_ptr()
@@ -212,8 +275,14 @@ def _recurrence_args(q, k, v, out, state, state_slots, starts, heads, groups, d,
         _require(tokens == batch, "without cu_seqlens every sequence brings one token")
     else:
         r.cu_seqlens = _flat("cu_seqlens", cu_seqlens, batch + 1, torch.int32)
-    _require(sum(x is not None for x in (decay, dt, channel_decay)) == 1, "give a constant decay, time steps or a decay per channel")
-    if channel_decay is not None:
+    _require(sum(x is not None for x in (decay, dt, channel_decay, gates)) == 1, "give a constant decay, time steps, a decay per channel or gates")
+    if gates is not None:
+        r.input_gate, r.forget_gate, r.gate_stride = gates.input.data_ptr(), gates.forget.data_ptr(), _rows("input gate", gates.input, heads, v.dtype)
+        _require(_rows("forget gate", gates.forget, heads, v.dtype) == r.gate_stride and gates.input.shape[0] == gates.forget.shape[0] == tokens,
+                 "the gates must have one row per token and the same stride")
+        r.input_bias, r.forget_bias = _flat("input bias", gates.input_bias, heads, torch.float32), _flat("forget bias", gates.forget_bias, heads, torch.float32)
+        r.top, r.gate_cap = _flat("top", gates.top, state.shape[0] * heads * copies, torch.float32), float(gates.cap)
+    elif channel_decay is not None:
         r.channel_decay, r.channel_decay_stride = channel_decay.data_ptr(), _rows("channel_decay", channel_decay, heads * d, torch.float32)
         _require(channel_decay.shape[0] == tokens, "channel_decay must have one row per token")
         r.bonus = _flat("bonus", bonus, heads * d, torch.float32)
@@ -245,11 +314,52 @@ def _recurrence_args(q, k, v, out, state, state_slots, starts, heads, groups, d,
 def decayed_recurrence(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, **options):
     """S <- a S + k (s v)^T, o = S^T q + skip v, token by token with the state of state_slots[b] in float32 (layout and options:
     mops_hip_recurrence in include/mops_hip.h).  Options: cu_seqlens (None: one token per sequence), decay | dt + dt_bias +
-    neg_a | channel_decay + bonus, skip, cos_sin (rotates q and k), k_scale, conv = (weight [taps, channels] float32, bias, ring, (q, k, v channel
+    neg_a | channel_decay + bonus | gates (a matrix memory), skip, cos_sin (rotates q and k), k_scale, conv = (weight [taps, channels] float32, bias, ring, (q, k, v channel
     offsets)).  Writes `out` and the state in place."""
     r = _recurrence_args(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, **options)
     st = _capi.load().mops_hip_decayed_recurrence(byref(r), _stream(v))
     _capi.check("mops_hip_decayed_recurrence", st)
+    return out
+
+
+def _delta_args(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, log_decay, beta, q_scale, unit_eps, cu_seqlens=None, conv=None):
+    a = _capi.Delta()
+    a.dtype = _dtype("v", v)
+    tokens, batch = v.shape[0], state_slots.numel()
+    _require(heads > 0 and groups > 0 and heads % groups == 0, "heads must be a multiple of groups")
+    _require(state.is_cuda and state.dtype == torch.float32 and state.is_contiguous() and state.dim() == 4
+             and tuple(state.shape[1:]) == (heads, vd, recurrence_state_pitch(d)), "state must be float32 [slots, heads, vd, pitch]")
+    a.q_stride, a.k_stride = _rows("q", q, groups * d, v.dtype), _rows("k", k, groups * d, v.dtype)
+    a.v_stride, a.out_stride = _rows("v", v, heads * vd, v.dtype), _rows("out", out, heads * vd, v.dtype)
+    a.q, a.k, a.v, a.out = q.data_ptr(), k.data_ptr(), v.data_ptr(), out.data_ptr()
+    a.log_decay, a.log_decay_stride = log_decay.data_ptr(), _rows("log_decay", log_decay, heads * d, torch.float32)
+    a.beta, a.beta_stride = beta.data_ptr(), _rows("beta", beta, heads, v.dtype)
+    _require(all(x.shape[0] == tokens for x in (q, k, out, log_decay, beta)), "all inputs must have the same number of tokens")
+    a.state, a.num_slots = state.data_ptr(), state.shape[0]
+    a.state_slots, a.starts = _flat("state_slots", state_slots, batch, torch.int32), _flat("starts", starts, batch, torch.int32)
+    if cu_seqlens is None:
+        _require(tokens == batch, "without cu_seqlens every sequence brings one token")
+    else:
+        a.cu_seqlens = _flat("cu_seqlens", cu_seqlens, batch + 1, torch.int32)
+    if conv is not None:
+        weight, ring, (a.q_channel, a.k_channel, a.v_channel) = conv
+        a.taps, a.channels = weight.shape
+        a.conv_weight = _flat("conv weight", weight, weight.numel(), torch.float32)
+        a.conv_ring = _flat("conv ring", ring, state.shape[0] * weight.numel(), v.dtype)
+    a.batch, a.heads, a.groups, a.d, a.vd = batch, heads, groups, d, vd
+    a.q_scale, a.unit_eps = float(q_scale), float(unit_eps)
+    return a
+
+
+@register_hip_op
+def delta_rule(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, **options):
+    """The gated delta rule token by token, S <- exp(log_decay) S, S <- S + k (sigmoid(beta) (v - S^T k))^T, o = S^T q, with q and k as unit
+    vectors and the state of state_slots[b] in float32 (mops_hip_delta in include/mops_hip.h).  Options: log_decay (float32 [tokens, heads *
+    d]), beta [tokens, heads], q_scale, unit_eps, cu_seqlens (None: one token per sequence), conv = (weight [taps, channels] float32, ring,
+    (q, k, v channel offsets)).  Writes `out` and the state in place."""
+    a = _delta_args(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, **options)
+    st = _capi.load().mops_hip_delta_rule(byref(a), _stream(v))
+    _capi.check("mops_hip_delta_rule", st)
     return out
 
 
@@ -321,7 +431,7 @@ def short_conv(x, weight, bias, ring, token_seq, cu_seqlens, starts, state_slots
     _require(ring.dim() == 3 and ring.shape[1:] == (taps, channels), "ring must be [slots, taps, channels]")
     out = torch.empty((tokens, channels), dtype=x.dtype, device=x.device)
     st = _capi.load().mops_hip_short_conv(x.data_ptr(), stride, _flat("weight", weight, taps * channels, torch.float32),
-                                          _flat("bias", bias, channels, torch.float32), _flat("ring", ring, ring.numel(), x.dtype), ring.shape[0],
+                                          None if bias is None else _flat("bias", bias, channels, torch.float32), _flat("ring", ring, ring.numel(), x.dtype), ring.shape[0],
                                           _flat("token_seq", token_seq, tokens, torch.int32), _flat("cu_seqlens", cu_seqlens, batch + 1, torch.int32),
                                           _flat("starts", starts, batch, torch.int32), _flat("state_slots", state_slots, batch, torch.int32),
                                           out.data_ptr(), code, tokens, channels, taps, _stream(x))
@@ -366,13 +476,15 @@ def token_mix(x, mu, before, starts, state_slots, token_seq=None, cu_seqlens=Non
 
 
 @register_hip_op
-def low_rank_decay(z, w2, w0):
-    """-exp(w2 tanh(z) + w0), float32: the logarithm of a decay per channel.  w2 in z's dtype, w0 float32."""
+def low_rank_decay(z, w2, w0, rate=None):
+    """-exp(w2 tanh(z) + w0), or with a rate per head (float32) rate softplus(w2 z + w0); float32: the logarithm of a decay per channel.  w2
+    in z's dtype, w0 float32."""
     code = _dtype("z", z)
     tokens, (channels, rank) = z.shape[0], w2.shape
     out = torch.empty((tokens, channels), dtype=torch.float32, device=z.device)
     st = _capi.load().mops_hip_low_rank_decay(z.data_ptr(), _rows("z", z, rank, z.dtype), _flat("w2", w2, channels * rank, z.dtype),
-                                              _flat("w0", w0, channels, torch.float32), out.data_ptr(), code, tokens, channels, rank, _stream(z))
+                                              _flat("w0", w0, channels, torch.float32), None if rate is None else _flat("rate", rate, rate.numel(), torch.float32),
+                                              0 if rate is None else channels // rate.numel(), out.data_ptr(), code, tokens, channels, rank, _stream(z))
     _capi.check("mops_hip_low_rank_decay", st)
     return out
 

@@ -193,7 +193,7 @@ def test_argument_validation_on_the_host():
     assert lib.mops_hip_layer_norm_f32(A, A, 1e-5, A, 0, 4, 64, None) == -1                       # out aliases x
     assert lib.mops_hip_layer_norm_f32(None, None, 1e-5, None, 0, 0, 64, None) == 0
     assert lib.mops_hip_add_norm_norm(A, 2 * A, 64, 1, A, A, A, 1e-5, 1, A, 0, 4, 64, None) == -1  # out aliases extra
-    assert lib.mops_hip_gelu_glu(A, 32, A, 64, A, 0, 4, 64, None) == -1
+    assert lib.mops_hip_gelu_glu(A, 32, A, 64, A, 64, 0, 4, 64, None) == -1
     e = _capi.EmbedPairs()
     e.ids = e.table = e.pairs = e.residual = e.before = e.starts = e.state_slots = A
     e.table_stride = e.pairs_stride = e.width = 64

@@ -210,8 +210,8 @@ def test_argument_validation_on_the_host():
     assert lib.mops_hip_token_mix(A, 64, A, 5, A, 4, A, None, A, A, A, 0, 3, 64, None) == -1      # token_seq without cu_seqlens
     assert lib.mops_hip_token_mix(A, 32, A, 5, A, 4, None, None, A, A, A, 0, 3, 64, None) == -1   # rows overlap
     assert lib.mops_hip_token_mix(None, 64, None, 5, None, 4, None, None, None, None, None, 0, 0, 64, None) == 0
-    assert lib.mops_hip_low_rank_decay(A, 8, A, A, A, 0, 3, 64, 16, None) == -1
-    assert lib.mops_hip_low_rank_decay(A, 5000, A, A, A, 0, 3, 64, 5000, None) == -2
+    assert lib.mops_hip_low_rank_decay(A, 8, A, A, None, 0, A, 0, 3, 64, 16, None) == -1
+    assert lib.mops_hip_low_rank_decay(A, 5000, A, A, None, 0, A, 0, 3, 64, 5000, None) == -2
     assert lib.mops_hip_add_norm_norm(A, A, 64, 1, None, A, A, 1e-5, 0, A, 0, 4, 64, None) == -1           # out aliases y
     assert lib.mops_hip_squared_relu(A, 8, A, 0, 4, 64, None) == -1
     m = _capi.Moe()
