@@ -465,10 +465,11 @@ typedef struct {
 } mops_hip_recurrence;
 /*
  * Matrix memory (input_gate given, in the place of a decay): gates are `dtype` [tokens, heads] with rows gate_stride apart, biases float
- * [heads]; state [num_slots, heads, vd + copies, pitch] and top float [num_slots, heads, copies], copies = mops_hip_matrix_memory_copies.
+ * [heads]; k_scale multiplies q; state [num_slots, heads, vd + copies, pitch] and top float [num_slots, heads, copies], copies = mops_hip_matrix_memory_copies.
  * The chunked form takes the gates from mops_hip_matrix_memory_gates instead: log_keep, input_scale and least, float [tokens, heads].
  */
 int64_t mops_hip_matrix_memory_copies(int64_t vd);
+int mops_hip_matrix_memory_gates(const mops_hip_recurrence* r, float* log_keep, float* input_scale, float* least, void* stream);
 int64_t mops_hip_recurrence_state_pitch(int64_t d);
 int mops_hip_decayed_recurrence(const mops_hip_recurrence* r, void* stream);
 
@@ -518,6 +519,16 @@ typedef struct {
   int dtype;
 } mops_hip_delta;
 int mops_hip_delta_rule(const mops_hip_delta* a, void* stream);
+
+/*
+ * The same for portions of many tokens, 16 tokens at a time on the matrix cores (csrc/delta_chunks.hip): bf16, d <= 256, cu_seqlens given,
+ * no convolution; a decay below 2^-28 counts as 2^-28.  chunks: int32 [num_chunks][2] = (first token, tokens <= 16): every sequence cut
+ * from its first token on, in order; seq_chunks: int32 [batch + 1] bounds each sequence's.  workspace: device scratch of at least
+ * mops_hip_delta_chunks_workspace_bytes(...), private to the call until it completes.
+ */
+int64_t mops_hip_delta_chunks_workspace_bytes(int64_t num_chunks, int64_t heads, int64_t d);
+int mops_hip_delta_chunks(const mops_hip_delta* a, const int32_t* chunks, int64_t num_chunks, const int32_t* seq_chunks, void* workspace,
+                          int64_t workspace_bytes, void* stream);
 
 /*
  * out[t, c] = silu(bias[c] (bias may be NULL) + sum over lags l < taps of weight[taps-1-l, c] * x(position - l)[c]) for packed portions.

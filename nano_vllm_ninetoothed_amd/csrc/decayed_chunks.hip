@@ -16,10 +16,15 @@
 // What the recurrence keeps in 32 bits - the state, the decayed scores, the decayed values - enters a product as the sum of two
 // bf16 numbers (value = hi + lo, 16 significant bits), at the price of a second MFMA.
 //
+// A matrix memory (MEMORY; decays and input scales per token from matrix_memory_gates_kernel) divides by its normalizer: n . q over the
+// state in front of the chunk is a dot product per token on vector units, the rest are sums over the weighted scores.  n is the sum of
+// four parts, one per wave and its sixteen tokens of every chunk.
+//
 // A sequence is one segment when there are enough sequences and heads to fill the chip.  Otherwise it is cut:
 //   pass 1 (STATE_ONLY)  every segment from a zero state: its contribution and its total decay
 //   pass 2 (scan)        the state at the start of every segment, and the final state into the sequence's slot
 //   pass 3               every segment again, with outputs, from its start state
+#include "matrix_memory.h"
 #include "mfma_tiles.h"
 
 namespace mops {
@@ -40,8 +45,10 @@ struct ChunkArgs {
   const float *log_decay, *dt_bias, *neg_a, *skip, *cos_sin;
   int rot;
   int64_t max_positions;
-  float k_scale;
-  float* seg_state;             // [n][heads][vd][pitch], or nullptr: one segment per sequence
+  float k_scale, q_scale;       // of a matrix memory the one is 1, of the others the other
+  const float *log_keep, *input_scale, *least;      // [tokens][heads]
+  int copies;                   // rows of a head's state behind its values: copies of the normalizer, one per 64 values
+  float* seg_state;             // [n][heads][vd + copies][pitch], or nullptr: one segment per sequence
   float* seg_decay;             // [n][heads]: base-2 logarithm of the segment's total decay
 };
 
@@ -54,7 +61,11 @@ struct ChunkShape {
   static constexpr int kK = kChunk * kPitch, kV = kChunk * kVPitch;
   static constexpr int kP = NH * 3 * 2 * kPTile;           // hi and lo of three tiles per head; takes the place of Q
   static constexpr int kQP = kK > kP ? kK : kP;
-  static constexpr int bytes(bool state_only) { return (kK + kV + (state_only ? 0 : kQP)) * 2 + NH * (3 * kChunk + 32) * 4; }
+  // floats of a matrix memory behind the tables: least [64], n . q [64], sums of weighted scores [3][32], n [DP], its parts [4][DP]
+  static constexpr int kMemory = 2 * kChunk + 96 + 5 * DP;
+  static constexpr int bytes(bool state_only, bool memory) {
+    return (kK + kV + (state_only ? 0 : kQP)) * 2 + (NH * (3 * kChunk + 32) + (memory ? kMemory : 0)) * 4;
+  }
 };
 
 // q, k and v rows of a chunk on their way from memory into the LDS tiles: q and k rotated, scaled and rounded to bf16, zeros
@@ -192,7 +203,7 @@ __device__ __forceinline__ void load_tile_scalar(uint16_t* tile, const uint16_t*
   }
 }
 
-template <int DP, int NH, bool STATE_ONLY, bool VEC>
+template <int DP, int NH, bool STATE_ONLY, bool VEC, bool MEMORY>
 __global__ __launch_bounds__(256, DP <= 128 ? 2 : 1) void decayed_chunk_kernel(const ChunkArgs a) {
   using S = ChunkShape<DP, NH>;
   constexpr int kDTiles = DP / 32, kSpan = kColumns / NH, kTilesPerHead = kSpan / 32;
@@ -204,6 +215,11 @@ __global__ __launch_bounds__(256, DP <= 128 ? 2 : 1) void decayed_chunk_kernel(c
   float* const tables = reinterpret_cast<float*>(tq + (STATE_ONLY ? 0 : S::kQP));
   // per head: [64] L, [64] input scale, [64] scale * 2^(L_end - L), [32] scale * 2^(L_31 - L), logarithms to base 2
   auto table = [&](int head) { return tables + head * (3 * kChunk + 32); };
+  float* const least = tables + NH * (3 * kChunk + 32);           // MEMORY
+  float* const n_dot_q = least + kChunk;
+  float* const weight_sums = n_dot_q + kChunk;
+  float* const n_all = weight_sums + 96;
+  float* const n_parts = n_all + DP;
 
   // consecutive workgroups go to different XCDs: give each XCD a contiguous run of items, so that the heads that read the
   // same q and k rows share an L2
@@ -232,6 +248,8 @@ __global__ __launch_bounds__(256, DP <= 128 ? 2 : 1) void decayed_chunk_kernel(c
   const float dt_bias = a.dt ? a.dt_bias[decay_head] : 0.f, neg_a = a.dt ? a.neg_a[decay_head] * kLog2e : 0.f;
   const float skip = a.skip ? a.skip[h] : 0.f;
 
+  const int rows = a.vd + (MEMORY ? a.copies : 0);
+
   // S: tile i, register 4 q + e = row d = 32 i + 8 q + 4 hh + e, column vx + (lane & 31)
   f32x16 st[kDTiles];
   const int v_col = vx + col;
@@ -240,10 +258,10 @@ __global__ __launch_bounds__(256, DP <= 128 ? 2 : 1) void decayed_chunk_kernel(c
   bool load_state = false;
   if (!STATE_ONLY) {
     if (a.seg_state) {
-      gstate = a.seg_state + (((int64_t)seg * a.heads + h) * a.vd + v0) * a.pitch;
+      gstate = a.seg_state + (((int64_t)seg * a.heads + h) * rows + v0) * a.pitch;
       load_state = true;
     } else {
-      gstate = a.state + (((int64_t)slot * a.heads + h) * a.vd + v0) * a.pitch;
+      gstate = a.state + (((int64_t)slot * a.heads + h) * rows + v0) * a.pitch;
       load_state = start > 0;
     }
   }
@@ -262,8 +280,20 @@ __global__ __launch_bounds__(256, DP <= 128 ? 2 : 1) void decayed_chunk_kernel(c
   constexpr int kPairsAll = (kChunk * (DP / 16) + 255) / 256;
   constexpr bool kAhead = VEC && kPairsAll <= 2;          // a whole chunk fits the registers next to the accumulators
   constexpr int kPairs = kPairsAll <= 2 ? kPairsAll : 2;
-  ChunkLoader<DP, STATE_ONLY, kPairs, NH == 1> ld;      // heads that rotate do not share keys
+  ChunkLoader<DP, STATE_ONLY, kPairs, NH == 1 && !MEMORY> ld;      // heads that rotate do not share keys
   uint32_t dt_next = 0;      // this lane's time step of the next chunk, raw
+  float keep_next = 0.f, scale_next = 0.f, least_next = 0.f;      // MEMORY: the same
+  constexpr int kNorm = (DP + 63) / 64;
+  float nn[MEMORY ? kNorm : 1];      // this wave's part of the normalizer: channels lane + 64 j
+  if (MEMORY) {
+#pragma unroll
+    for (int j = 0; j < kNorm; ++j) {
+      const int c = lane + 64 * j;
+      const bool ok = wave == 0 && load_state && c < a.pitch;
+      nn[MEMORY ? j : 0] = ok ? gstate[(int64_t)(a.vd - v0 + v0 / 64) * a.pitch + c] : 0.f;
+      if (c < DP) n_parts[wave * DP + c] = nn[MEMORY ? j : 0];
+    }
+  }
   auto fetch = [&](int t) {
     const int m = t_end - t < kChunk ? t_end - t : kChunk;
     ld.fetch_qk(0, kp + (int64_t)t * a.k_stride, qp + (int64_t)t * a.q_stride, m, a);
@@ -271,7 +301,16 @@ __global__ __launch_bounds__(256, DP <= 128 ? 2 : 1) void decayed_chunk_kernel(c
     ld.fetch_v(vp + (int64_t)t * a.v_stride, m, kSpan, vlen, a);
   };
   auto fetch_dt = [&](int t) {
-    if (a.dt) dt_next = a.dt[(int64_t)(t + lane < t_end ? t + lane : t_end - 1) * a.dt_stride + decay_head];
+    const int64_t row = t + lane < t_end ? t + lane : t_end - 1;
+    if (MEMORY) {
+      if (wave == 0) {
+        keep_next = a.log_keep[row * a.heads + h];
+        scale_next = a.input_scale[row * a.heads + h];
+        least_next = a.least[row * a.heads + h];
+      }
+    } else if (a.dt) {
+      dt_next = a.dt[row * a.dt_stride + decay_head];
+    }
   };
   if (kAhead) fetch(t_begin);
   fetch_dt(t_begin);
@@ -304,11 +343,12 @@ __global__ __launch_bounds__(256, DP <= 128 ? 2 : 1) void decayed_chunk_kernel(c
     }
     if (wave < NH) {     // decays of the chunk: lane = token
       float la = 0.f, s = 0.f, l;
-      if (a.dt) {
+      if (MEMORY || a.dt) {
         if (lane < n) {
-          s = softplus_f32(bf16lo_to_f32(dt_next) + dt_bias);
-          la = neg_a * s;
+          s = MEMORY ? scale_next : softplus_f32(bf16lo_to_f32(dt_next) + dt_bias);
+          la = MEMORY ? keep_next * kLog2e : neg_a * s;
         }
+        if (MEMORY) least[lane] = least_next;
         l = la;
 #pragma unroll
         for (int off = 1; off < 64; off <<= 1) {
@@ -326,6 +366,8 @@ __global__ __launch_bounds__(256, DP <= 128 ? 2 : 1) void decayed_chunk_kernel(c
       t[2 * kChunk + lane] = s * __builtin_amdgcn_exp2f(l_end - l);
       if (lane < 32) t[3 * kChunk + lane] = s * __builtin_amdgcn_exp2f(l_mid - l);
     }
+    if (MEMORY && !STATE_ONLY)
+      for (int c = threadIdx.x; c < DP; c += 256) n_all[c] = (n_parts[c] + n_parts[DP + c]) + (n_parts[2 * DP + c] + n_parts[3 * DP + c]);
     __syncthreads();
     const float* const mine = table(my_head);
     const float l_end = mine[kChunk - 1];
@@ -349,6 +391,7 @@ __global__ __launch_bounds__(256, DP <= 128 ? 2 : 1) void decayed_chunk_kernel(c
           for (int kk = 0; kk < DP / 16; ++kk)
             p = mfma32(tile_row(tk, S::kPitch, j_base + col, 16 * kk + 8 * hh), tile_row(tq, S::kPitch, i_tok, 16 * kk + 8 * hh), p);
           const float l_i = t[i_tok];
+          float sum = 0.f;
           const float e_mid = tile == 1 ? __builtin_amdgcn_exp2f(l_i - t[31]) : 0.f;
 #pragma unroll
           for (int half = 0; half < 2; ++half) {
@@ -363,11 +406,33 @@ __global__ __launch_bounds__(256, DP <= 128 ? 2 : 1) void decayed_chunk_kernel(c
                 // below the diagonal tiles the weight is a product of one factor per token on either side of the tile border
                 const float on = j0 + e <= i_tok ? s_j[e] * __builtin_amdgcn_exp2f(l_i - l_j[e]) : 0.f;
                 w[4 * q4 + e] = p[8 * half + 4 * q4 + e] * (tile == 1 ? m_j[e] * e_mid : on);
+                if (MEMORY) sum += w[4 * q4 + e];
               }
             }
             split8(w, p_hi[m][half], p_lo[m][half]);
           }
+          if (MEMORY) {
+            sum += __shfl_xor(sum, 32, kWave);
+            if (hh == 0) weight_sums[32 * tile + col] = sum;
+          }
         }
+      }
+      if (MEMORY) {      // four lanes per token
+        const int tok = threadIdx.x >> 2, part = threadIdx.x & 3;
+        float dot = 0.f;
+#pragma unroll
+        for (int j = 0; j < DP / 32; ++j) {
+          const int c = 32 * j + 8 * part;
+          const u32x4 qw = load16(tq + tok * S::kPitch + c);
+          const f32x4 n0 = *reinterpret_cast<const f32x4*>(n_all + c), n1 = *reinterpret_cast<const f32x4*>(n_all + c + 4);
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+            dot += (e & 1 ? bf16hi_to_f32(qw[e >> 1]) : bf16lo_to_f32(qw[e >> 1])) * n0[e] +
+                   (e & 1 ? bf16hi_to_f32(qw[2 + (e >> 1)]) : bf16lo_to_f32(qw[2 + (e >> 1)])) * n1[e];
+        }
+        dot += __shfl_xor(dot, 1, kWave);
+        dot += __shfl_xor(dot, 2, kWave);
+        if (part == 0) n_dot_q[tok] = dot * __builtin_amdgcn_exp2f(mine[tok]);
       }
       __builtin_amdgcn_sched_barrier(0);
       // ---- O^T = S^T Q^T, decayed
@@ -434,6 +499,10 @@ __global__ __launch_bounds__(256, DP <= 128 ? 2 : 1) void decayed_chunk_kernel(c
 #pragma unroll
         for (int it = 0; it < 2; ++it) {
           const int i_tok = 32 * it + col;
+          if (MEMORY) {
+            const float sum = it == 0 ? weight_sums[col] : weight_sums[32 + col] + weight_sums[64 + col];
+            o[it] *= a.q_scale / (fmaxf(a.q_scale * fabsf(n_dot_q[i_tok] + sum), least[i_tok]) + kMemoryEps);
+          }
           if (skip != 0.f) {
 #pragma unroll
             for (int q4 = 0; q4 < 4; ++q4)
@@ -492,10 +561,27 @@ __global__ __launch_bounds__(256, DP <= 128 ? 2 : 1) void decayed_chunk_kernel(c
         }
       }
     }
+    if (MEMORY) {
+      const float e_end = __builtin_amdgcn_exp2f(l_end);
+#pragma unroll
+      for (int j = 0; j < kNorm; ++j) {
+        const int c = lane + 64 * j;
+        float sum = nn[MEMORY ? j : 0] * e_end;
+        if (c < DP) {
+#pragma unroll
+          for (int i = 0; i < kChunk / 4; ++i) {
+            const int tok = kChunk / 4 * wave + i;
+            sum += mine[2 * kChunk + tok] * bf16lo_to_f32(tk[tok * S::kPitch + c]);
+          }
+          n_parts[wave * DP + c] = sum;
+        }
+        nn[MEMORY ? j : 0] = sum;
+      }
+    }
   }
 
   float* dst = nullptr;
-  if (STATE_ONLY) dst = a.seg_state + (((int64_t)seg * a.heads + h) * a.vd + v0) * a.pitch;
+  if (STATE_ONLY) dst = a.seg_state + (((int64_t)seg * a.heads + h) * rows + v0) * a.pitch;
   else if (!a.seg_state) dst = gstate;
   if (dst && active) {
 #pragma unroll
@@ -505,6 +591,13 @@ __global__ __launch_bounds__(256, DP <= 128 ? 2 : 1) void decayed_chunk_kernel(c
         if (v_col < vlen && state_d(i, q4) < a.pitch)
           *reinterpret_cast<f32x4*>(dst + v_col * a.pitch + state_d(i, q4)) = f32x4{st[i][4 * q4], st[i][4 * q4 + 1], st[i][4 * q4 + 2], st[i][4 * q4 + 3]};
   }
+  if (MEMORY && dst) {      // this workgroup's copies
+    __syncthreads();
+    for (int c = threadIdx.x; c < a.pitch; c += 256) {
+      const float sum = (n_parts[c] + n_parts[DP + c]) + (n_parts[2 * DP + c] + n_parts[3 * DP + c]);
+      for (int i = v0 / 64; i < v0 / 64 + kColumns / 64 && i < a.copies; ++i) dst[(int64_t)(a.vd - v0 + i) * a.pitch + c] = sum;
+    }
+  }
   if (STATE_ONLY && v0 == 0 && vx == 0 && lane == 0) a.seg_decay[(int64_t)seg * a.heads + h] = total_log;
 }
 
@@ -512,7 +605,7 @@ __global__ __launch_bounds__(256, DP <= 128 ? 2 : 1) void decayed_chunk_kernel(c
 // are consecutive; seq_segments[b], seq_segments[b + 1] bound them.
 __global__ __launch_bounds__(256) void decayed_segment_scan_kernel(const ChunkArgs a, const int32_t* __restrict__ seq_segments) {
   const int h = blockIdx.y, b = blockIdx.z;
-  const int64_t n = (int64_t)a.vd * a.pitch;
+  const int64_t n = (int64_t)(a.vd + a.copies) * a.pitch;
   const int64_t e = ((int64_t)blockIdx.x * 256 + threadIdx.x) * 4;
   const int slot = a.state_slots[b];
   if (e >= n || slot < 0 || slot >= a.num_slots) return;
@@ -530,33 +623,86 @@ __global__ __launch_bounds__(256) void decayed_segment_scan_kernel(const ChunkAr
   *reinterpret_cast<f32x4*>(gs) = s;
 }
 
-template <int DP, int NH, bool VEC>
+template <int DP, int NH, bool VEC, bool MEMORY>
 static int launch_chunks(const ChunkArgs& a, const int32_t* seq_segments, int64_t batch, hipStream_t s) {
   using S = ChunkShape<DP, NH>;
   const int64_t items = (int64_t)a.num_segments * (a.heads / NH) * (NH == 1 ? (a.vd + kColumns - 1) / kColumns : 1);
   const dim3 grid((unsigned)((items + 7) / 8 * 8)), block(256);
-  static const hipError_t lds = hipFuncSetAttribute(reinterpret_cast<const void*>(&decayed_chunk_kernel<DP, NH, false, VEC>),
-                                                    hipFuncAttributeMaxDynamicSharedMemorySize, S::bytes(false));
-  static const hipError_t lds_state = hipFuncSetAttribute(reinterpret_cast<const void*>(&decayed_chunk_kernel<DP, NH, true, VEC>),
-                                                          hipFuncAttributeMaxDynamicSharedMemorySize, S::bytes(true));
+  static const hipError_t lds = hipFuncSetAttribute(reinterpret_cast<const void*>(&decayed_chunk_kernel<DP, NH, false, VEC, MEMORY>),
+                                                    hipFuncAttributeMaxDynamicSharedMemorySize, S::bytes(false, MEMORY));
+  static const hipError_t lds_state = hipFuncSetAttribute(reinterpret_cast<const void*>(&decayed_chunk_kernel<DP, NH, true, VEC, MEMORY>),
+                                                          hipFuncAttributeMaxDynamicSharedMemorySize, S::bytes(true, MEMORY));
   if (lds != hipSuccess) return record_hip_error(lds);
   if (lds_state != hipSuccess) return record_hip_error(lds_state);
   if (a.seg_state) {
-    hipLaunchKernelGGL((decayed_chunk_kernel<DP, NH, true, VEC>), grid, block, S::bytes(true), s, a);
-    const int64_t quads = ((int64_t)a.vd * a.pitch / 4 + 255) / 256;
+    hipLaunchKernelGGL((decayed_chunk_kernel<DP, NH, true, VEC, MEMORY>), grid, block, S::bytes(true, MEMORY), s, a);
+    const int64_t quads = ((int64_t)(a.vd + a.copies) * a.pitch / 4 + 255) / 256;
     hipLaunchKernelGGL(decayed_segment_scan_kernel, dim3((unsigned)quads, (unsigned)a.heads, (unsigned)batch), dim3(256), 0, s, a, seq_segments);
   }
-  hipLaunchKernelGGL((decayed_chunk_kernel<DP, NH, false, VEC>), grid, block, S::bytes(false), s, a);
+  hipLaunchKernelGGL((decayed_chunk_kernel<DP, NH, false, VEC, MEMORY>), grid, block, S::bytes(false, MEMORY), s, a);
   return finish_launch();
 }
 
-template <int NH>
+template <int NH, bool MEMORY = false>
 static int launch_chunks_for(const ChunkArgs& a, const int32_t* seq_segments, int64_t batch, bool vec, hipStream_t s) {
-  if (!vec) return a.d <= 64 ? launch_chunks<64, NH, false>(a, seq_segments, batch, s) : launch_chunks<256, NH, false>(a, seq_segments, batch, s);
-  if (a.d <= 32) return launch_chunks<32, NH, true>(a, seq_segments, batch, s);
-  if (a.d <= 64) return launch_chunks<64, NH, true>(a, seq_segments, batch, s);
-  if (a.d <= 128) return launch_chunks<128, NH, true>(a, seq_segments, batch, s);
-  return launch_chunks<256, NH, true>(a, seq_segments, batch, s);
+  if (!vec) return a.d <= 64 ? launch_chunks<64, NH, false, MEMORY>(a, seq_segments, batch, s) : launch_chunks<256, NH, false, MEMORY>(a, seq_segments, batch, s);
+  if (a.d <= 32) return launch_chunks<32, NH, true, MEMORY>(a, seq_segments, batch, s);
+  if (a.d <= 64) return launch_chunks<64, NH, true, MEMORY>(a, seq_segments, batch, s);
+  if (a.d <= 128) return launch_chunks<128, NH, true, MEMORY>(a, seq_segments, batch, s);
+  return launch_chunks<256, NH, true, MEMORY>(a, seq_segments, batch, s);
+}
+
+// Gates of a matrix memory over the tokens of every (sequence, head), one wave each: with m_t = max(f_t + m_(t-1), i_t) the logarithm of
+// the decay f_t + m_(t-1) - m_t, the input scale exp(i_t - m_t) and exp(-m_t); files the last m in all copies.  m is a scan over pairs (sum
+// of f, greatest i carried to the end), 256 tokens at a time.
+__global__ __launch_bounds__(64) void matrix_memory_gates_kernel(const mops_hip_recurrence r, int copies, float* __restrict__ log_keep,
+                                                                 float* __restrict__ input_scale, float* __restrict__ least) {
+  const int heads = (int)r.heads, h = blockIdx.x % heads, b = blockIdx.x / heads, lane = threadIdx.x;
+  const int slot = r.state_slots[b];
+  if (slot < 0 || slot >= r.num_slots) return;
+  const int t_begin = r.cu_seqlens[b], t_end = r.cu_seqlens[b + 1];
+  float* const top = r.top + ((int64_t)slot * heads + h) * copies;
+  float m = r.starts[b] > 0 ? top[0] : 0.f;
+  const float input_bias = r.input_bias[h], forget_bias = r.forget_bias[h];
+  for (int t0 = t_begin; t0 < t_end; t0 += 256) {
+    float f[4], in[4], sum = 0.f, most = -INFINITY;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int64_t t = t0 + 4 * lane + e;
+      f[e] = 0.f;
+      in[e] = -INFINITY;      // behind the end: changes nothing
+      if (t < t_end) {
+        in[e] = capped_gate(bf16lo_to_f32(((const uint16_t*)r.input_gate)[t * r.gate_stride + h]) + input_bias, r.gate_cap);
+        f[e] = log_sigmoid(capped_gate(bf16lo_to_f32(((const uint16_t*)r.forget_gate)[t * r.gate_stride + h]) + forget_bias, r.gate_cap));
+      }
+      most = fmaxf(most + f[e], in[e]);
+      sum += f[e];
+    }
+#pragma unroll
+    for (int off = 1; off < 64; off <<= 1) {
+      const float sum_up = __shfl_up(sum, off, 64), most_up = __shfl_up(most, off, 64);
+      if (lane >= off) {
+        most = fmaxf(most_up + sum, most);
+        sum += sum_up;
+      }
+    }
+    float before = fmaxf(m + __shfl_up(sum, 1, 64), __shfl_up(most, 1, 64));
+    if (lane == 0) before = m;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const float now = fmaxf(f[e] + before, in[e]);
+      const int64_t at = (int64_t)(t0 + 4 * lane + e) * heads + h;
+      if (t0 + 4 * lane + e < t_end) {
+        log_keep[at] = f[e] + before - now;
+        input_scale[at] = expf(in[e] - now);
+        least[at] = expf(-now);
+      }
+      before = now;
+    }
+    m = __shfl(before, 63, 64);
+  }
+  if (t_end > t_begin)
+    for (int i = lane; i < copies; i += 64) top[i] = m;
 }
 
 // Heads of one workgroup: as many of a q/k group as fill its 128 value columns.
@@ -574,6 +720,20 @@ extern "C" int64_t mops_hip_decayed_chunks_workgroups(int64_t heads, int64_t gro
   return heads / nh * (nh == 1 ? (vd + mops::kColumns - 1) / mops::kColumns : 1);
 }
 
+extern "C" int mops_hip_matrix_memory_gates(const mops_hip_recurrence* r, float* log_keep, float* input_scale, float* least, void* stream) {
+  using namespace mops;
+  if (!r || r->batch < 0) return MOPS_HIP_EINVAL;
+  if (r->batch == 0) return MOPS_HIP_OK;
+  if (r->dtype != MOPS_HIP_BF16) return MOPS_HIP_EUNSUPPORTED;
+  if (!r->input_gate || !r->forget_gate || !r->input_bias || !r->forget_bias || !r->top || !r->state_slots || !r->starts || !r->cu_seqlens || !log_keep ||
+      !input_scale || !least || !(r->gate_cap > 0.f) || r->heads <= 0 || r->vd <= 0 || r->gate_stride < r->heads || r->num_slots <= 0)
+    return MOPS_HIP_EINVAL;
+  if (r->batch * r->heads > 0x7fffffffLL) return MOPS_HIP_EUNSUPPORTED;
+  hipLaunchKernelGGL(matrix_memory_gates_kernel, dim3((unsigned)(r->batch * r->heads)), dim3(64), 0, (hipStream_t)stream, *r,
+                     (int)mops_hip_matrix_memory_copies(r->vd), log_keep, input_scale, least);
+  return finish_launch();
+}
+
 extern "C" int mops_hip_decayed_chunks(const mops_hip_recurrence* r, const int32_t* segments, int64_t num_segments,
                                        const int32_t* seq_segments, float* seg_state, float* seg_decay, void* stream) {
   using namespace mops;
@@ -586,7 +746,8 @@ extern "C" int mops_hip_decayed_chunks(const mops_hip_recurrence* r, const int32
   if (r->d > 256 || r->heads > 65535 || r->batch > 65535 || r->vd > 65536) return MOPS_HIP_EUNSUPPORTED;
   if (r->q_stride < r->groups * r->d || r->k_stride < r->groups * r->d || r->v_stride < r->heads * r->vd || r->out_stride < r->heads * r->vd)
     return MOPS_HIP_EINVAL;
-  if (!r->log_decay == !r->dt) return MOPS_HIP_EINVAL;
+  if ((r->log_decay != nullptr) + (r->dt != nullptr) + (r->log_keep != nullptr) != 1) return MOPS_HIP_EINVAL;
+  if (r->log_keep && (!r->input_scale || !r->least || r->groups != r->heads || r->rot || r->skip)) return MOPS_HIP_EINVAL;
   if (r->dt && (!r->dt_bias || !r->neg_a || r->dt_stride < r->heads)) return MOPS_HIP_EINVAL;
   if (r->rot < 0 || (r->rot & 1) || r->rot > r->d || (r->rot && (!r->cos_sin || r->max_positions <= 0))) return MOPS_HIP_EINVAL;
   if (!aligned16(r->state) || (seg_state && !aligned16(seg_state))) return MOPS_HIP_EALIGN;
@@ -603,11 +764,15 @@ extern "C" int mops_hip_decayed_chunks(const mops_hip_recurrence* r, const int32
   a.heads = (int)r->heads; a.groups = (int)r->groups; a.d = (int)r->d; a.vd = (int)r->vd;
   a.pitch = (int)mops_hip_recurrence_state_pitch(r->d);
   a.log_decay = r->log_decay; a.dt_bias = r->dt_bias; a.neg_a = r->neg_a; a.skip = r->skip; a.cos_sin = r->cos_sin;
-  a.rot = (int)r->rot; a.max_positions = r->max_positions; a.k_scale = r->k_scale;
+  a.rot = (int)r->rot; a.max_positions = r->max_positions;
+  a.k_scale = r->log_keep ? 1.f : r->k_scale; a.q_scale = r->log_keep ? r->k_scale : 1.f;
+  a.log_keep = r->log_keep; a.input_scale = r->input_scale; a.least = r->least;
+  a.copies = r->log_keep ? (int)mops_hip_matrix_memory_copies(r->vd) : 0;
   a.seg_state = seg_state; a.seg_decay = seg_decay;
   const bool vec = r->d % 8 == 0 && r->q_stride % 8 == 0 && r->k_stride % 8 == 0 && aligned16(r->q) && aligned16(r->k) &&
                    (r->rot == 0 || (r->rot % 16 == 0 && aligned16(r->cos_sin))) && r->vd % 8 == 0 && r->v_stride % 8 == 0 &&
                    r->out_stride % 8 == 0 && aligned16(r->v) && aligned16(r->out);
+  if (a.log_keep) return launch_chunks_for<1, true>(a, seq_segments, r->batch, vec, (hipStream_t)stream);
   switch (heads_together(r->heads, r->groups, r->vd, r->rot > 0)) {
     case 4: return launch_chunks_for<4>(a, seq_segments, r->batch, vec, (hipStream_t)stream);
     case 2: return launch_chunks_for<2>(a, seq_segments, r->batch, vec, (hipStream_t)stream);

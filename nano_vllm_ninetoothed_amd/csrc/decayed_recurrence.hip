@@ -11,7 +11,7 @@
 //                 channel: o_t = (S_(t-1) + diag(u) k_t v_t^T)^T q_t
 //   matrix memory a = exp(f + m_(t-1) - m_t), s = exp(i - m_t) with gates i = cap tanh((x + bias) / cap) and f = log sigmoid(cap tanh((y +
 //                 bias) / cap)) per token and head, relative to a running maximum m_t = max(f + m_(t-1), i) that starts at 0; the same
-//                 recurrence with values of one gives n, and o_t = S_t^T q_t / (max(|n_t . q_t|, exp(-m_t)) + 1e-6).  n follows the value
+//                 recurrence with values of one gives n, and o_t = S_t^T q_t / (max(|n_t . q_t|, exp(-m_t)) + 1e-6).  k_scale multiplies q instead.  n follows the value
 //                 rows of a head's state, once per 64 of them, and so does m in `top`: every workgroup has a copy of its own.
 // q and k may be rotated on their first rot dimensions (dimension i with i + rot/2) by the row of a cos/sin table, and k is
 // multiplied by k_scale after that.  Query/key heads may be shared by heads / groups consecutive value heads.
@@ -164,7 +164,8 @@ __global__ __launch_bounds__(256) void decayed_recurrence_kernel(const Recurrenc
           qv = qv * c + to_f32(q[t * a.q_stride + mate]) * sn;
           kv = kv * c + to_f32(k[t * a.k_stride + mate]) * sn;
         }
-        kv *= a.k_scale;
+        if (MEMORY) qv *= a.k_scale;
+        else kv *= a.k_scale;
       }
       sq[i] = qv;
       sk[i] = kv;

@@ -1,0 +1,471 @@
+// The gated delta rule (delta_rule.hip) for portions of many tokens, 16 tokens at a time on the matrix cores (bf16 in, float32
+// accumulation and state).  With L_t = log2 of the product of the decays of a chunk up to token t (per channel), b_t the write strength
+// and S the state in front of the chunk, the writes u_t of a chunk solve a triangular system:
+//
+//   u_t = b_t (v_t - S^T (2^{L_t} k_t) - sum_{j<t} A[t, j] u_j),   A[t, j] = sum_d k_t k_j 2^{L_t - L_j}
+//   o_t = S^T (2^{L_t} q_t) + sum_{j<=t} P[t, j] u_j,              P[t, j] = sum_d q_t k_j 2^{L_t - L_j}
+//   S  <- 2^{L_15} S + sum_j (2^{L_15 - L_j} k_j) u_j^T
+//
+// With T = (1 + diag(b) A)^-1 diag(b) (1 + a strictly lower triangular matrix, inverted by substitution) the writes are
+// U = T V - W S, W = T (2^L k): everything but the products with S is known without S.  Two kernels:
+//
+//   delta_prepare_kernel   a wave per (chunk, head), all chunks in parallel: unit vectors, cumulative decays, A, P, T and W, left in memory
+//                          as the operands of the second kernel's products, lane by lane, so that it reads 16 bytes per lane in a row
+//   delta_scan_kernel      a wave per (sequence, head, 16 value columns) walks the chunks with S [d x 16] in its accumulators:
+//                          U = T V - W S, O^T = S^T q + U^T P^T, S <- 2^{L_15} S + k^T U.  No LDS and no barriers; an operand's next
+//                          value is loaded behind its last use
+//
+// A and P come apart into one factor per token on either side of a reference as in channel_chunks.hip: L_7 where t >= 8 > j, else the
+// middle of the half chunk both lie in (a decay below 2^-28 counts as 2^-28).  What is kept in 32 bits enters a product as the sum of two
+// bf16 numbers; where a product is 16 deep the two halves of the 32 deep instruction hold them.
+// A lane holds channels 32 s + 4 jj + 0..3 and 16 further on of step s in the first kernel, which is the order in which the accumulators
+// of S are an operand of the second.
+#include "mfma_tiles.h"
+
+namespace mops {
+
+constexpr int kDTokens = 16;
+constexpr float kLeastLog2Keep = -28.f;
+constexpr int kPieceBytes = 1024;      // an operand of a wave: 16 bytes per lane
+
+struct DeltaChunkArgs {
+  mops_hip_delta a;
+  const int32_t* chunks;        // [n][2]: first token, tokens
+  const int32_t* seq_chunks;    // [batch + 1]
+  int num_chunks, pitch;
+  unsigned char* operands;      // per (chunk, head): W hi, W lo, Q hi, Q lo [d / 32], K [d / 16], P, T as pieces, then 2^{L_15} float [d]
+  bool vec;
+};
+
+template <int DP>
+struct DeltaShape {
+  static constexpr int kSteps = DP / 32, kTiles = DP / 16;
+  static constexpr int kW = 0, kQ = 2 * kSteps, kK = 4 * kSteps, kP = kK + kTiles, kT = kP + 1, kPieces = kT + 1;
+  static constexpr int64_t kBytes = kPieces * kPieceBytes + DP * 4;
+};
+
+template <int N>
+__device__ __forceinline__ float row_up(float v) {       // the lane N places in front inside the row of 16; 0 where there is none
+  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x110 | N, 0xf, 0xf, true));
+}
+template <int N>
+__device__ __forceinline__ float row_take(float v) {     // lane N of the row of 16
+  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x150 | N, 0xf, 0xf, true));
+}
+__device__ __forceinline__ void wave_sync() {
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+}
+// Four values as hi (words 0, 1) and lo (words 2, 3).
+__device__ __forceinline__ u32x4 split4(const float (&v)[4]) {
+  u32x4 w;
+  w[0] = pack_bf16x2(v[0], v[1]);
+  w[1] = pack_bf16x2(v[2], v[3]);
+  w[2] = pack_bf16x2(v[0] - bf16lo_to_f32(w[0]), v[1] - bf16hi_to_f32(w[0]));
+  w[3] = pack_bf16x2(v[2] - bf16lo_to_f32(w[1]), v[3] - bf16hi_to_f32(w[1]));
+  return w;
+}
+__device__ __forceinline__ bf16x8 as_operand(u32x4 w) { return __builtin_bit_cast(bf16x8, w); }
+__device__ __forceinline__ bf16x8 high_twice(u32x4 w) { return as_operand(u32x4{w[0], w[1], w[0], w[1]}); }
+__device__ __forceinline__ bf16x8 low_once(u32x4 w) { return as_operand(u32x4{w[2], w[3], 0u, 0u}); }
+
+template <int DP, int WAVES>
+__global__ __launch_bounds__(64 * WAVES) void delta_prepare_kernel(const DeltaChunkArgs p) {
+  using Sh = DeltaShape<DP>;
+  constexpr int kS = Sh::kSteps, kPitch = DP + 8;
+  __shared__ __align__(16) uint16_t tiles[WAVES][2][kDTokens * kPitch];
+  const mops_hip_delta& a = p.a;
+  const int heads = (int)a.heads, d = (int)a.d;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, n16 = lane & 15, jj = lane >> 4;
+  const int64_t item = (int64_t)blockIdx.x * WAVES + wave;
+  if (item >= (int64_t)p.num_chunks * heads) return;      // no workgroup barriers below
+  const int h = (int)(item % heads), chunk = (int)(item / heads);
+  const int first = p.chunks[2 * chunk], n = p.chunks[2 * chunk + 1];
+  const bool in = n16 < n;
+  const int64_t t = first + (in ? n16 : n - 1);
+  const int g = h / (heads / (int)a.groups);
+  const uint16_t *qp = (const uint16_t*)a.q + t * a.q_stride + (int64_t)g * d, *kp = (const uint16_t*)a.k + t * a.k_stride + (int64_t)g * d;
+  const float* lp = a.log_decay + t * a.log_decay_stride + (int64_t)h * d;
+  float beta = sigmoid_for<float>(bf16lo_to_f32(((const uint16_t*)a.beta)[t * a.beta_stride + h]));
+  if (!in) beta = 0.f;
+
+  float q[kS][8], k[kS][8], L[kS][8];
+#pragma unroll
+  for (int s = 0; s < kS; ++s)
+#pragma unroll
+    for (int half = 0; half < 2; ++half) {
+      const int c = 32 * s + 16 * half + 4 * jj;
+      if (p.vec) {
+        const int cc = c < d ? c : 0;
+        const u32x2 x = *reinterpret_cast<const u32x2*>(qp + cc), y = *reinterpret_cast<const u32x2*>(kp + cc);
+        const f32x4 z = *reinterpret_cast<const f32x4*>(lp + cc);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          q[s][4 * half + e] = e & 1 ? bf16hi_to_f32(x[e >> 1]) : bf16lo_to_f32(x[e >> 1]);
+          k[s][4 * half + e] = e & 1 ? bf16hi_to_f32(y[e >> 1]) : bf16lo_to_f32(y[e >> 1]);
+          L[s][4 * half + e] = z[e];
+        }
+      } else {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const int cc = c + e < d ? c + e : 0;
+          q[s][4 * half + e] = bf16lo_to_f32(qp[cc]);
+          k[s][4 * half + e] = bf16lo_to_f32(kp[cc]);
+          L[s][4 * half + e] = lp[cc];
+        }
+      }
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const bool ok = in && c + e < d;
+        const int i = 4 * half + e;
+        q[s][i] = ok ? q[s][i] : 0.f;
+        k[s][i] = ok ? k[s][i] : 0.f;
+        L[s][i] = ok ? fmaxf(L[s][i] * 1.4426950408889634f, kLeastLog2Keep) : 0.f;
+      }
+    }
+  float qq = 0.f, kk = 0.f;
+#pragma unroll
+  for (int s = 0; s < kS; ++s)
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      qq += q[s][e] * q[s][e];
+      kk += k[s][e] * k[s][e];
+      float x = L[s][e];
+      x += row_up<1>(x);
+      x += row_up<2>(x);
+      x += row_up<4>(x);
+      x += row_up<8>(x);
+      L[s][e] = x;
+    }
+  qq += __shfl_xor(qq, 16, kWave);
+  kk += __shfl_xor(kk, 16, kWave);
+  qq += __shfl_xor(qq, 32, kWave);
+  kk += __shfl_xor(kk, 32, kWave);
+  const float rq = a.q_scale / sqrtf(qq + a.unit_eps), rk = 1.0f / sqrtf(kk + a.unit_eps);
+
+  unsigned char* const dst = p.operands + item * Sh::kBytes;
+  auto put = [&](int piece, u32x4 w) { store16(dst + piece * kPieceBytes + lane * 16, w); };
+  float* const decay = reinterpret_cast<float*>(dst + Sh::kPieces * kPieceBytes);
+  uint16_t* const hi_tile = tiles[wave][0];
+  uint16_t* const lo_tile = tiles[wave][1];
+  auto row_store = [&](int s, const float (&v)[8]) {      // a step's eight values of token n16 into the tiles
+#pragma unroll
+    for (int half = 0; half < 2; ++half) {
+      const float x[4] = {v[4 * half], v[4 * half + 1], v[4 * half + 2], v[4 * half + 3]};
+      const u32x4 w = split4(x);
+      const int at = n16 * kPitch + 32 * s + 16 * half + 4 * jj;
+      *reinterpret_cast<u32x2*>(hi_tile + at) = u32x2{w[0], w[1]};
+      *reinterpret_cast<u32x2*>(lo_tile + at) = u32x2{w[2], w[3]};
+    }
+  };
+
+  // ---- A and P: [j = 4 jj + e][t = n16], inside the halves of the chunk and across
+  f32x4 a_in = {0.f, 0.f, 0.f, 0.f}, p_in = a_in, a_over = a_in, p_over = a_in;
+#pragma unroll
+  for (int s = 0; s < kS; ++s) {
+    float kt[8], qt[8], kj[8], kb[8], qb[8], grown[8], qf[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      q[s][e] *= rq;
+      k[s][e] *= rk;
+      const float l = L[s][e], m3 = row_take<3>(l), m7 = row_take<7>(l), m11 = row_take<11>(l), mid = n16 < 8 ? m3 : m11;
+      const float up = __builtin_amdgcn_exp2f(l - mid), whole = __builtin_amdgcn_exp2f(l);
+      kt[e] = k[s][e] * up;
+      qt[e] = q[s][e] * up;
+      kj[e] = k[s][e] * __builtin_amdgcn_exp2f(mid - l);
+      const float over = __builtin_amdgcn_exp2f(n16 < 8 ? m7 - l : l - m7);
+      kb[e] = k[s][e] * over;
+      qb[e] = n16 < 8 ? 0.f : q[s][e] * over;
+      grown[e] = k[s][e] * whole;
+      qf[e] = q[s][e] * whole;
+    }
+    bf16x8 kth, ktl, qth, qtl, kjh, kjl, kbh, kbl, qbh, qbl, qfh, qfl;
+    split8(kt, kth, ktl);
+    split8(qt, qth, qtl);
+    split8(kj, kjh, kjl);
+    split8(kb, kbh, kbl);
+    split8(qb, qbh, qbl);
+    split8(qf, qfh, qfl);
+    a_in = mfma16(kjh, kth, a_in);
+    p_in = mfma16(kjh, qth, p_in);
+    a_over = mfma16(kbh, kbh, a_over);
+    p_over = mfma16(kbh, qbh, p_over);
+    a_in = mfma16(kjh, ktl, a_in);
+    p_in = mfma16(kjh, qtl, p_in);
+    a_over = mfma16(kbh, kbl, a_over);
+    p_over = mfma16(kbh, qbl, p_over);
+    a_in = mfma16(kjl, kth, a_in);
+    p_in = mfma16(kjl, qth, p_in);
+    a_over = mfma16(kbl, kbh, a_over);
+    p_over = mfma16(kbl, qbh, p_over);
+    put(Sh::kQ + s, __builtin_bit_cast(u32x4, qfh));
+    put(Sh::kQ + kS + s, __builtin_bit_cast(u32x4, qfl));
+    row_store(s, grown);
+  }
+  float below[4], weight[4], beta_j[4];
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    const int j = 4 * jj + e;
+    const bool over = n16 >= 8 && j < 8;
+    below[e] = j < n16 ? beta * (over ? a_over[e] : a_in[e]) : 0.f;
+    weight[e] = j <= n16 ? (over ? p_over[e] : p_in[e]) : 0.f;
+    beta_j[e] = __shfl(beta, j, kWave);
+  }
+  put(Sh::kP, split4(weight));
+
+  // ---- T: lane = row t, from the last column to the first; x[j] = [t == j] - sum_{i > j} x[i] below[i, j]
+  float x[kDTokens];
+#pragma unroll
+  for (int j = kDTokens - 1; j >= 0; --j) {
+    float acc = n16 == j ? 1.f : 0.f;
+#pragma unroll
+    for (int i = j + 1; i < kDTokens; ++i)
+      acc -= x[i] * __int_as_float(__builtin_amdgcn_readlane(__float_as_int(below[j & 3]), 16 * (j >> 2) + i));
+    x[j] = acc;
+  }
+  float tb[4];
+#pragma unroll
+  for (int e = 0; e < 4; ++e) tb[e] = (jj < 2 ? (jj == 0 ? x[e] : x[4 + e]) : (jj == 2 ? x[8 + e] : x[12 + e])) * beta_j[e];
+  const u32x4 tw = split4(tb);
+  put(Sh::kT, tw);
+
+  // ---- -W^T [d, t] = -(2^L k)^T T^T, in the order of an operand
+  wave_sync();
+  const bf16x8 t_high = high_twice(tw), t_low = low_once(tw);
+#pragma unroll
+  for (int s = 0; s < kS; ++s) {
+    float w[8];
+#pragma unroll
+    for (int half = 0; half < 2; ++half) {
+      const s16x4 kh = tile_block_columns(hi_tile, kPitch, 4 * jj, 32 * s + 16 * half, lane), kl = tile_block_columns(lo_tile, kPitch, 4 * jj, 32 * s + 16 * half, lane);
+      f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+      acc = mfma16(__builtin_bit_cast(bf16x8, join(kh, kl)), t_high, acc);
+      acc = mfma16(__builtin_bit_cast(bf16x8, join(kh, kh)), t_low, acc);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) w[4 * half + e] = -acc[e];
+    }
+    bf16x8 hi, lo;
+    split8(w, hi, lo);
+    put(Sh::kW + s, __builtin_bit_cast(u32x4, hi));
+    put(Sh::kW + kS + s, __builtin_bit_cast(u32x4, lo));
+  }
+  wave_sync();
+  // ---- 2^{L_15 - L} k, columns of it
+#pragma unroll
+  for (int s = 0; s < kS; ++s) {
+    float w[8], end[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      end[e] = row_take<15>(L[s][e]);
+      w[e] = k[s][e] * __builtin_amdgcn_exp2f(end[e] - L[s][e]);
+    }
+    row_store(s, w);
+    if (n16 == 0) {
+#pragma unroll
+      for (int half = 0; half < 2; ++half) {
+        f32x4 v;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = __builtin_amdgcn_exp2f(end[4 * half + e]);
+        *reinterpret_cast<f32x4*>(decay + 32 * s + 16 * half + 4 * jj) = v;
+      }
+    }
+  }
+  wave_sync();
+#pragma unroll
+  for (int i = 0; i < Sh::kTiles; ++i)
+    put(Sh::kK + i, __builtin_bit_cast(u32x4, join(tile_block_columns(hi_tile, kPitch, 4 * jj, 16 * i, lane), tile_block_columns(lo_tile, kPitch, 4 * jj, 16 * i, lane))));
+}
+
+constexpr int most_waves(int dp) { return dp <= 128 ? 8 : 4; }      // of a workgroup of the second kernel
+
+template <int DP>
+__global__ __launch_bounds__(64 * most_waves(DP)) void delta_scan_kernel(const DeltaChunkArgs p) {
+  using Sh = DeltaShape<DP>;
+  constexpr int kS = Sh::kSteps, kI = Sh::kTiles;
+  const mops_hip_delta& a = p.a;
+  const int heads = (int)a.heads, vd = (int)a.vd, columns = (int)blockDim.x >> 2;      // of a workgroup
+  const int blocks = (vd + columns - 1) / columns;
+  // each XCD a contiguous run of items, so that the workgroups of a head share an L2
+  const int total = (int)a.batch * heads * blocks, per_xcd = (total + 7) / 8;
+  const int item = (blockIdx.x % 8) * per_xcd + blockIdx.x / 8;
+  if ((int)blockIdx.x / 8 >= per_xcd || item >= total) return;
+  const int h = item / blocks % heads, b = item / (blocks * heads);
+  const int lane = threadIdx.x & 63, n16 = lane & 15, jj = lane >> 4;
+  const int v0 = item % blocks * columns + ((int)threadIdx.x >> 6) * 16;
+  if (v0 >= vd) return;      // no barriers below
+  const int slot = a.state_slots[b], t_begin = a.cu_seqlens[b], t_end = a.cu_seqlens[b + 1];
+  if (slot < 0 || slot >= a.num_slots || t_end <= t_begin) return;
+  const bool v_ok = v0 + n16 < vd;
+  const int v = v_ok ? v0 + n16 : vd - 1;
+  float* const state = a.state + (((int64_t)slot * heads + h) * vd + v) * p.pitch;
+  // S: tile i, element e = row d = 16 i + 4 jj + e, column v0 + n16
+  f32x4 st[kI];
+  const bool load_state = a.starts[b] > 0;
+#pragma unroll
+  for (int i = 0; i < kI; ++i) {
+    const int d = 16 * i + 4 * jj;
+    const bool ok = load_state && d < p.pitch;
+    const f32x4 w = *reinterpret_cast<const f32x4*>(state + (ok ? d : 0));
+#pragma unroll
+    for (int e = 0; e < 4; ++e) st[i][e] = ok ? w[e] : 0.f;
+  }
+  const uint16_t* const vp = (const uint16_t*)a.v + (int64_t)h * vd + v;
+  uint16_t* const op = (uint16_t*)a.out + (int64_t)h * vd + v0 + 4 * jj;
+
+  u32x4 wh[kS], wl[kS], qh[kS], ql[kS], kf[kI], pf, tf;
+  f32x4 dc[kI];
+  uint32_t vr[4];
+  const unsigned char* src = p.operands + ((int64_t)p.seq_chunks[b] * heads + h) * Sh::kBytes + lane * 16;
+  const int64_t step = heads * Sh::kBytes;
+  auto piece = [&](int i) { return load16(src + i * kPieceBytes); };
+  auto load_w = [&]() {
+#pragma unroll
+    for (int s = 0; s < kS; ++s) {
+      wh[s] = piece(Sh::kW + s);
+      wl[s] = piece(Sh::kW + kS + s);
+    }
+  };
+  auto load_q = [&]() {
+#pragma unroll
+    for (int s = 0; s < kS; ++s) {
+      qh[s] = piece(Sh::kQ + s);
+      ql[s] = piece(Sh::kQ + kS + s);
+    }
+  };
+  auto load_k = [&]() {
+#pragma unroll
+    for (int i = 0; i < kI; ++i) {
+      kf[i] = piece(Sh::kK + i);
+      dc[i] = *reinterpret_cast<const f32x4*>(src - lane * 16 + Sh::kPieces * kPieceBytes + (16 * i + 4 * jj) * 4);
+    }
+  };
+  auto load_v = [&](int t0) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) vr[e] = vp[(int64_t)(t0 + 4 * jj + e < t_end ? t0 + 4 * jj + e : t_end - 1) * a.v_stride];
+  };
+  load_v(t_begin);
+  tf = piece(Sh::kT);
+  load_w();
+  load_q();
+  pf = piece(Sh::kP);
+  load_k();
+  for (int t0 = t_begin; t0 < t_end; t0 += kDTokens) {
+    const bool more = t0 + kDTokens < t_end;
+    if (more) src += step;
+    const u32x2 vw = {vr[0] | vr[1] << 16, vr[2] | vr[3] << 16};
+    f32x4 u = {0.f, 0.f, 0.f, 0.f}, u2 = u, o = u, o2 = u;
+    u = mfma16(as_operand(tf), as_operand(u32x4{vw[0], vw[1], vw[0], vw[1]}), u);
+    if (more) {
+      load_v(t0 + kDTokens);
+      tf = piece(Sh::kT);
+    }
+#pragma unroll
+    for (int s = 0; s < kS; ++s) {
+      float x[8];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        x[e] = st[2 * s][e];
+        x[4 + e] = st[2 * s + 1][e];
+      }
+      bf16x8 hi, lo;
+      split8(x, hi, lo);
+      u = mfma16(as_operand(wh[s]), hi, u);
+      o = mfma16(hi, as_operand(qh[s]), o);
+      u2 = mfma16(as_operand(wh[s]), lo, u2);
+      o2 = mfma16(hi, as_operand(ql[s]), o2);
+      u = mfma16(as_operand(wl[s]), hi, u);
+      o = mfma16(lo, as_operand(qh[s]), o);
+    }
+    if (more) {
+      load_w();
+      load_q();
+    }
+    float uu[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) uu[e] = u[e] + u2[e];
+    const u32x4 uw = split4(uu);
+    const bf16x8 u_high = high_twice(uw), u_low = low_once(uw);
+    o = mfma16(u_high, as_operand(pf), o);
+    o2 = mfma16(u_low, as_operand(pf), o2);
+    if (more) pf = piece(Sh::kP);
+#pragma unroll
+    for (int i = 0; i < kI; ++i) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) st[i][e] *= dc[i][e];
+      st[i] = mfma16(as_operand(kf[i]), u_high, st[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < kI; ++i) st[i] = mfma16(as_operand(kf[i]), u_low, st[i]);
+    if (more) load_k();
+    if (t0 + n16 < t_end) {
+      uint16_t* const row = op + (int64_t)(t0 + n16) * a.out_stride;
+      const u32x2 w = {pack_bf16x2(o[0] + o2[0], o[1] + o2[1]), pack_bf16x2(o[2] + o2[2], o[3] + o2[3])};
+      if (p.vec && v0 + 4 * jj < vd) {
+        *reinterpret_cast<u32x2*>(row) = w;
+      } else {
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          if (v0 + 4 * jj + e < vd) row[e] = (uint16_t)(w[e >> 1] >> (16 * (e & 1)));
+      }
+    }
+  }
+  if (!v_ok) return;
+#pragma unroll
+  for (int i = 0; i < kI; ++i)
+    if (16 * i + 4 * jj < p.pitch) *reinterpret_cast<f32x4*>(state + 16 * i + 4 * jj) = st[i];
+}
+
+int check_delta(const mops_hip_delta* a);      // delta_rule.hip
+
+static int64_t operand_bytes(int64_t d) {
+  if (d <= 32) return DeltaShape<32>::kBytes;
+  if (d <= 64) return DeltaShape<64>::kBytes;
+  return d <= 128 ? DeltaShape<128>::kBytes : DeltaShape<256>::kBytes;
+}
+
+template <int DP>
+static int launch_delta_chunks(const DeltaChunkArgs& p, hipStream_t s) {
+  constexpr int kWaves = DP <= 128 ? 4 : 2;
+  const int64_t items = (int64_t)p.num_chunks * p.a.heads;
+  hipLaunchKernelGGL((delta_prepare_kernel<DP, kWaves>), dim3((unsigned)((items + kWaves - 1) / kWaves)), dim3(64 * kWaves), 0, s, p);
+  // as many waves in a workgroup as share a head's operands, fewer where that leaves most of the chip idle
+  const int64_t tiles = (p.a.vd + 15) / 16, rows = p.a.batch * p.a.heads;
+  int waves = tiles < most_waves(DP) ? (int)tiles : most_waves(DP);
+  if (rows * ((tiles + waves - 1) / waves) < 256 && waves > 4) waves = 4;
+  const int64_t total = rows * ((tiles + waves - 1) / waves);
+  hipLaunchKernelGGL((delta_scan_kernel<DP>), dim3((unsigned)((total + 7) / 8 * 8)), dim3(64 * waves), 0, s, p);
+  return finish_launch();
+}
+
+}  // namespace mops
+
+extern "C" int64_t mops_hip_delta_chunks_workspace_bytes(int64_t num_chunks, int64_t heads, int64_t d) {
+  return num_chunks <= 0 || heads <= 0 || d <= 0 || d > 256 ? 0 : num_chunks * heads * mops::operand_bytes(d);
+}
+
+extern "C" int mops_hip_delta_chunks(const mops_hip_delta* a, const int32_t* chunks, int64_t num_chunks, const int32_t* seq_chunks, void* workspace,
+                                     int64_t workspace_bytes, void* stream) {
+  using namespace mops;
+  const int pre = check_delta(a);
+  if (pre != 1) return pre;
+  if (a->dtype != MOPS_HIP_BF16 || a->d > 256 || a->conv_weight) return MOPS_HIP_EUNSUPPORTED;
+  if (num_chunks < 0 || !chunks || !seq_chunks || !a->cu_seqlens) return MOPS_HIP_EINVAL;
+  if (num_chunks == 0) return MOPS_HIP_OK;
+  if (num_chunks * a->heads > 0x7fffffffLL || a->batch * a->heads * ((a->vd + 15) / 16) > 0x3fffffffLL) return MOPS_HIP_EUNSUPPORTED;
+  if (!workspace || workspace_bytes < mops_hip_delta_chunks_workspace_bytes(num_chunks, a->heads, a->d)) return MOPS_HIP_EWORKSPACE;
+  if (!aligned16(workspace)) return MOPS_HIP_EALIGN;
+  DeltaChunkArgs p;
+  p.a = *a;
+  p.chunks = chunks;
+  p.seq_chunks = seq_chunks;
+  p.num_chunks = (int)num_chunks;
+  p.pitch = (int)mops_hip_recurrence_state_pitch(a->d);
+  p.operands = (unsigned char*)workspace;
+  p.vec = a->d % 4 == 0 && a->vd % 4 == 0 && a->q_stride % 4 == 0 && a->k_stride % 4 == 0 && a->log_decay_stride % 4 == 0 && a->out_stride % 4 == 0 &&
+          aligned16(a->q) && aligned16(a->k) && aligned16(a->log_decay) && aligned16(a->out);
+  hipStream_t s = (hipStream_t)stream;
+  if (a->d <= 32) return launch_delta_chunks<32>(p, s);
+  if (a->d <= 64) return launch_delta_chunks<64>(p, s);
+  return a->d <= 128 ? launch_delta_chunks<128>(p, s) : launch_delta_chunks<256>(p, s);
+}

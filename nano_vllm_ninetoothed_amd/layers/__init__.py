@@ -17,7 +17,7 @@ from dataclasses import dataclass
 import torch
 
 from .. import mops
-from ..mops.hip.recurrent_ops import CHUNK_MAX_DIM, channel_segments, recurrence_segments
+from ..mops.hip.recurrent_ops import CHUNK_MAX_DIM, channel_segments, delta_chunk_list, recurrence_segments
 
 MIXERS: dict = {}
 FEED_FORWARDS: dict = {}
@@ -102,12 +102,12 @@ class Rotary:
 class ChunkedRecurrence:
     """Runs a decayed recurrence over the portions of a batch: in chunks on the matrix cores in bf16, token by token for what
     those kernels do not cover (float32, head sizes beyond theirs)."""
-    CHUNKS = "decayed_chunks"
+    RECURRENCE, CHUNKS = "decayed_recurrence", "decayed_chunks"
 
     def __init__(self, heads, groups, d, vd, dtype):
         self.sizes = (heads, groups, d, vd)
         self.chunked = dtype == torch.bfloat16 and d <= CHUNK_MAX_DIM
-        self.recurrence, self.chunks = hip_op("decayed_recurrence"), hip_op(self.CHUNKS)
+        self.recurrence, self.chunks = hip_op(self.RECURRENCE), hip_op(self.CHUNKS)
 
     def segments(self, counts):
         heads, groups, _, vd = self.sizes
@@ -125,7 +125,8 @@ class ChunkedRecurrence:
         if key not in cuts:
             segments, bounds = self.segments(ctx["seq_counts"][nd:])
             flat = torch.tensor([x for s in segments for x in s] + bounds, dtype=torch.int32).to(v.device, non_blocking=True)
-            cuts[key] = (flat[:3 * len(segments)].view(-1, 3), flat[3 * len(segments):])
+            at = len(segments) * len(segments[0])
+            cuts[key] = (flat[:at].view(len(segments), -1), flat[at:])
         return self.chunks(q, k, v, out, state, slots, starts, *self.sizes, *cuts[key], cu_seqlens=cu, **options)
 
 
@@ -135,6 +136,14 @@ class ChannelRecurrence(ChunkedRecurrence):
 
     def segments(self, counts):
         return channel_segments(counts, self.sizes[0], self.sizes[3])
+
+
+class DeltaRecurrence(ChunkedRecurrence):
+    """The same for the gated delta rule; a cut is a list of chunks."""
+    RECURRENCE, CHUNKS = "delta_rule", "delta_chunks"
+
+    def segments(self, counts):
+        return delta_chunk_list(counts)
 
 
 def hip_op(name):

@@ -4,7 +4,7 @@ from __future__ import annotations
 
 import torch
 
-from . import Mixer, hip_op, register_mixer, require_size
+from . import DeltaRecurrence, Mixer, hip_op, register_mixer, require_size
 from .joined import TwoProducts
 from ..mops.hip.recurrent_ops import recurrence_state_pitch
 
@@ -38,6 +38,7 @@ class GatedDelta(TwoProducts, Mixer):
         self.dt_bias = take(prefix + "dt_bias", (h * d,), "vector").float().contiguous()
         self.rate = -torch.exp(take(prefix + "A_log", (h,), "vector").float()).contiguous()
         self.norm = take(prefix + "norm", (v,), "norm")
+        self.portions = DeltaRecurrence(h, g, d, v, m.dtype)
         self.recurrence, self.conv, self.conv_update = hip_op("delta_rule"), hip_op("short_conv"), hip_op("short_conv_update")
         self.decay, self.group_norm = hip_op("low_rank_decay"), hip_op("gated_group_norm")
         self.allocate(m.cache)
@@ -65,6 +66,6 @@ class GatedDelta(TwoProducts, Mixer):
         if nd < slots.numel():
             cu = ctx["portion_cu"]
             c = self.conv(qkv[nd:], self.conv_w, None, self.ring, ctx["portion_token_seq"], cu, starts[nd:], slots[nd:])
-            self.recurrence(*parts(c), o[nd:], self.state, slots[nd:], starts[nd:], *sizes, cu_seqlens=cu, **options(slice(nd, None)))
+            self.portions(*parts(c), o[nd:], self.state, ctx, **options(slice(nd, None)))
             self.conv_update(qkv[nd:], self.ring, cu, starts[nd:], slots[nd:])
         self.group_norm(o, gate, h, self.eps, weight=self.norm, activation="sigmoid", scale=scale, out=out)

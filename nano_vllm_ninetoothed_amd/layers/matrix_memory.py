@@ -4,7 +4,7 @@ from __future__ import annotations
 
 import torch
 
-from . import Mixer, hip_op, register_mixer, require_size
+from . import ChunkedRecurrence, Mixer, hip_op, register_mixer, require_size
 from .joined import TwoProducts
 from ..mops.hip.recurrent_ops import MemoryGates, matrix_memory_copies, recurrence_state_pitch
 
@@ -29,6 +29,7 @@ class MatrixMemory(TwoProducts, Mixer):
         self.products([qkv, gate, gates], take(prefix + "o", (m.width, h * v)))
         self.biases = [take(f"{prefix}{n}.b", (h,), "vector").float().contiguous() for n in ("i", "f")]
         self.norm = take(prefix + "norm", (h * v,), "norm")
+        self.portions = ChunkedRecurrence(h, h, d, v, m.dtype)
         self.recurrence, self.group_norm = hip_op("decayed_recurrence"), hip_op("gated_group_norm")
         self.allocate(m.cache)
 
@@ -45,11 +46,10 @@ class MatrixMemory(TwoProducts, Mixer):
         nd, slots, starts = ctx["n_decode"], ctx["state_slots"], ctx["starts"]
 
         def options(rows):
-            return dict(k_scale=d ** -0.5, gates=MemoryGates(both[rows, :h], both[rows, h:], *self.biases, self.cap, self.top))
+            return dict(gates=MemoryGates(both[rows, :h], both[rows, h:], *self.biases, self.cap, self.top, d ** -0.5))
 
         if nd:
             self.recurrence(q[:nd], k[:nd], vv[:nd], o[:nd], self.state, slots[:nd], starts[:nd], h, h, d, v, **options(slice(nd)))
         if nd < slots.numel():
-            self.recurrence(q[nd:], k[nd:], vv[nd:], o[nd:], self.state, slots[nd:], starts[nd:], h, h, d, v, cu_seqlens=ctx["portion_cu"],
-                            **options(slice(nd, None)))
+            self.portions(q[nd:], k[nd:], vv[nd:], o[nd:], self.state, ctx, **options(slice(nd, None)))
         self.group_norm(o, gate, h, self.eps, weight=self.norm, activation="sigmoid", scale=scale, out=out)

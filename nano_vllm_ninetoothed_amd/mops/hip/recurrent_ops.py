@@ -240,14 +240,15 @@ def matrix_memory_copies(vd: int) -> int:
 
 @dataclass(frozen=True)
 class MemoryGates:
-    """A matrix memory's gates: projections [tokens, heads] in front of bias and cap, biases (float32 [heads]), the cap, and the running
-    maximum of every slot (float32 [slots, heads, copies])."""
+    """A matrix memory's gates: projections [tokens, heads] in front of bias and cap, biases (float32 [heads]), the cap, the running maximum
+    of every slot (float32 [slots, heads, copies]), and a factor on the queries."""
     input: torch.Tensor
     forget: torch.Tensor
     input_bias: torch.Tensor
     forget_bias: torch.Tensor
     cap: float
     top: torch.Tensor
+    q_scale: float = 1.0
 
 
 def recurrence_state_pitch(d: int) -> int:
@@ -306,7 +307,7 @@ def _recurrence_args(q, k, v, out, state, state_slots, starts, heads, groups, d,
         r.conv_bias = _flat("conv bias", bias, weight.shape[1], torch.float32)
         r.conv_ring = _flat("conv ring", ring, state.shape[0] * weight.numel(), v.dtype)
     r.batch, r.heads, r.groups, r.d, r.vd = batch, heads, groups, d, vd
-    r.k_scale, r.dtype = float(k_scale), code
+    r.k_scale, r.dtype = float(k_scale if gates is None else gates.q_scale), code
     return r
 
 
@@ -363,6 +364,33 @@ def delta_rule(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, *
     return out
 
 
+DELTA_CHUNK = 16      # tokens
+
+
+def delta_chunk_list(counts):
+    """Cuts portions of counts[i] tokens (packed one behind the other) for delta_chunks: host lists (chunks, bounds per portion)."""
+    chunks, bounds, at = [], [0], 0
+    for n in counts:
+        chunks += [(at + begin, min(DELTA_CHUNK, n - begin)) for begin in range(0, n, DELTA_CHUNK)]
+        bounds.append(len(chunks))
+        at += n
+    return chunks, bounds
+
+
+@register_hip_op
+def delta_chunks(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, chunks, seq_chunks, **options):
+    """delta_rule for packed portions of many tokens, on the matrix cores (bf16, d up to CHUNK_MAX_DIM).  chunks [n, 2] and seq_chunks
+    [sequences + 1] are the int32 device copies of what delta_chunk_list returns; cu_seqlens is required."""
+    a = _delta_args(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, **options)
+    n, lib = chunks.shape[0], _capi.load()
+    _require(a.batch == seq_chunks.numel() - 1, "seq_chunks must bound the chunks of every sequence")
+    ws = torch.empty(max(16, lib.mops_hip_delta_chunks_workspace_bytes(n, heads, d)), dtype=torch.uint8, device=v.device)
+    st = lib.mops_hip_delta_chunks(byref(a), _flat("chunks", chunks, 2 * n, torch.int32), n, _flat("seq_chunks", seq_chunks, a.batch + 1, torch.int32),
+                                   ws.data_ptr(), ws.numel(), _stream(v))
+    _capi.check("mops_hip_delta_chunks", st)
+    return out
+
+
 CHUNK_MAX_DIM = 256       # head sizes (d) the chunked kernels cover
 
 
@@ -392,11 +420,16 @@ def _segments(counts, per_segment: int, wanted: int, enough: int):
 
 def _chunks(name, seg_decay_shape, q, k, v, out, state, state_slots, starts, heads, groups, d, vd, segments, seq_segments, **options):
     r = _recurrence_args(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, **options)
+    if options.get("gates") is not None:      # token by token, but numbers per head only
+        per_token = torch.empty((3, v.shape[0], heads), dtype=torch.float32, device=v.device)
+        r.log_keep, r.input_scale, r.least = (x.data_ptr() for x in per_token)
+        st = _capi.load().mops_hip_matrix_memory_gates(byref(r), r.log_keep, r.input_scale, r.least, _stream(v))
+        _capi.check("mops_hip_matrix_memory_gates", st)
     n = segments.shape[0]
     _require(r.batch == seq_segments.numel() - 1, "seq_segments must bound the segments of every sequence")
     seg_state = seg_decay = None
     if n > r.batch:
-        seg_state = torch.empty((n, heads, vd, state.shape[3]), dtype=torch.float32, device=v.device)
+        seg_state = torch.empty((n, *state.shape[1:]), dtype=torch.float32, device=v.device)
         seg_decay = torch.empty((n, *seg_decay_shape), dtype=torch.float32, device=v.device)
     st = getattr(_capi.load(), name)(byref(r), _flat("segments", segments, 3 * n, torch.int32), n,
                                      _flat("seq_segments", seq_segments, r.batch + 1, torch.int32),

@@ -146,18 +146,19 @@ def channel_decays(z, a_log, dt_bias, heads):
     return torch.exp(-torch.exp(a_log)[None, :, None] * softplus(z + dt_bias).view(z.shape[0], heads, -1))
 
 
-def delta_rule(q, k, v, g, beta):
-    """q, k [T, G, D], v [T, H, V], g [T, H, D], beta [T, H]: S <- g S; S <- S + k (beta (v - S^T k))^T; o = S^T q."""
+def delta_rule(q, k, v, g, beta, S=None):
+    """q, k [T, G, D], v [T, H, V], g [T, H, D], beta [T, H]: S <- g S; S <- S + k (beta (v - S^T k))^T; o = S^T q.  Returns (o [T, H, V],
+    the last S [H, D, V])."""
     T, H, V = v.shape
     q, k = (x.repeat_interleave(H // x.shape[1], dim=1) for x in (q, k))
-    S = torch.zeros((H, k.shape[2], V), dtype=v.dtype)
+    S = torch.zeros((H, k.shape[2], V), dtype=v.dtype) if S is None else S
     out = []
     for t in range(T):
         S = g[t][:, :, None] * S
         u = beta[t][:, None] * (v[t] - torch.einsum("hdv,hd->hv", S, k[t]))
         S = S + k[t][:, :, None] * u[:, None, :]
         out.append(torch.einsum("hdv,hd->hv", S, q[t]))
-    return torch.stack(out)
+    return torch.stack(out), S
 
 
 def gated_delta(h, w, m, eps):
@@ -166,7 +167,7 @@ def gated_delta(h, w, m, eps):
     q, k = unit(q.view(T, G, D)) * D ** -0.5, unit(k.view(T, G, D))
     beta = sigmoid(product(h, w["b"]))
     g = channel_decays(product(product(h, w["a1"]), w["a2"]), w["A_log"], w["dt_bias"], H)
-    o = stored(delta_rule(q, k, v.view(T, H, V), g, beta))
+    o = stored(delta_rule(q, k, v.view(T, H, V), g, beta)[0])
     o = over_rms(o, eps) * w["norm"] * sigmoid(product(product(h, w["g1"]), w["g2"])).view(T, H, V)
     return o.reshape(T, H * V)
 
@@ -183,10 +184,13 @@ def capped(x, cap):
     return cap * torch.tanh(x / cap)
 
 
-def matrix_memory(q, k, v, i, f):
-    """q, k [T, H, D], v [T, H, V], logarithms of the gates i, f [T, H]; everything relative to a running maximum m that starts at 0."""
+def matrix_memory(q, k, v, i, f, state=None):
+    """q, k [T, H, D], v [T, H, V], logarithms of the gates i, f [T, H]; everything relative to a running maximum m that starts at 0.
+    Returns (o [T, H, V], the last (S [H, D, V], n [H, D], m [H]))."""
     T, H, V = v.shape
-    S, n, m = torch.zeros((H, q.shape[2], V), dtype=v.dtype), torch.zeros((H, q.shape[2]), dtype=v.dtype), torch.zeros(H, dtype=v.dtype)
+    if state is None:
+        state = (torch.zeros((H, q.shape[2], V), dtype=v.dtype), torch.zeros((H, q.shape[2]), dtype=v.dtype), torch.zeros(H, dtype=v.dtype))
+    S, n, m = state
     out = []
     for t in range(T):
         m_new = torch.maximum(f[t] + m, i[t])
@@ -196,15 +200,19 @@ def matrix_memory(q, k, v, i, f):
         n = keep[:, None] * n + take[:, None] * k[t]
         den = torch.maximum((n * q[t]).sum(-1).abs(), torch.exp(-m)) + 1e-6
         out.append(torch.einsum("hdv,hd->hv", S, q[t]) / den[:, None])
-    return torch.stack(out)
+    return torch.stack(out), (S, n, m)
+
+
+def log_gates(i, f, cap):
+    """(input gate, forget gate), both logarithms, from their projections."""
+    return capped(i, cap), -softplus(-capped(f, cap))
 
 
 def mlstm(h, w, m, eps):
     H, D, V, T = m["heads"], m["dim"], m["vdim"], h.shape[0]
     q, k, v = product(h, w["q"]).view(T, H, D) * D ** -0.5, product(h, w["k"]).view(T, H, D), product(h, w["v"]).view(T, H, V)
-    i = capped(product(h, w["i"]) + w["i.b"], m["gate_cap"])
-    f = -softplus(-capped(product(h, w["f"]) + w["f.b"], m["gate_cap"]))
-    o = over_rms(stored(matrix_memory(q, k, v, i, f)), eps).reshape(T, H * V)
+    i, f = log_gates(product(h, w["i"]) + w["i.b"], product(h, w["f"]) + w["f.b"], m["gate_cap"])
+    o = over_rms(stored(matrix_memory(q, k, v, i, f)[0]), eps).reshape(T, H * V)
     return product(o * w["norm"] * sigmoid(product(h, w["g"])), w["o"])
 
 
