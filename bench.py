@@ -14,6 +14,7 @@ A step is one flash_attn_with_kvcache call over the whole batch, KV cache reside
          the line's value is the decode throughput of the last size at the largest batch.
   sozarax = the same for Sozarax, beside Nepulix and Qwen3 models of equal size and their kernels.
   lulizen = the same for Lulizen, beside Sozarax and Qwen3 models of equal size and their kernels.
+  fedovik = the same for Fedovik, beside Sozarax and Qwen3 models of equal size and their kernels.
   copy = a plain 1 GiB device-to-device tensor copy (not a mops op): the known-size kernel against which
          the FETCH_SIZE / WRITE_SIZE counters of a profile are calibrated.
   launch_floor = an empty kernel: the floor under the durations of the small operators (value 0, read the time).
@@ -62,13 +63,13 @@ def parse_args():
     ap.add_argument("--steps", type=int, default=None, help="timed steps (default 50; 500 for the prefill ops)")
     ap.add_argument("--warmup", type=int, default=None, help="untimed warm-up steps (default 10; 300 for the prefill ops)")
     ap.add_argument("--op", default="decode",
-                    choices=["decode", "decode8b", "prefill", "prefill_long", "prefix_prefill", "prefix_prefill_short", "store", "silu", "sampler", "qk_rope_store", "add_rms", "rms", "embedding", "copy", "launch_floor", "e2e", "nepulix", "sozarax", "lulizen"])
+                    choices=["decode", "decode8b", "prefill", "prefill_long", "prefix_prefill", "prefix_prefill_short", "store", "silu", "sampler", "qk_rope_store", "add_rms", "rms", "embedding", "copy", "launch_floor", "e2e", "nepulix", "sozarax", "lulizen", "fedovik"])
     ap.add_argument("--e2e-seqs", type=int, default=256, help="number of prompts of the e2e workload")
     ap.add_argument("--e2e-eager", action="store_true", help="e2e: no HIP-graph replay of the decode step")
     ap.add_argument("--e2e-stepwise", action="store_true", help="e2e: read every step's tokens back before the next step, as the reference does")
-    ap.add_argument("--part", "--nepulix-part", default="all", choices=["all", "models", "kernels"], help="nepulix, sozarax, lulizen: throughput of whole models, kernels, or both")
-    ap.add_argument("--kernels", "--nepulix-kernels", default="", help="nepulix, sozarax, lulizen: kernels to time, by the beginning of their names, with commas between them (default: all)")
-    ap.add_argument("--sizes", "--nepulix-sizes", default="", help="nepulix, sozarax, lulizen: sizes to run, with commas between them (default: all)")
+    ap.add_argument("--part", "--nepulix-part", default="all", choices=["all", "models", "kernels"], help="nepulix, sozarax, lulizen, fedovik: throughput of whole models, kernels, or both")
+    ap.add_argument("--kernels", "--nepulix-kernels", default="", help="nepulix, sozarax, lulizen, fedovik: kernels to time, by the beginning of their names, with commas between them (default: all)")
+    ap.add_argument("--sizes", "--nepulix-sizes", default="", help="nepulix, sozarax, lulizen, fedovik: sizes to run, with commas between them (default: all)")
     ap.add_argument("--no-cpu-baseline", action="store_true")
     ap.add_argument("--no-e2e", action="store_true", help="default op only: skip the end-to-end block of the line (profiling runs)")
     ap.add_argument("--seed", type=int, default=0)
@@ -172,7 +173,7 @@ def run_e2e(args, torch, dev, mops):
 
 
 def run_design(args, torch, dev):
-    """`--op nepulix`, `--op sozarax`, `--op lulizen`: throughput of the models and the table of kernels, in one line."""
+    """`--op nepulix`, `--op sozarax`, `--op lulizen`, `--op fedovik`: throughput of the models and the table of kernels, in one line."""
     from nano_vllm_ninetoothed_amd import bench_layers as B
     from nano_vllm_ninetoothed_amd.models import parse_config
     design = args.op
@@ -238,7 +239,7 @@ def main():
     if args.op == "e2e":
         run_e2e(args, torch, dev, mops)
         return
-    if args.op in ("nepulix", "sozarax", "lulizen"):
+    if args.op in ("nepulix", "sozarax", "lulizen", "fedovik"):
         run_design(args, torch, dev)
         return
     bound = "hbm"

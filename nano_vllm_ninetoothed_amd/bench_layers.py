@@ -1,4 +1,4 @@
-"""Measurements behind `bench.py --op nepulix`, `--op sozarax` and `--op lulizen`: prefill and decode throughput of models with layers
+"""Measurements behind `bench.py --op nepulix`, `--op sozarax`, `--op lulizen` and `--op fedovik`: prefill and decode throughput of models with layers
 of real sizes beside models of equal width, depth, feed-forward and vocabulary (Qwen3 and the designs that came before), and every
 kernel of the design beside the like kernel of those.  Random weights and inputs."""
 from __future__ import annotations
@@ -74,7 +74,29 @@ def lulizen_sizes():
             "w2048": (lulizen_dict(2048, 6, 6144, 32768, 16, 32, 4), *near["w2048"])}
 
 
-DESIGNS = {"nepulix": (sizes, "Qwen3"), "sozarax": (sozarax_sizes, "Nepulix and Qwen3"), "lulizen": (lulizen_sizes, "Sozarax and Qwen3")}
+def fedovik_dict(width, layers, ff, vocab, memory, att, left, right):
+    """A matrix memory, attention with sigmoid weights, and attention over a window beside a delta rule in turn; one pass of the loop, so
+    that a token runs through as many layers as in the other models."""
+    kinds = [("mlstm", memory), ("attention", att), ("parallel", {"left": left, "right": right, "left_scale": 0.7, "right_scale": 0.7})]
+    out = [{"type": kinds[i % 3][0], "mixer": kinds[i % 3][1], "mlp": {"kind": "dense", "ff": ff}} for i in range(layers)]
+    return {"architecture": "Fedovik", "width": width, "vocab": vocab, "norm": {"eps": 1e-6}, "embedding": {"scale": width ** 0.5}, "layers": out,
+            "loop": {"start": 0, "stop": layers, "times": 1}}
+
+
+def fedovik_sizes():
+    """name -> (Fedovik config.json dict, Sozarax dict and Qwen3Shape of equal size)"""
+    att = {"heads": 16, "kv_heads": 8, "dim": 128, "vdim": 128, "scale": 128 ** -0.5}
+    left = lambda heads: dict(att, heads=heads, kv_heads=heads // 2, mask={"size": 512})      # noqa: E731
+    near = {n: (c[0], c[-1]) for n, c in sozarax_sizes().items()}
+    rot = {"rot": {"base": 5e5, "dims": 128}}
+    return {"w1024": (fedovik_dict(1024, 12, 3072, 32768, {"heads": 8, "dim": 128, "vdim": 128, "gate_cap": 15.0}, {**att, **rot}, left(8),
+                                   {"heads": 8, "kv_heads": 8, "dim": 128, "vdim": 128, "conv": 4}), *near["w1024"]),
+            "w2048": (fedovik_dict(2048, 6, 6144, 32768, {"heads": 16, "dim": 128, "vdim": 128, "gate_cap": 15.0}, {**att, **rot}, left(16),
+                                   {"heads": 16, "kv_heads": 16, "dim": 128, "vdim": 128, "conv": 4}), *near["w2048"])}
+
+
+DESIGNS = {"nepulix": (sizes, "Qwen3"), "sozarax": (sozarax_sizes, "Nepulix and Qwen3"), "lulizen": (lulizen_sizes, "Sozarax and Qwen3"),
+           "fedovik": (fedovik_sizes, "Sozarax and Qwen3")}
 
 
 def _events(fn, warmup, steps):
@@ -510,6 +532,112 @@ def lulizen_kernels(t):
         like="add_rms prefill")
 
 
+def fedovik_attention(t):
+    from .layers import Rotary
+    from .mops.hip.attention_ops import Scores, biased_prefill_tiles
+    add, rnd, i32, dev = _handles(t)
+    ctx, blocks, table, lens_g = decode_contexts(t)
+    H, G, d = 16, 8, 128
+    far = (t.f32(H).abs(), t.f32(H).abs())
+    kp, vp, q, gate = rnd(blocks, 256, G, d), rnd(blocks, 256, G, d), rnd(256, H, d), rnd(256, H * d)
+    like = "biased_decode 256 x uniform[512,4096], 16/8 heads of 128"
+    for label, scores, g, seen in (
+            ("sigmoid weights, gates", Scores(weight_bias=t.f32(H)), gate, lambda n: n),
+            ("log distance", Scores(log_distance=far), None, lambda n: n),
+            ("log distance, window of 512", Scores(log_distance=far, window=512), None, lambda n: min(n, 512))):
+        add("biased_decode", f"256 x uniform[512,4096], {label}", lambda: graph_time(lambda i: op("biased_decode")(q, kp, vp, d, d, lens_g, table, 0.088, scores=scores, gate=g), 4),
+            nbytes=sum(map(seen, ctx)) * G * 2 * d * 2.0 + 256 * H * (2 if g is None else 3) * d * 2, like=like)
+    del kp, vp
+    kp, vp, q, gate = rnd(T // 256, 256, G, d), rnd(T // 256, 256, G, d), rnd(T, H, d), rnd(T, H * d)
+    out, lens = torch.empty((T, H * d), dtype=torch.bfloat16, device=dev), i32([0] * T)
+    for n, label, scores, g, seen in (
+            (1024, "sigmoid weights, gates", Scores(weight_bias=t.f32(H)), gate, lambda i: i + 1),
+            (1024, "log distance", Scores(log_distance=far), None, lambda i: i + 1),
+            (4096, "log distance, window of 512", Scores(log_distance=far, window=512), None, lambda i: min(i + 1, 512))):
+        b = T // n
+        tiles, ptab = i32(biased_prefill_tiles([n] * b, [0] * b, 0, 0)), torch.arange(T // 256, dtype=torch.int32, device=dev).view(b, -1)
+        add("biased_prefill", f"{b} x {n}, {label}", lambda: _events(lambda: op("biased_prefill")(
+            q, kp, vp, d, d, tiles, ptab, 0.088, lens, out=out, scores=scores, gate=g), 300, 200), flops=2.0 * H * 2 * d * b * sum(map(seen, range(n))),
+            like="biased_prefill 16 x 1024, 16/8 heads of 128")
+    qkv, w, bias = [rnd(T, (H + 2 * G) * d) for _ in range(2)], rnd(d), rnd((H + 2 * G) * d)
+    pos, slots = (torch.arange(T, device=dev) % 1024).to(torch.int32), torch.randperm(T, device=dev).to(torch.int32)
+    trig = Rotary(8192, dev).table(1e4, 128)
+    for label, more in (("biases, neighbours turned", {"cos_sin": trig}), ("biases, norms", {"q_weight": w, "k_weight": w})):
+        add("rotary_prepare", f"{T} tokens, 16/8 heads of 128, {label}", lambda: graph_time(lambda i: op("rotary_prepare")(
+            qkv[i % 2], pos, slots, kp, vp, H, G, d, d, eps=1e-6, bias=bias, neighbours=True, **more), 8), nbytes=T * (H + 2 * G) * d * 4.0,
+            like=f"attention_prepare {T} tokens, 16/8 heads of 128")
+
+
+def fedovik_recurrences(t):
+    from .mops.hip import recurrent_ops as R
+    add, rnd, i32, dev = _handles(t)
+    bs, heads = 256, 16
+    sl, st = torch.arange(bs, dtype=torch.int32, device=dev), torch.full((bs,), 1000, dtype=torch.int32, device=dev)
+    for dd in (64, 128):
+        n, pitch = heads * dd, R.recurrence_state_pitch(dd)
+        shape = f"{heads} x {dd} x {dd}"
+        state = torch.randn((bs, heads, dd, pitch), generator=t.g, device=dev) / 16
+        x, ld, o, beta = rnd(bs, 3 * n), -torch.exp(t.f32(bs, n) - 3), torch.empty((bs, n), dtype=torch.bfloat16, device=dev), rnd(bs, heads)
+        conv = (t.f32(4, 3 * n), torch.zeros((bs, 4, 3 * n), dtype=torch.bfloat16, device=dev), (0, n, 2 * n))
+        opts = dict(q_scale=dd ** -0.5, unit_eps=1e-6)
+        like = f"decayed_recurrence channels {bs} sequences, {shape}"
+        add("delta_rule", f"{bs} sequences, {shape}", lambda: graph_time(lambda i: op("delta_rule")(
+            x[:, :n], x[:, n:2 * n], x[:, 2 * n:], o, state, sl, st, heads, heads, dd, dd, log_decay=ld, beta=beta, **opts), 6),
+            nbytes=2.0 * bs * n * dd * 4 + bs * n * 12, like=like)
+        add("delta_rule", f"{bs} sequences, {shape}, convolutions of 4", lambda: graph_time(lambda i: op("delta_rule")(
+            x[:, :n], x[:, n:2 * n], x[:, 2 * n:], o, state, sl, st, heads, heads, dd, dd, log_decay=ld, beta=beta, conv=conv, **opts), 6),
+            nbytes=2.0 * bs * n * dd * 4 + bs * n * (12 + 24), like=like)
+        xs, ldT, oT, betas = rnd(T, 3 * n), -torch.exp(t.f32(T, n) - 3), torch.empty((T, n), dtype=torch.bfloat16, device=dev), rnd(T, heads)
+        for nseq in (16, 1):
+            chunks, ends = (i32(v) for v in R.delta_chunk_list([T // nseq] * nseq))
+            cu, zero = i32(list(range(0, T + 1, T // nseq))), torch.zeros(nseq, dtype=torch.int32, device=dev)
+            # least arithmetic at 16 tokens a chunk: the products inside it, the triangular system, state in and out and what a key finds there
+            add("delta_chunks", f"{nseq} x {T // nseq}, {shape}", lambda: _events(lambda: op("delta_chunks")(
+                xs[:, :n], xs[:, n:2 * n], xs[:, 2 * n:], oT, state, sl[:nseq], zero, heads, heads, dd, dd, chunks, ends, cu_seqlens=cu, log_decay=ldT, beta=betas, **opts), 20, 50),
+                flops=T * heads * (17.0 * 4 * dd + 6.0 * dd * dd), nbytes=T * n * 12.0, like=f"channel_chunks {nseq} x {T // nseq}, {shape}")
+        del xs, ldT, oT
+        copies = R.matrix_memory_copies(dd)
+        state, top = torch.randn((bs, heads, dd + copies, pitch), generator=t.g, device=dev), torch.zeros((bs, heads, copies), device=dev)
+        bi, bf = t.f32(heads), t.f32(heads) + 3
+        x, both = rnd(bs, 3 * n), rnd(bs, 2 * heads)
+        memory = lambda g: R.MemoryGates(g[:, :heads], g[:, heads:], bi, bf, 15.0, top, dd ** -0.5)      # noqa: E731
+        add("decayed_recurrence memory", f"{bs} sequences, {shape}", lambda: graph_time(lambda i: op("decayed_recurrence")(
+            x[:, :n], x[:, n:2 * n], x[:, 2 * n:], o, state, sl, st, heads, heads, dd, dd, gates=memory(both)), 6),
+            nbytes=2.0 * bs * n * dd * 4 + bs * n * 8, like="decayed_recurrence retention 256 sequences, 16 x 128 x 128")
+        xs, boths, oT = rnd(T, 3 * n), rnd(T, 2 * heads), torch.empty((T, n), dtype=torch.bfloat16, device=dev)
+        for nseq in (16, 1):
+            segs, ends = (i32(v) for v in R.recurrence_segments([T // nseq] * nseq, heads, heads, dd))
+            cu, zero = i32(list(range(0, T + 1, T // nseq))), torch.zeros(nseq, dtype=torch.int32, device=dev)
+            add("decayed_chunks memory", f"{nseq} x {T // nseq}, {shape}", lambda: _events(lambda: op("decayed_chunks")(
+                xs[:, :n], xs[:, n:2 * n], xs[:, 2 * n:], oT, state, sl[:nseq], zero, heads, heads, dd, dd, segs, ends, cu_seqlens=cu, gates=memory(boths)), 20, 50),
+                flops=T * heads * (65.0 * 2 * dd + 4.0 * dd * dd), nbytes=T * n * 8.0, like=f"decayed_chunks retention {nseq} x {T // nseq}, 16 x 128 x 128")
+        del xs, oT
+    rank = 32
+    z, w2, w0, rate = [rnd(T, rank) for _ in range(4)], rnd(1024, rank), t.f32(1024), -torch.exp(t.f32(16))
+    add("low_rank_decay", f"{T} x {rank} -> 1024, rates", lambda: graph_time(lambda i: op("low_rank_decay")(z[i % 4], w2, w0, rate=rate), 4), nbytes=T * (rank * 2 + 1024 * 4.0),
+        like=f"low_rank_decay {T} x {rank} -> 1024")
+    y, gate, wn = [rnd(T, 1024) for _ in range(4)], [rnd(T, 1024) for _ in range(4)], rnd(64)
+    add("gated_group_norm", f"{T} x 1024, 16 groups, sigmoid", lambda: graph_time(lambda i: op("gated_group_norm")(y[i % 4], gate[i % 4], 16, 1e-6, weight=wn, activation="sigmoid", scale=0.7), 8),
+        nbytes=T * 1024 * 6.0, like=f"gated_group_norm {T} x 1024, 16 groups")
+
+
+def fedovik_rows(t):
+    add, rnd, i32, dev = _handles(t)
+    halves = [rnd(T, 6144).chunk(2, dim=-1) for _ in range(4)]
+    add("relu_glu", f"{T} x 3072", lambda: graph_time(lambda i: op("relu_glu")(*halves[i % 4]), 8), nbytes=T * 3072 * 6.0, like="siluAndMul")
+    for rows, n in ((512, 4096), (T, 1024)):
+        sets = 24 if rows == 512 else 4
+        res, yy, w, b, shift = [t.f32(rows, n) for _ in range(sets)], [rnd(rows, n) for _ in range(sets)], rnd(n), rnd(n), t.f32(n)
+        add("add_norm", f"{rows} x {n}, layer norms", lambda: graph_time(lambda i: op("add_norm")(res[i % sets], yy[i % sets], shift, False, w, b, 1e-6, center=True), 24 if rows == 512 else 8),
+            nbytes=rows * n * 12.0, like=f"add_norm_norm {rows} x {n}, 1 part")
+
+
+def fedovik_kernels(t):
+    fedovik_attention(t)
+    fedovik_recurrences(t)
+    fedovik_rows(t)
+
+
 def kernel_table(dev, seed=0, only="", design="nepulix"):
     """The rows of a design's kernels behind those of the models it is measured against."""
     t = KernelTable(dev, seed, only)
@@ -522,6 +650,12 @@ def kernel_table(dev, seed=0, only="", design="nepulix"):
         sozarax_experts(t)
         sozarax_residual(t)
         lulizen_kernels(t)
+    elif design == "fedovik":
+        decayed_kernels(t, "retention", 16, 16, 128, 128, True)
+        sozarax_attention(t)
+        time_mixing_kernels(t)
+        sozarax_residual(t)
+        fedovik_kernels(t)
     else:
         nepulix_kernels(t)
     return t.rows
