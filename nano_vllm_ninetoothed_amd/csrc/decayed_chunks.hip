@@ -652,23 +652,26 @@ static int launch_chunks_for(const ChunkArgs& a, const int32_t* seq_segments, in
   return launch_chunks<256, NH, true, MEMORY>(a, seq_segments, batch, s);
 }
 
-// Gates of a matrix memory over the tokens of every (sequence, head), one wave each: with m_t = max(f_t + m_(t-1), i_t) the logarithm of
-// the decay f_t + m_(t-1) - m_t, the input scale exp(i_t - m_t) and exp(-m_t); files the last m in all copies.  m is a scan over pairs (sum
-// of f, greatest i carried to the end), 256 tokens at a time.
-__global__ __launch_bounds__(64) void matrix_memory_gates_kernel(const mops_hip_recurrence r, int copies, float* __restrict__ log_keep,
-                                                                 float* __restrict__ input_scale, float* __restrict__ least) {
-  const int heads = (int)r.heads, h = blockIdx.x % heads, b = blockIdx.x / heads, lane = threadIdx.x;
+// Gates of a matrix memory over the tokens of every (sequence, head), one workgroup each: with m_t = max(f_t + m_(t-1), i_t) the logarithm
+// of the decay f_t + m_(t-1) - m_t, the input scale exp(i_t - m_t) and exp(-m_t); files the last m in all copies.  m is a scan over pairs
+// (sum of f, greatest i carried to the end), four tokens per thread at a time.
+constexpr int kGateThreads = 1024;
+
+__global__ __launch_bounds__(kGateThreads) void matrix_memory_gates_kernel(const mops_hip_recurrence r, int copies, float* __restrict__ log_keep,
+                                                                           float* __restrict__ input_scale, float* __restrict__ least) {
+  __shared__ float wave_sum[kGateThreads / kWave], wave_most[kGateThreads / kWave];
+  const int heads = (int)r.heads, h = blockIdx.x % heads, b = blockIdx.x / heads, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int slot = r.state_slots[b];
   if (slot < 0 || slot >= r.num_slots) return;
   const int t_begin = r.cu_seqlens[b], t_end = r.cu_seqlens[b + 1];
   float* const top = r.top + ((int64_t)slot * heads + h) * copies;
   float m = r.starts[b] > 0 ? top[0] : 0.f;
   const float input_bias = r.input_bias[h], forget_bias = r.forget_bias[h];
-  for (int t0 = t_begin; t0 < t_end; t0 += 256) {
+  for (int t0 = t_begin; t0 < t_end; t0 += 4 * kGateThreads) {
     float f[4], in[4], sum = 0.f, most = -INFINITY;
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
-      const int64_t t = t0 + 4 * lane + e;
+      const int64_t t = t0 + 4 * tid + e;
       f[e] = 0.f;
       in[e] = -INFINITY;      // behind the end: changes nothing
       if (t < t_end) {
@@ -686,23 +689,31 @@ __global__ __launch_bounds__(64) void matrix_memory_gates_kernel(const mops_hip_
         sum += sum_up;
       }
     }
-    float before = fmaxf(m + __shfl_up(sum, 1, 64), __shfl_up(most, 1, 64));
-    if (lane == 0) before = m;
+    if (lane == 63) {
+      wave_sum[wave] = sum;
+      wave_most[wave] = most;
+    }
+    __syncthreads();
+    float start = m;      // the maximum in front of this wave's tokens, then in front of this thread's
+    for (int w = 0; w < wave; ++w) start = fmaxf(start + wave_sum[w], wave_most[w]);
+    for (int w = 0; w < kGateThreads / kWave; ++w) m = fmaxf(m + wave_sum[w], wave_most[w]);
+    float before = fmaxf(start + __shfl_up(sum, 1, 64), __shfl_up(most, 1, 64));
+    if (lane == 0) before = start;
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       const float now = fmaxf(f[e] + before, in[e]);
-      const int64_t at = (int64_t)(t0 + 4 * lane + e) * heads + h;
-      if (t0 + 4 * lane + e < t_end) {
+      const int64_t at = (int64_t)(t0 + 4 * tid + e) * heads + h;
+      if (t0 + 4 * tid + e < t_end) {
         log_keep[at] = f[e] + before - now;
         input_scale[at] = expf(in[e] - now);
         least[at] = expf(-now);
       }
       before = now;
     }
-    m = __shfl(before, 63, 64);
+    __syncthreads();
   }
   if (t_end > t_begin)
-    for (int i = lane; i < copies; i += 64) top[i] = m;
+    for (int i = tid; i < copies; i += kGateThreads) top[i] = m;
 }
 
 // Heads of one workgroup: as many of a q/k group as fill its 128 value columns.
@@ -729,7 +740,7 @@ extern "C" int mops_hip_matrix_memory_gates(const mops_hip_recurrence* r, float*
       !input_scale || !least || !(r->gate_cap > 0.f) || r->heads <= 0 || r->vd <= 0 || r->gate_stride < r->heads || r->num_slots <= 0)
     return MOPS_HIP_EINVAL;
   if (r->batch * r->heads > 0x7fffffffLL) return MOPS_HIP_EUNSUPPORTED;
-  hipLaunchKernelGGL(matrix_memory_gates_kernel, dim3((unsigned)(r->batch * r->heads)), dim3(64), 0, (hipStream_t)stream, *r,
+  hipLaunchKernelGGL(matrix_memory_gates_kernel, dim3((unsigned)(r->batch * r->heads)), dim3(kGateThreads), 0, (hipStream_t)stream, *r,
                      (int)mops_hip_matrix_memory_copies(r->vd), log_keep, input_scale, least);
   return finish_launch();
 }

@@ -12,8 +12,7 @@
 //   delta_prepare_kernel   a wave per (chunk, head), all chunks in parallel: unit vectors, cumulative decays, A, P, T and W, left in memory
 //                          as the operands of the second kernel's products, lane by lane, so that it reads 16 bytes per lane in a row
 //   delta_scan_kernel      a wave per (sequence, head, 16 value columns) walks the chunks with S [d x 16] in its accumulators:
-//                          U = T V - W S, O^T = S^T q + U^T P^T, S <- 2^{L_15} S + k^T U.  No LDS and no barriers; an operand's next
-//                          value is loaded behind its last use
+//                          U = T V - W S, O^T = S^T q + U^T P^T, S <- 2^{L_15} S + k^T U; the waves of a workgroup share the operands
 //
 // A and P come apart into one factor per token on either side of a reference as in channel_chunks.hip: L_7 where t >= 8 > j, else the
 // middle of the half chunk both lie in (a decay below 2^-28 counts as 2^-28).  What is kept in 32 bits enters a product as the sum of two
@@ -277,26 +276,25 @@ __global__ __launch_bounds__(64 * WAVES) void delta_prepare_kernel(const DeltaCh
     put(Sh::kK + i, __builtin_bit_cast(u32x4, join(tile_block_columns(hi_tile, kPitch, 4 * jj, 16 * i, lane), tile_block_columns(lo_tile, kPitch, 4 * jj, 16 * i, lane))));
 }
 
-constexpr int most_waves(int dp) { return dp <= 128 ? 8 : 4; }      // of a workgroup of the second kernel
-
-template <int DP>
-__global__ __launch_bounds__(64 * most_waves(DP)) void delta_scan_kernel(const DeltaChunkArgs p) {
+// WAVES waves of 16 value columns each.  The operands of a chunk go through LDS, two buffers; two more chunks are on their way in
+// registers, so that a load has two chunks' time to come back.
+template <int DP, int WAVES>
+__global__ __launch_bounds__(64 * WAVES) void delta_scan_kernel(const DeltaChunkArgs p) {
   using Sh = DeltaShape<DP>;
-  constexpr int kS = Sh::kSteps, kI = Sh::kTiles;
+  constexpr int kS = Sh::kSteps, kI = Sh::kTiles, kThreads = 64 * WAVES, kLoads16 = (int)(Sh::kBytes / 16), kLoads = (kLoads16 + kThreads - 1) / kThreads;
+  extern __shared__ __align__(16) unsigned char smem[];
   const mops_hip_delta& a = p.a;
-  const int heads = (int)a.heads, vd = (int)a.vd, columns = (int)blockDim.x >> 2;      // of a workgroup
-  const int blocks = (vd + columns - 1) / columns;
+  const int heads = (int)a.heads, vd = (int)a.vd, blocks = (vd + 16 * WAVES - 1) / (16 * WAVES);
   // each XCD a contiguous run of items, so that the workgroups of a head share an L2
   const int total = (int)a.batch * heads * blocks, per_xcd = (total + 7) / 8;
   const int item = (blockIdx.x % 8) * per_xcd + blockIdx.x / 8;
   if ((int)blockIdx.x / 8 >= per_xcd || item >= total) return;
   const int h = item / blocks % heads, b = item / (blocks * heads);
-  const int lane = threadIdx.x & 63, n16 = lane & 15, jj = lane >> 4;
-  const int v0 = item % blocks * columns + ((int)threadIdx.x >> 6) * 16;
-  if (v0 >= vd) return;      // no barriers below
+  const int tid = threadIdx.x, lane = tid & 63, n16 = lane & 15, jj = lane >> 4;
+  const int v0 = item % blocks * 16 * WAVES + (tid >> 6) * 16;
   const int slot = a.state_slots[b], t_begin = a.cu_seqlens[b], t_end = a.cu_seqlens[b + 1];
   if (slot < 0 || slot >= a.num_slots || t_end <= t_begin) return;
-  const bool v_ok = v0 + n16 < vd;
+  const bool active = v0 < vd, v_ok = v0 + n16 < vd;
   const int v = v_ok ? v0 + n16 : vd - 1;
   float* const state = a.state + (((int64_t)slot * heads + h) * vd + v) * p.pitch;
   // S: tile i, element e = row d = 16 i + 4 jj + e, column v0 + n16
@@ -312,54 +310,41 @@ __global__ __launch_bounds__(64 * most_waves(DP)) void delta_scan_kernel(const D
   }
   const uint16_t* const vp = (const uint16_t*)a.v + (int64_t)h * vd + v;
   uint16_t* const op = (uint16_t*)a.out + (int64_t)h * vd + v0 + 4 * jj;
-
-  u32x4 wh[kS], wl[kS], qh[kS], ql[kS], kf[kI], pf, tf;
-  f32x4 dc[kI];
-  uint32_t vr[4];
-  const unsigned char* src = p.operands + ((int64_t)p.seq_chunks[b] * heads + h) * Sh::kBytes + lane * 16;
+  const int n_chunks = (t_end - t_begin + kDTokens - 1) / kDTokens;
+  const unsigned char* const src = p.operands + ((int64_t)p.seq_chunks[b] * heads + h) * Sh::kBytes;
   const int64_t step = heads * Sh::kBytes;
-  auto piece = [&](int i) { return load16(src + i * kPieceBytes); };
-  auto load_w = [&]() {
+
+  // a chunk on its way: this thread's pieces of the operands, and its wave's values
+  struct Flight {
+    u32x4 w[kLoads];
+    uint32_t v[4];
+  } even, odd;
+  auto fetch = [&](Flight& f, int chunk) {
+    chunk = chunk < n_chunks ? chunk : n_chunks - 1;
+    const unsigned char* from = src + chunk * step;
 #pragma unroll
-    for (int s = 0; s < kS; ++s) {
-      wh[s] = piece(Sh::kW + s);
-      wl[s] = piece(Sh::kW + kS + s);
+    for (int i = 0; i < kLoads; ++i) {
+      const int at = i * kThreads + tid;
+      f.w[i] = load16(from + 16 * (at < kLoads16 ? at : 0));
+    }
+    const int t0 = t_begin + chunk * kDTokens + 4 * jj;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) f.v[e] = vp[(int64_t)(t0 + e < t_end ? t0 + e : t_end - 1) * a.v_stride];
+  };
+  auto file = [&](const Flight& f, int buffer) {
+#pragma unroll
+    for (int i = 0; i < kLoads; ++i) {
+      const int at = i * kThreads + tid;
+      if ((i + 1) * kThreads <= kLoads16 || at < kLoads16) store16(smem + buffer * Sh::kBytes + 16 * at, f.w[i]);
     }
   };
-  auto load_q = [&]() {
-#pragma unroll
-    for (int s = 0; s < kS; ++s) {
-      qh[s] = piece(Sh::kQ + s);
-      ql[s] = piece(Sh::kQ + kS + s);
-    }
-  };
-  auto load_k = [&]() {
-#pragma unroll
-    for (int i = 0; i < kI; ++i) {
-      kf[i] = piece(Sh::kK + i);
-      dc[i] = *reinterpret_cast<const f32x4*>(src - lane * 16 + Sh::kPieces * kPieceBytes + (16 * i + 4 * jj) * 4);
-    }
-  };
-  auto load_v = [&](int t0) {
-#pragma unroll
-    for (int e = 0; e < 4; ++e) vr[e] = vp[(int64_t)(t0 + 4 * jj + e < t_end ? t0 + 4 * jj + e : t_end - 1) * a.v_stride];
-  };
-  load_v(t_begin);
-  tf = piece(Sh::kT);
-  load_w();
-  load_q();
-  pf = piece(Sh::kP);
-  load_k();
-  for (int t0 = t_begin; t0 < t_end; t0 += kDTokens) {
-    const bool more = t0 + kDTokens < t_end;
-    if (more) src += step;
-    const u32x2 vw = {vr[0] | vr[1] << 16, vr[2] | vr[3] << 16};
+  u32x2 vw, vw_next;
+  auto values = [&](const Flight& f) { return u32x2{f.v[0] | f.v[1] << 16, f.v[2] | f.v[3] << 16}; };
+  auto run = [&](int chunk, int buffer) {
+    const unsigned char* const ops = smem + buffer * Sh::kBytes;
+    auto piece = [&](int i) { return as_operand(load16(ops + i * kPieceBytes + lane * 16)); };
     f32x4 u = {0.f, 0.f, 0.f, 0.f}, u2 = u, o = u, o2 = u;
-    u = mfma16(as_operand(tf), as_operand(u32x4{vw[0], vw[1], vw[0], vw[1]}), u);
-    if (more) {
-      load_v(t0 + kDTokens);
-      tf = piece(Sh::kT);
-    }
+    u = mfma16(piece(Sh::kT), as_operand(u32x4{vw[0], vw[1], vw[0], vw[1]}), u);
 #pragma unroll
     for (int s = 0; s < kS; ++s) {
       float x[8];
@@ -370,36 +355,34 @@ __global__ __launch_bounds__(64 * most_waves(DP)) void delta_scan_kernel(const D
       }
       bf16x8 hi, lo;
       split8(x, hi, lo);
-      u = mfma16(as_operand(wh[s]), hi, u);
-      o = mfma16(hi, as_operand(qh[s]), o);
-      u2 = mfma16(as_operand(wh[s]), lo, u2);
-      o2 = mfma16(hi, as_operand(ql[s]), o2);
-      u = mfma16(as_operand(wl[s]), hi, u);
-      o = mfma16(lo, as_operand(qh[s]), o);
-    }
-    if (more) {
-      load_w();
-      load_q();
+      const bf16x8 wh = piece(Sh::kW + s), wl = piece(Sh::kW + kS + s), qh = piece(Sh::kQ + s), ql = piece(Sh::kQ + kS + s);
+      u = mfma16(wh, hi, u);
+      o = mfma16(hi, qh, o);
+      u2 = mfma16(wh, lo, u2);
+      o2 = mfma16(hi, ql, o2);
+      u = mfma16(wl, hi, u);
+      o = mfma16(lo, qh, o);
     }
     float uu[4];
 #pragma unroll
     for (int e = 0; e < 4; ++e) uu[e] = u[e] + u2[e];
     const u32x4 uw = split4(uu);
     const bf16x8 u_high = high_twice(uw), u_low = low_once(uw);
-    o = mfma16(u_high, as_operand(pf), o);
-    o2 = mfma16(u_low, as_operand(pf), o2);
-    if (more) pf = piece(Sh::kP);
 #pragma unroll
     for (int i = 0; i < kI; ++i) {
+      const f32x4 keep = *reinterpret_cast<const f32x4*>(ops + Sh::kPieces * kPieceBytes + (16 * i + 4 * jj) * 4);
+      const bf16x8 k = piece(Sh::kK + i);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) st[i][e] *= dc[i][e];
-      st[i] = mfma16(as_operand(kf[i]), u_high, st[i]);
+      for (int e = 0; e < 4; ++e) st[i][e] *= keep[e];
+      st[i] = mfma16(k, u_high, st[i]);
+      st[i] = mfma16(k, u_low, st[i]);
     }
-#pragma unroll
-    for (int i = 0; i < kI; ++i) st[i] = mfma16(as_operand(kf[i]), u_low, st[i]);
-    if (more) load_k();
-    if (t0 + n16 < t_end) {
-      uint16_t* const row = op + (int64_t)(t0 + n16) * a.out_stride;
+    const bf16x8 weights = piece(Sh::kP);
+    o = mfma16(u_high, weights, o);
+    o2 = mfma16(u_low, weights, o2);
+    const int t = t_begin + chunk * kDTokens + n16;
+    if (t < t_end) {
+      uint16_t* const row = op + (int64_t)t * a.out_stride;
       const u32x2 w = {pack_bf16x2(o[0] + o2[0], o[1] + o2[1]), pack_bf16x2(o[2] + o2[2], o[3] + o2[3])};
       if (p.vec && v0 + 4 * jj < vd) {
         *reinterpret_cast<u32x2*>(row) = w;
@@ -409,6 +392,26 @@ __global__ __launch_bounds__(64 * most_waves(DP)) void delta_scan_kernel(const D
           if (v0 + 4 * jj + e < vd) row[e] = (uint16_t)(w[e >> 1] >> (16 * (e & 1)));
       }
     }
+  };
+  // one barrier per chunk: the chunk's buffer is filled, and everybody is done with the other one.  Only LDS is waited for.
+  auto turn = [&](Flight& f, int chunk) {
+    vw = vw_next;
+    asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+    if (chunk + 1 < n_chunks) {
+      file(f, (chunk + 1) & 1);
+      vw_next = values(f);
+      fetch(f, chunk + 3);
+    }
+    if (active) run(chunk, chunk & 1);
+  };
+  fetch(even, 0);
+  fetch(odd, 1);
+  file(even, 0);
+  vw_next = values(even);
+  fetch(even, 2);
+  for (int chunk = 0; chunk < n_chunks; chunk += 2) {
+    turn(odd, chunk);
+    if (chunk + 1 < n_chunks) turn(even, chunk + 1);
   }
   if (!v_ok) return;
 #pragma unroll
@@ -424,18 +427,25 @@ static int64_t operand_bytes(int64_t d) {
   return d <= 128 ? DeltaShape<128>::kBytes : DeltaShape<256>::kBytes;
 }
 
+template <int DP, int WAVES>
+static int launch_scan(const DeltaChunkArgs& p, hipStream_t s) {
+  constexpr int kLds = (int)(2 * DeltaShape<DP>::kBytes);
+  static const hipError_t lds = hipFuncSetAttribute(reinterpret_cast<const void*>(&delta_scan_kernel<DP, WAVES>), hipFuncAttributeMaxDynamicSharedMemorySize, kLds);
+  if (lds != hipSuccess) return record_hip_error(lds);
+  const int64_t total = p.a.batch * p.a.heads * ((p.a.vd + 16 * WAVES - 1) / (16 * WAVES));
+  hipLaunchKernelGGL((delta_scan_kernel<DP, WAVES>), dim3((unsigned)((total + 7) / 8 * 8)), dim3(64 * WAVES), kLds, s, p);
+  return finish_launch();
+}
+
 template <int DP>
 static int launch_delta_chunks(const DeltaChunkArgs& p, hipStream_t s) {
   constexpr int kWaves = DP <= 128 ? 4 : 2;
   const int64_t items = (int64_t)p.num_chunks * p.a.heads;
   hipLaunchKernelGGL((delta_prepare_kernel<DP, kWaves>), dim3((unsigned)((items + kWaves - 1) / kWaves)), dim3(64 * kWaves), 0, s, p);
-  // as many waves in a workgroup as share a head's operands, fewer where that leaves most of the chip idle
+  // eight waves share a head's operands, four where eight leave most of the chip idle or the registers do not allow them
   const int64_t tiles = (p.a.vd + 15) / 16, rows = p.a.batch * p.a.heads;
-  int waves = tiles < most_waves(DP) ? (int)tiles : most_waves(DP);
-  if (rows * ((tiles + waves - 1) / waves) < 256 && waves > 4) waves = 4;
-  const int64_t total = rows * ((tiles + waves - 1) / waves);
-  hipLaunchKernelGGL((delta_scan_kernel<DP>), dim3((unsigned)((total + 7) / 8 * 8)), dim3(64 * waves), 0, s, p);
-  return finish_launch();
+  const bool eight = DP <= 128 && tiles > 4 && rows * ((tiles + 7) / 8) >= 192;
+  return eight ? launch_scan<DP, DP <= 128 ? 8 : 4>(p, s) : launch_scan<DP, 4>(p, s);
 }
 
 }  // namespace mops
