@@ -523,12 +523,15 @@ int mops_hip_delta_rule(const mops_hip_delta* a, void* stream);
 /*
  * The same for portions of many tokens, 16 tokens at a time on the matrix cores (csrc/delta_chunks.hip): bf16, d <= 256, cu_seqlens given,
  * no convolution; a decay below 2^-28 counts as 2^-28.  chunks: int32 [num_chunks][2] = (first token, tokens <= 16): every sequence cut
- * from its first token on, in order; seq_chunks: int32 [batch + 1] bounds each sequence's.  workspace: device scratch of at least
- * mops_hip_delta_chunks_workspace_bytes(...), private to the call until it completes.
+ * from its first token on, in order.  segments: int32 [num_segments][4] = (sequence, first token, one past the last, number of its first
+ * chunk): runs of whole chunks that cover every sequence, in order; seq_segments: int32 [batch + 1] bounds each sequence's.  One segment
+ * per sequence, or more where that leaves the chip idle (mops_hip_delta_chunks_workgroups: what one segment gives).  workspace: device
+ * scratch of at least mops_hip_delta_chunks_workspace_bytes(...), private to the call until it completes.
  */
-int64_t mops_hip_delta_chunks_workspace_bytes(int64_t num_chunks, int64_t heads, int64_t d);
-int mops_hip_delta_chunks(const mops_hip_delta* a, const int32_t* chunks, int64_t num_chunks, const int32_t* seq_chunks, void* workspace,
-                          int64_t workspace_bytes, void* stream);
+int64_t mops_hip_delta_chunks_workgroups(int64_t heads, int64_t vd);
+int64_t mops_hip_delta_chunks_workspace_bytes(int64_t num_chunks, int64_t num_segments, int64_t batch, int64_t heads, int64_t d, int64_t vd);
+int mops_hip_delta_chunks(const mops_hip_delta* a, const int32_t* chunks, int64_t num_chunks, const int32_t* segments, int64_t num_segments,
+                          const int32_t* seq_segments, void* workspace, int64_t workspace_bytes, void* stream);
 
 /*
  * out[t, c] = silu(bias[c] (bias may be NULL) + sum over lags l < taps of weight[taps-1-l, c] * x(position - l)[c]) for packed portions.

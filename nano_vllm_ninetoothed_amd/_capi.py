@@ -150,8 +150,9 @@ SIGNATURES = {
     "mops_hip_relu_glu": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_int, c_int64, c_int64, c_void_p]),
     "mops_hip_matrix_memory_copies": (c_int64, [c_int64]),
     "mops_hip_delta_rule": (c_int, [POINTER(Delta), c_void_p]),
-    "mops_hip_delta_chunks_workspace_bytes": (c_int64, [c_int64] * 3),
-    "mops_hip_delta_chunks": (c_int, [POINTER(Delta), c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_void_p]),
+    "mops_hip_delta_chunks_workgroups": (c_int64, [c_int64] * 2),
+    "mops_hip_delta_chunks_workspace_bytes": (c_int64, [c_int64] * 6),
+    "mops_hip_delta_chunks": (c_int, [POINTER(Delta), c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_void_p]),
     "mops_hip_matrix_memory_gates": (c_int, [POINTER(Recurrence)] + [c_void_p] * 4),
     "mops_hip_recurrence_state_pitch": (c_int64, [c_int64]),
     "mops_hip_decayed_recurrence": (c_int, [POINTER(Recurrence), c_void_p]),

@@ -589,11 +589,11 @@ def fedovik_recurrences(t):
             nbytes=2.0 * bs * n * dd * 4 + bs * n * (12 + 24), like=like)
         xs, ldT, oT, betas = rnd(T, 3 * n), -torch.exp(t.f32(T, n) - 3), torch.empty((T, n), dtype=torch.bfloat16, device=dev), rnd(T, heads)
         for nseq in (16, 1):
-            chunks, ends = (i32(v) for v in R.delta_chunk_list([T // nseq] * nseq))
+            cuts = [i32(v) for v in R.delta_cuts([T // nseq] * nseq, heads, dd)]
             cu, zero = i32(list(range(0, T + 1, T // nseq))), torch.zeros(nseq, dtype=torch.int32, device=dev)
             # least arithmetic at 16 tokens a chunk: the products inside it, the triangular system, state in and out and what a key finds there
             add("delta_chunks", f"{nseq} x {T // nseq}, {shape}", lambda: _events(lambda: op("delta_chunks")(
-                xs[:, :n], xs[:, n:2 * n], xs[:, 2 * n:], oT, state, sl[:nseq], zero, heads, heads, dd, dd, chunks, ends, cu_seqlens=cu, log_decay=ldT, beta=betas, **opts), 20, 50),
+                xs[:, :n], xs[:, n:2 * n], xs[:, 2 * n:], oT, state, sl[:nseq], zero, heads, heads, dd, dd, *cuts, cu_seqlens=cu, log_decay=ldT, beta=betas, **opts), 20, 50),
                 flops=T * heads * (17.0 * 4 * dd + 6.0 * dd * dd), nbytes=T * n * 12.0, like=f"channel_chunks {nseq} x {T // nseq}, {shape}")
         del xs, ldT, oT
         copies = R.matrix_memory_copies(dd)

@@ -14,6 +14,12 @@
 //   delta_scan_kernel      a wave per (sequence, head, 16 value columns) walks the chunks with S [d x 16] in its accumulators:
 //                          U = T V - W S, O^T = S^T q + U^T P^T, S <- 2^{L_15} S + k^T U; the waves of a workgroup share the operands
 //
+// A sequence is one segment when sequences and heads fill the chip.  Otherwise it is cut, and three launches walk the segments side by side:
+//   states from zero   U = T V - W S without outputs, and beside the value columns d more with V = 0 that start from the identity: what the
+//                      segment makes of the state in front of it is S <- M S + C
+//   delta_join_kernel  S at the start of every segment, one after the other, and the last state into the sequence's slot
+//   outputs            delta_scan_kernel from these
+//
 // A and P come apart into one factor per token on either side of a reference as in channel_chunks.hip: L_7 where t >= 8 > j, else the
 // middle of the half chunk both lie in (a decay below 2^-28 counts as 2^-28).  What is kept in 32 bits enters a product as the sum of two
 // bf16 numbers; where a product is 16 deep the two halves of the 32 deep instruction hold them.
@@ -30,17 +36,23 @@ constexpr int kPieceBytes = 1024;      // an operand of a wave: 16 bytes per lan
 struct DeltaChunkArgs {
   mops_hip_delta a;
   const int32_t* chunks;        // [n][2]: first token, tokens
-  const int32_t* seq_chunks;    // [batch + 1]
-  int num_chunks, pitch;
-  unsigned char* operands;      // per (chunk, head): W hi, W lo, Q hi, Q lo [d / 32], K [d / 16], P, T as pieces, then 2^{L_15} float [d]
+  const int32_t* segments;      // [n][4]: sequence, first token, one past the last, first chunk
+  const int32_t* seq_segments;  // [batch + 1]
+  int num_chunks, num_segments, pitch;
+  unsigned char* operands;      // per (chunk, head): Q hi, Q lo [d / 32], P, W hi, W lo, K [d / 16], T as pieces, then 2^{L_15} float [d]
+  float* seg_state;             // [segments][heads][vd][pitch]: C, then the state at the start; nullptr: one segment per sequence
+  unsigned char* seg_map;       // [segments][heads]: M hi, M lo as pieces [d / 16][d / 32]
   bool vec;
 };
 
 template <int DP>
 struct DeltaShape {
   static constexpr int kSteps = DP / 32, kTiles = DP / 16;
-  static constexpr int kW = 0, kQ = 2 * kSteps, kK = 4 * kSteps, kP = kK + kTiles, kT = kP + 1, kPieces = kT + 1;
+  static constexpr int kQ = 0, kP = 2 * kSteps, kW = kP + 1, kK = kW + 2 * kSteps, kT = kK + kTiles, kPieces = kT + 1;
   static constexpr int64_t kBytes = kPieces * kPieceBytes + DP * 4;
+  static constexpr int64_t kMapBytes = 2 * kTiles * kSteps * kPieceBytes;
+  // the operands that a pass reads are in one run
+  static constexpr int from(bool states) { return states ? kW * kPieceBytes : 0; }
 };
 
 template <int N>
@@ -278,40 +290,44 @@ __global__ __launch_bounds__(64 * WAVES) void delta_prepare_kernel(const DeltaCh
 
 // WAVES waves of 16 value columns each.  The operands of a chunk go through LDS, two buffers; two more chunks are on their way in
 // registers, so that a load has two chunks' time to come back.
-template <int DP, int WAVES>
+template <int DP, int WAVES, bool STATES>
 __global__ __launch_bounds__(64 * WAVES) void delta_scan_kernel(const DeltaChunkArgs p) {
   using Sh = DeltaShape<DP>;
-  constexpr int kS = Sh::kSteps, kI = Sh::kTiles, kThreads = 64 * WAVES, kLoads16 = (int)(Sh::kBytes / 16), kLoads = (kLoads16 + kThreads - 1) / kThreads;
+  constexpr int kS = Sh::kSteps, kI = Sh::kTiles, kThreads = 64 * WAVES, kFrom = Sh::from(STATES);
+  constexpr int kBuffer = (int)Sh::kBytes - kFrom, kLoads16 = kBuffer / 16, kLoads = (kLoads16 + kThreads - 1) / kThreads;
   extern __shared__ __align__(16) unsigned char smem[];
   const mops_hip_delta& a = p.a;
-  const int heads = (int)a.heads, vd = (int)a.vd, blocks = (vd + 16 * WAVES - 1) / (16 * WAVES);
+  const int heads = (int)a.heads, vd = (int)a.vd, value_columns = (vd + 15) / 16 * 16;
+  const int columns = value_columns + (STATES ? ((int)a.d + 15) / 16 * 16 : 0), blocks = (columns + 16 * WAVES - 1) / (16 * WAVES);
   // each XCD a contiguous run of items, so that the workgroups of a head share an L2
-  const int total = (int)a.batch * heads * blocks, per_xcd = (total + 7) / 8;
+  const int total = p.num_segments * heads * blocks, per_xcd = (total + 7) / 8;
   const int item = (blockIdx.x % 8) * per_xcd + blockIdx.x / 8;
   if ((int)blockIdx.x / 8 >= per_xcd || item >= total) return;
-  const int h = item / blocks % heads, b = item / (blocks * heads);
+  const int h = item / blocks % heads, seg = item / (blocks * heads);
   const int tid = threadIdx.x, lane = tid & 63, n16 = lane & 15, jj = lane >> 4;
   const int v0 = item % blocks * 16 * WAVES + (tid >> 6) * 16;
-  const int slot = a.state_slots[b], t_begin = a.cu_seqlens[b], t_end = a.cu_seqlens[b + 1];
+  const int b = p.segments[4 * seg], t_begin = p.segments[4 * seg + 1], t_end = p.segments[4 * seg + 2], first_chunk = p.segments[4 * seg + 3];
+  const int slot = a.state_slots[b];
   if (slot < 0 || slot >= a.num_slots || t_end <= t_begin) return;
-  const bool active = v0 < vd, v_ok = v0 + n16 < vd;
+  const bool active = v0 < columns, v_ok = v0 + n16 < vd, maps = STATES && v0 >= value_columns;      // maps: columns of M
   const int v = v_ok ? v0 + n16 : vd - 1;
-  float* const state = a.state + (((int64_t)slot * heads + h) * vd + v) * p.pitch;
+  float* const state = (p.seg_state ? p.seg_state + ((int64_t)seg * heads + h) * vd * p.pitch : a.state + ((int64_t)slot * heads + h) * vd * p.pitch) +
+                       (int64_t)v * p.pitch;
   // S: tile i, element e = row d = 16 i + 4 jj + e, column v0 + n16
   f32x4 st[kI];
-  const bool load_state = a.starts[b] > 0;
+  const bool load_state = !STATES && (p.seg_state || a.starts[b] > 0);
 #pragma unroll
   for (int i = 0; i < kI; ++i) {
     const int d = 16 * i + 4 * jj;
     const bool ok = load_state && d < p.pitch;
     const f32x4 w = *reinterpret_cast<const f32x4*>(state + (ok ? d : 0));
 #pragma unroll
-    for (int e = 0; e < 4; ++e) st[i][e] = ok ? w[e] : 0.f;
+    for (int e = 0; e < 4; ++e) st[i][e] = ok ? w[e] : (maps && d + e == v0 - value_columns + n16 ? 1.f : 0.f);
   }
   const uint16_t* const vp = (const uint16_t*)a.v + (int64_t)h * vd + v;
   uint16_t* const op = (uint16_t*)a.out + (int64_t)h * vd + v0 + 4 * jj;
   const int n_chunks = (t_end - t_begin + kDTokens - 1) / kDTokens;
-  const unsigned char* const src = p.operands + ((int64_t)p.seq_chunks[b] * heads + h) * Sh::kBytes;
+  const unsigned char* const src = p.operands + ((int64_t)first_chunk * heads + h) * Sh::kBytes + kFrom;
   const int64_t step = heads * Sh::kBytes;
 
   // a chunk on its way: this thread's pieces of the operands, and its wave's values
@@ -335,13 +351,13 @@ __global__ __launch_bounds__(64 * WAVES) void delta_scan_kernel(const DeltaChunk
 #pragma unroll
     for (int i = 0; i < kLoads; ++i) {
       const int at = i * kThreads + tid;
-      if ((i + 1) * kThreads <= kLoads16 || at < kLoads16) store16(smem + buffer * Sh::kBytes + 16 * at, f.w[i]);
+      if ((i + 1) * kThreads <= kLoads16 || at < kLoads16) store16(smem + buffer * kBuffer + 16 * at, f.w[i]);
     }
   };
   u32x2 vw, vw_next;
-  auto values = [&](const Flight& f) { return u32x2{f.v[0] | f.v[1] << 16, f.v[2] | f.v[3] << 16}; };
+  auto values = [&](const Flight& f) { return maps ? u32x2{0u, 0u} : u32x2{f.v[0] | f.v[1] << 16, f.v[2] | f.v[3] << 16}; };
   auto run = [&](int chunk, int buffer) {
-    const unsigned char* const ops = smem + buffer * Sh::kBytes;
+    const unsigned char* const ops = smem + buffer * kBuffer - kFrom;
     auto piece = [&](int i) { return as_operand(load16(ops + i * kPieceBytes + lane * 16)); };
     f32x4 u = {0.f, 0.f, 0.f, 0.f}, u2 = u, o = u, o2 = u;
     u = mfma16(piece(Sh::kT), as_operand(u32x4{vw[0], vw[1], vw[0], vw[1]}), u);
@@ -355,13 +371,16 @@ __global__ __launch_bounds__(64 * WAVES) void delta_scan_kernel(const DeltaChunk
       }
       bf16x8 hi, lo;
       split8(x, hi, lo);
-      const bf16x8 wh = piece(Sh::kW + s), wl = piece(Sh::kW + kS + s), qh = piece(Sh::kQ + s), ql = piece(Sh::kQ + kS + s);
+      const bf16x8 wh = piece(Sh::kW + s), wl = piece(Sh::kW + kS + s);
       u = mfma16(wh, hi, u);
-      o = mfma16(hi, qh, o);
       u2 = mfma16(wh, lo, u2);
-      o2 = mfma16(hi, ql, o2);
+      if (!STATES) {
+        const bf16x8 qh = piece(Sh::kQ + s), ql = piece(Sh::kQ + kS + s);
+        o = mfma16(hi, qh, o);
+        o2 = mfma16(hi, ql, o2);
+        o = mfma16(lo, qh, o);
+      }
       u = mfma16(wl, hi, u);
-      o = mfma16(lo, qh, o);
     }
     float uu[4];
 #pragma unroll
@@ -377,6 +396,7 @@ __global__ __launch_bounds__(64 * WAVES) void delta_scan_kernel(const DeltaChunk
       st[i] = mfma16(k, u_high, st[i]);
       st[i] = mfma16(k, u_low, st[i]);
     }
+    if (STATES) return;
     const bf16x8 weights = piece(Sh::kP);
     o = mfma16(u_high, weights, o);
     o2 = mfma16(u_low, weights, o2);
@@ -413,10 +433,113 @@ __global__ __launch_bounds__(64 * WAVES) void delta_scan_kernel(const DeltaChunk
     turn(odd, chunk);
     if (chunk + 1 < n_chunks) turn(even, chunk + 1);
   }
-  if (!v_ok) return;
+  if (maps) {      // rows of M as operands: this wave's sixteen columns are half of a step, turned in the LDS that nobody reads any more
+    __syncthreads();
+    if (!active) return;
+    uint16_t* const hi_tile = reinterpret_cast<uint16_t*>(smem) + (tid >> 6) * 2 * 16 * 24;      // [column][16 rows], pitch 24
+    uint16_t* const lo_tile = hi_tile + 16 * 24;
+    unsigned char* const dst = p.seg_map + ((int64_t)seg * heads + h) * Sh::kMapBytes;
+    const int m0 = v0 - value_columns, s = m0 / 32, half = m0 / 16 & 1;
+#pragma unroll
+    for (int i = 0; i < kI; ++i) {
+      const float x[4] = {st[i][0], st[i][1], st[i][2], st[i][3]};
+      const u32x4 w = split4(x);
+      *reinterpret_cast<u32x2*>(hi_tile + n16 * 24 + 4 * jj) = u32x2{w[0], w[1]};
+      *reinterpret_cast<u32x2*>(lo_tile + n16 * 24 + 4 * jj) = u32x2{w[2], w[3]};
+      wave_sync();
+      const u32x2 kh = __builtin_bit_cast(u32x2, tile_block_columns(hi_tile, 24, 4 * jj, 0, lane)), kl = __builtin_bit_cast(u32x2, tile_block_columns(lo_tile, 24, 4 * jj, 0, lane));
+      wave_sync();
+      unsigned char* const at = dst + (i * kS + s) * kPieceBytes + lane * 16 + 8 * half;
+      *reinterpret_cast<u32x2*>(at) = kh;
+      *reinterpret_cast<u32x2*>(at + kI * kS * kPieceBytes) = kl;
+    }
+    return;
+  }
+  if (STATES) __syncthreads();      // beside the one above
+  if (!v_ok || (!STATES && p.seg_state)) return;
 #pragma unroll
   for (int i = 0; i < kI; ++i)
     if (16 * i + 4 * jj < p.pitch) *reinterpret_cast<f32x4*>(state + 16 * i + 4 * jj) = st[i];
+}
+
+// A workgroup per (sequence, head, 16 value columns): S <- M S + C over the segments of the sequence.  Its waves share the rows of S; all of
+// S goes round through LDS as operands.
+constexpr int join_waves(int dp) { return dp / 16 < 4 ? dp / 16 : 4; }
+
+template <int DP>
+__global__ __launch_bounds__(64 * join_waves(DP)) void delta_join_kernel(const DeltaChunkArgs p) {
+  using Sh = DeltaShape<DP>;
+  constexpr int kS = Sh::kSteps, kI = Sh::kTiles, kMine = kI / join_waves(DP);
+  __shared__ __align__(16) unsigned char ops[2][2][kS][kPieceBytes];      // two of them by turns: S hi, S lo
+  const mops_hip_delta& a = p.a;
+  const int heads = (int)a.heads, vd = (int)a.vd, blocks = (vd + 15) / 16;
+  const int h = blockIdx.x / blocks % heads, b = blockIdx.x / blocks / heads;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, n16 = lane & 15, jj = lane >> 4, v0 = blockIdx.x % blocks * 16;
+  const int slot = a.state_slots[b];
+  if (slot < 0 || slot >= a.num_slots) return;
+  const bool v_ok = v0 + n16 < vd, load_state = a.starts[b] > 0;
+  const int v = v_ok ? v0 + n16 : vd - 1;
+  float* const state = a.state + (((int64_t)slot * heads + h) * vd + v) * p.pitch;
+  auto row = [&](int i) { return 16 * (wave * kMine + i) + 4 * jj; };      // of element 0 of this wave's tile i
+  auto read = [&](const float* from, int i, bool on) {
+    const bool ok = on && row(i) < p.pitch;
+    const f32x4 w = *reinterpret_cast<const f32x4*>(from + (ok ? row(i) : 0));
+    return ok ? w : f32x4{0.f, 0.f, 0.f, 0.f};
+  };
+  f32x4 st[kMine], next[kMine];
+  u32x4 mh[kMine][kS], ml[kMine][kS];
+  auto part = [&](int seg) { return p.seg_state + (((int64_t)seg * heads + h) * vd + v) * p.pitch; };
+  auto fetch = [&](int seg) {
+    const unsigned char* const map = p.seg_map + ((int64_t)seg * heads + h) * Sh::kMapBytes + lane * 16;
+#pragma unroll
+    for (int i = 0; i < kMine; ++i) {
+      next[i] = read(part(seg), i, true);
+#pragma unroll
+      for (int s = 0; s < kS; ++s) {
+        const int at = (wave * kMine + i) * kS + s;
+        mh[i][s] = load16(map + at * kPieceBytes);
+        ml[i][s] = load16(map + (kI * kS + at) * kPieceBytes);
+      }
+    }
+  };
+#pragma unroll
+  for (int i = 0; i < kMine; ++i) st[i] = read(state, i, load_state);
+  const int first = p.seq_segments[b], end = p.seq_segments[b + 1];
+  if (first < end) fetch(first);
+  for (int seg = first; seg < end; ++seg) {
+    unsigned char(*const now)[kS][kPieceBytes] = ops[(seg - first) & 1];
+#pragma unroll
+    for (int i = 0; i < kMine; ++i) {
+      const float x[4] = {st[i][0], st[i][1], st[i][2], st[i][3]};
+      const u32x4 w = split4(x);
+      const int tile = wave * kMine + i, at = lane * 16 + 8 * (tile & 1);
+      *reinterpret_cast<u32x2*>(&now[0][tile >> 1][at]) = u32x2{w[0], w[1]};
+      *reinterpret_cast<u32x2*>(&now[1][tile >> 1][at]) = u32x2{w[2], w[3]};
+      if (v_ok && row(i) < p.pitch) *reinterpret_cast<f32x4*>(part(seg) + row(i)) = st[i];      // its lane has read C from there
+    }
+    __syncthreads();
+#pragma unroll
+    for (int s = 0; s < kS; ++s) {
+      const bf16x8 hi = as_operand(load16(&now[0][s][lane * 16])), lo = as_operand(load16(&now[1][s][lane * 16]));
+      const bool low = 32 * s < (int)a.d, high = 32 * s + 16 < (int)a.d;      // halves of the step that were written
+#pragma unroll
+      for (int i = 0; i < kMine; ++i) {
+        u32x4 x = mh[i][s], y = ml[i][s];
+        if (!low) x[0] = x[1] = y[0] = y[1] = 0u;
+        if (!high) x[2] = x[3] = y[2] = y[3] = 0u;
+        next[i] = mfma16(as_operand(x), hi, next[i]);
+        next[i] = mfma16(as_operand(x), lo, next[i]);
+        next[i] = mfma16(as_operand(y), hi, next[i]);
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < kMine; ++i) st[i] = next[i];
+    if (seg + 1 < end) fetch(seg + 1);
+  }
+  if (!v_ok) return;
+#pragma unroll
+  for (int i = 0; i < kMine; ++i)
+    if (row(i) < p.pitch) *reinterpret_cast<f32x4*>(state + row(i)) = st[i];
 }
 
 int check_delta(const mops_hip_delta* a);      // delta_rule.hip
@@ -427,51 +550,75 @@ static int64_t operand_bytes(int64_t d) {
   return d <= 128 ? DeltaShape<128>::kBytes : DeltaShape<256>::kBytes;
 }
 
-template <int DP, int WAVES>
+static int64_t map_bytes(int64_t d) {
+  if (d <= 32) return DeltaShape<32>::kMapBytes;
+  if (d <= 64) return DeltaShape<64>::kMapBytes;
+  return d <= 128 ? DeltaShape<128>::kMapBytes : DeltaShape<256>::kMapBytes;
+}
+
+template <int DP, int WAVES, bool STATES>
 static int launch_scan(const DeltaChunkArgs& p, hipStream_t s) {
-  constexpr int kLds = (int)(2 * DeltaShape<DP>::kBytes);
-  static const hipError_t lds = hipFuncSetAttribute(reinterpret_cast<const void*>(&delta_scan_kernel<DP, WAVES>), hipFuncAttributeMaxDynamicSharedMemorySize, kLds);
+  constexpr int kLds = (int)(2 * (DeltaShape<DP>::kBytes - DeltaShape<DP>::from(STATES)));
+  static const hipError_t lds = hipFuncSetAttribute(reinterpret_cast<const void*>(&delta_scan_kernel<DP, WAVES, STATES>), hipFuncAttributeMaxDynamicSharedMemorySize, kLds);
   if (lds != hipSuccess) return record_hip_error(lds);
-  const int64_t total = p.a.batch * p.a.heads * ((p.a.vd + 16 * WAVES - 1) / (16 * WAVES));
-  hipLaunchKernelGGL((delta_scan_kernel<DP, WAVES>), dim3((unsigned)((total + 7) / 8 * 8)), dim3(64 * WAVES), kLds, s, p);
+  const int64_t columns = (p.a.vd + 15) / 16 * 16 + (STATES ? (p.a.d + 15) / 16 * 16 : 0);
+  const int64_t total = p.num_segments * p.a.heads * ((columns + 16 * WAVES - 1) / (16 * WAVES));
+  hipLaunchKernelGGL((delta_scan_kernel<DP, WAVES, STATES>), dim3((unsigned)((total + 7) / 8 * 8)), dim3(64 * WAVES), kLds, s, p);
   return finish_launch();
 }
 
 template <int DP>
 static int launch_delta_chunks(const DeltaChunkArgs& p, hipStream_t s) {
-  constexpr int kWaves = DP <= 128 ? 4 : 2;
+  constexpr int kWaves = DP <= 128 ? 4 : 2, kMany = DP <= 128 ? 8 : 4;
   const int64_t items = (int64_t)p.num_chunks * p.a.heads;
   hipLaunchKernelGGL((delta_prepare_kernel<DP, kWaves>), dim3((unsigned)((items + kWaves - 1) / kWaves)), dim3(64 * kWaves), 0, s, p);
   // eight waves share a head's operands, four where eight leave most of the chip idle or the registers do not allow them
-  const int64_t tiles = (p.a.vd + 15) / 16, rows = p.a.batch * p.a.heads;
-  const bool eight = DP <= 128 && tiles > 4 && rows * ((tiles + 7) / 8) >= 192;
-  return eight ? launch_scan<DP, DP <= 128 ? 8 : 4>(p, s) : launch_scan<DP, 4>(p, s);
+  const int64_t tiles = (p.a.vd + 15) / 16, rows = p.num_segments * p.a.heads;
+  if (p.seg_state) {
+    const int st = launch_scan<DP, kMany, true>(p, s);
+    if (st != MOPS_HIP_OK) return st;
+    hipLaunchKernelGGL((delta_join_kernel<DP>), dim3((unsigned)(p.a.batch * p.a.heads * tiles)), dim3(64 * join_waves(DP)), 0, s, p);
+  }
+  return tiles > 4 && rows * ((tiles + 7) / 8) >= 192 ? launch_scan<DP, kMany, false>(p, s) : launch_scan<DP, 4, false>(p, s);
 }
 
 }  // namespace mops
 
-extern "C" int64_t mops_hip_delta_chunks_workspace_bytes(int64_t num_chunks, int64_t heads, int64_t d) {
-  return num_chunks <= 0 || heads <= 0 || d <= 0 || d > 256 ? 0 : num_chunks * heads * mops::operand_bytes(d);
+extern "C" int64_t mops_hip_delta_chunks_workspace_bytes(int64_t num_chunks, int64_t num_segments, int64_t batch, int64_t heads, int64_t d, int64_t vd) {
+  using namespace mops;
+  if (num_chunks <= 0 || heads <= 0 || d <= 0 || d > 256 || vd <= 0) return 0;
+  const int64_t cut = num_segments > batch ? num_segments * heads * (map_bytes(d) + (vd * mops_hip_recurrence_state_pitch(d) * 4 + 15) / 16 * 16) : 0;
+  return num_chunks * heads * operand_bytes(d) + cut;
 }
 
-extern "C" int mops_hip_delta_chunks(const mops_hip_delta* a, const int32_t* chunks, int64_t num_chunks, const int32_t* seq_chunks, void* workspace,
-                                     int64_t workspace_bytes, void* stream) {
+extern "C" int64_t mops_hip_delta_chunks_workgroups(int64_t heads, int64_t vd) {
+  return heads <= 0 || vd <= 0 ? MOPS_HIP_EINVAL : heads * ((vd + 127) / 128);
+}
+
+extern "C" int mops_hip_delta_chunks(const mops_hip_delta* a, const int32_t* chunks, int64_t num_chunks, const int32_t* segments, int64_t num_segments,
+                                     const int32_t* seq_segments, void* workspace, int64_t workspace_bytes, void* stream) {
   using namespace mops;
   const int pre = check_delta(a);
   if (pre != 1) return pre;
   if (a->dtype != MOPS_HIP_BF16 || a->d > 256 || a->conv_weight) return MOPS_HIP_EUNSUPPORTED;
-  if (num_chunks < 0 || !chunks || !seq_chunks || !a->cu_seqlens) return MOPS_HIP_EINVAL;
-  if (num_chunks == 0) return MOPS_HIP_OK;
-  if (num_chunks * a->heads > 0x7fffffffLL || a->batch * a->heads * ((a->vd + 15) / 16) > 0x3fffffffLL) return MOPS_HIP_EUNSUPPORTED;
-  if (!workspace || workspace_bytes < mops_hip_delta_chunks_workspace_bytes(num_chunks, a->heads, a->d)) return MOPS_HIP_EWORKSPACE;
+  if (num_chunks < 0 || num_segments < 0 || !chunks || !segments || !seq_segments || !a->cu_seqlens) return MOPS_HIP_EINVAL;
+  if (num_chunks == 0 || num_segments == 0) return MOPS_HIP_OK;
+  if (num_chunks * a->heads > 0x7fffffffLL || num_segments * a->heads * ((a->vd + a->d + 31) / 16) > 0x3fffffffLL ||
+      a->batch * a->heads * ((a->vd + 15) / 16) > 0x7fffffffLL)
+    return MOPS_HIP_EUNSUPPORTED;
+  if (!workspace || workspace_bytes < mops_hip_delta_chunks_workspace_bytes(num_chunks, num_segments, a->batch, a->heads, a->d, a->vd)) return MOPS_HIP_EWORKSPACE;
   if (!aligned16(workspace)) return MOPS_HIP_EALIGN;
   DeltaChunkArgs p;
   p.a = *a;
   p.chunks = chunks;
-  p.seq_chunks = seq_chunks;
+  p.segments = segments;
+  p.seq_segments = seq_segments;
   p.num_chunks = (int)num_chunks;
+  p.num_segments = (int)num_segments;
   p.pitch = (int)mops_hip_recurrence_state_pitch(a->d);
   p.operands = (unsigned char*)workspace;
+  p.seg_map = p.operands + num_chunks * a->heads * operand_bytes(a->d);
+  p.seg_state = num_segments > a->batch ? (float*)(p.seg_map + num_segments * a->heads * map_bytes(a->d)) : nullptr;
   p.vec = a->d % 4 == 0 && a->vd % 4 == 0 && a->q_stride % 4 == 0 && a->k_stride % 4 == 0 && a->log_decay_stride % 4 == 0 && a->out_stride % 4 == 0 &&
           aligned16(a->q) && aligned16(a->k) && aligned16(a->log_decay) && aligned16(a->out);
   hipStream_t s = (hipStream_t)stream;

@@ -17,7 +17,7 @@ from dataclasses import dataclass
 import torch
 
 from .. import mops
-from ..mops.hip.recurrent_ops import CHUNK_MAX_DIM, channel_segments, delta_chunk_list, recurrence_segments
+from ..mops.hip.recurrent_ops import CHUNK_MAX_DIM, channel_segments, delta_cuts, recurrence_segments
 
 MIXERS: dict = {}
 FEED_FORWARDS: dict = {}
@@ -110,6 +110,7 @@ class ChunkedRecurrence:
         self.recurrence, self.chunks = hip_op(self.RECURRENCE), hip_op(self.CHUNKS)
 
     def segments(self, counts):
+        """Host lists: tables of rows, then the bounds of every portion's segments."""
         heads, groups, _, vd = self.sizes
         return recurrence_segments(counts, heads, groups, vd)
 
@@ -123,10 +124,10 @@ class ChunkedRecurrence:
         cuts = ctx.setdefault("segment_cuts", {})
         key = (self.CHUNKS, heads, groups, vd)
         if key not in cuts:
-            segments, bounds = self.segments(ctx["seq_counts"][nd:])
-            flat = torch.tensor([x for s in segments for x in s] + bounds, dtype=torch.int32).to(v.device, non_blocking=True)
-            at = len(segments) * len(segments[0])
-            cuts[key] = (flat[:at].view(len(segments), -1), flat[at:])
+            *tables, bounds = self.segments(ctx["seq_counts"][nd:])
+            sizes = [len(t) * len(t[0]) for t in tables] + [len(bounds)]
+            flat = torch.tensor([x for t in tables for row in t for x in row] + bounds, dtype=torch.int32).to(v.device, non_blocking=True).split(sizes)
+            cuts[key] = [f.view(len(t), -1) for f, t in zip(flat, tables)] + [flat[-1]]
         return self.chunks(q, k, v, out, state, slots, starts, *self.sizes, *cuts[key], cu_seqlens=cu, **options)
 
 
@@ -139,11 +140,11 @@ class ChannelRecurrence(ChunkedRecurrence):
 
 
 class DeltaRecurrence(ChunkedRecurrence):
-    """The same for the gated delta rule; a cut is a list of chunks."""
+    """The same for the gated delta rule; a cut also lists the chunks."""
     RECURRENCE, CHUNKS = "delta_rule", "delta_chunks"
 
     def segments(self, counts):
-        return delta_chunk_list(counts)
+        return delta_cuts(counts, self.sizes[0], self.sizes[3])
 
 
 def hip_op(name):

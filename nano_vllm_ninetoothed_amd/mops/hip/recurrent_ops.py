@@ -367,26 +367,33 @@ def delta_rule(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, *
 DELTA_CHUNK = 16      # tokens
 
 
-def delta_chunk_list(counts):
-    """Cuts portions of counts[i] tokens (packed one behind the other) for delta_chunks: host lists (chunks, bounds per portion)."""
-    chunks, bounds, at = [], [0], 0
-    for n in counts:
+def delta_cuts(counts, heads: int, vd: int, wanted: int = 256, enough: int = 128):
+    """Cuts portions of counts[i] tokens (packed one behind the other) for delta_chunks: host lists (chunks, segments, bounds of the
+    segments per portion).  One segment per portion if those give enough workgroups, else about `wanted` workgroups in all."""
+    per_segment, length = _capi.load().mops_hip_delta_chunks_workgroups(heads, vd), max(counts)
+    if len(counts) * per_segment < enough and length > 256:
+        length = max(128, -(-sum(counts) * per_segment // wanted // DELTA_CHUNK) * DELTA_CHUNK)
+    length = -(-length // DELTA_CHUNK) * DELTA_CHUNK
+    chunks, segments, bounds, at = [], [], [0], 0
+    for i, n in enumerate(counts):
+        for begin in range(0, n, length):
+            segments.append((i, at + begin, at + min(n, begin + length), len(chunks) + begin // DELTA_CHUNK))
+        bounds.append(len(segments))
         chunks += [(at + begin, min(DELTA_CHUNK, n - begin)) for begin in range(0, n, DELTA_CHUNK)]
-        bounds.append(len(chunks))
         at += n
-    return chunks, bounds
+    return chunks, segments, bounds
 
 
 @register_hip_op
-def delta_chunks(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, chunks, seq_chunks, **options):
-    """delta_rule for packed portions of many tokens, on the matrix cores (bf16, d up to CHUNK_MAX_DIM).  chunks [n, 2] and seq_chunks
-    [sequences + 1] are the int32 device copies of what delta_chunk_list returns; cu_seqlens is required."""
+def delta_chunks(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, chunks, segments, seq_segments, **options):
+    """delta_rule for packed portions of many tokens, on the matrix cores (bf16, d up to CHUNK_MAX_DIM).  chunks [n, 2], segments [m, 4]
+    and seq_segments [sequences + 1] are the int32 device copies of what delta_cuts returns; cu_seqlens is required."""
     a = _delta_args(q, k, v, out, state, state_slots, starts, heads, groups, d, vd, **options)
-    n, lib = chunks.shape[0], _capi.load()
-    _require(a.batch == seq_chunks.numel() - 1, "seq_chunks must bound the chunks of every sequence")
-    ws = torch.empty(max(16, lib.mops_hip_delta_chunks_workspace_bytes(n, heads, d)), dtype=torch.uint8, device=v.device)
-    st = lib.mops_hip_delta_chunks(byref(a), _flat("chunks", chunks, 2 * n, torch.int32), n, _flat("seq_chunks", seq_chunks, a.batch + 1, torch.int32),
-                                   ws.data_ptr(), ws.numel(), _stream(v))
+    n, m, lib = chunks.shape[0], segments.shape[0], _capi.load()
+    _require(a.batch == seq_segments.numel() - 1, "seq_segments must bound the segments of every sequence")
+    ws = torch.empty(max(16, lib.mops_hip_delta_chunks_workspace_bytes(n, m, a.batch, heads, d, vd)), dtype=torch.uint8, device=v.device)
+    st = lib.mops_hip_delta_chunks(byref(a), _flat("chunks", chunks, 2 * n, torch.int32), n, _flat("segments", segments, 4 * m, torch.int32), m,
+                                   _flat("seq_segments", seq_segments, a.batch + 1, torch.int32), ws.data_ptr(), ws.numel(), _stream(v))
     _capi.check("mops_hip_delta_chunks", st)
     return out
 

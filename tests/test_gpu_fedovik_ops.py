@@ -294,7 +294,7 @@ def weak(g, shape):
     return -torch.exp(torch.randn(shape, generator=g) * 0.5 - 9)
 
 
-def run_delta(gpu, which, dtype, H, G, d, vd, counts, starts, log_decay, seed=0, slots=None, alike=0.0, beta_at=0.0):
+def run_delta(gpu, which, dtype, H, G, d, vd, counts, starts, log_decay, seed=0, slots=None, alike=0.0, beta_at=0.0, wanted=256):
     """Largest relative errors of outputs and states over the sequences.  alike: how much of a key all keys of a head share."""
     from nano_vllm_ninetoothed_amd.mops.hip import recurrent_ops as R
     g = torch.Generator().manual_seed(seed)
@@ -317,8 +317,8 @@ def run_delta(gpu, which, dtype, H, G, d, vd, counts, starts, log_decay, seed=0,
     args = [on[:, :G * d], on[:, G * d:2 * G * d], on[:, 2 * G * d:2 * G * d + H * vd], out, state, i32(slots, gpu), i32(starts, gpu), H, G, d, vd]
     options = dict(log_decay=lw.to(gpu), beta=beta.to(gpu)[:, :H], q_scale=d ** -0.5, unit_eps=1e-6, cu_seqlens=i32(cu, gpu))
     if which == "chunks":
-        chunks, ends = R.delta_chunk_list(counts)
-        op("delta_chunks")(*args, i32(chunks, gpu), i32(ends, gpu), **options)
+        cuts = R.delta_cuts(counts, H, vd, wanted)
+        op("delta_chunks")(*args, *(i32(x, gpu) for x in cuts), **options)
     else:
         if max(counts) == 1:
             del options["cu_seqlens"]
@@ -350,10 +350,10 @@ def test_delta_rule_token_by_token(gpu, dtype, H, G, d, vd):
 
 @pytest.mark.parametrize("H,G,d,vd", DELTA_SIZES)
 def test_delta_rule_in_chunks(gpu, H, G, d, vd):
-    """Portions shorter and longer than chunks; all strengths of decay; keys that are nearly the same throughout, so that every write
+    """Portions shorter and longer than chunks, and some that are cut into segments; all strengths of decay; keys that are nearly the same throughout, so that every write
     answers all those in front of it."""
     for seed, decay in enumerate((usual, strong, weak)):
-        for counts, starts, alike in (([2, 37, 16, 1, 100], [0, 5, 3, 2, 0], 0.0), ([17], [4], 6.0), ([300, 33], [0, 7], 2.0), ([64], [0], 30.0)):
+        for counts, starts, alike in (([2, 37, 16, 1, 100], [0, 5, 3, 2, 0], 0.0), ([17], [4], 6.0), ([300, 33], [0, 7], 2.0), ([64], [0], 30.0), ([290, 517], [9, 0], 0.0), ([700], [3], 1.0)):
             o, S = run_delta(gpu, "chunks", torch.bfloat16, H, G, d, vd, counts, starts, decay, seed=seed, alike=alike, beta_at=2.0 if alike else 0.0)
             assert o < 4e-3 and S < 1e-4, (decay.__name__, counts, o, S)
 
