@@ -50,41 +50,37 @@ __global__ __launch_bounds__(256) void delta_rule_kernel(const mops_hip_delta a,
   const int per_group = heads / (int)a.groups, g = h / per_group;
   const T *q = (const T*)a.q + (int64_t)g * d, *k = (const T*)a.k + (int64_t)g * d, *v = (const T*)a.v + (int64_t)h * vd + row0;
   T* ring = CONV ? (T*)a.conv_ring + (int64_t)slot * taps * a.channels : nullptr;
-  // channel c of the convolution, current input x: the output for position pos; `keep` also files x in the ring
-  auto conv = [&](float x, int64_t c, int pos, bool keep) {
+  // channel c of the convolution, current input x: the output for position start; `keep` also files x in the ring
+  const int ring_row = CONV ? start % taps : 0, lags = start < taps - 1 ? start : taps - 1;
+  auto conv = [&](float x, int64_t c, bool keep) {
     float acc = a.conv_weight[(int64_t)(taps - 1) * a.channels + c] * x;
-    for (int lag = 1; lag < taps; ++lag)
-      if (pos - lag >= 0)
-        acc += a.conv_weight[(int64_t)(taps - 1 - lag) * a.channels + c] * to_f32(ring[(int64_t)((pos - lag) % taps) * a.channels + c]);
-    if (keep) ring[(int64_t)(pos % taps) * a.channels + c] = from_f32<T>(x);
+#pragma unroll 4
+    for (int lag = 1; lag <= lags; ++lag) {
+      const int row = ring_row - lag < 0 ? ring_row - lag + taps : ring_row - lag;
+      acc += a.conv_weight[(int64_t)(taps - 1 - lag) * a.channels + c] * to_f32(ring[(int64_t)row * a.channels + c]);
+    }
+    if (keep) ring[(int64_t)ring_row * a.channels + c] = from_f32<T>(x);
     return silu_for<T>(acc);
   };
   for (int t = t_begin; t < t_end; ++t) {
-    const int pos = start + (t - t_begin);
     float q_squares = 0.f, k_squares = 0.f;
-    for (int i = tid; i < kDim; i += 256) {
-      float qv = 0.f, kv = 0.f, decay = 1.f;
+    for (int j = tid; j < 2 * kDim; j += 256) {      // q, then k
+      const bool is_k = j >= kDim;
+      const int i = is_k ? j - kDim : j;
+      float x = 0.f;
       if (i < d) {
-        qv = to_f32(q[t * a.q_stride + i]);
-        kv = to_f32(k[t * a.k_stride + i]);
-        if (CONV) {
-          const bool keep = tile == 0 && h % per_group == 0;
-          qv = conv(qv, a.q_channel + (int64_t)g * d + i, pos, keep);
-          kv = conv(kv, a.k_channel + (int64_t)g * d + i, pos, keep);
-        }
-        decay = expf(a.log_decay[t * a.log_decay_stride + (int64_t)h * d + i]);
+        x = to_f32((is_k ? k + t * a.k_stride : q + t * a.q_stride)[i]);
+        if (CONV) x = conv(x, (is_k ? a.k_channel : a.q_channel) + (int64_t)g * d + i, tile == 0 && h % per_group == 0);
       }
-      sq[i] = qv;
-      sk[i] = kv;
-      sa[i] = decay;
-      q_squares += qv * qv;
-      k_squares += kv * kv;
+      (is_k ? sk : sq)[i] = x;
+      (is_k ? k_squares : q_squares) += x * x;
     }
+    for (int i = tid; i < kDim; i += 256) sa[i] = i < d ? expf(a.log_decay[t * a.log_decay_stride + (int64_t)h * d + i]) : 1.f;
     for (int i = tid; i < kRows; i += 256) {
       float x = 0.f;
       if (row0 + i < vd) {
         x = to_f32(v[t * a.v_stride + i]);
-        if (CONV) x = conv(x, a.v_channel + (int64_t)h * vd + row0 + i, pos, true);
+        if (CONV) x = conv(x, a.v_channel + (int64_t)h * vd + row0 + i, true);
       }
       sv[i] = x;
     }
